@@ -546,7 +546,7 @@ def main():
             with open(tf) as fh:
                 doc = json.load(fh)
             traffic = doc["traffic_bytes_per_launch"]
-            with open(os.path.join(ROOT, "vllm-neuron_amd", "csrc", "linear_kernels.hip"), "rb") as fh:
+            with open(os.path.join(ROOT, "vllm-neuron_amd", "csrc", "linear_device.h"), "rb") as fh:
                 fresh = hashlib.sha1(fh.read()).hexdigest() == doc.get("kernel_source_sha1")
             traffic_src = ("profiles/r03_gemv_traffic.json (rocprofv3 --pmc FETCH_SIZE pass of this command, x2 gfx950 "
                            "correction: the counter tallies 128-B requests at 64 B)"

@@ -1,5 +1,5 @@
 """Dev tool: in-kernel phase timeline of the decode GEMVs (needs a -DMI_TRACE build of the library,
-passed as MI355X_VLLM_LIB=...; see the MI_TRACE block in csrc/linear_kernels.hip)."""
+passed as MI355X_VLLM_LIB=...; see the MI_TRACE block in csrc/linear_device.h)."""
 import ctypes, os, sys
 sys.path.insert(0, os.path.dirname(os.path.dirname(os.path.abspath(__file__))))
 import numpy as np

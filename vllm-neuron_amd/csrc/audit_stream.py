@@ -12,7 +12,7 @@ The check is a may-analysis over the kernel's control-flow graph: a register ran
 "in flight" at a point if it is in flight on ANY path reaching it.  build.py runs this on
 every build and fails the build on a finding.
 
-    python audit_stream.py linear_kernels.s
+    python audit_stream.py gemv_f8.s
 """
 import re
 import sys

@@ -12,12 +12,14 @@ import subprocess
 import sys
 
 HERE = os.path.dirname(os.path.abspath(__file__))
-SOURCES = ["linear_kernels.hip", "attn_kernels.hip", "misc_kernels.hip", "model.hip", "tp_group.hip"]
-HEADERS = ["mi_common.h", "linear_kernels.h", "attn_kernels.h", "misc_kernels.h", "model_internal.h", "tp_group.h",
+SOURCES = ["gemv_bf16.hip", "gemv_f8.hip", "gemv_i8.hip", "linear_kernels.hip", "attn_kernels.hip", "misc_kernels.hip", "model.hip", "tp_group.hip"]
+HEADERS = ["mi_common.h", "linear_device.h", "linear_kernels.h", "attn_kernels.h", "misc_kernels.h", "model_internal.h", "tp_group.h",
            os.path.join("..", "..", "include", "mi355x_vllm.h")]
 LIB = os.path.join(HERE, "libmi355x_vllm.so")
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function", "-Wno-unused-value",
-         "-Wno-unused-result", "-I/opt/rocm/include"]
+         "-Wno-unused-result", "-I/opt/rocm/include",
+         # no packed fp32 math (v_pk_{add,mul,fma}_f32): some of its forms are not reliable on these machines
+         "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 # extra flags for probe builds (e.g. MI_EXTRA_FLAGS="-DMI_TRACE"); part of the stamp below
 FLAGS += os.environ.get("MI_EXTRA_FLAGS", "").split()
 STAMP = os.path.join(HERE, "build", "flags.stamp")
@@ -56,7 +58,7 @@ def _compile(src, force=False):
 def build(verbose=True):
     os.makedirs(os.path.join(HERE, "build"), exist_ok=True)
     force = "--force" in sys.argv or _flags_changed()
-    with cf.ThreadPoolExecutor(max_workers=4) as ex:
+    with cf.ThreadPoolExecutor(max_workers=min(len(SOURCES), int(os.environ.get("MAX_JOBS") or os.cpu_count() or 4))) as ex:
         results = list(ex.map(lambda src: _compile(src, force), SOURCES))
     objs = [o for o, _ in results]
     for _, warn in results:

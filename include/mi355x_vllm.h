@@ -93,10 +93,42 @@ typedef struct mi_model_config {
 #define MI_TP_ALL_RANKS (-1)
 enum { MI_TP_TRANSPORT_P2P = 0, MI_TP_TRANSPORT_RCCL = 1 };
 
+/* ---- layer-stack decoders: a decoder given layer by layer, every size and constant a parameter ----
+ * (Vimesun is the first such design; the worker's model registry fills this from its config.json.)
+ *     x = embed[token] + pos[position]                        fp32 residual stream
+ *     layer:  x <- x + residual_mult (attention(norm1(x)) + feed-forward(norm2(x)))   both of the same x
+ *     norms:  layer norm with weight and bias
+ *     loop:   layers loop_start .. loop_stop - 1 run loop_times times in a row with the same weights, each pass with a
+ *             KV pool of its own; ahead of a pass's first layer  x <- W_in [x ; embedding output]
+ *     logits = head final_norm(x)
+ * Tensor names ("l<i>." = layer i): embed, pos, loop.in, l<i>.norm1(.b), l<i>.norm2(.b), l<i>.mix.{q,k,v,o},
+ * l<i>.mlp.{up,down}, final.norm(.b), head. */
+enum { MI_FF_NONE = 0, MI_FF_RELU2 = 1 };   /* down(max(up x, 0)^2) */
+typedef struct mi_layer_spec {
+  int32_t num_heads, num_kv_heads, qk_dim, v_dim;
+  int32_t window;         /* a query sees keys with 0 <= i - j < window; 0 = every earlier token */
+  float scale;            /* of q . k */
+  int32_t qk_unit_norm;   /* q and k heads divided by sqrt(mean square + norm_eps) */
+  int32_t distance_bias;  /* 2^(-8 (h + 1) / num_heads) (i - j) taken off the score of head h */
+  int32_t softmax_sink;   /* one added to the softmax denominator */
+  int32_t ff_kind, ff_size;
+} mi_layer_spec;
+typedef struct mi_stack_config {
+  int32_t num_layers;
+  const mi_layer_spec* layers;
+  int32_t width, vocab_size, max_positions;
+  float norm_eps, residual_mult;
+  int32_t loop_start, loop_stop, loop_times;   /* loop_times = 0: no loop (and no loop.in) */
+  int32_t compute_dtype;   /* MI_BF16: bf16 matrix products and KV; MI_F32: everything in fp32 (plain kernels: for checking) */
+} mi_stack_config;
+
 const char* mi_last_error(void);
-int mi_version(void);   /* 4 = this header (+ mi_tp_plan, mi_tp_info); 3 lacked them; 2 lacked tp_device_ids / tp_transport / MI_TP_ALL_RANKS; 1 lacked mi_forward_tokens, mi_op_sample, mi_tp_init_transport */
+int mi_version(void);   /* 5 = this header (+ mi_ctx_create_stack, mi_forward_rows, mi_layer_residuals, mi_op_* of the stack kernels); 4 (+ mi_tp_plan, mi_tp_info); 3 lacked them; 2 lacked tp_device_ids / tp_transport / MI_TP_ALL_RANKS; 1 lacked mi_forward_tokens, mi_op_sample, mi_tp_init_transport */
 
 int mi_ctx_create(const mi_model_config* cfg, mi_ctx** out);
+/* The same context around a layer stack.  Of cfg only the serving fields are read (pool, batch, buckets, device, graphs);
+ * geometry comes from `stack` (copied).  One GPU, unquantized weights. */
+int mi_ctx_create_stack(const mi_model_config* cfg, const mi_stack_config* stack, mi_ctx** out);
 int mi_ctx_destroy(mi_ctx* ctx);
 
 /* One HF-named tensor ("model.layers.3.self_attn.q_proj.weight", "lm_head.weight", ...),
@@ -165,6 +197,17 @@ int mi_forward_chunked(mi_ctx* ctx, int32_t n_req, int32_t total, const int64_t*
                        const int64_t* position_ids, const int64_t* slot_mapping, const int64_t* block_table,
                        int32_t MB, const int64_t* full_context_lens, const int64_t* computed_context_lens,
                        float* logits_out, const float* sampling_params, uint64_t seed, int64_t* tokens_out);
+
+/* The same ragged batch with the logits of chosen places: rows [n_rows] = indices into the token batch (any order, any
+ * number, none at all); logits_out [n_rows, vocab_size] in that order. */
+int mi_forward_rows(mi_ctx* ctx, int32_t n_req, int32_t total, const int64_t* input_ids, const int64_t* position_ids,
+                    const int64_t* slot_mapping, const int64_t* block_table, int32_t MB, const int64_t* full_context_lens,
+                    const int64_t* computed_context_lens, int32_t n_rows, const int64_t* rows, float* logits_out);
+
+/* Layer-stack contexts: keep a copy of the residual stream behind every layer run of the following ragged batches
+ * (on != 0).  mi_layer_residuals_read copies it out: [layer runs][rows of the last batch][width] fp32.  For checking. */
+int mi_layer_residuals(mi_ctx* ctx, int32_t on);
+int mi_layer_residuals_read(mi_ctx* ctx, int32_t rows, float* out);
 
 /* Fused speculation (the reference reaches it through NxDI's fused draft + target graph:
  * loader.py:349-355; output contract re-masked by _remask_fused_spec_output, loader.py:308-333; slots
@@ -337,6 +380,24 @@ int mi_op_paged_attn_prefill(const void* q, int32_t T, int32_t q_pos0, const voi
                              int32_t num_blocks, int32_t block_size, const int32_t* block_table,
                              int32_t MB, int32_t nh, int32_t nkv, int32_t hd, void* out,
                              void* stream);
+
+/* ---- kernels of the layer-stack decoders.  f32 != 0: activations / pools are fp32, else bf16 ----
+ * y1 / y2 [T, ldy] = layer norm of x [T, ld] fp32 over its first D columns (w, b [ld] fp32, zero beyond D; y2 may be NULL) */
+int mi_op_layernorm2(const float* x, int32_t T, int32_t D, int32_t ld, float eps, const float* w1, const float* b1, void* y1,
+                     const float* w2, const float* b2, void* y2, int32_t ldy, int32_t f32, void* stream);
+/* resid[t] (and x0[t], may be NULL) [T, ld] fp32 = table[ids[t]] + ptable[pos[t]], columns beyond D zero */
+int mi_op_embed_pos(const int32_t* ids, const int32_t* pos, const void* table, const void* ptable, int32_t T, int32_t D, int32_t ld,
+                    float* resid, float* x0, int32_t f32, void* stream);
+/* qkv [T, ldq] fp32 -> q [T, H, pad16(dk)], K pool [blocks][G][block_size][pad16(dk)], V pool [..][pad16(dv)] at slots (-1: skip) */
+int mi_op_qkv_scatter(const float* qkv, int32_t ldq, int32_t T, const mi_layer_spec* spec, float eps, const int32_t* slots,
+                      int32_t block_size, void* q, void* kpool, void* vpool, int32_t f32, void* stream);
+/* Windowed attention of a ragged batch over those pools.  segs_host [nseg][4] = (first row, rows, first position, block-table
+ * row); pos [T]; ctx_lens [block-table rows] (keys incl. the row's own) for one-row segments.  slopes [H] or NULL.
+ * path: 0 the model's choice, 1 the plain kernel.  out [T, H v_dim] (row stride ldo).  All device pointers but segs_host. */
+int mi_op_window_attn(const mi_layer_spec* spec, const float* slopes, const void* q, const void* kpool, const void* vpool,
+                      int32_t block_size, const int32_t* block_table, int32_t MB, const int32_t* pos, const int32_t* ctx_lens,
+                      const int32_t* segs_host, int32_t nseg, int32_t T, int32_t max_ctx, void* out, int32_t ldo, int32_t f32,
+                      int32_t path, void* stream);
 
 #ifdef __cplusplus
 }

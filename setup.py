@@ -37,7 +37,7 @@ setup(
     description="vLLM MI355X (gfx950) backend plugin: hand-written HIP hot path behind the vllm-neuron plugin boundary",
     license="Apache 2.0",
     package_dir={"vllm_neuron_amd": SRC},
-    packages=["vllm_neuron_amd", "vllm_neuron_amd.core", "vllm_neuron_amd.worker"],
+    packages=["vllm_neuron_amd", "vllm_neuron_amd.core", "vllm_neuron_amd.models", "vllm_neuron_amd.worker"],
     package_data={"vllm_neuron_amd": ["csrc/libmi355x_vllm.so", "csrc/*.h", "csrc/*.hip", "csrc/build.py"]},
     data_files=[("include", ["include/mi355x_vllm.h"])],
     cmdclass={"build_py": BuildWithHip},

@@ -53,6 +53,23 @@ class MiKvStats(C.Structure):
                 ("block_table_rows_sent", C.c_int64), ("block_table_rows_kept", C.c_int64)]
 
 
+MI_FF = {None: 0, "relu2": 1}
+MI_COMPUTE = {"bfloat16": MI_BF16, "float32": MI_F32}
+
+
+class MiLayerSpec(C.Structure):
+    _fields_ = [("num_heads", C.c_int32), ("num_kv_heads", C.c_int32), ("qk_dim", C.c_int32), ("v_dim", C.c_int32),
+                ("window", C.c_int32), ("scale", C.c_float), ("qk_unit_norm", C.c_int32), ("distance_bias", C.c_int32),
+                ("softmax_sink", C.c_int32), ("ff_kind", C.c_int32), ("ff_size", C.c_int32)]
+
+
+class MiStackConfig(C.Structure):
+    _fields_ = [("num_layers", C.c_int32), ("layers", C.POINTER(MiLayerSpec)), ("width", C.c_int32),
+                ("vocab_size", C.c_int32), ("max_positions", C.c_int32), ("norm_eps", C.c_float),
+                ("residual_mult", C.c_float), ("loop_start", C.c_int32), ("loop_stop", C.c_int32),
+                ("loop_times", C.c_int32), ("compute_dtype", C.c_int32)]
+
+
 class MiTpPlan(C.Structure):
     _fields_ = [("q_head0", C.c_int32), ("q_heads_real", C.c_int32), ("q_heads_local", C.c_int32),
                 ("kv_head0", C.c_int32), ("kv_heads_local", C.c_int32), ("inter0", C.c_int32), ("inter_local", C.c_int32),
@@ -72,6 +89,7 @@ _SIGS = {
     "mi_last_error": (C.c_char_p, []),
     "mi_version": (C.c_int, []),
     "mi_ctx_create": (C.c_int, [C.POINTER(MiModelConfig), C.POINTER(C.c_void_p)]),
+    "mi_ctx_create_stack": (C.c_int, [C.POINTER(MiModelConfig), C.POINTER(MiStackConfig), C.POINTER(C.c_void_p)]),
     "mi_ctx_destroy": (C.c_int, [C.c_void_p]),
     "mi_load_weight": (C.c_int, [C.c_void_p, C.c_char_p, C.c_void_p, C.c_int32,
                                  C.POINTER(C.c_int64), C.c_int32]),
@@ -88,6 +106,19 @@ _SIGS = {
                                     C.c_void_p, C.c_uint64, C.c_void_p]),
     "mi_forward_chunked": (C.c_int, [C.c_void_p, C.c_int32, C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p,
                                      C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p, C.c_uint64, C.c_void_p]),
+    "mi_forward_rows": (C.c_int, [C.c_void_p, C.c_int32, C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p,
+                                  C.c_int32, C.c_void_p, C.c_void_p, C.c_int32, C.c_void_p, C.c_void_p]),
+    "mi_layer_residuals": (C.c_int, [C.c_void_p, C.c_int32]),
+    "mi_layer_residuals_read": (C.c_int, [C.c_void_p, C.c_int32, C.c_void_p]),
+    "mi_op_layernorm2": (C.c_int, [C.c_void_p, C.c_int32, C.c_int32, C.c_int32, C.c_float, C.c_void_p, C.c_void_p, C.c_void_p,
+                                   C.c_void_p, C.c_void_p, C.c_void_p, C.c_int32, C.c_int32, C.c_void_p]),
+    "mi_op_embed_pos": (C.c_int, [C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p, C.c_int32, C.c_int32, C.c_int32, C.c_void_p,
+                                  C.c_void_p, C.c_int32, C.c_void_p]),
+    "mi_op_qkv_scatter": (C.c_int, [C.c_void_p, C.c_int32, C.c_int32, C.POINTER(MiLayerSpec), C.c_float, C.c_void_p, C.c_int32,
+                                    C.c_void_p, C.c_void_p, C.c_void_p, C.c_int32, C.c_void_p]),
+    "mi_op_window_attn": (C.c_int, [C.POINTER(MiLayerSpec), C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p, C.c_int32, C.c_void_p,
+                                    C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p, C.c_int32, C.c_int32, C.c_int32, C.c_void_p,
+                                    C.c_int32, C.c_int32, C.c_int32, C.c_void_p]),
     "mi_forward_spec": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int32, C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p,
                                   C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p]),
     "mi_replay_decode": (C.c_int, [C.c_void_p, C.c_int32, C.POINTER(C.c_float)]),
@@ -166,10 +197,35 @@ def _ptr(t) -> int:
     return 0 if t is None else t.data_ptr()
 
 
+def layer_spec(layer: dict) -> MiLayerSpec:
+    out = MiLayerSpec()
+    for k, v in layer.items():
+        if not hasattr(out, k):
+            raise ValueError(f"unknown layer field {k!r}")
+        setattr(out, k, v)
+    return out
+
+
+def stack_config(stack: dict) -> MiStackConfig:
+    st = MiStackConfig()
+    layers = [layer_spec(x) for x in stack["layers"]]
+    st._keep = (MiLayerSpec * len(layers))(*layers)      # the library copies it during the call
+    st.layers, st.num_layers = st._keep, len(layers)
+    for k, v in stack.items():
+        if k == "layers":
+            continue
+        if not hasattr(st, k):
+            raise ValueError(f"unknown stack field {k!r}")
+        setattr(st, k, v)
+    return st
+
+
 class NativeModel:
     """Owns one mi_ctx: device weights, paged KV pool, activations, stream."""
 
-    def __init__(self, **cfg):
+    def __init__(self, stack: dict | None = None, **cfg):
+        """`stack`: a layer-stack decoder (include/mi355x_vllm.h: mi_stack_config by field name, `layers` a list of
+        mi_layer_spec dicts) in place of the Llama-family geometry fields."""
         self.lib = load_library()
         c = MiModelConfig()
         buckets = list(cfg.pop("ctx_buckets", None) or [])
@@ -186,10 +242,17 @@ class NativeModel:
         for i, b in enumerate(buckets[:8]):
             c.ctx_buckets[i] = int(b)
         self.cfg = c
-        self.vocab_size = c.vocab_size
         self._logits_view = None
         self._ctx = C.c_void_p()
-        check(self.lib.mi_ctx_create(C.byref(c), C.byref(self._ctx)))
+        if stack is None:
+            check(self.lib.mi_ctx_create(C.byref(c), C.byref(self._ctx)))
+        else:
+            st = stack_config(stack)
+            c.vocab_size = st.vocab_size
+            self.width = st.width
+            self.layer_runs = st.num_layers + (max(st.loop_times - 1, 0)) * (st.loop_stop - st.loop_start)
+            check(self.lib.mi_ctx_create_stack(C.byref(c), C.byref(st), C.byref(self._ctx)))
+        self.vocab_size = c.vocab_size
 
     def close(self):
         if getattr(self, "_ctx", None) and self._ctx.value:
@@ -352,6 +415,31 @@ class NativeModel:
                                           None if tokens else out.data_ptr(),
                                           sp.data_ptr() if sp is not None else None, seed & (2 ** 64 - 1),
                                           out.data_ptr() if tokens else None))
+        return out
+
+    def forward_rows(self, input_ids, position_ids, slot_mapping, block_table, full_context_lens, computed_context_lens,
+                     rows) -> "torch.Tensor":
+        """The ragged batch of `forward_chunked` with the logits of chosen places: `rows` = indices into the token
+        batch (may be empty).  -> fp32 logits [len(rows), V]."""
+        def i64(t):
+            return torch.as_tensor(t).to(torch.int64).contiguous().reshape(-1)
+        ids, pos, sm, full, comp, want = (i64(t) for t in (input_ids, position_ids, slot_mapping, full_context_lens,
+                                                           computed_context_lens, rows))
+        n = full.numel()
+        bt = block_table.to(torch.int64).contiguous().reshape(n, -1)
+        out = torch.empty(want.numel(), self.vocab_size, dtype=torch.float32)
+        check(self.lib.mi_forward_rows(self._ctx, n, ids.numel(), ids.data_ptr(), pos.data_ptr(), sm.data_ptr(), bt.data_ptr(),
+                                       bt.shape[1], full.data_ptr(), comp.data_ptr(), want.numel(),
+                                       want.data_ptr() if want.numel() else None, out.data_ptr() if want.numel() else None))
+        return out
+
+    def keep_layer_residuals(self, on: bool) -> None:
+        check(self.lib.mi_layer_residuals(self._ctx, int(on)))
+
+    def layer_residuals(self, rows: int) -> "torch.Tensor":
+        """[layer runs, rows, width] fp32: the residual stream behind every layer run of the last batch."""
+        out = torch.empty(self.layer_runs, rows, self.width, dtype=torch.float32)
+        check(self.lib.mi_layer_residuals_read(self._ctx, rows, out.data_ptr()))
         return out
 
     def forward_spec(self, draft: "NativeModel", input_ids, position_ids, block_table, k: int, catchup_ids=None):

@@ -522,6 +522,20 @@ else:
             self.requests[request.request_id] = request
             self.waiting.append(request)
 
+        def finish_requests(self, request_ids, finished_status=RequestStatus.FINISHED_ABORTED):
+            """End requests from outside (vLLM's Scheduler.finish_requests): their blocks go back to the pool."""
+            for req_id in ([request_ids] if isinstance(request_ids, str) else request_ids):
+                req = self.requests.pop(req_id, None)
+                if req is None:
+                    continue
+                if req in self.running:
+                    self.running.remove(req)
+                    self.block_pool.release(req.block_ids)
+                    self.finished_req_ids.add(req_id)
+                elif req in self.waiting:
+                    self.waiting.remove(req)
+                req.status = finished_status
+
         def has_unfinished_requests(self):
             return bool(self.waiting or self.running)
 
@@ -538,6 +552,8 @@ else:
                 if budget <= 0:
                     break
                 n_tok = req.num_tokens - req.num_computed_tokens
+                if n_tok <= 0:
+                    continue                   # waits for more input (streaming requests)
                 if self.chunked_prefill:
                     n_tok = min(n_tok, budget)           # the next chunk of a long prompt
                 after = min(req.num_computed_tokens + n_tok + self.num_lookahead_tokens, self.max_model_len)

@@ -8,12 +8,15 @@ travels to the GPU box with the snapshot).
 """
 import concurrent.futures as cf
 import os
+import shutil
 import subprocess
 import sys
 
 HERE = os.path.dirname(os.path.abspath(__file__))
-SOURCES = ["gemv_bf16.hip", "gemv_f8.hip", "gemv_i8.hip", "linear_kernels.hip", "attn_kernels.hip", "misc_kernels.hip", "model.hip", "tp_group.hip"]
-HEADERS = ["mi_common.h", "linear_device.h", "linear_kernels.h", "attn_kernels.h", "misc_kernels.h", "model_internal.h", "tp_group.h",
+HIPCC = shutil.which("hipcc") or "/opt/rocm/bin/hipcc"
+SOURCES = ["gemv_bf16.hip", "gemv_f8.hip", "gemv_i8.hip", "linear_kernels.hip", "attn_kernels.hip", "misc_kernels.hip", "stack_kernels.hip",
+           "window_attn.hip", "stack.hip", "model.hip", "tp_group.hip"]
+HEADERS = ["mi_common.h", "linear_device.h", "linear_kernels.h", "attn_kernels.h", "misc_kernels.h", "model_internal.h", "stack_kernels.h", "window_attn.h", "stack.h", "tp_group.h",
            os.path.join("..", "..", "include", "mi355x_vllm.h")]
 LIB = os.path.join(HERE, "libmi355x_vllm.so")
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function", "-Wno-unused-value",
@@ -48,7 +51,7 @@ def _compile(src, force=False):
     deps = [os.path.join(HERE, src)] + [os.path.join(HERE, h) for h in HEADERS]
     if _mtime(obj) > max(_mtime(d) for d in deps) and not force:
         return obj, ""
-    cmd = ["hipcc", *FLAGS, "-c", os.path.join(HERE, src), "-o", obj]
+    cmd = [HIPCC, *FLAGS, "-c", os.path.join(HERE, src), "-o", obj]
     r = subprocess.run(cmd, capture_output=True, text=True)
     if r.returncode != 0:
         raise RuntimeError(f"hipcc failed for {src}:\n{r.stdout}\n{r.stderr}")
@@ -65,7 +68,7 @@ def build(verbose=True):
         if warn and verbose:
             sys.stderr.write(warn)
     if _mtime(LIB) < max(_mtime(o) for o in objs) or force:
-        cmd = ["hipcc", "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", LIB,
+        cmd = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", LIB,
                "-L/opt/rocm/lib", "-lrccl", "-Wl,-rpath,/opt/rocm/lib"]
         r = subprocess.run(cmd, capture_output=True, text=True)
         if r.returncode != 0:

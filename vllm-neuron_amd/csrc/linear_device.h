@@ -62,6 +62,9 @@ __device__ __forceinline__ void epilogue_store(const EpiArgs& e, int m, int n0, 
     const float a1 = v[2] / (1.f + __expf(-v[2])) * v[3];
     *reinterpret_cast<uint32_t*>(e.act_out + (size_t)m * e.ld_act + (n0 >> 1)) =
         pack_bf16x2(a0, a1);
+  } else if constexpr (EPI == EPI_RELU2) {
+    const float a0 = fmaxf(v[0], 0.f), a1 = fmaxf(v[1], 0.f), a2 = fmaxf(v[2], 0.f), a3 = fmaxf(v[3], 0.f);
+    *reinterpret_cast<uint2*>(e.act_out + (size_t)m * e.ld_act + n0) = make_uint2(pack_bf16x2(a0 * a0, a1 * a1), pack_bf16x2(a2 * a2, a3 * a3));
   } else {  // EPI_QKV
     const int qk_end = e.q_dim + e.kv_dim;
     if (n0 < qk_end) {  // rotary: (v0,v1) and (v2,v3) are (d, d + hd/2) pairs
@@ -906,7 +909,7 @@ static int launch_gemv_kstream(const LinearW& w, int M, const ProArgs& p, const 
 template <int WD, int PRO, int EPI>
 static int launch_gemv_t(const LinearW& w, int M, const ProArgs& p, const EpiArgs& e, hipStream_t s) {
   if (!gemv_fits_whole(M, w.K)) {
-    if constexpr (PRO == PRO_BF16 && (EPI == EPI_F32 || EPI == EPI_RESID)) {
+    if constexpr (PRO == PRO_BF16 && (EPI == EPI_F32 || EPI == EPI_RESID || EPI == EPI_RELU2)) {
       static const int min_m = [] { const char* v = getenv("MI355X_GEMV_KSTREAM_MIN_M"); return v ? atoi(v) : 1; }();
       if (gemv_kstream_enabled() && M >= min_m) return launch_gemv_kstream<WD, EPI>(w, M, p, e, s);
     }
@@ -1493,6 +1496,8 @@ int launch_gemv_wd(const LinearW& w, int M, int pro, const ProArgs& p, int epi, 
   if (pro == PRO_BF16) {
     if (epi == EPI_RESID) return launch_gemv_t<WD, PRO_BF16, EPI_RESID>(w, M, p, e, s);
     if (epi == EPI_F32) return launch_gemv_t<WD, PRO_BF16, EPI_F32>(w, M, p, e, s);
+    if constexpr (WD == MI_W_BF16)
+      if (epi == EPI_RELU2) return launch_gemv_t<WD, PRO_BF16, EPI_RELU2>(w, M, p, e, s);
   } else if (p.partial) {
     if (epi == EPI_QKV) return launch_gemv_t<WD, PRO_NORM_PARTIAL, EPI_QKV>(w, M, p, e, s);
     if (epi == EPI_SWIGLU) return launch_gemv_t<WD, PRO_NORM_PARTIAL, EPI_SWIGLU>(w, M, p, e, s);

@@ -7,7 +7,7 @@
 namespace mi {
 
 // What happens to the fp32 accumulator tile D[n][m] once the contraction is done.
-enum { EPI_F32 = 0, EPI_QKV = 1, EPI_SWIGLU = 2, EPI_RESID = 3 };
+enum { EPI_F32 = 0, EPI_QKV = 1, EPI_SWIGLU = 2, EPI_RESID = 3, EPI_RELU2 = 4 };
 // Where the bf16 activations come from.
 enum { PRO_BF16 = 0, PRO_NORM = 1, PRO_NORM_PARTIAL = 2 };  // callers pass PRO_BF16 / PRO_NORM; PARTIAL is picked when ProArgs::partial is set
 
@@ -32,6 +32,7 @@ struct EpiArgs {
   uint16_t* vpool;
   int block_size;
   // EPI_SWIGLU: rows interleaved (gate_i, up_i); act[m * ld_act + i] = silu(gate)*up
+  // EPI_RELU2 (bf16 weights): act[m * ld_act + n] = max(y, 0)^2
   uint16_t* act_out;
   int ld_act;
 };

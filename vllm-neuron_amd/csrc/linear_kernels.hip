@@ -212,7 +212,10 @@ static int launch_gemm_wd(const LinearW& w, int T, const uint16_t* x, int ldx, i
   if (epi == EPI_QKV) MI_G(EPI_QKV);
   else if (epi == EPI_SWIGLU) MI_G(EPI_SWIGLU);
   else if (epi == EPI_RESID) MI_G(EPI_RESID);
-  else MI_G(EPI_F32);
+  else if (epi == EPI_RELU2) {
+    if constexpr (WD == MI_W_BF16) MI_G(EPI_RELU2);
+    else { set_error("gemm: the squared-relu epilogue is built for bf16 weights"); return MI_EINVAL; }
+  } else MI_G(EPI_F32);
 #undef MI_G
   MI_HIP(hipGetLastError());
   return MI_OK;
@@ -488,7 +491,7 @@ int launch_gemm(const LinearW& w, int T, const uint16_t* x, int ldx, int epi, co
                 float* splitk_ws, size_t splitk_ws_bytes, SlabSum* defer) {
   if (defer) *defer = SlabSum();
   MI_CHECK(T >= 1, "gemm: T must be >= 1");
-  if (gemm_wide_wanted(w, T, splitk_ws ? splitk_ws_bytes : 0) && ldx % 8 == 0)
+  if (epi != EPI_RELU2 && gemm_wide_wanted(w, T, splitk_ws ? splitk_ws_bytes : 0) && ldx % 8 == 0)
     return launch_gemm_wide(w, T, x, ldx, epi, e, s, splitk_ws, splitk_ws_bytes, defer);
   MI_CHECK(w.N % 16 == 0 && w.K % 64 == 0, "gemm: N % 16 == 0 and K % 64 == 0 required");
   MI_CHECK(ldx % 8 == 0, "gemm: x row stride must be a multiple of 8 elements");

@@ -41,6 +41,7 @@ using namespace mi;
   } while (0)
 
 #include "model_internal.h"
+#include "stack.h"
 #include "tp_group.h"
 
 namespace {
@@ -65,28 +66,6 @@ int alloc_linear(mi_ctx* c, Linear& L, int N, int K, int wd, bool bias) {
   }
   return MI_OK;
 }
-
-// ---- profiling wrapper ---------------------------------------------------------------------
-struct Scope {
-  mi_ctx* c;
-  int cls;
-  hipEvent_t a = nullptr, b = nullptr;
-  Scope(mi_ctx* c_, int cls_) : c(c_), cls(cls_) {
-    if (c->prof.on) {
-      hipEventCreate(&a);
-      hipEventCreate(&b);
-      hipEventRecord(a, c->stream);
-    }
-  }
-  ~Scope() {
-    if (c->prof.on) {
-      hipEventRecord(b, c->stream);
-      c->prof.ev.push_back(a);
-      c->prof.ev.push_back(b);
-      c->prof.cls.push_back(cls);
-    }
-  }
-};
 
 int prof_collect(mi_ctx* c) {
   if (!c->prof.on || c->prof.ev.empty()) return MI_OK;
@@ -228,14 +207,18 @@ int all_reduce_partial(mi_ctx* c, int rows) {
 // positions pos0.. and block-table row i.  The projections see one [rows, K] matrix (the weights
 // cross the chip once for all requests); attention runs per request; the logits are those of
 // each request's last row (gathered through d_ctx, which holds the last-row indices).
-struct Seg { int row0, n, pos0; };
+// The trunk leaves the residual stream in c->resid[c->tail_cur] (+ c->partial when c->tail_partial); run_head makes the logits.
+using Seg = AttnSeg;
 static bool attn_early_kv() {   // MI355X_ATTN_EARLY_KV=0: the first K/V request of the decode attention waits for the context length
   static const bool on = [] { const char* v = getenv("MI355X_ATTN_EARLY_KV"); return !v || v[0] != '0'; }();
   return on;
 }
 
-int run_layers(mi_ctx* c, int rows, bool decode, int B, int MB, int q_pos0, int logits_rows,
-               int logits_row0, const Seg* segs = nullptr, int nseg = 0) {
+int run_trunk(mi_ctx* c, int rows, bool decode, int B, int MB, int q_pos0, const Seg* segs = nullptr, int nseg = 0) {
+  if (c->stack) {
+    const Seg whole{0, rows, q_pos0, 0};
+    return stack_trunk(c, rows, decode, MB, decode ? nullptr : (segs ? segs : &whole), decode ? 0 : (segs ? nseg : 1));
+  }
   const mi_model_config& k = c->cfg;
   hipStream_t s = c->stream;
   c->pend = SlabSum();   // (a call that failed half way may have left one behind)
@@ -342,20 +325,32 @@ int run_layers(mi_ctx* c, int rows, bool decode, int B, int MB, int q_pos0, int 
     }
   }
   MI_TRY(flush_pending(c));   // the last down projection's K-split sum: the final norm reads other rows (or a gather of rows)
+  c->tail_cur = cur;
+  c->tail_partial = have_partial;
+  return MI_OK;
+}
+
+// Final norm + lm_head over rows row0 .. + nrows of the trunk's output, or (gather) over the rows listed in c->d_ctx.
+int run_head(mi_ctx* c, int logits_rows, int logits_row0, bool gather) {
+  const mi_model_config& k = c->cfg;
+  hipStream_t s = c->stream;
+  const int cur = c->tail_cur;
+  const bool have_partial = !c->stack && c->tail_partial;
   {  // final norm + lm_head on the rows that are sampled (loader.py:363: logits[:, -1, :])
     ProArgs p{};
     p.resid_in = c->resid[cur] + (size_t)logits_row0 * c->H;
     p.partial = have_partial ? c->partial + (size_t)logits_row0 * c->H : nullptr;
-    if (segs) {   // the last row of every request, made contiguous in the K-split workspace
-      MI_CHECK((size_t)2 * nseg * c->H * 4 <= c->splitk_ws_bytes, "ragged batch: gather workspace too small");
+    if (gather) {   // the listed rows (the last one of every request), made contiguous in the K-split workspace
+      MI_CHECK((size_t)2 * logits_rows * c->H * 4 <= c->splitk_ws_bytes, "ragged batch: gather workspace too small");
       Scope sc(c, MI_K_OTHER);
       float* g0 = c->splitk_ws;
-      float* g1 = g0 + (size_t)nseg * c->H;
-      MI_TRY(launch_gather_rows(c->resid[cur], c->d_ctx, nseg, c->H, g0, s));
-      if (have_partial) MI_TRY(launch_gather_rows(c->partial, c->d_ctx, nseg, c->H, g1, s));
+      float* g1 = g0 + (size_t)logits_rows * c->H;
+      MI_TRY(launch_gather_rows(c->resid[cur], c->d_ctx, logits_rows, c->H, g0, s));
+      if (have_partial) MI_TRY(launch_gather_rows(c->partial, c->d_ctx, logits_rows, c->H, g1, s));
       p.resid_in = g0;
       p.partial = have_partial ? g1 : nullptr;
     }
+    if (c->stack) return stack_head(c, p.resid_in, logits_rows);
     p.resid_out = nullptr;
     p.gain = c->g_final; p.eps = k.rms_norm_eps;
     EpiArgs e{};
@@ -379,6 +374,12 @@ int run_layers(mi_ctx* c, int rows, bool decode, int B, int MB, int q_pos0, int 
     }
   }
   return MI_OK;
+}
+
+int run_layers(mi_ctx* c, int rows, bool decode, int B, int MB, int q_pos0, int logits_rows,
+               int logits_row0, const Seg* segs = nullptr, int nseg = 0) {
+  MI_TRY(run_trunk(c, rows, decode, B, MB, q_pos0, segs, nseg));
+  return run_head(c, logits_rows, logits_row0, segs != nullptr);
 }
 
 int fetch_logits(mi_ctx* c, int nrows, float* out) {
@@ -546,7 +547,7 @@ float bf16_bits_to_f32(uint16_t h) {
 int capture_or_launch_decode(mi_ctx* c, int B, int MB) {
   const int key = (B * 65536 + MB) ^ (int)((c->class_mask & 0xff) << 24) ^ ((c->attn_rows_per_seq - 1) << 12);
   // a caller-supplied transport runs on the host thread: never captured
-  if (!c->cfg.use_graphs || c->prof.on || c->xport_allreduce) return run_layers(c, B, true, B, MB, 0, B, 0);
+  if (!c->cfg.use_graphs || c->prof.on || c->xport_allreduce || (c->stack && c->stack->residuals)) return run_layers(c, B, true, B, MB, 0, B, 0);
   auto it = c->graphs.find(key);
   if (it == c->graphs.end()) {
     // one eager pass first: sets every kernel's attributes outside of capture
@@ -576,7 +577,7 @@ int capture_or_launch_decode(mi_ctx* c, int B, int MB) {
 extern "C" {
 
 const char* mi_last_error(void) { return mi::g_err.c_str(); }
-int mi_version(void) { return 4; }   // 3: + in-process tensor parallelism (tp_rank = MI_TP_ALL_RANKS, tp_device_ids, tp_transport)
+int mi_version(void) { return 5; }   // 3: + in-process tensor parallelism (tp_rank = MI_TP_ALL_RANKS, tp_device_ids, tp_transport)
 
 int mi_tp_plan(const mi_model_config* cfg, int32_t rank, mi_tp_plan_t* out) {
   MI_CHECK(cfg && out, "null argument");
@@ -694,6 +695,53 @@ int mi_ctx_create(const mi_model_config* cfg, mi_ctx** out) {
   return MI_OK;
 }
 
+int mi_ctx_create_stack(const mi_model_config* cfg, const mi_stack_config* stack, mi_ctx** out) {
+  MI_CHECK(cfg && stack && out && stack->layers, "null argument");
+  mi_model_config k = *cfg;
+  const mi_stack_config& t = *stack;
+  MI_CHECK(t.num_layers > 0 && t.width > 0 && t.width <= 32768 && t.vocab_size > 0 && t.max_positions > 0 && t.norm_eps >= 0.f, "stack: bad geometry");
+  MI_CHECK(t.compute_dtype == MI_BF16 || t.compute_dtype == MI_F32, "stack: compute_dtype must be MI_BF16 or MI_F32");
+  MI_CHECK(t.loop_times == 0 || (t.loop_times > 0 && t.loop_start >= 0 && t.loop_start < t.loop_stop && t.loop_stop <= t.num_layers), "stack: bad loop");
+  for (int i = 0; i < t.num_layers; ++i) {
+    const mi_layer_spec& p = t.layers[i];
+    MI_CHECK(p.num_heads > 0 && p.num_kv_heads > 0 && p.num_heads % p.num_kv_heads == 0 && p.qk_dim > 0 && p.v_dim > 0 && p.window >= 0,
+             "stack: layer " + std::to_string(i) + ": bad attention sizes");
+    MI_CHECK(p.ff_kind == MI_FF_NONE || (p.ff_kind == MI_FF_RELU2 && p.ff_size > 0), "stack: layer " + std::to_string(i) + ": bad feed-forward");
+  }
+  MI_CHECK(k.tp_degree <= 1, "stack: tensor parallelism is not built for layer-stack decoders");
+  MI_CHECK(k.weight_dtype == MI_W_BF16, "stack: weight quantization is not built for layer-stack decoders");
+  MI_CHECK(k.block_size > 0 && k.block_size % 16 == 0, "block_size must be a positive multiple of 16");
+  MI_CHECK(k.num_blocks >= 2, "num_blocks must include the null block and at least one real block");
+  MI_CHECK(k.max_num_seqs >= 1 && k.max_num_seqs <= 256, "max_num_seqs must be 1..256");
+  MI_CHECK(k.max_model_len >= 1 && k.max_model_len <= t.max_positions, "max_model_len must be 1..max_positions (learned positions)");
+  int ndev = 0;
+  MI_HIP(hipGetDeviceCount(&ndev));
+  MI_CHECK(ndev > 0, "no HIP device: this library has no CPU fallback");
+  MI_CHECK(k.device_id >= 0 && k.device_id < ndev, "device_id out of range");
+  MI_HIP(hipSetDevice(k.device_id));
+  k.num_layers = t.num_layers;
+  k.vocab_size = t.vocab_size;
+  k.hidden_size = t.width;
+  k.tp_degree = 1;
+  k.tp_rank = 0;
+  k.prefill_fp8_activations = 0;
+  mi_ctx* c = new mi_ctx();
+  c->cfg = k;
+  int maxb = k.max_model_len;
+  for (int i = 0; i < k.num_ctx_buckets && i < 8; ++i) maxb = std::max(maxb, k.ctx_buckets[i]);
+  c->max_rows = std::max(maxb, k.max_num_seqs);
+  int rc = hipStreamCreateWithFlags(&c->stream, hipStreamNonBlocking) == hipSuccess ? MI_OK : MI_EHIP;
+  if (rc == MI_OK) rc = stack_create(c, t);
+  if (rc != MI_OK) {
+    const std::string keep = mi::g_err;
+    mi_ctx_destroy(c);
+    set_error(keep);
+    return rc;
+  }
+  *out = c;
+  return MI_OK;
+}
+
 int mi_ctx_destroy(mi_ctx* c) {
   if (!c) return MI_OK;
   if (c->owned_group) {
@@ -710,6 +758,7 @@ int mi_ctx_destroy(mi_ctx* c) {
   for (auto& kv : c->graphs) hipGraphExecDestroy(kv.second);
   if (c->comm) ncclCommDestroy(c->comm);
   if (c->grp && c->grp->lockstep && c->cfg.tp_rank != 0) hipStreamSynchronize(c->stream);
+  if (c->stack) stack_destroy(c);
   auto fl = [](Linear& L) { hipFree(L.w); hipFree(L.scale); hipFree(L.bias); };
   for (auto& W : c->layers) { fl(W.qkv); fl(W.o); fl(W.gu); fl(W.down); hipFree(W.g_in); hipFree(W.g_post); }
   fl(c->lm_head);
@@ -737,6 +786,13 @@ int mi_load_weight(mi_ctx* c, const char* name_c, const void* host, int32_t dtyp
     std::vector<float> v((size_t)shape[0]);
     if (dtype == MI_F32) memcpy(v.data(), host, v.size() * 4);
     else for (size_t i = 0; i < v.size(); ++i) v[i] = bf16_bits_to_f32(reinterpret_cast<const uint16_t*>(host)[i]);
+    if (c->stack) {
+      MI_TRY(ensure_stage(c, v.size(), 1));
+      MI_HIP(hipMemcpyAsync(c->stage_f32, v.data(), v.size() * 4, hipMemcpyHostToDevice, c->stream));
+      MI_TRY(stack_load_tensor(c, name, c->stage_f32, (int)v.size(), 0));
+      MI_HIP(hipStreamSynchronize(c->stream));
+      return MI_OK;
+    }
     return route_vector(c, name, v);
   }
   const size_t elems = (size_t)shape[0] * (size_t)shape[1];
@@ -747,7 +803,8 @@ int mi_load_weight(mi_ctx* c, const char* name_c, const void* host, int32_t dtyp
     MI_HIP(hipMemcpyAsync(c->stage_raw, host, elems * 2, hipMemcpyHostToDevice, c->stream));
     MI_TRY(launch_bf16_to_f32(reinterpret_cast<const uint16_t*>(c->stage_raw), c->stage_f32, elems, c->stream));
   }
-  MI_TRY(route_matrix(c, name, c->stage_f32, (int)shape[0], (int)shape[1]));
+  if (c->stack) MI_TRY(stack_load_tensor(c, name, c->stage_f32, (int)shape[0], (int)shape[1]));
+  else MI_TRY(route_matrix(c, name, c->stage_f32, (int)shape[0], (int)shape[1]));
   MI_HIP(hipStreamSynchronize(c->stream));  // the host buffer / staging may be reused by the caller
   return MI_OK;
 }
@@ -758,6 +815,7 @@ int mi_init_synthetic_weights(mi_ctx* c, uint64_t seed, float std) {
     return group_run(c->owned_group, [&](mi_ctx* rc, int) { return mi_init_synthetic_weights(rc, seed, std); });
   MI_CHECK(!c->finalized, "bad state");
   MI_HIP(hipSetDevice(c->cfg.device_id));
+  if (c->stack) return stack_synthetic(c, seed, std);
   const mi_model_config& k = c->cfg;
   uint64_t tid = 1;
   auto gen = [&](const std::string& name, int rows, int cols, float sd) -> int {
@@ -824,10 +882,12 @@ void make_header(const mi_ctx* c, ArtifactHeader& h) {
   memcpy(h.geo, g, sizeof g);
   h.weight_dtype = k.weight_dtype; h.quant_type = k.quant_type; h.quantize_lm_head = k.quantize_lm_head;
   h.tp_degree = k.tp_degree; h.tp_rank = k.tp_rank;
+  if (c->stack) h.geo[8] = -1 - stack_geometry_hash(c);   // (negative: never the tie flag of a Llama-family file)
 }
 
 // every device tensor of a rank, in file order
 void artifact_tensors(mi_ctx* c, std::vector<std::pair<void*, size_t>>& out) {
+  if (c->stack) return stack_artifact_tensors(c, out);
   auto lin = [&](Linear& L) {
     out.push_back({L.w, L.bytes()});
     out.push_back({L.scale, (size_t)L.N * 4});
@@ -852,7 +912,7 @@ constexpr size_t kArtifactChunk = (size_t)64 << 20;
 int mi_save_weights(mi_ctx* c, const char* dir) {
   MI_CHECK(c && dir, "null argument");
   if (c->owned_group) return group_run(c->owned_group, [&](mi_ctx* rc, int) { return mi_save_weights(rc, dir); });
-  MI_CHECK(c->have_lm_head, "mi_save_weights: the weights are not loaded yet");
+  MI_CHECK(c->stack ? c->stack->missing.empty() : c->have_lm_head, "mi_save_weights: the weights are not loaded yet");
   MI_HIP(hipSetDevice(c->cfg.device_id));
   std::string path;
   artifact_file(c, dir, path);
@@ -919,6 +979,7 @@ int mi_load_weights_file(mi_ctx* c, const char* dir) {
   fclose(f);
   if (!ok) { set_error("weight artifacts at " + path + " are truncated or do not match this context's tensors"); return MI_EINVAL; }
   c->have_lm_head = true;
+  if (c->stack) c->stack->missing.clear();
   return MI_OK;
 }
 
@@ -937,6 +998,7 @@ int mi_set_num_blocks(mi_ctx* c, int32_t num_blocks) {
 // bytes mi_finalize allocates besides the KV pool (activations, exchange buffers, scratch): what
 // has to be kept out of the memory offered to vLLM for KV blocks
 static size_t workspace_estimate(const mi_ctx* c) {
+  if (c->stack) return stack_workspace_estimate(c);
   const mi_model_config& k = c->cfg;
   const size_t R = (size_t)c->max_rows, H = (size_t)c->H;
   size_t b = 3 * R * H * 4 + R * std::max<size_t>(H, c->I_l) * 2 + 2 * R * c->q_dim * 2 + R * c->I_l * 2;
@@ -952,6 +1014,7 @@ static size_t workspace_estimate(const mi_ctx* c) {
 int64_t mi_kv_bytes_per_block(mi_ctx* c) {
   if (!c) return 0;
   if (c->owned_group) c = c->owned_group->ranks[0];
+  if (c->stack) return (int64_t)stack_kv_bytes_per_block(c);
   return (int64_t)c->cfg.num_layers * 2 * c->nkv_l * c->cfg.block_size * c->hd * 2;
 }
 
@@ -965,7 +1028,7 @@ int mi_finalize(mi_ctx* c) {
     return MI_OK;
   }
   MI_CHECK(!c->finalized, "bad state");
-  MI_CHECK(c->have_lm_head, "lm_head.weight (or tied embed_tokens) was never loaded");
+  MI_CHECK(c->stack || c->have_lm_head, "lm_head.weight (or tied embed_tokens) was never loaded");
   MI_CHECK(c->cfg.tp_degree == 1 || c->collective(), "tp_degree > 1: call mi_tp_init before mi_finalize");
   const mi_model_config& k = c->cfg;
   MI_HIP(hipSetDevice(k.device_id));
@@ -973,6 +1036,11 @@ int mi_finalize(mi_ctx* c) {
   if (c->stage_raw) { hipFree(c->stage_raw); c->stage_raw = nullptr; }
   if (c->stage_f32) { hipFree(c->stage_f32); c->stage_f32 = nullptr; }
   c->stage_elems = 0;
+  const size_t R = (size_t)c->max_rows;
+  size_t* ws = &c->workspace_bytes;
+  if (c->stack) {
+    MI_TRY(stack_alloc(c));
+  } else {
   // KV pool, zero-filled: stale or never-written rows must hold finite values
   c->kv_half = (size_t)k.num_blocks * c->nkv_l * k.block_size * c->hd;
   const size_t kv_elems = c->kv_half * 2 * k.num_layers;
@@ -1020,8 +1088,6 @@ int mi_finalize(mi_ctx* c) {
     MI_HIP(hipMemcpyAsync(c->rope_sin, sn.data(), sn.size() * 4, hipMemcpyHostToDevice, s));
     MI_HIP(hipStreamSynchronize(s));
   }
-  const size_t R = (size_t)c->max_rows;
-  size_t* ws = &c->workspace_bytes;
   MI_TRY(dmalloc(&c->resid[0], R * c->H, ws));
   MI_TRY(dmalloc(&c->resid[1], R * c->H, ws));
   MI_TRY(dmalloc(&c->partial, R * c->H, ws));
@@ -1033,17 +1099,21 @@ int mi_finalize(mi_ctx* c) {
     MI_TRY(dmalloc(&c->x8, R * std::max(std::max(c->H, c->I_l), c->q_dim), ws));
     MI_TRY(dmalloc(&c->x8_scale, R, ws));
   }
+  }
   c->splitk_ws_bytes = (size_t)64 << 20;   // fp32 K-slice slabs of the short-prompt GEMMs
   MI_TRY(dmalloc(&c->splitk_ws, c->splitk_ws_bytes / 4, ws));
   MI_TRY(dmalloc(&c->logits, (size_t)k.max_num_seqs * c->V_l, ws));
   if (c->collective()) MI_TRY(dmalloc(&c->logits_all, (size_t)k.tp_degree * k.max_num_seqs * c->V_l, ws));
-  MI_HIP(hipMalloc(&c->attn_scratch, attn_scratch_bytes(k.max_num_seqs, c->nh_l, c->hd)));
-  MI_HIP(hipMemsetAsync(c->attn_scratch, 0, attn_scratch_bytes(k.max_num_seqs, c->nh_l, c->hd), s));   // incl. the merge tickets
-  *ws += attn_scratch_bytes(k.max_num_seqs, c->nh_l, c->hd);
+  if (!c->stack) {
+    MI_HIP(hipMalloc(&c->attn_scratch, attn_scratch_bytes(k.max_num_seqs, c->nh_l, c->hd)));
+    MI_HIP(hipMemsetAsync(c->attn_scratch, 0, attn_scratch_bytes(k.max_num_seqs, c->nh_l, c->hd), s));   // incl. the merge tickets
+    *ws += attn_scratch_bytes(k.max_num_seqs, c->nh_l, c->hd);
+  }
   c->MB_cap = ceil_div(k.max_model_len, k.block_size) + 1;
   const size_t nbt = (size_t)k.max_num_seqs * c->MB_cap;
   // inputs: [block tables][context lengths][ids][positions][slots], one block on each side
-  c->inputs_elems = nbt + (size_t)k.max_num_seqs + 3 * R + (size_t)k.max_num_seqs;   // [tables][per-request ints][ids][pos][slots][per-request context lengths]
+  // [tables][per-request ints][ids][pos][slots][per-request context lengths][per-request segments, 16-byte aligned]
+  c->inputs_elems = ((nbt + 2 * (size_t)k.max_num_seqs + 3 * R + 3) & ~(size_t)3) + 4 * (size_t)k.max_num_seqs;
   MI_TRY(dmalloc(&c->d_inputs, c->inputs_elems, ws));
   MI_HIP(hipHostMalloc(reinterpret_cast<void**>(&c->h_inputs), c->inputs_elems * 4, hipHostMallocDefault));
   memset(c->h_inputs, 0, c->inputs_elems * 4);
@@ -1100,6 +1170,7 @@ static void set_input_views(mi_ctx* c, bool decode_step) {
     c->d_bt = c->d_inputs; c->d_ctx = c->d_inputs + nbt; c->d_ids = c->d_ctx + ms; c->d_pos = c->d_ids + R; c->d_slots = c->d_pos + R;
     c->h_bt = c->h_inputs; c->h_ctx = c->h_inputs + nbt; c->h_ids = c->h_ctx + ms; c->h_pos = c->h_ids + R; c->h_slots = c->h_pos + R;
     c->d_seg_ctx = c->d_slots + R; c->h_seg_ctx = c->h_slots + R;
+    c->d_segs = c->d_inputs + c->inputs_elems - 4 * ms; c->h_segs = c->h_inputs + c->inputs_elems - 4 * ms;
   }
 }
 
@@ -1291,6 +1362,8 @@ static int forward_impl(mi_ctx* c, int32_t B, int32_t S, const int64_t* input_id
       c->h_slots[t] = (int32_t)slot;
     }
     for (int j = 0; j < MB; ++j) c->h_bt[j] = (int32_t)block_table[(size_t)b * MB + j];
+    c->h_seg_ctx[0] = full;
+    memcpy(c->h_segs, std::array<int32_t, 4>{0, n_new, comp, 0}.data(), 16);
     MI_TRY(push_inputs());
     MI_TRY(run_layers(c, n_new, false, 1, MB, comp, 1, n_new - 1));
     // (the copy engine reads the pinned block asynchronously: the next row's staging must not
@@ -1319,33 +1392,25 @@ int mi_forward_tokens(mi_ctx* c, int32_t B, int32_t S, const int64_t* input_ids,
                       computed_context_lens, nullptr, sampling_params, seed, tokens_out);
 }
 
-int mi_forward_chunked(mi_ctx* c, int32_t n_req, int32_t total, const int64_t* input_ids, const int64_t* position_ids,
-                       const int64_t* slot_mapping, const int64_t* block_table, int32_t MB,
-                       const int64_t* full_context_lens, const int64_t* computed_context_lens, float* logits_out,
-                       const float* sampling_params, uint64_t seed, int64_t* tokens_out) {
-  if (c && c->owned_group)
-    return group_run(c->owned_group, [&](mi_ctx* rc, int) {
-      return mi_forward_chunked(rc, n_req, total, input_ids, position_ids, slot_mapping, block_table, MB, full_context_lens,
-                                computed_context_lens, logits_out, sampling_params, seed, tokens_out);
-    });
-  MI_CHECK(c && c->finalized, "mi_forward_chunked before mi_finalize");
-  MI_CHECK(input_ids && position_ids && slot_mapping && block_table && full_context_lens && computed_context_lens, "null argument");
-  MI_CHECK((logits_out != nullptr) != (tokens_out != nullptr), "exactly one of logits_out / tokens_out");
+// A ragged batch through the trunk: checks, staging, one input copy, the layers.
+static int ragged_check(mi_ctx* c, int32_t n_req, int32_t total, int32_t MB, const int64_t* full_context_lens,
+                        const int64_t* computed_context_lens, bool* one_each) {
   const mi_model_config& k = c->cfg;
   MI_CHECK(n_req >= 1 && n_req <= k.max_num_seqs, "more requests than max_num_seqs");
   MI_CHECK(total >= n_req && total <= c->max_rows, "token batch larger than the largest context-encoding bucket");
   MI_CHECK(MB >= 1 && MB <= c->MB_cap, "bad block-table width");
   static const bool decode_shortcut = [] { const char* v = getenv("MI355X_CHUNKED_DECODE_SHORTCUT"); return !v || v[0] != '0'; }();
-  if (decode_shortcut && total == n_req) {
-    // every request contributes exactly one token: this IS a token-generation step (vLLM's native scheduler
-    // sends those through the same ragged record once all prompts are encoded) -- the weight-streaming
-    // kernels, the split-context attention and the step's hipGraph instead of a 1-row context encoding per request
-    bool one_each = true;
-    for (int i = 0; i < n_req; ++i) one_each = one_each && full_context_lens[i] - computed_context_lens[i] == 1;
-    if (one_each)
-      return forward_impl(c, n_req, 1, input_ids, position_ids, nullptr, block_table, MB, slot_mapping, 1, full_context_lens,
-                          computed_context_lens, logits_out, sampling_params, seed, tokens_out);
-  }
+  // every request contributes exactly one token: this IS a token-generation step (vLLM's native scheduler
+  // sends those through the same ragged record once all prompts are encoded) -- the weight-streaming
+  // kernels, the split-context attention and the step's hipGraph instead of a 1-row context encoding per request
+  *one_each = decode_shortcut && total == n_req;
+  for (int i = 0; *one_each && i < n_req; ++i) *one_each = full_context_lens[i] - computed_context_lens[i] == 1;
+  return MI_OK;
+}
+static int ragged_trunk(mi_ctx* c, int32_t n_req, int32_t total, const int64_t* input_ids, const int64_t* position_ids,
+                        const int64_t* slot_mapping, const int64_t* block_table, int32_t MB,
+                        const int64_t* full_context_lens, const int64_t* computed_context_lens) {
+  const mi_model_config& k = c->cfg;
   MI_HIP(hipSetDevice(k.device_id));
   hipStream_t s = c->stream;
   const int bs = k.block_size, V = k.vocab_size;
@@ -1372,17 +1437,92 @@ int mi_forward_chunked(mi_ctx* c, int32_t n_req, int32_t total, const int64_t* i
       c->h_pos[row + t] = (int32_t)pos;
       c->h_slots[row + t] = (int32_t)slot;
     }
-    segs[i] = Seg{row, n, comp};
+    segs[i] = Seg{row, n, comp, i};
     c->h_ctx[i] = row + n - 1;   // the request's last row: where its logits come from
     c->h_seg_ctx[i] = full;      // keys the request attends to (the decode-attention launch of 1-token requests)
     row += n;
   }
   MI_CHECK(row == total, "chunk lengths do not add up to the token batch");
+  memcpy(c->h_segs, segs.data(), (size_t)n_req * sizeof(Seg));
   MI_HIP(hipMemcpyAsync(c->d_inputs, c->h_inputs, c->inputs_elems * 4, hipMemcpyHostToDevice, s));
-  MI_TRY(run_layers(c, total, false, 1, MB, 0, n_req, 0, segs.data(), n_req));
+  return run_trunk(c, total, false, 1, MB, 0, segs.data(), n_req);
+}
+
+int mi_forward_chunked(mi_ctx* c, int32_t n_req, int32_t total, const int64_t* input_ids, const int64_t* position_ids,
+                       const int64_t* slot_mapping, const int64_t* block_table, int32_t MB,
+                       const int64_t* full_context_lens, const int64_t* computed_context_lens, float* logits_out,
+                       const float* sampling_params, uint64_t seed, int64_t* tokens_out) {
+  if (c && c->owned_group)
+    return group_run(c->owned_group, [&](mi_ctx* rc, int) {
+      return mi_forward_chunked(rc, n_req, total, input_ids, position_ids, slot_mapping, block_table, MB, full_context_lens,
+                                computed_context_lens, logits_out, sampling_params, seed, tokens_out);
+    });
+  MI_CHECK(c && c->finalized, "mi_forward_chunked before mi_finalize");
+  MI_CHECK(input_ids && position_ids && slot_mapping && block_table && full_context_lens && computed_context_lens, "null argument");
+  MI_CHECK((logits_out != nullptr) != (tokens_out != nullptr), "exactly one of logits_out / tokens_out");
+  bool one_each = false;
+  MI_TRY(ragged_check(c, n_req, total, MB, full_context_lens, computed_context_lens, &one_each));
+  if (one_each)
+    return forward_impl(c, n_req, 1, input_ids, position_ids, nullptr, block_table, MB, slot_mapping, 1, full_context_lens,
+                        computed_context_lens, logits_out, sampling_params, seed, tokens_out);
+  MI_TRY(ragged_trunk(c, n_req, total, input_ids, position_ids, slot_mapping, block_table, MB, full_context_lens, computed_context_lens));
+  MI_TRY(run_head(c, n_req, 0, true));
   if (tokens_out) MI_TRY(sample_on_device(c, n_req, 0, sampling_params, seed, tokens_out));
   else MI_TRY(fetch_logits(c, n_req, logits_out));
   return prof_collect(c);
+}
+
+int mi_forward_rows(mi_ctx* c, int32_t n_req, int32_t total, const int64_t* input_ids, const int64_t* position_ids,
+                    const int64_t* slot_mapping, const int64_t* block_table, int32_t MB, const int64_t* full_context_lens,
+                    const int64_t* computed_context_lens, int32_t n_rows, const int64_t* rows, float* logits_out) {
+  if (c && c->owned_group)
+    return group_run(c->owned_group, [&](mi_ctx* rc, int) {
+      return mi_forward_rows(rc, n_req, total, input_ids, position_ids, slot_mapping, block_table, MB, full_context_lens,
+                             computed_context_lens, n_rows, rows, logits_out);
+    });
+  MI_CHECK(c && c->finalized, "mi_forward_rows before mi_finalize");
+  MI_CHECK(input_ids && position_ids && slot_mapping && block_table && full_context_lens && computed_context_lens, "null argument");
+  MI_CHECK(n_rows >= 0 && (n_rows == 0 || (rows && logits_out)), "null argument");
+  for (int i = 0; i < n_rows; ++i) MI_CHECK(rows[i] >= 0 && rows[i] < total, "logits row outside the token batch");
+  bool one_each = false;
+  MI_TRY(ragged_check(c, n_req, total, MB, full_context_lens, computed_context_lens, &one_each));
+  const size_t V = (size_t)c->cfg.vocab_size, ms = (size_t)c->cfg.max_num_seqs;
+  if (one_each && !c->grp) {   // (a rank shard fills its columns of the caller's rows itself: no detour through a copy)
+    std::vector<float> all((size_t)n_req * V);
+    MI_TRY(forward_impl(c, n_req, 1, input_ids, position_ids, nullptr, block_table, MB, slot_mapping, 1, full_context_lens,
+                        computed_context_lens, all.data(), nullptr, 0, nullptr));
+    for (int i = 0; i < n_rows; ++i) memcpy(logits_out + (size_t)i * V, all.data() + (size_t)rows[i] * V, V * 4);
+    return MI_OK;
+  }
+  MI_TRY(ragged_trunk(c, n_req, total, input_ids, position_ids, slot_mapping, block_table, MB, full_context_lens, computed_context_lens));
+  for (int i0 = 0; i0 < n_rows; i0 += (int)ms) {   // the head and its buffers hold max_num_seqs rows at a time
+    const int n = std::min((int)ms, n_rows - i0);
+    MI_HIP(hipStreamSynchronize(c->stream));       // the pinned list behind d_ctx is free to be rewritten
+    for (int i = 0; i < n; ++i) c->h_ctx[i] = (int32_t)rows[i0 + i];
+    MI_HIP(hipMemcpyAsync(c->d_ctx, c->h_ctx, (size_t)n * 4, hipMemcpyHostToDevice, c->stream));
+    MI_TRY(run_head(c, n, 0, true));
+    MI_TRY(fetch_logits(c, n, logits_out + (size_t)i0 * V));
+  }
+  MI_HIP(hipStreamSynchronize(c->stream));
+  return prof_collect(c);
+}
+
+int mi_layer_residuals(mi_ctx* c, int32_t on) {
+  MI_CHECK(c && c->finalized && c->stack, "mi_layer_residuals: a finalized layer-stack context");
+  MI_HIP(hipSetDevice(c->cfg.device_id));
+  Stack* S = c->stack;
+  MI_HIP(hipStreamSynchronize(c->stream));
+  if (on && !S->residuals) MI_HIP(hipMalloc(reinterpret_cast<void**>(&S->residuals), S->runs.size() * c->max_rows * (size_t)S->ld * 4));
+  if (!on && S->residuals) { hipFree(S->residuals); S->residuals = nullptr; }
+  return MI_OK;
+}
+int mi_layer_residuals_read(mi_ctx* c, int32_t rows, float* out) {
+  MI_CHECK(c && c->stack && c->stack->residuals && out && rows >= 1 && rows <= c->max_rows, "mi_layer_residuals_read: not switched on, or bad rows");
+  Stack* S = c->stack;
+  MI_HIP(hipStreamSynchronize(c->stream));
+  for (size_t i = 0; i < S->runs.size(); ++i)
+    MI_HIP(hipMemcpy2D(out + i * rows * (size_t)S->D, (size_t)S->D * 4, S->residuals + i * c->max_rows * S->ld, (size_t)S->ld * 4, (size_t)S->D * 4, rows, hipMemcpyDeviceToHost));
+  return MI_OK;
 }
 
 // Fused speculation: k chained token-generation steps of the DRAFT context (its greedy token feeds its
@@ -1793,6 +1933,61 @@ int mi_op_qlinear_a8(const void* x, int32_t M, const void* w_tiled, const float*
   hipStreamSynchronize(s);
   hipFree(x8);
   hipFree(xs);
+  return rc;
+}
+static HeadGeom head_geom(const mi_layer_spec& p) {
+  return HeadGeom{p.num_heads, p.num_kv_heads, p.qk_dim, p.v_dim, (p.qk_dim + 15) / 16 * 16, (p.v_dim + 15) / 16 * 16};
+}
+int mi_op_layernorm2(const float* x, int32_t T, int32_t D, int32_t ld, float eps, const float* w1, const float* b1, void* y1,
+                     const float* w2, const float* b2, void* y2, int32_t ldy, int32_t f32, void* stream) {
+  MI_CHECK(x && w1 && b1 && y1 && (!y2 || (w2 && b2)) && T >= 1, "null argument");
+  return launch_layernorm_rows(x, nullptr, T, D, ld, eps, NormOut{w1, b1, y1}, NormOut{w2, b2, y2}, ldy, f32 != 0, (hipStream_t)stream);
+}
+int mi_op_embed_pos(const int32_t* ids, const int32_t* pos, const void* table, const void* ptable, int32_t T, int32_t D, int32_t ld,
+                    float* resid, float* x0, int32_t f32, void* stream) {
+  MI_CHECK(ids && pos && table && ptable && resid && T >= 1 && ld >= D, "bad argument");
+  return launch_embed_pos(ids, pos, table, ptable, f32 != 0, T, D, ld, resid, x0, (hipStream_t)stream);
+}
+int mi_op_qkv_scatter(const float* qkv, int32_t ldq, int32_t T, const mi_layer_spec* spec, float eps, const int32_t* slots,
+                      int32_t block_size, void* q, void* kpool, void* vpool, int32_t f32, void* stream) {
+  MI_CHECK(qkv && spec && slots && q && kpool && vpool && T >= 1, "null argument");
+  return launch_qkv_scatter(qkv, ldq, T, head_geom(*spec), spec->qk_unit_norm != 0, eps, slots, block_size, q, kpool, vpool, f32 != 0, (hipStream_t)stream);
+}
+int mi_op_window_attn(const mi_layer_spec* spec, const float* slopes, const void* q, const void* kpool, const void* vpool,
+                      int32_t block_size, const int32_t* block_table, int32_t MB, const int32_t* pos, const int32_t* ctx_lens,
+                      const int32_t* segs_host, int32_t nseg, int32_t T, int32_t max_ctx, void* out, int32_t ldo, int32_t f32,
+                      int32_t path, void* stream) {
+  MI_CHECK(spec && q && kpool && vpool && block_table && pos && ctx_lens && segs_host && out && nseg >= 1 && T >= 1, "null argument");
+  MI_CHECK(!spec->distance_bias || slopes, "distance bias without slopes");
+  const AttnSpec a{head_geom(*spec), spec->scale, spec->window, spec->distance_bias ? slopes : nullptr, spec->softmax_sink ? 1 : 0};
+  std::vector<AttnSeg> segs((size_t)nseg);
+  memcpy(segs.data(), segs_host, (size_t)nseg * sizeof(AttnSeg));
+  int row = 0;
+  for (const AttnSeg& g : segs) {
+    MI_CHECK(g.row0 == row && g.n >= 1 && g.pos0 >= 0 && ceil_div(g.pos0 + g.n, block_size) <= MB && g.pos0 + g.n <= max_ctx, "segments: contiguous rows, contexts within the block table");
+    row += g.n;
+  }
+  MI_CHECK(row == T, "segments do not add up to the rows");
+  hipStream_t s = (hipStream_t)stream;
+  AttnSeg* sd = nullptr;
+  void* scratch = nullptr;
+  MI_HIP(hipMalloc(reinterpret_cast<void**>(&sd), (size_t)nseg * sizeof(AttnSeg)));
+  MI_HIP(hipMalloc(&scratch, attn_window_scratch_bytes(nseg, a.g)));
+  MI_HIP(hipMemcpyAsync(sd, segs.data(), (size_t)nseg * sizeof(AttnSeg), hipMemcpyHostToDevice, s));
+  int rc = MI_OK;
+  if (f32 || path == 1 || !attn_window_supported(a.g)) {
+    rc = launch_attn_plain(a, q, kpool, vpool, block_size, block_table, MB, pos, sd, nseg, T, out, ldo, f32 != 0, s);
+  } else {
+    const uint16_t *qb = (const uint16_t*)q, *kb = (const uint16_t*)kpool, *vb = (const uint16_t*)vpool;
+    rc = launch_attn_window_prefill(a, qb, kb, vb, block_size, block_table, MB, sd, segs.data(), nseg, (uint16_t*)out, ldo, s);
+    for (int i = 0; i < nseg && rc == MI_OK; ++i)
+      if (segs[i].n == 1)
+        rc = launch_attn_window_decode(a, qb + (size_t)segs[i].row0 * a.g.H * a.g.dkp, kb, vb, block_size, block_table + (size_t)segs[i].seq * MB, MB,
+                                       ctx_lens + segs[i].seq, 1, max_ctx, (uint16_t*)out + (size_t)segs[i].row0 * ldo, ldo, scratch, s);
+  }
+  hipStreamSynchronize(s);
+  hipFree(sd);
+  hipFree(scratch);
   return rc;
 }
 int mi_op_rmsnorm(const float* x, const float* g, int32_t T, int32_t H, float eps, void* y, void* stream) {

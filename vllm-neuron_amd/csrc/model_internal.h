@@ -38,6 +38,7 @@ struct Prof {
 }  // namespace mi
 
 struct mi_group;
+namespace mi { struct Stack; }   // stack.h: the layer-stack decoders
 
 using mi::LayerW;
 using mi::Linear;
@@ -122,6 +123,36 @@ struct mi_ctx {
   mi_group* grp = nullptr;
   mi_group* owned_group = nullptr;
   bool stream_owned = true;
+  // a layer-stack decoder (stack.hip) in place of the Llama-family layers above
+  mi::Stack* stack = nullptr;
+  // ragged batches: (first row, rows, first position, block-table row) of every request
+  int32_t *d_segs = nullptr, *h_segs = nullptr;
+  // where the trunk left the residual stream for the final norm + lm_head (run_head)
+  int tail_cur = 0;
+  bool tail_partial = false;
   bool collective() const { return comm != nullptr || xport_allreduce != nullptr || grp != nullptr; }
 };
 
+namespace mi {
+// ---- profiling wrapper ---------------------------------------------------------------------
+struct Scope {
+  mi_ctx* c;
+  int cls;
+  hipEvent_t a = nullptr, b = nullptr;
+  Scope(mi_ctx* c_, int cls_) : c(c_), cls(cls_) {
+    if (c->prof.on) {
+      hipEventCreate(&a);
+      hipEventCreate(&b);
+      hipEventRecord(a, c->stream);
+    }
+  }
+  ~Scope() {
+    if (c->prof.on) {
+      hipEventRecord(b, c->stream);
+      c->prof.ev.push_back(a);
+      c->prof.ev.push_back(b);
+      c->prof.cls.push_back(cls);
+    }
+  }
+};
+}  // namespace mi

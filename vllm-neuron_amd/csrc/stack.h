@@ -1,0 +1,64 @@
+// Layer-stack decoders behind the same context, KV addressing and model calls as the Llama-family layers of model.hip:
+// what mi_ctx_create_stack adds to an mi_ctx.
+#pragma once
+#include <string>
+#include <vector>
+
+#include "model_internal.h"
+#include "window_attn.h"
+
+namespace mi {
+
+struct StackMat {   // a projection in the compute type: 16-row bf16 tiles (Linear) or row-major fp32
+  Linear L;
+  int N = 0, K = 0;   // padded: N % 16 == 0, K % 64 == 0
+};
+struct StackNorm { float *w = nullptr, *b = nullptr; };   // [ld], zero beyond the width
+
+struct StackLayer {
+  mi_layer_spec s{};
+  HeadGeom g;
+  AttnSpec attn;
+  int attn_cols = 0, ff_cols = 0;   // columns of the concatenated output projection's input: [heads x v_dim | feed-forward]
+  StackMat qkv, up, out;            // out = residual_mult [W_o | W_down]
+  StackNorm n1, n2;
+  float* slopes = nullptr;
+};
+struct StackRun { int layer; bool pass_start; };   // pass_start: the looped layers' input projection runs first
+
+struct Stack {
+  mi_stack_config cfg{};
+  std::vector<StackLayer> layers;
+  std::vector<StackRun> runs;
+  bool f32 = false;
+  int D = 0, ld = 0, Kd = 0;          // width; residual row stride (multiple of 16); activation row stride (multiple of 64)
+  void *embed = nullptr, *pos = nullptr;
+  StackMat loop_in, head;
+  StackNorm final_norm;
+  std::vector<size_t> kv_at;          // pool offset (elements) of every run's K; its V follows
+  std::vector<std::string> missing;   // tensors not loaded yet
+  // activations
+  float *x0 = nullptr, *qkv_out = nullptr, *logits_pad = nullptr;
+  void *n1 = nullptr, *n2 = nullptr, *q = nullptr, *cat = nullptr, *pair = nullptr;
+  int qkv_ld = 0, q_cols = 0, cat_ld = 0;
+  void* attn_scratch = nullptr;
+  SlabSum pend;                        // K-split sum of the last output projection, left for the next norm
+  float* residuals = nullptr;          // mi_layer_residuals: [runs][max_rows][ld]
+  size_t elem() const { return f32 ? 4 : 2; }
+};
+
+int stack_create(mi_ctx* c, const mi_stack_config& cfg);      // geometry + weight images (zeroed)
+void stack_destroy(mi_ctx* c);
+int stack_load_tensor(mi_ctx* c, const std::string& name, const float* dev, int rows, int cols);   // cols 0: a vector of `rows`
+int stack_synthetic(mi_ctx* c, uint64_t seed, float std);
+void stack_artifact_tensors(mi_ctx* c, std::vector<std::pair<void*, size_t>>& out);
+int stack_geometry_hash(const mi_ctx* c);
+size_t stack_kv_bytes_per_block(const mi_ctx* c);
+size_t stack_workspace_estimate(const mi_ctx* c);
+int stack_alloc(mi_ctx* c);                                    // KV pool + activations (mi_finalize)
+// the layers over `rows` rows; leaves the residual stream in c->resid[c->tail_cur]
+int stack_trunk(mi_ctx* c, int rows, bool decode, int MB, const AttnSeg* segs, int nseg);
+// final norm + head over nrows contiguous residual rows -> c->logits
+int stack_head(mi_ctx* c, const float* resid, int nrows);
+
+}  // namespace mi

@@ -1,0 +1,288 @@
+// Row-wise kernels of the layer-stack decoders.  See stack_kernels.h.
+#include "stack_kernels.h"
+
+#include "misc_kernels.h"
+
+namespace mi {
+
+namespace {
+
+__device__ __forceinline__ float to_f32(uint16_t v) { return bf16_to_f32(v); }
+__device__ __forceinline__ float to_f32(float v) { return v; }
+__device__ __forceinline__ void put4(uint16_t* p, float a, float b, float c, float d) {
+  *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf16x2(a, b), pack_bf16x2(c, d));
+}
+__device__ __forceinline__ void put4(float* p, float a, float b, float c, float d) { *reinterpret_cast<float4*>(p) = make_float4(a, b, c, d); }
+
+// sum over the work-group (256 threads); `red` has one float per wave and is free again after the next barrier
+__device__ __forceinline__ float block_sum(float v, float* red) {
+  v = wave_sum(v);
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+  __syncthreads();
+  return (red[0] + red[1]) + (red[2] + red[3]);
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void embed_pos_kernel(const int32_t* __restrict__ ids, const int32_t* __restrict__ pos,
+                                                        const T* __restrict__ table, const T* __restrict__ ptable, int D, int ld,
+                                                        float* __restrict__ resid, float* __restrict__ x0) {
+  const int t = blockIdx.x;
+  const T* e = table + (size_t)ids[t] * D;
+  const T* p = ptable + (size_t)pos[t] * D;
+  for (int d = threadIdx.x; d < ld; d += 256) {
+    const float v = d < D ? to_f32(e[d]) + to_f32(p[d]) : 0.f;
+    resid[(size_t)t * ld + d] = v;
+    if (x0) x0[(size_t)t * ld + d] = v;
+  }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void layernorm_rows_kernel(const float* __restrict__ resid_in, float* __restrict__ resid_out,
+                                                             int D, int ld, float eps, NormOut na, NormOut nb, int ldy, SlabSum sl) {
+  extern __shared__ __attribute__((aligned(16))) float hrow[];  // ld floats + 8
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const size_t o = (size_t)t * ld;
+  float* red = hrow + ld;
+  float sum = 0.f;
+  for (int c4 = tid; c4 < ld / 4; c4 += 256) {
+    float4 a = *reinterpret_cast<const float4*>(resid_in + o + c4 * 4);
+    if (sl.slab) {   // slabs in slice order, scale, + residual: the arithmetic of splitk_reduce + the residual epilogue
+      float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+      for (int z = 0; z < sl.KS; ++z) {
+        const float4 q = *reinterpret_cast<const float4*>(sl.slab + ((size_t)z * sl.T + t) * sl.N + c4 * 4);
+        v.x += q.x; v.y += q.y; v.z += q.z; v.w += q.w;
+      }
+      const float4 sc = *reinterpret_cast<const float4*>(sl.scale + c4 * 4);
+      a.x += v.x * sc.x; a.y += v.y * sc.y; a.z += v.z * sc.z; a.w += v.w * sc.w;
+      *reinterpret_cast<float4*>(resid_out + o + c4 * 4) = a;
+    }
+    *reinterpret_cast<float4*>(hrow + c4 * 4) = a;
+    sum += (a.x + a.y) + (a.z + a.w);     // columns beyond D are zero
+  }
+  const float mean = block_sum(sum, red) / (float)D;
+  float ss = 0.f;
+  for (int c4 = tid; c4 < ld / 4; c4 += 256) {   // (a thread reads back what it wrote itself)
+    float4 a = *reinterpret_cast<const float4*>(hrow + c4 * 4);
+    const int d = c4 * 4;
+    a.x = d < D ? a.x - mean : 0.f;
+    a.y = d + 1 < D ? a.y - mean : 0.f;
+    a.z = d + 2 < D ? a.z - mean : 0.f;
+    a.w = d + 3 < D ? a.w - mean : 0.f;
+    *reinterpret_cast<float4*>(hrow + c4 * 4) = a;
+    ss += (a.x * a.x + a.y * a.y) + (a.z * a.z + a.w * a.w);
+  }
+  const float rstd = 1.0f / sqrtf(block_sum(ss, red + 4) / (float)D + eps);
+  for (int c4 = tid; c4 < ld / 4; c4 += 256) {
+    const float4 a = *reinterpret_cast<const float4*>(hrow + c4 * 4);
+    auto emit = [&](const NormOut& n) {
+      const float4 w = *reinterpret_cast<const float4*>(n.w + c4 * 4), b = *reinterpret_cast<const float4*>(n.b + c4 * 4);
+      put4(reinterpret_cast<T*>(n.y) + (size_t)t * ldy + c4 * 4, a.x * rstd * w.x + b.x, a.y * rstd * w.y + b.y,
+           a.z * rstd * w.z + b.z, a.w * rstd * w.w + b.w);
+    };
+    if (na.y) emit(na);
+    if (nb.y) emit(nb);
+  }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void pair_rows_kernel(const float* __restrict__ x, const float* __restrict__ x0, int D4, int ld,
+                                                        int half, T* __restrict__ y) {
+  const int t = blockIdx.x;
+  T* row = y + (size_t)t * 2 * half;
+  for (int c4 = threadIdx.x; c4 < D4; c4 += 256) {
+    const float4 a = *reinterpret_cast<const float4*>(x + (size_t)t * ld + c4 * 4);
+    const float4 b = *reinterpret_cast<const float4*>(x0 + (size_t)t * ld + c4 * 4);
+    put4(row + c4 * 4, a.x, a.y, a.z, a.w);
+    put4(row + half + c4 * 4, b.x, b.y, b.z, b.w);
+  }
+}
+
+// 32 lanes per head: H q heads, G k heads, G v heads of one token row
+template <typename T>
+__global__ __launch_bounds__(256) void qkv_scatter_kernel(const float* __restrict__ qkv, int ldq, HeadGeom g, int unit_norm, float eps,
+                                                          const int32_t* __restrict__ slots, int bs, T* __restrict__ q,
+                                                          T* __restrict__ kpool, T* __restrict__ vpool) {
+  const int t = blockIdx.x, head = blockIdx.y * 8 + (threadIdx.x >> 5), l = threadIdx.x & 31;
+  if (head >= g.H + 2 * g.G) return;     // (whole 32-lane group: the shuffles below stay inside it)
+  const bool is_q = head < g.H, is_v = head >= g.H + g.G;
+  const int kvh = is_v ? head - g.H - g.G : head - g.H;
+  const int d_n = is_v ? g.dv : g.dk, d_p = is_v ? g.dvp : g.dkp;
+  const float* src = qkv + (size_t)t * ldq + (is_v ? (size_t)(g.H + g.G) * g.dk + (size_t)kvh * g.dv : (size_t)head * g.dk);
+  const bool vec = (d_n & 3) == 0 && (((is_v ? (g.H + g.G) * g.dk : 0)) & 3) == 0;
+  T* dst;
+  if (is_q) {
+    dst = q + ((size_t)t * g.H + head) * g.dkp;
+  } else {
+    const int slot = slots[t];
+    if (slot < 0) return;
+    const int blk = slot / bs, off = slot - blk * bs;
+    dst = (is_v ? vpool : kpool) + (((size_t)blk * g.G + kvh) * bs + off) * d_p;
+  }
+  auto get = [&](int d) -> float4 {
+    if (vec) return d < d_n ? *reinterpret_cast<const float4*>(src + d) : make_float4(0.f, 0.f, 0.f, 0.f);
+    return make_float4(d < d_n ? src[d] : 0.f, d + 1 < d_n ? src[d + 1] : 0.f, d + 2 < d_n ? src[d + 2] : 0.f, d + 3 < d_n ? src[d + 3] : 0.f);
+  };
+  float f = 1.f;
+  if (!is_v && unit_norm) {
+    float ss = 0.f;
+    for (int d = l * 4; d < d_n; d += 128) {
+      const float4 v = get(d);
+      ss += (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+    }
+#pragma unroll
+    for (int m = 16; m >= 1; m >>= 1) ss += __shfl_xor(ss, m);
+    f = 1.0f / sqrtf(ss / (float)d_n + eps);
+  }
+  for (int d = l * 4; d < d_p; d += 128) {
+    const float4 v = get(d);
+    put4(dst + d, v.x * f, v.y * f, v.z * f, v.w * f);
+  }
+}
+
+// 64 x 64 tile, 4 x 4 outputs per thread, fp32 FMAs: the 32-bit mode is for checking, not for speed
+template <int EPI>
+__global__ __launch_bounds__(256) void linear_f32_kernel(const float* __restrict__ w, int N, int K, const float* __restrict__ x, int ldx,
+                                                         int T, EpiArgs e) {
+  __shared__ float xs[16][68], ws[16][68];
+  const int n0 = blockIdx.x * 64, m0 = blockIdx.y * 64, tid = threadIdx.x;
+  const int tn = (tid & 15) * 4, tm = (tid >> 4) * 4, lr = tid >> 2, lk = (tid & 3) * 4;
+  float acc[4][4] = {};
+  for (int k0 = 0; k0 < K; k0 += 16) {
+    const float4 xv = *reinterpret_cast<const float4*>(x + (size_t)min(m0 + lr, T - 1) * ldx + k0 + lk);
+    const float4 wv = *reinterpret_cast<const float4*>(w + (size_t)min(n0 + lr, N - 1) * K + k0 + lk);
+    __syncthreads();
+    xs[lk][lr] = xv.x; xs[lk + 1][lr] = xv.y; xs[lk + 2][lr] = xv.z; xs[lk + 3][lr] = xv.w;
+    ws[lk][lr] = wv.x; ws[lk + 1][lr] = wv.y; ws[lk + 2][lr] = wv.z; ws[lk + 3][lr] = wv.w;
+    __syncthreads();
+#pragma unroll
+    for (int k = 0; k < 16; ++k)
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[i][j] = __builtin_fmaf(xs[k][tm + i], ws[k][tn + j], acc[i][j]);
+  }
+  if (n0 + tn >= N) return;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int m = m0 + tm + i;
+    if (m >= T) continue;
+    float v[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = acc[i][j] * e.scale[n0 + tn + j];
+    if constexpr (EPI == EPI_RELU2) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) { v[j] = fmaxf(v[j], 0.f); v[j] *= v[j]; }
+      put4(reinterpret_cast<float*>(e.act_out) + (size_t)m * e.ld_act + n0 + tn, v[0], v[1], v[2], v[3]);
+    } else {
+      if constexpr (EPI == EPI_RESID) {
+        const float4 r = *reinterpret_cast<const float4*>(e.resid_in + (size_t)m * e.ld_out + n0 + tn);
+        v[0] += r.x; v[1] += r.y; v[2] += r.z; v[3] += r.w;
+      }
+      put4(e.out_f32 + (size_t)m * e.ld_out + n0 + tn, v[0], v[1], v[2], v[3]);
+    }
+  }
+}
+
+__global__ void place_tiled_kernel(const float* __restrict__ src, int ld, int src_col0, int rows, int cols, uint16_t* __restrict__ dst,
+                                   int KT, int row0, int col0) {
+  const int c8n = (cols + 7) / 8;
+  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= (size_t)rows * c8n) return;
+  const int r = (int)(i / c8n), c = (int)(i % c8n) * 8;
+  const float* p = src + (size_t)r * ld + src_col0 + c;
+  float v[8];
+#pragma unroll
+  for (int k = 0; k < 8; ++k) v[k] = c + k < cols ? p[k] : 0.f;
+  const int R = row0 + r, C = col0 + c;
+  const size_t at = (((size_t)(R >> 4) * KT + (C >> 5)) * 64 + (R & 15) + 16 * ((C & 31) >> 3)) * 8;
+  *reinterpret_cast<uint4*>(dst + at) = make_uint4(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]), pack_bf16x2(v[4], v[5]), pack_bf16x2(v[6], v[7]));
+}
+__global__ void place_f32_kernel(const float* __restrict__ src, int ld, int src_col0, int rows, int cols, float* __restrict__ dst, int K,
+                                 int row0, int col0) {
+  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= (size_t)rows * cols) return;
+  const int r = (int)(i / cols), c = (int)(i % cols);
+  dst[(size_t)(row0 + r) * K + col0 + c] = src[(size_t)r * ld + src_col0 + c];
+}
+__global__ void pack_rows_kernel(const float* __restrict__ src, int ld_src, int V, float* __restrict__ dst) {
+  for (int v = blockIdx.x * blockDim.x + threadIdx.x; v < V; v += gridDim.x * blockDim.x)
+    dst[(size_t)blockIdx.y * V + v] = src[(size_t)blockIdx.y * ld_src + v];
+}
+
+}  // namespace
+
+int launch_embed_pos(const int32_t* ids, const int32_t* pos, const void* table, const void* ptable, bool f32, int T, int D,
+                     int ld, float* resid, float* x0, hipStream_t s) {
+  if (f32)
+    hipLaunchKernelGGL((embed_pos_kernel<float>), dim3(T), dim3(256), 0, s, ids, pos, (const float*)table, (const float*)ptable, D, ld, resid, x0);
+  else
+    hipLaunchKernelGGL((embed_pos_kernel<uint16_t>), dim3(T), dim3(256), 0, s, ids, pos, (const uint16_t*)table, (const uint16_t*)ptable, D, ld, resid, x0);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_layernorm_rows(const float* resid_in, float* resid_out, int T, int D, int ld, float eps, const NormOut& a,
+                          const NormOut& b, int ldy, bool f32, hipStream_t s, const SlabSum* slabs) {
+  MI_CHECK(ld % 4 == 0 && ld >= D && ld <= 32768 && ldy >= ld, "layer norm: row stride must be a multiple of 4, at least the width, at most 32768");
+  MI_CHECK(!slabs || (slabs->T == T && slabs->N == ld && resid_out && !slabs->bias && !slabs->row_scale), "layer norm: pending K-split sum of another shape");
+  const size_t lds = (size_t)(ld + 8) * sizeof(float);
+  const SlabSum sl = slabs ? *slabs : SlabSum();
+  if (lds > 64 * 1024)
+    MI_HIP(f32 ? hipFuncSetAttribute(reinterpret_cast<const void*>(layernorm_rows_kernel<float>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)
+               : hipFuncSetAttribute(reinterpret_cast<const void*>(layernorm_rows_kernel<uint16_t>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+  if (f32) hipLaunchKernelGGL((layernorm_rows_kernel<float>), dim3(T), dim3(256), lds, s, resid_in, resid_out, D, ld, eps, a, b, ldy, sl);
+  else hipLaunchKernelGGL((layernorm_rows_kernel<uint16_t>), dim3(T), dim3(256), lds, s, resid_in, resid_out, D, ld, eps, a, b, ldy, sl);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_pair_rows(const float* x, const float* x0, int T, int D, int ld, int half, void* y, bool f32, hipStream_t s) {
+  MI_CHECK(ld % 4 == 0 && half % 4 == 0 && half >= ld && ld >= D, "pair rows: strides");
+  if (f32) hipLaunchKernelGGL((pair_rows_kernel<float>), dim3(T), dim3(256), 0, s, x, x0, ld / 4, ld, half, (float*)y);
+  else hipLaunchKernelGGL((pair_rows_kernel<uint16_t>), dim3(T), dim3(256), 0, s, x, x0, ld / 4, ld, half, (uint16_t*)y);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_qkv_scatter(const float* qkv, int ldq, int T, const HeadGeom& g, bool unit_norm, float eps, const int32_t* slots,
+                       int block_size, void* q, void* kpool, void* vpool, bool f32, hipStream_t s) {
+  MI_CHECK(ldq % 4 == 0 && ldq >= (g.H + g.G) * g.dk + g.G * g.dv && g.dkp % 16 == 0 && g.dvp % 16 == 0 && g.dkp >= g.dk && g.dvp >= g.dv,
+           "qkv scatter: geometry");
+  const dim3 grid(T, ceil_div(g.H + 2 * g.G, 8));
+  if (f32) hipLaunchKernelGGL((qkv_scatter_kernel<float>), grid, dim3(256), 0, s, qkv, ldq, g, (int)unit_norm, eps, slots, block_size, (float*)q, (float*)kpool, (float*)vpool);
+  else hipLaunchKernelGGL((qkv_scatter_kernel<uint16_t>), grid, dim3(256), 0, s, qkv, ldq, g, (int)unit_norm, eps, slots, block_size, (uint16_t*)q, (uint16_t*)kpool, (uint16_t*)vpool);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_linear_f32(const float* w, int N, int K, const float* x, int ldx, int T, int epi, const EpiArgs& e, hipStream_t s) {
+  MI_CHECK(N % 16 == 0 && K % 16 == 0 && ldx % 4 == 0 && T >= 1, "linear_f32: N % 16 == 0, K % 16 == 0, ldx % 4 == 0");
+  const dim3 grid(ceil_div(N, 64), ceil_div(T, 64));
+  if (epi == EPI_F32) hipLaunchKernelGGL((linear_f32_kernel<EPI_F32>), grid, dim3(256), 0, s, w, N, K, x, ldx, T, e);
+  else if (epi == EPI_RESID) hipLaunchKernelGGL((linear_f32_kernel<EPI_RESID>), grid, dim3(256), 0, s, w, N, K, x, ldx, T, e);
+  else if (epi == EPI_RELU2) hipLaunchKernelGGL((linear_f32_kernel<EPI_RELU2>), grid, dim3(256), 0, s, w, N, K, x, ldx, T, e);
+  else { set_error("linear_f32: epilogue"); return MI_EINVAL; }
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_place(const float* src, int ld, int src_col0, int rows, int cols, void* dst, int K, bool f32, int row0, int col0, hipStream_t s) {
+  MI_CHECK(col0 % 8 == 0 && K % 64 == 0 && col0 + cols <= K && src_col0 + cols <= ld, "place: columns");
+  if (f32) {
+    const size_t n = (size_t)rows * cols;
+    hipLaunchKernelGGL(place_f32_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, src, ld, src_col0, rows, cols, (float*)dst, K, row0, col0);
+  } else {
+    const size_t n = (size_t)rows * ((cols + 7) / 8);
+    hipLaunchKernelGGL(place_tiled_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, src, ld, src_col0, rows, cols, (uint16_t*)dst, K / 32, row0, col0);
+  }
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_pack_rows(const float* src, int ld_src, int T, int V, float* dst, hipStream_t s) {
+  hipLaunchKernelGGL(pack_rows_kernel, dim3(ceil_div(V, 1024), T), dim3(256), 0, s, src, ld_src, V, dst);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+}  // namespace mi

@@ -1,0 +1,609 @@
+// Paged attention with a sliding window, distance bias and softmax sink.  See window_attn.h.
+//
+// MFMA forms: a column of the 16-wide MFMA tiles is one (query, head of the kv group) pair, column = query * r + head
+// with r = H / G, so the heads that share keys share the K / V tile, and a narrow window wastes little: a wave's columns
+// span few queries.  Scores are computed transposed (S^T = K.Q^T); the accumulator registers are then the B operand of
+// O^T += V^T.P^T as they stand, with V rows read transposed from LDS (ds_read_b64_tr_b16).  Scores, bias, softmax and
+// the sink are fp32 in the exp2 domain; the sink is the running state every column starts from (max 0, sum 1).
+
+#include "window_attn.h"
+
+namespace mi {
+
+namespace {
+
+typedef __attribute__((ext_vector_type(4))) short s16x4_t;
+constexpr float kLog2e = 1.4426950408889634f;
+constexpr int kMaxSplits = 16;
+
+__device__ __forceinline__ float fexp2(float x) { return __builtin_amdgcn_exp2f(x); }
+// exp2(x - m) with the -inf conventions of online softmax (m finite or -inf)
+__device__ __forceinline__ float sexp2(float x, float m) { return (x == -INFINITY) ? 0.f : fexp2(x - m); }
+__device__ __forceinline__ float ld_f32(const uint16_t* p) { return bf16_to_f32(*p); }
+__device__ __forceinline__ float ld_f32(const float* p) { return *p; }
+__device__ __forceinline__ void st_f32(uint16_t* p, float v) { *p = f32_to_bf16(v); }
+__device__ __forceinline__ void st_f32(float* p, float v) { *p = v; }
+
+// =====================================================================================
+// plain form
+// =====================================================================================
+// LDS: [q dk][o dv][p 64] floats, [V row offsets 64] int64
+template <typename T>
+__global__ __launch_bounds__(64) void attn_plain_kernel(AttnSpec a, const T* __restrict__ q, const T* __restrict__ kpool,
+                                                        const T* __restrict__ vpool, int bs, const int32_t* __restrict__ bt, int MB,
+                                                        const int32_t* __restrict__ pos, const AttnSeg* __restrict__ segs, int nseg,
+                                                        T* __restrict__ out, int ldo) {
+  extern __shared__ __attribute__((aligned(16))) unsigned char dsm[];
+  const HeadGeom& g = a.g;
+  long long* voff = reinterpret_cast<long long*>(dsm);
+  float* p = reinterpret_cast<float*>(voff + 64);
+  float* qs = p + 64;
+  float* o = qs + g.dk;
+  const int row = blockIdx.x, h = blockIdx.y, lane = threadIdx.x, kvh = h / (g.H / g.G);
+  int seq = row;
+  if (segs) {
+    int i = 0;
+    while (i < nseg - 1 && row >= segs[i].row0 + segs[i].n) ++i;
+    seq = segs[i].seq;
+  }
+  const int me = pos[row], lo = a.window > 0 ? max(0, me - a.window + 1) : 0;
+  const float slope = a.slopes ? a.slopes[h] : 0.f;
+  for (int d = lane; d < g.dk; d += 64) qs[d] = ld_f32(q + ((size_t)row * g.H + h) * g.dkp + d);
+  for (int d = lane; d < g.dv; d += 64) o[d] = 0.f;
+  __syncthreads();
+  float m = a.sink ? 0.f : -INFINITY, l = a.sink ? 1.f : 0.f;
+  for (int k0 = lo; k0 <= me; k0 += 64) {
+    const int j = k0 + lane;
+    float s = -INFINITY;
+    if (j <= me) {
+      const size_t r = ((size_t)bt[(size_t)seq * MB + j / bs] * g.G + kvh) * bs + j % bs;
+      const T* kr = kpool + r * g.dkp;
+      float dot = 0.f;
+      for (int d = 0; d < g.dk; ++d) dot = __builtin_fmaf(qs[d], ld_f32(kr + d), dot);
+      s = dot * a.scale - slope * (float)(me - j);
+      voff[lane] = (long long)(r * g.dvp);
+    }
+    float mx = s;
+#pragma unroll
+    for (int x = 32; x >= 1; x >>= 1) mx = fmaxf(mx, __shfl_xor(mx, x));
+    const float mn = fmaxf(m, mx), alpha = m == -INFINITY ? 0.f : expf(m - mn);
+    const float e = s == -INFINITY ? 0.f : expf(s - mn);
+    p[lane] = e;
+    l = l * alpha + wave_sum(e);
+    m = mn;
+    __syncthreads();
+    const int n = min(64, me - k0 + 1);
+    for (int d = lane; d < g.dv; d += 64) {
+      float acc = o[d] * alpha;
+      for (int k = 0; k < n; ++k) acc = __builtin_fmaf(p[k], ld_f32(vpool + voff[k] + d), acc);
+      o[d] = acc;
+    }
+    __syncthreads();
+  }
+  for (int d = lane; d < g.dv; d += 64) st_f32(out + (size_t)row * ldo + (size_t)h * g.dv + d, l > 0.f ? o[d] / l : 0.f);
+}
+
+// =====================================================================================
+// context encoding
+// =====================================================================================
+// 4 waves x NCG column groups of 16.  64-key tiles of K and V go through LDS (registers hold the next tile while the
+// current one is multiplied; the block ids run one tile further ahead).
+template <int DK, int DV>
+constexpr size_t prefill_lds() { return (size_t)64 * (DK + 8 + DV + 8) * 2; }
+
+template <int DK, int DV, int NCG>
+__global__ __launch_bounds__(256) void attn_window_prefill_kernel(AttnSpec a, const uint16_t* __restrict__ q, const uint16_t* __restrict__ kpool,
+                                                                  const uint16_t* __restrict__ vpool, int bs, const int32_t* __restrict__ bt,
+                                                                  int MB, const AttnSeg* __restrict__ segs, int nseg,
+                                                                  uint16_t* __restrict__ out, int ldo) {
+  constexpr int KP = DK + 8, VP = DV + 8;              // LDS row pitches (elements)
+  constexpr int KS = DK / 32, DN = DV / 16, KCH = DK / 8, VCH = DV / 8;
+  constexpr int NKL = 64 * KCH / 256, NVL = 64 * VCH / 256;   // 16-byte loads per thread and tile
+  extern __shared__ __attribute__((aligned(16))) unsigned char dsm[];
+  uint16_t* Ks = reinterpret_cast<uint16_t*>(dsm);
+  uint16_t* Vs = Ks + 64 * KP;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g4 = lane >> 4, c = lane & 15;
+  const int H = a.g.H, G = a.g.G, r = H / G, qpt = (64 * NCG) / r, kvh = blockIdx.y;
+
+  // this work-group's tile: segments with one row belong to the token-generation kernel.  Late tiles (long contexts) first.
+  int t = (int)(gridDim.x - 1 - blockIdx.x), si = 0;
+  AttnSeg sg{0, 0, 0, 0};
+  for (; si < nseg; ++si) {
+    sg = segs[si];
+    const int nt_s = sg.n > 1 ? ceil_div(sg.n, qpt) : 0;
+    if (t < nt_s) break;
+    t -= nt_s;
+  }
+  if (si == nseg) return;
+  const int q0 = t * qpt, nq = min(qpt, sg.n - q0), row0 = sg.row0 + q0, pos0 = sg.pos0 + q0;
+  const int32_t* btr = bt + (size_t)sg.seq * MB;
+  const int win = a.window > 0 ? a.window : 0x3fffffff;
+  const int klo = max(0, pos0 - win + 1) & ~15, khi = pos0 + nq - 1;
+  const int nt = ceil_div(khi + 1 - klo, 64);
+
+  const int dkc = a.g.dkp / 8 - 1, dvc = a.g.dvp / 8 - 1;   // last 16-byte chunk of a pool row
+  u32x4_t kr[NKL], vr[NVL];
+  int ids[4];
+  auto fetch_ids = [&](int k0) {     // block of each 16-token group (block_size is a multiple of 16); past the keys: the null block
+#pragma unroll
+    for (int u = 0; u < 4; ++u) ids[u] = (k0 + 16 * u <= khi) ? btr[(k0 + 16 * u) / bs] : 0;
+  };
+  auto issue = [&](int k0) {
+    size_t base[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u)
+      base[u] = (k0 + 16 * u <= khi) ? ((size_t)ids[u] * G + kvh) * bs + (k0 + 16 * u) % bs : 0;
+    auto row_of = [&](int row) -> size_t {
+      const int u = row >> 4;
+      return (u < 2 ? (u == 0 ? base[0] : base[1]) : (u == 2 ? base[2] : base[3])) + (row & 15);
+    };
+#pragma unroll
+    for (int i = 0; i < NKL; ++i) {
+      const int idx = tid + 256 * i, row = idx / KCH, ch = min(idx % KCH, dkc);
+      kr[i] = *reinterpret_cast<const u32x4_t*>(kpool + row_of(row) * a.g.dkp + ch * 8);
+    }
+#pragma unroll
+    for (int i = 0; i < NVL; ++i) {
+      const int idx = tid + 256 * i, row = idx / VCH, ch = min(idx % VCH, dvc);
+      vr[i] = *reinterpret_cast<const u32x4_t*>(vpool + row_of(row) * a.g.dvp + ch * 8);
+    }
+  };
+  fetch_ids(klo);
+  issue(klo);
+  fetch_ids(klo + 64);
+
+  // columns: position, bias slope, query fragments (zero beyond dkp and in dead columns)
+  int pc[NCG];
+  float sl2[NCG], mrow[NCG], lrow[NCG];
+  u32x4_t qf[NCG][KS];
+  f32x4_t acc[NCG][DN];
+#pragma unroll
+  for (int cg = 0; cg < NCG; ++cg) {
+    const int col = (wave * NCG + cg) * 16 + c, ql = col / r, h = kvh * r + col % r;
+    const bool live = ql < nq && ql < qpt;
+    pc[cg] = pos0 + (live ? ql : 0);
+    sl2[cg] = a.slopes ? a.slopes[h] * kLog2e : 0.f;
+    mrow[cg] = a.sink ? 0.f : -INFINITY;
+    lrow[cg] = (a.sink && g4 == 0) ? 1.f : 0.f;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks)
+      qf[cg][ks] = (live && ks * 32 + g4 * 8 < a.g.dkp) ? *reinterpret_cast<const u32x4_t*>(q + ((size_t)(row0 + ql) * H + h) * a.g.dkp + ks * 32 + g4 * 8)
+                                                        : u32x4_t{0, 0, 0, 0};
+#pragma unroll
+    for (int dn = 0; dn < DN; ++dn) acc[cg][dn] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  }
+  const float sc2 = a.scale * kLog2e;
+  // the wave's own query range (uniform)
+  const int wq0 = (wave * NCG * 16) / r, wq1 = min(nq - 1, (wave * NCG * 16 + NCG * 16 - 1) / r);
+  const bool wave_live = wq0 < nq;
+  const int pmin = pos0 + wq0, pmax = pos0 + wq1;
+  const int tr_row = (lane & 15) >> 2, tr_col = (lane & 3) * 4;
+
+  for (int n = 0; n < nt; ++n) {
+    const int k0 = klo + 64 * n;
+    __syncthreads();                     // the previous tile is consumed
+#pragma unroll
+    for (int i = 0; i < NKL; ++i) {
+      const int idx = tid + 256 * i;
+      *reinterpret_cast<u32x4_t*>(&Ks[(idx / KCH) * KP + (idx % KCH) * 8]) = kr[i];
+    }
+#pragma unroll
+    for (int i = 0; i < NVL; ++i) {
+      const int idx = tid + 256 * i;
+      *reinterpret_cast<u32x4_t*>(&Vs[(idx / VCH) * VP + (idx % VCH) * 8]) = vr[i];
+    }
+    __syncthreads();
+    if (n + 1 < nt) {
+      issue(k0 + 64);
+      fetch_ids(k0 + 128);
+    }
+    if (!wave_live || k0 > pmax || k0 + 63 <= pmin - win) continue;   // no key of this tile is seen by the wave (uniform)
+    f32x4_t st[NCG][4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+#pragma unroll
+      for (int cg = 0; cg < NCG; ++cg) st[cg][u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) {
+        const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(&Ks[(16 * u + c) * KP + ks * 32 + g4 * 8]);
+#pragma unroll
+        for (int cg = 0; cg < NCG; ++cg)
+          st[cg][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, __builtin_bit_cast(bf16x8_t, qf[cg][ks]), st[cg][u], 0, 0, 0);
+      }
+    }
+    const bool edge = k0 + 63 > pmin || k0 <= pmax - win;
+    union { uint32_t w[4]; bf16x8_t v; } pk[NCG][2];
+#pragma unroll
+    for (int cg = 0; cg < NCG; ++cg) {
+      const float b0 = sl2[cg] * (float)(k0 + 4 * g4 - pc[cg]);     // - slope (i - j), the lane's first key
+      float mx = -INFINITY;
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          float sv = __builtin_fmaf(st[cg][u][i], sc2, __builtin_fmaf(sl2[cg], (float)(16 * u + i), b0));
+          if (edge) {
+            const int j = k0 + 16 * u + 4 * g4 + i;
+            if (j > pc[cg] || j <= pc[cg] - win) sv = -INFINITY;
+          }
+          st[cg][u][i] = sv;
+          mx = fmaxf(mx, sv);
+        }
+      mx = fmaxf(mx, __shfl_xor(mx, 16));
+      mx = fmaxf(mx, __shfl_xor(mx, 32));
+      const float mn = fmaxf(mrow[cg], mx);
+      const float alpha = sexp2(mrow[cg], mn);
+      const bool moved = mn != mrow[cg];
+      mrow[cg] = mn;
+      const float ms = mn == -INFINITY ? 0.f : mn;   // (a column without a key so far: every score is -inf, exp2 gives 0)
+      float ps = 0.f;
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const float e = fexp2(st[cg][u][i] - ms);
+          st[cg][u][i] = e;
+          ps += e;
+        }
+      lrow[cg] = lrow[cg] * alpha + ps;
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        pk[cg][u >> 1].w[(u & 1) * 2] = pack_bf16x2(st[cg][u][0], st[cg][u][1]);
+        pk[cg][u >> 1].w[(u & 1) * 2 + 1] = pack_bf16x2(st[cg][u][2], st[cg][u][3]);
+      }
+      if (__any(moved)) {
+#pragma unroll
+        for (int dn = 0; dn < DN; ++dn) {
+          acc[cg][dn][0] *= alpha; acc[cg][dn][1] *= alpha; acc[cg][dn][2] *= alpha; acc[cg][dn][3] *= alpha;
+        }
+      }
+    }
+    // O^T += V^T.P^T: the k-slot (g4, j) of a 32-key half is key (j < 4 ? 4 g4 + j : 16 + 4 g4 + j - 4)
+#pragma unroll
+    for (int hf = 0; hf < 2; ++hf)
+#pragma unroll
+      for (int dn = 0; dn < DN; ++dn) {
+        const uint16_t* r0 = &Vs[(32 * hf + 4 * g4 + tr_row) * VP + 16 * dn + tr_col];
+        const s16x4_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4_t __attribute__((address_space(3)))*)r0);
+        const s16x4_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4_t __attribute__((address_space(3)))*)(r0 + 16 * VP));
+        const bf16x8_t av = {lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
+#pragma unroll
+        for (int cg = 0; cg < NCG; ++cg) acc[cg][dn] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(av, pk[cg][hf].v, acc[cg][dn], 0, 0, 0);
+      }
+  }
+
+#pragma unroll
+  for (int cg = 0; cg < NCG; ++cg) {
+    float L = lrow[cg];
+    L += __shfl_xor(L, 16);
+    L += __shfl_xor(L, 32);
+    const int col = (wave * NCG + cg) * 16 + c, ql = col / r, h = kvh * r + col % r;
+    if (ql >= nq || ql >= qpt) continue;
+    const float inv = L > 0.f ? 1.f / L : 0.f;
+    uint16_t* o = out + (size_t)(row0 + ql) * ldo + (size_t)h * a.g.dv;
+#pragma unroll
+    for (int dn = 0; dn < DN; ++dn) {
+      const int d = 16 * dn + 4 * g4;
+      if ((a.g.dv & 3) == 0) {
+        if (d < a.g.dv)
+          *reinterpret_cast<uint2*>(o + d) = make_uint2(pack_bf16x2(acc[cg][dn][0] * inv, acc[cg][dn][1] * inv), pack_bf16x2(acc[cg][dn][2] * inv, acc[cg][dn][3] * inv));
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (d + i < a.g.dv) o[d + i] = f32_to_bf16(acc[cg][dn][i] * inv);
+      }
+    }
+  }
+}
+
+// =====================================================================================
+// token generation
+// =====================================================================================
+// One work-group per (context split, kv head and group of 16 of its heads, sequence); its waves walk 32-key tiles
+// round-robin, two tiles in flight per wave.  K goes from the pool straight into A fragments, V through a wave-private LDS tile.
+template <int DV, int NW>
+constexpr size_t decode_lds() { return (size_t)NW * 32 * (DV + 8) * 2 + (size_t)NW * 16 * 2 * sizeof(float); }
+
+template <int DK, int DV, int NW, bool FINAL>
+__global__ __launch_bounds__(NW * 64) void attn_window_decode_kernel(AttnSpec a, const uint16_t* __restrict__ q, const uint16_t* __restrict__ kpool,
+                                                                     const uint16_t* __restrict__ vpool, int bs, const int32_t* __restrict__ bt,
+                                                                     int MB, const int32_t* __restrict__ ctx_lens, int NS,
+                                                                     float* __restrict__ o_part, float* __restrict__ ml_part,
+                                                                     uint16_t* __restrict__ out, int ldo) {
+  constexpr int VP = DV + 8, KS = DK / 32, DN = DV / 16, VCH = DV / 8;
+  constexpr int NV = 32 * VCH / 64;
+  constexpr int VT = 32 * VP;
+  extern __shared__ __attribute__((aligned(16))) unsigned char dsm[];
+  uint16_t* Vs = reinterpret_cast<uint16_t*>(dsm);                       // [NW][32][VP]
+  float* sm_ml = reinterpret_cast<float*>(dsm + (size_t)NW * VT * 2);    // [NW][16][2]
+  const int H = a.g.H, G = a.g.G, r = H / G;
+  const int split = blockIdx.x, kvh = blockIdx.y % G, hc = blockIdx.y / G, b = blockIdx.z;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g4 = lane >> 4, c = lane & 15;
+  const int nhc = min(16, r - hc * 16), h0 = kvh * r + hc * 16;          // this work-group's heads
+  const int ctx = ctx_lens[b], lo = a.window > 0 ? max(0, ctx - a.window) : 0;
+  const int32_t* btr = bt + (size_t)b * MB;
+  const int t_first = lo / 32 + split * NW + wave, t_end = ceil_div(ctx, 32), stride = NS * NW;
+  const int dkc = a.g.dkp / 8 - 1, dvc = a.g.dvp / 8 - 1;
+  uint16_t* Vw = Vs + wave * VT;
+
+  u32x4_t kA[2 * KS], vA[NV], kB[2 * KS], vB[NV];
+  auto issue = [&](u32x4_t (&kr)[2 * KS], u32x4_t (&vr)[NV], int tt) {
+    size_t rowh[2];   // pool row of the first token of each 16-token half (the null block where there is none)
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      const int tok = tt * 32 + 16 * u;
+      rowh[u] = (tt < t_end && tok < ctx) ? ((size_t)btr[tok / bs] * G + kvh) * bs + tok % bs : 0;
+    }
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks)
+        kr[u * KS + ks] = __builtin_nontemporal_load(reinterpret_cast<const u32x4_t*>(kpool + (rowh[u] + c) * a.g.dkp + min(ks * 4 + g4, dkc) * 8));
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int row = (lane + 64 * i) / VCH, ch = min((lane + 64 * i) % VCH, dvc);
+      vr[i] = __builtin_nontemporal_load(reinterpret_cast<const u32x4_t*>(vpool + (rowh[row >> 4] + (row & 15)) * a.g.dvp + ch * 8));
+    }
+  };
+  if (t_first < t_end) issue(kA, vA, t_first);
+
+  u32x4_t qf[KS];
+#pragma unroll
+  for (int ks = 0; ks < KS; ++ks)
+    qf[ks] = (c < nhc && ks * 32 + g4 * 8 < a.g.dkp) ? *reinterpret_cast<const u32x4_t*>(q + ((size_t)b * H + h0 + c) * a.g.dkp + ks * 32 + g4 * 8)
+                                                     : u32x4_t{0, 0, 0, 0};
+  const float sl2 = (a.slopes && c < nhc) ? a.slopes[h0 + c] * kLog2e : 0.f, sc2 = a.scale * kLog2e;
+  f32x4_t acc[DN];
+#pragma unroll
+  for (int dn = 0; dn < DN; ++dn) acc[dn] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  float mrow = -INFINITY, lrow = 0.f;
+  const int tr_row = (lane & 15) >> 2, tr_col = (lane & 3) * 4;
+
+  auto update = [&](const u32x4_t (&kr)[2 * KS], const u32x4_t (&vr)[NV], int tt) {
+    asm volatile("" ::: "memory");
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int idx = lane + 64 * i;
+      *reinterpret_cast<u32x4_t*>(&Vw[(idx / VCH) * VP + (idx % VCH) * 8]) = vr[i];
+    }
+    asm volatile("" ::: "memory");   // LDS ops of one wave execute in order; keep the compiler from reordering them
+    f32x4_t st[2];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      st[u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks)
+        st[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, kr[u * KS + ks]), __builtin_bit_cast(bf16x8_t, qf[ks]), st[u], 0, 0, 0);
+    }
+    s16x4_t vlo[DN], vhi[DN];
+#pragma unroll
+    for (int dn = 0; dn < DN; ++dn) {
+      const uint16_t* r0 = &Vw[(4 * g4 + tr_row) * VP + 16 * dn + tr_col];
+      vlo[dn] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4_t __attribute__((address_space(3)))*)r0);
+      vhi[dn] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4_t __attribute__((address_space(3)))*)(r0 + 16 * VP));
+    }
+    float pv[8], mx = -INFINITY;
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int j = tt * 32 + 16 * u + 4 * g4 + i;
+        float sv = __builtin_fmaf(st[u][i], sc2, sl2 * (float)(j - (ctx - 1)));
+        if (j >= ctx || j < lo) sv = -INFINITY;
+        pv[4 * u + i] = sv;
+        mx = fmaxf(mx, sv);
+      }
+    mx = fmaxf(mx, __shfl_xor(mx, 16));
+    mx = fmaxf(mx, __shfl_xor(mx, 32));
+    const float mn = fmaxf(mrow, mx);
+    const float alpha = sexp2(mrow, mn);
+    float ps = 0.f;
+#pragma unroll
+    for (int k = 0; k < 8; ++k) {
+      pv[k] = sexp2(pv[k], mn);
+      ps += pv[k];
+    }
+    const bool moved = mn != mrow;
+    mrow = mn;
+    lrow = lrow * alpha + ps;
+    union { uint32_t w[4]; bf16x8_t v; } pk;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) pk.w[k] = pack_bf16x2(pv[2 * k], pv[2 * k + 1]);
+    if (__any(moved)) {
+#pragma unroll
+      for (int dn = 0; dn < DN; ++dn) {
+        acc[dn][0] *= alpha; acc[dn][1] *= alpha; acc[dn][2] *= alpha; acc[dn][3] *= alpha;
+      }
+    }
+#pragma unroll
+    for (int dn = 0; dn < DN; ++dn) {
+      const s16x4_t l4 = vlo[dn], h4 = vhi[dn];
+      const bf16x8_t av = {l4[0], l4[1], l4[2], l4[3], h4[0], h4[1], h4[2], h4[3]};
+      acc[dn] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(av, pk.v, acc[dn], 0, 0, 0);
+    }
+  };
+
+  for (int tt = t_first; tt < t_end; tt += 2 * stride) {
+    if (tt + stride < t_end) issue(kB, vB, tt + stride);
+    update(kA, vA, tt);
+    if (tt + 2 * stride < t_end) issue(kA, vA, tt + 2 * stride);
+    if (tt + stride < t_end) update(kB, vB, tt + stride);
+  }
+
+  // merge the waves through their (now idle) LDS tiles, in wave order
+  lrow += __shfl_xor(lrow, 16);
+  lrow += __shfl_xor(lrow, 32);
+  asm volatile("" ::: "memory");
+  float* so = reinterpret_cast<float*>(Vw);            // [16 heads][DV] f32 <= the tile
+#pragma unroll
+  for (int dn = 0; dn < DN; ++dn) *reinterpret_cast<f32x4_t*>(&so[c * DV + 16 * dn + 4 * g4]) = acc[dn];
+  if (g4 == 0) {
+    sm_ml[(wave * 16 + c) * 2] = mrow;
+    sm_ml[(wave * 16 + c) * 2 + 1] = lrow;
+  }
+  __syncthreads();
+  for (int idx = tid; idx < nhc * DV; idx += NW * 64) {
+    const int h = idx / DV, d = idx % DV;
+    if (d >= a.g.dvp) continue;
+    float M = sm_ml[h * 2];
+#pragma unroll
+    for (int w = 1; w < NW; ++w) M = fmaxf(M, sm_ml[(w * 16 + h) * 2]);
+    if (FINAL && a.sink) M = fmaxf(M, 0.f);
+    float o = 0.f, L = 0.f;
+#pragma unroll
+    for (int w = 0; w < NW; ++w) {
+      const float f = sexp2(sm_ml[(w * 16 + h) * 2], M);
+      o += f * reinterpret_cast<const float*>(Vs + w * VT)[h * DV + d];
+      L += f * sm_ml[(w * 16 + h) * 2 + 1];
+    }
+    if constexpr (FINAL) {
+      if (a.sink) L += fexp2(-M);
+      if (d < a.g.dv) out[(size_t)b * ldo + (size_t)(h0 + h) * a.g.dv + d] = f32_to_bf16(L > 0.f ? o / L : 0.f);
+    } else {
+      const size_t row = ((size_t)b * H + h0 + h) * kMaxSplits + split;
+      o_part[row * a.g.dvp + d] = o;
+      if (d == 0) {
+        ml_part[row * 2] = M;
+        ml_part[row * 2 + 1] = L;
+      }
+    }
+  }
+}
+
+// merge the context splits of one (sequence, head) in split order, the sink last
+__global__ __launch_bounds__(128) void attn_window_combine_kernel(AttnSpec a, const float* __restrict__ o_part, const float* __restrict__ ml_part,
+                                                                  int NS, uint16_t* __restrict__ out, int ldo) {
+  const int head = blockIdx.x, b = blockIdx.y;
+  const size_t row0 = ((size_t)b * a.g.H + head) * kMaxSplits;
+  float mv[kMaxSplits], lv[kMaxSplits];
+  float M = a.sink ? 0.f : -INFINITY;
+#pragma unroll
+  for (int s = 0; s < kMaxSplits; ++s) {
+    const float2 ml = s < NS ? *reinterpret_cast<const float2*>(ml_part + (row0 + s) * 2) : make_float2(-INFINITY, 0.f);
+    mv[s] = ml.x;
+    lv[s] = ml.y;
+    M = fmaxf(M, ml.x);
+  }
+  float L = a.sink ? fexp2(-M) : 0.f;
+#pragma unroll
+  for (int s = 0; s < kMaxSplits; ++s) {
+    mv[s] = sexp2(mv[s], M);
+    L += mv[s] * lv[s];
+  }
+  for (int d = threadIdx.x; d < a.g.dv; d += 128) {
+    float ov[kMaxSplits];
+#pragma unroll
+    for (int s = 0; s < kMaxSplits; ++s) ov[s] = s < NS ? o_part[(row0 + s) * a.g.dvp + d] : 0.f;
+    float acc = 0.f;
+#pragma unroll
+    for (int s = 0; s < kMaxSplits; ++s) acc += mv[s] * ov[s];
+    out[(size_t)b * ldo + (size_t)head * a.g.dv + d] = f32_to_bf16(L > 0.f ? acc / L : 0.f);
+  }
+}
+
+// context splits: about one work-group per CU, every wave of a split with at least a tile to walk
+int decode_splits(int groups, int max_keys, int nw) {
+  const int by_cu = 256 / groups, by_len = ceil_div(ceil_div(max_keys, 32) + 1, nw);
+  const int ns = by_cu < by_len ? by_cu : by_len;
+  return ns < 1 ? 1 : (ns > kMaxSplits ? kMaxSplits : ns);
+}
+
+int check_spec(const AttnSpec& a, int block_size) {
+  MI_CHECK(a.g.H > 0 && a.g.G > 0 && a.g.H % a.g.G == 0, "attention: query heads must be a multiple of kv heads");
+  MI_CHECK(a.g.dk > 0 && a.g.dv > 0 && a.g.dkp % 16 == 0 && a.g.dvp % 16 == 0 && a.g.dkp >= a.g.dk && a.g.dvp >= a.g.dv, "attention: head sizes");
+  MI_CHECK(block_size > 0 && block_size % 16 == 0 && a.window >= 0, "attention: block_size % 16 == 0, window >= 0");
+  return MI_OK;
+}
+
+template <int DK, int DV>
+int launch_decode_t(const AttnSpec& a, const uint16_t* q, const uint16_t* kpool, const uint16_t* vpool, int bs, const int32_t* bt, int MB,
+                    const int32_t* ctx, int B, int max_ctx, uint16_t* out, int ldo, void* scratch, hipStream_t s) {
+  constexpr int NW = 4;
+  const int hcs = ceil_div(a.g.H / a.g.G, 16), groups = B * a.g.G * hcs;
+  const int max_keys = a.window > 0 && a.window < max_ctx ? a.window : max_ctx;
+  const int NS = decode_splits(groups, max_keys, NW);
+  constexpr size_t lds = decode_lds<DV, NW>();
+  const dim3 grid(NS, a.g.G * hcs, B);
+  if (NS == 1) {
+    auto kern = attn_window_decode_kernel<DK, DV, NW, true>;
+    if (lds > 64 * 1024) { int rc = ensure_dynamic_lds(reinterpret_cast<const void*>(kern), (int)lds); if (rc != MI_OK) return rc; }
+    hipLaunchKernelGGL(kern, grid, dim3(NW * 64), lds, s, a, q, kpool, vpool, bs, bt, MB, ctx, 1, nullptr, nullptr, out, ldo);
+  } else {
+    float* ml = reinterpret_cast<float*>(scratch);
+    float* op = ml + (size_t)B * a.g.H * kMaxSplits * 2;
+    auto kern = attn_window_decode_kernel<DK, DV, NW, false>;
+    if (lds > 64 * 1024) { int rc = ensure_dynamic_lds(reinterpret_cast<const void*>(kern), (int)lds); if (rc != MI_OK) return rc; }
+    hipLaunchKernelGGL(kern, grid, dim3(NW * 64), lds, s, a, q, kpool, vpool, bs, bt, MB, ctx, NS, op, ml, out, ldo);
+    hipLaunchKernelGGL(attn_window_combine_kernel, dim3(a.g.H, B), dim3(128), 0, s, a, op, ml, NS, out, ldo);
+  }
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+template <int DK, int DV, int NCG>
+int launch_prefill_t(const AttnSpec& a, const uint16_t* q, const uint16_t* kpool, const uint16_t* vpool, int bs, const int32_t* bt, int MB,
+                     const AttnSeg* sd, const AttnSeg* sh, int nseg, uint16_t* out, int ldo, hipStream_t s) {
+  const int qpt = 64 * NCG / (a.g.H / a.g.G);
+  int tiles = 0;
+  for (int i = 0; i < nseg; ++i) tiles += sh[i].n > 1 ? ceil_div(sh[i].n, qpt) : 0;
+  if (tiles == 0) return MI_OK;
+  constexpr size_t lds = prefill_lds<DK, DV>();
+  auto kern = attn_window_prefill_kernel<DK, DV, NCG>;
+  if (lds > 64 * 1024) { int rc = ensure_dynamic_lds(reinterpret_cast<const void*>(kern), (int)lds); if (rc != MI_OK) return rc; }
+  hipLaunchKernelGGL(kern, dim3(tiles, a.g.G), dim3(256), lds, s, a, q, kpool, vpool, bs, bt, MB, sd, nseg, out, ldo);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+// the built (dk, dv) sizes: the smallest that holds the layer's
+#define MI_BY_SIZE(CALL)                                                          \
+  do {                                                                            \
+    const int dk_ = a.g.dkp, dv_ = a.g.dvp;                                       \
+    if (dk_ <= 64 && dv_ <= 64) return CALL(64, 64, 2);                           \
+    if (dk_ <= 64 && dv_ <= 128) return CALL(64, 128, 2);                         \
+    if (dk_ <= 128 && dv_ <= 64) return CALL(128, 64, 2);                         \
+    if (dk_ <= 128 && dv_ <= 128) return CALL(128, 128, 2);                       \
+    return CALL(256, 256, 1);                                                     \
+  } while (0)
+
+}  // namespace
+
+bool attn_window_supported(const HeadGeom& g) { return g.dkp <= 256 && g.dvp <= 256 && g.H / g.G <= 64; }
+
+size_t attn_window_scratch_bytes(int B, const HeadGeom& g) { return (size_t)B * g.H * kMaxSplits * (g.dvp + 2) * sizeof(float); }
+
+int launch_attn_plain(const AttnSpec& a, const void* q, const void* kpool, const void* vpool, int bs, const int32_t* bt, int MB,
+                      const int32_t* pos, const AttnSeg* segs, int nseg, int T, void* out, int ldo, bool f32, hipStream_t s) {
+  int rc = check_spec(a, bs);
+  if (rc != MI_OK) return rc;
+  MI_CHECK(T >= 1 && ldo >= a.g.H * a.g.dv && (segs == nullptr || nseg >= 1), "attention: rows / output stride");
+  const size_t lds = 64 * 8 + (64 + (size_t)a.g.dk + a.g.dv) * 4;
+  MI_CHECK(lds <= 64 * 1024, "attention: head sizes too large");
+  const dim3 grid(T, a.g.H);
+  if (f32) hipLaunchKernelGGL((attn_plain_kernel<float>), grid, dim3(64), lds, s, a, (const float*)q, (const float*)kpool, (const float*)vpool, bs, bt, MB, pos, segs, nseg, (float*)out, ldo);
+  else hipLaunchKernelGGL((attn_plain_kernel<uint16_t>), grid, dim3(64), lds, s, a, (const uint16_t*)q, (const uint16_t*)kpool, (const uint16_t*)vpool, bs, bt, MB, pos, segs, nseg, (uint16_t*)out, ldo);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_attn_window_decode(const AttnSpec& a, const uint16_t* q, const uint16_t* kpool, const uint16_t* vpool, int bs, const int32_t* bt,
+                              int MB, const int32_t* ctx, int B, int max_ctx, uint16_t* out, int ldo, void* scratch, hipStream_t s) {
+  int rc = check_spec(a, bs);
+  if (rc != MI_OK) return rc;
+  MI_CHECK(attn_window_supported(a.g) && B >= 1 && max_ctx >= 1 && ldo >= a.g.H * a.g.dv, "windowed decode attention: shape");
+#define MI_CALL_D(DK, DV, NCG) launch_decode_t<DK, DV>(a, q, kpool, vpool, bs, bt, MB, ctx, B, max_ctx, out, ldo, scratch, s)
+  MI_BY_SIZE(MI_CALL_D);
+#undef MI_CALL_D
+}
+
+int launch_attn_window_prefill(const AttnSpec& a, const uint16_t* q, const uint16_t* kpool, const uint16_t* vpool, int bs, const int32_t* bt,
+                               int MB, const AttnSeg* sd, const AttnSeg* sh, int nseg, uint16_t* out, int ldo, hipStream_t s) {
+  int rc = check_spec(a, bs);
+  if (rc != MI_OK) return rc;
+  MI_CHECK(attn_window_supported(a.g) && nseg >= 1 && ldo >= a.g.H * a.g.dv && ((a.g.dv & 3) != 0 || ldo % 4 == 0), "windowed prefill attention: shape");
+#define MI_CALL_P(DK, DV, NCG) launch_prefill_t<DK, DV, NCG>(a, q, kpool, vpool, bs, bt, MB, sd, sh, nseg, out, ldo, s)
+  MI_BY_SIZE(MI_CALL_P);
+#undef MI_CALL_P
+}
+
+}  // namespace mi

@@ -14,10 +14,11 @@ import gc
 import time
 from dataclasses import dataclass, field
 
-from ._vllm_compat import (HAVE_VLLM, KVCacheConfig, Request, SamplingParams, Scheduler, SimpleCacheConfig,
+from ._vllm_compat import (HAVE_VLLM, KVCacheConfig, ModelRunnerOutput, Request, SamplingParams, Scheduler, SimpleCacheConfig,
                            SimpleDeviceConfig, SimpleModelConfig, SimpleParallelConfig,
                            SimpleSchedulerConfig, SimpleVllmConfig)
 from .core.scheduler import ContinuousBatchingMI355XScheduler
+from .models import load_config
 from .platform import MI355XPlatform
 from .worker.mi355x_worker import MI355XWorker
 
@@ -34,12 +35,14 @@ class RequestOutput:
 
 
 class MI355XEngine:
-    def __init__(self, hf_config, model: str = "", *, max_model_len=2048, max_num_seqs=4, block_size=32,
+    def __init__(self, hf_config=None, model: str = "", *, max_model_len=2048, max_num_seqs=4, block_size=32,
                  num_gpu_blocks_override=None, enable_prefix_caching=True, tensor_parallel_size=1,
                  dtype="bfloat16", override_mi355x_config: dict | None = None, seed=0, local_rank=0,
                  enable_chunked_prefill=False, max_num_batched_tokens=None, speculative_config=None):
         if HAVE_VLLM:  # pragma: no cover
             raise RuntimeError("vLLM is installed: use vllm.LLM(...) — the plugin registers itself")
+        if hf_config is None:
+            hf_config = load_config(model)        # config.json picks the model (models/__init__.py)
         cfg = SimpleVllmConfig(
             model_config=SimpleModelConfig(model=model, hf_config=hf_config, dtype=dtype,
                                            max_model_len=max_model_len, seed=seed),
@@ -121,6 +124,31 @@ class MI355XEngine:
             ro.token_ids.extend(out.new_token_ids)
             ro.finished = ro.finished or out.finished
         return sched_out, runner_out
+
+    def append_tokens(self, request_id: str, token_ids: list[int]) -> None:
+        """More input for a live request whose prompt is used up; it is scheduled again at the next step."""
+        self.scheduler.requests[request_id].prompt_token_ids.extend(token_ids)
+        self.worker.append_prompt_tokens(request_id, list(token_ids))
+
+    def score_step(self, places: dict[str, list[int]]):
+        """One engine step that samples nothing: schedule what is pending and return, per request, the fp32 logits at
+        `places` among the tokens scheduled for it.  -> ({request id: [places, vocab]}, SchedulerOutput)"""
+        sched_out = self.scheduler.schedule()
+        logits = self.worker.score_rows(sched_out, places)
+        ids = list(sched_out.num_scheduled_tokens)
+        self.scheduler.update_from_output(sched_out, ModelRunnerOutput(
+            req_ids=ids, req_id_to_index={r: i for i, r in enumerate(ids)}, sampled_token_ids=[[] for _ in ids]))
+        return logits, sched_out
+
+    def finish_requests(self, request_ids) -> None:
+        self.scheduler.finish_requests(request_ids)
+        for rid in request_ids:
+            self.outputs.pop(rid, None)
+
+    def close(self) -> None:
+        for native in (getattr(self.worker.model_runner.model, "draft", None), self.worker.model_runner.model.model):
+            if native is not None:
+                native.close()
 
     def generate(self, prompts: list[list[int]], sampling_params: SamplingParams | None = None,
                  eos_token_id=None) -> list[RequestOutput]:

@@ -15,6 +15,8 @@ working).  Extra keys understood here:
   synthetic_weights          {"seed","std"} random weights generated on the device (bench)
   state_dict                 dict[str, Tensor] in-memory HF-named weights (tests)
   use_graphs                 bool           hipGraph capture of token-generation steps
+  weight_artifacts           bool           False: no weight images are kept beside a local checkpoint
+  kv_overcommit              bool           a KV pool smaller than max_num_seqs x max_model_len is accepted
   tp_transport               "p2p" | "rccl" exchange between the rank shards of tensor_parallel_size > 1
   prefill_fp8_activations    bool           context-encoding GEMMs on FP8 weights quantize their bf16
                                             inputs per token to e4m3 and run on the MX-scaled MFMA
@@ -34,6 +36,7 @@ import torch
 import torch.nn as nn
 
 from .._vllm_compat import SamplerOutput
+from ..models import stack_of
 from .constants import (MI355X_MULTI_MODAL_MODELS, SUPPORTED_ARCHITECTURES,
                         TORCH_DTYPE_TO_MI355X_AMP)
 
@@ -254,6 +257,12 @@ class MI355XCausalLM(MI355XModelBase):
             slots = torch.where(ar < full[:, None], block_table * bs + ar, torch.full_like(ar, -1))
         return block_table, slots
 
+    def forward_rows(self, model_input, rows) -> torch.Tensor:
+        """Logits of chosen places of one ragged token batch (indices into it), nothing sampled."""
+        return self.model.forward_rows(model_input.input_tokens, model_input.position_ids, model_input.slot_mapping,
+                                       model_input.block_tables, model_input.full_context_lens,
+                                       model_input.computed_context_lens, rows)
+
     def sample(self, logits: torch.Tensor) -> SamplerOutput | None:
         if self.mi355x_config.on_device_sampling_config:
             return SamplerOutput(sampled_token_ids=logits.unsqueeze(-1), logprobs_tensors=None)
@@ -265,7 +274,7 @@ class MI355XCausalLM(MI355XModelBase):
         from .._native import NativeModel
         cfg: dict = kwargs["mi355x_config"]
         hf = self.hf_config
-        geo = _decoder_geometry(hf)
+        geo = _model_geometry(hf, cfg)
         max_model_len = cfg["seq_len"]
         if cfg["is_block_kv_layout"]:
             block_size, num_blocks = cfg["pa_block_size"], cfg["pa_num_blocks"]
@@ -414,8 +423,8 @@ class MI355XCausalLM(MI355XModelBase):
         draft_model_modules_to_not_convert says otherwise."""
         from .._native import NativeModel
         draft_cfg = speculative_config.draft_model_config
-        geo = _decoder_geometry(draft_cfg.hf_config)
-        if geo["vocab_size"] != self.hf_config.vocab_size:
+        geo = _model_geometry(draft_cfg.hf_config, {**cfg, "tp_degree": 1})
+        if draft_cfg.hf_config.vocab_size != self.hf_config.vocab_size:
             raise ValueError("fused speculation: draft and target must share the vocabulary")
         draft_skip = cfg.get("draft_model_modules_to_not_convert") or not_converted
         self._draft_catchup = {}
@@ -450,9 +459,12 @@ class MI355XCausalLM(MI355XModelBase):
           * MI355X_COMPILED_ARTIFACTS (the reference's NEURON_COMPILED_ARTIFACTS, loader.py:198-199): as given;
           * a local checkpoint directory: <model>/mi355x-compiled-artifacts/<md5 of the configuration>
             (loader.py:186-210);
-          * synthetic or in-memory weights without one of the two explicit paths: not cached."""
+          * synthetic or in-memory weights without one of the two explicit paths: not cached;
+          * override key weight_artifacts = False: nothing is kept."""
         import hashlib
         import json
+        if cfg.get("weight_artifacts") is False:
+            return None
         explicit = (cfg.get("quantized_checkpoints_path") if quantized else None) or os.getenv("MI355X_COMPILED_ARTIFACTS")
         if explicit:
             return str(explicit)
@@ -482,6 +494,16 @@ class MI355XCausalLM(MI355XModelBase):
                     t = sf.get_tensor(name)
                     if t.dim() in (1, 2):
                         self.model.load_weight(name, t)
+
+
+def _model_geometry(hf, cfg: dict) -> dict:
+    """NativeModel's geometry arguments: a layer stack, or the Llama-family fields."""
+    stack = stack_of(hf)
+    if stack is None:
+        return _decoder_geometry(hf)
+    if int(cfg["tp_degree"]) > 1 or cfg.get("quantized"):
+        raise NotImplementedError("layer-stack models: tensor parallelism and weight quantization are not built")
+    return dict(stack=dict(stack, compute_dtype={"bfloat16": 1, "float32": 0}[cfg.get("stack_dtype", "bfloat16")]))
 
 
 def _decoder_geometry(hf) -> dict:
@@ -562,6 +584,12 @@ def get_mi355x_model(model_config, cache_config, parallel_config, scheduler_conf
         cfg = _handle_pa_num_blocks(cache_config, cfg, override)
     cfg = _validate_mi355x_config(cache_config, scheduler_config, cfg)
     cfg["scheduler_max_num_seqs"] = scheduler_config.max_num_seqs
+    if stack_of(model_config.hf_config) is not None:
+        # the compute type follows the dtype asked for by name ("auto" is bf16: what the checkpoint holds)
+        dtype = "bfloat16" if model_config.dtype == "auto" else TORCH_DTYPE_TO_MI355X_AMP[model_config.dtype]
+        if dtype not in ("bfloat16", "float32"):
+            raise ValueError(f"{architecture}: dtype {dtype} is not served (bfloat16 or float32)")
+        cfg["stack_dtype"] = dtype
 
     if cfg.get("enable_fused_speculation") and not cfg.get("on_device_sampling_config"):
         # the fused step returns token ids, never logits (reference loader.py:349-355)
@@ -660,7 +688,9 @@ def _validate_mi355x_config(cache_config, scheduler_config, mi355x_config: dict)
             effective_blocks = cache_config.num_gpu_blocks_override - 1
         else:
             effective_blocks = mi355x_config.get("pa_num_blocks")
-        assert effective_blocks >= min_blocks_required, (
+        # kv_overcommit: the scheduler holds requests back when the pool runs out instead of every sequence having
+        # its worst case reserved
+        assert mi355x_config.get("kv_overcommit") or effective_blocks >= min_blocks_required, (
             f"At least {min_blocks_required} blocks are required for max_model_len "
             f"{scheduler_config.max_model_len}, but only {effective_blocks} blocks are available "
             "(user-intended blocks, excluding the +1 for null block)")

@@ -192,6 +192,33 @@ class MI355XModelRunner:
         sampler_outputs = self._execute_model_for_text(model_input, intermediate_tensors)
         return self._generate_model_runner_output(sampler_outputs)
 
+    @torch.inference_mode()
+    def score_rows(self, scheduler_output, places: dict):
+        """One engine step that samples nothing: {request id: places among its scheduled tokens} -> {request id: fp32
+        logits [places, vocab]}.  Same state update, input preparation and model call as a chunked-prefill step."""
+        if not self.is_chunked_prefill:
+            raise RuntimeError("score_rows needs the chunked-prefill engine (ragged token batches)")
+        if not self._kv_ready:
+            self.initialize_kv_cache(None)
+        self._update_states(scheduler_output)
+        if not scheduler_output.total_num_scheduled_tokens:
+            return {}
+        data = self._prepare_chunked_prefill_inputs(scheduler_output)
+        model_input = self._finalize_chunked_prefill_inputs(data)
+        rows, at, first = [], {}, 0
+        for req_id, full, computed in zip(data.request_ids, data.full_context_lens, data.computed_context_lens):
+            at[req_id] = (len(rows), len(places.get(req_id, ())))
+            rows.extend(first + int(p) for p in places.get(req_id, ()))
+            first += full - computed
+        logits = self.model.forward_rows(model_input, rows)
+        return {req_id: logits[i:i + n] for req_id, (i, n) in at.items()}
+
+    def append_prompt_tokens(self, req_id: str, token_ids: list) -> None:
+        """More input for a request that has used up its prompt (streaming input)."""
+        state = self.requests.get(req_id)
+        if state is not None:
+            state.prompt_token_ids.extend(token_ids)
+
     def _generate_model_runner_output(self, sampler_outputs: SamplerOutput | None):
         if sampler_outputs is None:
             return EMPTY_MODEL_RUNNER_OUTPUT

@@ -122,6 +122,12 @@ class MI355XWorker(WorkerBase):
         output = self.model_runner.execute_model(scheduler_output)
         return output if self.is_driver_worker else None
 
+    def score_rows(self, scheduler_output, places: dict) -> dict:
+        return self.model_runner.score_rows(scheduler_output, places)
+
+    def append_prompt_tokens(self, req_id: str, token_ids: list) -> None:
+        self.model_runner.append_prompt_tokens(req_id, token_ids)
+
     def profile(self, is_start: bool = True):
         """Per-kernel-class HIP-event timing of the following steps (eager launches)."""
         self.model_runner.model.model.profile_enable(bool(is_start))

@@ -269,6 +269,110 @@ def speculation_section(torch, HF, wd, plain_ms, steps, k=4):
                     "tests/test_spec_decode_gpu.py checks that the text equals the target's greedy text"}
 
 
+# ---- --vimesun: the layer-stack design beside a Llama of equal size, both bf16 (random weights) -------------------------
+# (label, width, q heads, kv heads, head size, Llama intermediate size, layers).  A Vimesun feed-forward has two matrices where
+# a Llama's has three: 1.5 x the intermediate size makes the layers equal in parameters.
+VIMESUN_SIZES = [("1b-like", 2048, 32, 8, 64, 8192, 16), ("8b-like", 4096, 32, 8, 128, 14336, 8)]
+VIMESUN_VOCAB, VIMESUN_WINDOW = 32768, 1024
+MFMA_BF16_PEAK_TFLOPS = 2500.0
+
+
+def vimesun_section(args):
+    """Prefill and decode of both models through the same library calls, per kernel class: milliseconds and the fraction of
+    the class's roofline (MFMA flops for GEMM and context attention, HBM bytes for the weight stream, decode attention and
+    the row-wise kernels).  `distance` = Llama's fraction / Vimesun's: how much further from its roofline the class is."""
+    import torch
+
+    from tests.helpers import decode_inputs, prefill_inputs
+    from vllm_neuron_amd._native import NativeModel
+    from vllm_neuron_amd.models import config_from_dict
+    from vllm_neuron_amd.worker.mi355x_model_loader import _decoder_geometry
+    max_len, mb = 4096, 4096 // BLOCK_SIZE
+    rows_max = 32
+    blocks = [[1 + b * mb + j for j in range(mb)] for b in range(rows_max)]
+
+    def build(kind, width, nh, nkv, hd, inter, layers, window):
+        common = dict(num_blocks=1 + rows_max * mb, block_size=BLOCK_SIZE, max_num_seqs=rows_max, max_model_len=max_len,
+                      ctx_buckets=[max_len], device_id=0, use_graphs=1)
+        if kind == "vimesun":
+            layer = {"type": "attention", "mixer": {"heads": nh, "kv_heads": nkv, "dim": hd, "vdim": hd, "mask": {"size": window},
+                                                    "scale": hd ** -0.5}, "mlp": {"kind": "dense", "ff": inter * 3 // 2}}
+            cfg = config_from_dict({"architecture": "Vimesun", "width": width, "vocab": VIMESUN_VOCAB, "layers": [layer] * layers,
+                                    "residual_mult": 0.5, "norm": {"eps": 1e-5}, "max_positions": max_len})
+            m = NativeModel(stack=dict(cfg.stack, compute_dtype=1), **common)
+        else:
+            hf = dict(MODELS["llama31_8b"], hidden_size=width, num_attention_heads=nh, num_key_value_heads=nkv, head_dim=hd,
+                      intermediate_size=inter, num_hidden_layers=layers, vocab_size=VIMESUN_VOCAB)
+            m = NativeModel(weight_dtype=0, quant_type=0, quantize_lm_head=0, tp_degree=1, tp_rank=0,
+                            prefill_fp8_activations=0, **common, **_decoder_geometry(SimpleNamespace(**hf)))
+        m.init_synthetic_weights(1, 0.02)
+        m.finalize()
+        return m
+
+    def keys_seen(first, n, window):          # keys of n consecutive queries
+        return sum(min(i + 1, window) for i in range(first, first + n))
+
+    out = []
+    for label, width, nh, nkv, hd, inter, layers in VIMESUN_SIZES:
+        per_layer = width * (2 * nh + 2 * nkv) * hd + 3 * width * inter
+        size = {"size": label, "layers": layers, "width": width, "heads": [nh, nkv, hd], "parameters": layers * per_layer + VIMESUN_VOCAB * width,
+                "prefill": [], "decode": []}
+        for kind, window in (("llama", max_len), ("vimesun", max_len), ("vimesun", VIMESUN_WINDOW)):
+            print(f"[bench] {label} {kind} window {window}", file=sys.stderr, flush=True)
+            m = build(kind, width, nh, nkv, hd, inter, layers, window)
+            name = "llama" if kind == "llama" else f"vimesun, {'every key' if window == max_len else f'window {window}'}"
+            for T in (512, 2048, 4000):
+                inp = prefill_inputs([(7 * i + 3) % VIMESUN_VOCAB for i in range(T)], blocks[0], BLOCK_SIZE, max_len, 0)
+                inp["slot_mapping"] = inp["slot_mapping"][:, :T].contiguous()
+                for _ in range(3):
+                    m.forward_tokens(**inp)
+                times = []
+                for _ in range(max(args.steps // 4, 8)):
+                    t = time.perf_counter()
+                    m.forward_tokens(**inp)
+                    times.append(time.perf_counter() - t)
+                m.profile_enable(True)
+                m.forward_tokens(**inp)
+                prof = m.profile_read()["ms"]
+                m.profile_enable(False)
+                ms = statistics.median(times) * 1e3
+                flops = {"gemm": 2.0 * T * layers * per_layer, "attn_prefill": 4.0 * layers * nh * hd * keys_seen(0, T, window)}
+                frac = {k: round(f / (prof[k] * 1e-3) / 1e12 / MFMA_BF16_PEAK_TFLOPS, 4) for k, f in flops.items() if prof[k] > 0}
+                size["prefill"].append({"model": name, "tokens": T, "ms": round(ms, 3), "tokens_per_s": round(T / ms * 1e3),
+                                        "class_ms": {k: round(v, 3) for k, v in prof.items() if v}, "mfma_fraction": frac})
+            for B, ctx in ((1, 1024), (4, 1024), (4, 4000), (16, 1024), (32, 1024)):
+                inp = decode_inputs(list(range(1, B + 1)), [ctx - 1] * B, blocks[:B], BLOCK_SIZE, max_len)
+                m.forward(**inp)
+                m.replay_decode(args.warmup)
+                ms = m.replay_decode(args.steps) / args.steps
+                m.profile_enable(True)
+                m.forward(**inp)
+                prof = m.profile_read()
+                m.profile_enable(False)
+                bytes_ = {"gemv": prof["gemv_weight_bytes"], "attn_decode": 4.0 * B * min(ctx, window) * nkv * hd * layers}
+                frac = {k: round(b / (prof["ms"][k] * 1e-3) / 1e9 / HBM_PEAK_GBS, 4) for k, b in bytes_.items() if prof["ms"][k] > 0}
+                gemv = m.replay_decode_classes(args.steps, ["gemv"]) / args.steps
+                attn = m.replay_decode_classes(args.steps, ["attn_decode"]) / args.steps
+                frac_graph = {k: round(b / (t * 1e-3) / 1e9 / HBM_PEAK_GBS, 4) for (k, b), t in zip(bytes_.items(), (gemv, attn)) if t > 0}
+                size["decode"].append({"model": name, "batch": B, "context": ctx, "ms": round(ms, 4), "tokens_per_s": round(B / ms * 1e3),
+                                       "class_ms_in_graph": {"gemv": round(gemv, 4), "attn_decode": round(attn, 4),
+                                                             "rest": round(ms - gemv - attn, 4)},
+                                       "launches": {k: v for k, v in prof["launches"].items() if v},
+                                       "hbm_fraction": frac_graph, "hbm_fraction_eager": frac})
+            m.close()
+        for table, key, fr in (("prefill", "tokens", "mfma_fraction"), ("decode", ("batch", "context"), "hbm_fraction")):
+            at = (lambda r: r[key]) if isinstance(key, str) else (lambda r: tuple(r[k] for k in key))
+            base = {at(r): r for r in size[table] if r["model"] == "llama"}
+            for r in size[table]:
+                if r["model"] != "llama":
+                    b = base[at(r)]
+                    r["distance"] = {k: round(b[fr][k] / v, 2) for k, v in r[fr].items() if k in b[fr] and v > 0}
+                    r["vs_llama_tokens_per_s"] = round(r["tokens_per_s"] / b["tokens_per_s"], 3)
+        out.append(size)
+    print(json.dumps({"metric": "Vimesun prefill / decode beside a Llama of equal size", "dtype": "bf16", "data": "synthetic",
+                      "higher_is_better": True, "steps": args.steps, "warmup": args.warmup, "n_gpus": 1, "sizes": out}), flush=True)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -283,7 +387,11 @@ def main():
     ap.add_argument("--tp-transport", default="p2p", choices=["p2p", "rccl"])
     ap.add_argument("--tp-loopback", action="store_true",
                     help="dev: place every rank shard of --gpus N on GPU 0 (functional check of the TP path on one GPU)")
+    ap.add_argument("--vimesun", action="store_true",
+                    help="instead of the headline workload: the Vimesun layer stack beside a Llama of equal size, both bf16")
     args = ap.parse_args()
+    if args.vimesun:
+        return vimesun_section(args)
     wd = args.weight_dtype or ("int8" if args.model == "qwen25_7b" else "f8e4m3")
     HF = MODELS[args.model]
 

@@ -1578,7 +1578,7 @@ int mi_forward_spec(mi_ctx* t, mi_ctx* d, int32_t B, int32_t k, const int64_t* i
   auto slot_of = [&](int b, int64_t p) { return block_table[(size_t)b * MB + p / bs] * bs + p % bs; };
   static const bool shared_cols = [] { const char* v = getenv("MI355X_SPEC_SHARED_ATTN"); return !v || v[0] != '0'; }();
   // the k rows of a sequence share the attention's MFMA columns where they fit (q heads per kv head x k <= 16)
-  const int rows_per_seq = (shared_cols && (t0->nh_l / t0->nkv_l) * k <= 16) ? k : 1;
+  const int rows_per_seq = (shared_cols && !t0->stack && (t0->nh_l / t0->nkv_l) * k <= 16) ? k : 1;
 
   // every shard: its copy of the B * k candidate rows (ids of candidates 1.. arrive on the device)
   auto stage_target = [&](mi_ctx* rc) -> int {

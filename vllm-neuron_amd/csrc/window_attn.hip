@@ -92,7 +92,7 @@ template <int DK, int DV>
 constexpr size_t prefill_lds() { return (size_t)64 * (DK + 8 + DV + 8) * 2; }
 
 template <int DK, int DV, int NCG>
-__global__ __launch_bounds__(256) void attn_window_prefill_kernel(AttnSpec a, const uint16_t* __restrict__ q, const uint16_t* __restrict__ kpool,
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(NCG == 1 ? 1 : 2, NCG == 1 ? 1 : 2))) void attn_window_prefill_kernel(AttnSpec a, const uint16_t* __restrict__ q, const uint16_t* __restrict__ kpool,
                                                                   const uint16_t* __restrict__ vpool, int bs, const int32_t* __restrict__ bt,
                                                                   int MB, const AttnSeg* __restrict__ segs, int nseg,
                                                                   uint16_t* __restrict__ out, int ldo) {

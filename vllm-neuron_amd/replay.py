@@ -21,17 +21,27 @@ MAX_LIVE_REQUESTS = 4
 
 
 class TraceReplay:
-    def __init__(self, model_dir: str, dtype: str, max_tokens: int):
-        from .engine import MI355XEngine
+    """`engine`: a chunked-prefill MI355XEngine without prefix caching (every token brought is computed)."""
+
+    def __init__(self, engine):
+        self.engine = engine
+        self.live: set = set()
+
+    @classmethod
+    def from_dir(cls, model_dir: str, dtype: str, max_tokens: int, max_live: int = MAX_LIVE_REQUESTS):
         from .models import load_config
-        config = load_config(model_dir)
-        self.engine = MI355XEngine(
-            config, model_dir, dtype=dtype, max_model_len=config.max_position_embeddings, max_num_seqs=MAX_LIVE_REQUESTS,
-            block_size=BLOCK_SIZE, num_gpu_blocks_override=-(-max_tokens // BLOCK_SIZE), enable_prefix_caching=False,
+        return cls.from_config(load_config(model_dir), dtype, max_tokens, max_live, model=model_dir)
+
+    @classmethod
+    def from_config(cls, config, dtype: str, max_tokens: int, max_live: int = MAX_LIVE_REQUESTS, block_size: int = BLOCK_SIZE,
+                    model: str = "", override: dict | None = None):
+        from .engine import MI355XEngine
+        return cls(MI355XEngine(
+            config, model, dtype=dtype, max_model_len=config.max_position_embeddings, max_num_seqs=max_live,
+            block_size=block_size, num_gpu_blocks_override=-(-max_tokens // block_size), enable_prefix_caching=False,
             enable_chunked_prefill=True, max_num_batched_tokens=max_tokens,
             override_mi355x_config={"is_block_kv_layout": True, "weight_artifacts": False, "kv_overcommit": True,
-                                    "chunked_prefill_config": {"max_num_seqs": MAX_LIVE_REQUESTS}})
-        self.live: set = set()
+                                    "chunked_prefill_config": {"max_num_seqs": max_live}, **(override or {})}))
 
     def step(self, entries: list, end: list):
         """-> the wanted logits, one [len(want), vocab] tensor per entry"""
@@ -60,7 +70,7 @@ def main(argv=None) -> int:
     ap.add_argument("--out", required=True, help="folder for <step>.f32 files")
     ap.add_argument("--max-tokens", type=int, required=True, help="most tokens live requests hold at any time (sizes the KV pool)")
     args = ap.parse_args(argv)
-    replay = TraceReplay(args.model, args.dtype, args.max_tokens)
+    replay = TraceReplay.from_dir(args.model, args.dtype, args.max_tokens)
     for line in sys.stdin:
         if not line.strip():
             continue

@@ -195,9 +195,24 @@ def test_window_attention(lib, H, G, dk, dv, window, bs, f32, path):
 @pytest.mark.parametrize("f32,path", PATHS)
 @pytest.mark.parametrize("bias,sink", [(0, 0), (1, 0), (0, 1)])
 def test_bias_and_sink_are_options(lib, bias, sink, f32, path):
-    spec = spec_of(lib, 6, 3, 48, 32, 50, 0.3, bias=bias, sink=sink)
+    spec = spec_of(lib, 6, 3, 48, 32, 50, 0.3, bias=bias, sink=sink, unit=bias)     # unit = 0: the running-maximum softmax
     got, ref = Paged(6, 3, 48, 32, SEGS, 16, seed=5).run(lib, spec, V.slopes(6), f32, path)
     assert ((got - ref).abs() <= (2e-5 if f32 else 1.5e-2) * (1 + ref.abs())).all()
+
+
+@pytest.mark.parametrize("f32,path", PATHS)
+@pytest.mark.parametrize("top,unit", [(40.0, 1), (90.0, 1), (700.0, 1), (60.0, 0)])
+def test_large_scores(lib, top, unit, f32, path):
+    """Scores up to `top` and down to -top: within and beyond what a fixed softmax reference can span; unit = 0 says nothing
+    about the heads' size, so q may be anything."""
+    p = Paged(4, 2, 64, 64, SEGS, 16, seed=16, q_gain=1.0 if unit else 3.0)
+    for i in range(len(p.k)):
+        for t in range(0, p.k[i].shape[0], 3):             # exact matches and exact opposites among the random keys
+            p.k[i][t] = V.unit_rms(p.q[i][t, ::2], 1e-6) * (1 if t % 2 else -1)
+    spec = spec_of(lib, 4, 2, 64, 64, 90, top / 64, unit=unit)
+    got, ref = p.run(lib, spec, V.slopes(4), f32, path)
+    # (the error of a score grows with its size)
+    assert ((got - ref).abs() <= (1e-3 if f32 else 3e-2) * (1 + ref.abs())).all(), (got - ref).abs().max()
 
 
 @pytest.mark.parametrize("f32,path", PATHS)

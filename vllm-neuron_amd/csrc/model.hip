@@ -1959,7 +1959,7 @@ int mi_op_window_attn(const mi_layer_spec* spec, const float* slopes, const void
                       int32_t path, void* stream) {
   MI_CHECK(spec && q && kpool && vpool && block_table && pos && ctx_lens && segs_host && out && nseg >= 1 && T >= 1, "null argument");
   MI_CHECK(!spec->distance_bias || slopes, "distance bias without slopes");
-  const AttnSpec a{head_geom(*spec), spec->scale, spec->window, spec->distance_bias ? slopes : nullptr, spec->softmax_sink ? 1 : 0};
+  const AttnSpec a{head_geom(*spec), spec->scale, spec->window, spec->distance_bias ? slopes : nullptr, spec->qk_unit_norm ? 1 : 0, spec->softmax_sink ? 1 : 0};
   std::vector<AttnSeg> segs((size_t)nseg);
   memcpy(segs.data(), segs_host, (size_t)nseg * sizeof(AttnSeg));
   int row = 0;

@@ -184,7 +184,7 @@ int stack_create(mi_ctx* c, const mi_stack_config& cfg) {
       MI_HIP(hipMemcpyAsync(W.slopes, sl.data(), sl.size() * 4, hipMemcpyHostToDevice, c->stream));
       MI_HIP(hipStreamSynchronize(c->stream));
     }
-    W.attn = AttnSpec{W.g, s.scale, s.window, W.slopes, s.softmax_sink ? 1 : 0};
+    W.attn = AttnSpec{W.g, s.scale, s.window, W.slopes, s.qk_unit_norm ? 1 : 0, s.softmax_sink ? 1 : 0};
     S->qkv_ld = std::max(S->qkv_ld, W.qkv.N);
     S->q_cols = std::max(S->q_cols, s.num_heads * W.g.dkp);
     S->cat_ld = std::max(S->cat_ld, W.out.K);

@@ -14,6 +14,7 @@ struct AttnSpec {
   float scale = 1.f;
   int window = 0;                  // keys a query sees, itself included; 0 = every earlier token
   const float* slopes = nullptr;   // [H] or null: no distance bias
+  int unit_norm = 0;               // q and k heads have unit root mean square: |q.k| <= dk
   int sink = 0;                    // 1: one more score of 0 in the denominator, without a value
 };
 struct AttnSeg { int row0, n, pos0, seq; };   // rows row0 .. + n of the batch = positions pos0 .. of the sequence in block-table row seq

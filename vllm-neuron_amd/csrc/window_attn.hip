@@ -88,25 +88,35 @@ __global__ __launch_bounds__(64) void attn_plain_kernel(AttnSpec a, const T* __r
 // =====================================================================================
 // 4 waves x NCG column groups of 16.  64-key tiles of K and V go through LDS (registers hold the next tile while the
 // current one is multiplied; the block ids run one tile further ahead).
+//
+// The softmax is VALU-bound (the exponential alone costs as much as the score's MFMAs), so it is kept short:
+//   * FIXED: the scores are bounded from above by s_max (unit-norm queries and keys: |q.k| <= dk; the bias only lowers a
+//     score), so exp2(s - s_max) needs no running maximum, no rescaling and no cross-lane step; the reference point is folded
+//     into the bias.  Taken where s_max is small enough for fp32's exponent range (fixed_reference below).
+//   * The denominator is one more row of the P.V product (A = ones): it sums what the numerator multiplies.
+// Row pitch dk + 16 / dv + 16 elements: fragment reads and transposed reads are bank-conflict-free (as in attn_kernels.hip).
+constexpr int kPitch = 16;
 template <int DK, int DV>
-constexpr size_t prefill_lds() { return (size_t)64 * (DK + 8 + DV + 8) * 2; }
+constexpr size_t prefill_lds() { return (size_t)64 * (DK + kPitch + DV + kPitch) * 2; }
 
-template <int DK, int DV, int NCG>
+template <int DK, int DV, int NCG, bool FIXED>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(NCG == 1 ? 1 : 2, NCG == 1 ? 1 : 2))) void attn_window_prefill_kernel(AttnSpec a, const uint16_t* __restrict__ q, const uint16_t* __restrict__ kpool,
                                                                   const uint16_t* __restrict__ vpool, int bs, const int32_t* __restrict__ bt,
                                                                   int MB, const AttnSeg* __restrict__ segs, int nseg,
-                                                                  uint16_t* __restrict__ out, int ldo) {
-  constexpr int KP = DK + 8, VP = DV + 8;              // LDS row pitches (elements)
+                                                                  uint16_t* __restrict__ out, int ldo, float s_max, int fold) {
+  constexpr int KP = DK + kPitch, VP = DV + kPitch;    // LDS row pitches (elements)
   constexpr int KS = DK / 32, DN = DV / 16, KCH = DK / 8, VCH = DV / 8;
   constexpr int NKL = 64 * KCH / 256, NVL = 64 * VCH / 256;   // 16-byte loads per thread and tile
   extern __shared__ __attribute__((aligned(16))) unsigned char dsm[];
   uint16_t* Ks = reinterpret_cast<uint16_t*>(dsm);
   uint16_t* Vs = Ks + 64 * KP;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g4 = lane >> 4, c = lane & 15;
-  const int H = a.g.H, G = a.g.G, r = H / G, qpt = (64 * NCG) / r, kvh = blockIdx.y;
+  const int H = a.g.H, G = a.g.G, r = H / G, qpt = (64 * NCG) / r, kvh = blockIdx.x;
 
-  // this work-group's tile: segments with one row belong to the token-generation kernel.  Late tiles (long contexts) first.
-  int t = (int)(gridDim.x - 1 - blockIdx.x), si = 0;
+  // this work-group's tile: segments with one row belong to the token-generation kernel.  Late tiles (long contexts) first; a
+  // grid that is resident at once deals its second half in ascending order, so that a CU's two work-groups add up evenly.
+  const int nty = (int)gridDim.y, ty = (int)blockIdx.y;
+  int t = (fold && ty >= (nty + 1) / 2) ? ty - (nty + 1) / 2 : nty - 1 - ty, si = 0;
   AttnSeg sg{0, 0, 0, 0};
   for (; si < nseg; ++si) {
     sg = segs[si];
@@ -154,17 +164,18 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(NCG == 1 ? 
 
   // columns: position, bias slope, query fragments (zero beyond dkp and in dead columns)
   int pc[NCG];
-  float sl2[NCG], mrow[NCG], lrow[NCG];
+  float sl2[NCG], mrow[NCG];
   u32x4_t qf[NCG][KS];
-  f32x4_t acc[NCG][DN];
+  f32x4_t acc[NCG][DN], den[NCG];     // den: the column's denominator, the same in every row
 #pragma unroll
   for (int cg = 0; cg < NCG; ++cg) {
     const int col = (wave * NCG + cg) * 16 + c, ql = col / r, h = kvh * r + col % r;
     const bool live = ql < nq && ql < qpt;
     pc[cg] = pos0 + (live ? ql : 0);
     sl2[cg] = a.slopes ? a.slopes[h] * kLog2e : 0.f;
-    mrow[cg] = a.sink ? 0.f : -INFINITY;
-    lrow[cg] = (a.sink && g4 == 0) ? 1.f : 0.f;
+    mrow[cg] = FIXED ? s_max : (a.sink ? 0.f : -INFINITY);
+    const float d0 = a.sink ? (FIXED ? fexp2(-s_max) : 1.f) : 0.f;
+    den[cg] = f32x4_t{d0, d0, d0, d0};
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks)
       qf[cg][ks] = (live && ks * 32 + g4 * 8 < a.g.dkp) ? *reinterpret_cast<const u32x4_t*>(q + ((size_t)(row0 + ql) * H + h) * a.g.dkp + ks * 32 + g4 * 8)
@@ -178,6 +189,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(NCG == 1 ? 
   const bool wave_live = wq0 < nq;
   const int pmin = pos0 + wq0, pmax = pos0 + wq1;
   const int tr_row = (lane & 15) >> 2, tr_col = (lane & 3) * 4;
+  const short one = 0x3f80;            // bf16 1.0
+  const bf16x8_t ones = {one, one, one, one, one, one, one, one};
 
   for (int n = 0; n < nt; ++n) {
     const int k0 = klo + 64 * n;
@@ -215,48 +228,54 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(NCG == 1 ? 
     union { uint32_t w[4]; bf16x8_t v; } pk[NCG][2];
 #pragma unroll
     for (int cg = 0; cg < NCG; ++cg) {
-      const float b0 = sl2[cg] * (float)(k0 + 4 * g4 - pc[cg]);     // - slope (i - j), the lane's first key
-      float mx = -INFINITY;
+      // - slope (i - j) of the lane's first key (- the fixed reference)
+      const float b0 = __builtin_fmaf(sl2[cg], (float)(k0 + 4 * g4 - pc[cg]), FIXED ? -s_max : 0.f);
 #pragma unroll
       for (int u = 0; u < 4; ++u)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          float sv = __builtin_fmaf(st[cg][u][i], sc2, __builtin_fmaf(sl2[cg], (float)(16 * u + i), b0));
-          if (edge) {
-            const int j = k0 + 16 * u + 4 * g4 + i;
-            if (j > pc[cg] || j <= pc[cg] - win) sv = -INFINITY;
+        for (int i = 0; i < 4; ++i)
+          st[cg][u][i] = __builtin_fmaf(st[cg][u][i], sc2, __builtin_fmaf(sl2[cg], (float)(16 * u + i), b0));
+      if (edge) {
+        const int j0 = k0 + 4 * g4;
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const int back = pc[cg] - (j0 + 16 * u + i);
+            if ((unsigned)back >= (unsigned)win) st[cg][u][i] = -INFINITY;   // ahead of the query, or out of its window
           }
-          st[cg][u][i] = sv;
-          mx = fmaxf(mx, sv);
-        }
-      mx = fmaxf(mx, __shfl_xor(mx, 16));
-      mx = fmaxf(mx, __shfl_xor(mx, 32));
-      const float mn = fmaxf(mrow[cg], mx);
-      const float alpha = sexp2(mrow[cg], mn);
-      const bool moved = mn != mrow[cg];
-      mrow[cg] = mn;
-      const float ms = mn == -INFINITY ? 0.f : mn;   // (a column without a key so far: every score is -inf, exp2 gives 0)
-      float ps = 0.f;
+      }
+      float ms = 0.f;
+      if constexpr (!FIXED) {
+        float mx = -INFINITY;
 #pragma unroll
-      for (int u = 0; u < 4; ++u)
+        for (int u = 0; u < 4; ++u)
+          mx = fmaxf(fmaxf(fmaxf(mx, st[cg][u][0]), fmaxf(st[cg][u][1], st[cg][u][2])), st[cg][u][3]);
+        mx = fmaxf(mx, __shfl_xor(mx, 16));
+        mx = fmaxf(mx, __shfl_xor(mx, 32));
+        const float mn = fmaxf(mrow[cg], mx);
+        const float alpha = sexp2(mrow[cg], mn);
+        const bool moved = mn != mrow[cg];
+        mrow[cg] = mn;
+        ms = mn == -INFINITY ? 0.f : mn;   // (a column without a key so far: every score is -inf, exp2 gives 0)
+        if (__any(moved)) {
+          den[cg][0] *= alpha; den[cg][1] *= alpha; den[cg][2] *= alpha; den[cg][3] *= alpha;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const float e = fexp2(st[cg][u][i] - ms);
-          st[cg][u][i] = e;
-          ps += e;
+          for (int dn = 0; dn < DN; ++dn) {
+            acc[cg][dn][0] *= alpha; acc[cg][dn][1] *= alpha; acc[cg][dn][2] *= alpha; acc[cg][dn][3] *= alpha;
+          }
         }
-      lrow[cg] = lrow[cg] * alpha + ps;
+      }
 #pragma unroll
       for (int u = 0; u < 4; ++u) {
-        pk[cg][u >> 1].w[(u & 1) * 2] = pack_bf16x2(st[cg][u][0], st[cg][u][1]);
-        pk[cg][u >> 1].w[(u & 1) * 2 + 1] = pack_bf16x2(st[cg][u][2], st[cg][u][3]);
-      }
-      if (__any(moved)) {
+        float e[4];
 #pragma unroll
-        for (int dn = 0; dn < DN; ++dn) {
-          acc[cg][dn][0] *= alpha; acc[cg][dn][1] *= alpha; acc[cg][dn][2] *= alpha; acc[cg][dn][3] *= alpha;
-        }
+        for (int i = 0; i < 4; ++i) e[i] = FIXED ? fexp2(st[cg][u][i]) : fexp2(st[cg][u][i] - ms);
+        pk[cg][u >> 1].w[(u & 1) * 2] = pack_bf16x2(e[0], e[1]);
+        pk[cg][u >> 1].w[(u & 1) * 2 + 1] = pack_bf16x2(e[2], e[3]);
       }
+#pragma unroll
+      for (int hf = 0; hf < 2; ++hf) den[cg] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pk[cg][hf].v, den[cg], 0, 0, 0);
     }
     // O^T += V^T.P^T: the k-slot (g4, j) of a 32-key half is key (j < 4 ? 4 g4 + j : 16 + 4 g4 + j - 4)
 #pragma unroll
@@ -274,9 +293,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(NCG == 1 ? 
 
 #pragma unroll
   for (int cg = 0; cg < NCG; ++cg) {
-    float L = lrow[cg];
-    L += __shfl_xor(L, 16);
-    L += __shfl_xor(L, 32);
+    const float L = den[cg][0];
     const int col = (wave * NCG + cg) * 16 + c, ql = col / r, h = kvh * r + col % r;
     if (ql >= nq || ql >= qpt) continue;
     const float inv = L > 0.f ? 1.f / L : 0.f;
@@ -540,6 +557,14 @@ int launch_decode_t(const AttnSpec& a, const uint16_t* q, const uint16_t* kpool,
   return MI_OK;
 }
 
+// FIXED softmax reference (exp2 domain): unit-norm heads bound the score by |scale| dk, 1 % for the rounding of q and k to bf16.
+// Up to 2^+-60 around it every weight that matters stays a normal fp32 number: the lowest unbiased score is 2^-120 of the
+// reference, and the sink (score 0) 2^-60.  0: not applicable, the running maximum is used.
+float fixed_reference(const AttnSpec& a) {
+  const float b = fabsf(a.scale) * (float)a.g.dk * 1.01f * kLog2e;
+  return a.unit_norm && b <= 60.f && b > 0.f ? b : 0.f;
+}
+
 template <int DK, int DV, int NCG>
 int launch_prefill_t(const AttnSpec& a, const uint16_t* q, const uint16_t* kpool, const uint16_t* vpool, int bs, const int32_t* bt, int MB,
                      const AttnSeg* sd, const AttnSeg* sh, int nseg, uint16_t* out, int ldo, hipStream_t s) {
@@ -548,9 +573,14 @@ int launch_prefill_t(const AttnSpec& a, const uint16_t* q, const uint16_t* kpool
   for (int i = 0; i < nseg; ++i) tiles += sh[i].n > 1 ? ceil_div(sh[i].n, qpt) : 0;
   if (tiles == 0) return MI_OK;
   constexpr size_t lds = prefill_lds<DK, DV>();
-  auto kern = attn_window_prefill_kernel<DK, DV, NCG>;
+  const float s_max = fixed_reference(a);
+  int num_cu = 0;
+  { int rc = device_num_cu(&num_cu); if (rc != MI_OK) return rc; }
+  const int fold = tiles * a.g.G <= 2 * num_cu;
+  auto kern = s_max > 0.f ? attn_window_prefill_kernel<DK, DV, NCG, true> : attn_window_prefill_kernel<DK, DV, NCG, false>;
   if (lds > 64 * 1024) { int rc = ensure_dynamic_lds(reinterpret_cast<const void*>(kern), (int)lds); if (rc != MI_OK) return rc; }
-  hipLaunchKernelGGL(kern, dim3(tiles, a.g.G), dim3(256), lds, s, a, q, kpool, vpool, bs, bt, MB, sd, nseg, out, ldo);
+  // kv head fastest: consecutive work-groups (one per XCD) read different heads, a head's tiles meet in one L2
+  hipLaunchKernelGGL(kern, dim3(a.g.G, tiles), dim3(256), lds, s, a, q, kpool, vpool, bs, bt, MB, sd, nseg, out, ldo, s_max, fold);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }

@@ -360,14 +360,16 @@ def vimesun_section(args):
                                        "launches": {k: v for k, v in prof["launches"].items() if v},
                                        "hbm_fraction": frac_graph, "hbm_fraction_eager": frac})
             m.close()
-        for table, key, fr in (("prefill", "tokens", "mfma_fraction"), ("decode", ("batch", "context"), "hbm_fraction")):
-            at = (lambda r: r[key]) if isinstance(key, str) else (lambda r: tuple(r[k] for k in key))
-            base = {at(r): r for r in size[table] if r["model"] == "llama"}
+        for table, fr in (("prefill", "mfma_fraction"), ("decode", "hbm_fraction")):
+            base = {(r.get("tokens"), r.get("batch"), r.get("context")): r for r in size[table] if r["model"] == "llama"}
             for r in size[table]:
-                if r["model"] != "llama":
-                    b = base[at(r)]
-                    r["distance"] = {k: round(b[fr][k] / v, 2) for k, v in r[fr].items() if k in b[fr] and v > 0}
-                    r["vs_llama_tokens_per_s"] = round(r["tokens_per_s"] / b["tokens_per_s"], 3)
+                if r["model"] == "llama":
+                    continue
+                b = base[r.get("tokens"), r.get("batch"), r.get("context")]
+                r["vs_llama_tokens_per_s"] = round(r["tokens_per_s"] / b["tokens_per_s"], 3)
+                if "window" in r["model"] and r.get("context", 0) > VIMESUN_WINDOW:     # the Llama step that reads as many keys
+                    b = base[None, r["batch"], VIMESUN_WINDOW]
+                r["distance"] = {k: round(b[fr][k] / v, 2) for k, v in r[fr].items() if k in b[fr] and v > 0}
         out.append(size)
     print(json.dumps({"metric": "Vimesun prefill / decode beside a Llama of equal size", "dtype": "bf16", "data": "synthetic",
                       "higher_is_better": True, "steps": args.steps, "warmup": args.warmup, "n_gpus": 1, "sizes": out}), flush=True)

@@ -1,6 +1,8 @@
 // Row-wise kernels of the layer-stack decoders.  See stack_kernels.h.
 #include "stack_kernels.h"
 
+#include <algorithm>
+
 #include "misc_kernels.h"
 
 namespace mi {
@@ -14,12 +16,20 @@ __device__ __forceinline__ void put4(uint16_t* p, float a, float b, float c, flo
 }
 __device__ __forceinline__ void put4(float* p, float a, float b, float c, float d) { *reinterpret_cast<float4*>(p) = make_float4(a, b, c, d); }
 
-// sum over the work-group (256 threads); `red` has one float per wave and is free again after the next barrier
+__device__ __forceinline__ float4 get4(const uint16_t* p) {
+  const uint2 v = *reinterpret_cast<const uint2*>(p);
+  return make_float4(bf16lo_to_f32(v.x), bf16hi_to_f32(v.x), bf16lo_to_f32(v.y), bf16hi_to_f32(v.y));
+}
+__device__ __forceinline__ float4 get4(const float* p) { return *reinterpret_cast<const float4*>(p); }
+
+// sum over the work-group (up to 16 waves), in wave order; `red` has 16 floats and is free again after the next barrier
 __device__ __forceinline__ float block_sum(float v, float* red) {
   v = wave_sum(v);
   if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
   __syncthreads();
-  return (red[0] + red[1]) + (red[2] + red[3]);
+  float t = 0.f;
+  for (int w = 0; w < (int)(blockDim.x >> 6); ++w) t += red[w];
+  return t;
 }
 
 template <typename T>
@@ -29,22 +39,33 @@ __global__ __launch_bounds__(256) void embed_pos_kernel(const int32_t* __restric
   const int t = blockIdx.x;
   const T* e = table + (size_t)ids[t] * D;
   const T* p = ptable + (size_t)pos[t] * D;
-  for (int d = threadIdx.x; d < ld; d += 256) {
-    const float v = d < D ? to_f32(e[d]) + to_f32(p[d]) : 0.f;
-    resid[(size_t)t * ld + d] = v;
-    if (x0) x0[(size_t)t * ld + d] = v;
+  for (int d = threadIdx.x * 4; d < ld; d += 1024) {
+    float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+    if ((D & 3) == 0) {
+      if (d < D) {
+        const float4 a = get4(e + d), b = get4(p + d);
+        v = make_float4(a.x + b.x, a.y + b.y, a.z + b.z, a.w + b.w);
+      }
+    } else {
+      if (d < D) v.x = to_f32(e[d]) + to_f32(p[d]);
+      if (d + 1 < D) v.y = to_f32(e[d + 1]) + to_f32(p[d + 1]);
+      if (d + 2 < D) v.z = to_f32(e[d + 2]) + to_f32(p[d + 2]);
+      if (d + 3 < D) v.w = to_f32(e[d + 3]) + to_f32(p[d + 3]);
+    }
+    *reinterpret_cast<float4*>(resid + (size_t)t * ld + d) = v;
+    if (x0) *reinterpret_cast<float4*>(x0 + (size_t)t * ld + d) = v;
   }
 }
 
 template <typename T>
-__global__ __launch_bounds__(256) void layernorm_rows_kernel(const float* __restrict__ resid_in, float* __restrict__ resid_out,
+__global__ __launch_bounds__(1024) void layernorm_rows_kernel(const float* __restrict__ resid_in, float* __restrict__ resid_out,
                                                              int D, int ld, float eps, NormOut na, NormOut nb, int ldy, SlabSum sl) {
-  extern __shared__ __attribute__((aligned(16))) float hrow[];  // ld floats + 8
-  const int t = blockIdx.x, tid = threadIdx.x;
+  extern __shared__ __attribute__((aligned(16))) float hrow[];  // ld floats + 32
+  const int t = blockIdx.x, tid = threadIdx.x, nthr = blockDim.x;
   const size_t o = (size_t)t * ld;
   float* red = hrow + ld;
   float sum = 0.f;
-  for (int c4 = tid; c4 < ld / 4; c4 += 256) {
+  for (int c4 = tid; c4 < ld / 4; c4 += nthr) {
     float4 a = *reinterpret_cast<const float4*>(resid_in + o + c4 * 4);
     if (sl.slab) {   // slabs in slice order, scale, + residual: the arithmetic of splitk_reduce + the residual epilogue
       float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
@@ -61,7 +82,7 @@ __global__ __launch_bounds__(256) void layernorm_rows_kernel(const float* __rest
   }
   const float mean = block_sum(sum, red) / (float)D;
   float ss = 0.f;
-  for (int c4 = tid; c4 < ld / 4; c4 += 256) {   // (a thread reads back what it wrote itself)
+  for (int c4 = tid; c4 < ld / 4; c4 += nthr) {   // (a thread reads back what it wrote itself)
     float4 a = *reinterpret_cast<const float4*>(hrow + c4 * 4);
     const int d = c4 * 4;
     a.x = d < D ? a.x - mean : 0.f;
@@ -71,8 +92,8 @@ __global__ __launch_bounds__(256) void layernorm_rows_kernel(const float* __rest
     *reinterpret_cast<float4*>(hrow + c4 * 4) = a;
     ss += (a.x * a.x + a.y * a.y) + (a.z * a.z + a.w * a.w);
   }
-  const float rstd = 1.0f / sqrtf(block_sum(ss, red + 4) / (float)D + eps);
-  for (int c4 = tid; c4 < ld / 4; c4 += 256) {
+  const float rstd = 1.0f / sqrtf(block_sum(ss, red + 16) / (float)D + eps);
+  for (int c4 = tid; c4 < ld / 4; c4 += nthr) {
     const float4 a = *reinterpret_cast<const float4*>(hrow + c4 * 4);
     auto emit = [&](const NormOut& n) {
       const float4 w = *reinterpret_cast<const float4*>(n.w + c4 * 4), b = *reinterpret_cast<const float4*>(n.b + c4 * 4);
@@ -225,13 +246,15 @@ int launch_layernorm_rows(const float* resid_in, float* resid_out, int T, int D,
                           const NormOut& b, int ldy, bool f32, hipStream_t s, const SlabSum* slabs) {
   MI_CHECK(ld % 4 == 0 && ld >= D && ld <= 32768 && ldy >= ld, "layer norm: row stride must be a multiple of 4, at least the width, at most 32768");
   MI_CHECK(!slabs || (slabs->T == T && slabs->N == ld && resid_out && !slabs->bias && !slabs->row_scale), "layer norm: pending K-split sum of another shape");
-  const size_t lds = (size_t)(ld + 8) * sizeof(float);
+  const size_t lds = (size_t)(ld + 32) * sizeof(float);
+  // few rows (token generation): one float4 per thread, the row is one round of loads; many rows: 256 threads, several rows per CU
+  const int threads = T <= 32 ? std::min(1024, ceil_div(ld / 4, 64) * 64) : 256;
   const SlabSum sl = slabs ? *slabs : SlabSum();
   if (lds > 64 * 1024)
     MI_HIP(f32 ? hipFuncSetAttribute(reinterpret_cast<const void*>(layernorm_rows_kernel<float>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds)
                : hipFuncSetAttribute(reinterpret_cast<const void*>(layernorm_rows_kernel<uint16_t>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
-  if (f32) hipLaunchKernelGGL((layernorm_rows_kernel<float>), dim3(T), dim3(256), lds, s, resid_in, resid_out, D, ld, eps, a, b, ldy, sl);
-  else hipLaunchKernelGGL((layernorm_rows_kernel<uint16_t>), dim3(T), dim3(256), lds, s, resid_in, resid_out, D, ld, eps, a, b, ldy, sl);
+  if (f32) hipLaunchKernelGGL((layernorm_rows_kernel<float>), dim3(T), dim3(threads), lds, s, resid_in, resid_out, D, ld, eps, a, b, ldy, sl);
+  else hipLaunchKernelGGL((layernorm_rows_kernel<uint16_t>), dim3(T), dim3(threads), lds, s, resid_in, resid_out, D, ld, eps, a, b, ldy, sl);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }

@@ -541,6 +541,21 @@ def test_trace_run_command(tmp_path, monkeypatch, capsys, dtype):
     assert error(read(7), torch.stack([rb[19], ra[30], ra[49]])) <= LIMIT[dtype]
 
 
+@pytest.mark.parametrize("chunk", [0, 24])
+def test_generate_command(tmp_path, capsys, chunk):
+    from vllm_neuron_amd.generate import main
+    cfg = CASES["looped"]()
+    w = weights(cfg, 5)
+    write_model(tmp_path / "m", cfg, w)
+    prompts = [tokens(cfg, 40, 1), tokens(cfg, 3, 2)]
+    argv = ["--model", str(tmp_path / "m"), "--dtype", "float32", "--max-tokens", "6", "--block-size", "16", "--chunked-prefill", str(chunk)]
+    for p in prompts:
+        argv += ["--prompt", ",".join(map(str, p))]
+    assert main(argv) == 0
+    lines = [json.loads(x) for x in capsys.readouterr().out.splitlines() if x.startswith("{")]
+    assert [x["tokens"] for x in lines] == [greedy(cfg, w, p, 6) for p in prompts]
+
+
 def test_weight_artifacts_round_trip(tmp_path):
     """A served checkpoint folder keeps its device images; the second start loads them and answers the same."""
     from vllm_neuron_amd._vllm_compat import SamplingParams

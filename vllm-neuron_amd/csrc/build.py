@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Build libmi355x_vllm.so for gfx950 with hipcc (cross-compiles without a GPU).
 
-    python vllm-neuron_amd/csrc/build.py [--force]
+    python vllm-neuron_amd/csrc/build.py [--force | --if-missing]
 
 Objects go to csrc/build/, the library next to the sources (in-tree, git-ignored: it
 travels to the GPU box with the snapshot).
@@ -77,4 +77,6 @@ def build(verbose=True):
 
 
 if __name__ == "__main__":
+    if "--if-missing" in sys.argv and os.path.exists(os.environ.get("MI355X_VLLM_LIB") or LIB):
+        sys.exit(0)
     print(build())

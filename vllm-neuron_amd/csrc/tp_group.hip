@@ -440,6 +440,43 @@ int group_create(const mi_model_config& cfg, mi_ctx* facade) {
   return MI_OK;
 }
 
+// Uncached device memory is never given back to the allocator while the process lives: once a kernel has read it, memory
+// allocated after such a free has been seen to hold wrong values.  Blocks of destroyed groups are handed to the next group.
+namespace {
+std::mutex g_uncached_mu;
+std::map<void*, std::pair<int, size_t>> g_uncached;                    // every uncached block: device, bytes
+std::map<std::pair<int, size_t>, std::vector<void*>> g_uncached_idle;  // ... and those no group uses
+}  // namespace
+static int alloc_uncached(void** p, size_t bytes) {
+  int dev = 0;
+  MI_HIP(hipGetDevice(&dev));
+  std::lock_guard<std::mutex> lk(g_uncached_mu);
+  auto& idle = g_uncached_idle[{dev, bytes}];
+  if (!idle.empty()) {
+    *p = idle.back();
+    idle.pop_back();
+    return MI_OK;
+  }
+  if (hipExtMallocWithFlags(p, bytes, hipDeviceMallocUncached) != hipSuccess) {
+    (void)hipGetLastError();
+    return MI_EHIP;
+  }
+  g_uncached[*p] = {dev, bytes};
+  return MI_OK;
+}
+static void free_exchange_mem(void* p) {
+  if (!p) return;
+  {
+    std::lock_guard<std::mutex> lk(g_uncached_mu);
+    auto it = g_uncached.find(p);
+    if (it != g_uncached.end()) {
+      g_uncached_idle[it->second].push_back(p);
+      return;
+    }
+  }
+  hipFree(p);
+}
+
 void group_destroy(mi_group* g) {
   if (!g) return;
   if (!g->threads.empty()) {
@@ -453,7 +490,7 @@ void group_destroy(mi_group* g) {
         if (c && (phase == 0) == (r != 0)) {
           if (g->counters[r]) hipFree(g->counters[r]);
           void* p[] = {g->peers.xbuf[r], g->peers.ybuf[r], g->peers.flag1[r], g->peers.flag2[r]};
-          for (void* q : p) if (q) hipFree(q);
+          for (void* q : p) free_exchange_mem(q);
           mi_ctx_destroy(c);
         }
         return MI_OK;
@@ -476,10 +513,7 @@ void group_destroy(mi_group* g) {
 // the allocation read zeros for 8 KiB..64 KiB of the peers' slots in about one process in six
 // (profiles/README.md, "exchange self-test"); ordinary memory never did in the same loop.
 static int alloc_exchange_mem(void** p, size_t bytes, bool uncached) {
-  if (uncached && !getenv("MI355X_TP_FLAGS_CACHED")) {
-    if (hipExtMallocWithFlags(p, bytes, hipDeviceMallocUncached) == hipSuccess) return MI_OK;
-    (void)hipGetLastError();
-  }
+  if (uncached && !getenv("MI355X_TP_FLAGS_CACHED") && alloc_uncached(p, bytes) == MI_OK) return MI_OK;
   MI_HIP(hipMalloc(p, bytes));
   return MI_OK;
 }

@@ -94,16 +94,30 @@ typedef struct mi_model_config {
 enum { MI_TP_TRANSPORT_P2P = 0, MI_TP_TRANSPORT_RCCL = 1 };
 
 /* ---- layer-stack decoders: a decoder given layer by layer, every size and constant a parameter ----
- * (Vimesun is the first such design; the worker's model registry fills this from its config.json.)
- *     x = embed[token] + pos[position]                        fp32 residual stream
- *     layer:  x <- x + residual_mult (attention(norm1(x)) + feed-forward(norm2(x)))   both of the same x
- *     norms:  layer norm with weight and bias
+ * (Vimesun and Rapodra are such designs; the worker's model registry fills this from their config.json.)
+ *     x = embed[token] (+ pos[position])                      fp32 residual stream
+ *     block MI_BLOCK_PARALLEL:  x <- x + residual_mult (mixer(norm1 x) + ff(norm2 x))     both of the same x
+ *     block MI_BLOCK_SANDWICH:  x <- x + norm1b(mixer(C1(norm1 x))); x <- x + norm2b(ff(C2(norm2 x)))
+ *             C(h) = h + causal convolution of h over time, conv_taps taps per channel; the last conv_taps - 1 inputs h
+ *             are part of a sequence's state
+ *     norms:  norm_groups = 0: layer norm with weight and bias; else RMS norm of norm_groups equal parts, each over its
+ *             own sqrt(mean square + norm_eps), times a weight
  *     loop:   layers loop_start .. loop_stop - 1 run loop_times times in a row with the same weights, each pass with a
  *             KV pool of its own; ahead of a pass's first layer  x <- W_in [x ; embedding output]
- *     logits = head final_norm(x)
+ *     logits = head final_norm(x); logit_softcap > 0: softcap tanh(logits / softcap)
+ * Mixers: MI_MIX_ATTENTION, grouped heads with K / V pools; MI_MIX_LATENT, per head k = W_uk c, v = W_uv c of a cached latent
+ *     c = RMSnorm(W_dkv h) [kv_rank]; kv_from >= 0: the latents of that earlier layer instead of own ones.
+ * Feed-forwards: MI_FF_RELU2 down(max(up x, 0)^2); MI_FF_GLU down(act(gate x, up x)); MI_FF_MOE the softmax-weighted sum of the
+ *     experts_top experts with the largest router logits (W_router x + b), each down(act(gate x, up x)).
+ * Gated activations: MI_ACT_SILU g sigmoid(g) u; MI_ACT_SWISH_CLIP, g = min(g, limit), u within +-limit: g sigmoid(alpha g) (u + 1).
+ * Built: parallel blocks of MI_MIX_ATTENTION with layer norms, sandwich blocks of MI_MIX_LATENT with RMS norms and no loop.
  * Tensor names ("l<i>." = layer i): embed, pos, loop.in, l<i>.norm1(.b), l<i>.norm2(.b), l<i>.mix.{q,k,v,o},
- * l<i>.mlp.{up,down}, final.norm(.b), head. */
-enum { MI_FF_NONE = 0, MI_FF_RELU2 = 1 };   /* down(max(up x, 0)^2) */
+ * l<i>.mlp.{up,down}, final.norm(.b), head; sandwich blocks: l<i>.norm1, .norm1b, .norm2, .norm2b, .canon1, .canon2
+ * [width, taps], l<i>.mix.{q,dkv,dkv.norm,uk,uv,o}, l<i>.mlp.{gate,up,down}, l<i>.mlp.router(.b), l<i>.mlp.e<n>.{gate,up,down}. */
+enum { MI_BLOCK_PARALLEL = 0, MI_BLOCK_SANDWICH = 1 };
+enum { MI_MIX_ATTENTION = 0, MI_MIX_LATENT = 1 };
+enum { MI_FF_NONE = 0, MI_FF_RELU2 = 1, MI_FF_GLU = 2, MI_FF_MOE = 3 };
+enum { MI_ACT_SILU = 0, MI_ACT_SWISH_CLIP = 1 };
 typedef struct mi_layer_spec {
   int32_t num_heads, num_kv_heads, qk_dim, v_dim;
   int32_t window;         /* a query sees keys with 0 <= i - j < window; 0 = every earlier token */
@@ -111,19 +125,27 @@ typedef struct mi_layer_spec {
   int32_t qk_unit_norm;   /* q and k heads divided by sqrt(mean square + norm_eps) */
   int32_t distance_bias;  /* 2^(-8 (h + 1) / num_heads) (i - j) taken off the score of head h */
   int32_t softmax_sink;   /* one added to the softmax denominator */
-  int32_t ff_kind, ff_size;
+  int32_t ff_kind, ff_size;   /* ff_size: of one expert where there are experts */
+  int32_t mixer_kind;
+  int32_t kv_rank, kv_from;   /* MI_MIX_LATENT; kv_from = -1: own latents */
+  int32_t ff_act;             /* MI_ACT_*, gated feed-forwards and experts */
+  float ff_limit, ff_alpha;   /* MI_ACT_SWISH_CLIP */
+  int32_t experts, experts_top;
 } mi_layer_spec;
 typedef struct mi_stack_config {
   int32_t num_layers;
   const mi_layer_spec* layers;
-  int32_t width, vocab_size, max_positions;
+  int32_t width, vocab_size, max_positions;    /* max_positions = 0: no learned positions, no bound on the sequence */
   float norm_eps, residual_mult;
   int32_t loop_start, loop_stop, loop_times;   /* loop_times = 0: no loop (and no loop.in) */
   int32_t compute_dtype;   /* MI_BF16: bf16 matrix products and KV; MI_F32: everything in fp32 (plain kernels: for checking) */
+  int32_t block_kind, norm_groups;
+  int32_t conv_taps;       /* sandwich blocks: 1 .. 16 */
+  float logit_softcap;     /* 0 = none */
 } mi_stack_config;
 
 const char* mi_last_error(void);
-int mi_version(void);   /* 5 = this header (+ mi_ctx_create_stack, mi_forward_rows, mi_layer_residuals, mi_op_* of the stack kernels); 4 (+ mi_tp_plan, mi_tp_info); 3 lacked them; 2 lacked tp_device_ids / tp_transport / MI_TP_ALL_RANKS; 1 lacked mi_forward_tokens, mi_op_sample, mi_tp_init_transport */
+int mi_version(void);   /* 6 = this header (+ sandwich blocks, latent attention, experts in mi_layer_spec / mi_stack_config and their mi_op_*); 5 (+ mi_ctx_create_stack, mi_forward_rows, mi_layer_residuals, mi_op_* of the stack kernels); 4 (+ mi_tp_plan, mi_tp_info); 3 lacked them; 2 lacked tp_device_ids / tp_transport / MI_TP_ALL_RANKS; 1 lacked mi_forward_tokens, mi_op_sample, mi_tp_init_transport */
 
 int mi_ctx_create(const mi_model_config* cfg, mi_ctx** out);
 /* The same context around a layer stack.  Of cfg only the serving fields are read (pool, batch, buckets, device, graphs);

@@ -14,6 +14,8 @@ import os
 
 import torch  # noqa: F401  (must precede CDLL, see module docstring)
 
+from ._stack_enums import MI_ACT, MI_BLOCK, MI_FF, MI_MIX  # noqa: F401
+
 _HERE = os.path.dirname(os.path.abspath(__file__))
 # MI355X_VLLM_LIB points at another build of the same library (A/B measurements)
 LIB_PATH = os.environ.get("MI355X_VLLM_LIB") or os.path.join(_HERE, "csrc", "libmi355x_vllm.so")
@@ -53,21 +55,23 @@ class MiKvStats(C.Structure):
                 ("block_table_rows_sent", C.c_int64), ("block_table_rows_kept", C.c_int64)]
 
 
-MI_FF = {None: 0, "relu2": 1}
 MI_COMPUTE = {"bfloat16": MI_BF16, "float32": MI_F32}
 
 
 class MiLayerSpec(C.Structure):
     _fields_ = [("num_heads", C.c_int32), ("num_kv_heads", C.c_int32), ("qk_dim", C.c_int32), ("v_dim", C.c_int32),
                 ("window", C.c_int32), ("scale", C.c_float), ("qk_unit_norm", C.c_int32), ("distance_bias", C.c_int32),
-                ("softmax_sink", C.c_int32), ("ff_kind", C.c_int32), ("ff_size", C.c_int32)]
+                ("softmax_sink", C.c_int32), ("ff_kind", C.c_int32), ("ff_size", C.c_int32), ("mixer_kind", C.c_int32),
+                ("kv_rank", C.c_int32), ("kv_from", C.c_int32), ("ff_act", C.c_int32), ("ff_limit", C.c_float),
+                ("ff_alpha", C.c_float), ("experts", C.c_int32), ("experts_top", C.c_int32)]
 
 
 class MiStackConfig(C.Structure):
     _fields_ = [("num_layers", C.c_int32), ("layers", C.POINTER(MiLayerSpec)), ("width", C.c_int32),
                 ("vocab_size", C.c_int32), ("max_positions", C.c_int32), ("norm_eps", C.c_float),
                 ("residual_mult", C.c_float), ("loop_start", C.c_int32), ("loop_stop", C.c_int32),
-                ("loop_times", C.c_int32), ("compute_dtype", C.c_int32)]
+                ("loop_times", C.c_int32), ("compute_dtype", C.c_int32), ("block_kind", C.c_int32),
+                ("norm_groups", C.c_int32), ("conv_taps", C.c_int32), ("logit_softcap", C.c_float)]
 
 
 class MiTpPlan(C.Structure):

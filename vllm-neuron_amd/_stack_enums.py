@@ -1,0 +1,7 @@
+# SPDX-License-Identifier: Apache-2.0
+"""Names of the layer-stack enumerations of include/mi355x_vllm.h (no torch, no library: the configuration readers use them)."""
+
+MI_BLOCK = {"parallel": 0, "sandwich": 1}
+MI_MIX = {"attention": 0, "latent": 1}
+MI_FF = {None: 0, "relu2": 1, "glu": 2, "moe": 3}
+MI_ACT = {"silu": 0, "swish_clip": 1}

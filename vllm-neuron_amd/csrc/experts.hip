@@ -1,0 +1,212 @@
+// Mixture-of-experts kernels.  See experts.h.
+#include "experts.h"
+
+namespace mi {
+
+namespace {
+
+constexpr int kMaxTop = 64;
+
+// ---- router: one work-group per row; a wave takes every fourth expert ----------------------------------------------------
+__device__ __forceinline__ float dot8(const uint16_t* w, const float* x) {
+  const uint4 v = *reinterpret_cast<const uint4*>(w);
+  float a = bf16lo_to_f32(v.x) * x[0];
+  a = __builtin_fmaf(bf16hi_to_f32(v.x), x[1], a); a = __builtin_fmaf(bf16lo_to_f32(v.y), x[2], a);
+  a = __builtin_fmaf(bf16hi_to_f32(v.y), x[3], a); a = __builtin_fmaf(bf16lo_to_f32(v.z), x[4], a);
+  a = __builtin_fmaf(bf16hi_to_f32(v.z), x[5], a); a = __builtin_fmaf(bf16lo_to_f32(v.w), x[6], a);
+  return __builtin_fmaf(bf16hi_to_f32(v.w), x[7], a);
+}
+__device__ __forceinline__ float dot8(const float* w, const float* x) {
+  float a = 0.f;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) a = __builtin_fmaf(w[i], x[i], a);
+  return a;
+}
+__device__ __forceinline__ void load8f(const uint16_t* p, float* o) {
+  const uint4 v = *reinterpret_cast<const uint4*>(p);
+  o[0] = bf16lo_to_f32(v.x); o[1] = bf16hi_to_f32(v.x); o[2] = bf16lo_to_f32(v.y); o[3] = bf16hi_to_f32(v.y);
+  o[4] = bf16lo_to_f32(v.z); o[5] = bf16hi_to_f32(v.z); o[6] = bf16lo_to_f32(v.w); o[7] = bf16hi_to_f32(v.w);
+}
+__device__ __forceinline__ void load8f(const float* p, float* o) {
+#pragma unroll
+  for (int i = 0; i < 8; ++i) o[i] = p[i];
+}
+
+// the `top` largest of z [E] (LDS; destroyed), by one wave; softmax over them
+__device__ __forceinline__ void pick_top(float* z, int E, int top, int32_t* ids, float* weights) {
+  const int lane = threadIdx.x & 63;
+  float first = 0.f, sum = 0.f;
+  float mine = 0.f;      // lane j keeps the j-th weight
+  int mine_id = 0;
+  for (int j = 0; j < top; ++j) {
+    float best = -INFINITY;
+    int at = 0x7fffffff;
+    for (int e = lane; e < E; e += 64)
+      if (z[e] > best) { best = z[e]; at = e; }
+#pragma unroll
+    for (int m = 32; m >= 1; m >>= 1) {
+      const float v = __shfl_xor(best, m);
+      const int i = __shfl_xor(at, m);
+      if (v > best || (v == best && i < at)) { best = v; at = i; }
+    }
+    if (at >= E) at = j;       // (nothing but -inf or NaN left)
+    if (j == 0) first = best;
+    const float w = expf(best - first);
+    sum += w;
+    if (lane == j) { mine = w; mine_id = at; }
+    if (lane == (at & 63)) z[at] = -INFINITY;
+  }
+  if (lane < top) { ids[lane] = mine_id; weights[lane] = mine / sum; }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void route_kernel(const T* __restrict__ x, int ldx, const T* __restrict__ w, const float* __restrict__ b, int E,
+                                                    int K, int top, int32_t* __restrict__ ids, float* __restrict__ weights) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];   // K + E floats
+  float *xs = sm, *z = sm + K;
+  const int t = blockIdx.x, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  for (int k = tid * 8; k < K; k += 2048) load8f(x + (size_t)t * ldx + k, xs + k);
+  __syncthreads();
+  for (int e = wave; e < E; e += 4) {
+    float a = 0.f;
+    for (int k = lane * 8; k < K; k += 512) a += dot8(w + (size_t)e * K + k, xs + k);
+    a = wave_sum(a);
+    if (lane == 0) z[e] = a + b[e];
+  }
+  __syncthreads();
+  if (wave == 0) pick_top(z, E, top, ids + (size_t)t * top, weights + (size_t)t * top);
+}
+
+// ---- experts' linear layers, few rows: weight streaming -------------------------------------------------------------------
+// One work-group per (16-row weight tile or KS = 1: four of them, expert).  The pairs that chose the expert are found by a scan
+// over the pair list, in pair order, and taken 16 at a time as the columns of the MFMA tiles.
+template <int KS, bool GLU>
+__global__ __launch_bounds__(256) void experts_stream_kernel(const uint4* __restrict__ w, int NT, int KT, const int32_t* __restrict__ ids, int P,
+                                                             const uint16_t* __restrict__ x, int ldx, int x_div, void* __restrict__ y, int ldy) {
+  __shared__ int list[256], count[4];
+  __shared__ f32x4_t red[KS == 1 ? 1 : 4 * 64];
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g4 = lane >> 4, c = lane & 15, e = blockIdx.y;
+  const int nt = KS == 1 ? (int)blockIdx.x * 4 + wave : (int)blockIdx.x;
+  const int per = KS == 1 ? KT : ceil_div(KT, KS), k0 = KS == 1 ? 0 : wave * per, k1 = min(k0 + per, KT);
+  for (int base = 0; base < P; base += 256) {
+    const bool hit = base + tid < P && ids[base + tid] == e;
+    const unsigned long long mask = __ballot(hit);
+    __syncthreads();                                  // the previous round's list is used up
+    if (lane == 0) count[wave] = __popcll(mask);
+    __syncthreads();
+    int before = 0, n = 0;
+#pragma unroll
+    for (int v = 0; v < 4; ++v) {
+      before += v < wave ? count[v] : 0;
+      n += count[v];
+    }
+    if (hit) list[before + __popcll(mask & ((1ull << lane) - 1))] = base + tid;
+    __syncthreads();
+    for (int p0 = 0; p0 < n; p0 += 16) {
+      const bool live = p0 + c < n;
+      const int pair = list[min(p0 + c, n - 1)];
+      const uint16_t* X = x + (size_t)(pair / x_div) * ldx + g4 * 8;
+      f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
+      if (nt < NT) {
+        const u32x4_t* W = reinterpret_cast<const u32x4_t*>(w) + ((size_t)e * NT + nt) * KT * 64 + lane;
+        constexpr int U = 8;
+        int kt = k0;
+        for (; kt + U <= k1; kt += U) {
+          u32x4_t a[U], b[U];
+#pragma unroll
+          for (int u = 0; u < U; ++u) a[u] = __builtin_nontemporal_load(W + (size_t)(kt + u) * 64);
+#pragma unroll
+          for (int u = 0; u < U; ++u) b[u] = live ? *reinterpret_cast<const u32x4_t*>(X + (kt + u) * 32) : u32x4_t{0, 0, 0, 0};
+#pragma unroll
+          for (int u = 0; u < U; ++u) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a[u]), __builtin_bit_cast(bf16x8_t, b[u]), acc, 0, 0, 0);
+        }
+        for (; kt < k1; ++kt) {
+          const u32x4_t a = W[(size_t)kt * 64], b = live ? *reinterpret_cast<const u32x4_t*>(X + kt * 32) : u32x4_t{0, 0, 0, 0};
+          acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, b), acc, 0, 0, 0);
+        }
+      }
+      if constexpr (KS > 1) {
+        if (p0) __syncthreads();                      // the previous chunk's sums are read
+        red[wave * 64 + lane] = acc;
+        __syncthreads();
+        if (wave == 0) {
+#pragma unroll
+          for (int v = 1; v < KS; ++v) {
+            const f32x4_t r = red[v * 64 + lane];
+            acc[0] += r[0]; acc[1] += r[1]; acc[2] += r[2]; acc[3] += r[3];
+          }
+        }
+      }
+      if ((KS == 1 || wave == 0) && live && nt < NT) {
+        const int n0 = nt * 16 + g4 * 4;
+        if constexpr (GLU) {
+          const float a0 = acc[0] / (1.f + __expf(-acc[0])) * acc[1], a1 = acc[2] / (1.f + __expf(-acc[2])) * acc[3];
+          *reinterpret_cast<uint32_t*>(reinterpret_cast<uint16_t*>(y) + (size_t)pair * ldy + (n0 >> 1)) = pack_bf16x2(a0, a1);
+        } else {
+          *reinterpret_cast<float4*>(reinterpret_cast<float*>(y) + (size_t)pair * ldy + n0) = make_float4(acc[0], acc[1], acc[2], acc[3]);
+        }
+      }
+    }
+  }
+}
+
+// 32-bit form: a wave per output of one pair (for checking)
+template <bool GLU>
+__global__ __launch_bounds__(256) void experts_f32_kernel(const float* __restrict__ w, int N, int K, const int32_t* __restrict__ ids,
+                                                          const float* __restrict__ x, int ldx, int x_div, float* __restrict__ y, int ldy) {
+  const int p = blockIdx.x, n = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (n >= (GLU ? N / 2 : N)) return;
+  const float *X = x + (size_t)(p / x_div) * ldx, *W = w + ((size_t)ids[p] * N + (GLU ? 2 * n : n)) * K;
+  float a = 0.f, b = 0.f;
+  for (int k = lane; k < K; k += 64) {
+    a = __builtin_fmaf(W[k], X[k], a);
+    if constexpr (GLU) b = __builtin_fmaf(W[K + k], X[k], b);
+  }
+  a = wave_sum(a);
+  if constexpr (GLU) {
+    b = wave_sum(b);
+    a = a / (1.f + expf(-a)) * b;
+  }
+  if (lane == 0) y[(size_t)p * ldy + n] = a;
+}
+
+template <int KS>
+int launch_stream(const ExpertsLinear& w, const int32_t* ids, int P, const uint16_t* x, int ldx, int x_div, bool glu, void* y, int ldy, hipStream_t s) {
+  const int NT = w.N / 16, KT = w.K / 32;
+  const dim3 grid(KS == 1 ? ceil_div(NT, 4) : NT, w.E);
+  if (glu) hipLaunchKernelGGL((experts_stream_kernel<KS, true>), grid, dim3(256), 0, s, (const uint4*)w.w, NT, KT, ids, P, x, ldx, x_div, y, ldy);
+  else hipLaunchKernelGGL((experts_stream_kernel<KS, false>), grid, dim3(256), 0, s, (const uint4*)w.w, NT, KT, ids, P, x, ldx, x_div, y, ldy);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+}  // namespace
+
+int launch_route(const void* x, int ldx, int T, const void* w, const float* b, int E, int K, int top, int32_t* ids, float* weights, bool f32, hipStream_t s) {
+  MI_CHECK(T >= 1 && E >= 1 && top >= 1 && top <= E && top <= kMaxTop && K % 64 == 0 && ldx >= K && ldx % 8 == 0, "router: 1 <= top <= min(experts, 64), row stride");
+  const size_t lds = (size_t)(K + E) * 4;
+  const void* kern = f32 ? reinterpret_cast<const void*>(route_kernel<float>) : reinterpret_cast<const void*>(route_kernel<uint16_t>);
+  MI_CHECK(lds <= 160 * 1024, "router: row and logits larger than the LDS");
+  if (lds > 64 * 1024) { int rc = ensure_dynamic_lds(kern, 160 * 1024); if (rc != MI_OK) return rc; }
+  if (f32) hipLaunchKernelGGL((route_kernel<float>), dim3(T), dim3(256), lds, s, (const float*)x, ldx, (const float*)w, b, E, K, top, ids, weights);
+  else hipLaunchKernelGGL((route_kernel<uint16_t>), dim3(T), dim3(256), lds, s, (const uint16_t*)x, ldx, (const uint16_t*)w, b, E, K, top, ids, weights);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_experts_linear(const ExpertsLinear& w, const int32_t* ids, int P, const void* x, int ldx, int x_div, bool glu, void* y, int ldy,
+                          bool f32, hipStream_t s) {
+  MI_CHECK(w.E >= 1 && w.E <= 65535 && w.N % 16 == 0 && w.K % 64 == 0 && ldx >= w.K && ldx % 8 == 0 && P >= 1 && x_div >= 1, "experts: shape");
+  MI_CHECK(ldy % 4 == 0 && ldy >= (glu ? w.N / 2 : w.N), "experts: output stride");
+  if (f32) {
+    const dim3 grid(P, ceil_div(glu ? w.N / 2 : w.N, 4));
+    if (glu) hipLaunchKernelGGL((experts_f32_kernel<true>), grid, dim3(256), 0, s, (const float*)w.w, w.N, w.K, ids, (const float*)x, ldx, x_div, (float*)y, ldy);
+    else hipLaunchKernelGGL((experts_f32_kernel<false>), grid, dim3(256), 0, s, (const float*)w.w, w.N, w.K, ids, (const float*)x, ldx, x_div, (float*)y, ldy);
+    MI_HIP(hipGetLastError());
+    return MI_OK;
+  }
+  return w.K / 32 >= 16 ? launch_stream<4>(w, ids, P, (const uint16_t*)x, ldx, x_div, glu, y, ldy, s)
+                        : launch_stream<1>(w, ids, P, (const uint16_t*)x, ldx, x_div, glu, y, ldy, s);
+}
+
+}  // namespace mi

@@ -15,6 +15,12 @@ namespace mi {
 // =====================================================================================
 // Epilogue
 // =====================================================================================
+// gated unit with clipped branches: g = min(gate, limit), u = up within +-limit -> g sigmoid(alpha g) (u + 1)
+__device__ __forceinline__ float glu_clip(float gate, float up, float limit, float alpha) {
+  const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+  return g / (1.f + __expf(-alpha * g)) * (u + 1.f);
+}
+
 template <int EPI>
 __device__ __forceinline__ void epilogue_store(const EpiArgs& e, int m, int n0, f32x4_t v);
 
@@ -65,6 +71,12 @@ __device__ __forceinline__ void epilogue_store(const EpiArgs& e, int m, int n0, 
   } else if constexpr (EPI == EPI_RELU2) {
     const float a0 = fmaxf(v[0], 0.f), a1 = fmaxf(v[1], 0.f), a2 = fmaxf(v[2], 0.f), a3 = fmaxf(v[3], 0.f);
     *reinterpret_cast<uint2*>(e.act_out + (size_t)m * e.ld_act + n0) = make_uint2(pack_bf16x2(a0 * a0, a1 * a1), pack_bf16x2(a2 * a2, a3 * a3));
+  } else if constexpr (EPI == EPI_GLU_CLIP) {
+    *reinterpret_cast<uint32_t*>(e.act_out + (size_t)m * e.ld_act + (n0 >> 1)) =
+        pack_bf16x2(glu_clip(v[0], v[1], e.glu_limit, e.glu_alpha), glu_clip(v[2], v[3], e.glu_limit, e.glu_alpha));
+  } else if constexpr (EPI == EPI_SOFTCAP) {
+    *reinterpret_cast<float4*>(e.out_f32 + (size_t)m * e.ld_out + n0) =
+        make_float4(e.softcap * tanhf(v[0] / e.softcap), e.softcap * tanhf(v[1] / e.softcap), e.softcap * tanhf(v[2] / e.softcap), e.softcap * tanhf(v[3] / e.softcap));
   } else {  // EPI_QKV
     const int qk_end = e.q_dim + e.kv_dim;
     if (n0 < qk_end) {  // rotary: (v0,v1) and (v2,v3) are (d, d + hd/2) pairs
@@ -909,7 +921,7 @@ static int launch_gemv_kstream(const LinearW& w, int M, const ProArgs& p, const 
 template <int WD, int PRO, int EPI>
 static int launch_gemv_t(const LinearW& w, int M, const ProArgs& p, const EpiArgs& e, hipStream_t s) {
   if (!gemv_fits_whole(M, w.K)) {
-    if constexpr (PRO == PRO_BF16 && (EPI == EPI_F32 || EPI == EPI_RESID || EPI == EPI_RELU2)) {
+    if constexpr (PRO == PRO_BF16 && (EPI == EPI_F32 || EPI == EPI_RESID || EPI >= EPI_RELU2)) {
       static const int min_m = [] { const char* v = getenv("MI355X_GEMV_KSTREAM_MIN_M"); return v ? atoi(v) : 1; }();
       if (gemv_kstream_enabled() && M >= min_m) return launch_gemv_kstream<WD, EPI>(w, M, p, e, s);
     }
@@ -1497,7 +1509,11 @@ int launch_gemv_wd(const LinearW& w, int M, int pro, const ProArgs& p, int epi, 
     if (epi == EPI_RESID) return launch_gemv_t<WD, PRO_BF16, EPI_RESID>(w, M, p, e, s);
     if (epi == EPI_F32) return launch_gemv_t<WD, PRO_BF16, EPI_F32>(w, M, p, e, s);
     if constexpr (WD == MI_W_BF16)
-      if (epi == EPI_RELU2) return launch_gemv_t<WD, PRO_BF16, EPI_RELU2>(w, M, p, e, s);
+      switch (epi) {
+        case EPI_RELU2: return launch_gemv_t<WD, PRO_BF16, EPI_RELU2>(w, M, p, e, s);
+        case EPI_GLU_CLIP: return launch_gemv_t<WD, PRO_BF16, EPI_GLU_CLIP>(w, M, p, e, s);
+        case EPI_SOFTCAP: return launch_gemv_t<WD, PRO_BF16, EPI_SOFTCAP>(w, M, p, e, s);
+      }
   } else if (p.partial) {
     if (epi == EPI_QKV) return launch_gemv_t<WD, PRO_NORM_PARTIAL, EPI_QKV>(w, M, p, e, s);
     if (epi == EPI_SWIGLU) return launch_gemv_t<WD, PRO_NORM_PARTIAL, EPI_SWIGLU>(w, M, p, e, s);

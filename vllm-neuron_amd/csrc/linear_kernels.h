@@ -7,7 +7,7 @@
 namespace mi {
 
 // What happens to the fp32 accumulator tile D[n][m] once the contraction is done.
-enum { EPI_F32 = 0, EPI_QKV = 1, EPI_SWIGLU = 2, EPI_RESID = 3, EPI_RELU2 = 4 };
+enum { EPI_F32 = 0, EPI_QKV = 1, EPI_SWIGLU = 2, EPI_RESID = 3, EPI_RELU2 = 4, EPI_GLU_CLIP = 5, EPI_SOFTCAP = 6 };
 // Where the bf16 activations come from.
 enum { PRO_BF16 = 0, PRO_NORM = 1, PRO_NORM_PARTIAL = 2 };  // callers pass PRO_BF16 / PRO_NORM; PARTIAL is picked when ProArgs::partial is set
 
@@ -33,8 +33,12 @@ struct EpiArgs {
   int block_size;
   // EPI_SWIGLU: rows interleaved (gate_i, up_i); act[m * ld_act + i] = silu(gate)*up
   // EPI_RELU2 (bf16 weights): act[m * ld_act + n] = max(y, 0)^2
+  // EPI_GLU_CLIP (bf16 weights; rows interleaved as for SWIGLU): g = min(gate, glu_limit), u = up within +-glu_limit,
+  //   act[m * ld_act + i] = g sigmoid(glu_alpha g) (u + 1)
   uint16_t* act_out;
   int ld_act;
+  float glu_limit, glu_alpha;
+  float softcap;         // EPI_SOFTCAP (bf16 weights): out[m * ld_out + n] = softcap tanh(y / softcap)
 };
 
 struct ProArgs {
@@ -58,7 +62,7 @@ struct LinearW {
 int launch_gemv(const LinearW& w, int M, int pro, const ProArgs& p, int epi, const EpiArgs& e,
                 hipStream_t s);
 // M > 16 context-encoding path (MFMA-bound).  x is always bf16 [T, K].
-// defer != null: a K-split residual projection (EPI_RESID) leaves its slabs unsummed and describes them in *defer
+// defer != null: a K-split projection (EPI_RESID, EPI_F32) leaves its slabs unsummed and describes them in *defer
 // (slab == null: nothing deferred); the caller hands them to the next row norm or to launch_splitk_flush
 int launch_gemm(const LinearW& w, int T, const uint16_t* x, int ldx, int epi, const EpiArgs& e,
                 hipStream_t s, float* splitk_ws = nullptr, size_t splitk_ws_bytes = 0, SlabSum* defer = nullptr);

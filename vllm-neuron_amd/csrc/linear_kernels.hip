@@ -205,16 +205,19 @@ static int launch_gemm_wd(const LinearW& w, int T, const uint16_t* x, int ldx, i
       hipLaunchKernelGGL((gemm_kernel<WD, EPI_, false>), grid, dim3(256), 0, s, W, NT, KT, T, w.K, x, ldx, e, nullptr); \
     } else { \
       hipLaunchKernelGGL((gemm_kernel<WD, EPI_, true>), grid, dim3(256), 0, s, W, NT, KT, T, w.K, x, ldx, e, splitk_ws); \
-      if (defer && EPI_ == EPI_RESID) { *defer = SlabSum{splitk_ws, KS, T, w.N, e.scale, e.bias, e.row_scale}; } \
+      if (defer && (EPI_ == EPI_RESID || EPI_ == EPI_F32)) { *defer = SlabSum{splitk_ws, KS, T, w.N, e.scale, e.bias, e.row_scale}; } \
       else hipLaunchKernelGGL((splitk_reduce_kernel<EPI_>), dim3(ceil_div(T * (w.N / 4), 256)), dim3(256), 0, s, splitk_ws, KS, T, w.N, e); \
     } \
   } while (0)
   if (epi == EPI_QKV) MI_G(EPI_QKV);
   else if (epi == EPI_SWIGLU) MI_G(EPI_SWIGLU);
   else if (epi == EPI_RESID) MI_G(EPI_RESID);
-  else if (epi == EPI_RELU2) {
-    if constexpr (WD == MI_W_BF16) MI_G(EPI_RELU2);
-    else { set_error("gemm: the squared-relu epilogue is built for bf16 weights"); return MI_EINVAL; }
+  else if (epi >= EPI_RELU2) {
+    if constexpr (WD == MI_W_BF16) {
+      if (epi == EPI_RELU2) MI_G(EPI_RELU2);
+      else if (epi == EPI_GLU_CLIP) MI_G(EPI_GLU_CLIP);
+      else MI_G(EPI_SOFTCAP);
+    } else { set_error("gemm: this epilogue is built for bf16 weights"); return MI_EINVAL; }
   } else MI_G(EPI_F32);
 #undef MI_G
   MI_HIP(hipGetLastError());
@@ -491,7 +494,7 @@ int launch_gemm(const LinearW& w, int T, const uint16_t* x, int ldx, int epi, co
                 float* splitk_ws, size_t splitk_ws_bytes, SlabSum* defer) {
   if (defer) *defer = SlabSum();
   MI_CHECK(T >= 1, "gemm: T must be >= 1");
-  if (epi != EPI_RELU2 && gemm_wide_wanted(w, T, splitk_ws ? splitk_ws_bytes : 0) && ldx % 8 == 0)
+  if (epi < EPI_RELU2 && gemm_wide_wanted(w, T, splitk_ws ? splitk_ws_bytes : 0) && ldx % 8 == 0)
     return launch_gemm_wide(w, T, x, ldx, epi, e, s, splitk_ws, splitk_ws_bytes, defer);
   MI_CHECK(w.N % 16 == 0 && w.K % 64 == 0, "gemm: N % 16 == 0 and K % 64 == 0 required");
   MI_CHECK(ldx % 8 == 0, "gemm: x row stride must be a multiple of 8 elements");

@@ -577,7 +577,7 @@ int capture_or_launch_decode(mi_ctx* c, int B, int MB) {
 extern "C" {
 
 const char* mi_last_error(void) { return mi::g_err.c_str(); }
-int mi_version(void) { return 5; }   // 3: + in-process tensor parallelism (tp_rank = MI_TP_ALL_RANKS, tp_device_ids, tp_transport)
+int mi_version(void) { return 6; }   // 3: + in-process tensor parallelism (tp_rank = MI_TP_ALL_RANKS, tp_device_ids, tp_transport)
 
 int mi_tp_plan(const mi_model_config* cfg, int32_t rank, mi_tp_plan_t* out) {
   MI_CHECK(cfg && out, "null argument");
@@ -699,21 +699,45 @@ int mi_ctx_create_stack(const mi_model_config* cfg, const mi_stack_config* stack
   MI_CHECK(cfg && stack && out && stack->layers, "null argument");
   mi_model_config k = *cfg;
   const mi_stack_config& t = *stack;
-  MI_CHECK(t.num_layers > 0 && t.width > 0 && t.width <= 32768 && t.vocab_size > 0 && t.max_positions > 0 && t.norm_eps >= 0.f, "stack: bad geometry");
+  MI_CHECK(t.num_layers > 0 && t.width > 0 && t.width <= 32768 && t.vocab_size > 0 && t.max_positions >= 0 && t.norm_eps >= 0.f, "stack: bad geometry");
   MI_CHECK(t.compute_dtype == MI_BF16 || t.compute_dtype == MI_F32, "stack: compute_dtype must be MI_BF16 or MI_F32");
   MI_CHECK(t.loop_times == 0 || (t.loop_times > 0 && t.loop_start >= 0 && t.loop_start < t.loop_stop && t.loop_stop <= t.num_layers), "stack: bad loop");
+  MI_CHECK(t.block_kind == MI_BLOCK_PARALLEL || t.block_kind == MI_BLOCK_SANDWICH, "stack: block_kind");
+  const bool sandwich = t.block_kind == MI_BLOCK_SANDWICH;
+  if (sandwich) {
+    MI_CHECK(t.norm_groups >= 1 && t.width % t.norm_groups == 0, "stack: the norm's groups must divide the width");
+    MI_CHECK(t.conv_taps >= 1 && t.conv_taps <= 16, "stack: convolutions of 1 .. 16 taps are built");
+    MI_CHECK(t.loop_times == 0, "stack: loops are not built for sandwich blocks");
+  } else {
+    MI_CHECK(t.norm_groups == 0 && t.conv_taps == 0 && t.max_positions > 0, "stack: parallel blocks are built with layer norms, learned positions and no convolution");
+  }
+  MI_CHECK(t.logit_softcap >= 0.f, "stack: logit_softcap");
   for (int i = 0; i < t.num_layers; ++i) {
     const mi_layer_spec& p = t.layers[i];
-    MI_CHECK(p.num_heads > 0 && p.num_kv_heads > 0 && p.num_heads % p.num_kv_heads == 0 && p.qk_dim > 0 && p.v_dim > 0 && p.window >= 0,
-             "stack: layer " + std::to_string(i) + ": bad attention sizes");
-    MI_CHECK(p.ff_kind == MI_FF_NONE || (p.ff_kind == MI_FF_RELU2 && p.ff_size > 0), "stack: layer " + std::to_string(i) + ": bad feed-forward");
+    const std::string who = "stack: layer " + std::to_string(i) + ": ";
+    MI_CHECK(p.mixer_kind == (sandwich ? MI_MIX_LATENT : MI_MIX_ATTENTION), who + "this mixer is not built for the block kind");
+    MI_CHECK(p.num_heads > 0 && p.qk_dim > 0 && p.v_dim > 0 && p.window >= 0, who + "bad attention sizes");
+    if (p.mixer_kind == MI_MIX_LATENT) {
+      MI_CHECK(p.kv_rank > 0 && p.kv_rank <= 4096 && p.qk_dim <= 4096 && p.v_dim <= 4096, who + "bad latent size");
+      MI_CHECK(!p.qk_unit_norm && !p.distance_bias && !p.softmax_sink, who + "latent attention has no unit norm, distance bias or sink");
+      MI_CHECK(p.kv_from < 0 || (p.kv_from < i && t.layers[p.kv_from].kv_from < 0 && t.layers[p.kv_from].kv_rank == p.kv_rank),
+               who + "kv_from must name an earlier layer with latents of its own and the same kv_rank");
+    } else {
+      MI_CHECK(p.num_kv_heads > 0 && p.num_heads % p.num_kv_heads == 0, who + "bad attention sizes");
+    }
+    const bool ff = p.ff_kind == MI_FF_NONE || (p.ff_size > 0 && (sandwich ? p.ff_kind == MI_FF_GLU || p.ff_kind == MI_FF_MOE : p.ff_kind == MI_FF_RELU2));
+    MI_CHECK(ff, who + "bad feed-forward");
+    if (p.ff_kind == MI_FF_GLU) MI_CHECK(p.ff_act == MI_ACT_SWISH_CLIP && p.ff_limit >= 0.f, who + "gated feed-forwards are built with the clipped activation");
+    if (p.ff_kind == MI_FF_MOE)
+      MI_CHECK(p.ff_act == MI_ACT_SILU && p.experts >= 1 && p.experts <= 4096 && p.experts_top >= 1 && p.experts_top <= std::min(p.experts, 64),
+               who + "experts: silu, 1 <= experts_top <= min(experts, 64)");
   }
   MI_CHECK(k.tp_degree <= 1, "stack: tensor parallelism is not built for layer-stack decoders");
   MI_CHECK(k.weight_dtype == MI_W_BF16, "stack: weight quantization is not built for layer-stack decoders");
   MI_CHECK(k.block_size > 0 && k.block_size % 16 == 0, "block_size must be a positive multiple of 16");
   MI_CHECK(k.num_blocks >= 2, "num_blocks must include the null block and at least one real block");
   MI_CHECK(k.max_num_seqs >= 1 && k.max_num_seqs <= 256, "max_num_seqs must be 1..256");
-  MI_CHECK(k.max_model_len >= 1 && k.max_model_len <= t.max_positions, "max_model_len must be 1..max_positions (learned positions)");
+  MI_CHECK(k.max_model_len >= 1 && (t.max_positions == 0 || k.max_model_len <= t.max_positions), "max_model_len must be 1..max_positions (learned positions)");
   int ndev = 0;
   MI_HIP(hipGetDeviceCount(&ndev));
   MI_CHECK(ndev > 0, "no HIP device: this library has no CPU fallback");
@@ -1556,6 +1580,9 @@ int mi_forward_spec(mi_ctx* t, mi_ctx* d, int32_t B, int32_t k, const int64_t* i
   MI_CHECK(kt.device_id == kd.device_id && kt.block_size == kd.block_size && kt.num_blocks == kd.num_blocks &&
            kt.vocab_size == kd.vocab_size && kt.max_model_len == kd.max_model_len,
            "mi_forward_spec: target (rank 0) and draft must share device, block_size, num_blocks, vocab_size and max_model_len");
+  // several rows of one sequence in a token-generation batch: a convolution's state follows one row per sequence
+  MI_CHECK(!(t0->stack && t0->stack->conv_keep > 0) && !(d->stack && d->stack->conv_keep > 0),
+           "mi_forward_spec: not built for models with convolution state");
   MI_CHECK(B >= 1 && k >= 1 && B * k <= kt.max_num_seqs && B <= kd.max_num_seqs,
            "mi_forward_spec: B * k rows exceed the target's max_num_seqs (or B the draft's)");
   int n_catch = 0;

@@ -4,8 +4,9 @@
 #include <string>
 #include <vector>
 
+#include "experts.h"
+#include "latent_attn.h"
 #include "model_internal.h"
-#include "window_attn.h"
 
 namespace mi {
 
@@ -23,6 +24,19 @@ struct StackLayer {
   StackMat qkv, up, out;            // out = residual_mult [W_o | W_down]
   StackNorm n1, n2;
   float* slopes = nullptr;
+  // sandwich blocks: qkv = [W_q | W_dkv], out = W_o, up = gate / up rows interleaved, down
+  StackNorm n1b, n2b;                            // post-norms
+  float *conv1 = nullptr, *conv2 = nullptr;      // [taps][ld]
+  StackMat down;
+  LatentGeom lg;
+  AttnSpec latent;                               // the attention over latents: one shared key / value row for all heads
+  float* c_norm = nullptr;                       // [rank]; null where the latents are another layer's
+  void *w_uk = nullptr, *w_uv = nullptr;         // per head: W_uk^T [rp, dkp], W_uv [dvp, rp]
+  void *router = nullptr, *expert_gu = nullptr, *expert_down = nullptr;
+  float* router_b = nullptr;
+  int ffk = 0;                                   // padded ff_size: contraction length of the experts' down projection
+  ExpertsLinear expert_up() const { return ExpertsLinear{expert_gu, s.experts, (2 * s.ff_size + 15) / 16 * 16, up.K}; }
+  ExpertsLinear expert_dn() const { return ExpertsLinear{expert_down, s.experts, out.N, ffk}; }
 };
 struct StackRun { int layer; bool pass_start; };   // pass_start: the looped layers' input projection runs first
 
@@ -35,12 +49,21 @@ struct Stack {
   void *embed = nullptr, *pos = nullptr;
   StackMat loop_in, head;
   StackNorm final_norm;
-  std::vector<size_t> kv_at;          // pool offset (elements) of every run's K; its V follows
+  std::vector<size_t> kv_at;          // pool offset (elements) of every run's K (V follows) or latents (its own, or the layer's it reads)
+  std::vector<size_t> conv_at;        // sandwich blocks: offset of every run's first convolution's state, the second's follows
+  int conv_keep = 0;                  // convolution inputs a block keeps
   std::vector<std::string> missing;   // tensors not loaded yet
   // activations
   float *x0 = nullptr, *qkv_out = nullptr, *logits_pad = nullptr;
   void *n1 = nullptr, *n2 = nullptr, *q = nullptr, *cat = nullptr, *pair = nullptr;
   int qkv_ld = 0, q_cols = 0, cat_ld = 0;
+  // sandwich blocks
+  float *y = nullptr, *pair_w = nullptr;       // a sublayer's output rows (experts: of every pair); the pairs' weights
+  int32_t* pair_ids = nullptr;
+  void *hb = nullptr, *act = nullptr, *qa = nullptr, *lat = nullptr;   // convolution inputs; gated units; queries / outputs in latent space
+  int act_ld = 0, lat_cols = 0, max_top = 0;
+  size_t act_elems = 0, y_rows = 0;
+  bool sandwich() const { return cfg.block_kind == MI_BLOCK_SANDWICH; }
   void* attn_scratch = nullptr;
   SlabSum pend;                        // K-split sum of the last output projection, left for the next norm
   float* residuals = nullptr;          // mi_layer_residuals: [runs][max_rows][ld]

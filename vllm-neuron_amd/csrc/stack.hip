@@ -9,6 +9,12 @@
 //   norm2 -> up projection, squared relu -> right part of the same row    GEMV / GEMM
 //   [W_o | W_down] x concatenated row, residual_mult in its row scale, + residual
 // The last one is both branches' output projection and the residual sum in one matrix product.
+//
+// A sandwich block's run (RMS norms around both sublayers, causal convolutions, latent attention, gated or expert feed-forward):
+//   row: x += post-norm of the previous sublayer's output; pre-norm; convolution    sandwich_rows / conv_rows
+//   [q | latent] projection; latent norm into the pool; W_uk^T q                    GEMV / GEMM, latent_scatter, head_linear
+//   attention over latents; W_uv; output projection
+//   row, as above; gated feed-forward, or router and experts                        experts.hip
 
 #include "stack.h"
 
@@ -133,6 +139,137 @@ int attention(mi_ctx* c, const StackLayer& W, size_t kv_at, int rows, bool decod
   return MI_OK;
 }
 
+// ---- sandwich blocks: geometry and weights of one layer --------------------------------------------------------------------
+int sandwich_layer_create(mi_ctx* c, StackLayer& W, const std::string& p) {
+  Stack* S = c->stack;
+  const mi_layer_spec& s = W.s;
+  size_t* wb = &c->weight_bytes;
+  auto want = [&](const char* n) { S->missing.push_back(p + n); };
+  auto norm = [&](StackNorm& n) { return alloc0(c, &n.w, (size_t)S->ld * 4, wb); };
+  const int taps = S->cfg.conv_taps;
+  const bool own = s.kv_from < 0;
+  W.lg = LatentGeom{s.num_heads, s.qk_dim, s.v_dim, s.kv_rank, pad_to(s.qk_dim, 32), pad_to(s.v_dim, 32), pad_to(s.kv_rank, 32)};
+  W.latent = AttnSpec{HeadGeom{s.num_heads, 1, W.lg.rp, W.lg.rp, W.lg.rp, W.lg.rp}, s.scale, s.window, nullptr, 0, 0};
+  MI_TRY(alloc_mat(c, W.qkv, s.num_heads * s.qk_dim + (own ? s.kv_rank : 0), S->D, 1.f));
+  MI_TRY(alloc_mat(c, W.out, S->D, s.num_heads * s.v_dim, 1.f));
+  MI_TRY(alloc0(c, &W.w_uk, (size_t)s.num_heads * W.lg.rp * W.lg.dkp * S->elem(), wb));
+  MI_TRY(alloc0(c, &W.w_uv, (size_t)s.num_heads * W.lg.dvp * W.lg.rp * S->elem(), wb));
+  if (own) MI_TRY(alloc0(c, &W.c_norm, (size_t)s.kv_rank * 4, wb));
+  MI_TRY(norm(W.n1)); MI_TRY(norm(W.n1b));
+  MI_TRY(alloc0(c, &W.conv1, (size_t)taps * S->ld * 4, wb));
+  for (const char* n : {"norm1", "norm1b", "canon1", "mix.q", "mix.uk", "mix.uv", "mix.o"}) want(n);
+  if (own) { want("mix.dkv"); want("mix.dkv.norm"); }
+  S->qkv_ld = std::max(S->qkv_ld, W.qkv.N);
+  S->q_cols = std::max(S->q_cols, s.num_heads * W.lg.dkp);
+  S->lat_cols = std::max(S->lat_cols, s.num_heads * W.lg.rp);
+  S->cat_ld = std::max(S->cat_ld, W.out.K);
+  if (s.ff_kind == MI_FF_NONE) return MI_OK;
+  MI_TRY(norm(W.n2)); MI_TRY(norm(W.n2b));
+  MI_TRY(alloc0(c, &W.conv2, (size_t)taps * S->ld * 4, wb));
+  for (const char* n : {"norm2", "norm2b", "canon2"}) want(n);
+  if (s.ff_kind == MI_FF_GLU) {
+    MI_TRY(alloc_mat(c, W.up, 2 * s.ff_size, S->D, 1.f));
+    MI_TRY(alloc_mat(c, W.down, S->D, s.ff_size, 1.f));
+    W.ffk = W.down.K;
+    for (const char* n : {"mlp.gate", "mlp.up", "mlp.down"}) want(n);
+  } else {
+    W.up.K = S->Kd;
+    W.ffk = pad_to(s.ff_size, 64);
+    S->max_top = std::max(S->max_top, s.experts_top);
+    const ExpertsLinear gu = W.expert_up(), dn = W.expert_dn();
+    MI_TRY(alloc0(c, &W.expert_gu, (size_t)gu.E * gu.N * gu.K * S->elem(), wb));
+    MI_TRY(alloc0(c, &W.expert_down, (size_t)dn.E * dn.N * dn.K * S->elem(), wb));
+    MI_TRY(alloc0(c, &W.router, (size_t)s.experts * S->Kd * S->elem(), wb));
+    MI_TRY(alloc0(c, &W.router_b, (size_t)s.experts * 4, wb));
+    want("mlp.router"); want("mlp.router.b");
+    for (int e = 0; e < s.experts; ++e)
+      for (const char* n : {".gate", ".up", ".down"}) want(("mlp.e" + std::to_string(e) + n).c_str());
+  }
+  S->act_ld = std::max(S->act_ld, W.ffk);
+  return MI_OK;
+}
+
+// shape of a tensor of a sandwich block's layer by its name behind "l<i>."; rows 0: not one of its tensors
+void sandwich_tensor_shape(const Stack* S, const StackLayer& W, const std::string& t, int* rows, int* cols) {
+  const mi_layer_spec& s = W.s;
+  *rows = *cols = 0;
+  const bool ff = s.ff_kind != MI_FF_NONE;
+  auto is = [&](int r, int k) { *rows = r; *cols = k; };
+  if (t == "norm1" || t == "norm1b" || (ff && (t == "norm2" || t == "norm2b"))) is(S->D, 0);
+  else if (t == "canon1" || (ff && t == "canon2")) is(S->D, S->cfg.conv_taps);
+  else if (t == "mix.q") is(s.num_heads * s.qk_dim, S->D);
+  else if (t == "mix.dkv" && s.kv_from < 0) is(s.kv_rank, S->D);
+  else if (t == "mix.dkv.norm" && s.kv_from < 0) is(s.kv_rank, 0);
+  else if (t == "mix.uk") is(s.num_heads * s.qk_dim, s.kv_rank);
+  else if (t == "mix.uv") is(s.num_heads * s.v_dim, s.kv_rank);
+  else if (t == "mix.o") is(S->D, s.num_heads * s.v_dim);
+  else if (s.ff_kind == MI_FF_GLU) {
+    if (t == "mlp.gate" || t == "mlp.up") is(s.ff_size, S->D);
+    else if (t == "mlp.down") is(S->D, s.ff_size);
+  } else if (s.ff_kind == MI_FF_MOE) {
+    int e = -1, at = 0;
+    if (t == "mlp.router") is(s.experts, S->D);
+    else if (t == "mlp.router.b") is(s.experts, 0);
+    else if (sscanf(t.c_str(), "mlp.e%d.%n", &e, &at) == 1 && at > 0 && e >= 0 && e < s.experts) {
+      const std::string m = t.substr(at);
+      if (m == "gate" || m == "up") is(s.ff_size, S->D);
+      else if (m == "down") is(S->D, s.ff_size);
+    }
+  }
+}
+
+int sandwich_place(mi_ctx* c, StackLayer& W, const std::string& t, const float* dev, int rows, int cols) {
+  Stack* S = c->stack;
+  const mi_layer_spec& s = W.s;
+  hipStream_t st = c->stream;
+  const size_t el = S->elem();
+  auto at = [&](void* base, size_t elems) -> void* { return reinterpret_cast<unsigned char*>(base) + elems * el; };
+  auto vec = [&](float* dst) -> int {
+    MI_HIP(hipMemcpyAsync(dst, dev, (size_t)rows * 4, hipMemcpyDeviceToDevice, st));
+    return MI_OK;
+  };
+  auto place = [&](void* dst, int K, int row0 = 0, int step = 1) { return launch_place(dev, cols, 0, rows, cols, dst, K, S->f32, row0, 0, st, step); };
+  if (t == "norm1") return vec(W.n1.w);
+  if (t == "norm1b") return vec(W.n1b.w);
+  if (t == "norm2") return vec(W.n2.w);
+  if (t == "norm2b") return vec(W.n2b.w);
+  if (t == "canon1" || t == "canon2") return launch_transpose(dev, rows, cols, t == "canon1" ? W.conv1 : W.conv2, S->ld, st);
+  if (t == "mix.q") return place(W.qkv.L.w, W.qkv.K);
+  if (t == "mix.dkv") return place(W.qkv.L.w, W.qkv.K, s.num_heads * s.qk_dim);
+  if (t == "mix.dkv.norm") return vec(W.c_norm);
+  if (t == "mix.o") return place(W.out.L.w, W.out.K);
+  if (t == "mix.uk" || t == "mix.uv") {
+    const bool k = t == "mix.uk";
+    const int n = k ? s.qk_dim : s.v_dim;
+    float* tmp = nullptr;
+    if (k) MI_HIP(hipMalloc(reinterpret_cast<void**>(&tmp), (size_t)n * cols * 4));
+    int rc = MI_OK;
+    for (int h = 0; h < s.num_heads && rc == MI_OK; ++h) {
+      const float* src = dev + (size_t)h * n * cols;
+      if (k) {
+        rc = launch_transpose(src, n, cols, tmp, n, st);
+        if (rc == MI_OK) rc = launch_place(tmp, n, 0, cols, n, at(W.w_uk, (size_t)h * W.lg.rp * W.lg.dkp), W.lg.dkp, S->f32, 0, 0, st);
+      } else {
+        rc = launch_place(src, cols, 0, n, cols, at(W.w_uv, (size_t)h * W.lg.dvp * W.lg.rp), W.lg.rp, S->f32, 0, 0, st);
+      }
+    }
+    hipStreamSynchronize(st);
+    hipFree(tmp);
+    return rc;
+  }
+  if (t == "mlp.gate") return place(W.up.L.w, W.up.K, 0, 2);
+  if (t == "mlp.up") return place(W.up.L.w, W.up.K, 1, 2);
+  if (t == "mlp.down") return place(W.down.L.w, W.down.K);
+  if (t == "mlp.router") return launch_place_rows(dev, rows, cols, W.router, S->Kd, S->f32, st);
+  if (t == "mlp.router.b") return vec(W.router_b);
+  int e = -1, off = 0;
+  sscanf(t.c_str(), "mlp.e%d.%n", &e, &off);
+  const std::string m = t.substr(off);
+  const ExpertsLinear gu = W.expert_up(), dn = W.expert_dn();
+  if (m == "down") return place(at(W.expert_down, (size_t)e * dn.N * dn.K), dn.K);
+  return place(at(W.expert_gu, (size_t)e * gu.N * gu.K), gu.K, m == "up" ? 1 : 0, 2);
+}
+
 }  // namespace
 
 int stack_create(mi_ctx* c, const mi_stack_config& cfg) {
@@ -158,8 +295,12 @@ int stack_create(mi_ctx* c, const mi_stack_config& cfg) {
   auto want = [&](const std::string& n) { S->missing.push_back(n); };
   size_t* wb = &c->weight_bytes;
   MI_TRY(alloc0(c, &S->embed, (size_t)cfg.vocab_size * S->D * S->elem(), wb));
-  MI_TRY(alloc0(c, &S->pos, (size_t)cfg.max_positions * S->D * S->elem(), wb));
-  want("embed"); want("pos");
+  want("embed");
+  if (cfg.max_positions > 0) {
+    MI_TRY(alloc0(c, &S->pos, (size_t)cfg.max_positions * S->D * S->elem(), wb));
+    want("pos");
+  }
+  S->conv_keep = std::min(c->cfg.block_size, std::max(cfg.conv_taps - 1, 0));
   if (loop) {
     MI_TRY(alloc_mat(c, S->loop_in, S->D, 2 * S->Kd, 1.f));
     want("loop.in");
@@ -169,6 +310,10 @@ int stack_create(mi_ctx* c, const mi_stack_config& cfg) {
     StackLayer& W = S->layers[i];
     W.s = cfg.layers[i];
     const mi_layer_spec& s = W.s;
+    if (S->sandwich()) {
+      MI_TRY(sandwich_layer_create(c, W, "l" + std::to_string(i) + "."));
+      continue;
+    }
     W.g = HeadGeom{s.num_heads, s.num_kv_heads, s.qk_dim, s.v_dim, pad_to(s.qk_dim, 16), pad_to(s.v_dim, 16)};
     W.attn_cols = pad_to(s.num_heads * s.v_dim, 16);
     W.ff_cols = s.ff_kind == MI_FF_NONE ? 0 : pad_to(s.ff_size, 16);
@@ -195,7 +340,8 @@ int stack_create(mi_ctx* c, const mi_stack_config& cfg) {
   }
   MI_TRY(alloc_norm(c, S->final_norm));
   MI_TRY(alloc_mat(c, S->head, cfg.vocab_size, S->D, 1.f));
-  want("final.norm"); want("final.norm.b"); want("head");
+  want("final.norm"); want("head");
+  if (cfg.norm_groups == 0) want("final.norm.b");
   MI_HIP(hipStreamSynchronize(c->stream));
   return MI_OK;
 }
@@ -204,12 +350,15 @@ void stack_destroy(mi_ctx* c) {
   Stack* S = c->stack;
   for (StackLayer& W : S->layers) {
     free_mat(W.qkv); free_mat(W.up); free_mat(W.out);
-    free_norm(W.n1); free_norm(W.n2);
-    hipFree(W.slopes);
+    free_mat(W.down);
+    free_norm(W.n1); free_norm(W.n2); free_norm(W.n1b); free_norm(W.n2b);
+    void* ps[] = {W.slopes, W.conv1, W.conv2, W.c_norm, W.w_uk, W.w_uv, W.router, W.router_b, W.expert_gu, W.expert_down};
+    for (void* p : ps) hipFree(p);
   }
   free_mat(S->loop_in); free_mat(S->head);
   free_norm(S->final_norm);
-  void* ptrs[] = {S->embed, S->pos, S->x0, S->qkv_out, S->logits_pad, S->n1, S->n2, S->q, S->cat, S->pair, S->attn_scratch, S->residuals};
+  void* ptrs[] = {S->embed, S->pos, S->x0, S->qkv_out, S->logits_pad, S->n1, S->n2, S->q, S->cat, S->pair, S->attn_scratch, S->residuals,
+                  S->y, S->pair_w, S->pair_ids, S->hb, S->act, S->qa, S->lat};
   for (void* p : ptrs) hipFree(p);
   delete S;
   c->stack = nullptr;
@@ -248,10 +397,10 @@ int stack_load_tensor(mi_ctx* c, const std::string& name, const float* dev, int 
     return done(MI_OK);
   };
   if (name == "embed") return table(S->embed, k.vocab_size);
-  if (name == "pos") return table(S->pos, k.max_positions);
+  if (name == "pos" && k.max_positions > 0) return table(S->pos, k.max_positions);
   if (name == "head") return place(S->head, k.vocab_size, S->D);
   if (name == "final.norm") return vec(S->final_norm.w);
-  if (name == "final.norm.b") return vec(S->final_norm.b);
+  if (name == "final.norm.b" && k.norm_groups == 0) return vec(S->final_norm.b);
   if (name == "loop.in" && k.loop_times > 0) {   // [x ; x0]: the halves at columns 0 and Kd
     if (rows != S->D || cols != 2 * S->D) return bad();
     for (int h = 0; h < 2; ++h) MI_TRY(launch_place(dev, cols, h * S->D, rows, S->D, S->loop_in.L.w, S->loop_in.K, S->f32, 0, h * S->Kd, s));
@@ -262,13 +411,20 @@ int stack_load_tensor(mi_ctx* c, const std::string& name, const float* dev, int 
     StackLayer& W = S->layers[l];
     const mi_layer_spec& p = W.s;
     const std::string t = name.substr(at);
+    if (S->sandwich()) {
+      int r = 0, cl = 0;
+      sandwich_tensor_shape(S, W, t, &r, &cl);
+      if (r > 0) return rows == r && cols == cl ? done(sandwich_place(c, W, t, dev, rows, cols)) : bad();
+    }
     const int qn = p.num_heads * p.qk_dim, kn = p.num_kv_heads * p.qk_dim;
-    if (t == "norm1") return vec(W.n1.w);
-    if (t == "norm1.b") return vec(W.n1.b);
-    if (t == "mix.q") return place(W.qkv, qn, S->D);
-    if (t == "mix.k") return place(W.qkv, kn, S->D, qn);
-    if (t == "mix.v") return place(W.qkv, p.num_kv_heads * p.v_dim, S->D, qn + kn);
-    if (t == "mix.o") return place(W.out, S->D, p.num_heads * p.v_dim);
+    if (!S->sandwich()) {
+      if (t == "norm1") return vec(W.n1.w);
+      if (t == "norm1.b") return vec(W.n1.b);
+      if (t == "mix.q") return place(W.qkv, qn, S->D);
+      if (t == "mix.k") return place(W.qkv, kn, S->D, qn);
+      if (t == "mix.v") return place(W.qkv, p.num_kv_heads * p.v_dim, S->D, qn + kn);
+      if (t == "mix.o") return place(W.out, S->D, p.num_heads * p.v_dim);
+    }
     if (W.ff_cols) {
       if (t == "norm2") return vec(W.n2.w);
       if (t == "norm2.b") return vec(W.n2.b);
@@ -291,7 +447,12 @@ int stack_synthetic(mi_ctx* c, uint64_t seed, float std) {
   for (const std::string& n : names) {
     int rows = S->D, cols = 0;
     float sd = std;
-    bool is_norm = n.find("norm") != std::string::npos;
+    bool is_norm = n.find("norm") != std::string::npos || (n.size() > 2 && n.compare(n.size() - 2, 2, ".b") == 0);
+    if (is_norm && S->sandwich() && n[0] == 'l') {
+      int r = 0, k0 = 0;
+      sandwich_tensor_shape(S, S->layers[atoi(n.c_str() + 1)], n.substr(n.find('.') + 1), &r, &k0);
+      rows = r;
+    }
     if (n == "embed" || n == "head") { rows = k.vocab_size; cols = S->D; if (n == "embed") sd = 1.f; }
     else if (n == "pos") { rows = k.max_positions; cols = S->D; sd = 0.1f; }
     else if (n == "loop.in") cols = 2 * S->D;
@@ -300,7 +461,10 @@ int stack_synthetic(mi_ctx* c, uint64_t seed, float std) {
       const mi_layer_spec& p = S->layers[l].s;
       const std::string t = n.substr(n.find('.') + 1);
       cols = S->D;
-      if (t == "mix.q") rows = p.num_heads * p.qk_dim;
+      if (S->sandwich()) {
+        sandwich_tensor_shape(S, S->layers[l], t, &rows, &cols);
+        if (t.compare(0, 5, "canon") == 0) sd = 0.3f;
+      } else if (t == "mix.q") rows = p.num_heads * p.qk_dim;
       else if (t == "mix.k") rows = p.num_kv_heads * p.qk_dim;
       else if (t == "mix.v") rows = p.num_kv_heads * p.v_dim;
       else if (t == "mlp.up") rows = p.ff_size;
@@ -327,11 +491,28 @@ void stack_artifact_tensors(mi_ctx* c, std::vector<std::pair<void*, size_t>>& ou
   Stack* S = c->stack;
   const size_t nb = (size_t)S->ld * 4;
   auto mat = [&](StackMat& m) { out.push_back({m.L.w, (size_t)m.N * m.K * S->elem()}); };
-  auto norm = [&](StackNorm& n) { out.push_back({n.w, nb}); out.push_back({n.b, nb}); };
+  auto norm = [&](StackNorm& n) { out.push_back({n.w, nb}); out.push_back({n.b, nb}); };   // (an RMS norm's bias is zero)
   out.push_back({S->embed, (size_t)S->cfg.vocab_size * S->D * S->elem()});
-  out.push_back({S->pos, (size_t)S->cfg.max_positions * S->D * S->elem()});
+  if (S->pos) out.push_back({S->pos, (size_t)S->cfg.max_positions * S->D * S->elem()});
   if (S->cfg.loop_times > 0) mat(S->loop_in);
   for (StackLayer& W : S->layers) {
+    if (S->sandwich()) {
+      const mi_layer_spec& p = W.s;
+      auto put = [&](void* q, size_t bytes) { if (q) out.push_back({q, bytes}); };
+      const size_t el = S->elem(), cb = (size_t)S->cfg.conv_taps * S->ld * 4;
+      mat(W.qkv); mat(W.out);
+      put(W.n1.w, nb); put(W.n1b.w, nb); put(W.n2.w, nb); put(W.n2b.w, nb);
+      put(W.conv1, cb); put(W.conv2, cb); put(W.c_norm, (size_t)p.kv_rank * 4);
+      put(W.w_uk, (size_t)p.num_heads * W.lg.rp * W.lg.dkp * el);
+      put(W.w_uv, (size_t)p.num_heads * W.lg.dvp * W.lg.rp * el);
+      if (p.ff_kind == MI_FF_GLU) { mat(W.up); mat(W.down); }
+      if (p.ff_kind == MI_FF_MOE) {
+        const ExpertsLinear gu = W.expert_up(), dn = W.expert_dn();
+        put(W.router, (size_t)p.experts * S->Kd * el); put(W.router_b, (size_t)p.experts * 4);
+        put(W.expert_gu, (size_t)gu.E * gu.N * gu.K * el); put(W.expert_down, (size_t)dn.E * dn.N * dn.K * el);
+      }
+      continue;
+    }
     mat(W.qkv); mat(W.out); norm(W.n1);
     if (W.ff_cols) { mat(W.up); norm(W.n2); }
   }
@@ -346,13 +527,18 @@ int stack_geometry_hash(const mi_ctx* c) {
     for (size_t i = 0; i < n; ++i) h = (h ^ reinterpret_cast<const unsigned char*>(p)[i]) * 16777619u;
   };
   const mi_stack_config& k = S->cfg;
-  const int32_t g[7] = {k.num_layers, k.width, k.vocab_size, k.max_positions, k.loop_times > 0, k.compute_dtype, 0};
+  const int32_t g[9] = {k.num_layers, k.width, k.vocab_size, k.max_positions, k.loop_times > 0, k.compute_dtype, k.block_kind, k.norm_groups, k.conv_taps};
   mix(g, sizeof g);
   for (const StackLayer& W : S->layers) mix(&W.s, sizeof W.s);
   return (int)(h & 0x7fffffff);
 }
 
-static size_t kv_run_elems_per_block(const mi_ctx* c, const StackLayer& W) { return (size_t)W.g.G * c->cfg.block_size * (W.g.dkp + W.g.dvp); }
+static size_t kv_run_elems_per_block(const mi_ctx* c, const StackLayer& W) {
+  const Stack* S = c->stack;
+  if (S->sandwich())   // latents (own ones) and both convolutions' state
+    return (W.s.kv_from < 0 ? (size_t)c->cfg.block_size * W.lg.rp : 0) + (size_t)S->conv_keep * S->Kd * (W.s.ff_kind == MI_FF_NONE ? 1 : 2);
+  return (size_t)W.g.G * c->cfg.block_size * (W.g.dkp + W.g.dvp);
+}
 size_t stack_kv_bytes_per_block(const mi_ctx* c) {
   size_t e = 0;
   for (const StackRun& r : c->stack->runs) e += kv_run_elems_per_block(c, c->stack->layers[r.layer]);
@@ -361,6 +547,7 @@ size_t stack_kv_bytes_per_block(const mi_ctx* c) {
 
 static size_t stack_scratch(const mi_ctx* c) {
   size_t b = 16;
+  if (c->stack->sandwich()) return b;
   for (const StackLayer& W : c->stack->layers) b = std::max(b, attn_window_scratch_bytes(c->cfg.max_num_seqs, W.g));
   return b;
 }
@@ -369,6 +556,10 @@ size_t stack_workspace_estimate(const mi_ctx* c) {
   const Stack* S = c->stack;
   const size_t R = (size_t)c->max_rows;
   size_t b = 3 * R * S->ld * 4 + R * S->qkv_ld * 4 + R * (4 * (size_t)S->Kd + S->q_cols + S->cat_ld) * S->elem();
+  if (S->sandwich()) {
+    const size_t pairs = R * std::max(1, S->max_top);
+    b += pairs * S->ld * 4 + pairs * 8 + R * S->Kd * S->elem() + pairs * S->act_ld * S->elem() + 2 * R * S->lat_cols * S->elem();
+  }
   b += (size_t)64 << 20;
   b += 2 * (size_t)c->cfg.max_num_seqs * pad_to(c->V_l, 16) * 4;
   return b + stack_scratch(c) + ((size_t)8 << 20);
@@ -395,15 +586,31 @@ int stack_alloc(mi_ctx* c) {
   MI_TRY(alloc0(c, &c->kv_pool, kv_bytes, &c->kv_bytes));
   size_t at = 0;
   for (const StackRun& r : S->runs) {
-    S->kv_at.push_back(at);
-    at += kv_run_elems_per_block(c, S->layers[r.layer]) * k.num_blocks;
+    const StackLayer& W = S->layers[r.layer];
+    const bool shared = S->sandwich() && W.s.kv_from >= 0;
+    S->kv_at.push_back(shared ? S->kv_at[W.s.kv_from] : at);
+    if (S->sandwich()) S->conv_at.push_back(at + (shared ? 0 : (size_t)k.num_blocks * k.block_size * W.lg.rp));
+    at += kv_run_elems_per_block(c, W) * k.num_blocks;
   }
   const size_t R = (size_t)c->max_rows;
   size_t* ws = &c->workspace_bytes;
   MI_TRY(alloc0(c, &c->resid[0], R * S->ld * 4, ws));
   MI_TRY(alloc0(c, &c->resid[1], R * S->ld * 4, ws));
   MI_TRY(alloc0(c, &S->n1, R * S->Kd * S->elem(), ws));
-  MI_TRY(alloc0(c, &S->n2, R * S->Kd * S->elem(), ws));
+  if (S->sandwich()) {
+    const size_t pairs = R * std::max(1, S->max_top);   // (a dense feed-forward: one "pair" per row)
+    MI_TRY(alloc0(c, &S->y, pairs * S->ld * 4, ws));
+    MI_TRY(alloc0(c, &S->hb, R * S->Kd * S->elem(), ws));
+    if (S->act_ld) MI_TRY(alloc0(c, &S->act, pairs * S->act_ld * S->elem(), ws));
+    MI_TRY(alloc0(c, &S->qa, R * S->lat_cols * S->elem(), ws));
+    MI_TRY(alloc0(c, &S->lat, R * S->lat_cols * S->elem(), ws));
+    if (S->max_top) {
+      MI_TRY(alloc0(c, &S->pair_w, pairs * 4, ws));
+      MI_TRY(alloc0(c, &S->pair_ids, pairs * 4, ws));
+    }
+  } else {
+    MI_TRY(alloc0(c, &S->n2, R * S->Kd * S->elem(), ws));
+  }
   MI_TRY(alloc0(c, &S->qkv_out, R * S->qkv_ld * 4, ws));
   MI_TRY(alloc0(c, &S->q, R * S->q_cols * S->elem(), ws));
   MI_TRY(alloc0(c, &S->cat, R * S->cat_ld * S->elem(), ws));
@@ -416,6 +623,122 @@ int stack_alloc(mi_ctx* c) {
   return MI_OK;
 }
 
+namespace {
+
+// ---- sandwich blocks ---------------------------------------------------------------------------------------------------------
+struct Batch { int rows; bool decode; int MB; const AttnSeg* segs; int nseg; };
+
+// x += post-norm of src; pre-norm and convolution -> S->n1.  cur: which residual buffer holds x
+int sandwich_norm(mi_ctx* c, int& cur, const Batch& b, RowSource& src, const float* w_post, const float* w_pre, const float* conv_w, size_t conv_at) {
+  Stack* S = c->stack;
+  if (!runs_other(c)) { if (src.any()) cur ^= 1; src = RowSource(); return MI_OK; }
+  Scope sc(c, MI_K_OTHER);
+  ConvState cs;
+  cs.w = conv_w;
+  cs.taps = S->cfg.conv_taps;
+  cs.keep = S->conv_keep;
+  cs.ring = reinterpret_cast<unsigned char*>(c->kv_pool) + conv_at * S->elem();
+  cs.block_size = c->cfg.block_size;
+  cs.MB = b.MB;
+  cs.bt = c->d_bt; cs.pos = c->d_pos; cs.slots = c->d_slots;
+  const bool fused = b.decode || !w_pre;
+  MI_TRY(launch_sandwich_rows(c->resid[cur], c->resid[cur ^ 1], src, w_post, w_pre, b.rows, S->D, S->ld, S->cfg.norm_groups, S->cfg.norm_eps,
+                              fused && w_pre ? &cs : nullptr, fused ? S->n1 : S->hb, S->Kd, S->f32, c->stream));
+  if (src.any()) cur ^= 1;
+  src = RowSource();
+  if (fused) return MI_OK;
+  return launch_conv_rows(S->hb, cs, reinterpret_cast<const AttnSeg*>(c->d_segs), b.segs, b.nseg, S->D, S->ld, S->n1, S->Kd, S->f32, c->stream);
+}
+
+int latent_mixer(mi_ctx* c, const StackLayer& W, size_t kv_at, const Batch& b, RowSource& out) {
+  Stack* S = c->stack;
+  const mi_model_config& k = c->cfg;
+  const LatentGeom& g = W.lg;
+  hipStream_t s = c->stream;
+  EpiArgs e{};
+  e.out_f32 = S->qkv_out; e.ld_out = S->qkv_ld;
+  MI_TRY(apply(c, W.qkv, b.rows, S->n1, S->Kd, EPI_F32, e));
+  unsigned char* pool = reinterpret_cast<unsigned char*>(c->kv_pool) + kv_at * S->elem();
+  if (runs_other(c)) {
+    Scope sc(c, MI_K_OTHER);
+    MI_TRY(launch_latent_scatter(S->qkv_out, S->qkv_ld, b.rows, g, W.c_norm, S->cfg.norm_eps, c->d_slots, k.block_size, S->q, pool, S->f32, s));
+    MI_TRY(launch_head_linear(W.w_uk, g.H, g.rp, g.dkp, S->q, b.rows, S->qa, g.H * g.rp, g.rp, g.rp, S->f32, s));
+  }
+  {
+    Scope sc(c, b.decode ? MI_K_ATTN_DECODE : MI_K_ATTN_PREFILL);
+    MI_TRY(launch_attn_plain(W.latent, S->qa, pool, pool, k.block_size, c->d_bt, b.MB, c->d_pos, b.decode ? nullptr : reinterpret_cast<const AttnSeg*>(c->d_segs),
+                             b.nseg, b.rows, S->lat, g.H * g.rp, S->f32, s));
+  }
+  if (runs_other(c)) {
+    Scope sc(c, MI_K_OTHER);
+    MI_TRY(launch_head_linear(W.w_uv, g.H, g.dvp, g.rp, S->lat, b.rows, S->cat, S->cat_ld, g.dv, g.dv, S->f32, s));
+  }
+  EpiArgs o{};
+  o.out_f32 = S->y; o.ld_out = S->ld;
+  out.y = S->y; out.ld = S->ld;
+  return apply(c, W.out, b.rows, S->cat, S->cat_ld, EPI_F32, o, b.rows >= 384 ? &out.slabs : nullptr);
+}
+
+int gated_ff(mi_ctx* c, const StackLayer& W, int rows, RowSource& out) {
+  Stack* S = c->stack;
+  EpiArgs e{};
+  e.act_out = reinterpret_cast<uint16_t*>(S->act); e.ld_act = S->act_ld;
+  e.glu_limit = W.s.ff_limit; e.glu_alpha = W.s.ff_alpha;
+  MI_TRY(apply(c, W.up, rows, S->n1, S->Kd, EPI_GLU_CLIP, e));
+  EpiArgs o{};
+  o.out_f32 = S->y; o.ld_out = S->ld;
+  out.y = S->y; out.ld = S->ld;
+  return apply(c, W.down, rows, S->act, S->act_ld, EPI_F32, o, rows >= 384 ? &out.slabs : nullptr);
+}
+
+int expert_ff(mi_ctx* c, const StackLayer& W, int rows, RowSource& out) {
+  Stack* S = c->stack;
+  const mi_layer_spec& p = W.s;
+  const int pairs = rows * p.experts_top;
+  if (runs_other(c)) {
+    Scope sc(c, MI_K_OTHER);
+    MI_TRY(launch_route(S->n1, S->Kd, rows, W.router, W.router_b, p.experts, S->Kd, p.experts_top, S->pair_ids, S->pair_w, S->f32, c->stream));
+  }
+  const int cls = rows <= 32 && !S->f32 ? MI_K_GEMV : MI_K_GEMM;
+  if (c->runs(cls)) {
+    Scope sc(c, cls);
+    MI_TRY(launch_experts_linear(W.expert_up(), S->pair_ids, pairs, S->n1, S->Kd, p.experts_top, true, S->act, S->act_ld, S->f32, c->stream));
+  }
+  if (c->runs(cls)) {
+    Scope sc(c, cls);
+    MI_TRY(launch_experts_linear(W.expert_dn(), S->pair_ids, pairs, S->act, S->act_ld, 1, false, S->y, S->ld, S->f32, c->stream));
+  }
+  out.y = S->y; out.ld = S->ld;
+  out.pair_w = S->pair_w; out.top = p.experts_top;
+  return MI_OK;
+}
+
+int sandwich_trunk(mi_ctx* c, const Batch& b, int& cur) {
+  Stack* S = c->stack;
+  RowSource src;
+  const float* w_post = nullptr;
+  auto keep = [&](size_t run) -> int {   // the stream behind layer run `run` is complete once its last sublayer is added
+    if (S->residuals)
+      MI_HIP(hipMemcpyAsync(S->residuals + run * c->max_rows * S->ld, c->resid[cur], (size_t)b.rows * S->ld * 4, hipMemcpyDeviceToDevice, c->stream));
+    return MI_OK;
+  };
+  for (size_t i = 0; i < S->runs.size(); ++i) {
+    const StackLayer& W = S->layers[S->runs[i].layer];
+    MI_TRY(sandwich_norm(c, cur, b, src, w_post, W.n1.w, W.conv1, S->conv_at[i]));
+    if (i > 0) MI_TRY(keep(i - 1));
+    MI_TRY(latent_mixer(c, W, S->kv_at[i], b, src));
+    w_post = W.n1b.w;
+    if (W.s.ff_kind == MI_FF_NONE) continue;
+    MI_TRY(sandwich_norm(c, cur, b, src, w_post, W.n2.w, W.conv2, S->conv_at[i] + (size_t)c->cfg.num_blocks * S->conv_keep * S->Kd));
+    MI_TRY(W.s.ff_kind == MI_FF_MOE ? expert_ff(c, W, b.rows, src) : gated_ff(c, W, b.rows, src));
+    w_post = W.n2b.w;
+  }
+  MI_TRY(sandwich_norm(c, cur, b, src, w_post, nullptr, nullptr, 0));
+  return keep(S->runs.size() - 1);
+}
+
+}  // namespace
+
 int stack_trunk(mi_ctx* c, int rows, bool decode, int MB, const AttnSeg* segs, int nseg) {
   Stack* S = c->stack;
   hipStream_t s = c->stream;
@@ -424,6 +747,11 @@ int stack_trunk(mi_ctx* c, int rows, bool decode, int MB, const AttnSeg* segs, i
   if (runs_other(c)) {
     Scope sc(c, MI_K_OTHER);
     MI_TRY(launch_embed_pos(c->d_ids, c->d_pos, S->embed, S->pos, S->f32, rows, S->D, S->ld, c->resid[0], S->x0, s));
+  }
+  if (S->sandwich()) {
+    MI_TRY(sandwich_trunk(c, Batch{rows, decode, MB, segs, nseg}, cur));
+    c->tail_cur = cur;
+    return MI_OK;
   }
   for (size_t i = 0; i < S->runs.size(); ++i) {
     const StackRun& run = S->runs[i];
@@ -474,13 +802,17 @@ int stack_head(mi_ctx* c, const float* resid, int nrows) {
   Stack* S = c->stack;
   if (runs_other(c)) {
     Scope sc(c, MI_K_OTHER);
-    MI_TRY(launch_layernorm_rows(resid, nullptr, nrows, S->D, S->ld, S->cfg.norm_eps, NormOut{S->final_norm.w, S->final_norm.b, S->n1}, NormOut{}, S->Kd, S->f32, c->stream));
+    if (S->cfg.norm_groups > 0)
+      MI_TRY(launch_sandwich_rows(resid, nullptr, RowSource(), nullptr, S->final_norm.w, nrows, S->D, S->ld, S->cfg.norm_groups, S->cfg.norm_eps, nullptr, S->n1, S->Kd, S->f32, c->stream));
+    else
+      MI_TRY(launch_layernorm_rows(resid, nullptr, nrows, S->D, S->ld, S->cfg.norm_eps, NormOut{S->final_norm.w, S->final_norm.b, S->n1}, NormOut{}, S->Kd, S->f32, c->stream));
   }
   const bool direct = c->V_l % 16 == 0;
   EpiArgs e{};
   e.out_f32 = direct ? c->logits : S->logits_pad;
   e.ld_out = S->head.N;
-  MI_TRY(apply(c, S->head, nrows, S->n1, S->Kd, EPI_F32, e));
+  e.softcap = S->cfg.logit_softcap;
+  MI_TRY(apply(c, S->head, nrows, S->n1, S->Kd, e.softcap > 0.f ? EPI_SOFTCAP : EPI_F32, e));
   if (!direct) {
     Scope sc(c, MI_K_OTHER);
     MI_TRY(launch_pack_rows(S->logits_pad, S->head.N, nrows, c->V_l, c->logits, c->stream));

@@ -38,14 +38,19 @@ __global__ __launch_bounds__(256) void embed_pos_kernel(const int32_t* __restric
                                                         float* __restrict__ resid, float* __restrict__ x0) {
   const int t = blockIdx.x;
   const T* e = table + (size_t)ids[t] * D;
-  const T* p = ptable + (size_t)pos[t] * D;
+  const T* p = ptable ? ptable + (size_t)pos[t] * D : nullptr;
   for (int d = threadIdx.x * 4; d < ld; d += 1024) {
     float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
     if ((D & 3) == 0) {
       if (d < D) {
-        const float4 a = get4(e + d), b = get4(p + d);
+        const float4 a = get4(e + d), b = p ? get4(p + d) : make_float4(0.f, 0.f, 0.f, 0.f);
         v = make_float4(a.x + b.x, a.y + b.y, a.z + b.z, a.w + b.w);
       }
+    } else if (!p) {
+      if (d < D) v.x = to_f32(e[d]);
+      if (d + 1 < D) v.y = to_f32(e[d + 1]);
+      if (d + 2 < D) v.z = to_f32(e[d + 2]);
+      if (d + 3 < D) v.w = to_f32(e[d + 3]);
     } else {
       if (d < D) v.x = to_f32(e[d]) + to_f32(p[d]);
       if (d + 1 < D) v.y = to_f32(e[d + 1]) + to_f32(p[d + 1]);
@@ -102,6 +107,164 @@ __global__ __launch_bounds__(1024) void layernorm_rows_kernel(const float* __res
     };
     if (na.y) emit(na);
     if (nb.y) emit(nb);
+  }
+}
+
+__device__ __forceinline__ float round_to(float v, const uint16_t*) { return bf16_to_f32(f32_to_bf16(v)); }
+__device__ __forceinline__ float round_to(float v, const float*) { return v; }
+
+// 1 / sqrt(mean square + eps) of every one of G equal parts of the D floats in `row`, into rstd [G].  A part is shared out to
+// several waves where there are fewer parts than waves; summed in wave order.  red: max(G, waves) floats.
+__device__ __forceinline__ void group_rstd(const float* row, int D, int G, float eps, float* red, float* rstd) {
+  const int nw = blockDim.x >> 6, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int gs = D / G, P = max(1, nw / G), len = ceil_div(gs, P);
+  __syncthreads();                      // the row is complete
+  for (int u = wave; u < G * P; u += nw) {
+    const int g = u / P, lo = g * gs + (u - g * P) * len, hi = min(lo + len, (g + 1) * gs);
+    float s = 0.f;
+    for (int i = lo + lane; i < hi; i += 64) s = __builtin_fmaf(row[i], row[i], s);
+    s = wave_sum(s);
+    if (lane == 0) red[u] = s;
+  }
+  __syncthreads();
+  for (int g = threadIdx.x; g < G; g += blockDim.x) {
+    float s = 0.f;
+    for (int p = 0; p < P; ++p) s += red[g * P + p];
+    rstd[g] = 1.0f / sqrtf(s / (float)gs + eps);
+  }
+  __syncthreads();
+}
+// part of element d (exact: d < 2^15, the quotient is at least 0.5 / gs away from an integer)
+__device__ __forceinline__ int part_of(int d, float inv_gs) { return (int)(((float)d + 0.5f) * inv_gs); }
+__device__ __forceinline__ float4 part_rstd(const float* rstd, int d, int G, float inv_gs) {
+  if (G == 1) return make_float4(rstd[0], rstd[0], rstd[0], rstd[0]);
+  auto at = [&](int i) { return rstd[min(part_of(d + i, inv_gs), G - 1)]; };
+  return make_float4(at(0), at(1), at(2), at(3));
+}
+
+__device__ __forceinline__ float4 source_row4(const RowSource& src, int t, int d) {
+  float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+  if (src.slabs.slab) {
+    for (int z = 0; z < src.slabs.KS; ++z) {
+      const float4 q = *reinterpret_cast<const float4*>(src.slabs.slab + ((size_t)z * src.slabs.T + t) * src.slabs.N + d);
+      v.x += q.x; v.y += q.y; v.z += q.z; v.w += q.w;
+    }
+    const float4 sc = *reinterpret_cast<const float4*>(src.slabs.scale + d);
+    v.x *= sc.x; v.y *= sc.y; v.z *= sc.z; v.w *= sc.w;
+  } else if (src.pair_w) {
+    for (int j = 0; j < src.top; ++j) {
+      const size_t r = (size_t)t * src.top + j;
+      const float w = src.pair_w[r];
+      const float4 q = *reinterpret_cast<const float4*>(src.y + r * src.ld + d);
+      v.x = __builtin_fmaf(w, q.x, v.x); v.y = __builtin_fmaf(w, q.y, v.y);
+      v.z = __builtin_fmaf(w, q.z, v.z); v.w = __builtin_fmaf(w, q.w, v.w);
+    }
+  } else {
+    v = *reinterpret_cast<const float4*>(src.y + (size_t)t * src.ld + d);
+  }
+  return v;
+}
+
+// the convolution's sum for channels d .. d + 3 at position p; past(back) = input `back` positions earlier (called where p >= back)
+template <typename F>
+__device__ __forceinline__ float4 conv_sum(const ConvState& cs, int ld, int d, int p, float4 h, F past) {
+  float4 a = make_float4(0.f, 0.f, 0.f, 0.f);
+  for (int j = 0; j < cs.taps; ++j) {
+    const int back = cs.taps - 1 - j;
+    if (back > p) continue;
+    const float4 v = back == 0 ? h : past(back), w = *reinterpret_cast<const float4*>(cs.w + (size_t)j * ld + d);
+    a.x = __builtin_fmaf(w.x, v.x, a.x); a.y = __builtin_fmaf(w.y, v.y, a.y);
+    a.z = __builtin_fmaf(w.z, v.z, a.z); a.w = __builtin_fmaf(w.w, v.w, a.w);
+  }
+  return make_float4(h.x + a.x, h.y + a.y, h.z + a.z, h.w + a.w);
+}
+template <typename T>
+__device__ __forceinline__ T* ring_at(const ConvState& cs, int blk, int off, int ldy) {
+  return reinterpret_cast<T*>(cs.ring) + ((size_t)blk * cs.keep + off % cs.keep) * ldy;
+}
+template <typename T>
+__device__ __forceinline__ float4 ring_get4(const ConvState& cs, int seq, int p, int ldy, int d) {
+  return get4(ring_at<T>(cs, cs.bt[(size_t)seq * cs.MB + p / cs.block_size], p % cs.block_size, ldy) + d);
+}
+
+template <typename T>
+__global__ __launch_bounds__(1024) void sandwich_rows_kernel(const float* __restrict__ resid_in, float* __restrict__ resid_out, RowSource src,
+                                                            const float* __restrict__ w_post, const float* __restrict__ w_pre, int D, int ld,
+                                                            int G, float eps, ConvState cs, T* __restrict__ y, int ldy) {
+  extern __shared__ __attribute__((aligned(16))) float row[];   // ld + max(G, 16) + G floats
+  float *red = row + ld, *rstd = red + max(G, 16);
+  const int t = blockIdx.x, tid = threadIdx.x, nthr = blockDim.x;
+  const size_t o = (size_t)t * ld;
+  const float inv_gs = 1.0f / (float)(D / G);
+  const bool add = src.y || src.slabs.slab;
+  if (add) {
+    for (int d = tid * 4; d < ld; d += nthr * 4) *reinterpret_cast<float4*>(row + d) = source_row4(src, t, d);
+    group_rstd(row, D, G, eps, red, rstd);
+  }
+  for (int d = tid * 4; d < ld; d += nthr * 4) {   // (a thread reads back what it wrote itself)
+    float4 x = *reinterpret_cast<const float4*>(resid_in + o + d);
+    if (add) {
+      const float4 v = *reinterpret_cast<const float4*>(row + d), w = *reinterpret_cast<const float4*>(w_post + d), r = part_rstd(rstd, d, G, inv_gs);
+      x.x = __builtin_fmaf(v.x * r.x, w.x, x.x); x.y = __builtin_fmaf(v.y * r.y, w.y, x.y);
+      x.z = __builtin_fmaf(v.z * r.z, w.z, x.z); x.w = __builtin_fmaf(v.w * r.w, w.w, x.w);
+      *reinterpret_cast<float4*>(resid_out + o + d) = x;
+    }
+    *reinterpret_cast<float4*>(row + d) = x;
+  }
+  if (!w_pre) return;
+  group_rstd(row, D, G, eps, red, rstd);
+  const int p = cs.w ? cs.pos[t] : 0, slot = cs.w ? cs.slots[t] : -1;
+  for (int d = tid * 4; d < ld; d += nthr * 4) {
+    const float4 x = *reinterpret_cast<const float4*>(row + d), w = *reinterpret_cast<const float4*>(w_pre + d), r = part_rstd(rstd, d, G, inv_gs);
+    float4 h = make_float4(x.x * r.x * w.x, x.y * r.y * w.y, x.z * r.z * w.z, x.w * r.w * w.w);
+    if (cs.w) {
+      h = make_float4(round_to(h.x, y), round_to(h.y, y), round_to(h.z, y), round_to(h.w, y));
+      const float4 a = conv_sum(cs, ld, d, p, h, [&](int back) { return ring_get4<T>(cs, t, p - back, ldy, d); });
+      if (slot >= 0 && cs.keep > 0) put4(ring_at<T>(cs, slot / cs.block_size, slot % cs.block_size, ldy) + d, h.x, h.y, h.z, h.w);
+      h = a;
+    }
+    put4(y + (size_t)t * ldy + d, h.x, h.y, h.z, h.w);
+  }
+}
+
+// One work-group: up to kConvRows rows of one segment x 1024 channels.
+// The rows at a segment's start read the state of the positions ahead of it, and rows further on renew it.  Both may meet in one
+// place only in the block that holds the position ahead of the segment; that block's renewal is left to the work-group of the
+// segment's first rows, whose threads have read their channels' state by then (kConvRows >= taps - 1).
+constexpr int kConvRows = 16;
+template <typename T>
+__global__ __launch_bounds__(256) void conv_rows_kernel(const T* __restrict__ hin, ConvState cs, const AttnSeg* __restrict__ segs, int nseg,
+                                                        int ld, T* __restrict__ y, int ldy) {
+  int tile = blockIdx.x, si = 0;
+  AttnSeg sg{0, 0, 0, 0};
+  for (; si < nseg; ++si) {
+    sg = segs[si];
+    const int n = ceil_div(sg.n, kConvRows);
+    if (tile < n) break;
+    tile -= n;
+  }
+  const int d = (blockIdx.y * 256 + threadIdx.x) * 4;
+  if (si == nseg || d >= ld) return;
+  const int bs = cs.block_size, first = tile * kConvRows, last = min(first + kConvRows, sg.n), end = sg.pos0 + sg.n;
+  const int shared_block = sg.pos0 % bs ? sg.pos0 / bs : -1;      // holds positions on both sides of the segment's start
+  auto renew = [&](int p, float4 h) {
+    const int slot = cs.slots[sg.row0 + p - sg.pos0];
+    if (slot >= 0) put4(ring_at<T>(cs, slot / bs, slot % bs, ldy) + d, h.x, h.y, h.z, h.w);
+  };
+  for (int i = first; i < last; ++i) {
+    const int p = sg.pos0 + i;
+    const size_t r = (size_t)(sg.row0 + i) * ldy + d;
+    const float4 h = get4(hin + r);
+    const float4 a = conv_sum(cs, ld, d, p, h, [&](int back) {
+      return back <= i ? get4(hin + r - (size_t)back * ldy) : ring_get4<T>(cs, sg.seq, p - back, ldy, d);
+    });
+    put4(y + r, a.x, a.y, a.z, a.w);
+    const int b = p / bs;
+    if (b != shared_block && p + cs.keep >= min(end, (b + 1) * bs)) renew(p, h);
+  }
+  if (tile == 0 && shared_block >= 0) {
+    const int stop = min(end, (shared_block + 1) * bs);
+    for (int p = max(sg.pos0, stop - cs.keep); p < stop; ++p) renew(p, get4(hin + (size_t)(sg.row0 + p - sg.pos0) * ldy + d));
   }
 }
 
@@ -194,6 +357,18 @@ __global__ __launch_bounds__(256) void linear_f32_kernel(const float* __restrict
 #pragma unroll
       for (int j = 0; j < 4; ++j) { v[j] = fmaxf(v[j], 0.f); v[j] *= v[j]; }
       put4(reinterpret_cast<float*>(e.act_out) + (size_t)m * e.ld_act + n0 + tn, v[0], v[1], v[2], v[3]);
+    } else if constexpr (EPI == EPI_GLU_CLIP) {
+      float a[2];
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        const float g = fminf(v[2 * j], e.glu_limit), u = fminf(fmaxf(v[2 * j + 1], -e.glu_limit), e.glu_limit);
+        a[j] = g / (1.f + expf(-e.glu_alpha * g)) * (u + 1.f);
+      }
+      *reinterpret_cast<float2*>(reinterpret_cast<float*>(e.act_out) + (size_t)m * e.ld_act + ((n0 + tn) >> 1)) = make_float2(a[0], a[1]);
+    } else if constexpr (EPI == EPI_SOFTCAP) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[j] = e.softcap * tanhf(v[j] / e.softcap);
+      put4(e.out_f32 + (size_t)m * e.ld_out + n0 + tn, v[0], v[1], v[2], v[3]);
     } else {
       if constexpr (EPI == EPI_RESID) {
         const float4 r = *reinterpret_cast<const float4*>(e.resid_in + (size_t)m * e.ld_out + n0 + tn);
@@ -205,7 +380,7 @@ __global__ __launch_bounds__(256) void linear_f32_kernel(const float* __restrict
 }
 
 __global__ void place_tiled_kernel(const float* __restrict__ src, int ld, int src_col0, int rows, int cols, uint16_t* __restrict__ dst,
-                                   int KT, int row0, int col0) {
+                                   int KT, int row0, int col0, int row_step) {
   const int c8n = (cols + 7) / 8;
   const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= (size_t)rows * c8n) return;
@@ -214,16 +389,26 @@ __global__ void place_tiled_kernel(const float* __restrict__ src, int ld, int sr
   float v[8];
 #pragma unroll
   for (int k = 0; k < 8; ++k) v[k] = c + k < cols ? p[k] : 0.f;
-  const int R = row0 + r, C = col0 + c;
+  const int R = row0 + r * row_step, C = col0 + c;
   const size_t at = (((size_t)(R >> 4) * KT + (C >> 5)) * 64 + (R & 15) + 16 * ((C & 31) >> 3)) * 8;
   *reinterpret_cast<uint4*>(dst + at) = make_uint4(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]), pack_bf16x2(v[4], v[5]), pack_bf16x2(v[6], v[7]));
 }
 __global__ void place_f32_kernel(const float* __restrict__ src, int ld, int src_col0, int rows, int cols, float* __restrict__ dst, int K,
-                                 int row0, int col0) {
+                                 int row0, int col0, int row_step) {
   const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= (size_t)rows * cols) return;
   const int r = (int)(i / cols), c = (int)(i % cols);
-  dst[(size_t)(row0 + r) * K + col0 + c] = src[(size_t)r * ld + src_col0 + c];
+  dst[(size_t)(row0 + r * row_step) * K + col0 + c] = src[(size_t)r * ld + src_col0 + c];
+}
+__global__ void place_rows_bf16_kernel(const float* __restrict__ src, int rows, int cols, uint16_t* __restrict__ dst, int K) {
+  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= (size_t)rows * cols) return;
+  dst[(i / cols) * K + i % cols] = f32_to_bf16(src[i]);
+}
+__global__ void transpose_kernel(const float* __restrict__ src, int rows, int cols, float* __restrict__ dst, int ld_dst) {
+  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= (size_t)rows * cols) return;
+  dst[(i % cols) * ld_dst + i / cols] = src[i];
 }
 __global__ void pack_rows_kernel(const float* __restrict__ src, int ld_src, int V, float* __restrict__ dst) {
   for (int v = blockIdx.x * blockDim.x + threadIdx.x; v < V; v += gridDim.x * blockDim.x)
@@ -259,6 +444,50 @@ int launch_layernorm_rows(const float* resid_in, float* resid_out, int T, int D,
   return MI_OK;
 }
 
+static int check_conv(const ConvState& c) {
+  MI_CHECK(c.taps >= 1 && c.taps <= kConvRows && c.block_size > 0 && c.bt && c.pos && c.slots && c.MB >= 1, "convolution: taps / block table");
+  MI_CHECK(c.taps == 1 || (c.ring && (c.keep >= c.taps - 1 || c.keep == c.block_size)), "convolution: state rows per block");
+  return MI_OK;
+}
+
+int launch_sandwich_rows(const float* resid_in, float* resid_out, const RowSource& src, const float* w_post, const float* w_pre, int T,
+                         int D, int ld, int groups, float eps, const ConvState* conv, void* y, int ldy, bool f32, hipStream_t s) {
+  MI_CHECK(T >= 1 && ld % 4 == 0 && ld >= D && ld <= 32768 && groups >= 1 && D % groups == 0, "sandwich rows: row stride / norm groups");
+  MI_CHECK(!src.any() || (resid_out && resid_out != resid_in && w_post), "sandwich rows: residual output / post-norm weight");
+  MI_CHECK(!src.slabs.slab || (src.slabs.T == T && src.slabs.N == ld && !src.slabs.bias && !src.slabs.row_scale), "sandwich rows: pending K-split sum of another shape");
+  MI_CHECK(src.slabs.slab || !src.y || src.ld >= ld, "sandwich rows: source stride");
+  MI_CHECK(!w_pre || (y && ldy >= ld && ldy % 4 == 0), "sandwich rows: output stride");
+  ConvState cs;
+  if (conv) {
+    int rc = check_conv(*conv);
+    if (rc != MI_OK) return rc;
+    cs = *conv;
+  }
+  const size_t lds = (size_t)(ld + std::max(groups, 16) + groups) * sizeof(float);
+  const int threads = T <= 32 ? std::min(1024, ceil_div(ld / 4, 64) * 64) : 256;
+  const void* kern = f32 ? reinterpret_cast<const void*>(sandwich_rows_kernel<float>) : reinterpret_cast<const void*>(sandwich_rows_kernel<uint16_t>);
+  MI_CHECK(lds <= 160 * 1024, "sandwich rows: row too long");
+  if (lds > 64 * 1024) { int rc = ensure_dynamic_lds(kern, 160 * 1024); if (rc != MI_OK) return rc; }
+  if (f32) hipLaunchKernelGGL((sandwich_rows_kernel<float>), dim3(T), dim3(threads), lds, s, resid_in, resid_out, src, w_post, w_pre, D, ld, groups, eps, cs, (float*)y, ldy);
+  else hipLaunchKernelGGL((sandwich_rows_kernel<uint16_t>), dim3(T), dim3(threads), lds, s, resid_in, resid_out, src, w_post, w_pre, D, ld, groups, eps, cs, (uint16_t*)y, ldy);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_conv_rows(const void* h, const ConvState& conv, const AttnSeg* sd, const AttnSeg* sh, int nseg, int D, int ld, void* y, int ldy,
+                     bool f32, hipStream_t s) {
+  int rc = check_conv(conv);
+  if (rc != MI_OK) return rc;
+  MI_CHECK(nseg >= 1 && ld % 4 == 0 && ld >= D && ldy >= ld && ldy % 4 == 0 && h != y, "convolution: strides");
+  int tiles = 0;
+  for (int i = 0; i < nseg; ++i) tiles += ceil_div(sh[i].n, kConvRows);
+  const dim3 grid(tiles, ceil_div(ld, 1024));
+  if (f32) hipLaunchKernelGGL((conv_rows_kernel<float>), grid, dim3(256), 0, s, (const float*)h, conv, sd, nseg, ld, (float*)y, ldy);
+  else hipLaunchKernelGGL((conv_rows_kernel<uint16_t>), grid, dim3(256), 0, s, (const uint16_t*)h, conv, sd, nseg, ld, (uint16_t*)y, ldy);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
 int launch_pair_rows(const float* x, const float* x0, int T, int D, int ld, int half, void* y, bool f32, hipStream_t s) {
   MI_CHECK(ld % 4 == 0 && half % 4 == 0 && half >= ld && ld >= D, "pair rows: strides");
   if (f32) hipLaunchKernelGGL((pair_rows_kernel<float>), dim3(T), dim3(256), 0, s, x, x0, ld / 4, ld, half, (float*)y);
@@ -284,20 +513,40 @@ int launch_linear_f32(const float* w, int N, int K, const float* x, int ldx, int
   if (epi == EPI_F32) hipLaunchKernelGGL((linear_f32_kernel<EPI_F32>), grid, dim3(256), 0, s, w, N, K, x, ldx, T, e);
   else if (epi == EPI_RESID) hipLaunchKernelGGL((linear_f32_kernel<EPI_RESID>), grid, dim3(256), 0, s, w, N, K, x, ldx, T, e);
   else if (epi == EPI_RELU2) hipLaunchKernelGGL((linear_f32_kernel<EPI_RELU2>), grid, dim3(256), 0, s, w, N, K, x, ldx, T, e);
+  else if (epi == EPI_GLU_CLIP) hipLaunchKernelGGL((linear_f32_kernel<EPI_GLU_CLIP>), grid, dim3(256), 0, s, w, N, K, x, ldx, T, e);
+  else if (epi == EPI_SOFTCAP) hipLaunchKernelGGL((linear_f32_kernel<EPI_SOFTCAP>), grid, dim3(256), 0, s, w, N, K, x, ldx, T, e);
   else { set_error("linear_f32: epilogue"); return MI_EINVAL; }
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
 
-int launch_place(const float* src, int ld, int src_col0, int rows, int cols, void* dst, int K, bool f32, int row0, int col0, hipStream_t s) {
-  MI_CHECK(col0 % 8 == 0 && K % 64 == 0 && col0 + cols <= K && src_col0 + cols <= ld, "place: columns");
+int launch_place(const float* src, int ld, int src_col0, int rows, int cols, void* dst, int K, bool f32, int row0, int col0, hipStream_t s,
+                 int row_step) {
+  MI_CHECK(col0 % 8 == 0 && K % 32 == 0 && col0 + cols <= K && src_col0 + cols <= ld, "place: columns");
   if (f32) {
     const size_t n = (size_t)rows * cols;
-    hipLaunchKernelGGL(place_f32_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, src, ld, src_col0, rows, cols, (float*)dst, K, row0, col0);
+    hipLaunchKernelGGL(place_f32_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, src, ld, src_col0, rows, cols, (float*)dst, K, row0, col0, row_step);
   } else {
     const size_t n = (size_t)rows * ((cols + 7) / 8);
-    hipLaunchKernelGGL(place_tiled_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, src, ld, src_col0, rows, cols, (uint16_t*)dst, K / 32, row0, col0);
+    hipLaunchKernelGGL(place_tiled_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, src, ld, src_col0, rows, cols, (uint16_t*)dst, K / 32, row0, col0, row_step);
   }
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_place_rows(const float* src, int rows, int cols, void* dst, int K, bool f32, hipStream_t s) {
+  MI_CHECK(rows > 0 && cols > 0 && cols <= K, "place rows: columns");
+  const dim3 grid((unsigned)(((size_t)rows * cols + 255) / 256));
+  if (f32) hipLaunchKernelGGL(place_f32_kernel, grid, dim3(256), 0, s, src, cols, 0, rows, cols, (float*)dst, K, 0, 0, 1);
+  else hipLaunchKernelGGL(place_rows_bf16_kernel, grid, dim3(256), 0, s, src, rows, cols, (uint16_t*)dst, K);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_transpose(const float* src, int rows, int cols, float* dst, int ld_dst, hipStream_t s) {
+  MI_CHECK(ld_dst >= rows && rows > 0 && cols > 0, "transpose: strides");
+  const size_t n = (size_t)rows * cols;
+  hipLaunchKernelGGL(transpose_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s, src, rows, cols, dst, ld_dst);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }

@@ -17,7 +17,6 @@ struct AttnSpec {
   int unit_norm = 0;               // q and k heads have unit root mean square: |q.k| <= dk
   int sink = 0;                    // 1: one more score of 0 in the denominator, without a value
 };
-struct AttnSeg { int row0, n, pos0, seq; };   // rows row0 .. + n of the batch = positions pos0 .. of the sequence in block-table row seq
 
 // Plain form (one wave per row and head, any sizes, bf16 or fp32 pool): the 32-bit mode, and sizes the MFMA kernels are not built for.
 // segs [nseg] on the device; null: row r is block-table row r (token generation).

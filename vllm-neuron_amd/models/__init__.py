@@ -11,6 +11,7 @@ import json
 import os
 from types import SimpleNamespace
 
+from .rapodra import RapodraConfig
 from .vimesun import VimesunConfig
 
 # served through multimodal model classes by the reference: out of this backend's scope
@@ -18,7 +19,7 @@ MULTI_MODAL_MODELS = [f"{family}ForConditionalGeneration" for family in ("Mllama
 
 LLAMA_FAMILY = ("LlamaForCausalLM", "Qwen2ForCausalLM", "MistralForCausalLM")
 # architecture name -> reader of its config.json dictionary
-STACK_DESIGNS = {VimesunConfig.architecture: VimesunConfig.from_dict}
+STACK_DESIGNS = {design.architecture: design.from_dict for design in (VimesunConfig, RapodraConfig)}
 SUPPORTED_ARCHITECTURES = LLAMA_FAMILY + tuple(STACK_DESIGNS)
 
 

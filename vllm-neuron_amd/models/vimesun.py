@@ -14,6 +14,8 @@ from __future__ import annotations
 
 from dataclasses import dataclass, field
 
+from .._stack_enums import MI_FF
+
 
 def _require(cond, what):
     if not cond:
@@ -28,11 +30,11 @@ def _layer(i: int, entry: dict) -> dict:
     window = int(mix["mask"]["size"])
     _require(window >= 1, f"layer {i}: mask.size must be at least 1")
     out = dict(num_heads=heads, num_kv_heads=kv, qk_dim=int(mix["dim"]), v_dim=int(mix["vdim"]), window=window,
-               scale=float(mix["scale"]), qk_unit_norm=1, distance_bias=1, softmax_sink=1, ff_kind=0, ff_size=0)
+               scale=float(mix["scale"]), qk_unit_norm=1, distance_bias=1, softmax_sink=1, ff_kind=MI_FF[None], ff_size=0)
     mlp = entry.get("mlp")
     if mlp is not None:
         _require(mlp.get("kind") == "dense", f"layer {i}: unknown feed-forward {mlp.get('kind')!r}")
-        out.update(ff_kind=1, ff_size=int(mlp["ff"]))      # MI_FF_RELU2
+        out.update(ff_kind=MI_FF["relu2"], ff_size=int(mlp["ff"]))
     return out
 
 

@@ -37,7 +37,7 @@ class TraceReplay:
                     model: str = "", override: dict | None = None):
         from .engine import MI355XEngine
         return cls(MI355XEngine(
-            config, model, dtype=dtype, max_model_len=config.max_position_embeddings, max_num_seqs=max_live,
+            config, model, dtype=dtype, max_model_len=min(config.max_position_embeddings, max_tokens), max_num_seqs=max_live,
             block_size=block_size, num_gpu_blocks_override=-(-max_tokens // block_size), enable_prefix_caching=False,
             enable_chunked_prefill=True, max_num_batched_tokens=max_tokens,
             override_mi355x_config={"is_block_kv_layout": True, "weight_artifacts": False, "kv_overcommit": True,

@@ -51,14 +51,26 @@ __global__ __launch_bounds__(256) void latent_scatter_kernel(const float* __rest
   }
 }
 
+struct RowAt { int row, seq; };
+__device__ __forceinline__ RowAt latent_row(const LatentRows& r, int z) {
+  if (!r.segs) return RowAt{z, z};
+  for (int i = 0; i < r.nseg; ++i) {
+    const AttnSeg sg = r.segs[i];
+    if (sg.n >= r.below_n) continue;
+    if (z < sg.n) return RowAt{sg.row0 + z, sg.seq};
+    z -= sg.n;
+  }
+  return RowAt{0, 0};    // (not reached: the grid has LatentRows::rows rows)
+}
+
 // a wave: one 16-row tile of W_h against 16 tokens
 __global__ __launch_bounds__(256) void head_linear_kernel(const uint4* __restrict__ w, int H, int NT, int KT, const uint16_t* __restrict__ x,
-                                                          int T, uint16_t* __restrict__ y, int ldy, int y_head, int n_valid) {
+                                                          LatentRows lr, uint16_t* __restrict__ y, int ldy, int y_head, int n_valid) {
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, g4 = lane >> 4, c = lane & 15;
-  const int nt = blockIdx.x * 4 + wave, h = blockIdx.y, m = blockIdx.z * 16 + c;
+  const int nt = blockIdx.x * 4 + wave, h = blockIdx.y, z = blockIdx.z * 16 + c, m = latent_row(lr, min(z, lr.rows - 1)).row;
   if (nt >= NT) return;
   const u32x4_t* W = reinterpret_cast<const u32x4_t*>(w) + ((size_t)h * NT + nt) * KT * 64 + lane;
-  const u32x4_t* X = reinterpret_cast<const u32x4_t*>(x + ((size_t)min(m, T - 1) * H + h) * (KT * 32)) + g4;
+  const u32x4_t* X = reinterpret_cast<const u32x4_t*>(x + ((size_t)m * H + h) * (KT * 32)) + g4;
   f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
   int kt = 0;
   for (; kt + 4 <= KT; kt += 4) {
@@ -70,7 +82,7 @@ __global__ __launch_bounds__(256) void head_linear_kernel(const uint4* __restric
   }
   for (; kt < KT; ++kt)
     acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, W[kt * 64]), __builtin_bit_cast(bf16x8_t, X[kt * 4]), acc, 0, 0, 0);
-  if (m >= T) return;
+  if (z >= lr.rows) return;
   const int n = nt * 16 + g4 * 4;
   uint16_t* o = y + (size_t)m * ldy + (size_t)h * y_head + n;
   if (n + 4 <= n_valid && ((y_head | ldy) & 3) == 0) {
@@ -92,6 +104,275 @@ __global__ __launch_bounds__(64) void head_linear_f32_kernel(const float* __rest
   y[(size_t)m * ldy + (size_t)h * y_head + n] = acc;
 }
 
+// =====================================================================================
+// attention over latents, MFMA form
+// =====================================================================================
+// One work-group per (context split, HG groups of 16 heads, row), four waves, 64-key tiles of latents in LDS: keys and values at
+// once.  Scores transposed (S^T = C.Q^T): wave w takes keys 16 w .. of the tile against every head; the softmax reference is
+// shared through LDS; O^T += C^T.P^T is split over the latent's columns, wave w takes a quarter, with C read transposed
+// (ds_read_b64_tr_b16) and the score registers as the B operand.  The next tile's rows are in flight in registers meanwhile.
+typedef __attribute__((ext_vector_type(4))) short s16x4_t;
+constexpr float kLog2e = 1.4426950408889634f;
+constexpr int kMaxSplits = 16;
+__device__ __forceinline__ float fexp2(float x) { return __builtin_amdgcn_exp2f(x); }
+__device__ __forceinline__ float sexp2(float x, float m) { return (x == -INFINITY) ? 0.f : fexp2(x - m); }
+
+constexpr int kCPitch = 16;
+template <int RP, int HG>
+constexpr size_t latent_lds() { return (size_t)64 * (RP + kCPitch) * 2 + (size_t)HG * RP * 32 + (size_t)HG * 4 * 64 * 8 + (size_t)HG * 4 * 16 * 4; }
+
+template <int RP, int HG, bool FINAL>
+__global__ __launch_bounds__(256) void latent_rows_kernel(LatentGeom g, float sc2, int window, const uint16_t* __restrict__ qa,
+                                                          const uint16_t* __restrict__ pool, int bs, const int32_t* __restrict__ bt, int MB,
+                                                          const int32_t* __restrict__ pos, LatentRows lr, int NS, float* __restrict__ o_part,
+                                                          float* __restrict__ ml_part, uint16_t* __restrict__ lat) {
+  constexpr int CP = RP + kCPitch, KS = RP / 32, DN = RP / 64, CCH = RP / 8, NL = 64 * CCH / 256;
+  extern __shared__ __attribute__((aligned(16))) unsigned char dsm[];
+  uint16_t* Cs = reinterpret_cast<uint16_t*>(dsm);                        // [64][CP]
+  u32x4_t* Qs = reinterpret_cast<u32x4_t*>(Cs + 64 * CP);                 // [HG][KS][64 lanes]
+  uint2* Ps = reinterpret_cast<uint2*>(Qs + HG * KS * 64);                // [HG][4 waves][64 lanes]
+  float* Ms = reinterpret_cast<float*>(Ps + HG * 4 * 64);                 // [HG][4 waves][16]
+  const int split = blockIdx.x, h0 = blockIdx.y * 16 * HG, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g4 = lane >> 4, c = lane & 15;
+  const RowAt at = latent_row(lr, blockIdx.z);
+  const int ctx = pos[at.row] + 1, lo = window > 0 ? max(0, ctx - window) : 0;
+  const int32_t* btr = bt + (size_t)at.seq * MB;
+  const int t_lo = lo / 64, t_hi = ceil_div(ctx, 64), per = ceil_div(t_hi - t_lo, NS);
+  const int t0 = t_lo + split * per, t1 = min(t0 + per, t_hi);
+  const int last_ch = g.rp / 8 - 1;
+
+  u32x4_t cr[NL];
+  int ids[4];
+  auto fetch_ids = [&](int tt) {     // the block of every 16-token group (block_size is a multiple of 16); past the keys: the null block
+#pragma unroll
+    for (int u = 0; u < 4; ++u) ids[u] = tt < t1 && tt * 64 + 16 * u < ctx ? btr[(tt * 64 + 16 * u) / bs] : 0;
+  };
+  auto issue = [&](int tt) {
+    size_t base[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) base[u] = tt * 64 + 16 * u < ctx ? (size_t)ids[u] * bs + (tt * 64 + 16 * u) % bs : 0;
+#pragma unroll
+    for (int i = 0; i < NL; ++i) {
+      const int idx = tid + 256 * i, row = idx / CCH, ch = min(idx % CCH, last_ch), u = row >> 4;
+      const size_t b = u < 2 ? (u == 0 ? base[0] : base[1]) : (u == 2 ? base[2] : base[3]);
+      cr[i] = *reinterpret_cast<const u32x4_t*>(pool + (b + (row & 15)) * g.rp + ch * 8);
+    }
+  };
+  if (t0 < t1) {
+    fetch_ids(t0);
+    issue(t0);
+    fetch_ids(t0 + 1);
+  }
+  for (int i = tid; i < HG * KS * 64; i += 256) {
+    const int l = i & 63, ks = (i >> 6) % KS, hg = (i >> 6) / KS, h = h0 + hg * 16 + (l & 15), d = ks * 32 + (l >> 4) * 8;
+    Qs[i] = h < g.H && d < g.rp ? *reinterpret_cast<const u32x4_t*>(qa + ((size_t)at.row * g.H + h) * g.rp + d) : u32x4_t{0, 0, 0, 0};
+  }
+  f32x4_t acc[HG][DN];
+  float mrow[HG], lrow[HG];
+#pragma unroll
+  for (int hg = 0; hg < HG; ++hg) {
+    mrow[hg] = -INFINITY;
+    lrow[hg] = 0.f;
+#pragma unroll
+    for (int dn = 0; dn < DN; ++dn) acc[hg][dn] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  }
+  const int tr_row = (lane & 15) >> 2, tr_col = (lane & 3) * 4, d_w = wave * (RP / 4);
+
+  for (int tt = t0; tt < t1; ++tt) {
+    __syncthreads();                       // the previous tile is used up
+#pragma unroll
+    for (int i = 0; i < NL; ++i) {
+      const int idx = tid + 256 * i;
+      *reinterpret_cast<u32x4_t*>(&Cs[(idx / CCH) * CP + (idx % CCH) * 8]) = cr[i];
+    }
+    __syncthreads();
+    if (tt + 1 < t1) {
+      issue(tt + 1);
+      fetch_ids(tt + 2);
+    }
+    f32x4_t st[HG];
+#pragma unroll
+    for (int hg = 0; hg < HG; ++hg) st[hg] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) {
+      const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(&Cs[(16 * wave + c) * CP + ks * 32 + g4 * 8]);
+#pragma unroll
+      for (int hg = 0; hg < HG; ++hg)
+        st[hg] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, __builtin_bit_cast(bf16x8_t, Qs[(hg * KS + ks) * 64 + lane]), st[hg], 0, 0, 0);
+    }
+    const int j0 = tt * 64 + 16 * wave + 4 * g4;
+#pragma unroll
+    for (int hg = 0; hg < HG; ++hg) {
+      float mx = -INFINITY;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        st[hg][i] = j0 + i >= lo && j0 + i < ctx ? st[hg][i] * sc2 : -INFINITY;
+        mx = fmaxf(mx, st[hg][i]);
+      }
+      mx = fmaxf(mx, __shfl_xor(mx, 16));
+      mx = fmaxf(mx, __shfl_xor(mx, 32));
+      if (g4 == 0) Ms[(hg * 4 + wave) * 16 + c] = mx;
+    }
+    __syncthreads();
+    float alpha[HG];
+#pragma unroll
+    for (int hg = 0; hg < HG; ++hg) {
+      const float* M = Ms + hg * 64 + c;
+      const float mn = fmaxf(mrow[hg], fmaxf(fmaxf(M[0], M[16]), fmaxf(M[32], M[48])));
+      alpha[hg] = sexp2(mrow[hg], mn);
+      mrow[hg] = mn;                       // (finite: a tile of the split's range has a key in sight)
+      float e[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) e[i] = sexp2(st[hg][i], mn);
+      lrow[hg] = lrow[hg] * alpha[hg] + ((e[0] + e[1]) + (e[2] + e[3]));
+      Ps[(hg * 4 + wave) * 64 + lane] = make_uint2(pack_bf16x2(e[0], e[1]), pack_bf16x2(e[2], e[3]));
+    }
+    __syncthreads();
+#pragma unroll
+    for (int hg = 0; hg < HG; ++hg)
+#pragma unroll
+      for (int dn = 0; dn < DN; ++dn) { acc[hg][dn][0] *= alpha[hg]; acc[hg][dn][1] *= alpha[hg]; acc[hg][dn][2] *= alpha[hg]; acc[hg][dn][3] *= alpha[hg]; }
+    // the k-slot (g4, j) of a 32-key half is key (j < 4 ? 4 g4 + j : 16 + 4 g4 + j - 4)
+#pragma unroll
+    for (int hf = 0; hf < 2; ++hf) {
+      bf16x8_t pf[HG];
+#pragma unroll
+      for (int hg = 0; hg < HG; ++hg) {
+        const uint2 a = Ps[(hg * 4 + 2 * hf) * 64 + lane], b = Ps[(hg * 4 + 2 * hf + 1) * 64 + lane];
+        pf[hg] = __builtin_bit_cast(bf16x8_t, u32x4_t{a.x, a.y, b.x, b.y});
+      }
+#pragma unroll
+      for (int dn = 0; dn < DN; ++dn) {
+        const uint16_t* r0 = &Cs[(32 * hf + 4 * g4 + tr_row) * CP + d_w + 16 * dn + tr_col];
+        const s16x4_t l4 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4_t __attribute__((address_space(3)))*)r0);
+        const s16x4_t h4 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4_t __attribute__((address_space(3)))*)(r0 + 16 * CP));
+        const bf16x8_t av = {l4[0], l4[1], l4[2], l4[3], h4[0], h4[1], h4[2], h4[3]};
+#pragma unroll
+        for (int hg = 0; hg < HG; ++hg) acc[hg][dn] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(av, pf[hg], acc[hg][dn], 0, 0, 0);
+      }
+    }
+  }
+
+  // denominators: over the lanes of a head, then over the waves, in wave order
+  __syncthreads();
+#pragma unroll
+  for (int hg = 0; hg < HG; ++hg) {
+    lrow[hg] += __shfl_xor(lrow[hg], 16);
+    lrow[hg] += __shfl_xor(lrow[hg], 32);
+    if (g4 == 0) Ms[(hg * 4 + wave) * 16 + c] = lrow[hg];
+  }
+  __syncthreads();
+#pragma unroll
+  for (int hg = 0; hg < HG; ++hg) {
+    const int h = h0 + hg * 16 + c;
+    if (h >= g.H) continue;
+    const float* M = Ms + hg * 64 + c;
+    const float L = (M[0] + M[16]) + (M[32] + M[48]);
+    const size_t hr = (size_t)at.row * g.H + h;
+    const float inv = FINAL ? (L > 0.f ? 1.f / L : 0.f) : 1.f;
+#pragma unroll
+    for (int dn = 0; dn < DN; ++dn) {
+      const int d = d_w + 16 * dn + 4 * g4;
+      if (d >= g.rp) continue;
+      const f32x4_t a = acc[hg][dn];
+      if constexpr (FINAL) put4(lat + hr * g.rp + d, make_float4(a[0] * inv, a[1] * inv, a[2] * inv, a[3] * inv));
+      else put4(o_part + (((size_t)blockIdx.z * g.H + h) * NS + split) * g.rp + d, make_float4(a[0], a[1], a[2], a[3]));
+    }
+    if (!FINAL && wave == 0 && g4 == 0) *reinterpret_cast<float2*>(ml_part + (((size_t)blockIdx.z * g.H + h) * NS + split) * 2) = make_float2(mrow[hg], L);
+  }
+}
+
+// merge the context splits of one head over up to RW rows (split order), then W_uv
+template <int RW>
+__global__ __launch_bounds__(256) void latent_merge_kernel(LatentGeom g, const float* __restrict__ o_part, const float* __restrict__ ml_part, int NS,
+                                                           LatentRows lr, const uint4* __restrict__ w_uv, uint16_t* __restrict__ out, int ldo) {
+  extern __shared__ __attribute__((aligned(16))) unsigned char dsm[];
+  uint16_t* os = reinterpret_cast<uint16_t*>(dsm);           // [RW][rp + 8]
+  const int h = blockIdx.x, z0 = blockIdx.y * RW, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g4 = lane >> 4, c = lane & 15;
+  const int pitch = g.rp + 8, n = min(RW, lr.rows - z0);
+  for (int i = tid; i < n * (g.rp / 4); i += 256) {
+    const int r = i / (g.rp / 4), d = (i % (g.rp / 4)) * 4;
+    const size_t at = ((size_t)(z0 + r) * g.H + h) * NS;
+    float M = -INFINITY, L = 0.f;
+    for (int k = 0; k < NS; ++k) M = fmaxf(M, ml_part[(at + k) * 2]);
+    float4 o = make_float4(0.f, 0.f, 0.f, 0.f);
+    for (int k = 0; k < NS; ++k) {
+      const float2 ml = *reinterpret_cast<const float2*>(ml_part + (at + k) * 2);
+      const float f = sexp2(ml.x, M);
+      const float4 v = *reinterpret_cast<const float4*>(o_part + (at + k) * g.rp + d);
+      L += f * ml.y;
+      o.x = __builtin_fmaf(f, v.x, o.x); o.y = __builtin_fmaf(f, v.y, o.y); o.z = __builtin_fmaf(f, v.z, o.z); o.w = __builtin_fmaf(f, v.w, o.w);
+    }
+    const float inv = L > 0.f ? 1.f / L : 0.f;
+    put4(os + r * pitch + d, make_float4(o.x * inv, o.y * inv, o.z * inv, o.w * inv));
+  }
+  __syncthreads();
+  const int NT = g.dvp / 16, KT = g.rp / 32;
+  const bool live = c < n;
+  const uint16_t* X = os + min(c, n - 1) * pitch + g4 * 8;
+  const int row = latent_row(lr, z0 + min(c, n - 1)).row;
+  for (int nt = wave; nt < NT; nt += 4) {
+    const u32x4_t* W = reinterpret_cast<const u32x4_t*>(w_uv) + ((size_t)h * NT + nt) * KT * 64 + lane;
+    f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
+    int kt = 0;
+    for (; kt + 4 <= KT; kt += 4) {
+      u32x4_t a[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) a[u] = W[(kt + u) * 64];
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a[u]), *reinterpret_cast<const bf16x8_t*>(X + (kt + u) * 32), acc, 0, 0, 0);
+    }
+    for (; kt < KT; ++kt)
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, W[kt * 64]), *reinterpret_cast<const bf16x8_t*>(X + kt * 32), acc, 0, 0, 0);
+    if (!live) continue;
+    const int d = nt * 16 + g4 * 4;
+    uint16_t* o = out + (size_t)row * ldo + (size_t)h * g.dv + d;
+    if (d + 4 <= g.dv && ((g.dv | ldo) & 3) == 0) {
+      put4(o, make_float4(acc[0], acc[1], acc[2], acc[3]));
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (d + i < g.dv) o[i] = f32_to_bf16(acc[i]);
+    }
+  }
+}
+
+// four gathered rows per work-group, a wave each
+__global__ __launch_bounds__(256) void latent_gather_kernel(LatentGeom g, int window, const uint16_t* __restrict__ pool, int bs,
+                                                            const int32_t* __restrict__ bt, int MB, const AttnSeg* __restrict__ segs, int nseg, int min_n,
+                                                            int rows, uint16_t* __restrict__ x, int ldx, int32_t* __restrict__ kv_bt, int kv_mb) {
+  const int m = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (m >= rows) return;
+  int at = m, i = 0;
+  AttnSeg sg{0, 0, 0, 0};
+  for (; i < nseg; ++i) {
+    sg = segs[i];
+    if (sg.n < min_n) continue;
+    const int n = latent_kv_rows(sg, window);
+    if (at < n) break;
+    at -= n;
+  }
+  if (i == nseg) return;
+  const int p_row = latent_kv_first(sg, window) + at, p = min(p_row, sg.pos0 + sg.n - 1);     // (padding rows: copies, never in sight)
+  if (lane == 0 && m % kKvBlock == 0) kv_bt[(size_t)sg.seq * kv_mb + p_row / kKvBlock] = m / kKvBlock;
+  const uint16_t* src = pool + ((size_t)bt[(size_t)sg.seq * MB + p / bs] * bs + p % bs) * g.rp;
+  for (int d = lane * 8; d < ldx; d += 512)
+    *reinterpret_cast<u32x4_t*>(x + (size_t)m * ldx + d) = d < g.rp ? *reinterpret_cast<const u32x4_t*>(src + d) : u32x4_t{0, 0, 0, 0};
+}
+
+// rows of the batch -> rows of a list (NS = 1: lat holds the normalised output of every row; the other rows are left alone)
+template <int RP, int HG>
+int launch_rows_t(const LatentGeom& g, float scale, int window, const uint16_t* qa, const uint16_t* pool, int bs, const int32_t* bt, int MB,
+                  const int32_t* pos, const LatentRows& lr, int NS, float* op, float* ml, uint16_t* lat, hipStream_t s) {
+  constexpr size_t lds = latent_lds<RP, HG>();
+  const dim3 grid(NS, ceil_div(g.H, 16 * HG), lr.rows);
+  auto kern = NS == 1 ? latent_rows_kernel<RP, HG, true> : latent_rows_kernel<RP, HG, false>;
+  if (lds > 64 * 1024) { int rc = ensure_dynamic_lds(reinterpret_cast<const void*>(kern), (int)lds); if (rc != MI_OK) return rc; }
+  hipLaunchKernelGGL(kern, grid, dim3(256), lds, s, g, scale * kLog2e, window, qa, pool, bs, bt, MB, pos, lr, NS, op, ml, lat);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
 }  // namespace
 
 int launch_latent_scatter(const float* qd, int ldq, int T, const LatentGeom& g, const float* c_norm, float eps, const int32_t* slots,
@@ -105,10 +386,67 @@ int launch_latent_scatter(const float* qd, int ldq, int T, const LatentGeom& g, 
   return MI_OK;
 }
 
+int launch_head_linear_rows(const void* w, int H, int N, int K, const uint16_t* x, const LatentRows& rows, uint16_t* y, int ldy, int y_head,
+                            int n_valid, hipStream_t s) {
+  MI_CHECK(H >= 1 && rows.rows >= 1 && N % 16 == 0 && K % 32 == 0 && n_valid <= N && y_head >= n_valid && ldy >= (H - 1) * y_head + n_valid, "head linear: shape");
+  hipLaunchKernelGGL(head_linear_kernel, dim3(ceil_div(N / 16, 4), H, ceil_div(rows.rows, 16)), dim3(256), 0, s, (const uint4*)w, H, N / 16, K / 32, x, rows, y, ldy, y_head, n_valid);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
 int launch_head_linear(const void* w, int H, int N, int K, const void* x, int T, void* y, int ldy, int y_head, int n_valid, bool f32, hipStream_t s) {
+  LatentRows all;
+  all.rows = T;
+  if (!f32) return launch_head_linear_rows(w, H, N, K, (const uint16_t*)x, all, (uint16_t*)y, ldy, y_head, n_valid, s);
   MI_CHECK(H >= 1 && T >= 1 && N % 16 == 0 && K % 32 == 0 && n_valid <= N && y_head >= n_valid && ldy >= (H - 1) * y_head + n_valid, "head linear: shape");
-  if (f32) hipLaunchKernelGGL(head_linear_f32_kernel, dim3(T, ceil_div(n_valid, 64), H), dim3(64), 0, s, (const float*)w, H, N, K, (const float*)x, (float*)y, ldy, y_head, n_valid);
-  else hipLaunchKernelGGL(head_linear_kernel, dim3(ceil_div(N / 16, 4), H, ceil_div(T, 16)), dim3(256), 0, s, (const uint4*)w, H, N / 16, K / 32, (const uint16_t*)x, T, (uint16_t*)y, ldy, y_head, n_valid);
+  hipLaunchKernelGGL(head_linear_f32_kernel, dim3(T, ceil_div(n_valid, 64), H), dim3(64), 0, s, (const float*)w, H, N, K, (const float*)x, (float*)y, ldy, y_head, n_valid);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+bool latent_attn_supported(const LatentGeom& g) { return g.rp <= 512; }
+
+// (rows x splits <= 256, launch_latent_attn_rows)
+size_t latent_attn_scratch_bytes(const LatentGeom& g) { return (size_t)256 * g.H * (g.rp + 2) * sizeof(float); }
+
+int launch_latent_attn_rows(const LatentGeom& g, float scale, int window, const uint16_t* qa, const uint16_t* pool, int bs, const int32_t* bt,
+                            int MB, const int32_t* pos, const LatentRows& lr, int max_ctx, const void* w_uv, uint16_t* lat, uint16_t* out, int ldo,
+                            void* scratch, hipStream_t s) {
+  MI_CHECK(latent_attn_supported(g) && lr.rows >= 1 && lr.rows <= 65535 && bs > 0 && bs % 16 == 0 && max_ctx >= 1 && window >= 0 && ldo >= g.H * g.dv, "latent attention: shape");
+  const int hgs = ceil_div(g.H, 16), max_keys = window > 0 && window < max_ctx ? window : max_ctx, tiles = ceil_div(max_keys, 64) + 1;
+  // head groups that share a tile: as many as leave the chip full
+  int hg = 1;
+  while (hg < 4 && hg < hgs && lr.rows * ceil_div(hgs, 2 * hg) >= 256) hg *= 2;
+  const int groups = lr.rows * ceil_div(hgs, hg);
+  int NS = min(min(256 / groups, tiles), kMaxSplits);
+  if (NS < 1) NS = 1;
+  float* ml = reinterpret_cast<float*>(scratch);
+  float* op = ml + (size_t)256 * g.H * 2;
+  int rc = MI_OK;
+#define MI_LR(RP) \
+  rc = hg == 1 ? launch_rows_t<RP, 1>(g, scale, window, qa, pool, bs, bt, MB, pos, lr, NS, op, ml, lat, s) \
+     : hg == 2 ? launch_rows_t<RP, 2>(g, scale, window, qa, pool, bs, bt, MB, pos, lr, NS, op, ml, lat, s) \
+               : launch_rows_t<RP, 4>(g, scale, window, qa, pool, bs, bt, MB, pos, lr, NS, op, ml, lat, s)
+  if (g.rp <= 64) MI_LR(64);
+  else if (g.rp <= 128) MI_LR(128);
+  else if (g.rp <= 256) MI_LR(256);
+  else MI_LR(512);
+#undef MI_LR
+  if (rc != MI_OK) return rc;
+  if (NS == 1) return launch_head_linear_rows(w_uv, g.H, g.dvp, g.rp, lat, lr, out, ldo, g.dv, g.dv, s);
+  const int rw = lr.rows <= 4 ? 1 : lr.rows <= 16 ? 4 : 16;
+  const size_t lds = (size_t)rw * (g.rp + 8) * 2;
+  const dim3 grid(g.H, ceil_div(lr.rows, rw));
+  if (rw == 1) hipLaunchKernelGGL((latent_merge_kernel<1>), grid, dim3(256), lds, s, g, op, ml, NS, lr, (const uint4*)w_uv, out, ldo);
+  else if (rw == 4) hipLaunchKernelGGL((latent_merge_kernel<4>), grid, dim3(256), lds, s, g, op, ml, NS, lr, (const uint4*)w_uv, out, ldo);
+  else hipLaunchKernelGGL((latent_merge_kernel<16>), grid, dim3(256), lds, s, g, op, ml, NS, lr, (const uint4*)w_uv, out, ldo);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_latent_gather(const LatentGeom& g, int window, const uint16_t* pool, int bs, const int32_t* bt, int MB, const AttnSeg* segs, int nseg,
+                         int min_n, int rows, uint16_t* x, int ldx, int32_t* kv_bt, int kv_mb, hipStream_t s) {
+  MI_CHECK(rows >= 1 && rows % kKvBlock == 0 && ldx % 8 == 0 && ldx >= g.rp && bs > 0 && nseg >= 1, "latent gather: shape");
+  hipLaunchKernelGGL(latent_gather_kernel, dim3(ceil_div(rows, 4)), dim3(256), 0, s, g, window, pool, bs, bt, MB, segs, nseg, min_n, rows, x, ldx, kv_bt, kv_mb);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }

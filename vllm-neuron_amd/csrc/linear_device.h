@@ -77,6 +77,12 @@ __device__ __forceinline__ void epilogue_store(const EpiArgs& e, int m, int n0, 
   } else if constexpr (EPI == EPI_SOFTCAP) {
     *reinterpret_cast<float4*>(e.out_f32 + (size_t)m * e.ld_out + n0) =
         make_float4(e.softcap * tanhf(v[0] / e.softcap), e.softcap * tanhf(v[1] / e.softcap), e.softcap * tanhf(v[2] / e.softcap), e.softcap * tanhf(v[3] / e.softcap));
+  } else if constexpr (EPI == EPI_HEADS_KV) {
+    const bool is_k = n0 < e.q_dim;
+    const int rel = is_k ? n0 : n0 - e.q_dim, w = is_k ? e.hd : e.kv_dim, head = rel / w, d = rel - head * w;
+    const int blk = m / e.block_size, off = m - blk * e.block_size;
+    *reinterpret_cast<uint2*>((is_k ? e.kpool : e.vpool) + (((size_t)blk * e.nkv + head) * e.block_size + off) * w + d) =
+        make_uint2(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]));
   } else {  // EPI_QKV
     const int qk_end = e.q_dim + e.kv_dim;
     if (n0 < qk_end) {  // rotary: (v0,v1) and (v2,v3) are (d, d + hd/2) pairs

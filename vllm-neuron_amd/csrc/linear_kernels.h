@@ -7,7 +7,7 @@
 namespace mi {
 
 // What happens to the fp32 accumulator tile D[n][m] once the contraction is done.
-enum { EPI_F32 = 0, EPI_QKV = 1, EPI_SWIGLU = 2, EPI_RESID = 3, EPI_RELU2 = 4, EPI_GLU_CLIP = 5, EPI_SOFTCAP = 6 };
+enum { EPI_F32 = 0, EPI_QKV = 1, EPI_SWIGLU = 2, EPI_RESID = 3, EPI_RELU2 = 4, EPI_GLU_CLIP = 5, EPI_SOFTCAP = 6, EPI_HEADS_KV = 7 };
 // Where the bf16 activations come from.
 enum { PRO_BF16 = 0, PRO_NORM = 1, PRO_NORM_PARTIAL = 2 };  // callers pass PRO_BF16 / PRO_NORM; PARTIAL is picked when ProArgs::partial is set
 
@@ -38,6 +38,8 @@ struct EpiArgs {
   uint16_t* act_out;
   int ld_act;
   float glu_limit, glu_alpha;
+  // EPI_HEADS_KV (bf16 weights, GEMM): rows [0, q_dim) are nkv heads of hd keys, the rest nkv heads of kv_dim values; token m goes
+  //   to row m % block_size of block m / block_size of kpool [blocks][nkv][block_size][hd] / vpool [..][kv_dim]
   float softcap;         // EPI_SOFTCAP (bf16 weights): out[m * ld_out + n] = softcap tanh(y / softcap)
 };
 

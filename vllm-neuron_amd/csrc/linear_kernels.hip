@@ -216,7 +216,8 @@ static int launch_gemm_wd(const LinearW& w, int T, const uint16_t* x, int ldx, i
     if constexpr (WD == MI_W_BF16) {
       if (epi == EPI_RELU2) MI_G(EPI_RELU2);
       else if (epi == EPI_GLU_CLIP) MI_G(EPI_GLU_CLIP);
-      else MI_G(EPI_SOFTCAP);
+      else if (epi == EPI_SOFTCAP) MI_G(EPI_SOFTCAP);
+      else MI_G(EPI_HEADS_KV);
     } else { set_error("gemm: this epilogue is built for bf16 weights"); return MI_EINVAL; }
   } else MI_G(EPI_F32);
 #undef MI_G

@@ -32,6 +32,9 @@ struct StackLayer {
   AttnSpec latent;                               // the attention over latents: one shared key / value row for all heads
   float* c_norm = nullptr;                       // [rank]; null where the latents are another layer's
   void *w_uk = nullptr, *w_uv = nullptr;         // per head: W_uk^T [rp, dkp], W_uv [dvp, rp]
+  StackMat ukv;                                  // [W_uk ; W_uv], heads padded to dkp / dvp rows: keys and values of a prompt (bf16)
+  HeadGeom kvg;                                  // ... as the context-encoding attention sees them: every head its own
+  bool fast() const { return ukv.L.w != nullptr; }   // the MFMA forms are built for the layer's sizes
   void *router = nullptr, *expert_gu = nullptr, *expert_down = nullptr;
   float* router_b = nullptr;
   int ffk = 0;                                   // padded ff_size: contraction length of the experts' down projection
@@ -62,7 +65,11 @@ struct Stack {
   int32_t* pair_ids = nullptr;
   void *hb = nullptr, *act = nullptr, *qa = nullptr, *lat = nullptr;   // convolution inputs; gated units; queries / outputs in latent space
   int act_ld = 0, lat_cols = 0, max_top = 0;
-  size_t act_elems = 0, y_rows = 0;
+  // keys and values of a prompt, written out per head
+  void *kv_x = nullptr, *kv_k = nullptr, *kv_v = nullptr;
+  int32_t* kv_bt = nullptr;
+  int kv_rows = 0, kv_mb = 0, kv_ldx = 0;
+  size_t kv_k_cols = 0, kv_v_cols = 0;
   bool sandwich() const { return cfg.block_kind == MI_BLOCK_SANDWICH; }
   void* attn_scratch = nullptr;
   SlabSum pend;                        // K-split sum of the last output projection, left for the next norm

@@ -154,6 +154,13 @@ int sandwich_layer_create(mi_ctx* c, StackLayer& W, const std::string& p) {
   MI_TRY(alloc_mat(c, W.out, S->D, s.num_heads * s.v_dim, 1.f));
   MI_TRY(alloc0(c, &W.w_uk, (size_t)s.num_heads * W.lg.rp * W.lg.dkp * S->elem(), wb));
   MI_TRY(alloc0(c, &W.w_uv, (size_t)s.num_heads * W.lg.dvp * W.lg.rp * S->elem(), wb));
+  W.kvg = HeadGeom{s.num_heads, s.num_heads, s.qk_dim, s.v_dim, W.lg.dkp, W.lg.dvp};
+  if (!S->f32 && latent_attn_supported(W.lg) && attn_window_supported(W.kvg)) {
+    MI_TRY(alloc_mat(c, W.ukv, s.num_heads * (W.lg.dkp + W.lg.dvp), s.kv_rank, 1.f));
+    S->kv_ldx = std::max(S->kv_ldx, W.ukv.K);
+    S->kv_k_cols = std::max(S->kv_k_cols, (size_t)s.num_heads * W.lg.dkp);
+    S->kv_v_cols = std::max(S->kv_v_cols, (size_t)s.num_heads * W.lg.dvp);
+  }
   if (own) MI_TRY(alloc0(c, &W.c_norm, (size_t)s.kv_rank * 4, wb));
   MI_TRY(norm(W.n1)); MI_TRY(norm(W.n1b));
   MI_TRY(alloc0(c, &W.conv1, (size_t)taps * S->ld * 4, wb));
@@ -252,6 +259,8 @@ int sandwich_place(mi_ctx* c, StackLayer& W, const std::string& t, const float* 
       } else {
         rc = launch_place(src, cols, 0, n, cols, at(W.w_uv, (size_t)h * W.lg.dvp * W.lg.rp), W.lg.rp, S->f32, 0, 0, st);
       }
+      if (rc == MI_OK && W.fast())
+        rc = launch_place(src, cols, 0, n, cols, W.ukv.L.w, W.ukv.K, false, k ? h * W.lg.dkp : s.num_heads * W.lg.dkp + h * W.lg.dvp, 0, st);
     }
     hipStreamSynchronize(st);
     hipFree(tmp);
@@ -350,7 +359,7 @@ void stack_destroy(mi_ctx* c) {
   Stack* S = c->stack;
   for (StackLayer& W : S->layers) {
     free_mat(W.qkv); free_mat(W.up); free_mat(W.out);
-    free_mat(W.down);
+    free_mat(W.down); free_mat(W.ukv);
     free_norm(W.n1); free_norm(W.n2); free_norm(W.n1b); free_norm(W.n2b);
     void* ps[] = {W.slopes, W.conv1, W.conv2, W.c_norm, W.w_uk, W.w_uv, W.router, W.router_b, W.expert_gu, W.expert_down};
     for (void* p : ps) hipFree(p);
@@ -358,7 +367,7 @@ void stack_destroy(mi_ctx* c) {
   free_mat(S->loop_in); free_mat(S->head);
   free_norm(S->final_norm);
   void* ptrs[] = {S->embed, S->pos, S->x0, S->qkv_out, S->logits_pad, S->n1, S->n2, S->q, S->cat, S->pair, S->attn_scratch, S->residuals,
-                  S->y, S->pair_w, S->pair_ids, S->hb, S->act, S->qa, S->lat};
+                  S->y, S->pair_w, S->pair_ids, S->hb, S->act, S->qa, S->lat, S->kv_x, S->kv_k, S->kv_v, S->kv_bt};
   for (void* p : ptrs) hipFree(p);
   delete S;
   c->stack = nullptr;
@@ -505,6 +514,7 @@ void stack_artifact_tensors(mi_ctx* c, std::vector<std::pair<void*, size_t>>& ou
       put(W.conv1, cb); put(W.conv2, cb); put(W.c_norm, (size_t)p.kv_rank * 4);
       put(W.w_uk, (size_t)p.num_heads * W.lg.rp * W.lg.dkp * el);
       put(W.w_uv, (size_t)p.num_heads * W.lg.dvp * W.lg.rp * el);
+      if (W.fast()) mat(W.ukv);
       if (p.ff_kind == MI_FF_GLU) { mat(W.up); mat(W.down); }
       if (p.ff_kind == MI_FF_MOE) {
         const ExpertsLinear gu = W.expert_up(), dn = W.expert_dn();
@@ -547,9 +557,18 @@ size_t stack_kv_bytes_per_block(const mi_ctx* c) {
 
 static size_t stack_scratch(const mi_ctx* c) {
   size_t b = 16;
-  if (c->stack->sandwich()) return b;
+  if (c->stack->sandwich()) {
+    for (const StackLayer& W : c->stack->layers)
+      if (W.fast()) b = std::max(b, latent_attn_scratch_bytes(W.lg));
+    return b;
+  }
   for (const StackLayer& W : c->stack->layers) b = std::max(b, attn_window_scratch_bytes(c->cfg.max_num_seqs, W.g));
   return b;
+}
+
+// rows of the written-out keys and values: the longest sequence, and as much again for batches of several prompts
+static int kv_work_rows(const mi_ctx* c) {
+  return c->stack->kv_ldx ? 2 * pad_to(std::max(c->max_rows, c->cfg.max_model_len), kKvBlock) + 2 * kKvBlock : 0;
 }
 
 size_t stack_workspace_estimate(const mi_ctx* c) {
@@ -558,6 +577,7 @@ size_t stack_workspace_estimate(const mi_ctx* c) {
   size_t b = 3 * R * S->ld * 4 + R * S->qkv_ld * 4 + R * (4 * (size_t)S->Kd + S->q_cols + S->cat_ld) * S->elem();
   if (S->sandwich()) {
     const size_t pairs = R * std::max(1, S->max_top);
+    b += (size_t)kv_work_rows(c) * (S->kv_ldx + S->kv_k_cols + S->kv_v_cols) * 2;
     b += pairs * S->ld * 4 + pairs * 8 + R * S->Kd * S->elem() + pairs * S->act_ld * S->elem() + 2 * R * S->lat_cols * S->elem();
   }
   b += (size_t)64 << 20;
@@ -604,6 +624,14 @@ int stack_alloc(mi_ctx* c) {
     if (S->act_ld) MI_TRY(alloc0(c, &S->act, pairs * S->act_ld * S->elem(), ws));
     MI_TRY(alloc0(c, &S->qa, R * S->lat_cols * S->elem(), ws));
     MI_TRY(alloc0(c, &S->lat, R * S->lat_cols * S->elem(), ws));
+    if (S->kv_ldx) {
+      S->kv_rows = kv_work_rows(c);
+      S->kv_mb = ceil_div(k.max_model_len, kKvBlock) + 1;
+      MI_TRY(alloc0(c, &S->kv_x, (size_t)S->kv_rows * S->kv_ldx * 2, ws));
+      MI_TRY(alloc0(c, &S->kv_k, (size_t)S->kv_rows * S->kv_k_cols * 2, ws));
+      MI_TRY(alloc0(c, &S->kv_v, (size_t)S->kv_rows * S->kv_v_cols * 2, ws));
+      MI_TRY(alloc0(c, &S->kv_bt, (size_t)k.max_num_seqs * S->kv_mb * 4, ws));
+    }
     if (S->max_top) {
       MI_TRY(alloc0(c, &S->pair_w, pairs * 4, ws));
       MI_TRY(alloc0(c, &S->pair_ids, pairs * 4, ws));
@@ -650,6 +678,72 @@ int sandwich_norm(mi_ctx* c, int& cur, const Batch& b, RowSource& src, const flo
   return launch_conv_rows(S->hb, cs, reinterpret_cast<const AttnSeg*>(c->d_segs), b.segs, b.nseg, S->D, S->ld, S->n1, S->Kd, S->f32, c->stream);
 }
 
+// any sizes, bf16 or fp32
+int latent_attention_plain(mi_ctx* c, const StackLayer& W, const void* pool, const Batch& b) {
+  Stack* S = c->stack;
+  const LatentGeom& g = W.lg;
+  Scope sc(c, b.decode ? MI_K_ATTN_DECODE : MI_K_ATTN_PREFILL);
+  MI_TRY(launch_head_linear(W.w_uk, g.H, g.rp, g.dkp, S->q, b.rows, S->qa, g.H * g.rp, g.rp, g.rp, S->f32, c->stream));
+  MI_TRY(launch_attn_plain(W.latent, S->qa, pool, pool, c->cfg.block_size, c->d_bt, b.MB, c->d_pos,
+                           b.decode ? nullptr : reinterpret_cast<const AttnSeg*>(c->d_segs), b.nseg, b.rows, S->lat, g.H * g.rp, S->f32, c->stream));
+  return launch_head_linear(W.w_uv, g.H, g.dvp, g.rp, S->lat, b.rows, S->cat, S->cat_ld, g.dv, g.dv, S->f32, c->stream);
+}
+
+// Rows of short portions (and token generation) stay in the latent space; longer ones get the keys and values in their sight
+// written out per head, which costs a matrix product over those tokens and then a quarter of the attention arithmetic or less.
+constexpr int kLatentRowsBelow = 64;
+int latent_attention(mi_ctx* c, const StackLayer& W, const uint16_t* pool, const Batch& b) {
+  Stack* S = c->stack;
+  const mi_model_config& k = c->cfg;
+  const LatentGeom& g = W.lg;
+  hipStream_t s = c->stream;
+  const uint16_t* q = reinterpret_cast<const uint16_t*>(S->q);
+  uint16_t *qa = reinterpret_cast<uint16_t*>(S->qa), *out = reinterpret_cast<uint16_t*>(S->cat);
+  const AttnSeg* segs_dev = reinterpret_cast<const AttnSeg*>(c->d_segs);
+  LatentRows lr;
+  lr.rows = b.rows;
+  if (!b.decode) {
+    lr = LatentRows{segs_dev, b.nseg, kLatentRowsBelow, 0};
+    for (int i = 0; i < b.nseg; ++i) lr.rows += b.segs[i].n < kLatentRowsBelow ? b.segs[i].n : 0;
+  }
+  const int cls = b.decode ? MI_K_ATTN_DECODE : MI_K_ATTN_PREFILL;
+  if (!c->runs(cls)) return MI_OK;
+  if (lr.rows > 0) {
+    Scope sc(c, cls);
+    MI_TRY(launch_head_linear_rows(W.w_uk, g.H, g.rp, g.dkp, q, lr, qa, g.H * g.rp, g.rp, g.rp, s));
+    MI_TRY(launch_latent_attn_rows(g, W.s.scale, W.s.window, qa, pool, k.block_size, c->d_bt, b.MB, c->d_pos, lr, k.max_model_len, W.w_uv,
+                                   reinterpret_cast<uint16_t*>(S->lat), out, S->cat_ld, S->attn_scratch, s));
+  }
+  const AttnSpec a{W.kvg, W.s.scale, W.s.window, nullptr, 0, 0};
+  uint16_t *kk = reinterpret_cast<uint16_t*>(S->kv_k), *vv = reinterpret_cast<uint16_t*>(S->kv_v);
+  for (int i = 0, j; i < b.nseg; i = j) {      // as many segments at a time as the written-out keys and values have room for
+    int rows = 0;
+    for (j = i; j < b.nseg; ++j) {
+      const int n = b.segs[j].n < kLatentRowsBelow ? 0 : latent_kv_rows(b.segs[j], W.s.window);
+      if (j > i && rows + n > S->kv_rows) break;
+      rows += n;
+    }
+    if (rows == 0) continue;
+    MI_CHECK(rows <= S->kv_rows, "latent attention: a sequence longer than the workspace");
+    {
+      Scope sc(c, MI_K_OTHER);
+      MI_TRY(launch_latent_gather(g, W.s.window, pool, k.block_size, c->d_bt, b.MB, segs_dev + i, j - i, kLatentRowsBelow, rows,
+                                  reinterpret_cast<uint16_t*>(S->kv_x), W.ukv.K, S->kv_bt, S->kv_mb, s));
+    }
+    {
+      Scope sc(c, MI_K_GEMM);
+      EpiArgs e{};
+      e.scale = W.ukv.L.scale;
+      e.q_dim = g.H * g.dkp; e.hd = g.dkp; e.kv_dim = g.dvp; e.nkv = g.H; e.block_size = kKvBlock;
+      e.kpool = kk; e.vpool = vv;
+      MI_TRY(launch_gemm(W.ukv.L.view(), rows, reinterpret_cast<const uint16_t*>(S->kv_x), W.ukv.K, EPI_HEADS_KV, e, s, c->splitk_ws, c->splitk_ws_bytes));
+    }
+    Scope sc(c, cls);
+    MI_TRY(launch_attn_window_prefill(a, q, kk, vv, kKvBlock, S->kv_bt, S->kv_mb, segs_dev + i, b.segs + i, j - i, out, S->cat_ld, s, kLatentRowsBelow));
+  }
+  return MI_OK;
+}
+
 int latent_mixer(mi_ctx* c, const StackLayer& W, size_t kv_at, const Batch& b, RowSource& out) {
   Stack* S = c->stack;
   const mi_model_config& k = c->cfg;
@@ -662,17 +756,8 @@ int latent_mixer(mi_ctx* c, const StackLayer& W, size_t kv_at, const Batch& b, R
   if (runs_other(c)) {
     Scope sc(c, MI_K_OTHER);
     MI_TRY(launch_latent_scatter(S->qkv_out, S->qkv_ld, b.rows, g, W.c_norm, S->cfg.norm_eps, c->d_slots, k.block_size, S->q, pool, S->f32, s));
-    MI_TRY(launch_head_linear(W.w_uk, g.H, g.rp, g.dkp, S->q, b.rows, S->qa, g.H * g.rp, g.rp, g.rp, S->f32, s));
   }
-  {
-    Scope sc(c, b.decode ? MI_K_ATTN_DECODE : MI_K_ATTN_PREFILL);
-    MI_TRY(launch_attn_plain(W.latent, S->qa, pool, pool, k.block_size, c->d_bt, b.MB, c->d_pos, b.decode ? nullptr : reinterpret_cast<const AttnSeg*>(c->d_segs),
-                             b.nseg, b.rows, S->lat, g.H * g.rp, S->f32, s));
-  }
-  if (runs_other(c)) {
-    Scope sc(c, MI_K_OTHER);
-    MI_TRY(launch_head_linear(W.w_uv, g.H, g.dvp, g.rp, S->lat, b.rows, S->cat, S->cat_ld, g.dv, g.dv, S->f32, s));
-  }
+  MI_TRY(W.fast() ? latent_attention(c, W, reinterpret_cast<const uint16_t*>(pool), b) : latent_attention_plain(c, W, pool, b));
   EpiArgs o{};
   o.out_f32 = S->y; o.ld_out = S->ld;
   out.y = S->y; out.ld = S->ld;

@@ -30,9 +30,9 @@ size_t attn_window_scratch_bytes(int B, const HeadGeom& g);
 int launch_attn_window_decode(const AttnSpec& a, const uint16_t* q, const uint16_t* kpool, const uint16_t* vpool, int block_size,
                               const int32_t* block_table, int MB, const int32_t* ctx_lens, int B, int max_ctx, uint16_t* out, int ldo,
                               void* scratch, hipStream_t s);
-// context encoding of every segment with more than one row (host copy of segs sizes the grid); others are left alone
+// context encoding of every segment with at least min_rows (>= 2) rows (host copy of segs sizes the grid); others are left alone
 int launch_attn_window_prefill(const AttnSpec& a, const uint16_t* q, const uint16_t* kpool, const uint16_t* vpool, int block_size,
                                const int32_t* block_table, int MB, const AttnSeg* segs_dev, const AttnSeg* segs_host, int nseg,
-                               uint16_t* out, int ldo, hipStream_t s);
+                               uint16_t* out, int ldo, hipStream_t s, int min_rows = 2);
 
 }  // namespace mi

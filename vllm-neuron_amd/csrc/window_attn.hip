@@ -103,7 +103,7 @@ template <int DK, int DV, int NCG, bool FIXED>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(NCG == 1 ? 1 : 2, NCG == 1 ? 1 : 2))) void attn_window_prefill_kernel(AttnSpec a, const uint16_t* __restrict__ q, const uint16_t* __restrict__ kpool,
                                                                   const uint16_t* __restrict__ vpool, int bs, const int32_t* __restrict__ bt,
                                                                   int MB, const AttnSeg* __restrict__ segs, int nseg,
-                                                                  uint16_t* __restrict__ out, int ldo, float s_max, int fold) {
+                                                                  uint16_t* __restrict__ out, int ldo, float s_max, int fold, int min_rows) {
   constexpr int KP = DK + kPitch, VP = DV + kPitch;    // LDS row pitches (elements)
   constexpr int KS = DK / 32, DN = DV / 16, KCH = DK / 8, VCH = DV / 8;
   constexpr int NKL = 64 * KCH / 256, NVL = 64 * VCH / 256;   // 16-byte loads per thread and tile
@@ -120,7 +120,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(NCG == 1 ? 
   AttnSeg sg{0, 0, 0, 0};
   for (; si < nseg; ++si) {
     sg = segs[si];
-    const int nt_s = sg.n > 1 ? ceil_div(sg.n, qpt) : 0;
+    const int nt_s = sg.n >= min_rows ? ceil_div(sg.n, qpt) : 0;
     if (t < nt_s) break;
     t -= nt_s;
   }
@@ -567,10 +567,10 @@ float fixed_reference(const AttnSpec& a) {
 
 template <int DK, int DV, int NCG>
 int launch_prefill_t(const AttnSpec& a, const uint16_t* q, const uint16_t* kpool, const uint16_t* vpool, int bs, const int32_t* bt, int MB,
-                     const AttnSeg* sd, const AttnSeg* sh, int nseg, uint16_t* out, int ldo, hipStream_t s) {
+                     const AttnSeg* sd, const AttnSeg* sh, int nseg, uint16_t* out, int ldo, hipStream_t s, int min_rows) {
   const int qpt = 64 * NCG / (a.g.H / a.g.G);
   int tiles = 0;
-  for (int i = 0; i < nseg; ++i) tiles += sh[i].n > 1 ? ceil_div(sh[i].n, qpt) : 0;
+  for (int i = 0; i < nseg; ++i) tiles += sh[i].n >= min_rows ? ceil_div(sh[i].n, qpt) : 0;
   if (tiles == 0) return MI_OK;
   constexpr size_t lds = prefill_lds<DK, DV>();
   const float s_max = fixed_reference(a);
@@ -580,7 +580,7 @@ int launch_prefill_t(const AttnSpec& a, const uint16_t* q, const uint16_t* kpool
   auto kern = s_max > 0.f ? attn_window_prefill_kernel<DK, DV, NCG, true> : attn_window_prefill_kernel<DK, DV, NCG, false>;
   if (lds > 64 * 1024) { int rc = ensure_dynamic_lds(reinterpret_cast<const void*>(kern), (int)lds); if (rc != MI_OK) return rc; }
   // kv head fastest: consecutive work-groups (one per XCD) read different heads, a head's tiles meet in one L2
-  hipLaunchKernelGGL(kern, dim3(a.g.G, tiles), dim3(256), lds, s, a, q, kpool, vpool, bs, bt, MB, sd, nseg, out, ldo, s_max, fold);
+  hipLaunchKernelGGL(kern, dim3(a.g.G, tiles), dim3(256), lds, s, a, q, kpool, vpool, bs, bt, MB, sd, nseg, out, ldo, s_max, fold, min_rows);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
@@ -627,11 +627,11 @@ int launch_attn_window_decode(const AttnSpec& a, const uint16_t* q, const uint16
 }
 
 int launch_attn_window_prefill(const AttnSpec& a, const uint16_t* q, const uint16_t* kpool, const uint16_t* vpool, int bs, const int32_t* bt,
-                               int MB, const AttnSeg* sd, const AttnSeg* sh, int nseg, uint16_t* out, int ldo, hipStream_t s) {
+                               int MB, const AttnSeg* sd, const AttnSeg* sh, int nseg, uint16_t* out, int ldo, hipStream_t s, int min_rows) {
   int rc = check_spec(a, bs);
   if (rc != MI_OK) return rc;
-  MI_CHECK(attn_window_supported(a.g) && nseg >= 1 && ldo >= a.g.H * a.g.dv && ((a.g.dv & 3) != 0 || ldo % 4 == 0), "windowed prefill attention: shape");
-#define MI_CALL_P(DK, DV, NCG) launch_prefill_t<DK, DV, NCG>(a, q, kpool, vpool, bs, bt, MB, sd, sh, nseg, out, ldo, s)
+  MI_CHECK(attn_window_supported(a.g) && nseg >= 1 && min_rows >= 2 && ldo >= a.g.H * a.g.dv && ((a.g.dv & 3) != 0 || ldo % 4 == 0), "windowed prefill attention: shape");
+#define MI_CALL_P(DK, DV, NCG) launch_prefill_t<DK, DV, NCG>(a, q, kpool, vpool, bs, bt, MB, sd, sh, nseg, out, ldo, s, min_rows)
   MI_BY_SIZE(MI_CALL_P);
 #undef MI_CALL_P
 }

@@ -421,6 +421,30 @@ int mi_op_window_attn(const mi_layer_spec* spec, const float* slopes, const void
                       const int32_t* segs_host, int32_t nseg, int32_t T, int32_t max_ctx, void* out, int32_t ldo, int32_t f32,
                       int32_t path, void* stream);
 
+/* ---- kernels of the sandwich blocks (device pointers but segs_host; segs_host [nseg][4] as above) ----
+ * resid_out [T, ld] = resid_in + RMS-norm(w_post) of y (may be NULL: nothing added); y [T, ld] fp32, or with pair_w [T, top] the sum over
+ * j of pair_w[t, j] y[t top + j].  Then, with w_pre, out [T, ldy] = RMS-norm(w_pre) of that row and, with conv_w [taps][ld] (row taps - 1
+ * meets the token itself), h + its causal convolution.  ring [blocks][keep][ldy]: the convolution's state, position p of a block at row
+ * (p % block_size) % keep, keep >= taps - 1 or block_size.  nseg = 0: token generation, row = block-table row. */
+int mi_op_sandwich_rows(const float* resid_in, float* resid_out, const float* y, const float* pair_w, int32_t top, const float* w_post,
+                        const float* w_pre, int32_t T, int32_t D, int32_t ld, int32_t groups, float eps, const float* conv_w, int32_t taps,
+                        void* ring, int32_t keep, int32_t block_size, const int32_t* block_table, int32_t MB, const int32_t* pos,
+                        const int32_t* slots, const int32_t* segs_host, int32_t nseg, void* out, int32_t ldy, int32_t f32, void* stream);
+/* qd [T, ldq] fp32 = [q heads | W_dkv h] -> q [T, H, pad32(dk)]; with c_norm [kv_rank] the RMS-normed latent into pool
+ * [blocks][block_size][pad32(kv_rank)] at slots (-1: skip) */
+int mi_op_latent_scatter(const float* qd, int32_t ldq, int32_t T, const mi_layer_spec* spec, const float* c_norm, float eps, const int32_t* slots,
+                         int32_t block_size, void* q, void* pool, int32_t f32, void* stream);
+/* Latent attention of a ragged batch over that pool: uk [H dk, rank], uv [H dv, rank] fp32.  path: 1 plain, 2 rows in the latent space,
+ * 3 keys and values written out (segments of two rows and more).  out [T, H v_dim] (row stride ldo). */
+int mi_op_latent_attn(const mi_layer_spec* spec, const float* uk, const float* uv, const void* q, const void* pool, int32_t block_size,
+                      const int32_t* block_table, int32_t MB, const int32_t* pos, const int32_t* segs_host, int32_t nseg, int32_t T,
+                      int32_t max_ctx, void* out, int32_t ldo, int32_t f32, int32_t path, void* stream);
+/* Router and experts: x [T, ldx]; router [E, D], router_b [E], gate / up [E, ff, D], down [E, D, ff] fp32 -> ids, weights [T, top],
+ * y [T top, ldy] fp32 = every pair's expert output, unweighted.  path: 1 weight streaming (or fp32), 2 pairs grouped by expert. */
+int mi_op_experts(const void* x, int32_t ldx, int32_t T, int32_t D, int32_t experts, int32_t top, int32_t ff, const float* router, const float* router_b,
+                  const float* gate, const float* up, const float* down, int32_t* ids, float* weights, float* y, int32_t ldy, int32_t f32, int32_t path,
+                  void* stream);
+
 #ifdef __cplusplus
 }
 #endif

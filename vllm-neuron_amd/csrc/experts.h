@@ -6,8 +6,12 @@
 
 namespace mi {
 
-// x [T, ldx], w [E, K] in the compute type, b [E] fp32 -> ids [T, top], weights [T, top] (largest logit first; ties: lowest expert)
-int launch_route(const void* x, int ldx, int T, const void* w, const float* b, int E, int K, int top, int32_t* ids, float* weights, bool f32, hipStream_t s);
+// x [T, ldx], w [E, K] row-major in the compute type, b [E] fp32 -> ids [T, top], weights [T, top] (largest logit first; ties:
+// lowest expert).  With z [T, E] and tickets [T] (zero, and left zero) a row's experts are shared out to several work-groups.
+int launch_route(const void* x, int ldx, int T, const void* w, const float* b, int E, int K, int top, int32_t* ids, float* weights, bool f32, hipStream_t s,
+                 float* z = nullptr, uint32_t* tickets = nullptr);
+// the same choice over given logits z [T, ldz]
+int launch_route_pick(const float* z, int ldz, int T, int E, int top, int32_t* ids, float* weights, hipStream_t s);
 
 struct ExpertsLinear {
   const void* w = nullptr;      // [E][N, K]: 16 x 32 bf16 tiles or row-major fp32
@@ -17,5 +21,19 @@ struct ExpertsLinear {
 // type = silu(gate) up; else y [P, ldy] fp32
 int launch_experts_linear(const ExpertsLinear& w, const int32_t* ids, int P, const void* x, int ldx, int x_div, bool glu, void* y, int ldy,
                           bool f32, hipStream_t s);
+
+// Many rows (bf16): the pairs are grouped by expert once, then every linear layer is one MFMA launch over (expert, block of its
+// pairs, block of its rows).
+struct ExpertPlan {
+  int32_t* order = nullptr;     // [P] pairs, expert by expert
+  int32_t* tiles = nullptr;     // [max_tiles][3] (expert, first place in order, pairs); then the number of tiles
+  int block = 0;                // pairs per tile: 64 or 128
+  int max_tiles = 0;
+};
+size_t experts_plan_ints(int P, int E);                                             // int32s of device memory behind a plan
+ExpertPlan experts_plan(int32_t* mem, int P, int E);
+int launch_experts_sort(const ExpertPlan& plan, const int32_t* ids, int P, int E, hipStream_t s);
+// y bf16 in both cases (glu or not)
+int launch_experts_gemm(const ExpertsLinear& w, const ExpertPlan& plan, int P, const uint16_t* x, int ldx, int x_div, bool glu, uint16_t* y, int ldy, hipStream_t s);
 
 }  // namespace mi

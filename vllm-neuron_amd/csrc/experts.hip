@@ -5,7 +5,7 @@ namespace mi {
 
 namespace {
 
-constexpr int kMaxTop = 64;
+constexpr int kMaxTop = 64, kRouteExperts = 16;
 
 // ---- router: one work-group per row; a wave takes every fourth expert ----------------------------------------------------
 __device__ __forceinline__ float dot8(const uint16_t* w, const float* x) {
@@ -54,27 +54,54 @@ __device__ __forceinline__ void pick_top(float* z, int E, int top, int32_t* ids,
     const float w = expf(best - first);
     sum += w;
     if (lane == j) { mine = w; mine_id = at; }
-    if (lane == (at & 63)) z[at] = -INFINITY;
+    if (lane == (at & 63)) z[at] = -INFINITY;     // (the lane that reads it)
   }
   if (lane < top) { ids[lane] = mine_id; weights[lane] = mine / sum; }
 }
 
 template <typename T>
 __global__ __launch_bounds__(256) void route_kernel(const T* __restrict__ x, int ldx, const T* __restrict__ w, const float* __restrict__ b, int E,
-                                                    int K, int top, int32_t* __restrict__ ids, float* __restrict__ weights) {
+                                                    int K, int top, int32_t* __restrict__ ids, float* __restrict__ weights, float* __restrict__ zg,
+                                                    uint32_t* __restrict__ tickets) {
   extern __shared__ __attribute__((aligned(16))) float sm[];   // K + E floats
+  __shared__ uint32_t arrived;
   float *xs = sm, *z = sm + K;
+  const int e0 = blockIdx.y * kRouteExperts, e1 = tickets ? min(e0 + kRouteExperts, E) : E;
   const int t = blockIdx.x, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   for (int k = tid * 8; k < K; k += 2048) load8f(x + (size_t)t * ldx + k, xs + k);
   __syncthreads();
-  for (int e = wave; e < E; e += 4) {
+  for (int e = e0 + wave; e < e1; e += 4) {
     float a = 0.f;
     for (int k = lane * 8; k < K; k += 512) a += dot8(w + (size_t)e * K + k, xs + k);
     a = wave_sum(a);
-    if (lane == 0) z[e] = a + b[e];
+    if (lane == 0) {
+      if (tickets) __hip_atomic_store(zg + (size_t)t * E + e, a + b[e], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      else z[e] = a + b[e];
+    }
+  }
+  if (tickets) {       // the row's last work-group to arrive picks; it leaves the ticket at zero for the next launch
+    __threadfence();
+    __syncthreads();
+    if (tid == 0) arrived = __hip_atomic_fetch_add(tickets + t, 1u, __ATOMIC_ACQ_REL, __HIP_MEMORY_SCOPE_AGENT);
+    __syncthreads();
+    if (arrived != gridDim.y - 1) return;
+    __threadfence();
+    for (int e = tid; e < E; e += 256) z[e] = __hip_atomic_load(zg + (size_t)t * E + e, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    if (tid == 0) __hip_atomic_store(tickets + t, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
   }
   __syncthreads();
   if (wave == 0) pick_top(z, E, top, ids + (size_t)t * top, weights + (size_t)t * top);
+}
+
+// a wave per row
+__global__ __launch_bounds__(256) void route_pick_kernel(const float* __restrict__ zg, int ldz, int T, int E, int top, int32_t* __restrict__ ids,
+                                                         float* __restrict__ weights) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];   // 4 E floats
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, t = blockIdx.x * 4 + wave;
+  if (t >= T) return;
+  float* z = sm + wave * E;            // (one wave's own: LDS operations of a wave execute in order)
+  for (int e = lane; e < E; e += 64) z[e] = zg[(size_t)t * ldz + e];
+  pick_top(z, E, top, ids + (size_t)t * top, weights + (size_t)t * top);
 }
 
 // ---- experts' linear layers, few rows: weight streaming -------------------------------------------------------------------
@@ -170,6 +197,133 @@ __global__ __launch_bounds__(256) void experts_f32_kernel(const float* __restric
   if (lane == 0) y[(size_t)p * ldy + n] = a;
 }
 
+// ---- experts' linear layers, many rows -----------------------------------------------------------------------------------
+// Group the pairs by expert: count, place, list the tiles.  One work-group.
+__global__ __launch_bounds__(1024) void experts_sort_kernel(const int32_t* __restrict__ ids, int P, int E, ExpertPlan plan) {
+  extern __shared__ __attribute__((aligned(16))) int cnt[];    // [E] counts, then places
+  __shared__ int wsum[2][16];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  for (int e = tid; e < E; e += 1024) cnt[e] = 0;
+  __syncthreads();
+  for (int p = tid; p < P; p += 1024) atomicAdd(&cnt[ids[p]], 1);
+  __syncthreads();
+  // exclusive sums of counts and tile counts over the experts; thread i owns experts [i per, (i + 1) per)
+  const int per = ceil_div(E, 1024), lo = min(tid * per, E), hi = min(lo + per, E);
+  int a = 0, b = 0;
+  for (int e = lo; e < hi; ++e) { a += cnt[e]; b += ceil_div(cnt[e], plan.block); }
+  int ia = a, ib = b;
+#pragma unroll
+  for (int m = 1; m < 64; m *= 2) {
+    const int va = __shfl_up(ia, m), vb = __shfl_up(ib, m);
+    if (lane >= m) { ia += va; ib += vb; }
+  }
+  if (lane == 63) { wsum[0][wave] = ia; wsum[1][wave] = ib; }
+  __syncthreads();
+  int at = ia - a, tt = ib - b, total = 0;
+  for (int v = 0; v < 16; ++v) {
+    if (v < wave) { at += wsum[0][v]; tt += wsum[1][v]; }
+    total += wsum[1][v];
+  }
+  for (int e = lo; e < hi; ++e) {
+    const int n = cnt[e];
+    for (int k = 0; k < n; k += plan.block) {
+      int* t = plan.tiles + (size_t)tt * 3;
+      t[0] = e; t[1] = at + k; t[2] = min(plan.block, n - k);
+      ++tt;
+    }
+    cnt[e] = at;
+    at += n;
+  }
+  if (tid == 0) plan.tiles[(size_t)plan.max_tiles * 3] = total;
+  __syncthreads();
+  for (int p = tid; p < P; p += 1024) plan.order[atomicAdd(&cnt[ids[p]], 1)] = p;    // (order inside an expert does not matter: rows are independent)
+}
+
+// 128 weight rows x BM pairs per work-group, four waves; pairs' rows through swizzled LDS, weights from their tiled image
+template <int BM, bool GLU>
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) void experts_gemm_kernel(
+    const uint4* __restrict__ w, int NT, int KT, ExpertPlan plan, const uint16_t* __restrict__ x, int ldx, int x_div, uint16_t* __restrict__ y, int ldy) {
+  constexpr int WM = BM / 64, WN = 4 / WM, NTW = 8 / WN, XL = BM / 32;
+  __shared__ __attribute__((aligned(16))) u32x4_t xs[BM * 8];
+  const int ntiles = ceil_div(NT, 8);
+  int mt_id, nblk;
+  if (ntiles % 8 == 0) {       // an XCD (linear id % 8) takes every eighth block of weight rows, all tiles of an expert back to back
+    const int per = ntiles / 8, seq = blockIdx.x >> 3;
+    mt_id = seq / per;
+    nblk = (seq % per) * 8 + (blockIdx.x & 7);
+  } else {
+    mt_id = blockIdx.x / ntiles;
+    nblk = blockIdx.x % ntiles;
+  }
+  if (mt_id >= plan.tiles[(size_t)plan.max_tiles * 3]) return;
+  const int e = plan.tiles[mt_id * 3], first = plan.tiles[mt_id * 3 + 1], n = plan.tiles[mt_id * 3 + 2];
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g = lane >> 4, c = lane & 15;
+  const int wn = wave / WM, wm = wave % WM, nt0 = nblk * 8 + wn * NTW;
+  const u32x4_t* W = reinterpret_cast<const u32x4_t*>(w) + (size_t)e * NT * KT * 64 + lane;
+  const int srow = tid >> 3, sch = tid & 7, nks = KT / 2;
+  const uint16_t* xp[XL];
+#pragma unroll
+  for (int i = 0; i < XL; ++i) xp[i] = x + (size_t)(plan.order[first + min(srow + 32 * i, n - 1)] / x_div) * ldx + sch * 8;
+  f32x4_t acc[NTW][4];
+#pragma unroll
+  for (int i = 0; i < NTW; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  u32x4_t xr[XL], wr[NTW][2];
+  auto load = [&](int ks) {
+#pragma unroll
+    for (int i = 0; i < XL; ++i) xr[i] = *reinterpret_cast<const u32x4_t*>(xp[i] + ks * 64);
+#pragma unroll
+    for (int i = 0; i < NTW; ++i)
+#pragma unroll
+      for (int t = 0; t < 2; ++t) wr[i][t] = W[((size_t)min(nt0 + i, NT - 1) * KT + ks * 2 + t) * 64];
+  };
+  load(0);
+  for (int ks = 0; ks < nks; ++ks) {
+#pragma unroll
+    for (int i = 0; i < XL; ++i) {
+      const int r = srow + 32 * i;
+      xs[r * 8 + (sch ^ (r & 7))] = xr[i];
+    }
+    bf16x8_t a0[NTW], a1[NTW];
+#pragma unroll
+    for (int i = 0; i < NTW; ++i) {
+      a0[i] = __builtin_bit_cast(bf16x8_t, wr[i][0]);
+      a1[i] = __builtin_bit_cast(bf16x8_t, wr[i][1]);
+    }
+    __syncthreads();
+    if (ks + 1 < nks) load(ks + 1);
+#pragma unroll
+    for (int mt = 0; mt < 4; ++mt) {
+      const int r = wm * 64 + mt * 16 + c;
+      const bf16x8_t b0 = __builtin_bit_cast(bf16x8_t, xs[r * 8 + (g ^ (r & 7))]);
+      const bf16x8_t b1 = __builtin_bit_cast(bf16x8_t, xs[r * 8 + ((4 + g) ^ (r & 7))]);
+#pragma unroll
+      for (int i = 0; i < NTW; ++i) {
+        acc[i][mt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a0[i], b0, acc[i][mt], 0, 0, 0);
+        acc[i][mt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a1[i], b1, acc[i][mt], 0, 0, 0);
+      }
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int mt = 0; mt < 4; ++mt) {
+    const int m = wm * 64 + mt * 16 + c;
+    if (m >= n) continue;
+    uint16_t* row = y + (size_t)plan.order[first + m] * ldy;
+#pragma unroll
+    for (int i = 0; i < NTW; ++i) {
+      if (nt0 + i >= NT) continue;
+      const f32x4_t v = acc[i][mt];
+      const int n0 = (nt0 + i) * 16 + g * 4;
+      if constexpr (GLU)
+        *reinterpret_cast<uint32_t*>(row + (n0 >> 1)) = pack_bf16x2(v[0] / (1.f + __expf(-v[0])) * v[1], v[2] / (1.f + __expf(-v[2])) * v[3]);
+      else
+        *reinterpret_cast<uint2*>(row + n0) = make_uint2(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]));
+    }
+  }
+}
+
 template <int KS>
 int launch_stream(const ExpertsLinear& w, const int32_t* ids, int P, const uint16_t* x, int ldx, int x_div, bool glu, void* y, int ldy, hipStream_t s) {
   const int NT = w.N / 16, KT = w.K / 32;
@@ -182,14 +336,50 @@ int launch_stream(const ExpertsLinear& w, const int32_t* ids, int P, const uint1
 
 }  // namespace
 
-int launch_route(const void* x, int ldx, int T, const void* w, const float* b, int E, int K, int top, int32_t* ids, float* weights, bool f32, hipStream_t s) {
+int launch_route(const void* x, int ldx, int T, const void* w, const float* b, int E, int K, int top, int32_t* ids, float* weights, bool f32, hipStream_t s,
+                 float* z, uint32_t* tickets) {
   MI_CHECK(T >= 1 && E >= 1 && top >= 1 && top <= E && top <= kMaxTop && K % 64 == 0 && ldx >= K && ldx % 8 == 0, "router: 1 <= top <= min(experts, 64), row stride");
   const size_t lds = (size_t)(K + E) * 4;
   const void* kern = f32 ? reinterpret_cast<const void*>(route_kernel<float>) : reinterpret_cast<const void*>(route_kernel<uint16_t>);
   MI_CHECK(lds <= 160 * 1024, "router: row and logits larger than the LDS");
   if (lds > 64 * 1024) { int rc = ensure_dynamic_lds(kern, 160 * 1024); if (rc != MI_OK) return rc; }
-  if (f32) hipLaunchKernelGGL((route_kernel<float>), dim3(T), dim3(256), lds, s, (const float*)x, ldx, (const float*)w, b, E, K, top, ids, weights);
-  else hipLaunchKernelGGL((route_kernel<uint16_t>), dim3(T), dim3(256), lds, s, (const uint16_t*)x, ldx, (const uint16_t*)w, b, E, K, top, ids, weights);
+  MI_CHECK(!tickets || z, "router: tickets without logits");
+  const dim3 grid(T, tickets ? ceil_div(E, kRouteExperts) : 1);
+  if (f32) hipLaunchKernelGGL((route_kernel<float>), grid, dim3(256), lds, s, (const float*)x, ldx, (const float*)w, b, E, K, top, ids, weights, z, tickets);
+  else hipLaunchKernelGGL((route_kernel<uint16_t>), grid, dim3(256), lds, s, (const uint16_t*)x, ldx, (const uint16_t*)w, b, E, K, top, ids, weights, z, tickets);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_route_pick(const float* z, int ldz, int T, int E, int top, int32_t* ids, float* weights, hipStream_t s) {
+  MI_CHECK(T >= 1 && E >= 1 && E <= 4096 && top >= 1 && top <= E && top <= kMaxTop && ldz >= E, "router: experts / top");
+  hipLaunchKernelGGL(route_pick_kernel, dim3(ceil_div(T, 4)), dim3(256), (size_t)16 * E, s, z, ldz, T, E, top, ids, weights);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+size_t experts_plan_ints(int P, int E) { return (size_t)P + 3 * ((size_t)P / 64 + min(P, E) + 1) + 1; }
+ExpertPlan experts_plan(int32_t* mem, int P, int E) {
+  const int block = P / E >= 96 ? 128 : 64;
+  return ExpertPlan{mem, mem + P, block, P / block + min(P, E) + 1};
+}
+int launch_experts_sort(const ExpertPlan& plan, const int32_t* ids, int P, int E, hipStream_t s) {
+  MI_CHECK(P >= 1 && E >= 1 && E <= 4096 && plan.order && plan.tiles, "experts: plan");
+  hipLaunchKernelGGL(experts_sort_kernel, dim3(1), dim3(1024), (size_t)4 * E, s, ids, P, E, plan);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+int launch_experts_gemm(const ExpertsLinear& w, const ExpertPlan& plan, int P, const uint16_t* x, int ldx, int x_div, bool glu, uint16_t* y, int ldy, hipStream_t s) {
+  MI_CHECK(w.E >= 1 && w.N % 16 == 0 && w.K % 64 == 0 && ldx >= w.K && ldx % 8 == 0 && P >= 1 && x_div >= 1, "experts: shape");
+  MI_CHECK(ldy % 4 == 0 && ldy >= (glu ? w.N / 2 : w.N), "experts: output stride");
+  const int NT = w.N / 16, KT = w.K / 32;
+  const dim3 grid((unsigned)(plan.max_tiles * ceil_div(NT, 8)));
+  const uint4* W = reinterpret_cast<const uint4*>(w.w);
+#define MI_EG(BM) \
+  if (glu) hipLaunchKernelGGL((experts_gemm_kernel<BM, true>), grid, dim3(256), 0, s, W, NT, KT, plan, x, ldx, x_div, y, ldy); \
+  else hipLaunchKernelGGL((experts_gemm_kernel<BM, false>), grid, dim3(256), 0, s, W, NT, KT, plan, x, ldx, x_div, y, ldy)
+  if (plan.block == 128) { MI_EG(128); } else { MI_EG(64); }
+#undef MI_EG
   MI_HIP(hipGetLastError());
   return MI_OK;
 }

@@ -36,7 +36,8 @@ struct StackLayer {
   HeadGeom kvg;                                  // ... as the context-encoding attention sees them: every head its own
   bool fast() const { return ukv.L.w != nullptr; }   // the MFMA forms are built for the layer's sizes
   void *router = nullptr, *expert_gu = nullptr, *expert_down = nullptr;
-  float* router_b = nullptr;
+  float* router_b = nullptr;                     // [experts padded to 16]
+  StackMat router_t;                             // the router as tiles: many rows (bf16)
   int ffk = 0;                                   // padded ff_size: contraction length of the experts' down projection
   ExpertsLinear expert_up() const { return ExpertsLinear{expert_gu, s.experts, (2 * s.ff_size + 15) / 16 * 16, up.K}; }
   ExpertsLinear expert_dn() const { return ExpertsLinear{expert_down, s.experts, out.N, ffk}; }
@@ -62,7 +63,10 @@ struct Stack {
   int qkv_ld = 0, q_cols = 0, cat_ld = 0;
   // sandwich blocks
   float *y = nullptr, *pair_w = nullptr;       // a sublayer's output rows (experts: of every pair); the pairs' weights
-  int32_t* pair_ids = nullptr;
+  int32_t *pair_ids = nullptr, *plan = nullptr;
+  uint32_t* tickets = nullptr;
+  float* route_z = nullptr;
+  int max_experts = 0;
   void *hb = nullptr, *act = nullptr, *qa = nullptr, *lat = nullptr;   // convolution inputs; gated units; queries / outputs in latent space
   int act_ld = 0, lat_cols = 0, max_top = 0;
   // keys and values of a prompt, written out per head

@@ -187,7 +187,9 @@ int sandwich_layer_create(mi_ctx* c, StackLayer& W, const std::string& p) {
     MI_TRY(alloc0(c, &W.expert_gu, (size_t)gu.E * gu.N * gu.K * S->elem(), wb));
     MI_TRY(alloc0(c, &W.expert_down, (size_t)dn.E * dn.N * dn.K * S->elem(), wb));
     MI_TRY(alloc0(c, &W.router, (size_t)s.experts * S->Kd * S->elem(), wb));
-    MI_TRY(alloc0(c, &W.router_b, (size_t)s.experts * 4, wb));
+    MI_TRY(alloc0(c, &W.router_b, (size_t)pad_to(s.experts, 16) * 4, wb));
+    if (!S->f32) MI_TRY(alloc_mat(c, W.router_t, s.experts, S->D, 1.f));
+    S->max_experts = std::max(S->max_experts, pad_to(s.experts, 16));
     want("mlp.router"); want("mlp.router.b");
     for (int e = 0; e < s.experts; ++e)
       for (const char* n : {".gate", ".up", ".down"}) want(("mlp.e" + std::to_string(e) + n).c_str());
@@ -269,6 +271,7 @@ int sandwich_place(mi_ctx* c, StackLayer& W, const std::string& t, const float* 
   if (t == "mlp.gate") return place(W.up.L.w, W.up.K, 0, 2);
   if (t == "mlp.up") return place(W.up.L.w, W.up.K, 1, 2);
   if (t == "mlp.down") return place(W.down.L.w, W.down.K);
+  if (t == "mlp.router" && !S->f32) MI_TRY(place(W.router_t.L.w, W.router_t.K));
   if (t == "mlp.router") return launch_place_rows(dev, rows, cols, W.router, S->Kd, S->f32, st);
   if (t == "mlp.router.b") return vec(W.router_b);
   int e = -1, off = 0;
@@ -359,7 +362,7 @@ void stack_destroy(mi_ctx* c) {
   Stack* S = c->stack;
   for (StackLayer& W : S->layers) {
     free_mat(W.qkv); free_mat(W.up); free_mat(W.out);
-    free_mat(W.down); free_mat(W.ukv);
+    free_mat(W.down); free_mat(W.ukv); free_mat(W.router_t);
     free_norm(W.n1); free_norm(W.n2); free_norm(W.n1b); free_norm(W.n2b);
     void* ps[] = {W.slopes, W.conv1, W.conv2, W.c_norm, W.w_uk, W.w_uv, W.router, W.router_b, W.expert_gu, W.expert_down};
     for (void* p : ps) hipFree(p);
@@ -367,7 +370,8 @@ void stack_destroy(mi_ctx* c) {
   free_mat(S->loop_in); free_mat(S->head);
   free_norm(S->final_norm);
   void* ptrs[] = {S->embed, S->pos, S->x0, S->qkv_out, S->logits_pad, S->n1, S->n2, S->q, S->cat, S->pair, S->attn_scratch, S->residuals,
-                  S->y, S->pair_w, S->pair_ids, S->hb, S->act, S->qa, S->lat, S->kv_x, S->kv_k, S->kv_v, S->kv_bt};
+                  S->y, S->pair_w, S->pair_ids, S->hb, S->act, S->qa, S->lat, S->kv_x, S->kv_k, S->kv_v, S->kv_bt, S->plan,
+                  S->tickets, S->route_z};
   for (void* p : ptrs) hipFree(p);
   delete S;
   c->stack = nullptr;
@@ -519,6 +523,7 @@ void stack_artifact_tensors(mi_ctx* c, std::vector<std::pair<void*, size_t>>& ou
       if (p.ff_kind == MI_FF_MOE) {
         const ExpertsLinear gu = W.expert_up(), dn = W.expert_dn();
         put(W.router, (size_t)p.experts * S->Kd * el); put(W.router_b, (size_t)p.experts * 4);
+        if (!S->f32) mat(W.router_t);
         put(W.expert_gu, (size_t)gu.E * gu.N * gu.K * el); put(W.expert_down, (size_t)dn.E * dn.N * dn.K * el);
       }
       continue;
@@ -578,7 +583,7 @@ size_t stack_workspace_estimate(const mi_ctx* c) {
   if (S->sandwich()) {
     const size_t pairs = R * std::max(1, S->max_top);
     b += (size_t)kv_work_rows(c) * (S->kv_ldx + S->kv_k_cols + S->kv_v_cols) * 2;
-    b += pairs * S->ld * 4 + pairs * 8 + R * S->Kd * S->elem() + pairs * S->act_ld * S->elem() + 2 * R * S->lat_cols * S->elem();
+    b += pairs * S->ld * 4 + pairs * 16 + R * (S->max_experts + 1) * 4 + R * S->Kd * S->elem() + pairs * S->act_ld * S->elem() + 2 * R * S->lat_cols * S->elem();
   }
   b += (size_t)64 << 20;
   b += 2 * (size_t)c->cfg.max_num_seqs * pad_to(c->V_l, 16) * 4;
@@ -635,6 +640,9 @@ int stack_alloc(mi_ctx* c) {
     if (S->max_top) {
       MI_TRY(alloc0(c, &S->pair_w, pairs * 4, ws));
       MI_TRY(alloc0(c, &S->pair_ids, pairs * 4, ws));
+      MI_TRY(alloc0(c, &S->route_z, R * S->max_experts * 4, ws));
+      MI_TRY(alloc0(c, &S->tickets, R * 4, ws));
+      MI_TRY(alloc0(c, &S->plan, experts_plan_ints((int)pairs, S->max_experts) * 4, ws));
     }
   } else {
     MI_TRY(alloc0(c, &S->n2, R * S->Kd * S->elem(), ws));
@@ -776,25 +784,52 @@ int gated_ff(mi_ctx* c, const StackLayer& W, int rows, RowSource& out) {
   return apply(c, W.down, rows, S->act, S->act_ld, EPI_F32, o, rows >= 384 ? &out.slabs : nullptr);
 }
 
+// few rows stream the weights of the experts they chose; many are grouped by expert
+constexpr int kExpertStreamRows = 32;
 int expert_ff(mi_ctx* c, const StackLayer& W, int rows, RowSource& out) {
   Stack* S = c->stack;
   const mi_layer_spec& p = W.s;
   const int pairs = rows * p.experts_top;
+  const bool grouped = rows > kExpertStreamRows && !S->f32;
+  hipStream_t s = c->stream;
+  const ExpertPlan plan = experts_plan(S->plan, pairs, p.experts);
+  out.ld = S->ld;
+  out.pair_w = S->pair_w; out.top = p.experts_top;
+  if (grouped) {
+    {
+      Scope sc(c, MI_K_GEMM);
+      EpiArgs e{};
+      e.scale = W.router_t.L.scale; e.bias = W.router_b;
+      e.out_f32 = S->route_z; e.ld_out = W.router_t.N;
+      MI_TRY(launch_gemm(W.router_t.L.view(), rows, reinterpret_cast<const uint16_t*>(S->n1), S->Kd, EPI_F32, e, s, c->splitk_ws, c->splitk_ws_bytes));
+    }
+    if (runs_other(c)) {
+      Scope sc(c, MI_K_OTHER);
+      MI_TRY(launch_route_pick(S->route_z, W.router_t.N, rows, p.experts, p.experts_top, S->pair_ids, S->pair_w, s));
+      MI_TRY(launch_experts_sort(plan, S->pair_ids, pairs, p.experts, s));
+    }
+    Scope sc(c, MI_K_GEMM);
+    uint16_t *act = reinterpret_cast<uint16_t*>(S->act), *y = reinterpret_cast<uint16_t*>(S->y);
+    MI_TRY(launch_experts_gemm(W.expert_up(), plan, pairs, reinterpret_cast<const uint16_t*>(S->n1), S->Kd, p.experts_top, true, act, S->act_ld, s));
+    MI_TRY(launch_experts_gemm(W.expert_dn(), plan, pairs, act, S->act_ld, 1, false, y, S->ld, s));
+    out.y16 = y;
+    return MI_OK;
+  }
   if (runs_other(c)) {
     Scope sc(c, MI_K_OTHER);
-    MI_TRY(launch_route(S->n1, S->Kd, rows, W.router, W.router_b, p.experts, S->Kd, p.experts_top, S->pair_ids, S->pair_w, S->f32, c->stream));
+    MI_TRY(launch_route(S->n1, S->Kd, rows, W.router, W.router_b, p.experts, S->Kd, p.experts_top, S->pair_ids, S->pair_w, S->f32, s,
+                        S->f32 ? nullptr : S->route_z, S->f32 ? nullptr : S->tickets));
   }
-  const int cls = rows <= 32 && !S->f32 ? MI_K_GEMV : MI_K_GEMM;
+  const int cls = S->f32 ? MI_K_GEMM : MI_K_GEMV;
   if (c->runs(cls)) {
     Scope sc(c, cls);
-    MI_TRY(launch_experts_linear(W.expert_up(), S->pair_ids, pairs, S->n1, S->Kd, p.experts_top, true, S->act, S->act_ld, S->f32, c->stream));
+    MI_TRY(launch_experts_linear(W.expert_up(), S->pair_ids, pairs, S->n1, S->Kd, p.experts_top, true, S->act, S->act_ld, S->f32, s));
   }
   if (c->runs(cls)) {
     Scope sc(c, cls);
-    MI_TRY(launch_experts_linear(W.expert_dn(), S->pair_ids, pairs, S->act, S->act_ld, 1, false, S->y, S->ld, S->f32, c->stream));
+    MI_TRY(launch_experts_linear(W.expert_dn(), S->pair_ids, pairs, S->act, S->act_ld, 1, false, S->y, S->ld, S->f32, s));
   }
-  out.y = S->y; out.ld = S->ld;
-  out.pair_w = S->pair_w; out.top = p.experts_top;
+  out.y = S->y;
   return MI_OK;
 }
 

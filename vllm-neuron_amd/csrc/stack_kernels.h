@@ -27,12 +27,13 @@ int launch_layernorm_rows(const float* resid_in, float* resid_out, int T, int D,
 // Norms are RMS norms over `groups` equal parts of the row, each over its own sqrt(mean square + eps).
 // A sublayer's output, in whatever form the sublayer leaves it:
 struct RowSource {
-  const float* y = nullptr;        // [T, ld] fp32
+  const float* y = nullptr;        // [T, ld] fp32 ...
+  const uint16_t* y16 = nullptr;   // ... or (experts) bf16
   int ld = 0;
   SlabSum slabs;                   // slabs.slab: the K-split sum of a projection, not summed yet
-  const float* pair_w = nullptr;   // experts: row t is sum_j pair_w[t top + j] y[t top + j]
+  const float* pair_w = nullptr;   // experts: row t is sum_j pair_w[t top + j] y(16)[t top + j]
   int top = 0;
-  bool any() const { return y || slabs.slab; }
+  __host__ __device__ bool any() const { return y || y16 || slabs.slab; }
 };
 // The convolution and its state.  The state lives in the KV blocks: every block keeps the last `keep` inputs h of its
 // positions, position p at row (p % block_size) % keep, so pages that are freed, shared or used again carry it along.

@@ -155,7 +155,7 @@ __device__ __forceinline__ float4 source_row4(const RowSource& src, int t, int d
     for (int j = 0; j < src.top; ++j) {
       const size_t r = (size_t)t * src.top + j;
       const float w = src.pair_w[r];
-      const float4 q = *reinterpret_cast<const float4*>(src.y + r * src.ld + d);
+      const float4 q = src.y16 ? get4(src.y16 + r * src.ld + d) : get4(src.y + r * src.ld + d);
       v.x = __builtin_fmaf(w, q.x, v.x); v.y = __builtin_fmaf(w, q.y, v.y);
       v.z = __builtin_fmaf(w, q.z, v.z); v.w = __builtin_fmaf(w, q.w, v.w);
     }
@@ -196,7 +196,7 @@ __global__ __launch_bounds__(1024) void sandwich_rows_kernel(const float* __rest
   const int t = blockIdx.x, tid = threadIdx.x, nthr = blockDim.x;
   const size_t o = (size_t)t * ld;
   const float inv_gs = 1.0f / (float)(D / G);
-  const bool add = src.y || src.slabs.slab;
+  const bool add = src.any();
   if (add) {
     for (int d = tid * 4; d < ld; d += nthr * 4) *reinterpret_cast<float4*>(row + d) = source_row4(src, t, d);
     group_rstd(row, D, G, eps, red, rstd);
@@ -455,7 +455,8 @@ int launch_sandwich_rows(const float* resid_in, float* resid_out, const RowSourc
   MI_CHECK(T >= 1 && ld % 4 == 0 && ld >= D && ld <= 32768 && groups >= 1 && D % groups == 0, "sandwich rows: row stride / norm groups");
   MI_CHECK(!src.any() || (resid_out && resid_out != resid_in && w_post), "sandwich rows: residual output / post-norm weight");
   MI_CHECK(!src.slabs.slab || (src.slabs.T == T && src.slabs.N == ld && !src.slabs.bias && !src.slabs.row_scale), "sandwich rows: pending K-split sum of another shape");
-  MI_CHECK(src.slabs.slab || !src.y || src.ld >= ld, "sandwich rows: source stride");
+  MI_CHECK(src.slabs.slab || !src.any() || src.ld >= ld, "sandwich rows: source stride");
+  MI_CHECK(!src.y16 || src.pair_w, "sandwich rows: bf16 sources are built for experts");
   MI_CHECK(!w_pre || (y && ldy >= ld && ldy % 4 == 0), "sandwich rows: output stride");
   ConvState cs;
   if (conv) {

@@ -308,6 +308,7 @@ class MI355XCausalLM(MI355XModelBase):
             if spec_len < 1 or speculative_config is None or chunked or not cfg["is_block_kv_layout"]:
                 raise NotImplementedError("fused speculation needs num_speculative_tokens >= 1, a draft model, the block "
                                           "KV layout (prefix caching on) and no chunked prefill")
+            check_speculation(stack_of(hf), stack_of(speculative_config.draft_model_config.hf_config))
         self.model = NativeModel(
             num_blocks=int(num_blocks), block_size=int(block_size),
             # the target scores every sequence's speculation window in one token-generation pass
@@ -494,6 +495,13 @@ class MI355XCausalLM(MI355XModelBase):
                     t = sf.get_tensor(name)
                     if t.dim() in (1, 2):
                         self.model.load_weight(name, t)
+
+
+def check_speculation(*stacks) -> None:
+    """Fused speculation runs several rows of one sequence in a token-generation pass; a convolution's state follows one."""
+    for stack in stacks:
+        if stack is not None and stack.get("conv_taps", 0) > 1:
+            raise NotImplementedError("fused speculation is not built for models with convolution state")
 
 
 def _model_geometry(hf, cfg: dict) -> dict:

@@ -70,22 +70,25 @@ __global__ __launch_bounds__(256) void route_kernel(const T* __restrict__ x, int
   const int t = blockIdx.x, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   for (int k = tid * 8; k < K; k += 2048) load8f(x + (size_t)t * ldx + k, xs + k);
   __syncthreads();
-  for (int e = e0 + wave; e < e1; e += 4) {
-    float a = 0.f;
-    for (int k = lane * 8; k < K; k += 512) a += dot8(w + (size_t)e * K + k, xs + k);
-    a = wave_sum(a);
-    if (lane == 0) {
-      if (tickets) __hip_atomic_store(zg + (size_t)t * E + e, a + b[e], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-      else z[e] = a + b[e];
+  for (int e = e0 + wave * 4; e < e1; e += 16) {       // four experts at a time: their rows are in flight together
+    float a[4] = {0.f, 0.f, 0.f, 0.f};
+    for (int k = lane * 8; k < K; k += 512)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) a[i] += dot8(w + (size_t)min(e + i, e1 - 1) * K + k, xs + k);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float v = wave_sum(a[i]);
+      if (lane != 0 || e + i >= e1) continue;
+      if (tickets) __hip_atomic_store(zg + (size_t)t * E + e + i, v + b[e + i], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+      else z[e + i] = v + b[e + i];
     }
   }
   if (tickets) {       // the row's last work-group to arrive picks; it leaves the ticket at zero for the next launch
-    __threadfence();
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // every storing wave drains its write-through stores
     __syncthreads();
-    if (tid == 0) arrived = __hip_atomic_fetch_add(tickets + t, 1u, __ATOMIC_ACQ_REL, __HIP_MEMORY_SCOPE_AGENT);
+    if (tid == 0) arrived = __hip_atomic_fetch_add(tickets + t, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
     __syncthreads();
     if (arrived != gridDim.y - 1) return;
-    __threadfence();
     for (int e = tid; e < E; e += 256) z[e] = __hip_atomic_load(zg + (size_t)t * E + e, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
     if (tid == 0) __hip_atomic_store(tickets + t, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
   }

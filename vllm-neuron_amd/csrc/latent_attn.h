@@ -18,6 +18,10 @@ struct LatentGeom {
 // square times c_norm [rank] into the pool at slots (-1: not written)
 int launch_latent_scatter(const float* qd, int ldq, int T, const LatentGeom& g, const float* c_norm, float eps, const int32_t* slots,
                           int block_size, void* q, void* pool, bool f32, hipStream_t s);
+// token generation: qa [rows, H, rp] = W_uk^T q (bf16) from the same projection, and the latents' scatter, in one launch
+inline bool latent_token_supported(const LatentGeom& g) { return g.dk % 4 == 0; }
+int launch_latent_token(const float* qd, int ldq, int rows, const LatentGeom& g, const void* w_uk, const float* c_norm, float eps, const int32_t* slots,
+                        uint16_t* qa, uint16_t* pool, hipStream_t s);
 // The rows of a batch that a kernel takes: every row (token generation: segs null, row = block-table row), or the rows of the
 // segments with fewer than below_n rows.
 struct LatentRows {

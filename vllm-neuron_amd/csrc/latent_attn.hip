@@ -8,6 +8,25 @@ namespace {
 __device__ __forceinline__ void put4(uint16_t* p, float4 v) { *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf16x2(v.x, v.y), pack_bf16x2(v.z, v.w)); }
 __device__ __forceinline__ void put4(float* p, float4 v) { *reinterpret_cast<float4*>(p) = v; }
 
+// one latent over its root mean square times c_norm, into its pool row; 256 threads
+template <typename T>
+__device__ __forceinline__ void latent_norm_row(const float* __restrict__ src, const LatentGeom& g, const float* __restrict__ c_norm, float eps, int slot,
+                                                T* __restrict__ pool, float* red) {
+  const int tid = threadIdx.x;
+  float ss = 0.f;
+  for (int d = tid; d < g.rank; d += 256) ss = __builtin_fmaf(src[d], src[d], ss);
+  ss = wave_sum(ss);
+  if ((tid & 63) == 0) red[tid >> 6] = ss;
+  __syncthreads();
+  const float f = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)g.rank + eps);
+  if (slot < 0) return;
+  T* dst = pool + (size_t)slot * g.rp;        // (a block's rows are consecutive: slot = block * block_size + offset)
+  for (int d = tid * 4; d < g.rp; d += 1024) {
+    auto at = [&](int i) { return d + i < g.rank ? src[d + i] * f * c_norm[d + i] : 0.f; };
+    put4(dst + d, make_float4(at(0), at(1), at(2), at(3)));
+  }
+}
+
 // blockIdx.y < q groups: 8 heads of 32 lanes each; the last one: the latent, one work-group per row
 template <typename T>
 __global__ __launch_bounds__(256) void latent_scatter_kernel(const float* __restrict__ qd, int ldq, LatentGeom g, const float* __restrict__ c_norm,
@@ -35,20 +54,7 @@ __global__ __launch_bounds__(256) void latent_scatter_kernel(const float* __rest
     }
     return;
   }
-  const float* src = qd + (size_t)t * ldq + (size_t)g.H * g.dk;
-  float ss = 0.f;
-  for (int d = tid; d < g.rank; d += 256) ss = __builtin_fmaf(src[d], src[d], ss);
-  ss = wave_sum(ss);
-  if ((tid & 63) == 0) red[tid >> 6] = ss;
-  __syncthreads();
-  const float f = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)g.rank + eps);
-  const int slot = slots[t];
-  if (slot < 0) return;
-  T* dst = pool + (size_t)slot * g.rp;        // (a block's rows are consecutive: slot = block * block_size + offset)
-  for (int d = tid * 4; d < g.rp; d += 1024) {
-    auto at = [&](int i) { return d + i < g.rank ? src[d + i] * f * c_norm[d + i] : 0.f; };
-    put4(dst + d, make_float4(at(0), at(1), at(2), at(3)));
-  }
+  latent_norm_row(qd + (size_t)t * ldq + (size_t)g.H * g.dk, g, c_norm, eps, slots[t], pool, red);
 }
 
 struct RowAt { int row, seq; };
@@ -92,6 +98,40 @@ __global__ __launch_bounds__(256) void head_linear_kernel(const uint4* __restric
     for (int i = 0; i < 4; ++i)
       if (n + i < n_valid) o[i] = f32_to_bf16(acc[i]);
   }
+}
+
+// Token generation: W_uk^T q straight from the projection's fp32 rows (rounded to bf16 on the way, as latent_scatter_kernel
+// leaves q), and the latents' norm and scatter in the same launch: blockIdx.y < H a head, = H the latents of row blockIdx.x.
+__global__ __launch_bounds__(256) void latent_token_kernel(const float* __restrict__ qd, int ldq, LatentGeom g, const uint4* __restrict__ w_uk, int rows,
+                                                           const float* __restrict__ c_norm, float eps, const int32_t* __restrict__ slots,
+                                                           uint16_t* __restrict__ qa, uint16_t* __restrict__ pool) {
+  __shared__ float red[4];
+  const int h = blockIdx.y;
+  if (h == g.H) {
+    if ((int)blockIdx.x < rows) latent_norm_row(qd + (size_t)blockIdx.x * ldq + (size_t)g.H * g.dk, g, c_norm, eps, slots[blockIdx.x], pool, red);
+    return;
+  }
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, g4 = lane >> 4, c = lane & 15;
+  const int NT = g.rp / 16, KT = g.dkp / 32, ntg = ceil_div(NT, 4), tt = blockIdx.x / ntg, nt = (blockIdx.x % ntg) * 4 + wave, m = tt * 16 + c;
+  if (tt * 16 >= rows || nt >= NT) return;
+  const u32x4_t* W = reinterpret_cast<const u32x4_t*>(w_uk) + ((size_t)h * NT + nt) * KT * 64 + lane;
+  const float* X = qd + (size_t)min(m, rows - 1) * ldq + (size_t)h * g.dk + g4 * 8;
+  f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
+  for (int k0 = 0; k0 < KT; k0 += 4) {       // (past the last tile: the last one's weights against zeros)
+    u32x4_t a[4], x[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      a[u] = W[min(k0 + u, KT - 1) * 64];
+      float4 x0 = make_float4(0.f, 0.f, 0.f, 0.f), x1 = x0;
+      const int d = (k0 + u) * 32 + g4 * 8;
+      if (d < g.dk) x0 = *reinterpret_cast<const float4*>(X + (k0 + u) * 32);
+      if (d + 4 < g.dk) x1 = *reinterpret_cast<const float4*>(X + (k0 + u) * 32 + 4);
+      x[u] = u32x4_t{pack_bf16x2(x0.x, x0.y), pack_bf16x2(x0.z, x0.w), pack_bf16x2(x1.x, x1.y), pack_bf16x2(x1.z, x1.w)};
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a[u]), __builtin_bit_cast(bf16x8_t, x[u]), acc, 0, 0, 0);
+  }
+  if (m < rows) put4(qa + ((size_t)m * g.H + h) * g.rp + nt * 16 + g4 * 4, make_float4(acc[0], acc[1], acc[2], acc[3]));
 }
 
 __global__ __launch_bounds__(64) void head_linear_f32_kernel(const float* __restrict__ w, int H, int N, int K, const float* __restrict__ x,
@@ -281,45 +321,64 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(LatentGeom g, float sc
   }
 }
 
-// merge the context splits of one head over up to RW rows (split order), then W_uv
+// merge the context splits of one head over up to RW rows (split order), then W_uv.  A thread owns four columns of one row; the first
+// weight tiles are requested ahead of the merge.
 template <int RW>
-__global__ __launch_bounds__(256) void latent_merge_kernel(LatentGeom g, const float* __restrict__ o_part, const float* __restrict__ ml_part, int NS,
+__global__ __launch_bounds__(512) void latent_merge_kernel(LatentGeom g, const float* __restrict__ o_part, const float* __restrict__ ml_part, int NS,
                                                            LatentRows lr, const uint4* __restrict__ w_uv, uint16_t* __restrict__ out, int ldo) {
   extern __shared__ __attribute__((aligned(16))) unsigned char dsm[];
   uint16_t* os = reinterpret_cast<uint16_t*>(dsm);           // [RW][rp + 8]
   const int h = blockIdx.x, z0 = blockIdx.y * RW, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g4 = lane >> 4, c = lane & 15;
-  const int pitch = g.rp + 8, n = min(RW, lr.rows - z0);
-  for (int i = tid; i < n * (g.rp / 4); i += 256) {
+  const int pitch = g.rp + 8, n = min(RW, lr.rows - z0), NT = g.dvp / 16, KT = g.rp / 32;
+  constexpr int PF = 8;
+  const u32x4_t* W0 = reinterpret_cast<const u32x4_t*>(w_uv) + ((size_t)h * NT + min(wave, NT - 1)) * KT * 64 + lane;
+  u32x4_t pre[PF];
+#pragma unroll
+  for (int u = 0; u < PF; ++u) pre[u] = W0[min(u, KT - 1) * 64];
+  for (int i = tid; i < n * (g.rp / 4); i += 512) {
     const int r = i / (g.rp / 4), d = (i % (g.rp / 4)) * 4;
     const size_t at = ((size_t)(z0 + r) * g.H + h) * NS;
+    float m[kMaxSplits], l[kMaxSplits];
+    float4 v[kMaxSplits];
+#pragma unroll
+    for (int k = 0; k < kMaxSplits; ++k) {
+      const float2 ml = k < NS ? *reinterpret_cast<const float2*>(ml_part + (at + k) * 2) : make_float2(-INFINITY, 0.f);
+      m[k] = ml.x; l[k] = ml.y;
+      v[k] = k < NS ? *reinterpret_cast<const float4*>(o_part + (at + k) * g.rp + d) : make_float4(0.f, 0.f, 0.f, 0.f);
+    }
     float M = -INFINITY, L = 0.f;
-    for (int k = 0; k < NS; ++k) M = fmaxf(M, ml_part[(at + k) * 2]);
+#pragma unroll
+    for (int k = 0; k < kMaxSplits; ++k) M = fmaxf(M, m[k]);
     float4 o = make_float4(0.f, 0.f, 0.f, 0.f);
-    for (int k = 0; k < NS; ++k) {
-      const float2 ml = *reinterpret_cast<const float2*>(ml_part + (at + k) * 2);
-      const float f = sexp2(ml.x, M);
-      const float4 v = *reinterpret_cast<const float4*>(o_part + (at + k) * g.rp + d);
-      L += f * ml.y;
-      o.x = __builtin_fmaf(f, v.x, o.x); o.y = __builtin_fmaf(f, v.y, o.y); o.z = __builtin_fmaf(f, v.z, o.z); o.w = __builtin_fmaf(f, v.w, o.w);
+#pragma unroll
+    for (int k = 0; k < kMaxSplits; ++k) {
+      const float f = sexp2(m[k], M);
+      L += f * l[k];
+      o.x = __builtin_fmaf(f, v[k].x, o.x); o.y = __builtin_fmaf(f, v[k].y, o.y); o.z = __builtin_fmaf(f, v[k].z, o.z); o.w = __builtin_fmaf(f, v[k].w, o.w);
     }
     const float inv = L > 0.f ? 1.f / L : 0.f;
     put4(os + r * pitch + d, make_float4(o.x * inv, o.y * inv, o.z * inv, o.w * inv));
   }
   __syncthreads();
-  const int NT = g.dvp / 16, KT = g.rp / 32;
   const bool live = c < n;
   const uint16_t* X = os + min(c, n - 1) * pitch + g4 * 8;
   const int row = latent_row(lr, z0 + min(c, n - 1)).row;
-  for (int nt = wave; nt < NT; nt += 4) {
+  for (int nt = wave; nt < NT; nt += 8) {
     const u32x4_t* W = reinterpret_cast<const u32x4_t*>(w_uv) + ((size_t)h * NT + nt) * KT * 64 + lane;
     f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
-    int kt = 0;
-    for (; kt + 4 <= KT; kt += 4) {
-      u32x4_t a[4];
 #pragma unroll
-      for (int u = 0; u < 4; ++u) a[u] = W[(kt + u) * 64];
+    for (int u = 0; u < PF; ++u) {
+      if (u >= KT) break;
+      const u32x4_t a = nt == wave ? pre[u] : W[u * 64];
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a), *reinterpret_cast<const bf16x8_t*>(X + u * 32), acc, 0, 0, 0);
+    }
+    int kt = PF;
+    for (; kt + 8 <= KT; kt += 8) {
+      u32x4_t a[8];
 #pragma unroll
-      for (int u = 0; u < 4; ++u)
+      for (int u = 0; u < 8; ++u) a[u] = W[(kt + u) * 64];
+#pragma unroll
+      for (int u = 0; u < 8; ++u)
         acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a[u]), *reinterpret_cast<const bf16x8_t*>(X + (kt + u) * 32), acc, 0, 0, 0);
     }
     for (; kt < KT; ++kt)
@@ -386,6 +445,16 @@ int launch_latent_scatter(const float* qd, int ldq, int T, const LatentGeom& g, 
   return MI_OK;
 }
 
+int launch_latent_token(const float* qd, int ldq, int rows, const LatentGeom& g, const void* w_uk, const float* c_norm, float eps, const int32_t* slots,
+                        uint16_t* qa, uint16_t* pool, hipStream_t s) {
+  MI_CHECK(rows >= 1 && latent_token_supported(g) && ldq % 4 == 0 && ldq >= g.H * g.dk + (c_norm ? g.rank : 0), "latent token: geometry");
+  const int heads_x = ceil_div(rows, 16) * ceil_div(g.rp / 16, 4);
+  const dim3 grid(c_norm && rows > heads_x ? rows : heads_x, g.H + (c_norm ? 1 : 0));
+  hipLaunchKernelGGL(latent_token_kernel, grid, dim3(256), 0, s, qd, ldq, g, (const uint4*)w_uk, rows, c_norm, eps, slots, qa, pool);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
 int launch_head_linear_rows(const void* w, int H, int N, int K, const uint16_t* x, const LatentRows& rows, uint16_t* y, int ldy, int y_head,
                             int n_valid, hipStream_t s) {
   MI_CHECK(H >= 1 && rows.rows >= 1 && N % 16 == 0 && K % 32 == 0 && n_valid <= N && y_head >= n_valid && ldy >= (H - 1) * y_head + n_valid, "head linear: shape");
@@ -433,12 +502,15 @@ int launch_latent_attn_rows(const LatentGeom& g, float scale, int window, const 
 #undef MI_LR
   if (rc != MI_OK) return rc;
   if (NS == 1) return launch_head_linear_rows(w_uv, g.H, g.dvp, g.rp, lat, lr, out, ldo, g.dv, g.dv, s);
-  const int rw = lr.rows <= 4 ? 1 : lr.rows <= 16 ? 4 : 16;
+  const int per = g.H * lr.rows / 256, rw = per <= 1 ? 1 : per <= 2 ? 2 : per <= 4 ? 4 : 16;
   const size_t lds = (size_t)rw * (g.rp + 8) * 2;
   const dim3 grid(g.H, ceil_div(lr.rows, rw));
-  if (rw == 1) hipLaunchKernelGGL((latent_merge_kernel<1>), grid, dim3(256), lds, s, g, op, ml, NS, lr, (const uint4*)w_uv, out, ldo);
-  else if (rw == 4) hipLaunchKernelGGL((latent_merge_kernel<4>), grid, dim3(256), lds, s, g, op, ml, NS, lr, (const uint4*)w_uv, out, ldo);
-  else hipLaunchKernelGGL((latent_merge_kernel<16>), grid, dim3(256), lds, s, g, op, ml, NS, lr, (const uint4*)w_uv, out, ldo);
+#define MI_LM(RW) hipLaunchKernelGGL((latent_merge_kernel<RW>), grid, dim3(512), lds, s, g, op, ml, NS, lr, (const uint4*)w_uv, out, ldo)
+  if (rw == 1) MI_LM(1);
+  else if (rw == 2) MI_LM(2);
+  else if (rw == 4) MI_LM(4);
+  else MI_LM(16);
+#undef MI_LM
   MI_HIP(hipGetLastError());
   return MI_OK;
 }

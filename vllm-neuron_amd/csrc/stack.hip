@@ -718,7 +718,8 @@ int latent_attention(mi_ctx* c, const StackLayer& W, const uint16_t* pool, const
   if (!c->runs(cls)) return MI_OK;
   if (lr.rows > 0) {
     Scope sc(c, cls);
-    MI_TRY(launch_head_linear_rows(W.w_uk, g.H, g.rp, g.dkp, q, lr, qa, g.H * g.rp, g.rp, g.rp, s));
+    if (!b.decode || !latent_token_supported(g))   // (token generation: done with the scatter)
+      MI_TRY(launch_head_linear_rows(W.w_uk, g.H, g.rp, g.dkp, q, lr, qa, g.H * g.rp, g.rp, g.rp, s));
     MI_TRY(launch_latent_attn_rows(g, W.s.scale, W.s.window, qa, pool, k.block_size, c->d_bt, b.MB, c->d_pos, lr, k.max_model_len, W.w_uv,
                                    reinterpret_cast<uint16_t*>(S->lat), out, S->cat_ld, S->attn_scratch, s));
   }
@@ -761,7 +762,13 @@ int latent_mixer(mi_ctx* c, const StackLayer& W, size_t kv_at, const Batch& b, R
   e.out_f32 = S->qkv_out; e.ld_out = S->qkv_ld;
   MI_TRY(apply(c, W.qkv, b.rows, S->n1, S->Kd, EPI_F32, e));
   unsigned char* pool = reinterpret_cast<unsigned char*>(c->kv_pool) + kv_at * S->elem();
-  if (runs_other(c)) {
+  if (b.decode && W.fast() && latent_token_supported(g)) {
+    if (runs_other(c)) {
+      Scope sc(c, MI_K_OTHER);
+      MI_TRY(launch_latent_token(S->qkv_out, S->qkv_ld, b.rows, g, W.w_uk, W.c_norm, S->cfg.norm_eps, c->d_slots, reinterpret_cast<uint16_t*>(S->qa),
+                                 reinterpret_cast<uint16_t*>(pool), s));
+    }
+  } else if (runs_other(c)) {
     Scope sc(c, MI_K_OTHER);
     MI_TRY(launch_latent_scatter(S->qkv_out, S->qkv_ld, b.rows, g, W.c_norm, S->cfg.norm_eps, c->d_slots, k.block_size, S->q, pool, S->f32, s));
   }

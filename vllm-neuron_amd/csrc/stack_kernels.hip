@@ -227,44 +227,150 @@ __global__ __launch_bounds__(1024) void sandwich_rows_kernel(const float* __rest
   }
 }
 
-// One work-group: up to kConvRows rows of one segment x 1024 channels.
+template <typename T> struct Raw4;
+template <> struct Raw4<uint16_t> { typedef uint2 type; };
+template <> struct Raw4<float> { typedef float4 type; };
+__device__ __forceinline__ float4 widen(uint2 v) { return make_float4(bf16lo_to_f32(v.x), bf16hi_to_f32(v.x), bf16lo_to_f32(v.y), bf16hi_to_f32(v.y)); }
+__device__ __forceinline__ float4 widen(float4 v) { return v; }
+
+// Token generation, rows of up to 4096: one float4 per thread and everything the row needs requested at once -- the sublayer's output,
+// the stream, both weights, the convolution's taps and state -- so that the two norms wait for memory once.  D / G a multiple of
+// 256: a wave's elements lie in one part, and a part's sum is a few waves' (in wave order).
+template <typename T, int TAPS>
+__global__ __launch_bounds__(1024) void sandwich_token_kernel(const float* __restrict__ resid_in, float* __restrict__ resid_out, RowSource src,
+                                                             const float* __restrict__ w_post, const float* __restrict__ w_pre, int D, int ld,
+                                                             int gs, float eps, ConvState cs, T* __restrict__ y, int ldy) {
+  typedef typename Raw4<T>::type raw_t;
+  __shared__ float red[2][16];
+  const int t = blockIdx.x, tid = threadIdx.x, wave = tid >> 6, d = tid * 4;
+  const bool in = d < ld, add = src.any();
+  const int dd = in ? d : 0;
+  const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+  float4 x = *reinterpret_cast<const float4*>(resid_in + (size_t)t * ld + dd);
+  float4 v = add ? source_row4(src, t, dd) : zero;
+  const float4 wp = add ? *reinterpret_cast<const float4*>(w_post + dd) : zero, wn = *reinterpret_cast<const float4*>(w_pre + dd);
+  float4 w[TAPS > 0 ? TAPS : 1];
+  raw_t past[TAPS > 1 ? TAPS - 1 : 1];
+  int slot = -1;
+  if constexpr (TAPS > 0) {
+    const int p = cs.pos[t];
+    slot = cs.slots[t];
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) w[j] = *reinterpret_cast<const float4*>(cs.w + (size_t)j * ld + dd);
+#pragma unroll
+    for (int j = 0; j + 1 < TAPS; ++j) {
+      const int q = p - (TAPS - 1 - j);
+      if (q >= 0) past[j] = *reinterpret_cast<const raw_t*>(ring_at<T>(cs, cs.bt[(size_t)t * cs.MB + q / cs.block_size], q % cs.block_size, ldy) + dd);
+      else past[j] = raw_t{};
+    }
+  }
+  const int wpg = gs >> 8, g0 = wave / wpg * wpg;              // waves of this element's part
+  auto rstd = [&](float4 a, float* r) {
+    const float s = wave_sum((a.x * a.x + a.y * a.y) + (a.z * a.z + a.w * a.w));   // (rows are whole parts: columns beyond D belong to no wave of a part)
+    if ((tid & 63) == 0) r[wave] = s;
+    __syncthreads();
+    float sum = 0.f;
+    for (int k = 0; k < wpg; ++k) sum += r[g0 + k];
+    return 1.0f / sqrtf(sum / (float)gs + eps);
+  };
+  if (add) {
+    const float r = rstd(in ? v : zero, red[0]);
+    x.x = __builtin_fmaf(v.x * r, wp.x, x.x); x.y = __builtin_fmaf(v.y * r, wp.y, x.y);
+    x.z = __builtin_fmaf(v.z * r, wp.z, x.z); x.w = __builtin_fmaf(v.w * r, wp.w, x.w);
+    if (in) *reinterpret_cast<float4*>(resid_out + (size_t)t * ld + d) = x;
+  }
+  const float r = rstd(in ? x : zero, red[1]);
+  if (!in) return;
+  float4 h = make_float4(x.x * r * wn.x, x.y * r * wn.y, x.z * r * wn.z, x.w * r * wn.w);
+  if constexpr (TAPS > 0) {
+    h = make_float4(round_to(h.x, y), round_to(h.y, y), round_to(h.z, y), round_to(h.w, y));
+    float4 a = zero;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) {
+      const float4 u = j + 1 < TAPS ? widen(past[j < TAPS - 1 ? j : 0]) : h;
+      a.x = __builtin_fmaf(w[j].x, u.x, a.x); a.y = __builtin_fmaf(w[j].y, u.y, a.y);
+      a.z = __builtin_fmaf(w[j].z, u.z, a.z); a.w = __builtin_fmaf(w[j].w, u.w, a.w);
+    }
+    if (TAPS > 1 && slot >= 0) put4(ring_at<T>(cs, slot / cs.block_size, slot % cs.block_size, ldy) + d, h.x, h.y, h.z, h.w);
+    h = make_float4(h.x + a.x, h.y + a.y, h.z + a.z, h.w + a.w);
+  }
+  put4(y + (size_t)t * ldy + d, h.x, h.y, h.z, h.w);
+}
+
+// One work-group: up to ROWS rows of one segment x 1024 channels, four channels per thread; a thread's rows and the inputs ahead of
+// them are all requested at once.  TAPS = 0: any number of taps, inputs read where they are needed.
 // The rows at a segment's start read the state of the positions ahead of it, and rows further on renew it.  Both may meet in one
 // place only in the block that holds the position ahead of the segment; that block's renewal is left to the work-group of the
-// segment's first rows, whose threads have read their channels' state by then (kConvRows >= taps - 1).
+// segment's first rows, whose threads have read their channels' state by then (ROWS >= taps - 1).
 constexpr int kConvRows = 16;
-template <typename T>
+template <typename T, int TAPS, int ROWS>
 __global__ __launch_bounds__(256) void conv_rows_kernel(const T* __restrict__ hin, ConvState cs, const AttnSeg* __restrict__ segs, int nseg,
                                                         int ld, T* __restrict__ y, int ldy) {
+  typedef typename Raw4<T>::type raw_t;
   int tile = blockIdx.x, si = 0;
   AttnSeg sg{0, 0, 0, 0};
   for (; si < nseg; ++si) {
     sg = segs[si];
-    const int n = ceil_div(sg.n, kConvRows);
+    const int n = ceil_div(sg.n, ROWS);
     if (tile < n) break;
     tile -= n;
   }
   const int d = (blockIdx.y * 256 + threadIdx.x) * 4;
   if (si == nseg || d >= ld) return;
-  const int bs = cs.block_size, first = tile * kConvRows, last = min(first + kConvRows, sg.n), end = sg.pos0 + sg.n;
+  const int bs = cs.block_size, first = tile * ROWS, last = min(first + ROWS, sg.n), end = sg.pos0 + sg.n;
   const int shared_block = sg.pos0 % bs ? sg.pos0 / bs : -1;      // holds positions on both sides of the segment's start
+  const T* hs = hin + (size_t)sg.row0 * ldy + d;
   auto renew = [&](int p, float4 h) {
     const int slot = cs.slots[sg.row0 + p - sg.pos0];
     if (slot >= 0) put4(ring_at<T>(cs, slot / bs, slot % bs, ldy) + d, h.x, h.y, h.z, h.w);
   };
-  for (int i = first; i < last; ++i) {
-    const int p = sg.pos0 + i;
-    const size_t r = (size_t)(sg.row0 + i) * ldy + d;
-    const float4 h = get4(hin + r);
-    const float4 a = conv_sum(cs, ld, d, p, h, [&](int back) {
-      return back <= i ? get4(hin + r - (size_t)back * ldy) : ring_get4<T>(cs, sg.seq, p - back, ldy, d);
-    });
-    put4(y + r, a.x, a.y, a.z, a.w);
+  auto renew_own = [&](int p, float4 h) {
     const int b = p / bs;
     if (b != shared_block && p + cs.keep >= min(end, (b + 1) * bs)) renew(p, h);
+  };
+  if constexpr (TAPS > 0) {
+    raw_t in[ROWS + TAPS - 1];
+    float4 w[TAPS];
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) w[j] = *reinterpret_cast<const float4*>(cs.w + (size_t)j * ld + d);
+#pragma unroll
+    for (int k = 0; k < ROWS + TAPS - 1; ++k) {
+      const int i = first + k - (TAPS - 1);                         // row of the segment; negative: ahead of it
+      if (i >= 0) in[k] = *reinterpret_cast<const raw_t*>(hs + (size_t)min(i, sg.n - 1) * ldy);
+      else if (sg.pos0 + i >= 0) {
+        const int p = sg.pos0 + i;
+        in[k] = *reinterpret_cast<const raw_t*>(ring_at<T>(cs, cs.bt[(size_t)sg.seq * cs.MB + p / bs], p % bs, ldy) + d);
+      } else in[k] = raw_t{};                                        // (ahead of the sequence: zeros)
+    }
+#pragma unroll
+    for (int k = 0; k < ROWS; ++k) {
+      if (first + k >= last) break;
+      const float4 h = widen(in[k + TAPS - 1]);
+      float4 a = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) {
+        const float4 v = widen(in[k + j]);
+        a.x = __builtin_fmaf(w[j].x, v.x, a.x); a.y = __builtin_fmaf(w[j].y, v.y, a.y);
+        a.z = __builtin_fmaf(w[j].z, v.z, a.z); a.w = __builtin_fmaf(w[j].w, v.w, a.w);
+      }
+      put4(y + (size_t)(sg.row0 + first + k) * ldy + d, h.x + a.x, h.y + a.y, h.z + a.z, h.w + a.w);
+      if constexpr (TAPS > 1) renew_own(sg.pos0 + first + k, h);
+    }
+  } else {
+    for (int i = first; i < last; ++i) {
+      const int p = sg.pos0 + i;
+      const T* r = hs + (size_t)i * ldy;
+      const float4 h = get4(r);
+      const float4 a = conv_sum(cs, ld, d, p, h, [&](int back) {
+        return back <= i ? get4(r - (size_t)back * ldy) : ring_get4<T>(cs, sg.seq, p - back, ldy, d);
+      });
+      put4(y + (size_t)(sg.row0 + i) * ldy + d, a.x, a.y, a.z, a.w);
+      renew_own(p, h);
+    }
   }
   if (tile == 0 && shared_block >= 0) {
     const int stop = min(end, (shared_block + 1) * bs);
-    for (int p = max(sg.pos0, stop - cs.keep); p < stop; ++p) renew(p, get4(hin + (size_t)(sg.row0 + p - sg.pos0) * ldy + d));
+    for (int p = max(sg.pos0, stop - cs.keep); p < stop; ++p) renew(p, get4(hs + (size_t)(p - sg.pos0) * ldy));
   }
 }
 
@@ -464,6 +570,22 @@ int launch_sandwich_rows(const float* resid_in, float* resid_out, const RowSourc
     if (rc != MI_OK) return rc;
     cs = *conv;
   }
+  if (T <= 32 && w_pre && ld <= 4096 && ld == D && (D / groups) % 256 == 0 && (!conv || conv->taps <= 4)) {
+    const int threads = ceil_div(ld / 4, 64) * 64, gs = D / groups;
+#define MI_TOKEN(TAPS) \
+    if (f32) hipLaunchKernelGGL((sandwich_token_kernel<float, TAPS>), dim3(T), dim3(threads), 0, s, resid_in, resid_out, src, w_post, w_pre, D, ld, gs, eps, cs, (float*)y, ldy); \
+    else hipLaunchKernelGGL((sandwich_token_kernel<uint16_t, TAPS>), dim3(T), dim3(threads), 0, s, resid_in, resid_out, src, w_post, w_pre, D, ld, gs, eps, cs, (uint16_t*)y, ldy)
+    switch (conv ? conv->taps : 0) {
+      case 0: MI_TOKEN(0); break;
+      case 1: MI_TOKEN(1); break;
+      case 2: MI_TOKEN(2); break;
+      case 3: MI_TOKEN(3); break;
+      default: MI_TOKEN(4);
+    }
+#undef MI_TOKEN
+    MI_HIP(hipGetLastError());
+    return MI_OK;
+  }
   const size_t lds = (size_t)(ld + std::max(groups, 16) + groups) * sizeof(float);
   const int threads = T <= 32 ? std::min(1024, ceil_div(ld / 4, 64) * 64) : 256;
   const void* kern = f32 ? reinterpret_cast<const void*>(sandwich_rows_kernel<float>) : reinterpret_cast<const void*>(sandwich_rows_kernel<uint16_t>);
@@ -480,11 +602,21 @@ int launch_conv_rows(const void* h, const ConvState& conv, const AttnSeg* sd, co
   int rc = check_conv(conv);
   if (rc != MI_OK) return rc;
   MI_CHECK(nseg >= 1 && ld % 4 == 0 && ld >= D && ldy >= ld && ldy % 4 == 0 && h != y, "convolution: strides");
+  const int rows = conv.taps <= 4 ? 8 : kConvRows;
   int tiles = 0;
-  for (int i = 0; i < nseg; ++i) tiles += ceil_div(sh[i].n, kConvRows);
+  for (int i = 0; i < nseg; ++i) tiles += ceil_div(sh[i].n, rows);
   const dim3 grid(tiles, ceil_div(ld, 1024));
-  if (f32) hipLaunchKernelGGL((conv_rows_kernel<float>), grid, dim3(256), 0, s, (const float*)h, conv, sd, nseg, ld, (float*)y, ldy);
-  else hipLaunchKernelGGL((conv_rows_kernel<uint16_t>), grid, dim3(256), 0, s, (const uint16_t*)h, conv, sd, nseg, ld, (uint16_t*)y, ldy);
+#define MI_CONV(TAPS, ROWS) \
+  if (f32) hipLaunchKernelGGL((conv_rows_kernel<float, TAPS, ROWS>), grid, dim3(256), 0, s, (const float*)h, conv, sd, nseg, ld, (float*)y, ldy); \
+  else hipLaunchKernelGGL((conv_rows_kernel<uint16_t, TAPS, ROWS>), grid, dim3(256), 0, s, (const uint16_t*)h, conv, sd, nseg, ld, (uint16_t*)y, ldy)
+  switch (conv.taps) {
+    case 2: MI_CONV(2, 8); break;
+    case 3: MI_CONV(3, 8); break;
+    case 4: MI_CONV(4, 8); break;
+    case 1: MI_CONV(1, 8); break;
+    default: MI_CONV(0, kConvRows);
+  }
+#undef MI_CONV
   MI_HIP(hipGetLastError());
   return MI_OK;
 }

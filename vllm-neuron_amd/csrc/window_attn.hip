@@ -100,7 +100,7 @@ template <int DK, int DV>
 constexpr size_t prefill_lds() { return (size_t)64 * (DK + kPitch + DV + kPitch) * 2; }
 
 template <int DK, int DV, int NCG, bool FIXED>
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(NCG == 1 ? 1 : 2, NCG == 1 ? 1 : 2))) void attn_window_prefill_kernel(AttnSpec a, const uint16_t* __restrict__ q, const uint16_t* __restrict__ kpool,
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK > 128 ? 1 : 2, DK > 128 ? 1 : 2))) void attn_window_prefill_kernel(AttnSpec a, const uint16_t* __restrict__ q, const uint16_t* __restrict__ kpool,
                                                                   const uint16_t* __restrict__ vpool, int bs, const int32_t* __restrict__ bt,
                                                                   int MB, const AttnSeg* __restrict__ segs, int nseg,
                                                                   uint16_t* __restrict__ out, int ldo, float s_max, int fold, int min_rows) {
@@ -631,7 +631,16 @@ int launch_attn_window_prefill(const AttnSpec& a, const uint16_t* q, const uint1
   int rc = check_spec(a, bs);
   if (rc != MI_OK) return rc;
   MI_CHECK(attn_window_supported(a.g) && nseg >= 1 && min_rows >= 2 && ldo >= a.g.H * a.g.dv && ((a.g.dv & 3) != 0 || ldo % 4 == 0), "windowed prefill attention: shape");
-#define MI_CALL_P(DK, DV, NCG) launch_prefill_t<DK, DV, NCG>(a, q, kpool, vpool, bs, bt, MB, sd, sh, nseg, out, ldo, s, min_rows)
+  // a grid that does not give every CU two work-groups takes tiles of half the queries (two waves per SIMD overlap, and light
+  // tiles pair up with heavy ones)
+  int num_cu = 0, tiles = 0;
+  rc = device_num_cu(&num_cu);
+  if (rc != MI_OK) return rc;
+  for (int i = 0; i < nseg; ++i) tiles += sh[i].n >= min_rows ? ceil_div(sh[i].n, 128 / (a.g.H / a.g.G)) : 0;
+  const bool half = tiles * a.g.G < 2 * num_cu;
+#define MI_CALL_P(DK, DV, NCG) \
+  half ? launch_prefill_t<DK, DV, 1>(a, q, kpool, vpool, bs, bt, MB, sd, sh, nseg, out, ldo, s, min_rows) \
+       : launch_prefill_t<DK, DV, NCG>(a, q, kpool, vpool, bs, bt, MB, sd, sh, nseg, out, ldo, s, min_rows)
   MI_BY_SIZE(MI_CALL_P);
 #undef MI_CALL_P
 }

@@ -5,7 +5,7 @@ namespace mi {
 
 namespace {
 
-constexpr int kMaxTop = 64, kRouteExperts = 16;
+constexpr int kMaxTop = 64, kRouteExperts = 8;
 
 // ---- router: one work-group per row; a wave takes every fourth expert ----------------------------------------------------
 __device__ __forceinline__ float dot8(const uint16_t* w, const float* x) {
@@ -32,9 +32,51 @@ __device__ __forceinline__ void load8f(const float* p, float* o) {
   for (int i = 0; i < 8; ++i) o[i] = p[i];
 }
 
-// the `top` largest of z [E] (LDS; destroyed), by one wave; softmax over them
+__device__ __forceinline__ float wave_max(float v) {
+#pragma unroll
+  for (int m = 32; m >= 1; m >>= 1) v = fmaxf(v, __shfl_xor(v, m));
+  return v;
+}
+// The `top` largest of z [E] (LDS; z[E .. E + 3] may be written), by one wave; softmax over them, largest first, ties to the lowest
+// expert.  Up to 256 experts: a logit's place is the number of logits ahead of it; beyond: one maximum after another (z destroyed).
 __device__ __forceinline__ void pick_top(float* z, int E, int top, int32_t* ids, float* weights) {
   const int lane = threadIdx.x & 63;
+  if (E <= 256) {
+    if (lane < 4) z[E + lane] = -INFINITY;
+    float v[4], w[4], mx = -INFINITY, sum = 0.f;
+    int place[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int e = lane + 64 * i;
+      v[i] = e < E ? z[e] : -INFINITY;
+      if (!(v[i] == v[i])) v[i] = -INFINITY;                    // (a NaN is refused)
+      place[i] = e < E ? 0 : 1 << 20;
+      mx = fmaxf(mx, v[i]);
+    }
+    for (int j = 0; j < E; j += 4) {
+      const float4 q = *reinterpret_cast<const float4*>(z + j);
+      const float u[4] = {q.x, q.y, q.z, q.w};
+#pragma unroll
+      for (int k = 0; k < 4; ++k)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          if (64 * i >= E) break;
+          const float t = u[k] == u[k] ? u[k] : -INFINITY;
+          place[i] += (t > v[i] || (t == v[i] && j + k < lane + 64 * i)) ? 1 : 0;
+        }
+    }
+    mx = wave_max(mx);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      w[i] = place[i] < top ? expf(v[i] - mx) : 0.f;
+      sum += w[i];
+    }
+    sum = wave_sum(sum);
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (place[i] < top) { ids[place[i]] = lane + 64 * i; weights[place[i]] = w[i] / sum; }
+    return;
+  }
   float first = 0.f, sum = 0.f;
   float mine = 0.f;      // lane j keeps the j-th weight
   int mine_id = 0;
@@ -63,25 +105,26 @@ template <typename T>
 __global__ __launch_bounds__(256) void route_kernel(const T* __restrict__ x, int ldx, const T* __restrict__ w, const float* __restrict__ b, int E,
                                                     int K, int top, int32_t* __restrict__ ids, float* __restrict__ weights, float* __restrict__ zg,
                                                     uint32_t* __restrict__ tickets) {
-  extern __shared__ __attribute__((aligned(16))) float sm[];   // K + E floats
+  extern __shared__ __attribute__((aligned(16))) float z[];   // E floats + 4
   __shared__ uint32_t arrived;
-  float *xs = sm, *z = sm + K;
   const int e0 = blockIdx.y * kRouteExperts, e1 = tickets ? min(e0 + kRouteExperts, E) : E;
   const int t = blockIdx.x, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
-  for (int k = tid * 8; k < K; k += 2048) load8f(x + (size_t)t * ldx + k, xs + k);
-  __syncthreads();
-  for (int e = e0 + wave * 4; e < e1; e += 16) {       // four experts at a time: their rows are in flight together
-    float a[4] = {0.f, 0.f, 0.f, 0.f};
-    for (int k = lane * 8; k < K; k += 512)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) a[i] += dot8(w + (size_t)min(e + i, e1 - 1) * K + k, xs + k);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const float v = wave_sum(a[i]);
-      if (lane != 0 || e + i >= e1) continue;
-      if (tickets) __hip_atomic_store(zg + (size_t)t * E + e + i, v + b[e + i], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-      else z[e + i] = v + b[e + i];
+  for (int e = e0 + wave * 2; e < e1; e += 8) {       // two experts at a time, their rows and x requested together
+    float a0 = 0.f, a1 = 0.f;
+    const T *w0 = w + (size_t)e * K, *w1 = w + (size_t)min(e + 1, e1 - 1) * K;
+#pragma unroll 4
+    for (int k = lane * 8; k < K; k += 512) {
+      float xv[8];
+      load8f(x + (size_t)t * ldx + k, xv);
+      a0 += dot8(w0 + k, xv);
+      a1 += dot8(w1 + k, xv);
     }
+    a0 = wave_sum(a0);
+    a1 = wave_sum(a1);
+    if (lane >= 2 || e + lane >= e1) continue;
+    const float v = (lane ? a1 : a0) + b[e + lane];
+    if (tickets) __hip_atomic_store(zg + (size_t)t * E + e + lane, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    else z[e + lane] = v;
   }
   if (tickets) {       // the row's last work-group to arrive picks; it leaves the ticket at zero for the next launch
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // every storing wave drains its write-through stores
@@ -99,10 +142,10 @@ __global__ __launch_bounds__(256) void route_kernel(const T* __restrict__ x, int
 // a wave per row
 __global__ __launch_bounds__(256) void route_pick_kernel(const float* __restrict__ zg, int ldz, int T, int E, int top, int32_t* __restrict__ ids,
                                                          float* __restrict__ weights) {
-  extern __shared__ __attribute__((aligned(16))) float sm[];   // 4 E floats
+  extern __shared__ __attribute__((aligned(16))) float sm[];   // 4 x (E padded to 4, + 4) floats
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, t = blockIdx.x * 4 + wave;
   if (t >= T) return;
-  float* z = sm + wave * E;            // (one wave's own: LDS operations of a wave execute in order)
+  float* z = sm + wave * ((E + 3) / 4 * 4 + 4);            // (one wave's own: LDS operations of a wave execute in order)
   for (int e = lane; e < E; e += 64) z[e] = zg[(size_t)t * ldz + e];
   pick_top(z, E, top, ids + (size_t)t * top, weights + (size_t)t * top);
 }
@@ -342,10 +385,8 @@ int launch_stream(const ExpertsLinear& w, const int32_t* ids, int P, const uint1
 int launch_route(const void* x, int ldx, int T, const void* w, const float* b, int E, int K, int top, int32_t* ids, float* weights, bool f32, hipStream_t s,
                  float* z, uint32_t* tickets) {
   MI_CHECK(T >= 1 && E >= 1 && top >= 1 && top <= E && top <= kMaxTop && K % 64 == 0 && ldx >= K && ldx % 8 == 0, "router: 1 <= top <= min(experts, 64), row stride");
-  const size_t lds = (size_t)(K + E) * 4;
-  const void* kern = f32 ? reinterpret_cast<const void*>(route_kernel<float>) : reinterpret_cast<const void*>(route_kernel<uint16_t>);
-  MI_CHECK(lds <= 160 * 1024, "router: row and logits larger than the LDS");
-  if (lds > 64 * 1024) { int rc = ensure_dynamic_lds(kern, 160 * 1024); if (rc != MI_OK) return rc; }
+  const size_t lds = (size_t)(E + 8) * 4;
+  MI_CHECK(E <= 4096, "router: up to 4096 experts");
   MI_CHECK(!tickets || z, "router: tickets without logits");
   const dim3 grid(T, tickets ? ceil_div(E, kRouteExperts) : 1);
   if (f32) hipLaunchKernelGGL((route_kernel<float>), grid, dim3(256), lds, s, (const float*)x, ldx, (const float*)w, b, E, K, top, ids, weights, z, tickets);
@@ -356,7 +397,7 @@ int launch_route(const void* x, int ldx, int T, const void* w, const float* b, i
 
 int launch_route_pick(const float* z, int ldz, int T, int E, int top, int32_t* ids, float* weights, hipStream_t s) {
   MI_CHECK(T >= 1 && E >= 1 && E <= 4096 && top >= 1 && top <= E && top <= kMaxTop && ldz >= E, "router: experts / top");
-  hipLaunchKernelGGL(route_pick_kernel, dim3(ceil_div(T, 4)), dim3(256), (size_t)16 * E, s, z, ldz, T, E, top, ids, weights);
+  hipLaunchKernelGGL(route_pick_kernel, dim3(ceil_div(T, 4)), dim3(256), (size_t)16 * (E + 8), s, z, ldz, T, E, top, ids, weights);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }

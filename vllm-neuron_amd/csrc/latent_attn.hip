@@ -159,18 +159,18 @@ __device__ __forceinline__ float sexp2(float x, float m) { return (x == -INFINIT
 
 constexpr int kCPitch = 16;
 template <int RP, int HG>
-constexpr size_t latent_lds() { return (size_t)64 * (RP + kCPitch) * 2 + (size_t)HG * RP * 32 + (size_t)HG * 4 * 64 * 8 + (size_t)HG * 4 * 16 * 4; }
+constexpr size_t latent_lds() { return (size_t)64 * (RP + kCPitch) * 2 + (HG == 1 ? 0 : (size_t)HG * RP * 32) + (size_t)HG * 4 * 64 * 8 + (size_t)HG * 4 * 16 * 4; }
 
 template <int RP, int HG, bool FINAL>
-__global__ __launch_bounds__(256) void latent_rows_kernel(LatentGeom g, float sc2, int window, const uint16_t* __restrict__ qa,
+__global__ __launch_bounds__(256, HG == 1 ? 2 : 1) void latent_rows_kernel(LatentGeom g, float sc2, int window, const uint16_t* __restrict__ qa,
                                                           const uint16_t* __restrict__ pool, int bs, const int32_t* __restrict__ bt, int MB,
-                                                          const int32_t* __restrict__ pos, LatentRows lr, int NS, float* __restrict__ o_part,
+                                                          const int32_t* __restrict__ pos, LatentRows lr, int NS, int bs_shift, float* __restrict__ o_part,
                                                           float* __restrict__ ml_part, uint16_t* __restrict__ lat) {
   constexpr int CP = RP + kCPitch, KS = RP / 32, DN = RP / 64, CCH = RP / 8, NL = 64 * CCH / 256;
   extern __shared__ __attribute__((aligned(16))) unsigned char dsm[];
   uint16_t* Cs = reinterpret_cast<uint16_t*>(dsm);                        // [64][CP]
-  u32x4_t* Qs = reinterpret_cast<u32x4_t*>(Cs + 64 * CP);                 // [HG][KS][64 lanes]
-  uint2* Ps = reinterpret_cast<uint2*>(Qs + HG * KS * 64);                // [HG][4 waves][64 lanes]
+  u32x4_t* Qs = reinterpret_cast<u32x4_t*>(Cs + 64 * CP);                 // [HG][KS][64 lanes]; one head group: in registers
+  uint2* Ps = reinterpret_cast<uint2*>(Qs + (HG == 1 ? 0 : HG * KS * 64));   // [HG][4 waves][64 lanes]
   float* Ms = reinterpret_cast<float*>(Ps + HG * 4 * 64);                 // [HG][4 waves][16]
   const int split = blockIdx.x, h0 = blockIdx.y * 16 * HG, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g4 = lane >> 4, c = lane & 15;
   const RowAt at = latent_row(lr, blockIdx.z);
@@ -181,30 +181,48 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(LatentGeom g, float sc
   const int last_ch = g.rp / 8 - 1;
 
   u32x4_t cr[NL];
-  int ids[4];
+  // (addresses: a uniform part per 16-token group and a per-lane part that never changes, as in window_attn.hip)
+  int blk[4], off[4];
   auto fetch_ids = [&](int tt) {     // the block of every 16-token group (block_size is a multiple of 16); past the keys: the null block
 #pragma unroll
-    for (int u = 0; u < 4; ++u) ids[u] = tt < t1 && tt * 64 + 16 * u < ctx ? btr[(tt * 64 + 16 * u) / bs] : 0;
+    for (int u = 0; u < 4; ++u) {
+      const int k = tt * 64 + 16 * u;
+      int bi;
+      if (bs_shift >= 0) { bi = k >> bs_shift; off[u] = k & (bs - 1); }
+      else { bi = k / bs; off[u] = k - bi * bs; }
+      const bool in = tt < t1 && k < ctx;
+      blk[u] = in ? btr[bi] : 0;
+      if (!in) off[u] = 0;
+    }
   };
-  auto issue = [&](int tt) {
-    size_t base[4];
+  constexpr int R = 256 / CCH;       // rows of a load
+  const int row0 = tid / CCH, lane_off = (row0 & 15) * g.rp + min(tid % CCH, last_ch) * 8;
+  auto issue = [&]() {               // the tile whose ids fetch_ids loaded last
+    const uint16_t* base[4];
 #pragma unroll
-    for (int u = 0; u < 4; ++u) base[u] = tt * 64 + 16 * u < ctx ? (size_t)ids[u] * bs + (tt * 64 + 16 * u) % bs : 0;
+    for (int u = 0; u < 4; ++u) base[u] = pool + ((size_t)blk[u] * bs + off[u]) * g.rp;
 #pragma unroll
     for (int i = 0; i < NL; ++i) {
-      const int idx = tid + 256 * i, row = idx / CCH, ch = min(idx % CCH, last_ch), u = row >> 4;
-      const size_t b = u < 2 ? (u == 0 ? base[0] : base[1]) : (u == 2 ? base[2] : base[3]);
-      cr[i] = *reinterpret_cast<const u32x4_t*>(pool + (b + (row & 15)) * g.rp + ch * 8);
+      const uint16_t* b = base[i * R / 16];
+      if constexpr (R == 32) b = row0 >= 16 ? base[i * 2 + 1] : base[i * 2];
+      cr[i] = *reinterpret_cast<const u32x4_t*>(b + (R < 16 ? (i * R % 16) * g.rp : 0) + lane_off);
     }
   };
   if (t0 < t1) {
     fetch_ids(t0);
-    issue(t0);
+    issue();
     fetch_ids(t0 + 1);
   }
-  for (int i = tid; i < HG * KS * 64; i += 256) {
-    const int l = i & 63, ks = (i >> 6) % KS, hg = (i >> 6) / KS, h = h0 + hg * 16 + (l & 15), d = ks * 32 + (l >> 4) * 8;
-    Qs[i] = h < g.H && d < g.rp ? *reinterpret_cast<const u32x4_t*>(qa + ((size_t)at.row * g.H + h) * g.rp + d) : u32x4_t{0, 0, 0, 0};
+  u32x4_t qr[KS];
+  auto q_frag = [&](int hg, int ks, int l) {
+    const int h = h0 + hg * 16 + (l & 15), d = ks * 32 + (l >> 4) * 8;
+    return h < g.H && d < g.rp ? *reinterpret_cast<const u32x4_t*>(qa + ((size_t)at.row * g.H + h) * g.rp + d) : u32x4_t{0, 0, 0, 0};
+  };
+  if constexpr (HG == 1) {
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) qr[ks] = q_frag(0, ks, lane);
+  } else {
+    for (int i = tid; i < HG * KS * 64; i += 256) Qs[i] = q_frag((i >> 6) / KS, (i >> 6) % KS, i & 63);
   }
   f32x4_t acc[HG][DN];
   float mrow[HG], lrow[HG];
@@ -226,7 +244,7 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(LatentGeom g, float sc
     }
     __syncthreads();
     if (tt + 1 < t1) {
-      issue(tt + 1);
+      issue();
       fetch_ids(tt + 2);
     }
     f32x4_t st[HG];
@@ -237,7 +255,7 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(LatentGeom g, float sc
       const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(&Cs[(16 * wave + c) * CP + ks * 32 + g4 * 8]);
 #pragma unroll
       for (int hg = 0; hg < HG; ++hg)
-        st[hg] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, __builtin_bit_cast(bf16x8_t, Qs[(hg * KS + ks) * 64 + lane]), st[hg], 0, 0, 0);
+        st[hg] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, __builtin_bit_cast(bf16x8_t, HG == 1 ? qr[ks] : Qs[(hg * KS + ks) * 64 + lane]), st[hg], 0, 0, 0);
     }
     const int j0 = tt * 64 + 16 * wave + 4 * g4;
 #pragma unroll
@@ -427,7 +445,7 @@ int launch_rows_t(const LatentGeom& g, float scale, int window, const uint16_t* 
   const dim3 grid(NS, ceil_div(g.H, 16 * HG), lr.rows);
   auto kern = NS == 1 ? latent_rows_kernel<RP, HG, true> : latent_rows_kernel<RP, HG, false>;
   if (lds > 64 * 1024) { int rc = ensure_dynamic_lds(reinterpret_cast<const void*>(kern), (int)lds); if (rc != MI_OK) return rc; }
-  hipLaunchKernelGGL(kern, grid, dim3(256), lds, s, g, scale * kLog2e, window, qa, pool, bs, bt, MB, pos, lr, NS, op, ml, lat);
+  hipLaunchKernelGGL(kern, grid, dim3(256), lds, s, g, scale * kLog2e, window, qa, pool, bs, bt, MB, pos, lr, NS, (bs & (bs - 1)) == 0 ? __builtin_ctz(bs) : -1, op, ml, lat);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
@@ -474,8 +492,8 @@ int launch_head_linear(const void* w, int H, int N, int K, const void* x, int T,
 
 bool latent_attn_supported(const LatentGeom& g) { return g.rp <= 512; }
 
-// (rows x splits <= 256, launch_latent_attn_rows)
-size_t latent_attn_scratch_bytes(const LatentGeom& g) { return (size_t)256 * g.H * (g.rp + 2) * sizeof(float); }
+// (rows x splits <= 512, launch_latent_attn_rows)
+size_t latent_attn_scratch_bytes(const LatentGeom& g) { return (size_t)512 * g.H * (g.rp + 2) * sizeof(float); }
 
 int launch_latent_attn_rows(const LatentGeom& g, float scale, int window, const uint16_t* qa, const uint16_t* pool, int bs, const int32_t* bt,
                             int MB, const int32_t* pos, const LatentRows& lr, int max_ctx, const void* w_uv, uint16_t* lat, uint16_t* out, int ldo,
@@ -486,10 +504,11 @@ int launch_latent_attn_rows(const LatentGeom& g, float scale, int window, const 
   int hg = 1;
   while (hg < 4 && hg < hgs && lr.rows * ceil_div(hgs, 2 * hg) >= 256) hg *= 2;
   const int groups = lr.rows * ceil_div(hgs, hg);
-  int NS = min(min(256 / groups, tiles), kMaxSplits);
+  // (one head group: 70 KiB of LDS at the largest rank, two work-groups per CU)
+  int NS = min(min((hg == 1 ? 512 : 256) / groups, tiles), kMaxSplits);
   if (NS < 1) NS = 1;
   float* ml = reinterpret_cast<float*>(scratch);
-  float* op = ml + (size_t)256 * g.H * 2;
+  float* op = ml + (size_t)512 * g.H * 2;
   int rc = MI_OK;
 #define MI_LR(RP) \
   rc = hg == 1 ? launch_rows_t<RP, 1>(g, scale, window, qa, pool, bs, bt, MB, pos, lr, NS, op, ml, lat, s) \

@@ -8,6 +8,8 @@
 
 #include "window_attn.h"
 
+#include <type_traits>
+
 namespace mi {
 
 namespace {
@@ -99,18 +101,21 @@ constexpr int kPitch = 16;
 template <int DK, int DV>
 constexpr size_t prefill_lds() { return (size_t)64 * (DK + kPitch + DV + kPitch) * 2; }
 
-template <int DK, int DV, int NCG, bool FIXED>
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK > 128 ? 1 : 2, DK > 128 ? 1 : 2))) void attn_window_prefill_kernel(AttnSpec a, const uint16_t* __restrict__ q, const uint16_t* __restrict__ kpool,
+// KS = 2: a second set of four waves takes every other key tile of the same queries (short grids, whose heaviest work-group is what
+// the launch waits for); the two sets' sums meet in LDS at the end.
+template <int DK, int DV, int NCG, int KS2, bool FIXED>
+__global__ __launch_bounds__(256 * KS2) __attribute__((amdgpu_waves_per_eu(DK > 128 ? KS2 : 2, DK > 128 ? KS2 : 2))) void attn_window_prefill_kernel(AttnSpec a, const uint16_t* __restrict__ q, const uint16_t* __restrict__ kpool,
                                                                   const uint16_t* __restrict__ vpool, int bs, const int32_t* __restrict__ bt,
                                                                   int MB, const AttnSeg* __restrict__ segs, int nseg,
-                                                                  uint16_t* __restrict__ out, int ldo, float s_max, int fold, int min_rows) {
+                                                                  uint16_t* __restrict__ out, int ldo, float s_max, int fold, int min_rows, int bs_shift) {
   constexpr int KP = DK + kPitch, VP = DV + kPitch;    // LDS row pitches (elements)
   constexpr int KS = DK / 32, DN = DV / 16, KCH = DK / 8, VCH = DV / 8;
   constexpr int NKL = 64 * KCH / 256, NVL = 64 * VCH / 256;   // 16-byte loads per thread and tile
   extern __shared__ __attribute__((aligned(16))) unsigned char dsm[];
-  uint16_t* Ks = reinterpret_cast<uint16_t*>(dsm);
+  const int set = KS2 == 1 ? 0 : (int)threadIdx.x >> 8;
+  uint16_t* Ks = reinterpret_cast<uint16_t*>(dsm) + set * (64 * (KP + VP));
   uint16_t* Vs = Ks + 64 * KP;
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g4 = lane >> 4, c = lane & 15;
+  const int tid = threadIdx.x & 255, wave = tid >> 6, lane = tid & 63, g4 = lane >> 4, c = lane & 15;
   const int H = a.g.H, G = a.g.G, r = H / G, qpt = (64 * NCG) / r, kvh = blockIdx.x;
 
   // this work-group's tile: segments with one row belong to the token-generation kernel.  Late tiles (long contexts) first; a
@@ -131,36 +136,48 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK > 128 ? 
   const int klo = max(0, pos0 - win + 1) & ~15, khi = pos0 + nq - 1;
   const int nt = ceil_div(khi + 1 - klo, 64);
 
+  // Addresses are a uniform part per 16-token group (block_size is a multiple of 16) and a per-lane part that never changes: thread
+  // load i covers rows i R .. of the tile, R = 256 / chunks per row.
   const int dkc = a.g.dkp / 8 - 1, dvc = a.g.dvp / 8 - 1;   // last 16-byte chunk of a pool row
   u32x4_t kr[NKL], vr[NVL];
-  int ids[4];
-  auto fetch_ids = [&](int k0) {     // block of each 16-token group (block_size is a multiple of 16); past the keys: the null block
+  int blk[4], off[4];
+  auto fetch_ids = [&](int k0) {     // block of each 16-token group; past the keys: the null block
 #pragma unroll
-    for (int u = 0; u < 4; ++u) ids[u] = (k0 + 16 * u <= khi) ? btr[(k0 + 16 * u) / bs] : 0;
+    for (int u = 0; u < 4; ++u) {
+      const int k = k0 + 16 * u;
+      int bi;
+      if (bs_shift >= 0) { bi = k >> bs_shift; off[u] = k & (bs - 1); }
+      else { bi = k / bs; off[u] = k - bi * bs; }
+      const bool in = k <= khi;
+      blk[u] = in ? btr[bi] : 0;
+      if (!in) off[u] = 0;
+    }
   };
-  auto issue = [&](int k0) {
+  auto load_tile = [&](auto& reg, const uint16_t* pool, const size_t (&base)[4], int rowp, int last, auto chunks) {
+    constexpr int CH = decltype(chunks)::value, R = 256 / CH, N = 64 / R;
+    const int row0 = tid / CH, lane_off = (row0 & 15) * rowp + min(tid % CH, last) * 8;
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      if constexpr (R >= 16) {
+        size_t b = base[i * R / 16];
+        if constexpr (R == 32) b = row0 >= 16 ? base[i * 2 + 1] : base[i * 2];
+        reg[i] = *reinterpret_cast<const u32x4_t*>(pool + b * rowp + lane_off);
+      } else {
+        reg[i] = *reinterpret_cast<const u32x4_t*>(pool + base[i * R / 16] * rowp + (i * R % 16) * rowp + lane_off);
+      }
+    }
+  };
+  auto issue = [&]() {               // the tile whose ids fetch_ids loaded last
     size_t base[4];
 #pragma unroll
-    for (int u = 0; u < 4; ++u)
-      base[u] = (k0 + 16 * u <= khi) ? ((size_t)ids[u] * G + kvh) * bs + (k0 + 16 * u) % bs : 0;
-    auto row_of = [&](int row) -> size_t {
-      const int u = row >> 4;
-      return (u < 2 ? (u == 0 ? base[0] : base[1]) : (u == 2 ? base[2] : base[3])) + (row & 15);
-    };
-#pragma unroll
-    for (int i = 0; i < NKL; ++i) {
-      const int idx = tid + 256 * i, row = idx / KCH, ch = min(idx % KCH, dkc);
-      kr[i] = *reinterpret_cast<const u32x4_t*>(kpool + row_of(row) * a.g.dkp + ch * 8);
-    }
-#pragma unroll
-    for (int i = 0; i < NVL; ++i) {
-      const int idx = tid + 256 * i, row = idx / VCH, ch = min(idx % VCH, dvc);
-      vr[i] = *reinterpret_cast<const u32x4_t*>(vpool + row_of(row) * a.g.dvp + ch * 8);
-    }
+    for (int u = 0; u < 4; ++u) base[u] = ((size_t)blk[u] * G + kvh) * bs + off[u];
+    load_tile(kr, kpool, base, a.g.dkp, dkc, std::integral_constant<int, KCH>{});
+    load_tile(vr, vpool, base, a.g.dvp, dvc, std::integral_constant<int, VCH>{});
   };
-  fetch_ids(klo);
-  issue(klo);
-  fetch_ids(klo + 64);
+  const int k_own = klo + 64 * set;        // this set's first tile
+  fetch_ids(k_own);
+  issue();
+  fetch_ids(k_own + 64 * KS2);
 
   // columns: position, bias slope, query fragments (zero beyond dkp and in dead columns)
   int pc[NCG];
@@ -173,8 +190,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK > 128 ? 
     const bool live = ql < nq && ql < qpt;
     pc[cg] = pos0 + (live ? ql : 0);
     sl2[cg] = a.slopes ? a.slopes[h] * kLog2e : 0.f;
-    mrow[cg] = FIXED ? s_max : (a.sink ? 0.f : -INFINITY);
-    const float d0 = a.sink ? (FIXED ? fexp2(-s_max) : 1.f) : 0.f;
+    mrow[cg] = FIXED ? s_max : (a.sink && set == 0 ? 0.f : -INFINITY);
+    const float d0 = a.sink && set == 0 ? (FIXED ? fexp2(-s_max) : 1.f) : 0.f;
     den[cg] = f32x4_t{d0, d0, d0, d0};
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks)
@@ -192,8 +209,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK > 128 ? 
   const short one = 0x3f80;            // bf16 1.0
   const bf16x8_t ones = {one, one, one, one, one, one, one, one};
 
-  for (int n = 0; n < nt; ++n) {
-    const int k0 = klo + 64 * n;
+  for (int n = 0; n < nt; n += KS2) {
+    const int k0 = k_own + 64 * n;       // (the second set's last tile may lie beyond the keys: no wave sees a key of it)
     __syncthreads();                     // the previous tile is consumed
 #pragma unroll
     for (int i = 0; i < NKL; ++i) {
@@ -206,35 +223,56 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK > 128 ? 
       *reinterpret_cast<u32x4_t*>(&Vs[(idx / VCH) * VP + (idx % VCH) * 8]) = vr[i];
     }
     __syncthreads();
-    if (n + 1 < nt) {
-      issue(k0 + 64);
-      fetch_ids(k0 + 128);
+    if (n + KS2 < nt) {
+      issue();
+      fetch_ids(k0 + 128 * KS2);
     }
     if (!wave_live || k0 > pmax || k0 + 63 <= pmin - win) continue;   // no key of this tile is seen by the wave (uniform)
+    // S^T = K.Q^T: the fragments of a 16-key group are requested one group ahead of the MFMAs that take them
     f32x4_t st[NCG][4];
+    {
+      bf16x8_t kf[KS];
 #pragma unroll
-    for (int u = 0; u < 4; ++u) {
+      for (int ks = 0; ks < KS; ++ks) kf[ks] = *reinterpret_cast<const bf16x8_t*>(&Ks[c * KP + ks * 32 + g4 * 8]);
 #pragma unroll
-      for (int cg = 0; cg < NCG; ++cg) st[cg][u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      for (int u = 0; u < 4; ++u) {
 #pragma unroll
-      for (int ks = 0; ks < KS; ++ks) {
-        const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(&Ks[(16 * u + c) * KP + ks * 32 + g4 * 8]);
+        for (int cg = 0; cg < NCG; ++cg) st[cg][u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int cg = 0; cg < NCG; ++cg)
-          st[cg][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, __builtin_bit_cast(bf16x8_t, qf[cg][ks]), st[cg][u], 0, 0, 0);
+        for (int ks = 0; ks < KS; ++ks) {
+#pragma unroll
+          for (int cg = 0; cg < NCG; ++cg)
+            st[cg][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[ks], __builtin_bit_cast(bf16x8_t, qf[cg][ks]), st[cg][u], 0, 0, 0);
+          if (u < 3) kf[ks] = *reinterpret_cast<const bf16x8_t*>(&Ks[(16 * (u + 1) + c) * KP + ks * 32 + g4 * 8]);
+        }
       }
+      __builtin_amdgcn_sched_group_barrier(0x100, KS, 0);
+#pragma unroll
+      for (int i = 0; i < 3 * KS; ++i) {
+        __builtin_amdgcn_sched_group_barrier(0x8, NCG, 0);
+        __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
+      }
+#pragma unroll
+      for (int i = 0; i < KS; ++i) __builtin_amdgcn_sched_group_barrier(0x8, NCG, 0);
     }
     const bool edge = k0 + 63 > pmin || k0 <= pmax - win;
     union { uint32_t w[4]; bf16x8_t v; } pk[NCG][2];
 #pragma unroll
     for (int cg = 0; cg < NCG; ++cg) {
-      // - slope (i - j) of the lane's first key (- the fixed reference)
-      const float b0 = __builtin_fmaf(sl2[cg], (float)(k0 + 4 * g4 - pc[cg]), FIXED ? -s_max : 0.f);
+      if (a.slopes) {
+        // - slope (i - j) of the lane's first key (- the fixed reference)
+        const float b0 = __builtin_fmaf(sl2[cg], (float)(k0 + 4 * g4 - pc[cg]), FIXED ? -s_max : 0.f);
 #pragma unroll
-      for (int u = 0; u < 4; ++u)
+        for (int u = 0; u < 4; ++u)
 #pragma unroll
-        for (int i = 0; i < 4; ++i)
-          st[cg][u][i] = __builtin_fmaf(st[cg][u][i], sc2, __builtin_fmaf(sl2[cg], (float)(16 * u + i), b0));
+          for (int i = 0; i < 4; ++i)
+            st[cg][u][i] = __builtin_fmaf(st[cg][u][i], sc2, __builtin_fmaf(sl2[cg], (float)(16 * u + i), b0));
+      } else {
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) st[cg][u][i] = FIXED ? __builtin_fmaf(st[cg][u][i], sc2, -s_max) : st[cg][u][i] * sc2;
+      }
       if (edge) {
         const int j0 = k0 + 4 * g4;
 #pragma unroll
@@ -277,20 +315,63 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DK > 128 ? 
 #pragma unroll
       for (int hf = 0; hf < 2; ++hf) den[cg] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pk[cg][hf].v, den[cg], 0, 0, 0);
     }
-    // O^T += V^T.P^T: the k-slot (g4, j) of a 32-key half is key (j < 4 ? 4 g4 + j : 16 + 4 g4 + j - 4)
+    // O^T += V^T.P^T: the k-slot (g4, j) of a 32-key half is key (j < 4 ? 4 g4 + j : 16 + 4 g4 + j - 4); fragments requested
+    // kAhead MFMAs ahead of their use
+    {
+      constexpr int NPV = 2 * DN, kAhead = NPV < 4 ? NPV : 4;
+      s16x4_t vlo[NPV], vhi[NPV];
+      auto vread = [&](int i) {
+        const uint16_t* r0 = &Vs[(32 * (i / DN) + 4 * g4 + tr_row) * VP + 16 * (i % DN) + tr_col];
+        vlo[i] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4_t __attribute__((address_space(3)))*)r0);
+        vhi[i] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4_t __attribute__((address_space(3)))*)(r0 + 16 * VP));
+      };
 #pragma unroll
-    for (int hf = 0; hf < 2; ++hf)
+      for (int i = 0; i < kAhead; ++i) vread(i);
 #pragma unroll
-      for (int dn = 0; dn < DN; ++dn) {
-        const uint16_t* r0 = &Vs[(32 * hf + 4 * g4 + tr_row) * VP + 16 * dn + tr_col];
-        const s16x4_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4_t __attribute__((address_space(3)))*)r0);
-        const s16x4_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4_t __attribute__((address_space(3)))*)(r0 + 16 * VP));
-        const bf16x8_t av = {lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
+      for (int i = 0; i < NPV; ++i) {
+        const bf16x8_t av = {vlo[i][0], vlo[i][1], vlo[i][2], vlo[i][3], vhi[i][0], vhi[i][1], vhi[i][2], vhi[i][3]};
 #pragma unroll
-        for (int cg = 0; cg < NCG; ++cg) acc[cg][dn] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(av, pk[cg][hf].v, acc[cg][dn], 0, 0, 0);
+        for (int cg = 0; cg < NCG; ++cg) acc[cg][i % DN] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(av, pk[cg][i / DN].v, acc[cg][i % DN], 0, 0, 0);
+        if (i + kAhead < NPV) vread(i + kAhead);
       }
+      __builtin_amdgcn_sched_group_barrier(0x100, 2 * kAhead, 0);
+#pragma unroll
+      for (int i = 0; i < NPV; ++i) {
+        __builtin_amdgcn_sched_group_barrier(0x8, NCG, 0);
+        if (i + kAhead < NPV) __builtin_amdgcn_sched_group_barrier(0x100, 2, 0);
+      }
+    }
   }
 
+  if constexpr (KS2 == 2) {              // the second set hands over its sums, lane by lane
+    float* x = reinterpret_cast<float*>(dsm) + (size_t)tid * 4;      // [DN + 1][256 lanes][4], one column group at a time
+#pragma unroll
+    for (int cg = 0; cg < NCG; ++cg) {
+      __syncthreads();
+      if (set == 1) {
+#pragma unroll
+        for (int dn = 0; dn < DN; ++dn) *reinterpret_cast<f32x4_t*>(x + dn * 1024) = acc[cg][dn];
+        *reinterpret_cast<float2*>(x + DN * 1024) = make_float2(mrow[cg], den[cg][0]);
+      }
+      __syncthreads();
+      if (set == 0) {
+        const float2 ml = *reinterpret_cast<const float2*>(x + DN * 1024);
+        float f0 = 1.f, f1 = 1.f;
+        if constexpr (!FIXED) {
+          const float M = fmaxf(mrow[cg], ml.x);
+          f0 = sexp2(mrow[cg], M); f1 = sexp2(ml.x, M);
+        }
+        den[cg][0] = den[cg][0] * f0 + ml.y * f1;
+#pragma unroll
+        for (int dn = 0; dn < DN; ++dn) {
+          const f32x4_t o = *reinterpret_cast<const f32x4_t*>(x + dn * 1024);
+#pragma unroll
+          for (int i = 0; i < 4; ++i) acc[cg][dn][i] = acc[cg][dn][i] * f0 + o[i] * f1;
+        }
+      }
+    }
+    if (set == 1) return;
+  }
 #pragma unroll
   for (int cg = 0; cg < NCG; ++cg) {
     const float L = den[cg][0];
@@ -565,22 +646,23 @@ float fixed_reference(const AttnSpec& a) {
   return a.unit_norm && b <= 60.f && b > 0.f ? b : 0.f;
 }
 
-template <int DK, int DV, int NCG>
+template <int DK, int DV, int NCG, int KS2>
 int launch_prefill_t(const AttnSpec& a, const uint16_t* q, const uint16_t* kpool, const uint16_t* vpool, int bs, const int32_t* bt, int MB,
                      const AttnSeg* sd, const AttnSeg* sh, int nseg, uint16_t* out, int ldo, hipStream_t s, int min_rows) {
   const int qpt = 64 * NCG / (a.g.H / a.g.G);
   int tiles = 0;
   for (int i = 0; i < nseg; ++i) tiles += sh[i].n >= min_rows ? ceil_div(sh[i].n, qpt) : 0;
   if (tiles == 0) return MI_OK;
-  constexpr size_t lds = prefill_lds<DK, DV>();
+  constexpr size_t lds = KS2 * prefill_lds<DK, DV>();
+  static_assert(KS2 == 1 || lds >= (size_t)(DV / 16 + 1) * 1024 * 4, "the handed-over sums fit the tiles");
   const float s_max = fixed_reference(a);
   int num_cu = 0;
   { int rc = device_num_cu(&num_cu); if (rc != MI_OK) return rc; }
-  const int fold = tiles * a.g.G <= 2 * num_cu;
-  auto kern = s_max > 0.f ? attn_window_prefill_kernel<DK, DV, NCG, true> : attn_window_prefill_kernel<DK, DV, NCG, false>;
+  const int fold = KS2 == 1 && tiles * a.g.G <= 2 * num_cu;
+  auto kern = s_max > 0.f ? attn_window_prefill_kernel<DK, DV, NCG, KS2, true> : attn_window_prefill_kernel<DK, DV, NCG, KS2, false>;
   if (lds > 64 * 1024) { int rc = ensure_dynamic_lds(reinterpret_cast<const void*>(kern), (int)lds); if (rc != MI_OK) return rc; }
   // kv head fastest: consecutive work-groups (one per XCD) read different heads, a head's tiles meet in one L2
-  hipLaunchKernelGGL(kern, dim3(a.g.G, tiles), dim3(256), lds, s, a, q, kpool, vpool, bs, bt, MB, sd, nseg, out, ldo, s_max, fold, min_rows);
+  hipLaunchKernelGGL(kern, dim3(a.g.G, tiles), dim3(256 * KS2), lds, s, a, q, kpool, vpool, bs, bt, MB, sd, nseg, out, ldo, s_max, fold, min_rows, (bs & (bs - 1)) == 0 ? __builtin_ctz(bs) : -1);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
@@ -631,16 +713,15 @@ int launch_attn_window_prefill(const AttnSpec& a, const uint16_t* q, const uint1
   int rc = check_spec(a, bs);
   if (rc != MI_OK) return rc;
   MI_CHECK(attn_window_supported(a.g) && nseg >= 1 && min_rows >= 2 && ldo >= a.g.H * a.g.dv && ((a.g.dv & 3) != 0 || ldo % 4 == 0), "windowed prefill attention: shape");
-  // a grid that does not give every CU two work-groups takes tiles of half the queries (two waves per SIMD overlap, and light
-  // tiles pair up with heavy ones)
+  // a grid that does not give every CU two work-groups takes tiles of half the queries, and two sets of waves to each
   int num_cu = 0, tiles = 0;
   rc = device_num_cu(&num_cu);
   if (rc != MI_OK) return rc;
   for (int i = 0; i < nseg; ++i) tiles += sh[i].n >= min_rows ? ceil_div(sh[i].n, 128 / (a.g.H / a.g.G)) : 0;
   const bool half = tiles * a.g.G < 2 * num_cu;
 #define MI_CALL_P(DK, DV, NCG) \
-  half ? launch_prefill_t<DK, DV, 1>(a, q, kpool, vpool, bs, bt, MB, sd, sh, nseg, out, ldo, s, min_rows) \
-       : launch_prefill_t<DK, DV, NCG>(a, q, kpool, vpool, bs, bt, MB, sd, sh, nseg, out, ldo, s, min_rows)
+  half ? launch_prefill_t<DK, DV, 1, (DK > 128 || DV > 128 ? 1 : 2)>(a, q, kpool, vpool, bs, bt, MB, sd, sh, nseg, out, ldo, s, min_rows) \
+       : launch_prefill_t<DK, DV, NCG, 1>(a, q, kpool, vpool, bs, bt, MB, sd, sh, nseg, out, ldo, s, min_rows)
   MI_BY_SIZE(MI_CALL_P);
 #undef MI_CALL_P
 }

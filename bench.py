@@ -273,106 +273,193 @@ def speculation_section(torch, HF, wd, plain_ms, steps, k=4):
 # (label, width, q heads, kv heads, head size, Llama intermediate size, layers).  A Vimesun feed-forward has two matrices where
 # a Llama's has three: 1.5 x the intermediate size makes the layers equal in parameters.
 VIMESUN_SIZES = [("1b-like", 2048, 32, 8, 64, 8192, 16), ("8b-like", 4096, 32, 8, 128, 14336, 8)]
-VIMESUN_VOCAB, VIMESUN_WINDOW = 32768, 1024
+STACK_VOCAB, STACK_WINDOW = 32768, 1024
 MFMA_BF16_PEAK_TFLOPS = 2500.0
 
 
-def vimesun_section(args):
-    """Prefill and decode of both models through the same library calls, per kernel class: milliseconds and the fraction of
-    the class's roofline (MFMA flops for GEMM and context attention, HBM bytes for the weight stream, decode attention and
-    the row-wise kernels).  `distance` = Llama's fraction / Vimesun's: how much further from its roofline the class is."""
-    import torch
+class StackBench:
+    """Prefill and decode of a model through the library calls, per kernel class: milliseconds and the fraction of the class's
+    roofline (prefill: MFMA flops, or the weights' bytes where they take longer; decode: HBM bytes of the weight stream and of
+    the attention)."""
 
-    from tests.helpers import decode_inputs, prefill_inputs
-    from vllm_neuron_amd._native import NativeModel
-    from vllm_neuron_amd.models import config_from_dict
-    from vllm_neuron_amd.worker.mi355x_model_loader import _decoder_geometry
-    max_len, mb = 4096, 4096 // BLOCK_SIZE
-    rows_max = 32
-    blocks = [[1 + b * mb + j for j in range(mb)] for b in range(rows_max)]
+    MAX_LEN, ROWS = 4096, 32
+    PREFILL = (512, 2048, 4000)
+    DECODE = ((1, 1024), (4, 1024), (4, 4000), (16, 1024), (32, 1024))
 
-    def build(kind, width, nh, nkv, hd, inter, layers, window):
-        common = dict(num_blocks=1 + rows_max * mb, block_size=BLOCK_SIZE, max_num_seqs=rows_max, max_model_len=max_len,
-                      ctx_buckets=[max_len], device_id=0, use_graphs=1)
-        if kind == "vimesun":
-            layer = {"type": "attention", "mixer": {"heads": nh, "kv_heads": nkv, "dim": hd, "vdim": hd, "mask": {"size": window},
-                                                    "scale": hd ** -0.5}, "mlp": {"kind": "dense", "ff": inter * 3 // 2}}
-            cfg = config_from_dict({"architecture": "Vimesun", "width": width, "vocab": VIMESUN_VOCAB, "layers": [layer] * layers,
-                                    "residual_mult": 0.5, "norm": {"eps": 1e-5}, "max_positions": max_len})
-            m = NativeModel(stack=dict(cfg.stack, compute_dtype=1), **common)
-        else:
-            hf = dict(MODELS["llama31_8b"], hidden_size=width, num_attention_heads=nh, num_key_value_heads=nkv, head_dim=hd,
-                      intermediate_size=inter, num_hidden_layers=layers, vocab_size=VIMESUN_VOCAB)
-            m = NativeModel(weight_dtype=0, quant_type=0, quantize_lm_head=0, tp_degree=1, tp_rank=0,
-                            prefill_fp8_activations=0, **common, **_decoder_geometry(SimpleNamespace(**hf)))
+    def __init__(self, args):
+        self.args = args
+        self.mb = self.MAX_LEN // BLOCK_SIZE
+        self.blocks = [[1 + b * self.mb + j for j in range(self.mb)] for b in range(self.ROWS)]
+
+    def common(self):
+        return dict(num_blocks=1 + self.ROWS * self.mb, block_size=BLOCK_SIZE, max_num_seqs=self.ROWS, max_model_len=self.MAX_LEN,
+                    ctx_buckets=[self.MAX_LEN], device_id=0, use_graphs=1)
+
+    def ready(self, m):
         m.init_synthetic_weights(1, 0.02)
         m.finalize()
         return m
 
-    def keys_seen(first, n, window):          # keys of n consecutive queries
-        return sum(min(i + 1, window) for i in range(first, first + n))
+    def llama(self, width, nh, nkv, hd, inter, layers):
+        from vllm_neuron_amd._native import NativeModel
+        from vllm_neuron_amd.worker.mi355x_model_loader import _decoder_geometry
+        hf = dict(MODELS["llama31_8b"], hidden_size=width, num_attention_heads=nh, num_key_value_heads=nkv, head_dim=hd,
+                  intermediate_size=inter, num_hidden_layers=layers, vocab_size=STACK_VOCAB)
+        return self.ready(NativeModel(weight_dtype=0, quant_type=0, quantize_lm_head=0, tp_degree=1, tp_rank=0,
+                                      prefill_fp8_activations=0, **self.common(), **_decoder_geometry(SimpleNamespace(**hf))))
 
-    out = []
-    for label, width, nh, nkv, hd, inter, layers in VIMESUN_SIZES:
-        per_layer = width * (2 * nh + 2 * nkv) * hd + 3 * width * inter
-        size = {"size": label, "layers": layers, "width": width, "heads": [nh, nkv, hd], "parameters": layers * per_layer + VIMESUN_VOCAB * width,
-                "prefill": [], "decode": []}
-        for kind, window in (("llama", max_len), ("vimesun", max_len), ("vimesun", VIMESUN_WINDOW)):
-            print(f"[bench] {label} {kind} window {window}", file=sys.stderr, flush=True)
-            m = build(kind, width, nh, nkv, hd, inter, layers, window)
-            name = "llama" if kind == "llama" else f"vimesun, {'every key' if window == max_len else f'window {window}'}"
-            for T in (512, 2048, 4000):
-                inp = prefill_inputs([(7 * i + 3) % VIMESUN_VOCAB for i in range(T)], blocks[0], BLOCK_SIZE, max_len, 0)
-                inp["slot_mapping"] = inp["slot_mapping"][:, :T].contiguous()
-                for _ in range(3):
-                    m.forward_tokens(**inp)
-                times = []
-                for _ in range(max(args.steps // 4, 8)):
-                    t = time.perf_counter()
-                    m.forward_tokens(**inp)
-                    times.append(time.perf_counter() - t)
-                m.profile_enable(True)
+    def stack(self, config):
+        from vllm_neuron_amd._native import NativeModel
+        from vllm_neuron_amd.models import config_from_dict
+        return self.ready(NativeModel(stack=dict(config_from_dict(config).stack, compute_dtype=1), **self.common()))
+
+    @staticmethod
+    def keys_seen(n, window):          # keys of the first n queries of a sequence
+        return sum(min(i + 1, window) for i in range(n))
+
+    def prefill(self, m, name, work):
+        """work(T) -> {class: (flops, bytes)}"""
+        from tests.helpers import prefill_inputs
+        rows = []
+        for T in self.PREFILL:
+            inp = prefill_inputs([(7 * i + 3) % STACK_VOCAB for i in range(T)], self.blocks[0], BLOCK_SIZE, self.MAX_LEN, 0)
+            inp["slot_mapping"] = inp["slot_mapping"][:, :T].contiguous()
+            for _ in range(3):
                 m.forward_tokens(**inp)
-                prof = m.profile_read()["ms"]
-                m.profile_enable(False)
-                ms = statistics.median(times) * 1e3
-                flops = {"gemm": 2.0 * T * layers * per_layer, "attn_prefill": 4.0 * layers * nh * hd * keys_seen(0, T, window)}
-                frac = {k: round(f / (prof[k] * 1e-3) / 1e12 / MFMA_BF16_PEAK_TFLOPS, 4) for k, f in flops.items() if prof[k] > 0}
-                size["prefill"].append({"model": name, "tokens": T, "ms": round(ms, 3), "tokens_per_s": round(T / ms * 1e3),
-                                        "class_ms": {k: round(v, 3) for k, v in prof.items() if v}, "mfma_fraction": frac})
-            for B, ctx in ((1, 1024), (4, 1024), (4, 4000), (16, 1024), (32, 1024)):
-                inp = decode_inputs(list(range(1, B + 1)), [ctx - 1] * B, blocks[:B], BLOCK_SIZE, max_len)
-                m.forward(**inp)
-                m.replay_decode(args.warmup)
-                ms = m.replay_decode(args.steps) / args.steps
-                m.profile_enable(True)
-                m.forward(**inp)
-                prof = m.profile_read()
-                m.profile_enable(False)
-                bytes_ = {"gemv": prof["gemv_weight_bytes"], "attn_decode": 4.0 * B * min(ctx, window) * nkv * hd * layers}
-                frac = {k: round(b / (prof["ms"][k] * 1e-3) / 1e9 / HBM_PEAK_GBS, 4) for k, b in bytes_.items() if prof["ms"][k] > 0}
-                gemv = m.replay_decode_classes(args.steps, ["gemv"]) / args.steps
-                attn = m.replay_decode_classes(args.steps, ["attn_decode"]) / args.steps
-                frac_graph = {k: round(b / (t * 1e-3) / 1e9 / HBM_PEAK_GBS, 4) for (k, b), t in zip(bytes_.items(), (gemv, attn)) if t > 0}
-                size["decode"].append({"model": name, "batch": B, "context": ctx, "ms": round(ms, 4), "tokens_per_s": round(B / ms * 1e3),
-                                       "class_ms_in_graph": {"gemv": round(gemv, 4), "attn_decode": round(attn, 4),
-                                                             "rest": round(ms - gemv - attn, 4)},
-                                       "launches": {k: v for k, v in prof["launches"].items() if v},
-                                       "hbm_fraction": frac_graph, "hbm_fraction_eager": frac})
-            m.close()
-        for table, fr in (("prefill", "mfma_fraction"), ("decode", "hbm_fraction")):
+            times = []
+            for _ in range(max(self.args.steps // 4, 8)):
+                t = time.perf_counter()
+                m.forward_tokens(**inp)
+                times.append(time.perf_counter() - t)
+            m.profile_enable(True)
+            m.forward_tokens(**inp)
+            prof = m.profile_read()["ms"]
+            m.profile_enable(False)
+            ms = statistics.median(times) * 1e3
+            frac = {k: round(max(f / MFMA_BF16_PEAK_TFLOPS / 1e12, b / HBM_PEAK_GBS / 1e9) / (prof[k] * 1e-3), 4)
+                    for k, (f, b) in work(T).items() if prof[k] > 0}
+            rows.append({"model": name, "tokens": T, "ms": round(ms, 3), "tokens_per_s": round(T / ms * 1e3),
+                         "class_ms": {k: round(v, 3) for k, v in prof.items() if v}, "roofline_fraction": frac})
+        return rows
+
+    def decode(self, m, name, attn_bytes, extra_gemv_bytes=lambda B: 0.0):
+        """attn_bytes(B, context), extra_gemv_bytes(B): bytes a step must read (the weight stream's own count is the library's)"""
+        from tests.helpers import decode_inputs
+        steps, rows = self.args.steps, []
+        for B, ctx in self.DECODE:
+            inp = decode_inputs([(37 * i + 1) % STACK_VOCAB for i in range(B)], [ctx - 1] * B, self.blocks[:B], BLOCK_SIZE, self.MAX_LEN)
+            m.forward(**inp)
+            m.replay_decode(self.args.warmup)
+            ms = m.replay_decode(steps) / steps
+            m.profile_enable(True)
+            m.forward(**inp)
+            prof = m.profile_read()
+            m.profile_enable(False)
+            bytes_ = {"gemv": prof["gemv_weight_bytes"] + extra_gemv_bytes(B), "attn_decode": attn_bytes(B, ctx)}
+            frac = {k: round(b / (prof["ms"][k] * 1e-3) / 1e9 / HBM_PEAK_GBS, 4) for k, b in bytes_.items() if prof["ms"][k] > 0}
+            gemv = m.replay_decode_classes(steps, ["gemv"]) / steps
+            attn = m.replay_decode_classes(steps, ["attn_decode"]) / steps
+            frac_graph = {k: round(b / (t * 1e-3) / 1e9 / HBM_PEAK_GBS, 4) for (k, b), t in zip(bytes_.items(), (gemv, attn)) if t > 0}
+            rows.append({"model": name, "batch": B, "context": ctx, "ms": round(ms, 4), "tokens_per_s": round(B / ms * 1e3),
+                         "class_ms_in_graph": {"gemv": round(gemv, 4), "attn_decode": round(attn, 4), "rest": round(ms - gemv - attn, 4)},
+                         "launches": {k: v for k, v in prof["launches"].items() if v},
+                         "hbm_fraction": frac_graph, "hbm_fraction_eager": frac})
+        return rows
+
+    @staticmethod
+    def compare(size, window):
+        """tokens/s and `distance` (how much further from its roofline a class is) against the Llama of the size"""
+        for table, fr in (("prefill", "roofline_fraction"), ("decode", "hbm_fraction")):
             base = {(r.get("tokens"), r.get("batch"), r.get("context")): r for r in size[table] if r["model"] == "llama"}
             for r in size[table]:
                 if r["model"] == "llama":
                     continue
                 b = base[r.get("tokens"), r.get("batch"), r.get("context")]
                 r["vs_llama_tokens_per_s"] = round(r["tokens_per_s"] / b["tokens_per_s"], 3)
-                if "window" in r["model"] and r.get("context", 0) > VIMESUN_WINDOW:     # the Llama step that reads as many keys
-                    b = base[None, r["batch"], VIMESUN_WINDOW]
+                if "window" in r["model"] and r.get("context", 0) > window:     # the Llama step that reads as many keys
+                    b = base[None, r["batch"], window]
                 r["distance"] = {k: round(b[fr][k] / v, 2) for k, v in r[fr].items() if k in b[fr] and v > 0}
+
+    def line(self, design, sizes):
+        print(json.dumps({"metric": f"{design} prefill / decode beside a Llama of equal size", "dtype": "bf16", "data": "synthetic",
+                          "higher_is_better": True, "steps": self.args.steps, "warmup": self.args.warmup, "n_gpus": 1, "sizes": sizes}),
+              flush=True)
+
+
+def vimesun_section(args):
+    bench, out = StackBench(args), []
+    every = bench.MAX_LEN
+    for label, width, nh, nkv, hd, inter, layers in VIMESUN_SIZES:
+        per_layer = width * (2 * nh + 2 * nkv) * hd + 3 * width * inter
+        size = {"size": label, "layers": layers, "width": width, "heads": [nh, nkv, hd], "parameters": layers * per_layer + STACK_VOCAB * width,
+                "prefill": [], "decode": []}
+        for kind, window in (("llama", every), ("vimesun", every), ("vimesun", STACK_WINDOW)):
+            print(f"[bench] {label} {kind} window {window}", file=sys.stderr, flush=True)
+            if kind == "llama":
+                m, name = bench.llama(width, nh, nkv, hd, inter, layers), "llama"
+            else:
+                layer = {"type": "attention", "mixer": {"heads": nh, "kv_heads": nkv, "dim": hd, "vdim": hd, "mask": {"size": window},
+                                                        "scale": hd ** -0.5}, "mlp": {"kind": "dense", "ff": inter * 3 // 2}}
+                m = bench.stack({"architecture": "Vimesun", "width": width, "vocab": STACK_VOCAB, "layers": [layer] * layers,
+                                 "residual_mult": 0.5, "norm": {"eps": 1e-5}, "max_positions": every})
+                name = f"vimesun, {'every key' if window == every else f'window {window}'}"
+            size["prefill"] += bench.prefill(m, name, lambda T: {
+                "gemm": (2.0 * T * layers * per_layer, 2.0 * layers * per_layer),
+                "attn_prefill": (4.0 * layers * nh * hd * bench.keys_seen(T, window), 0.0)})
+            size["decode"] += bench.decode(m, name, lambda B, ctx: 4.0 * B * min(ctx, window) * nkv * hd * layers)
+            m.close()
+        bench.compare(size, STACK_WINDOW)
         out.append(size)
-    print(json.dumps({"metric": "Vimesun prefill / decode beside a Llama of equal size", "dtype": "bf16", "data": "synthetic",
-                      "higher_is_better": True, "steps": args.steps, "warmup": args.warmup, "n_gpus": 1, "sizes": out}), flush=True)
+    bench.line("Vimesun", out)
+
+
+# ---- --rapodra: the latent-attention design beside a Llama of equal size ------------------------------------------------------
+# (label, width, latent heads of 128, latent rank, Llama q heads, kv heads, head size, Llama intermediate size, layers).  The dense
+# feed-forward makes the layers equal in parameters; the mixture (64 experts, 8 per token) makes them equal in what a token uses.
+RAPODRA_SIZES = [("2b-like", 2048, 16, 512, 32, 8, 64, 8192, 8), ("8b-like", 4096, 32, 512, 32, 8, 128, 14336, 4)]
+RAPODRA_EXPERTS, RAPODRA_TOP, RAPODRA_DIM = 64, 8, 128
+
+
+def rapodra_section(args):
+    bench, out = StackBench(args), []
+    every, E, top, dim = bench.MAX_LEN, RAPODRA_EXPERTS, RAPODRA_TOP, RAPODRA_DIM
+    for label, width, H, rank, nh, nkv, hd, inter, layers in RAPODRA_SIZES:
+        per_layer = width * (2 * nh + 2 * nkv) * hd + 3 * width * inter
+        proj = width * (H * dim + rank) + H * dim * width             # queries, latent, output
+        ff = (per_layer - proj - 2 * rank * H * dim) // (3 * width) // 512 * 512
+        size = {"size": label, "layers": layers, "width": width, "latent heads": [H, dim, rank], "ff": ff,
+                "experts": [E, top, ff // top], "llama heads": [nh, nkv, hd], "llama parameters": layers * per_layer + STACK_VOCAB * width,
+                "prefill": [], "decode": []}
+        for kind, window in (("llama", every), ("dense", every), ("dense", STACK_WINDOW), ("experts", STACK_WINDOW)):
+            print(f"[bench] {label} {kind} window {window}", file=sys.stderr, flush=True)
+            if kind == "llama":
+                m, name = bench.llama(width, nh, nkv, hd, inter, layers), "llama"
+                size["prefill"] += bench.prefill(m, name, lambda T: {
+                    "gemm": (2.0 * T * layers * per_layer, 2.0 * layers * per_layer),
+                    "attn_prefill": (4.0 * layers * nh * hd * bench.keys_seen(T, window), 0.0)})
+                size["decode"] += bench.decode(m, name, lambda B, ctx: 4.0 * B * min(ctx, window) * nkv * hd * layers)
+            else:
+                mlp = ({"kind": "dense", "ff": ff, "limit": 7.0} if kind == "dense" else
+                       {"kind": "moe", "router": {"experts": E, "top": top}, "expert": {"ff": ff // top}})
+                layer = {"type": "latent_attention", "mixer": {"heads": H, "dim": dim, "vdim": dim, "kv_rank": rank, "mask": {"size": window},
+                                                               "scale": dim ** -0.5}, "mlp": mlp}
+                m = bench.stack({"architecture": "Rapodra", "width": width, "vocab": STACK_VOCAB, "layers": [layer] * layers,
+                                 "canon": {"taps": 4}, "norm": {"eps": 1e-5, "groups": 4}, "logit_softcap": 30.0})
+                name = f"rapodra {kind}, {'every key' if window == every else f'window {window}'}"
+                router = E * width if kind == "experts" else 0
+                common = proj + 2 * rank * H * dim + router
+                # (experts: the expected number of different ones among B rows' choices)
+                hit = lambda B: E * (1 - (1 - top / E) ** B) if kind == "experts" else 0.0
+                size["prefill"] += bench.prefill(m, name, lambda T: {
+                    "gemm": (2.0 * T * layers * (common + 3 * width * ff),
+                             2.0 * layers * (common + 3 * width * (hit(T) * (ff // top) if kind == "experts" else ff))),
+                    "attn_prefill": (4.0 * layers * H * dim * bench.keys_seen(T, window), 0.0)})
+                size["decode"] += bench.decode(m, name, lambda B, ctx: 2.0 * layers * (B * min(ctx, window) * rank + rank * H * dim),
+                                               lambda B: 2.0 * layers * hit(B) * 3 * width * (ff // top))
+            m.close()
+        bench.compare(size, STACK_WINDOW)
+        out.append(size)
+    bench.line("Rapodra", out)
 
 
 def main():
@@ -391,9 +478,14 @@ def main():
                     help="dev: place every rank shard of --gpus N on GPU 0 (functional check of the TP path on one GPU)")
     ap.add_argument("--vimesun", action="store_true",
                     help="instead of the headline workload: the Vimesun layer stack beside a Llama of equal size, both bf16")
+    ap.add_argument("--rapodra", action="store_true",
+                    help="instead of the headline workload: Rapodra (latent attention; dense and expert feed-forwards) beside a Llama "
+                         "of equal size, all bf16")
     args = ap.parse_args()
     if args.vimesun:
         return vimesun_section(args)
+    if args.rapodra:
+        return rapodra_section(args)
     wd = args.weight_dtype or ("int8" if args.model == "qwen25_7b" else "f8e4m3")
     HF = MODELS[args.model]
 

@@ -7,7 +7,7 @@ namespace {
 
 constexpr int kMaxTop = 64, kRouteExperts = 8;
 
-// ---- router: one work-group per row; a wave takes every fourth expert ----------------------------------------------------
+// ---- router ----------------------------------------------------
 __device__ __forceinline__ float dot8(const uint16_t* w, const float* x) {
   const uint4 v = *reinterpret_cast<const uint4*>(w);
   float a = bf16lo_to_f32(v.x) * x[0];
@@ -101,28 +101,37 @@ __device__ __forceinline__ void pick_top(float* z, int E, int top, int32_t* ids,
   if (lane < top) { ids[lane] = mine_id; weights[lane] = mine / sum; }
 }
 
+// one work-group per row and kRouteExperts experts, or (no tickets) per row; a wave takes two experts at a time, their rows and x
+// requested together
 template <typename T>
 __global__ __launch_bounds__(256) void route_kernel(const T* __restrict__ x, int ldx, const T* __restrict__ w, const float* __restrict__ b, int E,
-                                                    int K, int top, int32_t* __restrict__ ids, float* __restrict__ weights, float* __restrict__ zg,
-                                                    uint32_t* __restrict__ tickets) {
+                                                        int K, int top, int32_t* __restrict__ ids, float* __restrict__ weights, float* __restrict__ zg,
+                                                        uint32_t* __restrict__ tickets) {
+  constexpr int NW = 4, EPW = 2;
   extern __shared__ __attribute__((aligned(16))) float z[];   // E floats + 4
   __shared__ uint32_t arrived;
   const int e0 = blockIdx.y * kRouteExperts, e1 = tickets ? min(e0 + kRouteExperts, E) : E;
   const int t = blockIdx.x, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
-  for (int e = e0 + wave * 2; e < e1; e += 8) {       // two experts at a time, their rows and x requested together
-    float a0 = 0.f, a1 = 0.f;
-    const T *w0 = w + (size_t)e * K, *w1 = w + (size_t)min(e + 1, e1 - 1) * K;
+  for (int e = e0 + wave * EPW; e < e1; e += NW * EPW) {
+    float a[EPW];
+    const T* we[EPW];
+#pragma unroll
+    for (int i = 0; i < EPW; ++i) { a[i] = 0.f; we[i] = w + (size_t)min(e + i, e1 - 1) * K; }
 #pragma unroll 4
     for (int k = lane * 8; k < K; k += 512) {
       float xv[8];
       load8f(x + (size_t)t * ldx + k, xv);
-      a0 += dot8(w0 + k, xv);
-      a1 += dot8(w1 + k, xv);
+#pragma unroll
+      for (int i = 0; i < EPW; ++i) a[i] += dot8(we[i] + k, xv);
     }
-    a0 = wave_sum(a0);
-    a1 = wave_sum(a1);
-    if (lane >= 2 || e + lane >= e1) continue;
-    const float v = (lane ? a1 : a0) + b[e + lane];
+    float v = 0.f;
+#pragma unroll
+    for (int i = 0; i < EPW; ++i) {
+      const float s = wave_sum(a[i]);
+      v = lane == i ? s : v;
+    }
+    if (lane >= EPW || e + lane >= e1) continue;
+    v += b[e + lane];
     if (tickets) __hip_atomic_store(zg + (size_t)t * E + e + lane, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
     else z[e + lane] = v;
   }
@@ -132,7 +141,7 @@ __global__ __launch_bounds__(256) void route_kernel(const T* __restrict__ x, int
     if (tid == 0) arrived = __hip_atomic_fetch_add(tickets + t, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
     __syncthreads();
     if (arrived != gridDim.y - 1) return;
-    for (int e = tid; e < E; e += 256) z[e] = __hip_atomic_load(zg + (size_t)t * E + e, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    for (int e = tid; e < E; e += NW * 64) z[e] = __hip_atomic_load(zg + (size_t)t * E + e, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
     if (tid == 0) __hip_atomic_store(tickets + t, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
   }
   __syncthreads();
@@ -287,7 +296,7 @@ __global__ __launch_bounds__(1024) void experts_sort_kernel(const int32_t* __res
 
 // 128 weight rows x BM pairs per work-group, four waves; pairs' rows through swizzled LDS, weights from their tiled image
 template <int BM, bool GLU>
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) void experts_gemm_kernel(
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(BM == 64 ? 4 : 2, BM == 64 ? 4 : 2))) void experts_gemm_kernel(
     const uint4* __restrict__ w, int NT, int KT, ExpertPlan plan, const uint16_t* __restrict__ x, int ldx, int x_div, uint16_t* __restrict__ y, int ldy) {
   constexpr int WM = BM / 64, WN = 4 / WM, NTW = 8 / WN, XL = BM / 32;
   __shared__ __attribute__((aligned(16))) u32x4_t xs[BM * 8];

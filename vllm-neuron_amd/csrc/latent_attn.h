@@ -15,9 +15,10 @@ struct LatentGeom {
   int dkp = 0, dvp = 0, rp = 0;      // padded to 32
 };
 // qd [T, ldq] fp32 (q heads, then the latent's projection where c_norm is given) -> q [T, H, dkp]; latent over its root mean
-// square times c_norm [rank] into the pool at slots (-1: not written)
+// square times c_norm [rank] into the pool at slots (-1: not written).  slabs (slabs->slab): the projection as a K-split of row
+// stride ldq that is not summed yet, instead of qd
 int launch_latent_scatter(const float* qd, int ldq, int T, const LatentGeom& g, const float* c_norm, float eps, const int32_t* slots,
-                          int block_size, void* q, void* pool, bool f32, hipStream_t s);
+                          int block_size, void* q, void* pool, bool f32, hipStream_t s, const SlabSum* slabs = nullptr);
 // token generation: qa [rows, H, rp] = W_uk^T q (bf16) from the same projection, and the latents' scatter, in one launch
 inline bool latent_token_supported(const LatentGeom& g) { return g.dk % 4 == 0; }
 int launch_latent_token(const float* qd, int ldq, int rows, const LatentGeom& g, const void* w_uk, const float* c_norm, float eps, const int32_t* slots,

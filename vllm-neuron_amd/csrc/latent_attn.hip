@@ -8,13 +8,35 @@ namespace {
 __device__ __forceinline__ void put4(uint16_t* p, float4 v) { *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf16x2(v.x, v.y), pack_bf16x2(v.z, v.w)); }
 __device__ __forceinline__ void put4(float* p, float4 v) { *reinterpret_cast<float4*>(p) = v; }
 
-// one latent over its root mean square times c_norm, into its pool row; 256 threads
+// the projection's row t: summed, or slabs of a K-split still to be summed (slice order, as splitk_reduce does)
+struct QdRow {
+  const float* p;
+  const SlabSum& sl;
+  __device__ __forceinline__ float at(int c) const {
+    if (!sl.slab) return p[c];
+    float v = 0.f;
+    for (int z = 0; z < sl.KS; ++z) v += p[(size_t)z * sl.T * sl.N + c];
+    return v * sl.scale[c];
+  }
+  __device__ __forceinline__ float4 at4(int c) const {      // c % 4 == 0
+    float4 v = *reinterpret_cast<const float4*>(p + c);
+    if (!sl.slab) return v;
+    for (int z = 1; z < sl.KS; ++z) {
+      const float4 q = *reinterpret_cast<const float4*>(p + (size_t)z * sl.T * sl.N + c);
+      v.x += q.x; v.y += q.y; v.z += q.z; v.w += q.w;
+    }
+    const float4 s = *reinterpret_cast<const float4*>(sl.scale + c);
+    return make_float4(v.x * s.x, v.y * s.y, v.z * s.z, v.w * s.w);
+  }
+};
+
+// one latent (columns c0 .. of the row) over its root mean square times c_norm, into its pool row; 256 threads
 template <typename T>
-__device__ __forceinline__ void latent_norm_row(const float* __restrict__ src, const LatentGeom& g, const float* __restrict__ c_norm, float eps, int slot,
+__device__ __forceinline__ void latent_norm_row(const QdRow& row, int c0, const LatentGeom& g, const float* __restrict__ c_norm, float eps, int slot,
                                                 T* __restrict__ pool, float* red) {
   const int tid = threadIdx.x;
   float ss = 0.f;
-  for (int d = tid; d < g.rank; d += 256) ss = __builtin_fmaf(src[d], src[d], ss);
+  for (int d = tid; d < g.rank; d += 256) { const float v = row.at(c0 + d); ss = __builtin_fmaf(v, v, ss); }
   ss = wave_sum(ss);
   if ((tid & 63) == 0) red[tid >> 6] = ss;
   __syncthreads();
@@ -22,39 +44,40 @@ __device__ __forceinline__ void latent_norm_row(const float* __restrict__ src, c
   if (slot < 0) return;
   T* dst = pool + (size_t)slot * g.rp;        // (a block's rows are consecutive: slot = block * block_size + offset)
   for (int d = tid * 4; d < g.rp; d += 1024) {
-    auto at = [&](int i) { return d + i < g.rank ? src[d + i] * f * c_norm[d + i] : 0.f; };
+    auto at = [&](int i) { return d + i < g.rank ? row.at(c0 + d + i) * f * c_norm[d + i] : 0.f; };
     put4(dst + d, make_float4(at(0), at(1), at(2), at(3)));
   }
 }
 
 // blockIdx.y < q groups: 8 heads of 32 lanes each; the last one: the latent, one work-group per row
 template <typename T>
-__global__ __launch_bounds__(256) void latent_scatter_kernel(const float* __restrict__ qd, int ldq, LatentGeom g, const float* __restrict__ c_norm,
+__global__ __launch_bounds__(256) void latent_scatter_kernel(const float* __restrict__ qd, int ldq, SlabSum sl, LatentGeom g, const float* __restrict__ c_norm,
                                                              float eps, const int32_t* __restrict__ slots, int bs, T* __restrict__ q,
                                                              T* __restrict__ pool) {
   __shared__ float red[4];
   const int t = blockIdx.x, tid = threadIdx.x;
+  const QdRow row{sl.slab ? sl.slab + (size_t)t * sl.N : qd + (size_t)t * ldq, sl};
   if ((int)blockIdx.y < ceil_div(g.H, 8)) {
     const int h = blockIdx.y * 8 + (tid >> 5);
     if (h >= g.H) return;
-    const float* src = qd + (size_t)t * ldq + (size_t)h * g.dk;
+    const int c0 = h * g.dk;
     T* dst = q + ((size_t)t * g.H + h) * g.dkp;
     const bool vec = (g.dk & 3) == 0;
     for (int d = (tid & 31) * 4; d < g.dkp; d += 128) {
       float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
       if (vec) {
-        if (d < g.dk) v = *reinterpret_cast<const float4*>(src + d);
+        if (d < g.dk) v = row.at4(c0 + d);
       } else {
-        if (d < g.dk) v.x = src[d];
-        if (d + 1 < g.dk) v.y = src[d + 1];
-        if (d + 2 < g.dk) v.z = src[d + 2];
-        if (d + 3 < g.dk) v.w = src[d + 3];
+        if (d < g.dk) v.x = row.at(c0 + d);
+        if (d + 1 < g.dk) v.y = row.at(c0 + d + 1);
+        if (d + 2 < g.dk) v.z = row.at(c0 + d + 2);
+        if (d + 3 < g.dk) v.w = row.at(c0 + d + 3);
       }
       put4(dst + d, v);
     }
     return;
   }
-  latent_norm_row(qd + (size_t)t * ldq + (size_t)g.H * g.dk, g, c_norm, eps, slots[t], pool, red);
+  latent_norm_row(row, g.H * g.dk, g, c_norm, eps, slots[t], pool, red);
 }
 
 struct RowAt { int row, seq; };
@@ -108,7 +131,8 @@ __global__ __launch_bounds__(256) void latent_token_kernel(const float* __restri
   __shared__ float red[4];
   const int h = blockIdx.y;
   if (h == g.H) {
-    if ((int)blockIdx.x < rows) latent_norm_row(qd + (size_t)blockIdx.x * ldq + (size_t)g.H * g.dk, g, c_norm, eps, slots[blockIdx.x], pool, red);
+    const SlabSum none;
+    if ((int)blockIdx.x < rows) latent_norm_row(QdRow{qd + (size_t)blockIdx.x * ldq, none}, g.H * g.dk, g, c_norm, eps, slots[blockIdx.x], pool, red);
     return;
   }
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, g4 = lane >> 4, c = lane & 15;
@@ -250,12 +274,35 @@ __global__ __launch_bounds__(256, HG == 1 ? 2 : 1) void latent_rows_kernel(Laten
     f32x4_t st[HG];
 #pragma unroll
     for (int hg = 0; hg < HG; ++hg) st[hg] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    {   // fragments requested kAhead MFMAs ahead of their use
+      constexpr int kAhead = KS < 8 ? KS : 8;
+      bf16x8_t kf[KS];
+      auto kread = [&](int ks) { kf[ks] = *reinterpret_cast<const bf16x8_t*>(&Cs[(16 * wave + c) * CP + ks * 32 + g4 * 8]); };
 #pragma unroll
-    for (int ks = 0; ks < KS; ++ks) {
-      const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(&Cs[(16 * wave + c) * CP + ks * 32 + g4 * 8]);
+      for (int ks = 0; ks < kAhead; ++ks) kread(ks);
+      f32x4_t s2[HG];                    // two chains of sums, added at the end
 #pragma unroll
-      for (int hg = 0; hg < HG; ++hg)
-        st[hg] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, __builtin_bit_cast(bf16x8_t, HG == 1 ? qr[ks] : Qs[(hg * KS + ks) * 64 + lane]), st[hg], 0, 0, 0);
+      for (int hg = 0; hg < HG; ++hg) s2[hg] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int ks = 0; ks < KS; ++ks) {
+#pragma unroll
+        for (int hg = 0; hg < HG; ++hg) {
+          const bf16x8_t qf = __builtin_bit_cast(bf16x8_t, HG == 1 ? qr[ks] : Qs[(hg * KS + ks) * 64 + lane]);
+          if (ks & 1) s2[hg] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[ks], qf, s2[hg], 0, 0, 0);
+          else st[hg] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[ks], qf, st[hg], 0, 0, 0);
+        }
+        if (ks + kAhead < KS) kread(ks + kAhead);
+      }
+      if constexpr (HG == 1) {
+        __builtin_amdgcn_sched_group_barrier(0x100, kAhead, 0);
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) {
+          __builtin_amdgcn_sched_group_barrier(0x8, 1, 0);
+          if (ks + kAhead < KS) __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
+        }
+      }
+#pragma unroll
+      for (int hg = 0; hg < HG; ++hg) { st[hg][0] += s2[hg][0]; st[hg][1] += s2[hg][1]; st[hg][2] += s2[hg][2]; st[hg][3] += s2[hg][3]; }
     }
     const int j0 = tt * 64 + 16 * wave + 4 * g4;
 #pragma unroll
@@ -290,22 +337,30 @@ __global__ __launch_bounds__(256, HG == 1 ? 2 : 1) void latent_rows_kernel(Laten
 #pragma unroll
       for (int dn = 0; dn < DN; ++dn) { acc[hg][dn][0] *= alpha[hg]; acc[hg][dn][1] *= alpha[hg]; acc[hg][dn][2] *= alpha[hg]; acc[hg][dn][3] *= alpha[hg]; }
     // the k-slot (g4, j) of a 32-key half is key (j < 4 ? 4 g4 + j : 16 + 4 g4 + j - 4)
+    bf16x8_t pf[2][HG];
 #pragma unroll
-    for (int hf = 0; hf < 2; ++hf) {
-      bf16x8_t pf[HG];
+    for (int hf = 0; hf < 2; ++hf)
 #pragma unroll
       for (int hg = 0; hg < HG; ++hg) {
         const uint2 a = Ps[(hg * 4 + 2 * hf) * 64 + lane], b = Ps[(hg * 4 + 2 * hf + 1) * 64 + lane];
-        pf[hg] = __builtin_bit_cast(bf16x8_t, u32x4_t{a.x, a.y, b.x, b.y});
+        pf[hf][hg] = __builtin_bit_cast(bf16x8_t, u32x4_t{a.x, a.y, b.x, b.y});
       }
+    {
+      constexpr int NPV = 2 * DN, kAhead = NPV < 6 ? NPV : 6;
+      s16x4_t vlo[NPV], vhi[NPV];
+      auto vread = [&](int i) {
+        const uint16_t* r0 = &Cs[(32 * (i / DN) + 4 * g4 + tr_row) * CP + d_w + 16 * (i % DN) + tr_col];
+        vlo[i] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4_t __attribute__((address_space(3)))*)r0);
+        vhi[i] = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4_t __attribute__((address_space(3)))*)(r0 + 16 * CP));
+      };
 #pragma unroll
-      for (int dn = 0; dn < DN; ++dn) {
-        const uint16_t* r0 = &Cs[(32 * hf + 4 * g4 + tr_row) * CP + d_w + 16 * dn + tr_col];
-        const s16x4_t l4 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4_t __attribute__((address_space(3)))*)r0);
-        const s16x4_t h4 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4_t __attribute__((address_space(3)))*)(r0 + 16 * CP));
-        const bf16x8_t av = {l4[0], l4[1], l4[2], l4[3], h4[0], h4[1], h4[2], h4[3]};
+      for (int i = 0; i < kAhead; ++i) vread(i);
 #pragma unroll
-        for (int hg = 0; hg < HG; ++hg) acc[hg][dn] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(av, pf[hg], acc[hg][dn], 0, 0, 0);
+      for (int i = 0; i < NPV; ++i) {
+        const bf16x8_t av = {vlo[i][0], vlo[i][1], vlo[i][2], vlo[i][3], vhi[i][0], vhi[i][1], vhi[i][2], vhi[i][3]};
+#pragma unroll
+        for (int hg = 0; hg < HG; ++hg) acc[hg][i % DN] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(av, pf[i / DN][hg], acc[hg][i % DN], 0, 0, 0);
+        if (i + kAhead < NPV) vread(i + kAhead);
       }
     }
   }
@@ -453,12 +508,14 @@ int launch_rows_t(const LatentGeom& g, float scale, int window, const uint16_t* 
 }  // namespace
 
 int launch_latent_scatter(const float* qd, int ldq, int T, const LatentGeom& g, const float* c_norm, float eps, const int32_t* slots,
-                          int bs, void* q, void* pool, bool f32, hipStream_t s) {
+                          int bs, void* q, void* pool, bool f32, hipStream_t s, const SlabSum* slabs) {
+  const SlabSum sl = slabs ? *slabs : SlabSum();
+  MI_CHECK(!sl.slab || (sl.T == T && sl.N == ldq && !sl.bias && !sl.row_scale), "latent scatter: pending K-split sum of another shape");
   MI_CHECK(T >= 1 && ldq % 4 == 0 && ldq >= g.H * g.dk + (c_norm ? g.rank : 0) && g.dkp >= g.dk && g.dkp % 32 == 0 && g.rp >= g.rank && g.rp % 32 == 0 && bs > 0,
            "latent scatter: geometry");
   const dim3 grid(T, ceil_div(g.H, 8) + (c_norm ? 1 : 0));
-  if (f32) hipLaunchKernelGGL((latent_scatter_kernel<float>), grid, dim3(256), 0, s, qd, ldq, g, c_norm, eps, slots, bs, (float*)q, (float*)pool);
-  else hipLaunchKernelGGL((latent_scatter_kernel<uint16_t>), grid, dim3(256), 0, s, qd, ldq, g, c_norm, eps, slots, bs, (uint16_t*)q, (uint16_t*)pool);
+  if (f32) hipLaunchKernelGGL((latent_scatter_kernel<float>), grid, dim3(256), 0, s, qd, ldq, sl, g, c_norm, eps, slots, bs, (float*)q, (float*)pool);
+  else hipLaunchKernelGGL((latent_scatter_kernel<uint16_t>), grid, dim3(256), 0, s, qd, ldq, sl, g, c_norm, eps, slots, bs, (uint16_t*)q, (uint16_t*)pool);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }

@@ -759,18 +759,19 @@ int latent_mixer(mi_ctx* c, const StackLayer& W, size_t kv_at, const Batch& b, R
   const LatentGeom& g = W.lg;
   hipStream_t s = c->stream;
   EpiArgs e{};
-  e.out_f32 = S->qkv_out; e.ld_out = S->qkv_ld;
-  MI_TRY(apply(c, W.qkv, b.rows, S->n1, S->Kd, EPI_F32, e));
+  e.out_f32 = S->qkv_out; e.ld_out = W.qkv.N;
+  SlabSum slabs;       // (many rows: a K-split's sum is left to the scatter)
+  MI_TRY(apply(c, W.qkv, b.rows, S->n1, S->Kd, EPI_F32, e, b.rows >= 384 ? &slabs : nullptr));
   unsigned char* pool = reinterpret_cast<unsigned char*>(c->kv_pool) + kv_at * S->elem();
   if (b.decode && W.fast() && latent_token_supported(g)) {
     if (runs_other(c)) {
       Scope sc(c, MI_K_OTHER);
-      MI_TRY(launch_latent_token(S->qkv_out, S->qkv_ld, b.rows, g, W.w_uk, W.c_norm, S->cfg.norm_eps, c->d_slots, reinterpret_cast<uint16_t*>(S->qa),
+      MI_TRY(launch_latent_token(S->qkv_out, W.qkv.N, b.rows, g, W.w_uk, W.c_norm, S->cfg.norm_eps, c->d_slots, reinterpret_cast<uint16_t*>(S->qa),
                                  reinterpret_cast<uint16_t*>(pool), s));
     }
   } else if (runs_other(c)) {
     Scope sc(c, MI_K_OTHER);
-    MI_TRY(launch_latent_scatter(S->qkv_out, S->qkv_ld, b.rows, g, W.c_norm, S->cfg.norm_eps, c->d_slots, k.block_size, S->q, pool, S->f32, s));
+    MI_TRY(launch_latent_scatter(S->qkv_out, W.qkv.N, b.rows, g, W.c_norm, S->cfg.norm_eps, c->d_slots, k.block_size, S->q, pool, S->f32, s, &slabs));
   }
   MI_TRY(W.fast() ? latent_attention(c, W, reinterpret_cast<const uint16_t*>(pool), b) : latent_attention_plain(c, W, pool, b));
   EpiArgs o{};

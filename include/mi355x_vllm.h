@@ -142,6 +142,7 @@ typedef struct mi_stack_config {
   int32_t block_kind, norm_groups;
   int32_t conv_taps;       /* sandwich blocks: 1 .. 16 */
   float logit_softcap;     /* 0 = none */
+  int32_t state_lookahead; /* sandwich blocks: a step may write this many positions behind the last accepted one (speculation: k - 1) */
 } mi_stack_config;
 
 const char* mi_last_error(void);

@@ -110,15 +110,12 @@ def test_logits_of_a_prefix_do_not_depend_on_what_follows(case):
     assert torch.allclose(a[:41], b, atol=1e-9)
 
 
-def test_speculation_is_refused_at_load():
-    from vllm_neuron_amd.worker.mi355x_model_loader import check_speculation
-    stack = stack_of(config_from_dict(CASES["uneven"]()))
+def test_a_draft_with_convolution_state_is_refused():
+    from vllm_neuron_amd.worker.mi355x_model_loader import check_draft
     with pytest.raises(NotImplementedError, match="convolution"):
-        check_speculation(stack, None)
-    with pytest.raises(NotImplementedError, match="convolution"):
-        check_speculation(None, stack)
-    check_speculation(None, None)
-    check_speculation(stack_of(config_from_dict(CASES["wide"]())), None)      # one tap: no state
+        check_draft(stack_of(config_from_dict(CASES["uneven"]())))
+    check_draft(None)
+    check_draft(stack_of(config_from_dict(CASES["wide"]())))      # one tap: no state
 
 
 # ---- the GPU tests' cases show a mistake in any mechanism (the mistakes are planted here, in the oracle) -------------

@@ -305,7 +305,7 @@ def test_far_key_of_a_long_context(lib, f32, path):
 
 # ---- router and experts ----------------------------------------------------------------------------------------------------
 @pytest.mark.parametrize("f32,path", [(1, 1), (0, 1), (0, 2)])
-@pytest.mark.parametrize("T,D,E,top,ff", [(1, 64, 4, 1, 16), (5, 120, 7, 3, 22), (32, 320, 64, 8, 40), (3, 1024, 200, 5, 64), (150, 192, 6, 6, 72),
+@pytest.mark.parametrize("T,D,E,top,ff", [(1, 64, 4, 1, 16), (5, 120, 7, 3, 22), (32, 320, 64, 8, 40), (3, 1024, 300, 5, 64), (150, 192, 6, 6, 72),
                                           (700, 128, 12, 2, 130)])
 def test_router_and_experts(lib, T, D, E, top, ff, f32, path):
     g = torch.Generator().manual_seed(T + E)
@@ -591,7 +591,59 @@ def test_batch_line_kv_layout():
     eng.close()
 
 
-def test_speculation_is_refused():
+@pytest.mark.parametrize("k,max_len", [(3, 128), (5, 48)])
+def test_speculation_yields_the_greedy_text(k, max_len):
+    """Candidates of a step are segments of k tokens: rejected ones leave latents and convolution inputs behind that the next
+    step must not see.  The draft is the target without the convolutions' past, right about half of the time.  max_len 48:
+    sequences end at the model length, inside a speculation window."""
+    import copy
+    from types import SimpleNamespace
+
+    from vllm_neuron_amd._vllm_compat import SamplingParams, SimpleSpeculativeConfig
+    from vllm_neuron_amd.engine import MI355XEngine
+    from vllm_neuron_amd.models import config_from_dict
+    cfg, w = case("uneven")
+    w = dict(w)
+    for name in w:
+        if "canon" in name:
+            w[name] = torch.cat([w[name][:, :-1] * 0.35, w[name][:, -1:]], 1)
+    small = copy.deepcopy(cfg)
+    small["canon"]["taps"] = 1
+    wd = {n: (t[:, -1:].contiguous() if "canon" in n else t) for n, t in w.items()}
+    spec = SimpleSpeculativeConfig(num_speculative_tokens=k, draft_model_config=SimpleNamespace(model="", hf_config=config_from_dict(small)))
+    eng = MI355XEngine(config_from_dict(cfg), dtype="float32", max_model_len=max_len, max_num_seqs=2, block_size=16, speculative_config=spec,
+                       override_mi355x_config={"state_dict": w, "draft_state_dict": wd})
+    prompts = [torch.randint(0, 203, (n,), generator=torch.Generator().manual_seed(n)).tolist() for n in (30, 12)]
+    ids = [eng.add_request(p, SamplingParams(temperature=0.0, max_tokens=30)) for p in prompts]
+    steps = 0
+    while eng.has_unfinished_requests():
+        eng.step()
+        steps += 1
+    texts = [eng.outputs[i].token_ids for i in ids]
+    assert texts == [greedy(cfg, w, p, min(30, max_len - len(p))) for p in prompts]
+    assert steps < 0.85 * max(map(len, texts)) + 2, steps           # some candidates were accepted ...
+    assert steps > max(map(len, texts)) / k + 2, steps               # ... and some were not
+    eng.close()
+
+
+def test_speculation_with_an_accepting_draft():
+    """A model without state (one tap) as its own draft: every candidate is accepted."""
+    from types import SimpleNamespace
+
+    from vllm_neuron_amd._vllm_compat import SamplingParams, SimpleSpeculativeConfig
+    from vllm_neuron_amd.engine import MI355XEngine
+    from vllm_neuron_amd.models import config_from_dict
+    cfg, w = case("wide")
+    spec = SimpleSpeculativeConfig(num_speculative_tokens=4, draft_model_config=SimpleNamespace(model="", hf_config=config_from_dict(cfg)))
+    eng = MI355XEngine(config_from_dict(cfg), dtype="float32", max_model_len=128, max_num_seqs=2, block_size=16, speculative_config=spec,
+                       override_mi355x_config={"state_dict": w, "draft_state_dict": w})
+    prompts = [torch.randint(0, 336, (n,), generator=torch.Generator().manual_seed(n)).tolist() for n in (20, 9)]
+    outs = eng.generate(prompts, SamplingParams(temperature=0.0, max_tokens=12))
+    assert [o.token_ids for o in outs] == [greedy(cfg, w, p, 12) for p in prompts]
+    eng.close()
+
+
+def test_a_draft_with_convolution_state_is_refused():
     from types import SimpleNamespace
 
     from vllm_neuron_amd._vllm_compat import SimpleSpeculativeConfig

@@ -71,7 +71,8 @@ class MiStackConfig(C.Structure):
                 ("vocab_size", C.c_int32), ("max_positions", C.c_int32), ("norm_eps", C.c_float),
                 ("residual_mult", C.c_float), ("loop_start", C.c_int32), ("loop_stop", C.c_int32),
                 ("loop_times", C.c_int32), ("compute_dtype", C.c_int32), ("block_kind", C.c_int32),
-                ("norm_groups", C.c_int32), ("conv_taps", C.c_int32), ("logit_softcap", C.c_float)]
+                ("norm_groups", C.c_int32), ("conv_taps", C.c_int32), ("logit_softcap", C.c_float),
+                ("state_lookahead", C.c_int32)]
 
 
 class MiTpPlan(C.Structure):

@@ -706,7 +706,7 @@ int mi_ctx_create_stack(const mi_model_config* cfg, const mi_stack_config* stack
   const bool sandwich = t.block_kind == MI_BLOCK_SANDWICH;
   if (sandwich) {
     MI_CHECK(t.norm_groups >= 1 && t.width % t.norm_groups == 0, "stack: the norm's groups must divide the width");
-    MI_CHECK(t.conv_taps >= 1 && t.conv_taps <= 16, "stack: convolutions of 1 .. 16 taps are built");
+    MI_CHECK(t.conv_taps >= 1 && t.conv_taps <= 16 && t.state_lookahead >= 0, "stack: convolutions of 1 .. 16 taps are built");
     MI_CHECK(t.loop_times == 0, "stack: loops are not built for sandwich blocks");
   } else {
     MI_CHECK(t.norm_groups == 0 && t.conv_taps == 0 && t.max_positions > 0, "stack: parallel blocks are built with layer norms, learned positions and no convolution");
@@ -1580,9 +1580,13 @@ int mi_forward_spec(mi_ctx* t, mi_ctx* d, int32_t B, int32_t k, const int64_t* i
   MI_CHECK(kt.device_id == kd.device_id && kt.block_size == kd.block_size && kt.num_blocks == kd.num_blocks &&
            kt.vocab_size == kd.vocab_size && kt.max_model_len == kd.max_model_len,
            "mi_forward_spec: target (rank 0) and draft must share device, block_size, num_blocks, vocab_size and max_model_len");
-  // several rows of one sequence in a token-generation batch: a convolution's state follows one row per sequence
-  MI_CHECK(!(t0->stack && t0->stack->conv_keep > 0) && !(d->stack && d->stack->conv_keep > 0),
-           "mi_forward_spec: not built for models with convolution state");
+  // Several rows of one sequence in a pass: a convolution's state follows one row per sequence.  Such a target takes the candidates as
+  // segments of k tokens, and its blocks keep the state far enough back to continue behind any accepted one; the draft's own steps
+  // (one row per sequence, a catch-up row beside it) have no such form.
+  const bool conv_target = t0->stack && t0->stack->cfg.conv_taps > 1;
+  MI_CHECK(!conv_target || t0->stack->conv_keep >= std::min(kt.block_size, t0->stack->cfg.conv_taps - 1 + k - 1),
+           "mi_forward_spec: the target keeps its convolution state for fewer candidates (mi_stack_config.state_lookahead)");
+  MI_CHECK(!(d->stack && d->stack->cfg.conv_taps > 1), "mi_forward_spec: a draft with convolution state is not built");
   MI_CHECK(B >= 1 && k >= 1 && B * k <= kt.max_num_seqs && B <= kd.max_num_seqs,
            "mi_forward_spec: B * k rows exceed the target's max_num_seqs (or B the draft's)");
   int n_catch = 0;
@@ -1675,6 +1679,20 @@ int mi_forward_spec(mi_ctx* t, mi_ctx* d, int32_t B, int32_t k, const int64_t* i
     return MI_OK;
   };
   auto target_pass = [&](mi_ctx* rc) -> int {
+    if (conv_target) {   // rows past a sequence's limit belong to no segment: computed, never read
+      const size_t at = rc->inputs_elems - 4 * (size_t)rc->cfg.max_num_seqs;
+      rc->d_segs = rc->d_inputs + at;
+      rc->h_segs = rc->h_inputs + at;
+      std::vector<Seg> segs((size_t)B);
+      for (int b = 0; b < B; ++b) segs[b] = Seg{b * k, lim_of(b), (int)position_ids[b], b * k};
+      memcpy(rc->h_segs, segs.data(), (size_t)B * sizeof(Seg));
+      MI_HIP(hipMemcpyAsync(rc->d_segs, rc->h_segs, (size_t)B * sizeof(Seg), hipMemcpyHostToDevice, rc->stream));
+      MI_TRY(run_trunk(rc, B * k, false, B, MB, 0, segs.data(), B));
+      MI_TRY(run_head(rc, B * k, 0, false));
+      rc->last_B = B * k;
+      rc->last_MB = MB;
+      return MI_OK;
+    }
     rc->attn_rows_per_seq = rows_per_seq;
     const int rc_pass = capture_or_launch_decode(rc, B * k, MB);
     rc->attn_rows_per_seq = 1;

@@ -312,7 +312,7 @@ int stack_create(mi_ctx* c, const mi_stack_config& cfg) {
     MI_TRY(alloc0(c, &S->pos, (size_t)cfg.max_positions * S->D * S->elem(), wb));
     want("pos");
   }
-  S->conv_keep = std::min(c->cfg.block_size, std::max(cfg.conv_taps - 1, 0));
+  S->conv_keep = cfg.conv_taps > 1 ? std::min(c->cfg.block_size, cfg.conv_taps - 1 + cfg.state_lookahead) : 0;
   if (loop) {
     MI_TRY(alloc_mat(c, S->loop_in, S->D, 2 * S->Kd, 1.f));
     want("loop.in");

@@ -308,7 +308,9 @@ class MI355XCausalLM(MI355XModelBase):
             if spec_len < 1 or speculative_config is None or chunked or not cfg["is_block_kv_layout"]:
                 raise NotImplementedError("fused speculation needs num_speculative_tokens >= 1, a draft model, the block "
                                           "KV layout (prefix caching on) and no chunked prefill")
-            check_speculation(stack_of(hf), stack_of(speculative_config.draft_model_config.hf_config))
+            check_draft(stack_of(speculative_config.draft_model_config.hf_config))
+            if "stack" in geo and geo["stack"].get("conv_taps", 0) > 1:
+                geo["stack"]["state_lookahead"] = spec_len - 1
         self.model = NativeModel(
             num_blocks=int(num_blocks), block_size=int(block_size),
             # the target scores every sequence's speculation window in one token-generation pass
@@ -497,11 +499,11 @@ class MI355XCausalLM(MI355XModelBase):
                         self.model.load_weight(name, t)
 
 
-def check_speculation(*stacks) -> None:
-    """Fused speculation runs several rows of one sequence in a token-generation pass; a convolution's state follows one."""
-    for stack in stacks:
-        if stack is not None and stack.get("conv_taps", 0) > 1:
-            raise NotImplementedError("fused speculation is not built for models with convolution state")
+def check_draft(stack: dict | None) -> None:
+    """The draft's chained steps run one row per sequence with a catch-up row beside it; a convolution's state would need
+    them in order."""
+    if stack is not None and stack.get("conv_taps", 0) > 1:
+        raise NotImplementedError("fused speculation: a draft model with convolution state is not built")
 
 
 def _model_geometry(hf, cfg: dict) -> dict:

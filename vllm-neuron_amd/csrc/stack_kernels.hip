@@ -297,16 +297,31 @@ __global__ __launch_bounds__(1024) void sandwich_token_kernel(const float* __res
   put4(y + (size_t)t * ldy + d, h.x, h.y, h.z, h.w);
 }
 
-// One work-group: up to ROWS rows of one segment x 1024 channels, four channels per thread; a thread's rows and the inputs ahead of
-// them are all requested at once.  TAPS = 0: any number of taps, inputs read where they are needed.
+// One work-group: up to ROWS rows of one segment x 256 C channels, C channels (16 bytes) per thread; a thread's rows and the inputs
+// ahead of them are all requested at once.  TAPS = 0: any number of taps, inputs read where they are needed.
 // The rows at a segment's start read the state of the positions ahead of it, and rows further on renew it.  Both may meet in one
 // place only in the block that holds the position ahead of the segment; that block's renewal is left to the work-group of the
 // segment's first rows, whose threads have read their channels' state by then (ROWS >= taps - 1).
 constexpr int kConvRows = 16;
+template <typename T> struct Chunk16 { static constexpr int C = 16 / sizeof(T); };
+
+__device__ __forceinline__ void widen16(const u32x4_t& v, float (&o)[8]) {
+#pragma unroll
+  for (int i = 0; i < 4; ++i) { o[2 * i] = bf16lo_to_f32(v[i]); o[2 * i + 1] = bf16hi_to_f32(v[i]); }
+}
+__device__ __forceinline__ void widen16(const u32x4_t& v, float (&o)[4]) {
+#pragma unroll
+  for (int i = 0; i < 4; ++i) o[i] = __builtin_bit_cast(float, (unsigned)v[i]);
+}
+__device__ __forceinline__ void put16(uint16_t* p, const float (&v)[8]) {
+  *reinterpret_cast<uint4*>(p) = make_uint4(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]), pack_bf16x2(v[4], v[5]), pack_bf16x2(v[6], v[7]));
+}
+__device__ __forceinline__ void put16(float* p, const float (&v)[4]) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
+
 template <typename T, int TAPS, int ROWS>
 __global__ __launch_bounds__(256) void conv_rows_kernel(const T* __restrict__ hin, ConvState cs, const AttnSeg* __restrict__ segs, int nseg,
                                                         int ld, T* __restrict__ y, int ldy) {
-  typedef typename Raw4<T>::type raw_t;
+  constexpr int C = Chunk16<T>::C;
   int tile = blockIdx.x, si = 0;
   AttnSeg sg{0, 0, 0, 0};
   for (; si < nseg; ++si) {
@@ -315,62 +330,78 @@ __global__ __launch_bounds__(256) void conv_rows_kernel(const T* __restrict__ hi
     if (tile < n) break;
     tile -= n;
   }
-  const int d = (blockIdx.y * 256 + threadIdx.x) * 4;
+  const int d = (blockIdx.y * 256 + threadIdx.x) * C;
   if (si == nseg || d >= ld) return;
   const int bs = cs.block_size, first = tile * ROWS, last = min(first + ROWS, sg.n), end = sg.pos0 + sg.n;
   const int shared_block = sg.pos0 % bs ? sg.pos0 / bs : -1;      // holds positions on both sides of the segment's start
   const T* hs = hin + (size_t)sg.row0 * ldy + d;
-  auto renew = [&](int p, float4 h) {
+  auto get = [&](const T* p) { return *reinterpret_cast<const u32x4_t*>(p); };
+  auto state = [&](int p) { return get(ring_at<T>(cs, cs.bt[(size_t)sg.seq * cs.MB + p / bs], p % bs, ldy) + d); };
+  auto renew = [&](int p, const u32x4_t& h) {
     const int slot = cs.slots[sg.row0 + p - sg.pos0];
-    if (slot >= 0) put4(ring_at<T>(cs, slot / bs, slot % bs, ldy) + d, h.x, h.y, h.z, h.w);
+    if (slot >= 0) *reinterpret_cast<u32x4_t*>(ring_at<T>(cs, slot / bs, slot % bs, ldy) + d) = h;
   };
-  auto renew_own = [&](int p, float4 h) {
+  auto renew_own = [&](int p, const u32x4_t& h) {
     const int b = p / bs;
     if (b != shared_block && p + cs.keep >= min(end, (b + 1) * bs)) renew(p, h);
   };
-  if constexpr (TAPS > 0) {
-    raw_t in[ROWS + TAPS - 1];
-    float4 w[TAPS];
+  auto tap = [&](int j, float (&w)[C]) {
 #pragma unroll
-    for (int j = 0; j < TAPS; ++j) w[j] = *reinterpret_cast<const float4*>(cs.w + (size_t)j * ld + d);
+    for (int c = 0; c < C; c += 4) *reinterpret_cast<float4*>(w + c) = *reinterpret_cast<const float4*>(cs.w + (size_t)j * ld + d + c);
+  };
+  if constexpr (TAPS > 0) {
+    u32x4_t in[ROWS + TAPS - 1];
+    float w[TAPS][C];
 #pragma unroll
     for (int k = 0; k < ROWS + TAPS - 1; ++k) {
       const int i = first + k - (TAPS - 1);                         // row of the segment; negative: ahead of it
-      if (i >= 0) in[k] = *reinterpret_cast<const raw_t*>(hs + (size_t)min(i, sg.n - 1) * ldy);
-      else if (sg.pos0 + i >= 0) {
-        const int p = sg.pos0 + i;
-        in[k] = *reinterpret_cast<const raw_t*>(ring_at<T>(cs, cs.bt[(size_t)sg.seq * cs.MB + p / bs], p % bs, ldy) + d);
-      } else in[k] = raw_t{};                                        // (ahead of the sequence: zeros)
+      if (i >= 0) in[k] = get(hs + (size_t)min(i, sg.n - 1) * ldy);
+      else if (sg.pos0 + i >= 0) in[k] = state(sg.pos0 + i);
+      else in[k] = u32x4_t{0, 0, 0, 0};                              // (ahead of the sequence: zeros)
     }
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) tap(j, w[j]);
 #pragma unroll
     for (int k = 0; k < ROWS; ++k) {
       if (first + k >= last) break;
-      const float4 h = widen(in[k + TAPS - 1]);
-      float4 a = make_float4(0.f, 0.f, 0.f, 0.f);
+      float a[C], h[C];
+#pragma unroll
+      for (int c = 0; c < C; ++c) a[c] = 0.f;
 #pragma unroll
       for (int j = 0; j < TAPS; ++j) {
-        const float4 v = widen(in[k + j]);
-        a.x = __builtin_fmaf(w[j].x, v.x, a.x); a.y = __builtin_fmaf(w[j].y, v.y, a.y);
-        a.z = __builtin_fmaf(w[j].z, v.z, a.z); a.w = __builtin_fmaf(w[j].w, v.w, a.w);
+        widen16(in[k + j], h);
+#pragma unroll
+        for (int c = 0; c < C; ++c) a[c] = __builtin_fmaf(w[j][c], h[c], a[c]);
       }
-      put4(y + (size_t)(sg.row0 + first + k) * ldy + d, h.x + a.x, h.y + a.y, h.z + a.z, h.w + a.w);
-      if constexpr (TAPS > 1) renew_own(sg.pos0 + first + k, h);
+#pragma unroll
+      for (int c = 0; c < C; ++c) a[c] += h[c];                      // (the last tap met the token itself)
+      put16(y + (size_t)(sg.row0 + first + k) * ldy + d, a);
+      if constexpr (TAPS > 1) renew_own(sg.pos0 + first + k, in[k + TAPS - 1]);
     }
   } else {
     for (int i = first; i < last; ++i) {
       const int p = sg.pos0 + i;
       const T* r = hs + (size_t)i * ldy;
-      const float4 h = get4(r);
-      const float4 a = conv_sum(cs, ld, d, p, h, [&](int back) {
-        return back <= i ? get4(r - (size_t)back * ldy) : ring_get4<T>(cs, sg.seq, p - back, ldy, d);
-      });
-      put4(y + (size_t)(sg.row0 + i) * ldy + d, a.x, a.y, a.z, a.w);
-      renew_own(p, h);
+      float a[C], h[C], w[C];
+#pragma unroll
+      for (int c = 0; c < C; ++c) a[c] = 0.f;
+      for (int j = 0; j < cs.taps; ++j) {
+        const int back = cs.taps - 1 - j;
+        if (back > p) continue;
+        widen16(back <= i ? get(r - (size_t)back * ldy) : state(p - back), h);
+        tap(j, w);
+#pragma unroll
+        for (int c = 0; c < C; ++c) a[c] = __builtin_fmaf(w[c], h[c], a[c]);
+      }
+#pragma unroll
+      for (int c = 0; c < C; ++c) a[c] += h[c];
+      put16(y + (size_t)(sg.row0 + i) * ldy + d, a);
+      renew_own(p, get(r));
     }
   }
   if (tile == 0 && shared_block >= 0) {
     const int stop = min(end, (shared_block + 1) * bs);
-    for (int p = max(sg.pos0, stop - cs.keep); p < stop; ++p) renew(p, get4(hs + (size_t)(p - sg.pos0) * ldy));
+    for (int p = max(sg.pos0, stop - cs.keep); p < stop; ++p) renew(p, get(hs + (size_t)(p - sg.pos0) * ldy));
   }
 }
 
@@ -601,11 +632,11 @@ int launch_conv_rows(const void* h, const ConvState& conv, const AttnSeg* sd, co
                      bool f32, hipStream_t s) {
   int rc = check_conv(conv);
   if (rc != MI_OK) return rc;
-  MI_CHECK(nseg >= 1 && ld % 4 == 0 && ld >= D && ldy >= ld && ldy % 4 == 0 && h != y, "convolution: strides");
+  MI_CHECK(nseg >= 1 && ld % 8 == 0 && ld >= D && ldy >= ld && ldy % 8 == 0 && h != y, "convolution: strides");
   const int rows = conv.taps <= 4 ? 8 : kConvRows;
   int tiles = 0;
   for (int i = 0; i < nseg; ++i) tiles += ceil_div(sh[i].n, rows);
-  const dim3 grid(tiles, ceil_div(ld, 1024));
+  const dim3 grid(tiles, ceil_div(ld, f32 ? 1024 : 2048));
 #define MI_CONV(TAPS, ROWS) \
   if (f32) hipLaunchKernelGGL((conv_rows_kernel<float, TAPS, ROWS>), grid, dim3(256), 0, s, (const float*)h, conv, sd, nseg, ld, (float*)y, ldy); \
   else hipLaunchKernelGGL((conv_rows_kernel<uint16_t, TAPS, ROWS>), grid, dim3(256), 0, s, (const uint16_t*)h, conv, sd, nseg, ld, (uint16_t*)y, ldy)

@@ -240,7 +240,7 @@ def close(got, ref, f32, tol=2e-2):
 
 @pytest.mark.parametrize("f32,path", PATHS)
 @pytest.mark.parametrize("H,dk,dv,rank,window,bs", [
-    (4, 64, 48, 64, 96, 16), (3, 20, 13, 36, 37, 32), (18, 32, 32, 160, 0, 48), (34, 16, 24, 64, 5, 16), (2, 160, 200, 288, 129, 32),
+    (4, 64, 40, 96, 96, 16), (3, 20, 13, 36, 37, 32), (18, 32, 32, 160, 0, 48), (34, 16, 24, 64, 5, 16), (2, 160, 200, 288, 129, 32),
     (70, 8, 8, 32, 1, 16), (5, 128, 128, 512, 64, 16)])
 def test_latent_attention(lib, H, dk, dv, rank, window, bs, f32, path):
     got, ref = Paged(H, dk, dv, rank, SEGS, bs, seed=H + window).run(lib, window, 1.5 / math.sqrt(dk), f32, path)

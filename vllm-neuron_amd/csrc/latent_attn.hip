@@ -561,8 +561,10 @@ int launch_latent_attn_rows(const LatentGeom& g, float scale, int window, const 
   int hg = 1;
   while (hg < 4 && hg < hgs && lr.rows * ceil_div(hgs, 2 * hg) >= 256) hg *= 2;
   const int groups = lr.rows * ceil_div(hgs, hg);
-  // (one head group: 70 KiB of LDS at the largest rank, two work-groups per CU)
-  int NS = min(min((hg == 1 ? 512 : 256) / groups, tiles), kMaxSplits);
+  // One head group: 70 KiB of LDS at the largest rank, two work-groups per CU.  The second one is worth its partial results
+  // (the merge reads every split's) up to eight splits.
+  const int most = hg == 1 ? min(512 / groups, max(256 / groups, 8)) : 256 / groups;
+  int NS = min(min(most, tiles), kMaxSplits);
   if (NS < 1) NS = 1;
   float* ml = reinterpret_cast<float*>(scratch);
   float* op = ml + (size_t)512 * g.H * 2;

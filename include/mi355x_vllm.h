@@ -94,30 +94,50 @@ typedef struct mi_model_config {
 enum { MI_TP_TRANSPORT_P2P = 0, MI_TP_TRANSPORT_RCCL = 1 };
 
 /* ---- layer-stack decoders: a decoder given layer by layer, every size and constant a parameter ----
- * (Vimesun and Rapodra are such designs; the worker's model registry fills this from their config.json.)
- *     x = embed[token] (+ pos[position])                      fp32 residual stream
+ * (Vimesun, Rapodra and Bokulorn are such designs; the worker's model registry fills this from their config.json.)
+ *     x = embed_scale embed[token] (+ pos[position])          fp32 residual stream
  *     block MI_BLOCK_PARALLEL:  x <- x + residual_mult (mixer(norm1 x) + ff(norm2 x))     both of the same x
  *     block MI_BLOCK_SANDWICH:  x <- x + norm1b(mixer(C1(norm1 x))); x <- x + norm2b(ff(C2(norm2 x)))
  *             C(h) = h + causal convolution of h over time, conv_taps taps per channel; the last conv_taps - 1 inputs h
  *             are part of a sequence's state
+ *     block MI_BLOCK_ONE_NORM:  h = norm1 x;  x <- x + mixer(h) + ff(h)
  *     norms:  norm_groups = 0: layer norm with weight and bias; else RMS norm of norm_groups equal parts, each over its
- *             own sqrt(mean square + norm_eps), times a weight
+ *             own sqrt(mean square + norm_eps), times a weight (norm_offset = 1: times 1 + weight, also the final norm)
  *     loop:   layers loop_start .. loop_stop - 1 run loop_times times in a row with the same weights, each pass with a
  *             KV pool of its own; ahead of a pass's first layer  x <- W_in [x ; embedding output]
+ *     weights_of >= 0: the layer has no tensors of its own, it runs that other layer's with a cache and state of its own
  *     logits = head final_norm(x); logit_softcap > 0: softcap tanh(logits / softcap)
  * Mixers: MI_MIX_ATTENTION, grouped heads with K / V pools; MI_MIX_LATENT, per head k = W_uk c, v = W_uv c of a cached latent
  *     c = RMSnorm(W_dkv h) [kv_rank]; kv_from >= 0: the latents of that earlier layer instead of own ones.
+ *     q_rank > 0: queries q = W_uq RMSnorm(W_dq h) [q_rank] instead of W_q h.  rot_dim > 0: a head's query has rot_dim more
+ *     elements behind its qk_dim, W_dkv that many more rows (one more key part for all heads, not normed); both parts rotate over their
+ *     first rot_dims elements, pair (i, i + rot_dims / 2) by position * rot_base^(-2 i / rot_dims), and their product joins the
+ *     score.  out_gate: MI_GATE_HEAD, a head's output times sigmoid(W_g h)_head; MI_GATE_ELEMENT, every element of the heads'.
+ *   MI_MIX_DELTA, a gated delta rule with one decay per head and key channel, num_kv_heads query / key heads shared by
+ *     num_heads heads with a state S [qk_dim, v_dim] each: q, k, v = W h through a causal convolution of conv_taps taps and
+ *     silu; q and k over sqrt(sum of squares + 1e-6), q times qk_dim^-1/2; beta = sigmoid(W_b h); g = exp(-exp(A_log)
+ *     softplus(W_a2 W_a1 h + dt_bias)) (decay_rank rows in W_a1);  S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q;
+ *     output W_o (RMSnorm(o) sigmoid(W_g2 W_g1 h)) (gate_rank rows in W_g1).  Everything fp32 but the projections.  S and the
+ *     last inputs of the convolution live in a state slot per sequence (seq_ids of the model calls).
  * Feed-forwards: MI_FF_RELU2 down(max(up x, 0)^2); MI_FF_GLU down(act(gate x, up x)); MI_FF_MOE the softmax-weighted sum of the
  *     experts_top experts with the largest router logits (W_router x + b), each down(act(gate x, up x)).
+ *     router_score MI_ROUTE_SIGMOID: s = sigmoid(W_router x); choice scores s + correction; the experts lie in router_groups equal
+ *     groups, of which the router_keep with the largest sum of their two best choice scores are eligible; weights s over their sum.
  * Gated activations: MI_ACT_SILU g sigmoid(g) u; MI_ACT_SWISH_CLIP, g = min(g, limit), u within +-limit: g sigmoid(alpha g) (u + 1).
- * Built: parallel blocks of MI_MIX_ATTENTION with layer norms, sandwich blocks of MI_MIX_LATENT with RMS norms and no loop.
+ * MI_ACT_RELU2 (experts): no gate, max(up x, 0)^2.
+ * Built: parallel blocks of MI_MIX_ATTENTION with layer norms, sandwich blocks of MI_MIX_LATENT with RMS norms and no loop,
+ * one-norm blocks of MI_MIX_LATENT (every earlier token in sight) and MI_MIX_DELTA with RMS norms, experts or no feed-forward and no loop.
  * Tensor names ("l<i>." = layer i): embed, pos, loop.in, l<i>.norm1(.b), l<i>.norm2(.b), l<i>.mix.{q,k,v,o},
  * l<i>.mlp.{up,down}, final.norm(.b), head; sandwich blocks: l<i>.norm1, .norm1b, .norm2, .norm2b, .canon1, .canon2
- * [width, taps], l<i>.mix.{q,dkv,dkv.norm,uk,uv,o}, l<i>.mlp.{gate,up,down}, l<i>.mlp.router(.b), l<i>.mlp.e<n>.{gate,up,down}. */
-enum { MI_BLOCK_PARALLEL = 0, MI_BLOCK_SANDWICH = 1 };
-enum { MI_MIX_ATTENTION = 0, MI_MIX_LATENT = 1 };
+ * [width, taps], l<i>.mix.{q,dkv,dkv.norm,uk,uv,o}, l<i>.mlp.{gate,up,down}, l<i>.mlp.router(.b), l<i>.mlp.e<n>.{gate,up,down};
+ * one-norm blocks: l<i>.norm1, l<i>.mix.{dq,dq.norm,uq | q}, l<i>.mix.{dkv,dkv.norm,uk,uv,g,o}, or l<i>.mix.{q,k,v,q.conv,k.conv,v.conv,
+ * b,A_log,a1,a2,dt_bias,g1,g2,norm,o}, l<i>.mlp.router, .correction (or .router.b), l<i>.mlp.e<n>.{gate,up,down}. */
+enum { MI_BLOCK_PARALLEL = 0, MI_BLOCK_SANDWICH = 1, MI_BLOCK_ONE_NORM = 2 };
+enum { MI_MIX_ATTENTION = 0, MI_MIX_LATENT = 1, MI_MIX_DELTA = 2 };
 enum { MI_FF_NONE = 0, MI_FF_RELU2 = 1, MI_FF_GLU = 2, MI_FF_MOE = 3 };
-enum { MI_ACT_SILU = 0, MI_ACT_SWISH_CLIP = 1 };
+enum { MI_ACT_SILU = 0, MI_ACT_SWISH_CLIP = 1, MI_ACT_RELU2 = 2 };
+enum { MI_GATE_NONE = 0, MI_GATE_HEAD = 1, MI_GATE_ELEMENT = 2 };
+enum { MI_ROUTE_SOFTMAX = 0, MI_ROUTE_SIGMOID = 1 };
 typedef struct mi_layer_spec {
   int32_t num_heads, num_kv_heads, qk_dim, v_dim;
   int32_t window;         /* a query sees keys with 0 <= i - j < window; 0 = every earlier token */
@@ -131,6 +151,13 @@ typedef struct mi_layer_spec {
   int32_t ff_act;             /* MI_ACT_*, gated feed-forwards and experts */
   float ff_limit, ff_alpha;   /* MI_ACT_SWISH_CLIP */
   int32_t experts, experts_top;
+  int32_t router_score, router_groups, router_keep;   /* MI_ROUTE_SIGMOID: groups >= 1, 1 <= keep <= groups */
+  int32_t weights_of;         /* -1: tensors of its own (one-norm blocks) */
+  int32_t q_rank;             /* MI_MIX_LATENT: 0 = W_q h */
+  int32_t rot_dim, rot_dims;
+  float rot_base;
+  int32_t out_gate;           /* MI_GATE_* */
+  int32_t conv_taps, decay_rank, gate_rank;   /* MI_MIX_DELTA */
 } mi_layer_spec;
 typedef struct mi_stack_config {
   int32_t num_layers;
@@ -143,10 +170,11 @@ typedef struct mi_stack_config {
   int32_t conv_taps;       /* sandwich blocks: 1 .. 16 */
   float logit_softcap;     /* 0 = none */
   int32_t state_lookahead; /* sandwich blocks: a step may write this many positions behind the last accepted one (speculation: k - 1) */
+  float embed_scale, norm_offset;
 } mi_stack_config;
 
 const char* mi_last_error(void);
-int mi_version(void);   /* 6 = this header (+ sandwich blocks, latent attention, experts in mi_layer_spec / mi_stack_config and their mi_op_*); 5 (+ mi_ctx_create_stack, mi_forward_rows, mi_layer_residuals, mi_op_* of the stack kernels); 4 (+ mi_tp_plan, mi_tp_info); 3 lacked them; 2 lacked tp_device_ids / tp_transport / MI_TP_ALL_RANKS; 1 lacked mi_forward_tokens, mi_op_sample, mi_tp_init_transport */
+int mi_version(void);   /* 7 = this header (+ one-norm blocks, recurrent mixers and their state slots: seq_ids of mi_forward_chunked / mi_forward_rows); 6 (+ sandwich blocks, latent attention, experts in mi_layer_spec / mi_stack_config and their mi_op_*); 5 (+ mi_ctx_create_stack, mi_forward_rows, mi_layer_residuals, mi_op_* of the stack kernels); 4 (+ mi_tp_plan, mi_tp_info); 3 lacked them; 2 lacked tp_device_ids / tp_transport / MI_TP_ALL_RANKS; 1 lacked mi_forward_tokens, mi_op_sample, mi_tp_init_transport */
 
 int mi_ctx_create(const mi_model_config* cfg, mi_ctx** out);
 /* The same context around a layer stack.  Of cfg only the serving fields are read (pool, batch, buckets, device, graphs);
@@ -183,6 +211,8 @@ int mi_finalize(mi_ctx* ctx);
  *   input_ids, position_ids [B, S]; seq_ids [B]; block_table [B, MB];
  *   slot_mapping [B, SM]; full_context_lens, computed_context_lens [B];
  *   logits_out [B, vocab_size] fp32 (last-token logits, loader.py:363).
+ * seq_ids: models with recurrent mixers keep a sequence's state in slot seq_ids[b] (0 .. max_num_seqs - 1, no two rows
+ * alike; a sequence whose first token is in the call starts from a zero state, whatever the slot held); otherwise not read.
  * S == 1 -> token generation;  S > 1 -> context encoding of tokens
  * computed..full-1 of each row (the FULL prompt is passed, runner.py:721-726,754).
  * Slot -1 = no write; block-table entries past full_context_lens are never read. */
@@ -215,16 +245,17 @@ int mi_forward_tokens(mi_ctx* ctx, int32_t B, int32_t S, const int64_t* input_id
  * once over all rows.  logits_out [n_req, vocab_size] = logits of each request's LAST scheduled
  * token (the caller ignores rows whose prompt is not complete: prefill_completion_state);
  * or tokens_out [n_req] with sampling_params as in mi_forward_tokens.  total may not exceed the
- * largest context-encoding bucket (pass max_num_batched_tokens as a bucket). */
+ * largest context-encoding bucket (pass max_num_batched_tokens as a bucket).  seq_ids [n_req]: as mi_forward; may be NULL for
+ * models without recurrent mixers. */
 int mi_forward_chunked(mi_ctx* ctx, int32_t n_req, int32_t total, const int64_t* input_ids,
-                       const int64_t* position_ids, const int64_t* slot_mapping, const int64_t* block_table,
+                       const int64_t* position_ids, const int64_t* seq_ids, const int64_t* slot_mapping, const int64_t* block_table,
                        int32_t MB, const int64_t* full_context_lens, const int64_t* computed_context_lens,
                        float* logits_out, const float* sampling_params, uint64_t seed, int64_t* tokens_out);
 
 /* The same ragged batch with the logits of chosen places: rows [n_rows] = indices into the token batch (any order, any
  * number, none at all); logits_out [n_rows, vocab_size] in that order. */
 int mi_forward_rows(mi_ctx* ctx, int32_t n_req, int32_t total, const int64_t* input_ids, const int64_t* position_ids,
-                    const int64_t* slot_mapping, const int64_t* block_table, int32_t MB, const int64_t* full_context_lens,
+                    const int64_t* seq_ids, const int64_t* slot_mapping, const int64_t* block_table, int32_t MB, const int64_t* full_context_lens,
                     const int64_t* computed_context_lens, int32_t n_rows, const int64_t* rows, float* logits_out);
 
 /* Layer-stack contexts: keep a copy of the residual stream behind every layer run of the following ragged batches

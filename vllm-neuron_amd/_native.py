@@ -14,7 +14,7 @@ import os
 
 import torch  # noqa: F401  (must precede CDLL, see module docstring)
 
-from ._stack_enums import MI_ACT, MI_BLOCK, MI_FF, MI_MIX  # noqa: F401
+from ._stack_enums import MI_ACT, MI_BLOCK, MI_FF, MI_GATE, MI_MIX, MI_ROUTE  # noqa: F401
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 # MI355X_VLLM_LIB points at another build of the same library (A/B measurements)
@@ -63,7 +63,10 @@ class MiLayerSpec(C.Structure):
                 ("window", C.c_int32), ("scale", C.c_float), ("qk_unit_norm", C.c_int32), ("distance_bias", C.c_int32),
                 ("softmax_sink", C.c_int32), ("ff_kind", C.c_int32), ("ff_size", C.c_int32), ("mixer_kind", C.c_int32),
                 ("kv_rank", C.c_int32), ("kv_from", C.c_int32), ("ff_act", C.c_int32), ("ff_limit", C.c_float),
-                ("ff_alpha", C.c_float), ("experts", C.c_int32), ("experts_top", C.c_int32)]
+                ("ff_alpha", C.c_float), ("experts", C.c_int32), ("experts_top", C.c_int32),
+                ("router_score", C.c_int32), ("router_groups", C.c_int32), ("router_keep", C.c_int32), ("weights_of", C.c_int32),
+                ("q_rank", C.c_int32), ("rot_dim", C.c_int32), ("rot_dims", C.c_int32), ("rot_base", C.c_float),
+                ("out_gate", C.c_int32), ("conv_taps", C.c_int32), ("decay_rank", C.c_int32), ("gate_rank", C.c_int32)]
 
 
 class MiStackConfig(C.Structure):
@@ -72,7 +75,7 @@ class MiStackConfig(C.Structure):
                 ("residual_mult", C.c_float), ("loop_start", C.c_int32), ("loop_stop", C.c_int32),
                 ("loop_times", C.c_int32), ("compute_dtype", C.c_int32), ("block_kind", C.c_int32),
                 ("norm_groups", C.c_int32), ("conv_taps", C.c_int32), ("logit_softcap", C.c_float),
-                ("state_lookahead", C.c_int32)]
+                ("state_lookahead", C.c_int32), ("embed_scale", C.c_float), ("norm_offset", C.c_float)]
 
 
 class MiTpPlan(C.Structure):
@@ -109,9 +112,9 @@ _SIGS = {
     "mi_forward_tokens": (C.c_int, [C.c_void_p, C.c_int32, C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p,
                                     C.c_void_p, C.c_int32, C.c_void_p, C.c_int32, C.c_void_p, C.c_void_p,
                                     C.c_void_p, C.c_uint64, C.c_void_p]),
-    "mi_forward_chunked": (C.c_int, [C.c_void_p, C.c_int32, C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p,
+    "mi_forward_chunked": (C.c_int, [C.c_void_p, C.c_int32, C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p,
                                      C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p, C.c_uint64, C.c_void_p]),
-    "mi_forward_rows": (C.c_int, [C.c_void_p, C.c_int32, C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p,
+    "mi_forward_rows": (C.c_int, [C.c_void_p, C.c_int32, C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p, C.c_void_p,
                                   C.c_int32, C.c_void_p, C.c_void_p, C.c_int32, C.c_void_p, C.c_void_p]),
     "mi_layer_residuals": (C.c_int, [C.c_void_p, C.c_int32]),
     "mi_layer_residuals_read": (C.c_int, [C.c_void_p, C.c_int32, C.c_void_p]),
@@ -211,7 +214,7 @@ def _ptr(t) -> int:
 
 
 def layer_spec(layer: dict) -> MiLayerSpec:
-    out = MiLayerSpec()
+    out = MiLayerSpec(weights_of=-1)
     for k, v in layer.items():
         if not hasattr(out, k):
             raise ValueError(f"unknown layer field {k!r}")
@@ -220,7 +223,7 @@ def layer_spec(layer: dict) -> MiLayerSpec:
 
 
 def stack_config(stack: dict) -> MiStackConfig:
-    st = MiStackConfig()
+    st = MiStackConfig(embed_scale=1.0)
     layers = [layer_spec(x) for x in stack["layers"]]
     st._keep = (MiLayerSpec * len(layers))(*layers)      # the library copies it during the call
     st.layers, st.num_layers = st._keep, len(layers)
@@ -409,9 +412,10 @@ class NativeModel:
         return out
 
     def forward_chunked(self, input_ids, position_ids, slot_mapping, block_table, full_context_lens,
-                        computed_context_lens, sampling_params=None, seed: int = 0, tokens: bool = False):
+                        computed_context_lens, sampling_params=None, seed: int = 0, tokens: bool = False, seq_ids=None):
         """Chunked prefill: one ragged token batch (reference runner.py:1000-1051).  input_ids,
-        position_ids, slot_mapping: flat [total]; block_table [n, MB]; the context lengths [n].
+        position_ids, slot_mapping: flat [total]; block_table [n, MB]; the context lengths [n]; seq_ids [n]: state slots of
+        models with recurrent mixers.
         -> fp32 logits [n, V] of every request's last scheduled token, or sampled ids [n] (tokens=True)."""
         def i64(t):
             return t.to(torch.int64).contiguous()
@@ -423,7 +427,9 @@ class NativeModel:
         if tokens and sampling_params is not None:
             sp = sampling_params.to(torch.float32).contiguous()
         out = torch.empty(n, dtype=torch.int64) if tokens else torch.empty(n, self.vocab_size, dtype=torch.float32)
-        check(self.lib.mi_forward_chunked(self._ctx, n, ids.numel(), ids.data_ptr(), pos.data_ptr(), sm.data_ptr(),
+        seq = i64(seq_ids).reshape(n) if seq_ids is not None else None
+        check(self.lib.mi_forward_chunked(self._ctx, n, ids.numel(), ids.data_ptr(), pos.data_ptr(),
+                                          seq.data_ptr() if seq is not None else None, sm.data_ptr(),
                                           bt.data_ptr(), bt.shape[1], full.data_ptr(), comp.data_ptr(),
                                           None if tokens else out.data_ptr(),
                                           sp.data_ptr() if sp is not None else None, seed & (2 ** 64 - 1),
@@ -431,7 +437,7 @@ class NativeModel:
         return out
 
     def forward_rows(self, input_ids, position_ids, slot_mapping, block_table, full_context_lens, computed_context_lens,
-                     rows) -> "torch.Tensor":
+                     rows, seq_ids=None) -> "torch.Tensor":
         """The ragged batch of `forward_chunked` with the logits of chosen places: `rows` = indices into the token
         batch (may be empty).  -> fp32 logits [len(rows), V]."""
         def i64(t):
@@ -441,7 +447,9 @@ class NativeModel:
         n = full.numel()
         bt = block_table.to(torch.int64).contiguous().reshape(n, -1)
         out = torch.empty(want.numel(), self.vocab_size, dtype=torch.float32)
-        check(self.lib.mi_forward_rows(self._ctx, n, ids.numel(), ids.data_ptr(), pos.data_ptr(), sm.data_ptr(), bt.data_ptr(),
+        seq = i64(seq_ids) if seq_ids is not None else None
+        check(self.lib.mi_forward_rows(self._ctx, n, ids.numel(), ids.data_ptr(), pos.data_ptr(),
+                                       seq.data_ptr() if seq is not None else None, sm.data_ptr(), bt.data_ptr(),
                                        bt.shape[1], full.data_ptr(), comp.data_ptr(), want.numel(),
                                        want.data_ptr() if want.numel() else None, out.data_ptr() if want.numel() else None))
         return out

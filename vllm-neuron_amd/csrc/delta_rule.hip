@@ -1,0 +1,562 @@
+// Gated delta rule.  See delta_rule.h.
+#include "delta_rule.h"
+
+#include <algorithm>
+
+namespace mi {
+
+namespace {
+
+constexpr int kC = kDeltaChunk;
+
+__device__ __forceinline__ float silu(float v) { return v / (1.f + expf(-v)); }
+__device__ __forceinline__ float sigmoid(float v) { return 1.f / (1.f + expf(-v)); }
+__device__ __forceinline__ float softplus(float v) { return fmaxf(v, 0.f) + log1pf(expf(-fabsf(v))); }
+__device__ __forceinline__ float log_decay(float z, float dt, float a_log) { return -expf(a_log) * softplus(z + dt); }
+__device__ __forceinline__ void put1(uint16_t* p, float v) { *p = f32_to_bf16(v); }
+__device__ __forceinline__ void put1(float* p, float v) { *p = v; }
+
+// ---- token generation ---------------------------------------------------------------------------------------------------------
+// One work-group per (head, row): the whole state of the head in registers, requested first; thread (vq, dg) owns columns
+// 4 vq .. + 3 of rows dg RPT .. + RPT - 1.  Both products with the decayed state are taken in one pass (o = S^T q + (k.q) u).
+constexpr int kTokenThreads = 512;
+template <typename T, int VQ, int RPT>
+__global__ __launch_bounds__(kTokenThreads) void delta_token_kernel(DeltaGeom g, DeltaIn in, const AttnSeg* __restrict__ segs, T* __restrict__ y, int ldy) {
+  constexpr int NW = kTokenThreads / 64;
+  __shared__ float qs[256], ks[256], gs[256], vs[256];
+  __shared__ float norms[3];
+  __shared__ __attribute__((aligned(16))) float red[2][NW][VQ * 4];
+  const int h = blockIdx.x, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  int row = blockIdx.y, seq = blockIdx.y;
+  if (segs) {
+    const AttnSeg sg = segs[blockIdx.y];
+    if (sg.n != 1) return;
+    row = sg.row0; seq = sg.seq;
+  }
+  const int slot = in.slots[seq], p = in.pos[row], vq = tid % VQ, dg = tid / VQ;
+  const bool vin = vq * 4 < g.dvp;
+  float* S0 = in.state + ((size_t)slot * g.H + h) * g.dkp * g.dvp + vq * 4;
+  float4 S[RPT];
+#pragma unroll
+  for (int i = 0; i < RPT; ++i) {
+    const int d = dg * RPT + i;
+    S[i] = p > 0 && vin && d < g.dkp ? *reinterpret_cast<const float4*>(S0 + (size_t)d * g.dvp) : make_float4(0.f, 0.f, 0.f, 0.f);
+  }
+  // convolutions of the head's channels; position p goes to a row of the ring that nobody reads in this launch
+  const int C = g.channels(), r = g.H / g.G, kvh = h / r;
+  const float* x = in.proj + (size_t)row * in.ldp;
+  float* ring = in.ring + (size_t)slot * g.taps * C;
+  for (int i = tid; i < 2 * g.dk + g.dv; i += kTokenThreads) {
+    const int part = i < g.dk ? 0 : i < 2 * g.dk ? 1 : 2, d = i - part * g.dk;
+    const int ch = part == 2 ? 2 * g.G * g.dk + h * g.dv + d : (part * g.G + kvh) * g.dk + d;
+    const float now = x[ch];
+    float a = 0.f;
+    for (int j = 0; j + 1 < g.taps; ++j) {
+      const int q = p - (g.taps - 1 - j);
+      if (q >= 0) a = __builtin_fmaf(in.conv[(size_t)j * C + ch], ring[(size_t)(q % g.taps) * C + ch], a);
+    }
+    a = silu(__builtin_fmaf(in.conv[(size_t)(g.taps - 1) * C + ch], now, a));
+    if (part == 2 || h % r == 0) ring[(size_t)(p % g.taps) * C + ch] = now;
+    (part == 0 ? qs : part == 1 ? ks : vs)[d] = a;
+  }
+  for (int d = tid; d < g.dkp; d += kTokenThreads) {
+    if (d >= g.dk) { qs[d] = ks[d] = 0.f; gs[d] = 1.f; continue; }
+    gs[d] = expf(log_decay(in.z[(size_t)row * in.ldz + h * g.dk + d], in.dt[h * g.dk + d], in.a_log[h]));
+  }
+  for (int d = g.dv + tid; d < g.dvp; d += kTokenThreads) vs[d] = 0.f;
+  const float beta = sigmoid(x[in.beta + h]);
+  __syncthreads();
+  if (wave < 3) {
+    float s = 0.f;
+    for (int d = lane; d < g.dk; d += 64) s = __builtin_fmaf(wave == 1 ? ks[d] : qs[d], wave == 0 ? qs[d] : ks[d], s);
+    s = wave_sum(s);
+    if (lane == 0) norms[wave] = s;
+  }
+  __syncthreads();
+  const float fq = 1.f / sqrtf(norms[0] + 1e-6f) * (1.f / sqrtf((float)g.dk)), fk = 1.f / sqrtf(norms[1] + 1e-6f), qk = norms[2] * fq * fk;
+  float4 r1 = make_float4(0.f, 0.f, 0.f, 0.f), r2 = r1;
+#pragma unroll
+  for (int i = 0; i < RPT; ++i) {
+    const int d = dg * RPT + i;
+    if (d >= g.dkp) continue;
+    const float gd = gs[d], kd = ks[d] * fk, qd = qs[d] * fq;
+    S[i].x *= gd; S[i].y *= gd; S[i].z *= gd; S[i].w *= gd;
+    r1.x = __builtin_fmaf(S[i].x, kd, r1.x); r1.y = __builtin_fmaf(S[i].y, kd, r1.y); r1.z = __builtin_fmaf(S[i].z, kd, r1.z); r1.w = __builtin_fmaf(S[i].w, kd, r1.w);
+    r2.x = __builtin_fmaf(S[i].x, qd, r2.x); r2.y = __builtin_fmaf(S[i].y, qd, r2.y); r2.z = __builtin_fmaf(S[i].z, qd, r2.z); r2.w = __builtin_fmaf(S[i].w, qd, r2.w);
+  }
+#pragma unroll
+  for (int m = VQ; m < 64; m *= 2) {
+    r1.x += __shfl_xor(r1.x, m); r1.y += __shfl_xor(r1.y, m); r1.z += __shfl_xor(r1.z, m); r1.w += __shfl_xor(r1.w, m);
+    r2.x += __shfl_xor(r2.x, m); r2.y += __shfl_xor(r2.y, m); r2.z += __shfl_xor(r2.z, m); r2.w += __shfl_xor(r2.w, m);
+  }
+  if (lane < VQ) {
+    *reinterpret_cast<float4*>(&red[0][wave][vq * 4]) = r1;
+    *reinterpret_cast<float4*>(&red[1][wave][vq * 4]) = r2;
+  }
+  __syncthreads();
+  r1 = make_float4(0.f, 0.f, 0.f, 0.f);
+  r2 = r1;
+#pragma unroll
+  for (int w = 0; w < NW; ++w) {
+    const float4 a = *reinterpret_cast<const float4*>(&red[0][w][vq * 4]), b = *reinterpret_cast<const float4*>(&red[1][w][vq * 4]);
+    r1.x += a.x; r1.y += a.y; r1.z += a.z; r1.w += a.w;
+    r2.x += b.x; r2.y += b.y; r2.z += b.z; r2.w += b.w;
+  }
+  if (!vin) r1 = r2 = make_float4(0.f, 0.f, 0.f, 0.f);
+  float4 u = make_float4(0.f, 0.f, 0.f, 0.f);
+  if (vin) u = make_float4(beta * (vs[vq * 4] - r1.x), beta * (vs[vq * 4 + 1] - r1.y), beta * (vs[vq * 4 + 2] - r1.z), beta * (vs[vq * 4 + 3] - r1.w));
+#pragma unroll
+  for (int i = 0; i < RPT; ++i) {
+    const int d = dg * RPT + i;
+    if (!vin || d >= g.dkp) continue;
+    const float kd = ks[d] * fk;
+    S[i].x = __builtin_fmaf(kd, u.x, S[i].x); S[i].y = __builtin_fmaf(kd, u.y, S[i].y); S[i].z = __builtin_fmaf(kd, u.z, S[i].z); S[i].w = __builtin_fmaf(kd, u.w, S[i].w);
+    *reinterpret_cast<float4*>(S0 + (size_t)d * g.dvp) = S[i];
+  }
+  if (wave) return;                                  // (VQ <= 64 lanes of the first wave hold every column)
+  float o[4] = {__builtin_fmaf(qk, u.x, r2.x), __builtin_fmaf(qk, u.y, r2.y), __builtin_fmaf(qk, u.z, r2.z), __builtin_fmaf(qk, u.w, r2.w)};
+  float ss = lane < VQ ? (o[0] * o[0] + o[1] * o[1]) + (o[2] * o[2] + o[3] * o[3]) : 0.f;     // (padding columns are zero)
+  ss = wave_sum(ss);
+  const float f = 1.f / sqrtf(ss / (float)g.dv + in.eps);
+  if (lane >= VQ) return;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int v = vq * 4 + i;
+    if (v < g.dv) put1(y + (size_t)row * ldy + h * g.dv + v, o[i] * f * in.norm[v] * sigmoid(in.z[(size_t)row * in.ldz + in.gate + h * g.dv + v]));
+  }
+}
+
+// ---- prompts: the chunks of a ragged batch ------------------------------------------------------------------------------------
+struct ChunkAt { AttnSeg sg; int t0, n; bool ok, last; };     // rows t0 .. + n of the segment
+__device__ __forceinline__ ChunkAt chunk_at(const AttnSeg* segs, int nseg, int c) {
+  for (int i = 0; i < nseg; ++i) {
+    const AttnSeg sg = segs[i];
+    if (sg.n < 2) continue;
+    const int k = ceil_div(sg.n, kC);
+    if (c < k) return ChunkAt{sg, c * kC, min(kC, sg.n - c * kC), true, c == k - 1};
+    c -= k;
+  }
+  return ChunkAt{AttnSeg{0, 0, 0, 0}, 0, 0, false, false};
+}
+
+// factors of a chunk and head, in floats: -W, Q', K' as [dkp / 16] tiles of 16 x 16 (W, Q': token x channel; K': channel x token),
+// exp L_end [dkp], T and P T [16][16]
+struct Factors { float *w, *q, *k, *e, *t, *m; };
+__host__ __device__ __forceinline__ size_t factor_floats(int dkp) { return (size_t)49 * dkp + 512; }
+__device__ __forceinline__ Factors factors_at(float* base, size_t index, int dkp) {
+  float* p = base + index * factor_floats(dkp);
+  return Factors{p, p + 16 * dkp, p + 32 * dkp, p + 48 * dkp, p + 49 * dkp, p + 49 * dkp + 256};
+}
+
+// the input of a convolution `i` rows behind the segment's start (negative: ahead of it)
+__device__ __forceinline__ float conv_in(const DeltaIn& in, const AttnSeg& sg, const float* ring, int taps, int C, int ch, int i) {
+  if (i >= 0) return in.proj[(size_t)(sg.row0 + i) * in.ldp + ch];
+  const int p = sg.pos0 + i;
+  return p >= 0 ? ring[(size_t)(p % taps) * C + ch] : 0.f;
+}
+
+template <int TAPS>
+__global__ __launch_bounds__(256) void delta_factors_kernel(DeltaGeom g, DeltaIn in, const AttnSeg* __restrict__ segs, int nseg, int c0, float* __restrict__ out) {
+  extern __shared__ __attribute__((aligned(16))) float sm[];
+  const int pitch = g.dkp + 4;
+  float *qs = sm, *ks = qs + kC * pitch, *Ls = ks + kC * pitch, *gs = Ls + kC * pitch, *red = gs + kC * pitch;   // red [4][64][8]
+  __shared__ float As[kC][kC + 1], Ps[kC][kC + 1], Ts[kC][kC + 1], Ms[kC][kC + 1], bs[kC], rn[2 * kC];
+  const ChunkAt at = chunk_at(segs, nseg, c0 + blockIdx.x);
+  if (!at.ok) return;
+  const int h = blockIdx.y, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, n = at.n, C = g.channels(), kvh = h / (g.H / g.G);
+  const Factors F = factors_at(out, (size_t)blockIdx.x * g.H + h, g.dkp);
+  const float* ring = in.ring + (size_t)in.slots[at.sg.seq] * g.taps * C;
+  const float* rows = in.proj + (size_t)(at.sg.row0 + at.t0) * in.ldp;
+  // convolutions: a thread walks one channel down the chunk
+  for (int i = tid; i < 2 * g.dkp; i += 256) {
+    const int part = i < g.dkp ? 0 : 1, d = i - part * g.dkp;
+    float* dst = (part ? ks : qs) + d;
+    if (d >= g.dk) {
+      for (int t = 0; t < kC; ++t) dst[t * pitch] = 0.f;
+      continue;
+    }
+    const int ch = (part * g.G + kvh) * g.dk + d;
+    if constexpr (TAPS > 0) {
+      float x[kC + TAPS - 1], w[TAPS];
+#pragma unroll
+      for (int k = 0; k < kC + TAPS - 1; ++k) {
+        const int t = k - (TAPS - 1);
+        x[k] = t < 0 ? conv_in(in, at.sg, ring, TAPS, C, ch, at.t0 + t) : rows[(size_t)min(t, n - 1) * in.ldp + ch];
+      }
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) w[j] = in.conv[(size_t)j * C + ch];
+#pragma unroll
+      for (int t = 0; t < kC; ++t) {
+        float a = 0.f;
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) a = __builtin_fmaf(w[j], x[t + j], a);
+        dst[t * pitch] = t < n ? silu(a) : 0.f;
+      }
+    } else {
+      for (int t = 0; t < kC; ++t) {
+        float a = 0.f;
+        for (int j = 0; j < g.taps; ++j) a = __builtin_fmaf(in.conv[(size_t)j * C + ch], conv_in(in, at.sg, ring, g.taps, C, ch, at.t0 + min(t, n - 1) - (g.taps - 1 - j)), a);
+        dst[t * pitch] = t < n ? silu(a) : 0.f;
+      }
+    }
+  }
+  {
+    const float a_log = in.a_log[h];
+    for (int d = tid; d < g.dkp; d += 256) {
+      float zt[kC];
+#pragma unroll
+      for (int t = 0; t < kC; ++t) zt[t] = d < g.dk ? in.z[(size_t)(at.sg.row0 + at.t0 + min(t, n - 1)) * in.ldz + h * g.dk + d] : 0.f;
+      const float dt = d < g.dk ? in.dt[h * g.dk + d] : 0.f;
+      float L = 0.f;
+#pragma unroll
+      for (int t = 0; t < kC; ++t) {
+        const float lg = d < g.dk && t < n ? log_decay(zt[t], dt, a_log) : 0.f;
+        L += lg;
+        Ls[t * pitch + d] = L;
+        gs[t * pitch + d] = expf(lg);
+      }
+    }
+  }
+  if (tid < kC) bs[tid] = tid < n ? sigmoid(rows[(size_t)tid * in.ldp + in.beta + h]) : 0.f;
+  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const int v = wave * 8 + i;
+    const float* r = (v < kC ? qs : ks) + (v & (kC - 1)) * pitch;
+    float s = 0.f;
+    for (int d = lane; d < g.dkp; d += 64) s = __builtin_fmaf(r[d], r[d], s);
+    s = wave_sum(s);
+    if (lane == 0) rn[v] = 1.f / sqrtf(s + 1e-6f) * (v < kC ? 1.f / sqrtf((float)g.dk) : 1.f);
+  }
+  __syncthreads();
+  for (int i = tid; i < 2 * kC * (g.dkp / 4); i += 256) {
+    const int v = i / (g.dkp / 4), d = (i % (g.dkp / 4)) * 4;
+    float4* r = reinterpret_cast<float4*>((v < kC ? qs : ks) + (v & (kC - 1)) * pitch + d);
+    float4 x = *r;
+    const float f = rn[v];
+    *r = make_float4(x.x * f, x.y * f, x.z * f, x.w * f);
+  }
+  __syncthreads();
+  {   // pairs: lane (I, J) takes tokens 2 I, 2 I + 1 against 2 J, 2 J + 1, a wave a quarter of the channels
+    const int I = lane >> 3, J = lane & 7, i0 = 2 * I, j0 = 2 * J;
+    float a[4] = {0.f, 0.f, 0.f, 0.f}, p[4] = {0.f, 0.f, 0.f, 0.f};        // (i0,j0) (i0,j1) (i1,j0) (i1,j1)
+    if (J <= I) {
+      const bool diag = I == J;
+      for (int d = wave * (g.dkp / 4); d < (wave + 1) * (g.dkp / 4); d += 4) {
+        const float4 ki0 = *reinterpret_cast<const float4*>(ks + i0 * pitch + d), ki1 = *reinterpret_cast<const float4*>(ks + (i0 + 1) * pitch + d);
+        const float4 qi0 = *reinterpret_cast<const float4*>(qs + i0 * pitch + d), qi1 = *reinterpret_cast<const float4*>(qs + (i0 + 1) * pitch + d);
+        const float4 kj0 = *reinterpret_cast<const float4*>(ks + j0 * pitch + d), kj1 = *reinterpret_cast<const float4*>(ks + (j0 + 1) * pitch + d);
+        const float4 Li = *reinterpret_cast<const float4*>(Ls + i0 * pitch + d), Lj = *reinterpret_cast<const float4*>(Ls + (j0 + 1) * pitch + d);
+        const float4 gi = *reinterpret_cast<const float4*>(gs + (i0 + 1) * pitch + d), gj = *reinterpret_cast<const float4*>(gs + (j0 + 1) * pitch + d);
+        auto one = [&](float k0, float k1, float q0, float q1, float c0, float c1, float li, float lj, float g1, float h1) {
+          const float e = diag ? 0.f : __expf(li - lj);
+          const float e01 = e, e11 = diag ? 1.f : e * g1, e00 = diag ? 1.f : e * h1, e10 = e00 * g1;
+          const float x00 = c0 * e00, x01 = c1 * e01, x10 = c0 * e10, x11 = c1 * e11;
+          a[0] = __builtin_fmaf(k0, x00, a[0]); a[1] = __builtin_fmaf(k0, x01, a[1]); a[2] = __builtin_fmaf(k1, x10, a[2]); a[3] = __builtin_fmaf(k1, x11, a[3]);
+          p[0] = __builtin_fmaf(q0, x00, p[0]); p[1] = __builtin_fmaf(q0, x01, p[1]); p[2] = __builtin_fmaf(q1, x10, p[2]); p[3] = __builtin_fmaf(q1, x11, p[3]);
+        };
+        one(ki0.x, ki1.x, qi0.x, qi1.x, kj0.x, kj1.x, Li.x, Lj.x, gi.x, gj.x);
+        one(ki0.y, ki1.y, qi0.y, qi1.y, kj0.y, kj1.y, Li.y, Lj.y, gi.y, gj.y);
+        one(ki0.z, ki1.z, qi0.z, qi1.z, kj0.z, kj1.z, Li.z, Lj.z, gi.z, gj.z);
+        one(ki0.w, ki1.w, qi0.w, qi1.w, kj0.w, kj1.w, Li.w, Lj.w, gi.w, gj.w);
+      }
+    }
+    float4* r = reinterpret_cast<float4*>(red + (wave * 64 + lane) * 8);
+    r[0] = make_float4(a[0], a[1], a[2], a[3]);
+    r[1] = make_float4(p[0], p[1], p[2], p[3]);
+  }
+  __syncthreads();
+  {
+    const int i = tid >> 4, j = tid & 15, at8 = ((i >> 1) * 8 + (j >> 1)) * 8 + (i & 1) * 2 + (j & 1);
+    float a = 0.f, p = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) { a += red[w * 512 + at8]; p += red[w * 512 + at8 + 4]; }
+    As[i][j] = j < i ? a * bs[i] : 0.f;
+    Ps[i][j] = j <= i ? p : 0.f;
+  }
+  __syncthreads();
+  if (wave == 0) {   // (I + A)^-1, a lane per column, by forward substitution
+    float x[kC];
+    const int j = lane & 15;
+#pragma unroll
+    for (int i = 0; i < kC; ++i) {
+      float v = i == j ? 1.f : 0.f;
+#pragma unroll
+      for (int m = 0; m < i; ++m) v = __builtin_fmaf(-As[i][m], x[m], v);
+      x[i] = v;
+    }
+    if (lane < kC) {
+#pragma unroll
+      for (int i = 0; i < kC; ++i) Ts[i][j] = x[i] * bs[j];
+    }
+  } else {           // k exp L and q exp L in place of k and q, K' out
+    for (int d = tid - 64; d < g.dkp; d += 192) {
+      const float end = Ls[(kC - 1) * pitch + d];
+      float* kt = F.k + (d >> 4) * 256 + (d & 15) * 16;
+      float o[kC];
+#pragma unroll
+      for (int t = 0; t < kC; ++t) {
+        const float L = Ls[t * pitch + d], e = expf(L), k = ks[t * pitch + d];
+        o[t] = k * expf(end - L);
+        ks[t * pitch + d] = k * e;
+        qs[t * pitch + d] *= e;
+      }
+#pragma unroll
+      for (int t = 0; t < kC; t += 4) *reinterpret_cast<float4*>(kt + t) = make_float4(o[t], o[t + 1], o[t + 2], o[t + 3]);
+      F.e[d] = expf(end);
+    }
+  }
+  __syncthreads();
+  {
+    const int i = tid >> 4, j = tid & 15;
+    float m = 0.f;
+#pragma unroll
+    for (int k = 0; k < kC; ++k) m = __builtin_fmaf(Ps[i][k], Ts[k][j], m);
+    Ms[i][j] = m;
+    F.t[tid] = Ts[i][j];
+    F.m[tid] = m;
+  }
+  __syncthreads();
+  const int g4 = lane >> 4, c = lane & 15;
+  for (int t = wave; t < g.dkp / 16; t += 4) {
+    f32x4_t w = {0.f, 0.f, 0.f, 0.f}, q = w;
+#pragma unroll
+    for (int s = 0; s < 4; ++s) {
+      const float b = ks[(4 * s + g4) * pitch + 16 * t + c];
+      w = __builtin_amdgcn_mfma_f32_16x16x4f32(Ts[c][4 * s + g4], b, w, 0, 0, 0);
+      q = __builtin_amdgcn_mfma_f32_16x16x4f32(Ms[c][4 * s + g4], b, q, 0, 0, 0);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int i = 4 * g4 + r;
+      F.w[t * 256 + i * 16 + c] = -w[r];
+      F.q[t * 256 + i * 16 + c] = qs[i * pitch + 16 * t + c] - q[r];
+    }
+  }
+}
+
+// One work-group per (head, 16 value columns, segment): the chunks of the segment in order.  A wave holds NT 16-channel tiles of the
+// state as MFMA accumulators, which are the B operands of the next chunk's products as they stand; the partial sums of u and
+// o over the channels meet in LDS, once per chunk.
+template <int NT, int TAPS>
+__global__ __launch_bounds__(256) void delta_scan_kernel(DeltaGeom g, DeltaIn in, const AttnSeg* __restrict__ segs, int nseg, int c0, int c1, int nvt,
+                                                         float* __restrict__ factors, float* __restrict__ o) {
+  __shared__ f32x4_t ps[2][2][4][64];
+  int id = blockIdx.x, h, vt;
+  if (g.H % 8 == 0) {        // the column blocks of a head on one XCD: they read the same factors
+    const int k = id >> 3;
+    h = (id & 7) + 8 * (k / nvt);
+    vt = k % nvt;
+  } else {
+    h = id / nvt;
+    vt = id % nvt;
+  }
+  const int si = blockIdx.y;
+  const AttnSeg sg = segs[si];
+  if (sg.n < 2) return;
+  int first = 0;             // the segment's first chunk among all
+  for (int i = 0; i < si; ++i) first += segs[i].n < 2 ? 0 : ceil_div(segs[i].n, kC);
+  const int k0 = max(c0 - first, 0), k1 = min(c1 - first, ceil_div(sg.n, kC));
+  if (k0 >= k1) return;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g4 = lane >> 4, c = lane & 15;
+  const int tiles = g.dkp / 16, v = vt * 16 + c, slot = in.slots[sg.seq], C = g.channels();
+  const bool vin = v < g.dv;
+  float* S0 = in.state + ((size_t)slot * g.H + h) * g.dkp * g.dvp + v;
+  const float* ring = in.ring + (size_t)slot * g.taps * C;
+  const int ch = 2 * g.G * g.dk + h * g.dv + min(v, g.dv - 1);
+  f32x4_t S[NT];
+  int tile[NT];
+#pragma unroll
+  for (int t = 0; t < NT; ++t) {
+    tile[t] = wave * NT + t;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) S[t][r] = sg.pos0 + k0 > 0 && tile[t] < tiles ? S0[(size_t)(tile[t] * 16 + 4 * g4 + r) * g.dvp] : 0.f;
+  }
+  float cw[TAPS > 0 ? TAPS : 1];
+  if constexpr (TAPS > 0) {
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) cw[j] = in.conv[(size_t)j * C + ch];
+  }
+  struct Frag { f32x4_t w[NT], q[NT], k[NT], e[NT]; float t, m, x[TAPS > 0 ? TAPS : 1]; };
+  auto load = [&](int k, Frag& f) {
+    const Factors F = factors_at(factors, (size_t)(first + k - c0) * g.H + h, g.dkp);
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+      const int tl = min(tile[t], tiles - 1), off = tl * 256 + c * 16 + 4 * g4;     // (past the last tile: S stays zero)
+      f.w[t] = *reinterpret_cast<const f32x4_t*>(F.w + off);
+      f.q[t] = *reinterpret_cast<const f32x4_t*>(F.q + off);
+      f.k[t] = *reinterpret_cast<const f32x4_t*>(F.k + off);
+      f.e[t] = *reinterpret_cast<const f32x4_t*>(F.e + tl * 16 + 4 * g4);
+    }
+    f.t = F.t[c * 16 + 4 * wave + g4];
+    f.m = F.m[c * 16 + 4 * wave + g4];
+    const int tok = min(k * kC + 4 * wave + g4, sg.n - 1);
+    if constexpr (TAPS > 0) {
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) f.x[j] = conv_in(in, sg, ring, TAPS, C, ch, tok - (TAPS - 1 - j));
+    } else {
+      float a = 0.f;
+      for (int j = 0; j < g.taps; ++j) a = __builtin_fmaf(in.conv[(size_t)j * C + ch], conv_in(in, sg, ring, g.taps, C, ch, tok - (g.taps - 1 - j)), a);
+      f.x[0] = a;
+    }
+  };
+  Frag f;
+  load(k0, f);
+  for (int k = k0; k < k1; ++k) {
+    Frag nx;
+    load(min(k + 1, k1 - 1), nx);
+    float x = 0.f;
+    if constexpr (TAPS > 0) {
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) x = __builtin_fmaf(cw[j], f.x[j], x);
+    } else {
+      x = f.x[0];
+    }
+    x = vin && k * kC + 4 * wave + g4 < sg.n ? silu(x) : 0.f;
+    f32x4_t u = {0.f, 0.f, 0.f, 0.f}, ov = u;
+#pragma unroll
+    for (int t = 0; t < NT; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        u = __builtin_amdgcn_mfma_f32_16x16x4f32(f.w[t][r], S[t][r], u, 0, 0, 0);
+        ov = __builtin_amdgcn_mfma_f32_16x16x4f32(f.q[t][r], S[t][r], ov, 0, 0, 0);
+      }
+    u = __builtin_amdgcn_mfma_f32_16x16x4f32(f.t, x, u, 0, 0, 0);
+    ov = __builtin_amdgcn_mfma_f32_16x16x4f32(f.m, x, ov, 0, 0, 0);
+    const int b = k & 1;
+    ps[b][0][wave][lane] = u;
+    ps[b][1][wave][lane] = ov;
+    __syncthreads();
+#pragma unroll
+    for (int t = 0; t < NT; ++t) { S[t][0] *= f.e[t][0]; S[t][1] *= f.e[t][1]; S[t][2] *= f.e[t][2]; S[t][3] *= f.e[t][3]; }
+    u = ps[b][0][0][lane];
+#pragma unroll
+    for (int w = 1; w < 4; ++w) {
+      const f32x4_t a = ps[b][0][w][lane];
+      u[0] += a[0]; u[1] += a[1]; u[2] += a[2]; u[3] += a[3];
+    }
+#pragma unroll
+    for (int t = 0; t < NT; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (tile[t] < tiles) S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.k[t][r], u[r], S[t], 0, 0, 0);
+    {
+      const float* po = reinterpret_cast<const float*>(&ps[b][1][0][0]);
+      const int tok = k * kC + 4 * g4 + wave;
+      float s = 0.f;
+#pragma unroll
+      for (int w = 0; w < 4; ++w) s += po[(w * 64 + lane) * 4 + wave];
+      if (tok < sg.n) o[(size_t)(sg.row0 + tok) * g.H * g.dvp + h * g.dvp + v] = s;
+    }
+    f = nx;
+  }
+#pragma unroll
+  for (int t = 0; t < NT; ++t)
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (tile[t] < tiles) S0[(size_t)(tile[t] * 16 + 4 * g4 + r) * g.dvp] = S[t][r];
+}
+
+// norm and gate, a wave per head and token; the work-groups of a segment's last chunk renew its ring
+template <typename T>
+__global__ __launch_bounds__(256) void delta_out_kernel(DeltaGeom g, DeltaIn in, const AttnSeg* __restrict__ segs, int nseg, int c0, const float* __restrict__ o,
+                                                        T* __restrict__ y, int ldy) {
+  const ChunkAt at = chunk_at(segs, nseg, c0 + blockIdx.x);
+  if (!at.ok) return;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, h = blockIdx.y * 4 + wave;
+  if (h < g.H) {
+    for (int t = 0; t < at.n; ++t) {
+      const size_t row = at.sg.row0 + at.t0 + t;
+      const float* src = o + row * g.H * g.dvp + h * g.dvp;
+      float x[4], ss = 0.f;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int v = lane + 64 * i;
+        x[i] = v < g.dv ? src[v] : 0.f;
+        ss = __builtin_fmaf(x[i], x[i], ss);
+      }
+      const float f = 1.f / sqrtf(wave_sum(ss) / (float)g.dv + in.eps);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int v = lane + 64 * i;
+        if (v < g.dv) put1(y + row * ldy + h * g.dv + v, x[i] * f * in.norm[v] * sigmoid(in.z[row * in.ldz + in.gate + h * g.dv + v]));
+      }
+    }
+  }
+  if (!at.last) return;
+  const int C = g.channels();
+  float* ring = in.ring + (size_t)in.slots[at.sg.seq] * g.taps * C;
+  for (int ch = blockIdx.y * 256 + threadIdx.x; ch < C; ch += gridDim.y * 256)
+    for (int i = max(0, at.sg.n - g.taps); i < at.sg.n; ++i)
+      ring[(size_t)((at.sg.pos0 + i) % g.taps) * C + ch] = in.proj[(size_t)(at.sg.row0 + i) * in.ldp + ch];
+}
+
+int check_in(const DeltaGeom& g, const DeltaIn& in) {
+  MI_CHECK(delta_supported(g), "delta rule: heads must be a multiple of the key heads, head sizes 1 .. 256, 1 .. 16 taps");
+  MI_CHECK(g.dkp % 16 == 0 && g.dkp >= g.dk && g.dkp < g.dk + 16 && g.dvp % 16 == 0 && g.dvp >= g.dv && g.dvp < g.dv + 16, "delta rule: padding");
+  MI_CHECK(in.proj && in.z && in.conv && in.a_log && in.dt && in.norm && in.state && in.ring && in.slots && in.pos, "delta rule: null argument");
+  MI_CHECK(in.beta >= g.channels() && in.ldp >= in.beta + g.H && in.gate >= g.H * g.dk && in.ldz >= in.gate + g.H * g.dv, "delta rule: columns");
+  return MI_OK;
+}
+
+}  // namespace
+
+bool delta_supported(const DeltaGeom& g) {
+  return g.H >= 1 && g.G >= 1 && g.H % g.G == 0 && g.dk >= 1 && g.dk <= 256 && g.dv >= 1 && g.dv <= 256 && g.taps >= 1 && g.taps <= 16;
+}
+size_t delta_factor_floats(const DeltaGeom& g) { return (size_t)g.H * factor_floats(g.dkp); }
+
+int launch_delta_token(const DeltaGeom& g, const DeltaIn& in, int rows, const AttnSeg* segs, void* y, int ldy, bool f32, hipStream_t s) {
+  int rc = check_in(g, in);
+  if (rc != MI_OK) return rc;
+  MI_CHECK(rows >= 1 && rows <= 65535 && y && ldy >= g.H * g.dv, "delta rule: rows");
+  const dim3 grid(g.H, rows);
+  const int vq = g.dvp <= 16 ? 4 : g.dvp <= 32 ? 8 : g.dvp <= 64 ? 16 : g.dvp <= 128 ? 32 : 64, need = ceil_div(g.dkp, kTokenThreads / vq);
+#define MI_DT(VQ, RPT) \
+  if (f32) hipLaunchKernelGGL((delta_token_kernel<float, VQ, RPT>), grid, dim3(kTokenThreads), 0, s, g, in, segs, (float*)y, ldy); \
+  else hipLaunchKernelGGL((delta_token_kernel<uint16_t, VQ, RPT>), grid, dim3(kTokenThreads), 0, s, g, in, segs, (uint16_t*)y, ldy)
+  if (vq == 4) { if (need <= 1) { MI_DT(4, 1); } else { MI_DT(4, 2); } }
+  else if (vq == 8) { if (need <= 1) { MI_DT(8, 1); } else if (need <= 2) { MI_DT(8, 2); } else { MI_DT(8, 4); } }
+  else if (vq == 16) { if (need <= 2) { MI_DT(16, 2); } else if (need <= 4) { MI_DT(16, 4); } else { MI_DT(16, 8); } }
+  else if (vq == 32) { if (need <= 4) { MI_DT(32, 4); } else if (need <= 8) { MI_DT(32, 8); } else { MI_DT(32, 16); } }
+  else { if (need <= 8) { MI_DT(64, 8); } else if (need <= 16) { MI_DT(64, 16); } else { MI_DT(64, 32); } }
+#undef MI_DT
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_delta_prompt(const DeltaGeom& g, const DeltaIn& in, const AttnSeg* sd, const AttnSeg* sh, int nseg, float* factors, int max_chunks,
+                        float* o, void* y, int ldy, bool f32, hipStream_t s) {
+  int rc = check_in(g, in);
+  if (rc != MI_OK) return rc;
+  MI_CHECK(nseg >= 1 && nseg <= 65535 && factors && max_chunks >= 1 && o && y && ldy >= g.H * g.dv, "delta rule: segments / workspace");
+  int chunks = 0;
+  for (int i = 0; i < nseg; ++i) chunks += sh[i].n < 2 ? 0 : ceil_div(sh[i].n, kC);
+  const int nvt = g.dvp / 16, nt = ceil_div(g.dkp / 16, 4);
+  const size_t lds = (size_t)(4 * kC * (g.dkp + 4) + 4 * 64 * 8) * sizeof(float);
+  for (int c0 = 0; c0 < chunks; c0 += max_chunks) {
+    const int n = std::min(max_chunks, chunks - c0);
+    const dim3 gf(n, g.H), gs(g.H * nvt, nseg), go(n, ceil_div(g.H, 4));
+#define MI_DF(TAPS) { \
+    if (lds > 48 * 1024) { rc = ensure_dynamic_lds(reinterpret_cast<const void*>(delta_factors_kernel<TAPS>), (int)lds); if (rc != MI_OK) return rc; } \
+    hipLaunchKernelGGL((delta_factors_kernel<TAPS>), gf, dim3(256), lds, s, g, in, sd, nseg, c0, factors); \
+    if (nt == 1) hipLaunchKernelGGL((delta_scan_kernel<1, TAPS>), gs, dim3(256), 0, s, g, in, sd, nseg, c0, c0 + n, nvt, factors, o); \
+    else if (nt == 2) hipLaunchKernelGGL((delta_scan_kernel<2, TAPS>), gs, dim3(256), 0, s, g, in, sd, nseg, c0, c0 + n, nvt, factors, o); \
+    else if (nt == 3) hipLaunchKernelGGL((delta_scan_kernel<3, TAPS>), gs, dim3(256), 0, s, g, in, sd, nseg, c0, c0 + n, nvt, factors, o); \
+    else hipLaunchKernelGGL((delta_scan_kernel<4, TAPS>), gs, dim3(256), 0, s, g, in, sd, nseg, c0, c0 + n, nvt, factors, o); }
+    switch (g.taps) {
+      case 1: MI_DF(1); break;
+      case 2: MI_DF(2); break;
+      case 3: MI_DF(3); break;
+      case 4: MI_DF(4); break;
+      default: MI_DF(0);
+    }
+#undef MI_DF
+    if (f32) hipLaunchKernelGGL((delta_out_kernel<float>), go, dim3(256), 0, s, g, in, sd, nseg, c0, o, (float*)y, ldy);
+    else hipLaunchKernelGGL((delta_out_kernel<uint16_t>), go, dim3(256), 0, s, g, in, sd, nseg, c0, o, (uint16_t*)y, ldy);
+    MI_HIP(hipGetLastError());
+  }
+  return MI_OK;
+}
+
+}  // namespace mi

@@ -37,24 +37,66 @@ __device__ __forceinline__ float wave_max(float v) {
   for (int m = 32; m >= 1; m >>= 1) v = fmaxf(v, __shfl_xor(v, m));
   return v;
 }
-// The `top` largest of z [E] (LDS; z[E .. E + 3] may be written), by one wave; softmax over them, largest first, ties to the lowest
-// expert.  Up to 256 experts: a logit's place is the number of logits ahead of it; beyond: one maximum after another (z destroyed).
-__device__ __forceinline__ void pick_top(float* z, int E, int top, int32_t* ids, float* weights) {
+// LDS written by some lanes of a wave, read by others of it: a wave's LDS operations execute in order, the compiler must keep them so
+__device__ __forceinline__ void wave_lds_order() {
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+}
+__host__ __device__ __forceinline__ int pick_stride(int E) { return (E + 3) / 4 * 4 + 4; }
+__device__ __forceinline__ float route_sigmoid(float z) { return 1.f / (1.f + expf(-z)); }
+
+// sigmoid rule: z [E] logits -> c [E] choice scores, -inf outside the best groups; gs [groups] is scratch
+__device__ __forceinline__ void choice_scores(const float* z, float* c, float* gs, int E, const RouterRule& rule) {
+  const int lane = threadIdx.x & 63, per = E / rule.groups;
+  for (int e = lane; e < E; e += 64) c[e] = route_sigmoid(z[e]) + rule.b[e];
+  if (rule.groups == 1 || rule.keep == rule.groups) return;
+  wave_lds_order();
+  for (int k = lane; k < rule.groups; k += 64) {
+    float a = -INFINITY, b = -INFINITY;
+    for (int e = k * per; e < (k + 1) * per; ++e) {
+      const float v = c[e];
+      b = fmaxf(b, fminf(a, v));
+      a = fmaxf(a, v);
+    }
+    gs[k] = per > 1 ? a + b : a;
+  }
+  wave_lds_order();
+  for (int e = lane; e < E; e += 64) {
+    const int k = e / per;
+    const float mine = gs[k];
+    int ahead = 0;
+    for (int i = 0; i < rule.groups; ++i) ahead += gs[i] > mine || (gs[i] == mine && i < k) ? 1 : 0;
+    if (ahead >= rule.keep) c[e] = -INFINITY;
+  }
+}
+
+// The `top` best of z [E] (LDS, pick_stride(E) floats and as many for each further array), by one wave; weights, best first, ties to
+// the lowest expert.  Up to 256 experts: an expert's place is the number of experts ahead of it; beyond: one maximum after
+// another (destroys the scores).
+__device__ __forceinline__ void pick_top(float* z, int E, int top, const RouterRule& rule, int32_t* ids, float* weights) {
   const int lane = threadIdx.x & 63;
+  float* c = z;
+  wave_lds_order();
+  if (rule.sigmoid) {
+    c = z + pick_stride(E);
+    choice_scores(z, c, c + pick_stride(E), E, rule);
+    wave_lds_order();
+  }
   if (E <= 256) {
-    if (lane < 4) z[E + lane] = -INFINITY;
+    if (lane < 4) c[E + lane] = -INFINITY;
+    wave_lds_order();
     float v[4], w[4], mx = -INFINITY, sum = 0.f;
     int place[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int e = lane + 64 * i;
-      v[i] = e < E ? z[e] : -INFINITY;
+      v[i] = e < E ? c[e] : -INFINITY;
       if (!(v[i] == v[i])) v[i] = -INFINITY;                    // (a NaN is refused)
       place[i] = e < E ? 0 : 1 << 20;
       mx = fmaxf(mx, v[i]);
     }
     for (int j = 0; j < E; j += 4) {
-      const float4 q = *reinterpret_cast<const float4*>(z + j);
+      const float4 q = *reinterpret_cast<const float4*>(c + j);
       const float u[4] = {q.x, q.y, q.z, q.w};
 #pragma unroll
       for (int k = 0; k < 4; ++k)
@@ -68,10 +110,10 @@ __device__ __forceinline__ void pick_top(float* z, int E, int top, int32_t* ids,
     mx = wave_max(mx);
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      w[i] = place[i] < top ? expf(v[i] - mx) : 0.f;
+      w[i] = place[i] >= top ? 0.f : rule.sigmoid ? route_sigmoid(z[lane + 64 * i]) : expf(v[i] - mx);
       sum += w[i];
     }
-    sum = wave_sum(sum);
+    sum = wave_sum(sum) + (rule.sigmoid ? 1e-20f : 0.f);
 #pragma unroll
     for (int i = 0; i < 4; ++i)
       if (place[i] < top) { ids[place[i]] = lane + 64 * i; weights[place[i]] = w[i] / sum; }
@@ -84,7 +126,7 @@ __device__ __forceinline__ void pick_top(float* z, int E, int top, int32_t* ids,
     float best = -INFINITY;
     int at = 0x7fffffff;
     for (int e = lane; e < E; e += 64)
-      if (z[e] > best) { best = z[e]; at = e; }
+      if (c[e] > best) { best = c[e]; at = e; }
 #pragma unroll
     for (int m = 32; m >= 1; m >>= 1) {
       const float v = __shfl_xor(best, m);
@@ -93,22 +135,23 @@ __device__ __forceinline__ void pick_top(float* z, int E, int top, int32_t* ids,
     }
     if (at >= E) at = j;       // (nothing but -inf or NaN left)
     if (j == 0) first = best;
-    const float w = expf(best - first);
+    const float w = rule.sigmoid ? route_sigmoid(z[at]) : expf(best - first);
     sum += w;
     if (lane == j) { mine = w; mine_id = at; }
-    if (lane == (at & 63)) z[at] = -INFINITY;     // (the lane that reads it)
+    if (lane == (at & 63)) c[at] = -INFINITY;     // (the lane that reads it)
   }
+  if (rule.sigmoid) sum += 1e-20f;
   if (lane < top) { ids[lane] = mine_id; weights[lane] = mine / sum; }
 }
 
 // one work-group per row and kRouteExperts experts, or (no tickets) per row; a wave takes two experts at a time, their rows and x
 // requested together
 template <typename T>
-__global__ __launch_bounds__(256) void route_kernel(const T* __restrict__ x, int ldx, const T* __restrict__ w, const float* __restrict__ b, int E,
+__global__ __launch_bounds__(256) void route_kernel(const T* __restrict__ x, int ldx, const T* __restrict__ w, RouterRule rule, int E,
                                                         int K, int top, int32_t* __restrict__ ids, float* __restrict__ weights, float* __restrict__ zg,
                                                         uint32_t* __restrict__ tickets) {
   constexpr int NW = 4, EPW = 2;
-  extern __shared__ __attribute__((aligned(16))) float z[];   // E floats + 4
+  extern __shared__ __attribute__((aligned(16))) float z[];   // as pick_top
   __shared__ uint32_t arrived;
   const int e0 = blockIdx.y * kRouteExperts, e1 = tickets ? min(e0 + kRouteExperts, E) : E;
   const int t = blockIdx.x, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
@@ -131,7 +174,7 @@ __global__ __launch_bounds__(256) void route_kernel(const T* __restrict__ x, int
       v = lane == i ? s : v;
     }
     if (lane >= EPW || e + lane >= e1) continue;
-    v += b[e + lane];
+    if (!rule.sigmoid) v += rule.b[e + lane];
     if (tickets) __hip_atomic_store(zg + (size_t)t * E + e + lane, v, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
     else z[e + lane] = v;
   }
@@ -145,24 +188,29 @@ __global__ __launch_bounds__(256) void route_kernel(const T* __restrict__ x, int
     if (tid == 0) __hip_atomic_store(tickets + t, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
   }
   __syncthreads();
-  if (wave == 0) pick_top(z, E, top, ids + (size_t)t * top, weights + (size_t)t * top);
+  if (wave == 0) pick_top(z, E, top, rule, ids + (size_t)t * top, weights + (size_t)t * top);
 }
 
 // a wave per row
-__global__ __launch_bounds__(256) void route_pick_kernel(const float* __restrict__ zg, int ldz, int T, int E, int top, int32_t* __restrict__ ids,
+__global__ __launch_bounds__(256) void route_pick_kernel(const float* __restrict__ zg, int ldz, int T, RouterRule rule, int E, int top, int32_t* __restrict__ ids,
                                                          float* __restrict__ weights) {
-  extern __shared__ __attribute__((aligned(16))) float sm[];   // 4 x (E padded to 4, + 4) floats
+  extern __shared__ __attribute__((aligned(16))) float sm[];   // 4 x pick_top's
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, t = blockIdx.x * 4 + wave;
   if (t >= T) return;
-  float* z = sm + wave * ((E + 3) / 4 * 4 + 4);            // (one wave's own: LDS operations of a wave execute in order)
+  float* z = sm + wave * (rule.sigmoid ? 3 : 1) * pick_stride(E);            // (one wave's own: LDS operations of a wave execute in order)
   for (int e = lane; e < E; e += 64) z[e] = zg[(size_t)t * ldz + e];
-  pick_top(z, E, top, ids + (size_t)t * top, weights + (size_t)t * top);
+  pick_top(z, E, top, rule, ids + (size_t)t * top, weights + (size_t)t * top);
+}
+
+__device__ __forceinline__ uint2 relu2x4(f32x4_t v) {
+  auto f = [](float x) { x = fmaxf(x, 0.f); return x * x; };
+  return make_uint2(pack_bf16x2(f(v[0]), f(v[1])), pack_bf16x2(f(v[2]), f(v[3])));
 }
 
 // ---- experts' linear layers, few rows: weight streaming -------------------------------------------------------------------
 // One work-group per (16-row weight tile or KS = 1: four of them, expert).  The pairs that chose the expert are found by a scan
 // over the pair list, in pair order, and taken 16 at a time as the columns of the MFMA tiles.
-template <int KS, bool GLU>
+template <int KS, int ACT>
 __global__ __launch_bounds__(256) void experts_stream_kernel(const uint4* __restrict__ w, int NT, int KT, const int32_t* __restrict__ ids, int P,
                                                              const uint16_t* __restrict__ x, int ldx, int x_div, void* __restrict__ y, int ldy) {
   __shared__ int list[256], count[4];
@@ -221,7 +269,9 @@ __global__ __launch_bounds__(256) void experts_stream_kernel(const uint4* __rest
       }
       if ((KS == 1 || wave == 0) && live && nt < NT) {
         const int n0 = nt * 16 + g4 * 4;
-        if constexpr (GLU) {
+        if constexpr (ACT == EXPERT_RELU2) {
+          *reinterpret_cast<uint2*>(reinterpret_cast<uint16_t*>(y) + (size_t)pair * ldy + n0) = relu2x4(acc);
+        } else if constexpr (ACT == EXPERT_SILU_GLU) {
           const float a0 = acc[0] / (1.f + __expf(-acc[0])) * acc[1], a1 = acc[2] / (1.f + __expf(-acc[2])) * acc[3];
           *reinterpret_cast<uint32_t*>(reinterpret_cast<uint16_t*>(y) + (size_t)pair * ldy + (n0 >> 1)) = pack_bf16x2(a0, a1);
         } else {
@@ -233,9 +283,10 @@ __global__ __launch_bounds__(256) void experts_stream_kernel(const uint4* __rest
 }
 
 // 32-bit form: a wave per output of one pair (for checking)
-template <bool GLU>
+template <int ACT>
 __global__ __launch_bounds__(256) void experts_f32_kernel(const float* __restrict__ w, int N, int K, const int32_t* __restrict__ ids,
                                                           const float* __restrict__ x, int ldx, int x_div, float* __restrict__ y, int ldy) {
+  constexpr bool GLU = ACT == EXPERT_SILU_GLU;
   const int p = blockIdx.x, n = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
   if (n >= (GLU ? N / 2 : N)) return;
   const float *X = x + (size_t)(p / x_div) * ldx, *W = w + ((size_t)ids[p] * N + (GLU ? 2 * n : n)) * K;
@@ -249,6 +300,7 @@ __global__ __launch_bounds__(256) void experts_f32_kernel(const float* __restric
     b = wave_sum(b);
     a = a / (1.f + expf(-a)) * b;
   }
+  if constexpr (ACT == EXPERT_RELU2) { a = fmaxf(a, 0.f); a *= a; }
   if (lane == 0) y[(size_t)p * ldy + n] = a;
 }
 
@@ -295,7 +347,7 @@ __global__ __launch_bounds__(1024) void experts_sort_kernel(const int32_t* __res
 }
 
 // 128 weight rows x BM pairs per work-group, four waves; pairs' rows through swizzled LDS, weights from their tiled image
-template <int BM, bool GLU>
+template <int BM, int ACT>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(BM == 64 ? 4 : 2, BM == 64 ? 4 : 2))) void experts_gemm_kernel(
     const uint4* __restrict__ w, int NT, int KT, ExpertPlan plan, const uint16_t* __restrict__ x, int ldx, int x_div, uint16_t* __restrict__ y, int ldy) {
   constexpr int WM = BM / 64, WN = 4 / WM, NTW = 8 / WN, XL = BM / 32;
@@ -371,7 +423,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(BM == 64 ? 
       if (nt0 + i >= NT) continue;
       const f32x4_t v = acc[i][mt];
       const int n0 = (nt0 + i) * 16 + g * 4;
-      if constexpr (GLU)
+      if constexpr (ACT == EXPERT_RELU2)
+        *reinterpret_cast<uint2*>(row + n0) = relu2x4(v);
+      else if constexpr (ACT == EXPERT_SILU_GLU)
         *reinterpret_cast<uint32_t*>(row + (n0 >> 1)) = pack_bf16x2(v[0] / (1.f + __expf(-v[0])) * v[1], v[2] / (1.f + __expf(-v[2])) * v[3]);
       else
         *reinterpret_cast<uint2*>(row + n0) = make_uint2(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]));
@@ -380,33 +434,37 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(BM == 64 ? 
 }
 
 template <int KS>
-int launch_stream(const ExpertsLinear& w, const int32_t* ids, int P, const uint16_t* x, int ldx, int x_div, bool glu, void* y, int ldy, hipStream_t s) {
+int launch_stream(const ExpertsLinear& w, const int32_t* ids, int P, const uint16_t* x, int ldx, int x_div, int act, void* y, int ldy, hipStream_t s) {
   const int NT = w.N / 16, KT = w.K / 32;
   const dim3 grid(KS == 1 ? ceil_div(NT, 4) : NT, w.E);
-  if (glu) hipLaunchKernelGGL((experts_stream_kernel<KS, true>), grid, dim3(256), 0, s, (const uint4*)w.w, NT, KT, ids, P, x, ldx, x_div, y, ldy);
-  else hipLaunchKernelGGL((experts_stream_kernel<KS, false>), grid, dim3(256), 0, s, (const uint4*)w.w, NT, KT, ids, P, x, ldx, x_div, y, ldy);
+  if (act == EXPERT_SILU_GLU) hipLaunchKernelGGL((experts_stream_kernel<KS, EXPERT_SILU_GLU>), grid, dim3(256), 0, s, (const uint4*)w.w, NT, KT, ids, P, x, ldx, x_div, y, ldy);
+  else if (act == EXPERT_RELU2) hipLaunchKernelGGL((experts_stream_kernel<KS, EXPERT_RELU2>), grid, dim3(256), 0, s, (const uint4*)w.w, NT, KT, ids, P, x, ldx, x_div, y, ldy);
+  else hipLaunchKernelGGL((experts_stream_kernel<KS, EXPERT_LINEAR>), grid, dim3(256), 0, s, (const uint4*)w.w, NT, KT, ids, P, x, ldx, x_div, y, ldy);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
 
 }  // namespace
 
-int launch_route(const void* x, int ldx, int T, const void* w, const float* b, int E, int K, int top, int32_t* ids, float* weights, bool f32, hipStream_t s,
+int launch_route(const void* x, int ldx, int T, const void* w, const RouterRule& rule, int E, int K, int top, int32_t* ids, float* weights, bool f32, hipStream_t s,
                  float* z, uint32_t* tickets) {
   MI_CHECK(T >= 1 && E >= 1 && top >= 1 && top <= E && top <= kMaxTop && K % 64 == 0 && ldx >= K && ldx % 8 == 0, "router: 1 <= top <= min(experts, 64), row stride");
-  const size_t lds = (size_t)(E + 8) * 4;
-  MI_CHECK(E <= 4096, "router: up to 4096 experts");
+  const size_t lds = (size_t)(rule.sigmoid ? 3 : 1) * pick_stride(E) * 4;
+  MI_CHECK(rule.b && E <= (rule.sigmoid ? 1024 : 4096), "router: up to 4096 experts, 1024 with the sigmoid rule");
+  MI_CHECK(rule.groups >= 1 && E % rule.groups == 0 && rule.keep >= 1 && rule.keep <= rule.groups, "router: groups");
   MI_CHECK(!tickets || z, "router: tickets without logits");
   const dim3 grid(T, tickets ? ceil_div(E, kRouteExperts) : 1);
-  if (f32) hipLaunchKernelGGL((route_kernel<float>), grid, dim3(256), lds, s, (const float*)x, ldx, (const float*)w, b, E, K, top, ids, weights, z, tickets);
-  else hipLaunchKernelGGL((route_kernel<uint16_t>), grid, dim3(256), lds, s, (const uint16_t*)x, ldx, (const uint16_t*)w, b, E, K, top, ids, weights, z, tickets);
+  if (f32) hipLaunchKernelGGL((route_kernel<float>), grid, dim3(256), lds, s, (const float*)x, ldx, (const float*)w, rule, E, K, top, ids, weights, z, tickets);
+  else hipLaunchKernelGGL((route_kernel<uint16_t>), grid, dim3(256), lds, s, (const uint16_t*)x, ldx, (const uint16_t*)w, rule, E, K, top, ids, weights, z, tickets);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
 
-int launch_route_pick(const float* z, int ldz, int T, int E, int top, int32_t* ids, float* weights, hipStream_t s) {
-  MI_CHECK(T >= 1 && E >= 1 && E <= 4096 && top >= 1 && top <= E && top <= kMaxTop && ldz >= E, "router: experts / top");
-  hipLaunchKernelGGL(route_pick_kernel, dim3(ceil_div(T, 4)), dim3(256), (size_t)16 * (E + 8), s, z, ldz, T, E, top, ids, weights);
+int launch_route_pick(const float* z, int ldz, int T, const RouterRule& rule, int E, int top, int32_t* ids, float* weights, hipStream_t s) {
+  MI_CHECK(T >= 1 && E >= 1 && E <= (rule.sigmoid ? 1024 : 4096) && top >= 1 && top <= E && top <= kMaxTop && ldz >= E, "router: experts / top");
+  MI_CHECK((!rule.sigmoid || rule.b) && rule.groups >= 1 && E % rule.groups == 0 && rule.keep >= 1 && rule.keep <= rule.groups, "router: groups");
+  const size_t lds = (size_t)4 * (rule.sigmoid ? 3 : 1) * pick_stride(E) * 4;
+  hipLaunchKernelGGL(route_pick_kernel, dim3(ceil_div(T, 4)), dim3(256), lds, s, z, ldz, T, rule, E, top, ids, weights);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
@@ -422,34 +480,36 @@ int launch_experts_sort(const ExpertPlan& plan, const int32_t* ids, int P, int E
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
-int launch_experts_gemm(const ExpertsLinear& w, const ExpertPlan& plan, int P, const uint16_t* x, int ldx, int x_div, bool glu, uint16_t* y, int ldy, hipStream_t s) {
+int launch_experts_gemm(const ExpertsLinear& w, const ExpertPlan& plan, int P, const uint16_t* x, int ldx, int x_div, int act, uint16_t* y, int ldy, hipStream_t s) {
   MI_CHECK(w.E >= 1 && w.N % 16 == 0 && w.K % 64 == 0 && ldx >= w.K && ldx % 8 == 0 && P >= 1 && x_div >= 1, "experts: shape");
-  MI_CHECK(ldy % 4 == 0 && ldy >= (glu ? w.N / 2 : w.N), "experts: output stride");
+  MI_CHECK(ldy % 4 == 0 && ldy >= (act == EXPERT_SILU_GLU ? w.N / 2 : w.N), "experts: output stride");
   const int NT = w.N / 16, KT = w.K / 32;
   const dim3 grid((unsigned)(plan.max_tiles * ceil_div(NT, 8)));
   const uint4* W = reinterpret_cast<const uint4*>(w.w);
 #define MI_EG(BM) \
-  if (glu) hipLaunchKernelGGL((experts_gemm_kernel<BM, true>), grid, dim3(256), 0, s, W, NT, KT, plan, x, ldx, x_div, y, ldy); \
-  else hipLaunchKernelGGL((experts_gemm_kernel<BM, false>), grid, dim3(256), 0, s, W, NT, KT, plan, x, ldx, x_div, y, ldy)
+  if (act == EXPERT_SILU_GLU) hipLaunchKernelGGL((experts_gemm_kernel<BM, EXPERT_SILU_GLU>), grid, dim3(256), 0, s, W, NT, KT, plan, x, ldx, x_div, y, ldy); \
+  else if (act == EXPERT_RELU2) hipLaunchKernelGGL((experts_gemm_kernel<BM, EXPERT_RELU2>), grid, dim3(256), 0, s, W, NT, KT, plan, x, ldx, x_div, y, ldy); \
+  else hipLaunchKernelGGL((experts_gemm_kernel<BM, EXPERT_LINEAR>), grid, dim3(256), 0, s, W, NT, KT, plan, x, ldx, x_div, y, ldy)
   if (plan.block == 128) { MI_EG(128); } else { MI_EG(64); }
 #undef MI_EG
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
 
-int launch_experts_linear(const ExpertsLinear& w, const int32_t* ids, int P, const void* x, int ldx, int x_div, bool glu, void* y, int ldy,
+int launch_experts_linear(const ExpertsLinear& w, const int32_t* ids, int P, const void* x, int ldx, int x_div, int act, void* y, int ldy,
                           bool f32, hipStream_t s) {
   MI_CHECK(w.E >= 1 && w.E <= 65535 && w.N % 16 == 0 && w.K % 64 == 0 && ldx >= w.K && ldx % 8 == 0 && P >= 1 && x_div >= 1, "experts: shape");
-  MI_CHECK(ldy % 4 == 0 && ldy >= (glu ? w.N / 2 : w.N), "experts: output stride");
+  MI_CHECK(ldy % 4 == 0 && ldy >= (act == EXPERT_SILU_GLU ? w.N / 2 : w.N), "experts: output stride");
   if (f32) {
-    const dim3 grid(P, ceil_div(glu ? w.N / 2 : w.N, 4));
-    if (glu) hipLaunchKernelGGL((experts_f32_kernel<true>), grid, dim3(256), 0, s, (const float*)w.w, w.N, w.K, ids, (const float*)x, ldx, x_div, (float*)y, ldy);
-    else hipLaunchKernelGGL((experts_f32_kernel<false>), grid, dim3(256), 0, s, (const float*)w.w, w.N, w.K, ids, (const float*)x, ldx, x_div, (float*)y, ldy);
+    const dim3 grid(P, ceil_div(act == EXPERT_SILU_GLU ? w.N / 2 : w.N, 4));
+    if (act == EXPERT_RELU2) hipLaunchKernelGGL((experts_f32_kernel<EXPERT_RELU2>), grid, dim3(256), 0, s, (const float*)w.w, w.N, w.K, ids, (const float*)x, ldx, x_div, (float*)y, ldy);
+    else if (act == EXPERT_SILU_GLU) hipLaunchKernelGGL((experts_f32_kernel<EXPERT_SILU_GLU>), grid, dim3(256), 0, s, (const float*)w.w, w.N, w.K, ids, (const float*)x, ldx, x_div, (float*)y, ldy);
+    else hipLaunchKernelGGL((experts_f32_kernel<EXPERT_LINEAR>), grid, dim3(256), 0, s, (const float*)w.w, w.N, w.K, ids, (const float*)x, ldx, x_div, (float*)y, ldy);
     MI_HIP(hipGetLastError());
     return MI_OK;
   }
-  return w.K / 32 >= 16 ? launch_stream<4>(w, ids, P, (const uint16_t*)x, ldx, x_div, glu, y, ldy, s)
-                        : launch_stream<1>(w, ids, P, (const uint16_t*)x, ldx, x_div, glu, y, ldy, s);
+  return w.K / 32 >= 16 ? launch_stream<4>(w, ids, P, (const uint16_t*)x, ldx, x_div, act, y, ldy, s)
+                        : launch_stream<1>(w, ids, P, (const uint16_t*)x, ldx, x_div, act, y, ldy, s);
 }
 
 }  // namespace mi

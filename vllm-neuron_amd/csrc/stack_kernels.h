@@ -9,8 +9,8 @@ namespace mi {
 
 struct AttnSeg { int row0, n, pos0, seq; };   // rows row0 .. + n of the batch = positions pos0 .. of the sequence in block-table row seq
 
-// resid[t, :] = E[ids[t], :] (+ P[pos[t], :], ptable not null) in fp32, also to x0 when given; columns D .. ld - 1 are zero
-int launch_embed_pos(const int32_t* ids, const int32_t* pos, const void* table, const void* ptable, bool f32, int T,
+// resid[t, :] = scale E[ids[t], :] (+ P[pos[t], :], ptable not null) in fp32, also to x0 when given; columns D .. ld - 1 are zero
+int launch_embed_pos(const int32_t* ids, const int32_t* pos, const void* table, const void* ptable, float scale, bool f32, int T,
                      int D, int ld, float* resid, float* x0, hipStream_t s);
 
 struct NormOut {
@@ -25,7 +25,7 @@ int launch_layernorm_rows(const float* resid_in, float* resid_out, int T, int D,
 
 // ---- sandwich blocks: x <- x + post_norm(sublayer output); h = pre_norm(x); a = h + causal convolution of h ----------
 // Norms are RMS norms over `groups` equal parts of the row, each over its own sqrt(mean square + eps).
-// A sublayer's output, in whatever form the sublayer leaves it:
+// A sublayer's output, in whatever form the sublayer leaves it (slabs and pairs: their sum):
 struct RowSource {
   const float* y = nullptr;        // [T, ld] fp32 ...
   const uint16_t* y16 = nullptr;   // ... or (experts) bf16
@@ -44,13 +44,20 @@ struct ConvState {
   int block_size = 0, MB = 0;
   const int32_t *bt = nullptr, *pos = nullptr, *slots = nullptr;
 };
-// resid_out = resid_in (+ post-normed src); then, with w_pre, y [T, ldy] = h in the compute type, or (conv, every row its own
+// resid_out = resid_in (+ post-normed src; w_post null: + src as it is); then, with w_pre, y [T, ldy] = h in the compute type, or (conv, every row its own
 // sequence: block-table row = row) a with the state read and renewed.  Without w_pre only the residual sum.
 int launch_sandwich_rows(const float* resid_in, float* resid_out, const RowSource& src, const float* w_post, const float* w_pre, int T,
                          int D, int ld, int groups, float eps, const ConvState* conv, void* y, int ldy, bool f32, hipStream_t s);
 // a = h + conv(h) over a ragged batch: h [T, ldy] as launch_sandwich_rows leaves it
 int launch_conv_rows(const void* h, const ConvState& conv, const AttnSeg* segs_dev, const AttnSeg* segs_host, int nseg, int D, int ld,
                      void* y, int ldy, bool f32, hipStream_t s);
+
+// y [T, ldy] = columns col .. col + n of x [T, ld] fp32 in the compute type, zeros behind them; w [n]: over their root mean square, times w
+int launch_columns(const float* x, int ld, int col, int n, const float* w, float eps, int T, void* y, int ldy, bool f32, hipStream_t s);
+// y[t, h dv + d] *= sigmoid(g[t, ...]): one gate per head, or (per_element) per element; g [T, ldg] fp32, y [T, ldy] in the compute type
+int launch_gate_rows(void* y, int ldy, int T, int H, int dv, const float* g, int ldg, bool per_element, bool f32, hipStream_t s);
+// dst = src + offset
+int launch_offset_copy(const float* src, int n, float offset, float* dst, hipStream_t s);
 
 // y[t] = [x ; x0] in the compute type, the second half at column half
 int launch_pair_rows(const float* x, const float* x0, int T, int D, int ld, int half, void* y, bool f32, hipStream_t s);

@@ -34,7 +34,7 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
 
 template <typename T>
 __global__ __launch_bounds__(256) void embed_pos_kernel(const int32_t* __restrict__ ids, const int32_t* __restrict__ pos,
-                                                        const T* __restrict__ table, const T* __restrict__ ptable, int D, int ld,
+                                                        const T* __restrict__ table, const T* __restrict__ ptable, float sc, int D, int ld,
                                                         float* __restrict__ resid, float* __restrict__ x0) {
   const int t = blockIdx.x;
   const T* e = table + (size_t)ids[t] * D;
@@ -44,18 +44,11 @@ __global__ __launch_bounds__(256) void embed_pos_kernel(const int32_t* __restric
     if ((D & 3) == 0) {
       if (d < D) {
         const float4 a = get4(e + d), b = p ? get4(p + d) : make_float4(0.f, 0.f, 0.f, 0.f);
-        v = make_float4(a.x + b.x, a.y + b.y, a.z + b.z, a.w + b.w);
+        v = make_float4(__builtin_fmaf(sc, a.x, b.x), __builtin_fmaf(sc, a.y, b.y), __builtin_fmaf(sc, a.z, b.z), __builtin_fmaf(sc, a.w, b.w));
       }
-    } else if (!p) {
-      if (d < D) v.x = to_f32(e[d]);
-      if (d + 1 < D) v.y = to_f32(e[d + 1]);
-      if (d + 2 < D) v.z = to_f32(e[d + 2]);
-      if (d + 3 < D) v.w = to_f32(e[d + 3]);
     } else {
-      if (d < D) v.x = to_f32(e[d]) + to_f32(p[d]);
-      if (d + 1 < D) v.y = to_f32(e[d + 1]) + to_f32(p[d + 1]);
-      if (d + 2 < D) v.z = to_f32(e[d + 2]) + to_f32(p[d + 2]);
-      if (d + 3 < D) v.w = to_f32(e[d + 3]) + to_f32(p[d + 3]);
+      auto at = [&](int i) { return d + i < D ? __builtin_fmaf(sc, to_f32(e[d + i]), p ? to_f32(p[d + i]) : 0.f) : 0.f; };
+      v = make_float4(at(0), at(1), at(2), at(3));
     }
     *reinterpret_cast<float4*>(resid + (size_t)t * ld + d) = v;
     if (x0) *reinterpret_cast<float4*>(x0 + (size_t)t * ld + d) = v;
@@ -151,7 +144,8 @@ __device__ __forceinline__ float4 source_row4(const RowSource& src, int t, int d
     }
     const float4 sc = *reinterpret_cast<const float4*>(src.slabs.scale + d);
     v.x *= sc.x; v.y *= sc.y; v.z *= sc.z; v.w *= sc.w;
-  } else if (src.pair_w) {
+  }
+  if (src.pair_w) {
     for (int j = 0; j < src.top; ++j) {
       const size_t r = (size_t)t * src.top + j;
       const float w = src.pair_w[r];
@@ -159,7 +153,7 @@ __device__ __forceinline__ float4 source_row4(const RowSource& src, int t, int d
       v.x = __builtin_fmaf(w, q.x, v.x); v.y = __builtin_fmaf(w, q.y, v.y);
       v.z = __builtin_fmaf(w, q.z, v.z); v.w = __builtin_fmaf(w, q.w, v.w);
     }
-  } else {
+  } else if (!src.slabs.slab) {
     v = *reinterpret_cast<const float4*>(src.y + (size_t)t * src.ld + d);
   }
   return v;
@@ -197,13 +191,17 @@ __global__ __launch_bounds__(1024) void sandwich_rows_kernel(const float* __rest
   const size_t o = (size_t)t * ld;
   const float inv_gs = 1.0f / (float)(D / G);
   const bool add = src.any();
-  if (add) {
+  if (add && w_post) {
     for (int d = tid * 4; d < ld; d += nthr * 4) *reinterpret_cast<float4*>(row + d) = source_row4(src, t, d);
     group_rstd(row, D, G, eps, red, rstd);
   }
   for (int d = tid * 4; d < ld; d += nthr * 4) {   // (a thread reads back what it wrote itself)
     float4 x = *reinterpret_cast<const float4*>(resid_in + o + d);
-    if (add) {
+    if (add && !w_post) {
+      const float4 v = source_row4(src, t, d);
+      x = make_float4(x.x + v.x, x.y + v.y, x.z + v.z, x.w + v.w);
+      *reinterpret_cast<float4*>(resid_out + o + d) = x;
+    } else if (add) {
       const float4 v = *reinterpret_cast<const float4*>(row + d), w = *reinterpret_cast<const float4*>(w_post + d), r = part_rstd(rstd, d, G, inv_gs);
       x.x = __builtin_fmaf(v.x * r.x, w.x, x.x); x.y = __builtin_fmaf(v.y * r.y, w.y, x.y);
       x.z = __builtin_fmaf(v.z * r.z, w.z, x.z); x.w = __builtin_fmaf(v.w * r.w, w.w, x.w);
@@ -248,7 +246,7 @@ __global__ __launch_bounds__(1024) void sandwich_token_kernel(const float* __res
   const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
   float4 x = *reinterpret_cast<const float4*>(resid_in + (size_t)t * ld + dd);
   float4 v = add ? source_row4(src, t, dd) : zero;
-  const float4 wp = add ? *reinterpret_cast<const float4*>(w_post + dd) : zero, wn = *reinterpret_cast<const float4*>(w_pre + dd);
+  const float4 wp = add && w_post ? *reinterpret_cast<const float4*>(w_post + dd) : zero, wn = *reinterpret_cast<const float4*>(w_pre + dd);
   float4 w[TAPS > 0 ? TAPS : 1];
   raw_t past[TAPS > 1 ? TAPS - 1 : 1];
   int slot = -1;
@@ -273,7 +271,10 @@ __global__ __launch_bounds__(1024) void sandwich_token_kernel(const float* __res
     for (int k = 0; k < wpg; ++k) sum += r[g0 + k];
     return 1.0f / sqrtf(sum / (float)gs + eps);
   };
-  if (add) {
+  if (add && !w_post) {
+    x = make_float4(x.x + v.x, x.y + v.y, x.z + v.z, x.w + v.w);
+    if (in) *reinterpret_cast<float4*>(resid_out + (size_t)t * ld + d) = x;
+  } else if (add) {
     const float r = rstd(in ? v : zero, red[0]);
     x.x = __builtin_fmaf(v.x * r, wp.x, x.x); x.y = __builtin_fmaf(v.y * r, wp.y, x.y);
     x.z = __builtin_fmaf(v.z * r, wp.z, x.z); x.w = __builtin_fmaf(v.w * r, wp.w, x.w);
@@ -403,6 +404,36 @@ __global__ __launch_bounds__(256) void conv_rows_kernel(const T* __restrict__ hi
     const int stop = min(end, (shared_block + 1) * bs);
     for (int p = max(sg.pos0, stop - cs.keep); p < stop; ++p) renew(p, get(hs + (size_t)(p - sg.pos0) * ldy));
   }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void columns_kernel(const float* __restrict__ x, int ld, int n, const float* __restrict__ w, float eps,
+                                                      T* __restrict__ y, int ldy) {
+  __shared__ float red[4];
+  const float* src = x + (size_t)blockIdx.x * ld;
+  const int tid = threadIdx.x;
+  float f = 1.f;
+  if (w) {
+    float ss = 0.f;
+    for (int d = tid; d < n; d += 256) ss = __builtin_fmaf(src[d], src[d], ss);
+    f = 1.0f / sqrtf(block_sum(ss, red) / (float)n + eps);
+  }
+  for (int d = tid * 4; d < ldy; d += 1024) {
+    auto at = [&](int i) { return d + i < n ? src[d + i] * f * (w ? w[d + i] : 1.f) : 0.f; };
+    put4(y + (size_t)blockIdx.x * ldy + d, at(0), at(1), at(2), at(3));
+  }
+}
+__device__ __forceinline__ void gate1(uint16_t* p, float g) { *p = f32_to_bf16(bf16_to_f32(*p) * g); }
+__device__ __forceinline__ void gate1(float* p, float g) { *p *= g; }
+template <typename T, bool ELEM>
+__global__ __launch_bounds__(256) void gate_rows_kernel(T* __restrict__ y, int ldy, int n, int dv, const float* __restrict__ g, int ldg) {
+  const int t = blockIdx.x;
+  for (int i = blockIdx.y * 256 + threadIdx.x; i < n; i += gridDim.y * 256)
+    gate1(y + (size_t)t * ldy + i, 1.f / (1.f + expf(-g[(size_t)t * ldg + (ELEM ? i : i / dv)])));
+}
+__global__ void offset_copy_kernel(const float* __restrict__ src, int n, float offset, float* __restrict__ dst) {
+  const int i = blockIdx.x * blockDim.x + threadIdx.x;
+  if (i < n) dst[i] = src[i] + offset;
 }
 
 template <typename T>
@@ -554,12 +585,12 @@ __global__ void pack_rows_kernel(const float* __restrict__ src, int ld_src, int 
 
 }  // namespace
 
-int launch_embed_pos(const int32_t* ids, const int32_t* pos, const void* table, const void* ptable, bool f32, int T, int D,
+int launch_embed_pos(const int32_t* ids, const int32_t* pos, const void* table, const void* ptable, float scale, bool f32, int T, int D,
                      int ld, float* resid, float* x0, hipStream_t s) {
   if (f32)
-    hipLaunchKernelGGL((embed_pos_kernel<float>), dim3(T), dim3(256), 0, s, ids, pos, (const float*)table, (const float*)ptable, D, ld, resid, x0);
+    hipLaunchKernelGGL((embed_pos_kernel<float>), dim3(T), dim3(256), 0, s, ids, pos, (const float*)table, (const float*)ptable, scale, D, ld, resid, x0);
   else
-    hipLaunchKernelGGL((embed_pos_kernel<uint16_t>), dim3(T), dim3(256), 0, s, ids, pos, (const uint16_t*)table, (const uint16_t*)ptable, D, ld, resid, x0);
+    hipLaunchKernelGGL((embed_pos_kernel<uint16_t>), dim3(T), dim3(256), 0, s, ids, pos, (const uint16_t*)table, (const uint16_t*)ptable, scale, D, ld, resid, x0);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
@@ -590,7 +621,7 @@ static int check_conv(const ConvState& c) {
 int launch_sandwich_rows(const float* resid_in, float* resid_out, const RowSource& src, const float* w_post, const float* w_pre, int T,
                          int D, int ld, int groups, float eps, const ConvState* conv, void* y, int ldy, bool f32, hipStream_t s) {
   MI_CHECK(T >= 1 && ld % 4 == 0 && ld >= D && ld <= 32768 && groups >= 1 && D % groups == 0, "sandwich rows: row stride / norm groups");
-  MI_CHECK(!src.any() || (resid_out && resid_out != resid_in && w_post), "sandwich rows: residual output / post-norm weight");
+  MI_CHECK(!src.any() || (resid_out && resid_out != resid_in), "sandwich rows: residual output");
   MI_CHECK(!src.slabs.slab || (src.slabs.T == T && src.slabs.N == ld && !src.slabs.bias && !src.slabs.row_scale), "sandwich rows: pending K-split sum of another shape");
   MI_CHECK(src.slabs.slab || !src.any() || src.ld >= ld, "sandwich rows: source stride");
   MI_CHECK(!src.y16 || src.pair_w, "sandwich rows: bf16 sources are built for experts");
@@ -648,6 +679,33 @@ int launch_conv_rows(const void* h, const ConvState& conv, const AttnSeg* sd, co
     default: MI_CONV(0, kConvRows);
   }
 #undef MI_CONV
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_columns(const float* x, int ld, int col, int n, const float* w, float eps, int T, void* y, int ldy, bool f32, hipStream_t s) {
+  MI_CHECK(T >= 1 && n >= 1 && col >= 0 && ld >= col + n && ldy >= n && ldy % 4 == 0, "columns: strides");
+  if (f32) hipLaunchKernelGGL((columns_kernel<float>), dim3(T), dim3(256), 0, s, x + col, ld, n, w, eps, (float*)y, ldy);
+  else hipLaunchKernelGGL((columns_kernel<uint16_t>), dim3(T), dim3(256), 0, s, x + col, ld, n, w, eps, (uint16_t*)y, ldy);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_gate_rows(void* y, int ldy, int T, int H, int dv, const float* g, int ldg, bool per_element, bool f32, hipStream_t s) {
+  const int n = H * dv;
+  MI_CHECK(T >= 1 && H >= 1 && dv >= 1 && ldy >= n && ldg >= (per_element ? n : H), "gate rows: strides");
+  const dim3 grid(T, std::min(ceil_div(n, 256), 16));
+  if (f32 && per_element) hipLaunchKernelGGL((gate_rows_kernel<float, true>), grid, dim3(256), 0, s, (float*)y, ldy, n, dv, g, ldg);
+  else if (f32) hipLaunchKernelGGL((gate_rows_kernel<float, false>), grid, dim3(256), 0, s, (float*)y, ldy, n, dv, g, ldg);
+  else if (per_element) hipLaunchKernelGGL((gate_rows_kernel<uint16_t, true>), grid, dim3(256), 0, s, (uint16_t*)y, ldy, n, dv, g, ldg);
+  else hipLaunchKernelGGL((gate_rows_kernel<uint16_t, false>), grid, dim3(256), 0, s, (uint16_t*)y, ldy, n, dv, g, ldg);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+
+int launch_offset_copy(const float* src, int n, float offset, float* dst, hipStream_t s) {
+  MI_CHECK(n >= 1, "offset copy: size");
+  hipLaunchKernelGGL(offset_copy_kernel, dim3(ceil_div(n, 256)), dim3(256), 0, s, src, n, offset, dst);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }

@@ -11,6 +11,8 @@ import json
 import os
 from types import SimpleNamespace
 
+from .._stack_enums import MI_MIX
+from .bokulorn import BokulornConfig
 from .rapodra import RapodraConfig
 from .vimesun import VimesunConfig
 
@@ -19,7 +21,7 @@ MULTI_MODAL_MODELS = [f"{family}ForConditionalGeneration" for family in ("Mllama
 
 LLAMA_FAMILY = ("LlamaForCausalLM", "Qwen2ForCausalLM", "MistralForCausalLM")
 # architecture name -> reader of its config.json dictionary
-STACK_DESIGNS = {design.architecture: design.from_dict for design in (VimesunConfig, RapodraConfig)}
+STACK_DESIGNS = {design.architecture: design.from_dict for design in (VimesunConfig, RapodraConfig, BokulornConfig)}
 SUPPORTED_ARCHITECTURES = LLAMA_FAMILY + tuple(STACK_DESIGNS)
 
 
@@ -44,3 +46,20 @@ def load_config(model_dir: str):
 def stack_of(config) -> dict | None:
     """The library's description of a layer-stack model; None for the Llama family."""
     return getattr(config, "stack", None)
+
+
+def has_recurrent_state(config) -> bool:
+    """Whether a sequence owns state that is not in KV blocks (a slot per sequence; no prefix to be taken over from the cache)."""
+    stack = stack_of(config)
+    return stack is not None and any(x.get("mixer_kind") == MI_MIX["delta"] for x in stack["layers"])
+
+
+def fill_sizes(config, shape_of) -> None:
+    """Sizes a design's config.json leaves to the checkpoint: `shape_of`(tensor name) -> its shape, or None."""
+    for (layer, name), tensor in getattr(config, "sizes_from", {}).items():
+        if config.stack["layers"][layer].get(name):
+            continue
+        shape = shape_of(tensor)
+        if shape is None:
+            raise ValueError(f"{config.architecture}: tensor {tensor}, whose shape gives {name} of layer {layer}, is not in the checkpoint")
+        config.stack["layers"][layer][name] = int(shape[0])

@@ -17,6 +17,7 @@ import os
 from typing import TYPE_CHECKING
 
 from ._vllm_compat import Platform, PlatformEnum
+from .models import has_recurrent_state
 
 if TYPE_CHECKING:  # pragma: no cover
     from vllm.config import ModelConfig, ParallelConfig, VllmConfig
@@ -120,6 +121,11 @@ class MI355XPlatform(Platform):
                         cache_config.num_gpu_blocks_override, cache_config.num_gpu_blocks_override + 1)
             cache_config.num_gpu_blocks_override += 1
             setattr(cache_config, _NULL_BLOCK_MARK, True)
+
+        if cache_config and cache_config.enable_prefix_caching and has_recurrent_state(vllm_config.model_config.hf_config):
+            # the state behind a cached prefix is not kept: every prompt is computed from its first token
+            logger.info("prefix caching switched off: the model's sequences own recurrent state")
+            cache_config.enable_prefix_caching = False
 
         parallel_config = vllm_config.parallel_config
         if parallel_config.worker_cls == "auto":

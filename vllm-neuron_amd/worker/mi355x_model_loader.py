@@ -36,7 +36,7 @@ import torch
 import torch.nn as nn
 
 from .._vllm_compat import SamplerOutput
-from ..models import stack_of
+from ..models import fill_sizes, has_recurrent_state, stack_of
 from .constants import (MI355X_MULTI_MODAL_MODELS, SUPPORTED_ARCHITECTURES,
                         TORCH_DTYPE_TO_MI355X_AMP)
 
@@ -118,6 +118,7 @@ class MI355XCausalLM(MI355XModelBase):
     """`forward` = one call of libmi355x_vllm's mi_forward (reference loader.py:336-365)."""
 
     draft = None     # NativeModel of the draft model when fused speculation is on
+    recurrent = False    # sequences own state slots (models/__init__.py: has_recurrent_state)
     _draft_catchup: dict = {}    # sequence id -> (position of its next step, token the draft has not seen)
 
     def _remask_fused_spec_output(self, fused, inputs):
@@ -194,7 +195,7 @@ class MI355XCausalLM(MI355XModelBase):
     def forward(self, input_ids, input_block_ids, **kwargs):
         cfg = self.mi355x_config
         if cfg.get("chunked_prefill_config") is not None:
-            return self._forward_chunked(input_ids, **kwargs)
+            return self._forward_chunked(input_ids, input_block_ids=input_block_ids, **kwargs)
         with self._reordered(input_block_ids, input_ids=input_ids, **kwargs) as (seq_ids, inputs, restore):
             ids = inputs["input_ids"]
             if cfg.is_block_kv_layout:
@@ -236,11 +237,12 @@ class MI355XCausalLM(MI355XModelBase):
         cfg = self.mi355x_config
         args = (input_ids, inputs["position_ids"], inputs["slot_mapping"], inputs["block_tables"],
                 inputs["full_context_lens"], inputs["computed_context_lens"])
+        seq_ids = inputs.get("input_block_ids") if self.recurrent else None
         if cfg.on_device_sampling_config:
             self._sample_calls += 1
             return self.model.forward_chunked(*args, sampling_params=inputs.get("sampling_params"),
-                                              seed=(self._sample_seed << 32) + self._sample_calls, tokens=True)
-        return self.model.forward_chunked(*args)
+                                              seed=(self._sample_seed << 32) + self._sample_calls, tokens=True, seq_ids=seq_ids)
+        return self.model.forward_chunked(*args, seq_ids=seq_ids)
 
     def _batch_line_addressing(self, seq_ids, position_ids, full_context_lens, computed, S):
         """Contiguous ('batch line') KV expressed through the block pool: sequence id s owns
@@ -261,7 +263,8 @@ class MI355XCausalLM(MI355XModelBase):
         """Logits of chosen places of one ragged token batch (indices into it), nothing sampled."""
         return self.model.forward_rows(model_input.input_tokens, model_input.position_ids, model_input.slot_mapping,
                                        model_input.block_tables, model_input.full_context_lens,
-                                       model_input.computed_context_lens, rows)
+                                       model_input.computed_context_lens, rows,
+                                       seq_ids=model_input.input_block_ids if self.recurrent else None)
 
     def sample(self, logits: torch.Tensor) -> SamplerOutput | None:
         if self.mi355x_config.on_device_sampling_config:
@@ -274,6 +277,9 @@ class MI355XCausalLM(MI355XModelBase):
         from .._native import NativeModel
         cfg: dict = kwargs["mi355x_config"]
         hf = self.hf_config
+        if getattr(hf, "sizes_from", None):
+            fill_sizes(hf, _checkpoint_shapes(model_name_or_path, cfg))
+        self.recurrent = has_recurrent_state(hf)
         geo = _model_geometry(hf, cfg)
         max_model_len = cfg["seq_len"]
         if cfg["is_block_kv_layout"]:
@@ -300,6 +306,8 @@ class MI355XCausalLM(MI355XModelBase):
             # the reference compiles a batch-1 model over max_num_batched_tokens (loader.py:734-736);
             # the ragged batch here holds up to chunked_prefill_config.max_num_seqs requests
             max_num_seqs = int(getattr(chunked, "max_num_seqs", None) or cfg.get("scheduler_max_num_seqs") or max_num_seqs)
+            if self.recurrent:      # (the library's rows are its state slots too)
+                max_num_seqs = max(max_num_seqs, int(cfg.get("scheduler_max_num_seqs") or 0))
             buckets = sorted(set(buckets + [int(cfg["max_context_length"])]))
         speculative_config = kwargs.get("speculative_config")
         fused_spec = bool(cfg.get("enable_fused_speculation"))
@@ -308,6 +316,9 @@ class MI355XCausalLM(MI355XModelBase):
             if spec_len < 1 or speculative_config is None or chunked or not cfg["is_block_kv_layout"]:
                 raise NotImplementedError("fused speculation needs num_speculative_tokens >= 1, a draft model, the block "
                                           "KV layout (prefix caching on) and no chunked prefill")
+            if self.recurrent:
+                raise NotImplementedError("fused speculation: a target with recurrent state is not built (its state cannot be "
+                                          "taken back to the last accepted token)")
             check_draft(stack_of(speculative_config.draft_model_config.hf_config))
             if "stack" in geo and geo["stack"].get("conv_taps", 0) > 1:
                 geo["stack"]["state_lookahead"] = spec_len - 1
@@ -500,10 +511,23 @@ class MI355XCausalLM(MI355XModelBase):
 
 
 def check_draft(stack: dict | None) -> None:
-    """The draft's chained steps run one row per sequence with a catch-up row beside it; a convolution's state would need
-    them in order."""
-    if stack is not None and stack.get("conv_taps", 0) > 1:
-        raise NotImplementedError("fused speculation: a draft model with convolution state is not built")
+    """The draft's chained steps run one row per sequence with a catch-up row beside it; a convolution's or a recurrence's
+    state would need them in order."""
+    if stack is not None and (stack.get("conv_taps", 0) > 1 or has_recurrent_state(SimpleNamespace(stack=stack))):
+        raise NotImplementedError("fused speculation: a draft model with sequence state beside its KV blocks is not built")
+
+
+def _checkpoint_shapes(path: str, cfg: dict):
+    """Tensor name -> shape, from the in-memory weights or the safetensors files' headers."""
+    if cfg.get("state_dict") is not None:
+        shapes = {n: tuple(t.shape) for n, t in cfg["state_dict"].items()}
+    else:
+        from safetensors import safe_open
+        shapes = {}
+        for f in sorted(glob.glob(os.path.join(path, "*.safetensors"))) if path else []:
+            with safe_open(f, "pt") as sf:
+                shapes.update({name: tuple(sf.get_slice(name).get_shape()) for name in sf.keys()})
+    return shapes.get
 
 
 def _model_geometry(hf, cfg: dict) -> dict:

@@ -259,6 +259,10 @@ class MI355XModelRunner:
             self.requests.pop(req_id, None)
         for req_id in scheduler_output.finished_req_ids:
             self.input_batch.remove_request(req_id)
+        if self.is_chunked_prefill:
+            # (state slots of recurrent models; a preempted request starts over from its first token)
+            for req_id in (*scheduler_output.finished_req_ids, *(getattr(scheduler_output, "preempted_req_ids", None) or ())):
+                self._release_state_slot(req_id)
         scheduled = scheduler_output.num_scheduled_tokens.keys()
         for req_id in self.input_batch.req_id_to_index.keys() - scheduled:
             self.input_batch.remove_request(req_id)
@@ -397,21 +401,46 @@ class MI355XModelRunner:
         either the next chunk of a prompt or the single next token of a request that generates."""
         data = IntermediateInputData()
         num_scheduled = scheduler_output.num_scheduled_tokens
+        scheduled = num_scheduled if getattr(self.model, "recurrent", False) else None
         for request_data in scheduler_output.scheduled_new_reqs:
             if request_data.mm_features:
                 raise NotImplementedError("multimodal inputs are not supported on the MI355X plugin")
             assert len(request_data.block_ids) == 1
             self._append_chunk(data, request_data.req_id, request_data.prompt_token_ids, [],
                                request_data.block_ids[0], request_data.num_computed_tokens,
-                               num_scheduled[request_data.req_id])
+                               num_scheduled[request_data.req_id], scheduled)
         cached = scheduler_output.scheduled_cached_reqs
         for i, req_id in enumerate(cached.req_ids):
             state = self.requests[req_id]
             self._append_chunk(data, req_id, state.prompt_token_ids, state.output_token_ids, state.block_ids[0],
-                               cached.num_computed_tokens[i], num_scheduled[req_id])
+                               cached.num_computed_tokens[i], num_scheduled[req_id], scheduled)
         return data
 
-    def _append_chunk(self, data: IntermediateInputData, req_id, prompt, outputs, block_table, start, n) -> None:
+    def _release_state_slot(self, req_id) -> None:
+        slot = self.vllm_req_to_seq_id_mapping.pop(req_id, None)
+        if slot is not None:
+            self.free_seq_ids.add(slot)
+
+    def _state_slot(self, req_id, start, scheduled) -> int:
+        """The slot a request's recurrent state lives in: taken with its first token, kept until it ends.  A scheduler that does
+        not report preemptions leaves slots with requests that will start over; when all are taken, one of a request that is
+        not in this step goes (should that request continue after all, it is refused below)."""
+        slots = self.vllm_req_to_seq_id_mapping
+        if req_id in slots:
+            return slots[req_id]
+        if start > 0:
+            raise RuntimeError(f"request {req_id} continues at token {start} but its recurrent state is not held any more")
+        if not self.free_seq_ids:
+            idle = next((r for r in reversed(slots) if r not in scheduled), None)
+            if idle is None:
+                raise RuntimeError("more requests in one step than state slots")
+            self._release_state_slot(idle)
+        slots[req_id] = slot = min(self.free_seq_ids)
+        self.free_seq_ids.remove(slot)
+        return slot
+
+    def _append_chunk(self, data: IntermediateInputData, req_id, prompt, outputs, block_table, start, n,
+                      scheduled=None) -> None:
         end = start + n
         data.request_ids.append(req_id)
         # tokens start .. end-1 of the sequence (prompt, then what was generated so far)
@@ -421,7 +450,7 @@ class MI355XModelRunner:
             seq = list(prompt) + list(outputs)
             data.input_tokens.extend(seq[start:end])
         data.position_ids.extend(range(start, end))
-        data.input_block_ids.append(0)
+        data.input_block_ids.append(0 if scheduled is None else self._state_slot(req_id, start, scheduled))
         bs = self.cache_config.block_size
         data.slot_mapping.extend(block_table[i // bs] * bs + i % bs for i in range(start, end))
         data.block_tables.append(list(block_table))
@@ -437,7 +466,8 @@ class MI355XModelRunner:
         return ModelInputForMI355X(
             request_ids=data.request_ids, input_tokens=input_tokens,
             position_ids=torch.tensor(data.position_ids, dtype=torch.long).reshape(1, -1),
-            input_block_ids=torch.tensor(data.input_block_ids[:1], dtype=torch.long),
+            input_block_ids=torch.tensor(data.input_block_ids if getattr(self.model, "recurrent", False) else data.input_block_ids[:1],
+                                         dtype=torch.long),
             slot_mapping=torch.tensor(data.slot_mapping, dtype=torch.long), block_tables=block_tables,
             full_context_lens=torch.tensor(data.full_context_lens, dtype=torch.long),
             computed_context_lens=torch.tensor(data.computed_context_lens, dtype=torch.long),

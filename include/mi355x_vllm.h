@@ -462,20 +462,30 @@ int mi_op_sandwich_rows(const float* resid_in, float* resid_out, const float* y,
                         const float* w_pre, int32_t T, int32_t D, int32_t ld, int32_t groups, float eps, const float* conv_w, int32_t taps,
                         void* ring, int32_t keep, int32_t block_size, const int32_t* block_table, int32_t MB, const int32_t* pos,
                         const int32_t* slots, const int32_t* segs_host, int32_t nseg, void* out, int32_t ldy, int32_t f32, void* stream);
-/* qd [T, ldq] fp32 = [q heads | W_dkv h] -> q [T, H, pad32(dk)]; with c_norm [kv_rank] the RMS-normed latent into pool
- * [blocks][block_size][pad32(kv_rank)] at slots (-1: skip) */
-int mi_op_latent_scatter(const float* qd, int32_t ldq, int32_t T, const mi_layer_spec* spec, const float* c_norm, float eps, const int32_t* slots,
-                         int32_t block_size, void* q, void* pool, int32_t f32, void* stream);
+/* qd [T, ldq] fp32 = [q heads | W_dkv h] -> q [T, H, pad32(dk + rot_dim)]; with c_norm [kv_rank] the RMS-normed latent and the rotated
+ * key part into pool [blocks][block_size][pad32(kv_rank) + pad32(rot_dim)] at slots (-1: skip).  rot [positions][rot_dims / 2][2]: cosines and
+ * sines, pos [T]; both NULL without a rotated part */
+int mi_op_latent_scatter(const float* qd, int32_t ldq, int32_t T, const mi_layer_spec* spec, const float* rot, const int32_t* pos, const float* c_norm,
+                         float eps, const int32_t* slots, int32_t block_size, void* q, void* pool, int32_t f32, void* stream);
+/* Gated delta rule of a ragged batch (spec: MI_MIX_DELTA).  proj [T, ldp] fp32: [q | k | v] at column 0, beta's projection at column beta; z
+ * [T, ldz]: decays at column 0, output gates at column gate; conv [taps][channels]; state [num_slots][H][pad16(dk)][pad16(dv)], ring
+ * [num_slots][taps][channels], row p % taps = the inputs of position p.  slots_host: slot of every block-table row (segs_host's last column; nseg = 0: of
+ * every row, token generation).  max_chunks: chunks of 16 tokens whose factors are kept at a time.  out [T, ldo] in the compute type. */
+int mi_op_delta_rule(const mi_layer_spec* spec, const float* proj, int32_t ldp, int32_t beta, const float* z, int32_t ldz, int32_t gate, const float* conv,
+                     const float* a_log, const float* dt, const float* norm, float eps, float* state, float* ring, int32_t num_slots,
+                     const int32_t* slots_host, const int32_t* pos_host, const int32_t* segs_host, int32_t nseg, int32_t T, int32_t max_chunks,
+                     void* out, int32_t ldo, int32_t f32, void* stream);
 /* Latent attention of a ragged batch over that pool: uk [H dk, rank], uv [H dv, rank] fp32.  path: 1 plain, 2 rows in the latent space,
  * 3 keys and values written out (segments of two rows and more).  out [T, H v_dim] (row stride ldo). */
 int mi_op_latent_attn(const mi_layer_spec* spec, const float* uk, const float* uv, const void* q, const void* pool, int32_t block_size,
                       const int32_t* block_table, int32_t MB, const int32_t* pos, const int32_t* segs_host, int32_t nseg, int32_t T,
                       int32_t max_ctx, void* out, int32_t ldo, int32_t f32, int32_t path, void* stream);
 /* Router and experts: x [T, ldx]; router [E, D], router_b [E], gate / up [E, ff, D], down [E, D, ff] fp32 -> ids, weights [T, top],
- * y [T top, ldy] fp32 = every pair's expert output, unweighted.  path: 1 weight streaming (or fp32), 2 pairs grouped by expert. */
+ * y [T top, ldy] fp32 = every pair's expert output, unweighted.  path: 1 weight streaming (or fp32), 2 pairs grouped by expert.
+ * groups > 0: the sigmoid rule over that many groups, `keep` of them eligible, router_b its correction; squared-relu experts, gate NULL. */
 int mi_op_experts(const void* x, int32_t ldx, int32_t T, int32_t D, int32_t experts, int32_t top, int32_t ff, const float* router, const float* router_b,
-                  const float* gate, const float* up, const float* down, int32_t* ids, float* weights, float* y, int32_t ldy, int32_t f32, int32_t path,
-                  void* stream);
+                  const float* gate, const float* up, const float* down, int32_t* ids, float* weights, float* y, int32_t ldy, int32_t groups, int32_t keep,
+                  int32_t f32, int32_t path, void* stream);
 
 #ifdef __cplusplus
 }

@@ -157,7 +157,7 @@ def test_latent_norm_and_scatter(lib, H, dk, rank, f32):
     q = torch.full((T, H, pad(dk, 32)), 7.0, dtype=dt, device="cuda")
     pool = torch.full((nb * bs, pad(rank, 32)), 7.0, dtype=dt, device="cuda")
     a = [dev(t) for t in (qd, cn, slots)]
-    lib.check(lib.load_library().mi_op_latent_scatter(ptr(a[0]), ldq, T, spec_of(lib, H, dk, 8, rank, 4, 1.0), ptr(a[1]), 1e-3, ptr(a[2]), bs,
+    lib.check(lib.load_library().mi_op_latent_scatter(ptr(a[0]), ldq, T, spec_of(lib, H, dk, 8, rank, 4, 1.0), None, None, ptr(a[1]), 1e-3, ptr(a[2]), bs,
                                                       ptr(q), ptr(pool), f32, None))
     torch.cuda.synchronize()
     tol = 1e-5 if f32 else 1.2e-2
@@ -332,7 +332,7 @@ def test_router_and_experts(lib, T, D, E, top, ff, f32, path):
     y = torch.zeros(T * top, ldy, device="cuda")
     for _ in range(2):                        # (the second call finds what the first left behind, as a layer's next step does)
         lib.check(lib.load_library().mi_op_experts(ptr(a[0]), Kd, T, D, E, top, ff, ptr(a[1]), ptr(a[2]), ptr(a[3]), ptr(a[4]), ptr(a[5]),
-                                                   ptr(ids), ptr(p), ptr(y), ldy, f32, path, None))
+                                                   ptr(ids), ptr(p), ptr(y), ldy, 0, 0, f32, path, None))
     torch.cuda.synchronize()
     ref_ids, ref_p = R.route(x.double(), w.double(), b.double(), top)
     assert torch.equal(ids.cpu().long(), ref_ids)
@@ -354,7 +354,7 @@ def test_router_prefers_the_lower_of_equal_experts(lib):
         ids, p = torch.full((T, 4), -1, dtype=torch.int32, device="cuda"), torch.zeros(T, 4, device="cuda")
         y = torch.zeros(T * 4, D, device="cuda")
         lib.check(lib.load_library().mi_op_experts(ptr(a[0]), 64, T, D, E, 4, 16, ptr(a[1]), ptr(a[2]), ptr(a[3]), ptr(a[4]), ptr(a[5]), ptr(ids),
-                                                   ptr(p), ptr(y), D, 0, path, None))
+                                                   ptr(p), ptr(y), D, 0, 0, 0, path, None))
         torch.cuda.synchronize()
         assert ids.cpu().tolist() == [[0, 1, 2, 3]] * T and torch.allclose(p.cpu(), torch.full((T, 4), 0.25))
 

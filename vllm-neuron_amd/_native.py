@@ -130,11 +130,13 @@ _SIGS = {
     "mi_op_sandwich_rows": (C.c_int, [C.c_void_p] * 4 + [C.c_int32] + [C.c_void_p] * 2 + [C.c_int32] * 4 + [C.c_float, C.c_void_p, C.c_int32,
                                       C.c_void_p, C.c_int32, C.c_int32, C.c_void_p, C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p,
                                       C.c_int32, C.c_void_p, C.c_int32, C.c_int32, C.c_void_p]),
-    "mi_op_latent_scatter": (C.c_int, [C.c_void_p, C.c_int32, C.c_int32, C.POINTER(MiLayerSpec), C.c_void_p, C.c_float, C.c_void_p,
+    "mi_op_latent_scatter": (C.c_int, [C.c_void_p, C.c_int32, C.c_int32, C.POINTER(MiLayerSpec), C.c_void_p, C.c_void_p, C.c_void_p, C.c_float, C.c_void_p,
                                        C.c_int32, C.c_void_p, C.c_void_p, C.c_int32, C.c_void_p]),
     "mi_op_latent_attn": (C.c_int, [C.POINTER(MiLayerSpec)] + [C.c_void_p] * 4 + [C.c_int32, C.c_void_p, C.c_int32, C.c_void_p, C.c_void_p,
                                     C.c_int32, C.c_int32, C.c_int32, C.c_void_p, C.c_int32, C.c_int32, C.c_int32, C.c_void_p]),
-    "mi_op_experts": (C.c_int, [C.c_void_p] + [C.c_int32] * 6 + [C.c_void_p] * 8 + [C.c_int32] * 3 + [C.c_void_p]),
+    "mi_op_experts": (C.c_int, [C.c_void_p] + [C.c_int32] * 6 + [C.c_void_p] * 8 + [C.c_int32] * 5 + [C.c_void_p]),
+    "mi_op_delta_rule": (C.c_int, [C.POINTER(MiLayerSpec), C.c_void_p, C.c_int32, C.c_int32, C.c_void_p, C.c_int32, C.c_int32] + [C.c_void_p] * 4
+                         + [C.c_float, C.c_void_p, C.c_void_p, C.c_int32] + [C.c_void_p] * 3 + [C.c_int32] * 3 + [C.c_void_p, C.c_int32, C.c_int32, C.c_void_p]),
     "mi_forward_spec": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int32, C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p,
                                   C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p]),
     "mi_replay_decode": (C.c_int, [C.c_void_p, C.c_int32, C.POINTER(C.c_float)]),

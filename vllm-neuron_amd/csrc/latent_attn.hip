@@ -30,10 +30,19 @@ struct QdRow {
   }
 };
 
+// element d of a query head with its last nr elements rotated, at(i) the unrotated ones (rotate-half pairs)
+template <typename F>
+__device__ __forceinline__ float rotated(int i, int dims, const float2* cs, F at) {
+  if (i >= dims) return at(i);
+  const int half = dims >> 1;
+  if (i < half) return at(i) * cs[i].x - at(i + half) * cs[i].y;
+  return at(i) * cs[i - half].x + at(i - half) * cs[i - half].y;
+}
+
 // one latent (columns c0 .. of the row) over its root mean square times c_norm, into its pool row; 256 threads
 template <typename T>
-__device__ __forceinline__ void latent_norm_row(const QdRow& row, int c0, const LatentGeom& g, const float* __restrict__ c_norm, float eps, int slot,
-                                                T* __restrict__ pool, float* red) {
+__device__ __forceinline__ void latent_norm_row(const QdRow& row, int c0, const LatentGeom& g, const float2* cs, const float* __restrict__ c_norm, float eps,
+                                                int slot, T* __restrict__ pool, float* red) {
   const int tid = threadIdx.x;
   float ss = 0.f;
   for (int d = tid; d < g.rank; d += 256) { const float v = row.at(c0 + d); ss = __builtin_fmaf(v, v, ss); }
@@ -42,30 +51,41 @@ __device__ __forceinline__ void latent_norm_row(const QdRow& row, int c0, const 
   __syncthreads();
   const float f = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)g.rank + eps);
   if (slot < 0) return;
-  T* dst = pool + (size_t)slot * g.rp;        // (a block's rows are consecutive: slot = block * block_size + offset)
+  T* dst = pool + (size_t)slot * g.cp;        // (a block's rows are consecutive: slot = block * block_size + offset)
   for (int d = tid * 4; d < g.rp; d += 1024) {
     auto at = [&](int i) { return d + i < g.rank ? row.at(c0 + d + i) * f * c_norm[d + i] : 0.f; };
     put4(dst + d, make_float4(at(0), at(1), at(2), at(3)));
+  }
+  for (int d = tid * 4; d < g.cp - g.rp; d += 1024) {
+    auto at = [&](int i) { return d + i < g.nr ? rotated(d + i, g.dims, cs, [&](int k) { return row.at(c0 + g.rank + k); }) : 0.f; };
+    put4(dst + g.rp + d, make_float4(at(0), at(1), at(2), at(3)));
   }
 }
 
 // blockIdx.y < q groups: 8 heads of 32 lanes each; the last one: the latent, one work-group per row
 template <typename T>
-__global__ __launch_bounds__(256) void latent_scatter_kernel(const float* __restrict__ qd, int ldq, SlabSum sl, LatentGeom g, const float* __restrict__ c_norm,
+__global__ __launch_bounds__(256) void latent_scatter_kernel(LatentRowsIn in, SlabSum sl, LatentGeom g, Rotation rot, const float* __restrict__ c_norm,
                                                              float eps, const int32_t* __restrict__ slots, int bs, T* __restrict__ q,
                                                              T* __restrict__ pool) {
   __shared__ float red[4];
   const int t = blockIdx.x, tid = threadIdx.x;
-  const QdRow row{sl.slab ? sl.slab + (size_t)t * sl.N : qd + (size_t)t * ldq, sl};
+  const QdRow row{sl.slab ? sl.slab + (size_t)t * sl.N : in.q + (size_t)t * in.ldq, sl};
+  const float2* cs = g.nr ? rot.table + (size_t)rot.pos[t] * (g.dims / 2) : nullptr;
   if ((int)blockIdx.y < ceil_div(g.H, 8)) {
     const int h = blockIdx.y * 8 + (tid >> 5);
     if (h >= g.H) return;
-    const int c0 = h * g.dk;
+    const int c0 = h * (g.dk + g.nr);
     T* dst = q + ((size_t)t * g.H + h) * g.dkp;
-    const bool vec = (g.dk & 3) == 0;
+    const bool vec = ((g.dk | g.nr) & 3) == 0;
     for (int d = (tid & 31) * 4; d < g.dkp; d += 128) {
       float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
-      if (vec) {
+      if (d + 3 >= g.dk && g.nr) {
+        auto at = [&](int i) {
+          if (d + i < g.dk) return row.at(c0 + d + i);
+          return d + i < g.dk + g.nr ? rotated(d + i - g.dk, g.dims, cs, [&](int k) { return row.at(c0 + g.dk + k); }) : 0.f;
+        };
+        v = make_float4(at(0), at(1), at(2), at(3));
+      } else if (vec) {
         if (d < g.dk) v = row.at4(c0 + d);
       } else {
         if (d < g.dk) v.x = row.at(c0 + d);
@@ -77,7 +97,8 @@ __global__ __launch_bounds__(256) void latent_scatter_kernel(const float* __rest
     }
     return;
   }
-  latent_norm_row(row, g.H * g.dk, g, c_norm, eps, slots[t], pool, red);
+  if (sl.slab) { latent_norm_row(row, g.H * (g.dk + g.nr), g, cs, c_norm, eps, slots[t], pool, red); return; }
+  latent_norm_row(QdRow{in.lat + (size_t)t * in.ldl, sl}, 0, g, cs, c_norm, eps, slots[t], pool, red);
 }
 
 struct RowAt { int row, seq; };
@@ -125,21 +146,29 @@ __global__ __launch_bounds__(256) void head_linear_kernel(const uint4* __restric
 
 // Token generation: W_uk^T q straight from the projection's fp32 rows (rounded to bf16 on the way, as latent_scatter_kernel
 // leaves q), and the latents' norm and scatter in the same launch: blockIdx.y < H a head, = H the latents of row blockIdx.x.
-__global__ __launch_bounds__(256) void latent_token_kernel(const float* __restrict__ qd, int ldq, LatentGeom g, const uint4* __restrict__ w_uk, int rows,
+__global__ __launch_bounds__(256) void latent_token_kernel(LatentRowsIn in, LatentGeom g, Rotation rot, const uint4* __restrict__ w_uk, int rows,
                                                            const float* __restrict__ c_norm, float eps, const int32_t* __restrict__ slots,
                                                            uint16_t* __restrict__ qa, uint16_t* __restrict__ pool) {
   __shared__ float red[4];
   const int h = blockIdx.y;
   if (h == g.H) {
     const SlabSum none;
-    if ((int)blockIdx.x < rows) latent_norm_row(QdRow{qd + (size_t)blockIdx.x * ldq, none}, g.H * g.dk, g, c_norm, eps, slots[blockIdx.x], pool, red);
+    const int t = blockIdx.x;
+    if (t < rows)
+      latent_norm_row(QdRow{in.lat + (size_t)t * in.ldl, none}, 0, g, g.nr ? rot.table + (size_t)rot.pos[t] * (g.dims / 2) : nullptr, c_norm, eps, slots[t], pool, red);
     return;
   }
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, g4 = lane >> 4, c = lane & 15;
-  const int NT = g.rp / 16, KT = g.dkp / 32, ntg = ceil_div(NT, 4), tt = blockIdx.x / ntg, nt = (blockIdx.x % ntg) * 4 + wave, m = tt * 16 + c;
+  const int NT = g.cp / 16, KT = g.dkp / 32, ntg = ceil_div(NT, 4), tt = blockIdx.x / ntg, nt = (blockIdx.x % ntg) * 4 + wave, m = tt * 16 + c;
   if (tt * 16 >= rows || nt >= NT) return;
   const u32x4_t* W = reinterpret_cast<const u32x4_t*>(w_uk) + ((size_t)h * NT + nt) * KT * 64 + lane;
-  const float* X = qd + (size_t)min(m, rows - 1) * ldq + (size_t)h * g.dk + g4 * 8;
+  const float* X0 = in.q + (size_t)min(m, rows - 1) * in.ldq + (size_t)h * (g.dk + g.nr);
+  const float* X = X0 + g4 * 8;
+  const float2* cs = g.nr ? rot.table + (size_t)rot.pos[min(m, rows - 1)] * (g.dims / 2) : nullptr;
+  auto turned = [&](int d) {          // four elements of the rotated part
+    auto at = [&](int i) { return rotated(d - g.dk + i, g.dims, cs, [&](int k) { return X0[g.dk + k]; }); };
+    return make_float4(at(0), at(1), at(2), at(3));
+  };
   f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
   for (int k0 = 0; k0 < KT; k0 += 4) {       // (past the last tile: the last one's weights against zeros)
     u32x4_t a[4], x[4];
@@ -149,13 +178,15 @@ __global__ __launch_bounds__(256) void latent_token_kernel(const float* __restri
       float4 x0 = make_float4(0.f, 0.f, 0.f, 0.f), x1 = x0;
       const int d = (k0 + u) * 32 + g4 * 8;
       if (d < g.dk) x0 = *reinterpret_cast<const float4*>(X + (k0 + u) * 32);
+      else if (d < g.dk + g.nr) x0 = turned(d);
       if (d + 4 < g.dk) x1 = *reinterpret_cast<const float4*>(X + (k0 + u) * 32 + 4);
+      else if (d + 4 < g.dk + g.nr) x1 = turned(d + 4);
       x[u] = u32x4_t{pack_bf16x2(x0.x, x0.y), pack_bf16x2(x0.z, x0.w), pack_bf16x2(x1.x, x1.y), pack_bf16x2(x1.z, x1.w)};
     }
 #pragma unroll
     for (int u = 0; u < 4; ++u) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a[u]), __builtin_bit_cast(bf16x8_t, x[u]), acc, 0, 0, 0);
   }
-  if (m < rows) put4(qa + ((size_t)m * g.H + h) * g.rp + nt * 16 + g4 * 4, make_float4(acc[0], acc[1], acc[2], acc[3]));
+  if (m < rows) put4(qa + ((size_t)m * g.H + h) * g.cp + nt * 16 + g4 * 4, make_float4(acc[0], acc[1], acc[2], acc[3]));
 }
 
 __global__ __launch_bounds__(64) void head_linear_f32_kernel(const float* __restrict__ w, int H, int N, int K, const float* __restrict__ x,
@@ -182,15 +213,16 @@ __device__ __forceinline__ float fexp2(float x) { return __builtin_amdgcn_exp2f(
 __device__ __forceinline__ float sexp2(float x, float m) { return (x == -INFINITY) ? 0.f : fexp2(x - m); }
 
 constexpr int kCPitch = 16;
-template <int RP, int HG>
-constexpr size_t latent_lds() { return (size_t)64 * (RP + kCPitch) * 2 + (HG == 1 ? 0 : (size_t)HG * RP * 32) + (size_t)HG * 4 * 64 * 8 + (size_t)HG * 4 * 16 * 4; }
+template <int RP, int RX, int HG>
+constexpr size_t latent_lds() { return (size_t)64 * (RP + RX + kCPitch) * 2 + (HG == 1 ? 0 : (size_t)HG * (RP + RX) * 32) + (size_t)HG * 4 * 64 * 8 + (size_t)HG * 4 * 16 * 4; }
 
-template <int RP, int HG, bool FINAL>
+// RX: columns of the rotated part (behind the latent's RP in LDS; scores only)
+template <int RP, int RX, int HG, bool FINAL>
 __global__ __launch_bounds__(256, HG == 1 ? 2 : 1) void latent_rows_kernel(LatentGeom g, float sc2, int window, const uint16_t* __restrict__ qa,
                                                           const uint16_t* __restrict__ pool, int bs, const int32_t* __restrict__ bt, int MB,
                                                           const int32_t* __restrict__ pos, LatentRows lr, int NS, int bs_shift, float* __restrict__ o_part,
                                                           float* __restrict__ ml_part, uint16_t* __restrict__ lat) {
-  constexpr int CP = RP + kCPitch, KS = RP / 32, DN = RP / 64, CCH = RP / 8, NL = 64 * CCH / 256;
+  constexpr int CP = RP + RX + kCPitch, KS = (RP + RX) / 32, DN = RP / 64, CCH = RP / 8, NL = 64 * CCH / 256, NX = RX / 32;
   extern __shared__ __attribute__((aligned(16))) unsigned char dsm[];
   uint16_t* Cs = reinterpret_cast<uint16_t*>(dsm);                        // [64][CP]
   u32x4_t* Qs = reinterpret_cast<u32x4_t*>(Cs + 64 * CP);                 // [HG][KS][64 lanes]; one head group: in registers
@@ -204,7 +236,7 @@ __global__ __launch_bounds__(256, HG == 1 ? 2 : 1) void latent_rows_kernel(Laten
   const int t0 = t_lo + split * per, t1 = min(t0 + per, t_hi);
   const int last_ch = g.rp / 8 - 1;
 
-  u32x4_t cr[NL];
+  u32x4_t cr[NL], xr[NX > 0 ? NX : 1];     // (rotated part: eight chunks a row, row tid / 8 + 32 i)
   // (addresses: a uniform part per 16-token group and a per-lane part that never changes, as in window_attn.hip)
   int blk[4], off[4];
   auto fetch_ids = [&](int tt) {     // the block of every 16-token group (block_size is a multiple of 16); past the keys: the null block
@@ -220,16 +252,21 @@ __global__ __launch_bounds__(256, HG == 1 ? 2 : 1) void latent_rows_kernel(Laten
     }
   };
   constexpr int R = 256 / CCH;       // rows of a load
-  const int row0 = tid / CCH, lane_off = (row0 & 15) * g.rp + min(tid % CCH, last_ch) * 8;
+  const int row0 = tid / CCH, lane_off = (row0 & 15) * g.cp + min(tid % CCH, last_ch) * 8;
+  const int x_off = ((tid >> 3) & 15) * g.cp + g.rp + min((tid & 7) * 8, g.cp - g.rp - 8);
   auto issue = [&]() {               // the tile whose ids fetch_ids loaded last
     const uint16_t* base[4];
 #pragma unroll
-    for (int u = 0; u < 4; ++u) base[u] = pool + ((size_t)blk[u] * bs + off[u]) * g.rp;
+    for (int u = 0; u < 4; ++u) base[u] = pool + ((size_t)blk[u] * bs + off[u]) * g.cp;
 #pragma unroll
     for (int i = 0; i < NL; ++i) {
       const uint16_t* b = base[i * R / 16];
       if constexpr (R == 32) b = row0 >= 16 ? base[i * 2 + 1] : base[i * 2];
-      cr[i] = *reinterpret_cast<const u32x4_t*>(b + (R < 16 ? (i * R % 16) * g.rp : 0) + lane_off);
+      cr[i] = *reinterpret_cast<const u32x4_t*>(b + (R < 16 ? (i * R % 16) * g.cp : 0) + lane_off);
+    }
+    if constexpr (NX > 0) {
+#pragma unroll
+      for (int i = 0; i < NX; ++i) xr[i] = *reinterpret_cast<const u32x4_t*>((tid >= 128 ? base[2 * i + 1] : base[2 * i]) + x_off);
     }
   };
   if (t0 < t1) {
@@ -239,8 +276,8 @@ __global__ __launch_bounds__(256, HG == 1 ? 2 : 1) void latent_rows_kernel(Laten
   }
   u32x4_t qr[KS];
   auto q_frag = [&](int hg, int ks, int l) {
-    const int h = h0 + hg * 16 + (l & 15), d = ks * 32 + (l >> 4) * 8;
-    return h < g.H && d < g.rp ? *reinterpret_cast<const u32x4_t*>(qa + ((size_t)at.row * g.H + h) * g.rp + d) : u32x4_t{0, 0, 0, 0};
+    const int h = h0 + hg * 16 + (l & 15), e = ks * 32 + (l >> 4) * 8, d = e < RP ? e : g.rp + e - RP;
+    return h < g.H && d < (e < RP ? g.rp : g.cp) ? *reinterpret_cast<const u32x4_t*>(qa + ((size_t)at.row * g.H + h) * g.cp + d) : u32x4_t{0, 0, 0, 0};
   };
   if constexpr (HG == 1) {
 #pragma unroll
@@ -265,6 +302,10 @@ __global__ __launch_bounds__(256, HG == 1 ? 2 : 1) void latent_rows_kernel(Laten
     for (int i = 0; i < NL; ++i) {
       const int idx = tid + 256 * i;
       *reinterpret_cast<u32x4_t*>(&Cs[(idx / CCH) * CP + (idx % CCH) * 8]) = cr[i];
+    }
+    if constexpr (NX > 0) {
+#pragma unroll
+      for (int i = 0; i < NX; ++i) *reinterpret_cast<u32x4_t*>(&Cs[((tid >> 3) + 32 * i) * CP + RP + (tid & 7) * 8]) = xr[i];
     }
     __syncthreads();
     if (tt + 1 < t1) {
@@ -487,18 +528,18 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(LatentGeom g, int wi
   if (i == nseg) return;
   const int p_row = latent_kv_first(sg, window) + at, p = min(p_row, sg.pos0 + sg.n - 1);     // (padding rows: copies, never in sight)
   if (lane == 0 && m % kKvBlock == 0) kv_bt[(size_t)sg.seq * kv_mb + p_row / kKvBlock] = m / kKvBlock;
-  const uint16_t* src = pool + ((size_t)bt[(size_t)sg.seq * MB + p / bs] * bs + p % bs) * g.rp;
+  const uint16_t* src = pool + ((size_t)bt[(size_t)sg.seq * MB + p / bs] * bs + p % bs) * g.cp;
   for (int d = lane * 8; d < ldx; d += 512)
-    *reinterpret_cast<u32x4_t*>(x + (size_t)m * ldx + d) = d < g.rp ? *reinterpret_cast<const u32x4_t*>(src + d) : u32x4_t{0, 0, 0, 0};
+    *reinterpret_cast<u32x4_t*>(x + (size_t)m * ldx + d) = d < g.cp ? *reinterpret_cast<const u32x4_t*>(src + d) : u32x4_t{0, 0, 0, 0};
 }
 
 // rows of the batch -> rows of a list (NS = 1: lat holds the normalised output of every row; the other rows are left alone)
-template <int RP, int HG>
+template <int RP, int RX, int HG>
 int launch_rows_t(const LatentGeom& g, float scale, int window, const uint16_t* qa, const uint16_t* pool, int bs, const int32_t* bt, int MB,
                   const int32_t* pos, const LatentRows& lr, int NS, float* op, float* ml, uint16_t* lat, hipStream_t s) {
-  constexpr size_t lds = latent_lds<RP, HG>();
+  constexpr size_t lds = latent_lds<RP, RX, HG>();
   const dim3 grid(NS, ceil_div(g.H, 16 * HG), lr.rows);
-  auto kern = NS == 1 ? latent_rows_kernel<RP, HG, true> : latent_rows_kernel<RP, HG, false>;
+  auto kern = NS == 1 ? latent_rows_kernel<RP, RX, HG, true> : latent_rows_kernel<RP, RX, HG, false>;
   if (lds > 64 * 1024) { int rc = ensure_dynamic_lds(reinterpret_cast<const void*>(kern), (int)lds); if (rc != MI_OK) return rc; }
   hipLaunchKernelGGL(kern, grid, dim3(256), lds, s, g, scale * kLog2e, window, qa, pool, bs, bt, MB, pos, lr, NS, (bs & (bs - 1)) == 0 ? __builtin_ctz(bs) : -1, op, ml, lat);
   MI_HIP(hipGetLastError());
@@ -507,25 +548,37 @@ int launch_rows_t(const LatentGeom& g, float scale, int window, const uint16_t* 
 
 }  // namespace
 
-int launch_latent_scatter(const float* qd, int ldq, int T, const LatentGeom& g, const float* c_norm, float eps, const int32_t* slots,
+static int check_latent(const LatentRowsIn& in, int T, const LatentGeom& g, const Rotation& rot, const float* c_norm) {
+  MI_CHECK(T >= 1 && in.q && in.ldq % 4 == 0 && in.ldq >= g.H * g.dq() && g.dkp >= g.dq() && g.dkp % 32 == 0 && g.rp >= g.rank && g.rp % 32 == 0 &&
+           g.cp >= g.rp + g.nr && g.cp % 32 == 0, "latent rows: geometry");
+  MI_CHECK(g.nr == 0 || (rot.table && rot.pos && g.dims % 2 == 0 && g.dims <= g.nr), "latent rows: rotation");
+  MI_CHECK(!c_norm || (in.lat && in.ldl >= g.rank + g.nr), "latent rows: latents");
+  return MI_OK;
+}
+
+int launch_latent_scatter(const LatentRowsIn& in, int T, const LatentGeom& g, const Rotation& rot, const float* c_norm, float eps, const int32_t* slots,
                           int bs, void* q, void* pool, bool f32, hipStream_t s, const SlabSum* slabs) {
   const SlabSum sl = slabs ? *slabs : SlabSum();
-  MI_CHECK(!sl.slab || (sl.T == T && sl.N == ldq && !sl.bias && !sl.row_scale), "latent scatter: pending K-split sum of another shape");
-  MI_CHECK(T >= 1 && ldq % 4 == 0 && ldq >= g.H * g.dk + (c_norm ? g.rank : 0) && g.dkp >= g.dk && g.dkp % 32 == 0 && g.rp >= g.rank && g.rp % 32 == 0 && bs > 0,
-           "latent scatter: geometry");
+  int rc = check_latent(in, T, g, rot, c_norm);
+  if (rc != MI_OK) return rc;
+  MI_CHECK(!sl.slab || (sl.T == T && sl.N == in.ldq && !sl.bias && !sl.row_scale && sl.N >= g.H * g.dq() + (c_norm ? g.rank + g.nr : 0)),
+           "latent scatter: pending K-split sum of another shape");
+  MI_CHECK(bs > 0, "latent scatter: block size");
   const dim3 grid(T, ceil_div(g.H, 8) + (c_norm ? 1 : 0));
-  if (f32) hipLaunchKernelGGL((latent_scatter_kernel<float>), grid, dim3(256), 0, s, qd, ldq, sl, g, c_norm, eps, slots, bs, (float*)q, (float*)pool);
-  else hipLaunchKernelGGL((latent_scatter_kernel<uint16_t>), grid, dim3(256), 0, s, qd, ldq, sl, g, c_norm, eps, slots, bs, (uint16_t*)q, (uint16_t*)pool);
+  if (f32) hipLaunchKernelGGL((latent_scatter_kernel<float>), grid, dim3(256), 0, s, in, sl, g, rot, c_norm, eps, slots, bs, (float*)q, (float*)pool);
+  else hipLaunchKernelGGL((latent_scatter_kernel<uint16_t>), grid, dim3(256), 0, s, in, sl, g, rot, c_norm, eps, slots, bs, (uint16_t*)q, (uint16_t*)pool);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
 
-int launch_latent_token(const float* qd, int ldq, int rows, const LatentGeom& g, const void* w_uk, const float* c_norm, float eps, const int32_t* slots,
-                        uint16_t* qa, uint16_t* pool, hipStream_t s) {
-  MI_CHECK(rows >= 1 && latent_token_supported(g) && ldq % 4 == 0 && ldq >= g.H * g.dk + (c_norm ? g.rank : 0), "latent token: geometry");
-  const int heads_x = ceil_div(rows, 16) * ceil_div(g.rp / 16, 4);
+int launch_latent_token(const LatentRowsIn& in, int rows, const LatentGeom& g, const Rotation& rot, const void* w_uk, const float* c_norm, float eps,
+                        const int32_t* slots, uint16_t* qa, uint16_t* pool, hipStream_t s) {
+  int rc = check_latent(in, rows, g, rot, c_norm);
+  if (rc != MI_OK) return rc;
+  MI_CHECK(latent_token_supported(g), "latent token: head sizes must be multiples of 4");
+  const int heads_x = ceil_div(rows, 16) * ceil_div(g.cp / 16, 4);
   const dim3 grid(c_norm && rows > heads_x ? rows : heads_x, g.H + (c_norm ? 1 : 0));
-  hipLaunchKernelGGL(latent_token_kernel, grid, dim3(256), 0, s, qd, ldq, g, (const uint4*)w_uk, rows, c_norm, eps, slots, qa, pool);
+  hipLaunchKernelGGL(latent_token_kernel, grid, dim3(256), 0, s, in, g, rot, (const uint4*)w_uk, rows, c_norm, eps, slots, qa, pool);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
@@ -547,7 +600,7 @@ int launch_head_linear(const void* w, int H, int N, int K, const void* x, int T,
   return MI_OK;
 }
 
-bool latent_attn_supported(const LatentGeom& g) { return g.rp <= 512; }
+bool latent_attn_supported(const LatentGeom& g) { return g.rp <= 512 && g.cp - g.rp <= 64; }
 
 // (rows x splits <= 512, launch_latent_attn_rows)
 size_t latent_attn_scratch_bytes(const LatentGeom& g) { return (size_t)512 * g.H * (g.rp + 2) * sizeof(float); }
@@ -569,15 +622,17 @@ int launch_latent_attn_rows(const LatentGeom& g, float scale, int window, const 
   float* ml = reinterpret_cast<float*>(scratch);
   float* op = ml + (size_t)512 * g.H * 2;
   int rc = MI_OK;
-#define MI_LR(RP) \
-  rc = hg == 1 ? launch_rows_t<RP, 1>(g, scale, window, qa, pool, bs, bt, MB, pos, lr, NS, op, ml, lat, s) \
-     : hg == 2 ? launch_rows_t<RP, 2>(g, scale, window, qa, pool, bs, bt, MB, pos, lr, NS, op, ml, lat, s) \
-               : launch_rows_t<RP, 4>(g, scale, window, qa, pool, bs, bt, MB, pos, lr, NS, op, ml, lat, s)
-  if (g.rp <= 64) MI_LR(64);
-  else if (g.rp <= 128) MI_LR(128);
-  else if (g.rp <= 256) MI_LR(256);
-  else MI_LR(512);
+#define MI_LX(RP, RX) \
+  rc = hg == 1 ? launch_rows_t<RP, RX, 1>(g, scale, window, qa, pool, bs, bt, MB, pos, lr, NS, op, ml, lat, s) \
+     : hg == 2 ? launch_rows_t<RP, RX, 2>(g, scale, window, qa, pool, bs, bt, MB, pos, lr, NS, op, ml, lat, s) \
+               : launch_rows_t<RP, RX, 4>(g, scale, window, qa, pool, bs, bt, MB, pos, lr, NS, op, ml, lat, s)
+#define MI_LR(RP) { if (g.cp > g.rp) MI_LX(RP, 64); else MI_LX(RP, 0); }
+  if (g.rp <= 64) MI_LR(64)
+  else if (g.rp <= 128) MI_LR(128)
+  else if (g.rp <= 256) MI_LR(256)
+  else MI_LR(512)
 #undef MI_LR
+#undef MI_LX
   if (rc != MI_OK) return rc;
   if (NS == 1) return launch_head_linear_rows(w_uv, g.H, g.dvp, g.rp, lat, lr, out, ldo, g.dv, g.dv, s);
   const int per = g.H * lr.rows / 256, rw = per <= 1 ? 1 : per <= 2 ? 2 : per <= 4 ? 4 : 16;
@@ -595,7 +650,7 @@ int launch_latent_attn_rows(const LatentGeom& g, float scale, int window, const 
 
 int launch_latent_gather(const LatentGeom& g, int window, const uint16_t* pool, int bs, const int32_t* bt, int MB, const AttnSeg* segs, int nseg,
                          int min_n, int rows, uint16_t* x, int ldx, int32_t* kv_bt, int kv_mb, hipStream_t s) {
-  MI_CHECK(rows >= 1 && rows % kKvBlock == 0 && ldx % 8 == 0 && ldx >= g.rp && bs > 0 && nseg >= 1, "latent gather: shape");
+  MI_CHECK(rows >= 1 && rows % kKvBlock == 0 && ldx % 8 == 0 && ldx >= g.cp && bs > 0 && nseg >= 1, "latent gather: shape");
   hipLaunchKernelGGL(latent_gather_kernel, dim3(ceil_div(rows, 4)), dim3(256), 0, s, g, window, pool, bs, bt, MB, segs, nseg, min_n, rows, x, ldx, kv_bt, kv_mb);
   MI_HIP(hipGetLastError());
   return MI_OK;

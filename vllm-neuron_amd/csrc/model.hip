@@ -702,35 +702,60 @@ int mi_ctx_create_stack(const mi_model_config* cfg, const mi_stack_config* stack
   MI_CHECK(t.num_layers > 0 && t.width > 0 && t.width <= 32768 && t.vocab_size > 0 && t.max_positions >= 0 && t.norm_eps >= 0.f, "stack: bad geometry");
   MI_CHECK(t.compute_dtype == MI_BF16 || t.compute_dtype == MI_F32, "stack: compute_dtype must be MI_BF16 or MI_F32");
   MI_CHECK(t.loop_times == 0 || (t.loop_times > 0 && t.loop_start >= 0 && t.loop_start < t.loop_stop && t.loop_stop <= t.num_layers), "stack: bad loop");
-  MI_CHECK(t.block_kind == MI_BLOCK_PARALLEL || t.block_kind == MI_BLOCK_SANDWICH, "stack: block_kind");
-  const bool sandwich = t.block_kind == MI_BLOCK_SANDWICH;
+  MI_CHECK(t.block_kind >= MI_BLOCK_PARALLEL && t.block_kind <= MI_BLOCK_ONE_NORM, "stack: block_kind");
+  const bool sandwich = t.block_kind == MI_BLOCK_SANDWICH, one_norm = t.block_kind == MI_BLOCK_ONE_NORM;
   if (sandwich) {
     MI_CHECK(t.norm_groups >= 1 && t.width % t.norm_groups == 0, "stack: the norm's groups must divide the width");
     MI_CHECK(t.conv_taps >= 1 && t.conv_taps <= 16 && t.state_lookahead >= 0, "stack: convolutions of 1 .. 16 taps are built");
     MI_CHECK(t.loop_times == 0, "stack: loops are not built for sandwich blocks");
+  } else if (one_norm) {
+    MI_CHECK(t.norm_groups == 1 && t.conv_taps == 0 && t.loop_times == 0 && t.residual_mult == 1.f, "stack: one-norm blocks are built with a whole-row RMS norm and no loop");
   } else {
     MI_CHECK(t.norm_groups == 0 && t.conv_taps == 0 && t.max_positions > 0, "stack: parallel blocks are built with layer norms, learned positions and no convolution");
   }
+  MI_CHECK(one_norm || (t.norm_offset == 0.f && t.embed_scale == 1.f), "stack: norm_offset and embed_scale are built for one-norm blocks");
   MI_CHECK(t.logit_softcap >= 0.f, "stack: logit_softcap");
   for (int i = 0; i < t.num_layers; ++i) {
     const mi_layer_spec& p = t.layers[i];
     const std::string who = "stack: layer " + std::to_string(i) + ": ";
-    MI_CHECK(p.mixer_kind == (sandwich ? MI_MIX_LATENT : MI_MIX_ATTENTION), who + "this mixer is not built for the block kind");
+    if (one_norm && p.weights_of >= 0) {
+      int j = i, steps = 0;
+      while (j >= 0 && j < t.num_layers && t.layers[j].weights_of >= 0 && steps++ < t.num_layers) j = t.layers[j].weights_of;
+      MI_CHECK(j >= 0 && j < t.num_layers && t.layers[j].weights_of < 0, who + "weights_of must lead to a layer with tensors of its own");
+      continue;
+    }
+    MI_CHECK(one_norm ? p.mixer_kind == MI_MIX_LATENT || p.mixer_kind == MI_MIX_DELTA : p.mixer_kind == (sandwich ? MI_MIX_LATENT : MI_MIX_ATTENTION),
+             who + "this mixer is not built for the block kind");
     MI_CHECK(p.num_heads > 0 && p.qk_dim > 0 && p.v_dim > 0 && p.window >= 0, who + "bad attention sizes");
-    if (p.mixer_kind == MI_MIX_LATENT) {
+    MI_CHECK(one_norm || (!p.q_rank && !p.rot_dim && !p.out_gate && !p.router_score), who + "query latents, rotation, output gates and sigmoid routers are built for one-norm blocks");
+    if (p.mixer_kind == MI_MIX_DELTA) {
+      const DeltaGeom g{p.num_heads, p.num_kv_heads, p.qk_dim, p.v_dim, 0, 0, p.conv_taps};
+      MI_CHECK(delta_supported(g), who + "delta rule: num_heads a multiple of num_kv_heads, head sizes 1 .. 256, 1 .. 16 taps");
+      MI_CHECK(p.decay_rank >= 1 && p.gate_rank >= 1, who + "delta rule: decay_rank / gate_rank");
+    } else if (p.mixer_kind == MI_MIX_LATENT) {
       MI_CHECK(p.kv_rank > 0 && p.kv_rank <= 4096 && p.qk_dim <= 4096 && p.v_dim <= 4096, who + "bad latent size");
       MI_CHECK(!p.qk_unit_norm && !p.distance_bias && !p.softmax_sink, who + "latent attention has no unit norm, distance bias or sink");
       MI_CHECK(p.kv_from < 0 || (p.kv_from < i && t.layers[p.kv_from].kv_from < 0 && t.layers[p.kv_from].kv_rank == p.kv_rank),
                who + "kv_from must name an earlier layer with latents of its own and the same kv_rank");
+      MI_CHECK(!one_norm || (p.kv_from < 0 && p.window == 0), who + "one-norm blocks: latents of another layer and windows are not built");
+      MI_CHECK(p.q_rank >= 0 && p.rot_dim >= 0 && p.rot_dim <= 4096 && p.rot_dims >= 0 && p.rot_dims <= p.rot_dim && p.rot_dims % 2 == 0 && (p.rot_dims == 0 || p.rot_base > 0.f),
+               who + "rotation: rot_dims even, at most rot_dim, rot_base positive");
+      MI_CHECK(p.out_gate >= MI_GATE_NONE && p.out_gate <= MI_GATE_ELEMENT, who + "out_gate");
     } else {
       MI_CHECK(p.num_kv_heads > 0 && p.num_heads % p.num_kv_heads == 0, who + "bad attention sizes");
     }
-    const bool ff = p.ff_kind == MI_FF_NONE || (p.ff_size > 0 && (sandwich ? p.ff_kind == MI_FF_GLU || p.ff_kind == MI_FF_MOE : p.ff_kind == MI_FF_RELU2));
-    MI_CHECK(ff, who + "bad feed-forward");
+    const bool kind = one_norm ? p.ff_kind == MI_FF_MOE : sandwich ? p.ff_kind == MI_FF_GLU || p.ff_kind == MI_FF_MOE : p.ff_kind == MI_FF_RELU2;
+    MI_CHECK(p.ff_kind == MI_FF_NONE || (p.ff_size > 0 && kind), who + "bad feed-forward");
     if (p.ff_kind == MI_FF_GLU) MI_CHECK(p.ff_act == MI_ACT_SWISH_CLIP && p.ff_limit >= 0.f, who + "gated feed-forwards are built with the clipped activation");
-    if (p.ff_kind == MI_FF_MOE)
-      MI_CHECK(p.ff_act == MI_ACT_SILU && p.experts >= 1 && p.experts <= 4096 && p.experts_top >= 1 && p.experts_top <= std::min(p.experts, 64),
-               who + "experts: silu, 1 <= experts_top <= min(experts, 64)");
+    if (p.ff_kind == MI_FF_MOE) {
+      MI_CHECK((p.ff_act == MI_ACT_SILU || p.ff_act == MI_ACT_RELU2) && p.experts >= 1 && p.experts <= 4096 && p.experts_top >= 1 && p.experts_top <= std::min(p.experts, 64),
+               who + "experts: silu or relu2, 1 <= experts_top <= min(experts, 64)");
+      if (p.router_score == MI_ROUTE_SIGMOID)
+        MI_CHECK(p.experts <= 1024 && p.router_groups >= 1 && p.experts % p.router_groups == 0 && p.router_keep >= 1 && p.router_keep <= p.router_groups &&
+                 p.experts_top <= p.experts / p.router_groups * p.router_keep, who + "sigmoid router: up to 1024 experts, groups that divide them and hold the chosen ones");
+      else
+        MI_CHECK(p.router_score == MI_ROUTE_SOFTMAX, who + "router_score");
+    }
   }
   MI_CHECK(k.tp_degree <= 1, "stack: tensor parallelism is not built for layer-stack decoders");
   MI_CHECK(k.weight_dtype == MI_W_BF16, "stack: weight quantization is not built for layer-stack decoders");
@@ -1136,8 +1161,8 @@ int mi_finalize(mi_ctx* c) {
   c->MB_cap = ceil_div(k.max_model_len, k.block_size) + 1;
   const size_t nbt = (size_t)k.max_num_seqs * c->MB_cap;
   // inputs: [block tables][context lengths][ids][positions][slots], one block on each side
-  // [tables][per-request ints][ids][pos][slots][per-request context lengths][per-request segments, 16-byte aligned]
-  c->inputs_elems = ((nbt + 2 * (size_t)k.max_num_seqs + 3 * R + 3) & ~(size_t)3) + 4 * (size_t)k.max_num_seqs;
+  // [tables][per-request ints][ids][pos][slots][per-request context lengths][per-request state slots][per-request segments, 16-byte aligned]
+  c->inputs_elems = ((nbt + 3 * (size_t)k.max_num_seqs + 3 * R + 3) & ~(size_t)3) + 4 * (size_t)k.max_num_seqs;
   MI_TRY(dmalloc(&c->d_inputs, c->inputs_elems, ws));
   MI_HIP(hipHostMalloc(reinterpret_cast<void**>(&c->h_inputs), c->inputs_elems * 4, hipHostMallocDefault));
   memset(c->h_inputs, 0, c->inputs_elems * 4);
@@ -1157,11 +1182,11 @@ int mi_finalize(mi_ctx* c) {
   }
   {   // token-generation inputs: small per-step block + device-resident block tables
     const size_t ms = (size_t)k.max_num_seqs;
-    MI_TRY(dmalloc(&c->d_dec, 4 * ms, ws));
+    MI_TRY(dmalloc(&c->d_dec, 5 * ms, ws));
     MI_TRY(dmalloc(&c->d_dec_bt, nbt, ws));
-    MI_HIP(hipHostMalloc(reinterpret_cast<void**>(&c->h_dec), 4 * ms * 4, hipHostMallocDefault));
+    MI_HIP(hipHostMalloc(reinterpret_cast<void**>(&c->h_dec), 5 * ms * 4, hipHostMallocDefault));
     MI_HIP(hipHostMalloc(reinterpret_cast<void**>(&c->h_dec_bt), nbt * 4, hipHostMallocDefault));
-    memset(c->h_dec, 0, 4 * ms * 4);
+    memset(c->h_dec, 0, 5 * ms * 4);
     memset(c->h_dec_bt, 0, nbt * 4);
     MI_HIP(hipMemsetAsync(c->d_dec_bt, 0, nbt * 4, s));
     c->bt_checked.assign(ms, 0);
@@ -1189,16 +1214,18 @@ static void set_input_views(mi_ctx* c, bool decode_step) {
   if (decode_step) {
     c->d_ctx = c->d_dec; c->d_ids = c->d_dec + ms; c->d_pos = c->d_dec + 2 * ms; c->d_slots = c->d_dec + 3 * ms;
     c->h_ctx = c->h_dec; c->h_ids = c->h_dec + ms; c->h_pos = c->h_dec + 2 * ms; c->h_slots = c->h_dec + 3 * ms;
+    c->d_state = c->d_dec + 4 * ms; c->h_state = c->h_dec + 4 * ms;
     c->d_bt = c->d_dec_bt; c->h_bt = c->h_dec_bt;
   } else {
     c->d_bt = c->d_inputs; c->d_ctx = c->d_inputs + nbt; c->d_ids = c->d_ctx + ms; c->d_pos = c->d_ids + R; c->d_slots = c->d_pos + R;
     c->h_bt = c->h_inputs; c->h_ctx = c->h_inputs + nbt; c->h_ids = c->h_ctx + ms; c->h_pos = c->h_ids + R; c->h_slots = c->h_pos + R;
     c->d_seg_ctx = c->d_slots + R; c->h_seg_ctx = c->h_slots + R;
+    c->d_state = c->d_seg_ctx + ms; c->h_state = c->h_seg_ctx + ms;
     c->d_segs = c->d_inputs + c->inputs_elems - 4 * ms; c->h_segs = c->h_inputs + c->inputs_elems - 4 * ms;
   }
 }
 
-// ---- staging of a token-generation batch: 4 ints per row + the block-table rows that changed ----
+// ---- staging of a token-generation batch: 5 ints per row + the block-table rows that changed ----
 // (block tables are resident on the device; a row is re-sent only when it differs from the host
 //  shadow of what the device holds, and only entries that became live are range-checked)
 struct DecodeStage { int row_lo = 0, row_hi = -1; };
@@ -1250,9 +1277,9 @@ static int decode_stage_row(mi_ctx* c, int b, int MB, int64_t id, int64_t pos, i
   c->h_ctx[b] = full;
   return MI_OK;
 }
-static int decode_stage_push(mi_ctx* c, int MB, const DecodeStage& st) {   // 4 x max_num_seqs ints, + the table rows that changed
+static int decode_stage_push(mi_ctx* c, int MB, const DecodeStage& st) {   // 5 x max_num_seqs ints, + the table rows that changed
   hipStream_t s = c->stream;
-  MI_HIP(hipMemcpyAsync(c->d_dec, c->h_dec, (size_t)c->cfg.max_num_seqs * 16, hipMemcpyHostToDevice, s));
+  MI_HIP(hipMemcpyAsync(c->d_dec, c->h_dec, (size_t)c->cfg.max_num_seqs * 20, hipMemcpyHostToDevice, s));
   if (st.row_hi >= st.row_lo)
     MI_HIP(hipMemcpyAsync(c->d_dec_bt + (size_t)st.row_lo * MB, c->h_dec_bt + (size_t)st.row_lo * MB,
                           (size_t)(st.row_hi - st.row_lo + 1) * MB * 4, hipMemcpyHostToDevice, s));
@@ -1300,6 +1327,19 @@ static int sample_on_device(mi_ctx* c, int nrows, int row0, const float* samplin
   return MI_OK;
 }
 
+// the state slots of a step's sequences (set_input_views first)
+static int stage_state(mi_ctx* c, int n, const int64_t* seq_ids) {
+  if (!stack_has_state(c)) return MI_OK;
+  MI_CHECK(seq_ids, "models with recurrent mixers need a state slot per sequence (seq_ids)");
+  std::vector<bool> seen((size_t)c->cfg.max_num_seqs, false);
+  for (int i = 0; i < n; ++i) {
+    MI_CHECK(seq_ids[i] >= 0 && seq_ids[i] < c->cfg.max_num_seqs && !seen[seq_ids[i]], "state slots (seq_ids) must be distinct and below max_num_seqs");
+    seen[seq_ids[i]] = true;
+    c->h_state[i] = (int32_t)seq_ids[i];
+  }
+  return MI_OK;
+}
+
 static int forward_impl(mi_ctx* c, int32_t B, int32_t S, const int64_t* input_ids, const int64_t* position_ids,
                         const int64_t* seq_ids, const int64_t* block_table, int32_t MB, const int64_t* slot_mapping,
                         int32_t SM, const int64_t* full_context_lens, const int64_t* computed_context_lens,
@@ -1312,7 +1352,6 @@ static int forward_impl(mi_ctx* c, int32_t B, int32_t S, const int64_t* input_id
   MI_CHECK(c && c->finalized, "mi_forward before mi_finalize");
   MI_CHECK(input_ids && position_ids && block_table && slot_mapping && full_context_lens && computed_context_lens, "null argument");
   MI_CHECK((logits_out != nullptr) != (tokens_out != nullptr), "exactly one of logits_out / tokens_out");
-  (void)seq_ids;  // block-layout KV: rows are addressed through block_table, not batch lines
   const mi_model_config& k = c->cfg;
   MI_CHECK(B >= 1 && B <= k.max_num_seqs, "batch size exceeds max_num_seqs");
   MI_CHECK(S >= 1 && MB >= 1 && MB <= c->MB_cap && SM >= 1, "bad S / MB / SM");
@@ -1347,6 +1386,7 @@ static int forward_impl(mi_ctx* c, int32_t B, int32_t S, const int64_t* input_id
     for (int b = 0; b < B; ++b)
       MI_TRY(decode_stage_row(c, b, MB, input_ids[b], position_ids[b], slot_mapping[(size_t)b * SM], (int)full_context_lens[b],
                               block_table + (size_t)b * MB, st));
+    MI_TRY(stage_state(c, B, seq_ids));
     auto push_inputs = [&]() -> int { return decode_stage_push(c, MB, st); };
     g_ht.lap(0);
     MI_TRY(push_inputs());
@@ -1387,6 +1427,7 @@ static int forward_impl(mi_ctx* c, int32_t B, int32_t S, const int64_t* input_id
     }
     for (int j = 0; j < MB; ++j) c->h_bt[j] = (int32_t)block_table[(size_t)b * MB + j];
     c->h_seg_ctx[0] = full;
+    MI_TRY(stage_state(c, 1, seq_ids ? seq_ids + b : nullptr));
     memcpy(c->h_segs, std::array<int32_t, 4>{0, n_new, comp, 0}.data(), 16);
     MI_TRY(push_inputs());
     MI_TRY(run_layers(c, n_new, false, 1, MB, comp, 1, n_new - 1));
@@ -1432,13 +1473,14 @@ static int ragged_check(mi_ctx* c, int32_t n_req, int32_t total, int32_t MB, con
   return MI_OK;
 }
 static int ragged_trunk(mi_ctx* c, int32_t n_req, int32_t total, const int64_t* input_ids, const int64_t* position_ids,
-                        const int64_t* slot_mapping, const int64_t* block_table, int32_t MB,
+                        const int64_t* seq_ids, const int64_t* slot_mapping, const int64_t* block_table, int32_t MB,
                         const int64_t* full_context_lens, const int64_t* computed_context_lens) {
   const mi_model_config& k = c->cfg;
   MI_HIP(hipSetDevice(k.device_id));
   hipStream_t s = c->stream;
   const int bs = k.block_size, V = k.vocab_size;
   set_input_views(c, false);
+  MI_TRY(stage_state(c, n_req, seq_ids));
   std::vector<Seg> segs((size_t)n_req);
   int row = 0;
   for (int i = 0; i < n_req; ++i) {
@@ -1473,12 +1515,12 @@ static int ragged_trunk(mi_ctx* c, int32_t n_req, int32_t total, const int64_t* 
 }
 
 int mi_forward_chunked(mi_ctx* c, int32_t n_req, int32_t total, const int64_t* input_ids, const int64_t* position_ids,
-                       const int64_t* slot_mapping, const int64_t* block_table, int32_t MB,
+                       const int64_t* seq_ids, const int64_t* slot_mapping, const int64_t* block_table, int32_t MB,
                        const int64_t* full_context_lens, const int64_t* computed_context_lens, float* logits_out,
                        const float* sampling_params, uint64_t seed, int64_t* tokens_out) {
   if (c && c->owned_group)
     return group_run(c->owned_group, [&](mi_ctx* rc, int) {
-      return mi_forward_chunked(rc, n_req, total, input_ids, position_ids, slot_mapping, block_table, MB, full_context_lens,
+      return mi_forward_chunked(rc, n_req, total, input_ids, position_ids, seq_ids, slot_mapping, block_table, MB, full_context_lens,
                                 computed_context_lens, logits_out, sampling_params, seed, tokens_out);
     });
   MI_CHECK(c && c->finalized, "mi_forward_chunked before mi_finalize");
@@ -1487,9 +1529,9 @@ int mi_forward_chunked(mi_ctx* c, int32_t n_req, int32_t total, const int64_t* i
   bool one_each = false;
   MI_TRY(ragged_check(c, n_req, total, MB, full_context_lens, computed_context_lens, &one_each));
   if (one_each)
-    return forward_impl(c, n_req, 1, input_ids, position_ids, nullptr, block_table, MB, slot_mapping, 1, full_context_lens,
+    return forward_impl(c, n_req, 1, input_ids, position_ids, seq_ids, block_table, MB, slot_mapping, 1, full_context_lens,
                         computed_context_lens, logits_out, sampling_params, seed, tokens_out);
-  MI_TRY(ragged_trunk(c, n_req, total, input_ids, position_ids, slot_mapping, block_table, MB, full_context_lens, computed_context_lens));
+  MI_TRY(ragged_trunk(c, n_req, total, input_ids, position_ids, seq_ids, slot_mapping, block_table, MB, full_context_lens, computed_context_lens));
   MI_TRY(run_head(c, n_req, 0, true));
   if (tokens_out) MI_TRY(sample_on_device(c, n_req, 0, sampling_params, seed, tokens_out));
   else MI_TRY(fetch_logits(c, n_req, logits_out));
@@ -1497,11 +1539,11 @@ int mi_forward_chunked(mi_ctx* c, int32_t n_req, int32_t total, const int64_t* i
 }
 
 int mi_forward_rows(mi_ctx* c, int32_t n_req, int32_t total, const int64_t* input_ids, const int64_t* position_ids,
-                    const int64_t* slot_mapping, const int64_t* block_table, int32_t MB, const int64_t* full_context_lens,
+                    const int64_t* seq_ids, const int64_t* slot_mapping, const int64_t* block_table, int32_t MB, const int64_t* full_context_lens,
                     const int64_t* computed_context_lens, int32_t n_rows, const int64_t* rows, float* logits_out) {
   if (c && c->owned_group)
     return group_run(c->owned_group, [&](mi_ctx* rc, int) {
-      return mi_forward_rows(rc, n_req, total, input_ids, position_ids, slot_mapping, block_table, MB, full_context_lens,
+      return mi_forward_rows(rc, n_req, total, input_ids, position_ids, seq_ids, slot_mapping, block_table, MB, full_context_lens,
                              computed_context_lens, n_rows, rows, logits_out);
     });
   MI_CHECK(c && c->finalized, "mi_forward_rows before mi_finalize");
@@ -1513,12 +1555,12 @@ int mi_forward_rows(mi_ctx* c, int32_t n_req, int32_t total, const int64_t* inpu
   const size_t V = (size_t)c->cfg.vocab_size, ms = (size_t)c->cfg.max_num_seqs;
   if (one_each && !c->grp) {   // (a rank shard fills its columns of the caller's rows itself: no detour through a copy)
     std::vector<float> all((size_t)n_req * V);
-    MI_TRY(forward_impl(c, n_req, 1, input_ids, position_ids, nullptr, block_table, MB, slot_mapping, 1, full_context_lens,
+    MI_TRY(forward_impl(c, n_req, 1, input_ids, position_ids, seq_ids, block_table, MB, slot_mapping, 1, full_context_lens,
                         computed_context_lens, all.data(), nullptr, 0, nullptr));
     for (int i = 0; i < n_rows; ++i) memcpy(logits_out + (size_t)i * V, all.data() + (size_t)rows[i] * V, V * 4);
     return MI_OK;
   }
-  MI_TRY(ragged_trunk(c, n_req, total, input_ids, position_ids, slot_mapping, block_table, MB, full_context_lens, computed_context_lens));
+  MI_TRY(ragged_trunk(c, n_req, total, input_ids, position_ids, seq_ids, slot_mapping, block_table, MB, full_context_lens, computed_context_lens));
   for (int i0 = 0; i0 < n_rows; i0 += (int)ms) {   // the head and its buffers hold max_num_seqs rows at a time
     const int n = std::min((int)ms, n_rows - i0);
     MI_HIP(hipStreamSynchronize(c->stream));       // the pinned list behind d_ctx is free to be rewritten
@@ -1570,6 +1612,7 @@ int mi_forward_spec(mi_ctx* t, mi_ctx* d, int32_t B, int32_t k, const int64_t* i
   MI_CHECK(!d->owned_group && !d->grp && !d->collective() && !t->grp && (t->owned_group || !t->collective()),
            "mi_forward_spec: the draft is a single-GPU context; the target a single-GPU context or an in-process tensor-parallel group");
   MI_CHECK(input_ids && position_ids && block_table && accepted_out && next_pos_out, "null argument");
+  MI_CHECK(!stack_has_state(t) && !stack_has_state(d), "mi_forward_spec: recurrent state cannot be taken back to the last accepted token");
   // the target's rank shards (one: the context itself).  Everything the step keeps on the device besides the
   // shards' own inputs lives with shard 0, on whose GPU (and stream) the draft runs.
   mi_group* g = t->owned_group;
@@ -1991,7 +2034,7 @@ int mi_op_layernorm2(const float* x, int32_t T, int32_t D, int32_t ld, float eps
 int mi_op_embed_pos(const int32_t* ids, const int32_t* pos, const void* table, const void* ptable, int32_t T, int32_t D, int32_t ld,
                     float* resid, float* x0, int32_t f32, void* stream) {
   MI_CHECK(ids && pos && table && ptable && resid && T >= 1 && ld >= D, "bad argument");
-  return launch_embed_pos(ids, pos, table, ptable, f32 != 0, T, D, ld, resid, x0, (hipStream_t)stream);
+  return launch_embed_pos(ids, pos, table, ptable, 1.f, f32 != 0, T, D, ld, resid, x0, (hipStream_t)stream);
 }
 int mi_op_qkv_scatter(const float* qkv, int32_t ldq, int32_t T, const mi_layer_spec* spec, float eps, const int32_t* slots,
                       int32_t block_size, void* q, void* kpool, void* vpool, int32_t f32, void* stream) {

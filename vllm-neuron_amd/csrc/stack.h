@@ -4,6 +4,7 @@
 #include <string>
 #include <vector>
 
+#include "delta_rule.h"
 #include "experts.h"
 #include "latent_attn.h"
 #include "model_internal.h"
@@ -35,11 +36,25 @@ struct StackLayer {
   StackMat ukv;                                  // [W_uk ; W_uv], heads padded to dkp / dvp rows: keys and values of a prompt (bf16)
   HeadGeom kvg;                                  // ... as the context-encoding attention sees them: every head its own
   bool fast() const { return ukv.L.w != nullptr; }   // the MFMA forms are built for the layer's sizes
+  // one-norm blocks: qkv = every product with h the mixer needs, columns at col_*; latent mixer: [dkv | dq (or q) | g]; delta rule:
+  // [q | k | v | b | a1 | g1]
+  int col_q = 0, col_g = 0, col_b = 0, col_a = 0;
+  StackMat uq, a2, g2;
+  float *q_norm = nullptr, *conv = nullptr, *a_log = nullptr, *dt = nullptr, *o_norm = nullptr;
+  DeltaGeom dg;
+  const float2* rot = nullptr;                   // cosines and sines of the layer's rotation (Stack::rot)
+  int ff_act() const { return s.ff_act == MI_ACT_RELU2 ? EXPERT_RELU2 : EXPERT_SILU_GLU; }
+  RouterRule rule() const {
+    RouterRule r;
+    r.sigmoid = s.router_score == MI_ROUTE_SIGMOID; r.b = router_b;
+    if (r.sigmoid) { r.groups = s.router_groups; r.keep = s.router_keep; }
+    return r;
+  }
   void *router = nullptr, *expert_gu = nullptr, *expert_down = nullptr;
   float* router_b = nullptr;                     // [experts padded to 16]
   StackMat router_t;                             // the router as tiles: many rows (bf16)
   int ffk = 0;                                   // padded ff_size: contraction length of the experts' down projection
-  ExpertsLinear expert_up() const { return ExpertsLinear{expert_gu, s.experts, (2 * s.ff_size + 15) / 16 * 16, up.K}; }
+  ExpertsLinear expert_up() const { return ExpertsLinear{expert_gu, s.experts, ((s.ff_act == MI_ACT_RELU2 ? 1 : 2) * s.ff_size + 15) / 16 * 16, up.K}; }
   ExpertsLinear expert_dn() const { return ExpertsLinear{expert_down, s.experts, out.N, ffk}; }
 };
 struct StackRun { int layer; bool pass_start; };   // pass_start: the looped layers' input projection runs first
@@ -74,6 +89,16 @@ struct Stack {
   int32_t* kv_bt = nullptr;
   int kv_rows = 0, kv_mb = 0, kv_ldx = 0;
   size_t kv_k_cols = 0, kv_v_cols = 0;
+  // one-norm blocks
+  struct RotTable { float base; int dims; float2* t; };
+  std::vector<RotTable> rot;
+  std::vector<float*> state_at;       // every run's recurrent state, then its ring (null: none)
+  int state_slots = 0;                // 0: no layer has any
+  int z_ld = 0, z_gate = 0, low_ld = 0, cq_ld = 0, q2_ld = 0, delta_chunks = 0;
+  size_t delta_o_cols = 0, factor_floats = 0;
+  void *cq = nullptr, *low = nullptr; // normed query latents; the inputs of the decay's and the gate's second product [2][rows][low_ld]
+  float *q2 = nullptr, *z = nullptr, *delta_o = nullptr, *factors = nullptr;
+  bool one_norm() const { return cfg.block_kind == MI_BLOCK_ONE_NORM; }
   bool sandwich() const { return cfg.block_kind == MI_BLOCK_SANDWICH; }
   void* attn_scratch = nullptr;
   SlabSum pend;                        // K-split sum of the last output projection, left for the next norm
@@ -88,7 +113,8 @@ int stack_synthetic(mi_ctx* c, uint64_t seed, float std);
 void stack_artifact_tensors(mi_ctx* c, std::vector<std::pair<void*, size_t>>& out);
 int stack_geometry_hash(const mi_ctx* c);
 size_t stack_kv_bytes_per_block(const mi_ctx* c);
-size_t stack_workspace_estimate(const mi_ctx* c);
+size_t stack_workspace_estimate(const mi_ctx* c);               // recurrent state included
+bool stack_has_state(const mi_ctx* c);
 int stack_alloc(mi_ctx* c);                                    // KV pool + activations (mi_finalize)
 // the layers over `rows` rows; leaves the residual stream in c->resid[c->tail_cur]
 int stack_trunk(mi_ctx* c, int rows, bool decode, int MB, const AttnSeg* segs, int nseg);

@@ -15,6 +15,13 @@
 //   [q | latent] projection; latent norm into the pool; W_uk^T q                    GEMV / GEMM, latent_scatter, head_linear
 //   attention over latents; W_uv; output projection
 //   row, as above; gated feed-forward, or router and experts                        experts.hip
+//
+// A one-norm block's run (RMS norm, then mixer and experts of the same row):
+//   row: x += what the previous run left unsummed; norm                             sandwich_rows
+//   router, experts                                                                 experts.hip
+//   latent attention: [dkv | dq | g] product; query latent's norm; W_uq; rotation, scatter, attention as above; output gate
+//   delta rule: [q | k | v | b | a1 | g1] product; a2, g2; recurrence               delta_rule.hip
+//   output projection + residual; the experts' weighted sum and a K-split's are left to the next row kernel
 
 #include "stack.h"
 
@@ -139,6 +146,53 @@ int attention(mi_ctx* c, const StackLayer& W, size_t kv_at, int rows, bool decod
   return MI_OK;
 }
 
+// what latent attention needs in either block: W_uk, W_uv, W_o and the workspace's columns
+int latent_layer_create(mi_ctx* c, StackLayer& W) {
+  Stack* S = c->stack;
+  const mi_layer_spec& s = W.s;
+  size_t* wb = &c->weight_bytes;
+  const LatentGeom& g = W.lg = latent_geom(s.num_heads, s.qk_dim, s.v_dim, s.kv_rank, s.rot_dim, s.rot_dims);
+  W.latent = AttnSpec{HeadGeom{s.num_heads, 1, g.cp, g.rp, g.cp, g.cp}, s.scale, s.window, nullptr, 0, 0};
+  MI_TRY(alloc_mat(c, W.out, S->D, s.num_heads * s.v_dim, 1.f));
+  MI_TRY(alloc0(c, &W.w_uk, (size_t)s.num_heads * g.cp * g.dkp * S->elem(), wb));
+  MI_TRY(alloc0(c, &W.w_uv, (size_t)s.num_heads * g.dvp * g.rp * S->elem(), wb));
+  W.kvg = HeadGeom{s.num_heads, s.num_heads, g.dq(), s.v_dim, g.dkp, g.dvp};
+  if (!S->f32 && latent_attn_supported(g) && attn_window_supported(W.kvg)) {
+    MI_TRY(alloc_mat(c, W.ukv, s.num_heads * (g.dkp + g.dvp), g.nr ? g.rp + g.nr : s.kv_rank, 1.f));
+    S->kv_ldx = std::max(S->kv_ldx, W.ukv.K);
+    S->kv_k_cols = std::max(S->kv_k_cols, (size_t)s.num_heads * g.dkp);
+    S->kv_v_cols = std::max(S->kv_v_cols, (size_t)s.num_heads * g.dvp);
+  }
+  S->q_cols = std::max(S->q_cols, s.num_heads * g.dkp);
+  S->lat_cols = std::max(S->lat_cols, s.num_heads * g.cp);
+  S->cat_ld = std::max(S->cat_ld, W.out.K);
+  return MI_OK;
+}
+
+int experts_create(mi_ctx* c, StackLayer& W, const std::string& p) {
+  Stack* S = c->stack;
+  const mi_layer_spec& s = W.s;
+  size_t* wb = &c->weight_bytes;
+  auto want = [&](const char* n) { S->missing.push_back(p + n); };
+  W.up.K = S->Kd;
+  W.ffk = pad_to(s.ff_size, 64);
+  S->max_top = std::max(S->max_top, s.experts_top);
+  const ExpertsLinear gu = W.expert_up(), dn = W.expert_dn();
+  MI_TRY(alloc0(c, &W.expert_gu, (size_t)gu.E * gu.N * gu.K * S->elem(), wb));
+  MI_TRY(alloc0(c, &W.expert_down, (size_t)dn.E * dn.N * dn.K * S->elem(), wb));
+  MI_TRY(alloc0(c, &W.router, (size_t)s.experts * S->Kd * S->elem(), wb));
+  MI_TRY(alloc0(c, &W.router_b, (size_t)pad_to(s.experts, 16) * 4, wb));
+  if (!S->f32) MI_TRY(alloc_mat(c, W.router_t, s.experts, S->D, 1.f));
+  S->max_experts = std::max(S->max_experts, pad_to(s.experts, 16));
+  want("mlp.router");
+  want(s.router_score == MI_ROUTE_SIGMOID ? "mlp.correction" : "mlp.router.b");
+  for (int e = 0; e < s.experts; ++e)
+    for (const char* n : {".gate", ".up", ".down"})
+      if (n[1] != 'g' || s.ff_act != MI_ACT_RELU2) want(("mlp.e" + std::to_string(e) + n).c_str());
+  S->act_ld = std::max(S->act_ld, W.ffk);
+  return MI_OK;
+}
+
 // ---- sandwich blocks: geometry and weights of one layer --------------------------------------------------------------------
 int sandwich_layer_create(mi_ctx* c, StackLayer& W, const std::string& p) {
   Stack* S = c->stack;
@@ -148,28 +202,14 @@ int sandwich_layer_create(mi_ctx* c, StackLayer& W, const std::string& p) {
   auto norm = [&](StackNorm& n) { return alloc0(c, &n.w, (size_t)S->ld * 4, wb); };
   const int taps = S->cfg.conv_taps;
   const bool own = s.kv_from < 0;
-  W.lg = LatentGeom{s.num_heads, s.qk_dim, s.v_dim, s.kv_rank, pad_to(s.qk_dim, 32), pad_to(s.v_dim, 32), pad_to(s.kv_rank, 32)};
-  W.latent = AttnSpec{HeadGeom{s.num_heads, 1, W.lg.rp, W.lg.rp, W.lg.rp, W.lg.rp}, s.scale, s.window, nullptr, 0, 0};
   MI_TRY(alloc_mat(c, W.qkv, s.num_heads * s.qk_dim + (own ? s.kv_rank : 0), S->D, 1.f));
-  MI_TRY(alloc_mat(c, W.out, S->D, s.num_heads * s.v_dim, 1.f));
-  MI_TRY(alloc0(c, &W.w_uk, (size_t)s.num_heads * W.lg.rp * W.lg.dkp * S->elem(), wb));
-  MI_TRY(alloc0(c, &W.w_uv, (size_t)s.num_heads * W.lg.dvp * W.lg.rp * S->elem(), wb));
-  W.kvg = HeadGeom{s.num_heads, s.num_heads, s.qk_dim, s.v_dim, W.lg.dkp, W.lg.dvp};
-  if (!S->f32 && latent_attn_supported(W.lg) && attn_window_supported(W.kvg)) {
-    MI_TRY(alloc_mat(c, W.ukv, s.num_heads * (W.lg.dkp + W.lg.dvp), s.kv_rank, 1.f));
-    S->kv_ldx = std::max(S->kv_ldx, W.ukv.K);
-    S->kv_k_cols = std::max(S->kv_k_cols, (size_t)s.num_heads * W.lg.dkp);
-    S->kv_v_cols = std::max(S->kv_v_cols, (size_t)s.num_heads * W.lg.dvp);
-  }
+  MI_TRY(latent_layer_create(c, W));
   if (own) MI_TRY(alloc0(c, &W.c_norm, (size_t)s.kv_rank * 4, wb));
   MI_TRY(norm(W.n1)); MI_TRY(norm(W.n1b));
   MI_TRY(alloc0(c, &W.conv1, (size_t)taps * S->ld * 4, wb));
   for (const char* n : {"norm1", "norm1b", "canon1", "mix.q", "mix.uk", "mix.uv", "mix.o"}) want(n);
   if (own) { want("mix.dkv"); want("mix.dkv.norm"); }
   S->qkv_ld = std::max(S->qkv_ld, W.qkv.N);
-  S->q_cols = std::max(S->q_cols, s.num_heads * W.lg.dkp);
-  S->lat_cols = std::max(S->lat_cols, s.num_heads * W.lg.rp);
-  S->cat_ld = std::max(S->cat_ld, W.out.K);
   if (s.ff_kind == MI_FF_NONE) return MI_OK;
   MI_TRY(norm(W.n2)); MI_TRY(norm(W.n2b));
   MI_TRY(alloc0(c, &W.conv2, (size_t)taps * S->ld * 4, wb));
@@ -180,22 +220,23 @@ int sandwich_layer_create(mi_ctx* c, StackLayer& W, const std::string& p) {
     W.ffk = W.down.K;
     for (const char* n : {"mlp.gate", "mlp.up", "mlp.down"}) want(n);
   } else {
-    W.up.K = S->Kd;
-    W.ffk = pad_to(s.ff_size, 64);
-    S->max_top = std::max(S->max_top, s.experts_top);
-    const ExpertsLinear gu = W.expert_up(), dn = W.expert_dn();
-    MI_TRY(alloc0(c, &W.expert_gu, (size_t)gu.E * gu.N * gu.K * S->elem(), wb));
-    MI_TRY(alloc0(c, &W.expert_down, (size_t)dn.E * dn.N * dn.K * S->elem(), wb));
-    MI_TRY(alloc0(c, &W.router, (size_t)s.experts * S->Kd * S->elem(), wb));
-    MI_TRY(alloc0(c, &W.router_b, (size_t)pad_to(s.experts, 16) * 4, wb));
-    if (!S->f32) MI_TRY(alloc_mat(c, W.router_t, s.experts, S->D, 1.f));
-    S->max_experts = std::max(S->max_experts, pad_to(s.experts, 16));
-    want("mlp.router"); want("mlp.router.b");
-    for (int e = 0; e < s.experts; ++e)
-      for (const char* n : {".gate", ".up", ".down"}) want(("mlp.e" + std::to_string(e) + n).c_str());
+    MI_TRY(experts_create(c, W, p));
   }
   S->act_ld = std::max(S->act_ld, W.ffk);
   return MI_OK;
+}
+
+void experts_tensor_shape(const Stack* S, const mi_layer_spec& s, const std::string& t, int* rows, int* cols) {
+  int e = -1, at = 0;
+  auto is = [&](int r, int k) { *rows = r; *cols = k; };
+  const bool sigmoid = s.router_score == MI_ROUTE_SIGMOID;
+  if (t == "mlp.router") is(s.experts, S->D);
+  else if (t == (sigmoid ? "mlp.correction" : "mlp.router.b")) is(s.experts, 0);
+  else if (sscanf(t.c_str(), "mlp.e%d.%n", &e, &at) == 1 && at > 0 && e >= 0 && e < s.experts) {
+    const std::string m = t.substr(at);
+    if ((m == "gate" && s.ff_act != MI_ACT_RELU2) || m == "up") is(s.ff_size, S->D);
+    else if (m == "down") is(S->D, s.ff_size);
+  }
 }
 
 // shape of a tensor of a sandwich block's layer by its name behind "l<i>."; rows 0: not one of its tensors
@@ -216,23 +257,72 @@ void sandwich_tensor_shape(const Stack* S, const StackLayer& W, const std::strin
     if (t == "mlp.gate" || t == "mlp.up") is(s.ff_size, S->D);
     else if (t == "mlp.down") is(S->D, s.ff_size);
   } else if (s.ff_kind == MI_FF_MOE) {
-    int e = -1, at = 0;
-    if (t == "mlp.router") is(s.experts, S->D);
-    else if (t == "mlp.router.b") is(s.experts, 0);
-    else if (sscanf(t.c_str(), "mlp.e%d.%n", &e, &at) == 1 && at > 0 && e >= 0 && e < s.experts) {
-      const std::string m = t.substr(at);
-      if (m == "gate" || m == "up") is(s.ff_size, S->D);
-      else if (m == "down") is(S->D, s.ff_size);
+    experts_tensor_shape(S, s, t, rows, cols);
+  }
+}
+
+// W_uk: transposed, with ones on the rotated part's diagonal; and, as W_uv, a block of rows of the prompts' matrix
+int latent_place(mi_ctx* c, StackLayer& W, bool k, const float* dev, int cols) {
+  Stack* S = c->stack;
+  const LatentGeom& g = W.lg;
+  hipStream_t st = c->stream;
+  const int n = k ? g.dk : g.dv, dq = g.dq();
+  auto at = [&](void* base, size_t elems) -> void* { return reinterpret_cast<unsigned char*>(base) + elems * S->elem(); };
+  float *tmp = nullptr, *ones = nullptr;      // [rank][dq]: W_uk^T, zeros behind it; [nr][dq]: zeros, then the unit matrix
+  int rc = MI_OK;
+  if (k) {
+    std::vector<float> u((size_t)std::max(g.nr, 1) * dq, 0.f);
+    for (int i = 0; i < g.nr; ++i) u[(size_t)i * dq + g.dk + i] = 1.f;
+    MI_HIP(hipMalloc(reinterpret_cast<void**>(&tmp), (size_t)cols * dq * 4));
+    MI_HIP(hipMalloc(reinterpret_cast<void**>(&ones), u.size() * 4));
+    MI_HIP(hipMemcpyAsync(ones, u.data(), u.size() * 4, hipMemcpyHostToDevice, st));
+    MI_HIP(hipMemsetAsync(tmp, 0, (size_t)cols * dq * 4, st));
+    MI_HIP(hipStreamSynchronize(st));
+  }
+  for (int h = 0; h < g.H && rc == MI_OK; ++h) {
+    const float* src = dev + (size_t)h * n * cols;
+    if (k) {
+      void* dst = at(W.w_uk, (size_t)h * g.cp * g.dkp);
+      rc = launch_transpose(src, n, cols, tmp, dq, st);
+      if (rc == MI_OK) rc = launch_place(tmp, dq, 0, cols, dq, dst, g.dkp, S->f32, 0, 0, st);
+      if (rc == MI_OK && g.nr) rc = launch_place(ones, dq, 0, g.nr, dq, dst, g.dkp, S->f32, g.rp, 0, st);
+    } else {
+      rc = launch_place(src, cols, 0, n, cols, at(W.w_uv, (size_t)h * g.dvp * g.rp), g.rp, S->f32, 0, 0, st);
+    }
+    if (rc == MI_OK && W.fast()) {
+      const int row0 = k ? h * g.dkp : g.H * g.dkp + h * g.dvp;
+      rc = launch_place(src, cols, 0, n, cols, W.ukv.L.w, W.ukv.K, false, row0, 0, st);
+      if (rc == MI_OK && k && g.nr) rc = launch_place(ones, dq, g.dk, g.nr, g.nr, W.ukv.L.w, W.ukv.K, false, row0 + g.dk, g.rp, st);
     }
   }
+  hipStreamSynchronize(st);
+  hipFree(tmp);
+  hipFree(ones);
+  return rc;
+}
+
+int experts_place(mi_ctx* c, StackLayer& W, const std::string& t, const float* dev, int rows, int cols) {
+  Stack* S = c->stack;
+  const mi_layer_spec& s = W.s;
+  hipStream_t st = c->stream;
+  auto at = [&](void* base, size_t elems) -> void* { return reinterpret_cast<unsigned char*>(base) + elems * S->elem(); };
+  auto place = [&](void* dst, int K, int row0 = 0, int step = 1) { return launch_place(dev, cols, 0, rows, cols, dst, K, S->f32, row0, 0, st, step); };
+  if (t == "mlp.router" && !S->f32) MI_TRY(place(W.router_t.L.w, W.router_t.K));
+  if (t == "mlp.router") return launch_place_rows(dev, rows, cols, W.router, S->Kd, S->f32, st);
+  if (t == "mlp.router.b" || t == "mlp.correction") return launch_offset_copy(dev, rows, 0.f, W.router_b, st);
+  int e = -1, off = 0;
+  sscanf(t.c_str(), "mlp.e%d.%n", &e, &off);
+  const std::string m = t.substr(off);
+  const ExpertsLinear gu = W.expert_up(), dn = W.expert_dn();
+  if (m == "down") return place(at(W.expert_down, (size_t)e * dn.N * dn.K), dn.K);
+  if (s.ff_act == MI_ACT_RELU2) return place(at(W.expert_gu, (size_t)e * gu.N * gu.K), gu.K);
+  return place(at(W.expert_gu, (size_t)e * gu.N * gu.K), gu.K, m == "up" ? 1 : 0, 2);
 }
 
 int sandwich_place(mi_ctx* c, StackLayer& W, const std::string& t, const float* dev, int rows, int cols) {
   Stack* S = c->stack;
   const mi_layer_spec& s = W.s;
   hipStream_t st = c->stream;
-  const size_t el = S->elem();
-  auto at = [&](void* base, size_t elems) -> void* { return reinterpret_cast<unsigned char*>(base) + elems * el; };
   auto vec = [&](float* dst) -> int {
     MI_HIP(hipMemcpyAsync(dst, dev, (size_t)rows * 4, hipMemcpyDeviceToDevice, st));
     return MI_OK;
@@ -247,39 +337,140 @@ int sandwich_place(mi_ctx* c, StackLayer& W, const std::string& t, const float* 
   if (t == "mix.dkv") return place(W.qkv.L.w, W.qkv.K, s.num_heads * s.qk_dim);
   if (t == "mix.dkv.norm") return vec(W.c_norm);
   if (t == "mix.o") return place(W.out.L.w, W.out.K);
-  if (t == "mix.uk" || t == "mix.uv") {
-    const bool k = t == "mix.uk";
-    const int n = k ? s.qk_dim : s.v_dim;
-    float* tmp = nullptr;
-    if (k) MI_HIP(hipMalloc(reinterpret_cast<void**>(&tmp), (size_t)n * cols * 4));
-    int rc = MI_OK;
-    for (int h = 0; h < s.num_heads && rc == MI_OK; ++h) {
-      const float* src = dev + (size_t)h * n * cols;
-      if (k) {
-        rc = launch_transpose(src, n, cols, tmp, n, st);
-        if (rc == MI_OK) rc = launch_place(tmp, n, 0, cols, n, at(W.w_uk, (size_t)h * W.lg.rp * W.lg.dkp), W.lg.dkp, S->f32, 0, 0, st);
-      } else {
-        rc = launch_place(src, cols, 0, n, cols, at(W.w_uv, (size_t)h * W.lg.dvp * W.lg.rp), W.lg.rp, S->f32, 0, 0, st);
-      }
-      if (rc == MI_OK && W.fast())
-        rc = launch_place(src, cols, 0, n, cols, W.ukv.L.w, W.ukv.K, false, k ? h * W.lg.dkp : s.num_heads * W.lg.dkp + h * W.lg.dvp, 0, st);
-    }
-    hipStreamSynchronize(st);
-    hipFree(tmp);
-    return rc;
-  }
+  if (t == "mix.uk" || t == "mix.uv") return latent_place(c, W, t == "mix.uk", dev, cols);
   if (t == "mlp.gate") return place(W.up.L.w, W.up.K, 0, 2);
   if (t == "mlp.up") return place(W.up.L.w, W.up.K, 1, 2);
   if (t == "mlp.down") return place(W.down.L.w, W.down.K);
-  if (t == "mlp.router" && !S->f32) MI_TRY(place(W.router_t.L.w, W.router_t.K));
-  if (t == "mlp.router") return launch_place_rows(dev, rows, cols, W.router, S->Kd, S->f32, st);
-  if (t == "mlp.router.b") return vec(W.router_b);
-  int e = -1, off = 0;
-  sscanf(t.c_str(), "mlp.e%d.%n", &e, &off);
-  const std::string m = t.substr(off);
-  const ExpertsLinear gu = W.expert_up(), dn = W.expert_dn();
-  if (m == "down") return place(at(W.expert_down, (size_t)e * dn.N * dn.K), dn.K);
-  return place(at(W.expert_gu, (size_t)e * gu.N * gu.K), gu.K, m == "up" ? 1 : 0, 2);
+  return experts_place(c, W, t, dev, rows, cols);
+}
+
+// ---- one-norm blocks: geometry and weights of one layer ----------------------------------------------------------------------
+int delta_layer_create(mi_ctx* c, StackLayer& W) {
+  Stack* S = c->stack;
+  const mi_layer_spec& s = W.s;
+  size_t* wb = &c->weight_bytes;
+  DeltaGeom& g = W.dg;
+  g = DeltaGeom{s.num_heads, s.num_kv_heads, s.qk_dim, s.v_dim, pad_to(s.qk_dim, 16), pad_to(s.v_dim, 16), s.conv_taps};
+  W.col_b = pad_to(g.channels(), 16);
+  W.col_a = W.col_b + pad_to(g.H, 16);
+  W.col_g = W.col_a + pad_to(s.decay_rank, 16);
+  MI_TRY(alloc_mat(c, W.qkv, W.col_g + s.gate_rank, S->D, 1.f));
+  MI_TRY(alloc_mat(c, W.a2, g.H * g.dk, s.decay_rank, 1.f));
+  MI_TRY(alloc_mat(c, W.g2, g.H * g.dv, s.gate_rank, 1.f));
+  MI_TRY(alloc_mat(c, W.out, S->D, g.H * g.dv, 1.f));
+  MI_TRY(alloc0(c, &W.conv, (size_t)g.taps * g.channels() * 4, wb));
+  MI_TRY(alloc0(c, &W.a_log, (size_t)g.H * 4, wb));
+  MI_TRY(alloc0(c, &W.dt, (size_t)g.H * g.dk * 4, wb));
+  MI_TRY(alloc0(c, &W.o_norm, (size_t)g.dv * 4, wb));
+  S->z_ld = std::max(S->z_ld, W.a2.N + W.g2.N);
+  S->low_ld = std::max(S->low_ld, std::max(W.a2.K, W.g2.K));
+  S->delta_o_cols = std::max(S->delta_o_cols, (size_t)g.H * g.dvp);
+  S->factor_floats = std::max(S->factor_floats, delta_factor_floats(g));
+  S->cat_ld = std::max(S->cat_ld, W.out.K);
+  S->state_slots = c->cfg.max_num_seqs;
+  return MI_OK;
+}
+
+int one_norm_layer_create(mi_ctx* c, StackLayer& W, const std::string& p) {
+  Stack* S = c->stack;
+  const mi_layer_spec& s = W.s;
+  size_t* wb = &c->weight_bytes;
+  auto want = [&](const char* n) { S->missing.push_back(p + n); };
+  MI_TRY(alloc0(c, &W.n1.w, (size_t)S->ld * 4, wb));
+  want("norm1");
+  if (s.mixer_kind == MI_MIX_DELTA) {
+    MI_TRY(delta_layer_create(c, W));
+    for (const char* n : {"q", "q.conv", "k", "k.conv", "v", "v.conv", "b", "A_log", "a1", "a2", "dt_bias", "g1", "g2", "norm", "o"}) want((std::string("mix.") + n).c_str());
+  } else {
+    const int dq = s.num_heads * (s.qk_dim + s.rot_dim), gates = s.out_gate == MI_GATE_HEAD ? s.num_heads : s.out_gate == MI_GATE_ELEMENT ? s.num_heads * s.v_dim : 0;
+    W.col_q = pad_to(s.kv_rank + s.rot_dim, 16);
+    W.col_g = W.col_q + pad_to(s.q_rank ? s.q_rank : dq, 16);
+    MI_TRY(alloc_mat(c, W.qkv, W.col_g + gates, S->D, 1.f));
+    MI_TRY(latent_layer_create(c, W));
+    MI_TRY(alloc0(c, &W.c_norm, (size_t)s.kv_rank * 4, wb));
+    if (s.q_rank) {
+      MI_TRY(alloc_mat(c, W.uq, dq, s.q_rank, 1.f));
+      MI_TRY(alloc0(c, &W.q_norm, (size_t)s.q_rank * 4, wb));
+      S->cq_ld = std::max(S->cq_ld, W.uq.K);
+      S->q2_ld = std::max(S->q2_ld, W.uq.N);
+      for (const char* n : {"mix.dq", "mix.dq.norm", "mix.uq"}) want(n);
+    } else {
+      want("mix.q");
+    }
+    for (const char* n : {"mix.dkv", "mix.dkv.norm", "mix.uk", "mix.uv", "mix.o"}) want(n);
+    if (gates) want("mix.g");
+  }
+  S->qkv_ld = std::max(S->qkv_ld, W.qkv.N);
+  return s.ff_kind == MI_FF_MOE ? experts_create(c, W, p) : MI_OK;
+}
+
+void one_norm_tensor_shape(const Stack* S, const StackLayer& W, const std::string& t, int* rows, int* cols) {
+  const mi_layer_spec& s = W.s;
+  *rows = *cols = 0;
+  auto is = [&](int r, int k) { *rows = r; *cols = k; };
+  if (t == "norm1") return is(S->D, 0);
+  if (s.ff_kind == MI_FF_MOE && t.compare(0, 4, "mlp.") == 0) return experts_tensor_shape(S, s, t, rows, cols);
+  if (t.compare(0, 4, "mix.") != 0) return;
+  const std::string m = t.substr(4);
+  const int H = s.num_heads, G = s.num_kv_heads;
+  if (s.mixer_kind == MI_MIX_DELTA) {
+    const int qk = G * s.qk_dim, v = H * s.v_dim;
+    if (m == "q" || m == "k") is(qk, S->D);
+    else if (m == "q.conv" || m == "k.conv") is(qk, s.conv_taps);
+    else if (m == "v") is(v, S->D);
+    else if (m == "v.conv") is(v, s.conv_taps);
+    else if (m == "b") is(H, S->D);
+    else if (m == "A_log") is(H, 0);
+    else if (m == "a1") is(s.decay_rank, S->D);
+    else if (m == "a2") is(H * s.qk_dim, s.decay_rank);
+    else if (m == "dt_bias") is(H * s.qk_dim, 0);
+    else if (m == "g1") is(s.gate_rank, S->D);
+    else if (m == "g2") is(v, s.gate_rank);
+    else if (m == "norm") is(s.v_dim, 0);
+    else if (m == "o") is(S->D, v);
+    return;
+  }
+  const int dq = H * (s.qk_dim + s.rot_dim);
+  if (m == "dq" && s.q_rank) is(s.q_rank, S->D);
+  else if (m == "dq.norm" && s.q_rank) is(s.q_rank, 0);
+  else if (m == "uq" && s.q_rank) is(dq, s.q_rank);
+  else if (m == "q" && !s.q_rank) is(dq, S->D);
+  else if (m == "dkv") is(s.kv_rank + s.rot_dim, S->D);
+  else if (m == "dkv.norm") is(s.kv_rank, 0);
+  else if (m == "uk") is(H * s.qk_dim, s.kv_rank);
+  else if (m == "uv") is(H * s.v_dim, s.kv_rank);
+  else if (m == "g" && s.out_gate != MI_GATE_NONE) is(s.out_gate == MI_GATE_HEAD ? H : H * s.v_dim, S->D);
+  else if (m == "o") is(S->D, H * s.v_dim);
+}
+
+int one_norm_place(mi_ctx* c, StackLayer& W, const std::string& t, const float* dev, int rows, int cols) {
+  Stack* S = c->stack;
+  const mi_layer_spec& s = W.s;
+  hipStream_t st = c->stream;
+  auto vec = [&](float* dst, float offset = 0.f) { return launch_offset_copy(dev, rows, offset, dst, st); };
+  auto place = [&](const StackMat& m, int row0 = 0) { return launch_place(dev, cols, 0, rows, cols, m.L.w, m.K, S->f32, row0, 0, st); };
+  if (t == "norm1") return vec(W.n1.w, S->cfg.norm_offset);
+  if (t.compare(0, 4, "mlp.") == 0) return experts_place(c, W, t, dev, rows, cols);
+  const std::string m = t.substr(4);
+  if (m == "o") return place(W.out);
+  if (s.mixer_kind == MI_MIX_DELTA) {
+    const DeltaGeom& g = W.dg;
+    const int part = m[0] == 'q' ? 0 : m[0] == 'k' ? g.G * g.dk : 2 * g.G * g.dk;      // the tensor's channels
+    if (m == "q" || m == "k" || m == "v") return place(W.qkv, part);
+    if (m == "q.conv" || m == "k.conv" || m == "v.conv") return launch_transpose(dev, rows, cols, W.conv + part, g.channels(), st);
+    if (m == "b") return place(W.qkv, W.col_b);
+    if (m == "a1") return place(W.qkv, W.col_a);
+    if (m == "g1") return place(W.qkv, W.col_g);
+    if (m == "a2") return place(W.a2);
+    if (m == "g2") return place(W.g2);
+    return vec(m == "A_log" ? W.a_log : m == "dt_bias" ? W.dt : W.o_norm);
+  }
+  if (m == "uk" || m == "uv") return latent_place(c, W, m == "uk", dev, cols);
+  if (m == "dkv") return place(W.qkv);
+  if (m == "dq" || m == "q") return place(W.qkv, W.col_q);
+  if (m == "g") return place(W.qkv, W.col_g);
+  if (m == "uq") return place(W.uq);
+  return vec(m == "dq.norm" ? W.q_norm : W.c_norm);
 }
 
 }  // namespace
@@ -296,6 +487,12 @@ int stack_create(mi_ctx* c, const mi_stack_config& cfg) {
   c->V_l = cfg.vocab_size;
   const bool loop = cfg.loop_times > 0;
   for (int i = 0; i < cfg.num_layers; ++i) {
+    if (S->one_norm()) {
+      int j = i;
+      while (cfg.layers[j].weights_of >= 0) j = cfg.layers[j].weights_of;     // (checked by mi_ctx_create_stack)
+      S->runs.push_back({j, false});
+      continue;
+    }
     if (!loop || i < cfg.loop_start || i >= cfg.loop_stop) {
       S->runs.push_back({i, false});
       continue;
@@ -322,6 +519,10 @@ int stack_create(mi_ctx* c, const mi_stack_config& cfg) {
     StackLayer& W = S->layers[i];
     W.s = cfg.layers[i];
     const mi_layer_spec& s = W.s;
+    if (S->one_norm()) {
+      if (s.weights_of < 0) MI_TRY(one_norm_layer_create(c, W, "l" + std::to_string(i) + "."));
+      continue;
+    }
     if (S->sandwich()) {
       MI_TRY(sandwich_layer_create(c, W, "l" + std::to_string(i) + "."));
       continue;
@@ -364,15 +565,18 @@ void stack_destroy(mi_ctx* c) {
     free_mat(W.qkv); free_mat(W.up); free_mat(W.out);
     free_mat(W.down); free_mat(W.ukv); free_mat(W.router_t);
     free_norm(W.n1); free_norm(W.n2); free_norm(W.n1b); free_norm(W.n2b);
-    void* ps[] = {W.slopes, W.conv1, W.conv2, W.c_norm, W.w_uk, W.w_uv, W.router, W.router_b, W.expert_gu, W.expert_down};
+    free_mat(W.uq); free_mat(W.a2); free_mat(W.g2);
+    void* ps[] = {W.q_norm, W.conv, W.a_log, W.dt, W.o_norm, W.slopes, W.conv1, W.conv2, W.c_norm, W.w_uk, W.w_uv, W.router, W.router_b, W.expert_gu, W.expert_down};
     for (void* p : ps) hipFree(p);
   }
   free_mat(S->loop_in); free_mat(S->head);
   free_norm(S->final_norm);
   void* ptrs[] = {S->embed, S->pos, S->x0, S->qkv_out, S->logits_pad, S->n1, S->n2, S->q, S->cat, S->pair, S->attn_scratch, S->residuals,
                   S->y, S->pair_w, S->pair_ids, S->hb, S->act, S->qa, S->lat, S->kv_x, S->kv_k, S->kv_v, S->kv_bt, S->plan,
-                  S->tickets, S->route_z};
+                  S->tickets, S->route_z, S->cq, S->low, S->q2, S->z, S->delta_o, S->factors};
   for (void* p : ptrs) hipFree(p);
+  for (float* p : S->state_at) hipFree(p);
+  for (Stack::RotTable& r : S->rot) hipFree(r.t);
   delete S;
   c->stack = nullptr;
 }
@@ -412,6 +616,8 @@ int stack_load_tensor(mi_ctx* c, const std::string& name, const float* dev, int 
   if (name == "embed") return table(S->embed, k.vocab_size);
   if (name == "pos" && k.max_positions > 0) return table(S->pos, k.max_positions);
   if (name == "head") return place(S->head, k.vocab_size, S->D);
+  if (name == "final.norm" && k.norm_offset != 0.f)
+    return rows == S->D && cols == 0 ? done(launch_offset_copy(dev, rows, k.norm_offset, S->final_norm.w, s)) : bad();
   if (name == "final.norm") return vec(S->final_norm.w);
   if (name == "final.norm.b" && k.norm_groups == 0) return vec(S->final_norm.b);
   if (name == "loop.in" && k.loop_times > 0) {   // [x ; x0]: the halves at columns 0 and Kd
@@ -424,6 +630,13 @@ int stack_load_tensor(mi_ctx* c, const std::string& name, const float* dev, int 
     StackLayer& W = S->layers[l];
     const mi_layer_spec& p = W.s;
     const std::string t = name.substr(at);
+    if (S->one_norm()) {
+      int r = 0, cl = 0;
+      if (p.weights_of < 0) one_norm_tensor_shape(S, W, t, &r, &cl);
+      if (r > 0) return rows == r && cols == cl ? done(one_norm_place(c, W, t, dev, rows, cols)) : bad();
+      set_error("tensor " + name + " is not part of this model's configuration");
+      return MI_EINVAL;
+    }
     if (S->sandwich()) {
       int r = 0, cl = 0;
       sandwich_tensor_shape(S, W, t, &r, &cl);
@@ -469,7 +682,12 @@ int stack_synthetic(mi_ctx* c, uint64_t seed, float std) {
     if (n == "embed" || n == "head") { rows = k.vocab_size; cols = S->D; if (n == "embed") sd = 1.f; }
     else if (n == "pos") { rows = k.max_positions; cols = S->D; sd = 0.1f; }
     else if (n == "loop.in") cols = 2 * S->D;
-    else if (!is_norm) {
+    else if (S->one_norm() && n[0] == 'l') {
+      const StackLayer& W = S->layers[atoi(n.c_str() + 1)];
+      one_norm_tensor_shape(S, W, n.substr(n.find('.') + 1), &rows, &cols);
+      if (n.find(".conv") != std::string::npos) sd = 0.3f;
+      is_norm = cols == 0;
+    } else if (!is_norm) {
       const int l = atoi(n.c_str() + 1);
       const mi_layer_spec& p = S->layers[l].s;
       const std::string t = n.substr(n.find('.') + 1);
@@ -489,7 +707,9 @@ int stack_synthetic(mi_ctx* c, uint64_t seed, float std) {
       MI_HIP(hipMalloc(reinterpret_cast<void**>(&buf), elems * 4));
       cap = elems;
     }
-    if (is_norm) rc = launch_fill_f32(buf, elems, n.size() > 2 && n.compare(n.size() - 2, 2, ".b") == 0 ? 0.f : 1.f, c->stream);
+    if (is_norm && S->one_norm())     // norms around zero; plain ones; decays, biases and corrections zero
+      rc = launch_fill_f32(buf, elems, n.find(".mix.") != std::string::npos && n.find("norm") != std::string::npos ? 1.f : 0.f, c->stream);
+    else if (is_norm) rc = launch_fill_f32(buf, elems, n.size() > 2 && n.compare(n.size() - 2, 2, ".b") == 0 ? 0.f : 1.f, c->stream);
     else rc = launch_randn(buf, elems, seed, tid, sd, c->stream);
     ++tid;
     if (rc == MI_OK) rc = stack_load_tensor(c, n, buf, rows, cols);
@@ -509,16 +729,27 @@ void stack_artifact_tensors(mi_ctx* c, std::vector<std::pair<void*, size_t>>& ou
   if (S->pos) out.push_back({S->pos, (size_t)S->cfg.max_positions * S->D * S->elem()});
   if (S->cfg.loop_times > 0) mat(S->loop_in);
   for (StackLayer& W : S->layers) {
-    if (S->sandwich()) {
+    if (S->one_norm() && W.s.weights_of >= 0) continue;
+    if (!S->sandwich() && !S->one_norm()) {
+      mat(W.qkv); mat(W.out); norm(W.n1);
+      if (W.ff_cols) { mat(W.up); norm(W.n2); }
+      continue;
+    }
+    {
       const mi_layer_spec& p = W.s;
       auto put = [&](void* q, size_t bytes) { if (q) out.push_back({q, bytes}); };
       const size_t el = S->elem(), cb = (size_t)S->cfg.conv_taps * S->ld * 4;
       mat(W.qkv); mat(W.out);
       put(W.n1.w, nb); put(W.n1b.w, nb); put(W.n2.w, nb); put(W.n2b.w, nb);
       put(W.conv1, cb); put(W.conv2, cb); put(W.c_norm, (size_t)p.kv_rank * 4);
-      put(W.w_uk, (size_t)p.num_heads * W.lg.rp * W.lg.dkp * el);
+      put(W.w_uk, (size_t)p.num_heads * W.lg.cp * W.lg.dkp * el);
       put(W.w_uv, (size_t)p.num_heads * W.lg.dvp * W.lg.rp * el);
       if (W.fast()) mat(W.ukv);
+      for (StackMat* m : {&W.uq, &W.a2, &W.g2})
+        if (m->L.w) mat(*m);
+      put(W.q_norm, (size_t)p.q_rank * 4);
+      put(W.conv, (size_t)W.dg.taps * W.dg.channels() * 4); put(W.a_log, (size_t)W.dg.H * 4);
+      put(W.dt, (size_t)W.dg.H * W.dg.dk * 4); put(W.o_norm, (size_t)W.dg.dv * 4);
       if (p.ff_kind == MI_FF_GLU) { mat(W.up); mat(W.down); }
       if (p.ff_kind == MI_FF_MOE) {
         const ExpertsLinear gu = W.expert_up(), dn = W.expert_dn();
@@ -526,10 +757,7 @@ void stack_artifact_tensors(mi_ctx* c, std::vector<std::pair<void*, size_t>>& ou
         if (!S->f32) mat(W.router_t);
         put(W.expert_gu, (size_t)gu.E * gu.N * gu.K * el); put(W.expert_down, (size_t)dn.E * dn.N * dn.K * el);
       }
-      continue;
     }
-    mat(W.qkv); mat(W.out); norm(W.n1);
-    if (W.ff_cols) { mat(W.up); norm(W.n2); }
   }
   norm(S->final_norm);
   mat(S->head);
@@ -544,14 +772,17 @@ int stack_geometry_hash(const mi_ctx* c) {
   const mi_stack_config& k = S->cfg;
   const int32_t g[9] = {k.num_layers, k.width, k.vocab_size, k.max_positions, k.loop_times > 0, k.compute_dtype, k.block_kind, k.norm_groups, k.conv_taps};
   mix(g, sizeof g);
+  const float f[2] = {k.embed_scale, k.norm_offset};
+  if (S->one_norm()) mix(f, sizeof f);
   for (const StackLayer& W : S->layers) mix(&W.s, sizeof W.s);
   return (int)(h & 0x7fffffff);
 }
 
 static size_t kv_run_elems_per_block(const mi_ctx* c, const StackLayer& W) {
   const Stack* S = c->stack;
+  if (S->one_norm()) return W.s.mixer_kind == MI_MIX_LATENT ? (size_t)c->cfg.block_size * W.lg.cp : 0;
   if (S->sandwich())   // latents (own ones) and both convolutions' state
-    return (W.s.kv_from < 0 ? (size_t)c->cfg.block_size * W.lg.rp : 0) + (size_t)S->conv_keep * S->Kd * (W.s.ff_kind == MI_FF_NONE ? 1 : 2);
+    return (W.s.kv_from < 0 ? (size_t)c->cfg.block_size * W.lg.cp : 0) + (size_t)S->conv_keep * S->Kd * (W.s.ff_kind == MI_FF_NONE ? 1 : 2);
   return (size_t)W.g.G * c->cfg.block_size * (W.g.dkp + W.g.dvp);
 }
 size_t stack_kv_bytes_per_block(const mi_ctx* c) {
@@ -562,7 +793,7 @@ size_t stack_kv_bytes_per_block(const mi_ctx* c) {
 
 static size_t stack_scratch(const mi_ctx* c) {
   size_t b = 16;
-  if (c->stack->sandwich()) {
+  if (c->stack->sandwich() || c->stack->one_norm()) {
     for (const StackLayer& W : c->stack->layers)
       if (W.fast()) b = std::max(b, latent_attn_scratch_bytes(W.lg));
     return b;
@@ -576,11 +807,27 @@ static int kv_work_rows(const mi_ctx* c) {
   return c->stack->kv_ldx ? 2 * pad_to(std::max(c->max_rows, c->cfg.max_model_len), kKvBlock) + 2 * kKvBlock : 0;
 }
 
+bool stack_has_state(const mi_ctx* c) { return c->stack && c->stack->state_slots > 0; }
+
+static size_t state_floats(const mi_ctx* c, const StackLayer& W) {
+  return W.s.mixer_kind == MI_MIX_DELTA ? c->stack->state_slots * (W.dg.state_floats() + W.dg.ring_floats()) : 0;
+}
+// chunks of prompts whose factors are in memory at a time
+static int delta_chunks(const mi_ctx* c) { return std::min(512, c->max_rows / kDeltaChunk + c->cfg.max_num_seqs); }
+
 size_t stack_workspace_estimate(const mi_ctx* c) {
   const Stack* S = c->stack;
   const size_t R = (size_t)c->max_rows;
+  size_t extra = 0;
+  if (S->one_norm()) {
+    for (const StackRun& r : S->runs) extra += state_floats(c, S->layers[r.layer]) * 4;
+    if (S->state_slots) extra += (size_t)delta_chunks(c) * S->factor_floats * 4;
+    extra += R * ((size_t)S->z_ld + S->delta_o_cols + S->q2_ld) * 4 + R * (2 * (size_t)S->low_ld + S->cq_ld) * S->elem();
+    for (const StackLayer& W : S->layers) extra += W.s.mixer_kind == MI_MIX_LATENT ? (size_t)c->cfg.max_model_len * W.s.rot_dims * 4 : 0;
+  }
   size_t b = 3 * R * S->ld * 4 + R * S->qkv_ld * 4 + R * (4 * (size_t)S->Kd + S->q_cols + S->cat_ld) * S->elem();
-  if (S->sandwich()) {
+  b += extra;
+  if (S->sandwich() || S->one_norm()) {
     const size_t pairs = R * std::max(1, S->max_top);
     b += (size_t)kv_work_rows(c) * (S->kv_ldx + S->kv_k_cols + S->kv_v_cols) * 2;
     b += pairs * S->ld * 4 + pairs * 16 + R * (S->max_experts + 1) * 4 + R * S->Kd * S->elem() + pairs * S->act_ld * S->elem() + 2 * R * S->lat_cols * S->elem();
@@ -588,6 +835,48 @@ size_t stack_workspace_estimate(const mi_ctx* c) {
   b += (size_t)64 << 20;
   b += 2 * (size_t)c->cfg.max_num_seqs * pad_to(c->V_l, 16) * 4;
   return b + stack_scratch(c) + ((size_t)8 << 20);
+}
+
+// recurrent state, rotation tables and the workspace only one-norm blocks have
+static int one_norm_alloc(mi_ctx* c) {
+  Stack* S = c->stack;
+  const size_t R = (size_t)c->max_rows;
+  size_t* ws = &c->workspace_bytes;
+  for (const StackRun& r : S->runs) {
+    float* p = nullptr;
+    if (const size_t n = state_floats(c, S->layers[r.layer])) MI_TRY(alloc0(c, &p, n * 4, &c->kv_bytes));
+    S->state_at.push_back(p);
+  }
+  for (StackLayer& W : S->layers) {
+    if (W.s.weights_of >= 0 || W.s.mixer_kind != MI_MIX_LATENT || W.s.rot_dim == 0) continue;
+    for (const Stack::RotTable& r : S->rot)
+      if (r.base == W.s.rot_base && r.dims == W.s.rot_dims) W.rot = r.t;
+    if (W.rot) continue;
+    const int half = W.s.rot_dims / 2, P = c->cfg.max_model_len;
+    std::vector<float2> t(std::max<size_t>((size_t)P * half, 1));
+    for (int i = 0; i < half; ++i) {
+      const double f = std::pow((double)W.s.rot_base, -2.0 * i / W.s.rot_dims);
+      for (int p = 0; p < P; ++p) t[(size_t)p * half + i] = make_float2((float)std::cos(p * f), (float)std::sin(p * f));
+    }
+    float2* d = nullptr;
+    MI_TRY(alloc0(c, &d, t.size() * sizeof(float2), ws));
+    S->rot.push_back({W.s.rot_base, W.s.rot_dims, d});
+    MI_HIP(hipMemcpyAsync(d, t.data(), t.size() * sizeof(float2), hipMemcpyHostToDevice, c->stream));
+    MI_HIP(hipStreamSynchronize(c->stream));
+    W.rot = d;
+  }
+  if (S->cq_ld) {
+    MI_TRY(alloc0(c, &S->cq, R * S->cq_ld * S->elem(), ws));
+    MI_TRY(alloc0(c, &S->q2, R * S->q2_ld * 4, ws));
+  }
+  if (S->state_slots) {
+    S->delta_chunks = delta_chunks(c);
+    MI_TRY(alloc0(c, &S->low, 2 * R * S->low_ld * S->elem(), ws));
+    MI_TRY(alloc0(c, &S->z, R * S->z_ld * 4, ws));
+    MI_TRY(alloc0(c, &S->delta_o, R * S->delta_o_cols * 4, ws));
+    MI_TRY(alloc0(c, &S->factors, (size_t)S->delta_chunks * S->factor_floats * 4, ws));
+  }
+  return MI_OK;
 }
 
 int stack_alloc(mi_ctx* c) {
@@ -608,27 +897,28 @@ int stack_alloc(mi_ctx* c) {
     return MI_ENOMEM;
   }
   // zero-filled: rows that were never written must hold finite values
-  MI_TRY(alloc0(c, &c->kv_pool, kv_bytes, &c->kv_bytes));
+  MI_TRY(alloc0(c, &c->kv_pool, std::max<size_t>(kv_bytes, 16), &c->kv_bytes));
   size_t at = 0;
   for (const StackRun& r : S->runs) {
     const StackLayer& W = S->layers[r.layer];
     const bool shared = S->sandwich() && W.s.kv_from >= 0;
     S->kv_at.push_back(shared ? S->kv_at[W.s.kv_from] : at);
-    if (S->sandwich()) S->conv_at.push_back(at + (shared ? 0 : (size_t)k.num_blocks * k.block_size * W.lg.rp));
+    if (S->sandwich()) S->conv_at.push_back(at + (shared ? 0 : (size_t)k.num_blocks * k.block_size * W.lg.cp));
     at += kv_run_elems_per_block(c, W) * k.num_blocks;
   }
+  if (S->one_norm()) MI_TRY(one_norm_alloc(c));
   const size_t R = (size_t)c->max_rows;
   size_t* ws = &c->workspace_bytes;
   MI_TRY(alloc0(c, &c->resid[0], R * S->ld * 4, ws));
   MI_TRY(alloc0(c, &c->resid[1], R * S->ld * 4, ws));
   MI_TRY(alloc0(c, &S->n1, R * S->Kd * S->elem(), ws));
-  if (S->sandwich()) {
+  if (S->sandwich() || S->one_norm()) {
     const size_t pairs = R * std::max(1, S->max_top);   // (a dense feed-forward: one "pair" per row)
     MI_TRY(alloc0(c, &S->y, pairs * S->ld * 4, ws));
     MI_TRY(alloc0(c, &S->hb, R * S->Kd * S->elem(), ws));
     if (S->act_ld) MI_TRY(alloc0(c, &S->act, pairs * S->act_ld * S->elem(), ws));
-    MI_TRY(alloc0(c, &S->qa, R * S->lat_cols * S->elem(), ws));
-    MI_TRY(alloc0(c, &S->lat, R * S->lat_cols * S->elem(), ws));
+    MI_TRY(alloc0(c, &S->qa, std::max<size_t>(R * S->lat_cols * S->elem(), 16), ws));
+    MI_TRY(alloc0(c, &S->lat, std::max<size_t>(R * S->lat_cols * S->elem(), 16), ws));
     if (S->kv_ldx) {
       S->kv_rows = kv_work_rows(c);
       S->kv_mb = ceil_div(k.max_model_len, kKvBlock) + 1;
@@ -648,7 +938,7 @@ int stack_alloc(mi_ctx* c) {
     MI_TRY(alloc0(c, &S->n2, R * S->Kd * S->elem(), ws));
   }
   MI_TRY(alloc0(c, &S->qkv_out, R * S->qkv_ld * 4, ws));
-  MI_TRY(alloc0(c, &S->q, R * S->q_cols * S->elem(), ws));
+  MI_TRY(alloc0(c, &S->q, std::max<size_t>(R * S->q_cols * S->elem(), 16), ws));
   MI_TRY(alloc0(c, &S->cat, R * S->cat_ld * S->elem(), ws));
   if (S->cfg.loop_times > 0) {
     MI_TRY(alloc0(c, &S->x0, R * S->ld * 4, ws));
@@ -691,7 +981,7 @@ int latent_attention_plain(mi_ctx* c, const StackLayer& W, const void* pool, con
   Stack* S = c->stack;
   const LatentGeom& g = W.lg;
   Scope sc(c, b.decode ? MI_K_ATTN_DECODE : MI_K_ATTN_PREFILL);
-  MI_TRY(launch_head_linear(W.w_uk, g.H, g.rp, g.dkp, S->q, b.rows, S->qa, g.H * g.rp, g.rp, g.rp, S->f32, c->stream));
+  MI_TRY(launch_head_linear(W.w_uk, g.H, g.cp, g.dkp, S->q, b.rows, S->qa, g.H * g.cp, g.cp, g.cp, S->f32, c->stream));
   MI_TRY(launch_attn_plain(W.latent, S->qa, pool, pool, c->cfg.block_size, c->d_bt, b.MB, c->d_pos,
                            b.decode ? nullptr : reinterpret_cast<const AttnSeg*>(c->d_segs), b.nseg, b.rows, S->lat, g.H * g.rp, S->f32, c->stream));
   return launch_head_linear(W.w_uv, g.H, g.dvp, g.rp, S->lat, b.rows, S->cat, S->cat_ld, g.dv, g.dv, S->f32, c->stream);
@@ -719,7 +1009,7 @@ int latent_attention(mi_ctx* c, const StackLayer& W, const uint16_t* pool, const
   if (lr.rows > 0) {
     Scope sc(c, cls);
     if (!b.decode || !latent_token_supported(g))   // (token generation: done with the scatter)
-      MI_TRY(launch_head_linear_rows(W.w_uk, g.H, g.rp, g.dkp, q, lr, qa, g.H * g.rp, g.rp, g.rp, s));
+      MI_TRY(launch_head_linear_rows(W.w_uk, g.H, g.cp, g.dkp, q, lr, qa, g.H * g.cp, g.cp, g.cp, s));
     MI_TRY(launch_latent_attn_rows(g, W.s.scale, W.s.window, qa, pool, k.block_size, c->d_bt, b.MB, c->d_pos, lr, k.max_model_len, W.w_uv,
                                    reinterpret_cast<uint16_t*>(S->lat), out, S->cat_ld, S->attn_scratch, s));
   }
@@ -763,15 +1053,16 @@ int latent_mixer(mi_ctx* c, const StackLayer& W, size_t kv_at, const Batch& b, R
   SlabSum slabs;       // (many rows: a K-split's sum is left to the scatter)
   MI_TRY(apply(c, W.qkv, b.rows, S->n1, S->Kd, EPI_F32, e, b.rows >= 384 ? &slabs : nullptr));
   unsigned char* pool = reinterpret_cast<unsigned char*>(c->kv_pool) + kv_at * S->elem();
+  const LatentRowsIn in{S->qkv_out, S->qkv_out + g.H * g.dk, W.qkv.N, W.qkv.N};
   if (b.decode && W.fast() && latent_token_supported(g)) {
     if (runs_other(c)) {
       Scope sc(c, MI_K_OTHER);
-      MI_TRY(launch_latent_token(S->qkv_out, W.qkv.N, b.rows, g, W.w_uk, W.c_norm, S->cfg.norm_eps, c->d_slots, reinterpret_cast<uint16_t*>(S->qa),
+      MI_TRY(launch_latent_token(in, b.rows, g, Rotation(), W.w_uk, W.c_norm, S->cfg.norm_eps, c->d_slots, reinterpret_cast<uint16_t*>(S->qa),
                                  reinterpret_cast<uint16_t*>(pool), s));
     }
   } else if (runs_other(c)) {
     Scope sc(c, MI_K_OTHER);
-    MI_TRY(launch_latent_scatter(S->qkv_out, W.qkv.N, b.rows, g, W.c_norm, S->cfg.norm_eps, c->d_slots, k.block_size, S->q, pool, S->f32, s, &slabs));
+    MI_TRY(launch_latent_scatter(in, b.rows, g, Rotation(), W.c_norm, S->cfg.norm_eps, c->d_slots, k.block_size, S->q, pool, S->f32, s, &slabs));
   }
   MI_TRY(W.fast() ? latent_attention(c, W, reinterpret_cast<const uint16_t*>(pool), b) : latent_attention_plain(c, W, pool, b));
   EpiArgs o{};
@@ -807,35 +1098,35 @@ int expert_ff(mi_ctx* c, const StackLayer& W, int rows, RowSource& out) {
     {
       Scope sc(c, MI_K_GEMM);
       EpiArgs e{};
-      e.scale = W.router_t.L.scale; e.bias = W.router_b;
+      e.scale = W.router_t.L.scale; e.bias = W.rule().sigmoid ? nullptr : W.router_b;
       e.out_f32 = S->route_z; e.ld_out = W.router_t.N;
       MI_TRY(launch_gemm(W.router_t.L.view(), rows, reinterpret_cast<const uint16_t*>(S->n1), S->Kd, EPI_F32, e, s, c->splitk_ws, c->splitk_ws_bytes));
     }
     if (runs_other(c)) {
       Scope sc(c, MI_K_OTHER);
-      MI_TRY(launch_route_pick(S->route_z, W.router_t.N, rows, p.experts, p.experts_top, S->pair_ids, S->pair_w, s));
+      MI_TRY(launch_route_pick(S->route_z, W.router_t.N, rows, W.rule(), p.experts, p.experts_top, S->pair_ids, S->pair_w, s));
       MI_TRY(launch_experts_sort(plan, S->pair_ids, pairs, p.experts, s));
     }
     Scope sc(c, MI_K_GEMM);
     uint16_t *act = reinterpret_cast<uint16_t*>(S->act), *y = reinterpret_cast<uint16_t*>(S->y);
-    MI_TRY(launch_experts_gemm(W.expert_up(), plan, pairs, reinterpret_cast<const uint16_t*>(S->n1), S->Kd, p.experts_top, true, act, S->act_ld, s));
-    MI_TRY(launch_experts_gemm(W.expert_dn(), plan, pairs, act, S->act_ld, 1, false, y, S->ld, s));
+    MI_TRY(launch_experts_gemm(W.expert_up(), plan, pairs, reinterpret_cast<const uint16_t*>(S->n1), S->Kd, p.experts_top, W.ff_act(), act, S->act_ld, s));
+    MI_TRY(launch_experts_gemm(W.expert_dn(), plan, pairs, act, S->act_ld, 1, EXPERT_LINEAR, y, S->ld, s));
     out.y16 = y;
     return MI_OK;
   }
   if (runs_other(c)) {
     Scope sc(c, MI_K_OTHER);
-    MI_TRY(launch_route(S->n1, S->Kd, rows, W.router, W.router_b, p.experts, S->Kd, p.experts_top, S->pair_ids, S->pair_w, S->f32, s,
+    MI_TRY(launch_route(S->n1, S->Kd, rows, W.router, W.rule(), p.experts, S->Kd, p.experts_top, S->pair_ids, S->pair_w, S->f32, s,
                         S->f32 ? nullptr : S->route_z, S->f32 ? nullptr : S->tickets));
   }
   const int cls = S->f32 ? MI_K_GEMM : MI_K_GEMV;
   if (c->runs(cls)) {
     Scope sc(c, cls);
-    MI_TRY(launch_experts_linear(W.expert_up(), S->pair_ids, pairs, S->n1, S->Kd, p.experts_top, true, S->act, S->act_ld, S->f32, s));
+    MI_TRY(launch_experts_linear(W.expert_up(), S->pair_ids, pairs, S->n1, S->Kd, p.experts_top, W.ff_act(), S->act, S->act_ld, S->f32, s));
   }
   if (c->runs(cls)) {
     Scope sc(c, cls);
-    MI_TRY(launch_experts_linear(W.expert_dn(), S->pair_ids, pairs, S->act, S->act_ld, 1, false, S->y, S->ld, S->f32, s));
+    MI_TRY(launch_experts_linear(W.expert_dn(), S->pair_ids, pairs, S->act, S->act_ld, 1, EXPERT_LINEAR, S->y, S->ld, S->f32, s));
   }
   out.y = S->y;
   return MI_OK;
@@ -865,6 +1156,114 @@ int sandwich_trunk(mi_ctx* c, const Batch& b, int& cur) {
   return keep(S->runs.size() - 1);
 }
 
+// ---- one-norm blocks -----------------------------------------------------------------------------------------------------------
+int one_norm_latent(mi_ctx* c, const StackLayer& W, size_t kv_at, const Batch& b) {
+  Stack* S = c->stack;
+  const LatentGeom& g = W.lg;
+  hipStream_t s = c->stream;
+  EpiArgs e{};
+  e.out_f32 = S->qkv_out; e.ld_out = W.qkv.N;
+  MI_TRY(apply(c, W.qkv, b.rows, S->n1, S->Kd, EPI_F32, e));
+  LatentRowsIn in{S->qkv_out + W.col_q, S->qkv_out, W.qkv.N, W.qkv.N};
+  if (W.s.q_rank) {
+    if (runs_other(c)) {
+      Scope sc(c, MI_K_OTHER);
+      MI_TRY(launch_columns(S->qkv_out, W.qkv.N, W.col_q, W.s.q_rank, W.q_norm, S->cfg.norm_eps, b.rows, S->cq, W.uq.K, S->f32, s));
+    }
+    EpiArgs u{};
+    u.out_f32 = S->q2; u.ld_out = W.uq.N;
+    MI_TRY(apply(c, W.uq, b.rows, S->cq, W.uq.K, EPI_F32, u));
+    in.q = S->q2; in.ldq = W.uq.N;
+  }
+  const Rotation rot{W.rot, c->d_pos};
+  unsigned char* pool = reinterpret_cast<unsigned char*>(c->kv_pool) + kv_at * S->elem();
+  if (runs_other(c)) {
+    Scope sc(c, MI_K_OTHER);
+    if (b.decode && W.fast() && latent_token_supported(g))
+      MI_TRY(launch_latent_token(in, b.rows, g, rot, W.w_uk, W.c_norm, S->cfg.norm_eps, c->d_slots, reinterpret_cast<uint16_t*>(S->qa),
+                                 reinterpret_cast<uint16_t*>(pool), s));
+    else
+      MI_TRY(launch_latent_scatter(in, b.rows, g, rot, W.c_norm, S->cfg.norm_eps, c->d_slots, c->cfg.block_size, S->q, pool, S->f32, s));
+  }
+  MI_TRY(W.fast() ? latent_attention(c, W, reinterpret_cast<const uint16_t*>(pool), b) : latent_attention_plain(c, W, pool, b));
+  if (W.s.out_gate == MI_GATE_NONE || !runs_other(c)) return MI_OK;
+  Scope sc(c, MI_K_OTHER);
+  return launch_gate_rows(S->cat, S->cat_ld, b.rows, g.H, g.dv, S->qkv_out + W.col_g, W.qkv.N, W.s.out_gate == MI_GATE_ELEMENT, S->f32, s);
+}
+
+int one_norm_delta(mi_ctx* c, const StackLayer& W, float* state, const Batch& b) {
+  Stack* S = c->stack;
+  const DeltaGeom& g = W.dg;
+  hipStream_t s = c->stream;
+  EpiArgs e{};
+  e.out_f32 = S->qkv_out; e.ld_out = W.qkv.N;
+  MI_TRY(apply(c, W.qkv, b.rows, S->n1, S->Kd, EPI_F32, e));
+  void* low2 = reinterpret_cast<unsigned char*>(S->low) + (size_t)c->max_rows * S->low_ld * S->elem();
+  if (runs_other(c)) {
+    Scope sc(c, MI_K_OTHER);
+    MI_TRY(launch_columns(S->qkv_out, W.qkv.N, W.col_a, W.s.decay_rank, nullptr, 0.f, b.rows, S->low, S->low_ld, S->f32, s));
+    MI_TRY(launch_columns(S->qkv_out, W.qkv.N, W.col_g, W.s.gate_rank, nullptr, 0.f, b.rows, low2, S->low_ld, S->f32, s));
+  }
+  const int ldz = W.a2.N + W.g2.N;
+  EpiArgs z{};
+  z.out_f32 = S->z; z.ld_out = ldz;
+  MI_TRY(apply(c, W.a2, b.rows, S->low, S->low_ld, EPI_F32, z));
+  z.out_f32 = S->z + W.a2.N;
+  MI_TRY(apply(c, W.g2, b.rows, low2, S->low_ld, EPI_F32, z));
+  DeltaIn in;
+  in.proj = S->qkv_out; in.ldp = W.qkv.N; in.beta = W.col_b;
+  in.z = S->z; in.ldz = ldz; in.gate = W.a2.N;
+  in.conv = W.conv; in.a_log = W.a_log; in.dt = W.dt; in.norm = W.o_norm;
+  in.eps = S->cfg.norm_eps;
+  in.state = state; in.ring = state + (size_t)S->state_slots * g.state_floats();
+  in.slots = c->d_state; in.pos = c->d_pos;
+  const int cls = b.decode ? MI_K_ATTN_DECODE : MI_K_ATTN_PREFILL;
+  if (!c->runs(cls)) return MI_OK;
+  Scope sc(c, cls);
+  if (b.decode) return launch_delta_token(g, in, b.rows, nullptr, S->cat, S->cat_ld, S->f32, s);
+  int ones = 0;
+  for (int i = 0; i < b.nseg; ++i) ones += b.segs[i].n == 1;
+  const AttnSeg* segs = reinterpret_cast<const AttnSeg*>(c->d_segs);
+  if (ones) MI_TRY(launch_delta_token(g, in, b.nseg, segs, S->cat, S->cat_ld, S->f32, s));
+  if (ones < b.nseg) MI_TRY(launch_delta_prompt(g, in, segs, b.segs, b.nseg, S->factors, S->delta_chunks, S->delta_o, S->cat, S->cat_ld, S->f32, s));
+  return MI_OK;
+}
+
+// The feed-forward runs ahead of the mixer: the mixer's output projection may leave a K-split's sum in the workspace that the
+// router's product uses too.
+int one_norm_trunk(mi_ctx* c, const Batch& b, int& cur) {
+  Stack* S = c->stack;
+  RowSource src;
+  auto keep = [&](size_t run) -> int {
+    if (S->residuals)
+      MI_HIP(hipMemcpyAsync(S->residuals + run * c->max_rows * S->ld, c->resid[cur], (size_t)b.rows * S->ld * 4, hipMemcpyDeviceToDevice, c->stream));
+    return MI_OK;
+  };
+  auto row = [&](const float* w_norm) -> int {
+    const bool add = src.any();
+    if (runs_other(c) && (add || w_norm)) {
+      Scope sc(c, MI_K_OTHER);
+      MI_TRY(launch_sandwich_rows(c->resid[cur], c->resid[cur ^ 1], src, nullptr, w_norm, b.rows, S->D, S->ld, 1, S->cfg.norm_eps, nullptr, S->n1, S->Kd, S->f32, c->stream));
+    }
+    if (add) cur ^= 1;
+    src = RowSource();
+    return MI_OK;
+  };
+  for (size_t i = 0; i < S->runs.size(); ++i) {
+    const StackLayer& W = S->layers[S->runs[i].layer];
+    MI_TRY(row(W.n1.w));
+    if (i > 0) MI_TRY(keep(i - 1));
+    if (W.s.ff_kind == MI_FF_MOE) MI_TRY(expert_ff(c, W, b.rows, src));
+    MI_TRY(W.s.mixer_kind == MI_MIX_DELTA ? one_norm_delta(c, W, S->state_at[i], b) : one_norm_latent(c, W, S->kv_at[i], b));
+    EpiArgs e{};
+    e.out_f32 = c->resid[cur ^ 1]; e.resid_in = c->resid[cur]; e.ld_out = S->ld;
+    MI_TRY(apply(c, W.out, b.rows, S->cat, S->cat_ld, EPI_RESID, e, b.rows >= 384 ? &src.slabs : nullptr));
+    if (!src.slabs.slab) cur ^= 1;
+  }
+  MI_TRY(row(nullptr));
+  return keep(S->runs.size() - 1);
+}
+
 }  // namespace
 
 int stack_trunk(mi_ctx* c, int rows, bool decode, int MB, const AttnSeg* segs, int nseg) {
@@ -874,7 +1273,12 @@ int stack_trunk(mi_ctx* c, int rows, bool decode, int MB, const AttnSeg* segs, i
   int cur = 0;
   if (runs_other(c)) {
     Scope sc(c, MI_K_OTHER);
-    MI_TRY(launch_embed_pos(c->d_ids, c->d_pos, S->embed, S->pos, S->f32, rows, S->D, S->ld, c->resid[0], S->x0, s));
+    MI_TRY(launch_embed_pos(c->d_ids, c->d_pos, S->embed, S->pos, S->cfg.embed_scale, S->f32, rows, S->D, S->ld, c->resid[0], S->x0, s));
+  }
+  if (S->one_norm()) {
+    MI_TRY(one_norm_trunk(c, Batch{rows, decode, MB, segs, nseg}, cur));
+    c->tail_cur = cur;
+    return MI_OK;
   }
   if (S->sandwich()) {
     MI_TRY(sandwich_trunk(c, Batch{rows, decode, MB, segs, nseg}, cur));

@@ -50,10 +50,10 @@ int latent_op(const mi_layer_spec& p, const float* uk, const float* uv, const vo
               const int32_t* pos, const int32_t* segs_host, int nseg, int T, int max_ctx, void* out, int ldo, bool f32, int path, hipStream_t s) {
   Arena mem;
   const int H = p.num_heads;
-  const LatentGeom g{H, p.qk_dim, p.v_dim, p.kv_rank, pad_to(p.qk_dim, 32), pad_to(p.v_dim, 32), pad_to(p.kv_rank, 32)};
-  const HeadGeom kvg{H, H, g.dk, g.dv, g.dkp, g.dvp};
+  const LatentGeom g = latent_geom(H, p.qk_dim, p.v_dim, p.kv_rank, p.rot_dim, p.rot_dims);
+  const HeadGeom kvg{H, H, g.dq(), g.dv, g.dkp, g.dvp};
   const size_t el = f32 ? 4 : 2;
-  const int Kc = pad_to(g.rank, 64), nkv = H * (g.dkp + g.dvp);
+  const int dq = g.dq(), Kc = pad_to(g.nr ? g.rp + g.nr : g.rank, 64), nkv = H * (g.dkp + g.dvp);
   std::vector<AttnSeg> segs;
   AttnSeg* sd = nullptr;
   MI_TRY(take_segs(mem, segs_host, nseg, T, bs, MB, segs, &sd, s));
@@ -64,26 +64,35 @@ int latent_op(const mi_layer_spec& p, const float* uk, const float* uv, const vo
   }
   unsigned char *w_uk, *w_uv, *qa, *lat;
   uint16_t* ukv;
-  float *tmp, *ones;
-  MI_TRY(mem.take(&w_uk, (size_t)H * g.rp * g.dkp * el, s));
+  float *tmp, *ones, *unit;
+  MI_TRY(mem.take(&w_uk, (size_t)H * g.cp * g.dkp * el, s));
   MI_TRY(mem.take(&w_uv, (size_t)H * g.dvp * g.rp * el, s));
   MI_TRY(mem.take(&ukv, (size_t)nkv * Kc * 2, s));
-  MI_TRY(mem.take(&tmp, (size_t)g.dk * g.rank * 4, s));
+  MI_TRY(mem.take(&tmp, (size_t)dq * g.rank * 4, s));
   MI_TRY(mem.take(&ones, (size_t)nkv * 4, s));
-  MI_TRY(mem.take(&qa, (size_t)T * H * g.rp * el, s));
-  MI_TRY(mem.take(&lat, (size_t)T * H * g.rp * el, s));
+  MI_TRY(mem.take(&qa, (size_t)T * H * g.cp * el, s));
+  MI_TRY(mem.take(&lat, (size_t)T * H * g.cp * el, s));
   MI_TRY(launch_fill_f32(ones, nkv, 1.f, s));
+  std::vector<float> u((size_t)std::max(g.nr, 1) * dq, 0.f);
+  for (int i = 0; i < g.nr; ++i) u[(size_t)i * dq + g.dk + i] = 1.f;
+  MI_TRY(mem.take(&unit, u.size() * 4, s));
+  MI_HIP(hipMemcpyAsync(unit, u.data(), u.size() * 4, hipMemcpyHostToDevice, s));
+  MI_HIP(hipStreamSynchronize(s));
   for (int h = 0; h < H; ++h) {
     const float *k = uk + (size_t)h * g.dk * g.rank, *v = uv + (size_t)h * g.dv * g.rank;
-    MI_TRY(launch_transpose(k, g.dk, g.rank, tmp, g.dk, s));
-    MI_TRY(launch_place(tmp, g.dk, 0, g.rank, g.dk, w_uk + (size_t)h * g.rp * g.dkp * el, g.dkp, f32, 0, 0, s));
+    MI_TRY(launch_transpose(k, g.dk, g.rank, tmp, dq, s));
+    MI_TRY(launch_place(tmp, dq, 0, g.rank, dq, w_uk + (size_t)h * g.cp * g.dkp * el, g.dkp, f32, 0, 0, s));
+    if (g.nr) {
+      MI_TRY(launch_place(unit, dq, 0, g.nr, dq, w_uk + (size_t)h * g.cp * g.dkp * el, g.dkp, f32, g.rp, 0, s));
+      MI_TRY(launch_place(unit, dq, g.dk, g.nr, g.nr, ukv, Kc, false, h * g.dkp + g.dk, g.rp, s));
+    }
     MI_TRY(launch_place(v, g.rank, 0, g.dv, g.rank, w_uv + (size_t)h * g.dvp * g.rp * el, g.rp, f32, 0, 0, s));
     MI_TRY(launch_place(k, g.rank, 0, g.dk, g.rank, ukv, Kc, false, h * g.dkp, 0, s));
     MI_TRY(launch_place(v, g.rank, 0, g.dv, g.rank, ukv, Kc, false, H * g.dkp + h * g.dvp, 0, s));
   }
   if (f32 || path == 1) {
-    const AttnSpec a{HeadGeom{H, 1, g.rp, g.rp, g.rp, g.rp}, p.scale, p.window, nullptr, 0, 0};
-    MI_TRY(launch_head_linear(w_uk, H, g.rp, g.dkp, q, T, qa, H * g.rp, g.rp, g.rp, f32, s));
+    const AttnSpec a{HeadGeom{H, 1, g.cp, g.rp, g.cp, g.cp}, p.scale, p.window, nullptr, 0, 0};
+    MI_TRY(launch_head_linear(w_uk, H, g.cp, g.dkp, q, T, qa, H * g.cp, g.cp, g.cp, f32, s));
     MI_TRY(launch_attn_plain(a, qa, pool, pool, bs, bt, MB, pos, sd, nseg, T, lat, H * g.rp, f32, s));
     MI_TRY(launch_head_linear(w_uv, H, g.dvp, g.rp, lat, T, out, ldo, g.dv, g.dv, f32, s));
   } else if (path == 2) {
@@ -91,7 +100,7 @@ int latent_op(const mi_layer_spec& p, const float* uk, const float* uv, const vo
     void* scratch = nullptr;
     MI_TRY(mem.take(&scratch, latent_attn_scratch_bytes(g), s));
     const LatentRows lr{sd, nseg, 1 << 30, T};
-    MI_TRY(launch_head_linear_rows(w_uk, H, g.rp, g.dkp, (const uint16_t*)q, lr, (uint16_t*)qa, H * g.rp, g.rp, g.rp, s));
+    MI_TRY(launch_head_linear_rows(w_uk, H, g.cp, g.dkp, (const uint16_t*)q, lr, (uint16_t*)qa, H * g.cp, g.cp, g.cp, s));
     MI_TRY(launch_latent_attn_rows(g, p.scale, p.window, (const uint16_t*)qa, (const uint16_t*)pool, bs, bt, MB, pos, lr, max_ctx, w_uv, (uint16_t*)lat,
                                    (uint16_t*)out, ldo, scratch, s));
   } else {
@@ -154,12 +163,56 @@ int mi_op_sandwich_rows(const float* resid_in, float* resid_out, const float* y,
   return MI_OK;
 }
 
-int mi_op_latent_scatter(const float* qd, int32_t ldq, int32_t T, const mi_layer_spec* spec, const float* c_norm, float eps, const int32_t* slots,
-                         int32_t block_size, void* q, void* pool, int32_t f32, void* stream) {
+int mi_op_latent_scatter(const float* qd, int32_t ldq, int32_t T, const mi_layer_spec* spec, const float* rot, const int32_t* pos, const float* c_norm,
+                         float eps, const int32_t* slots, int32_t block_size, void* q, void* pool, int32_t f32, void* stream) {
   MI_CHECK(qd && spec && slots && q && pool, "null argument");
   const mi_layer_spec& p = *spec;
-  const LatentGeom g{p.num_heads, p.qk_dim, p.v_dim, p.kv_rank, pad_to(p.qk_dim, 32), pad_to(p.v_dim, 32), pad_to(p.kv_rank, 32)};
-  return launch_latent_scatter(qd, ldq, T, g, c_norm, eps, slots, block_size, q, pool, f32 != 0, (hipStream_t)stream);
+  const LatentGeom g = latent_geom(p.num_heads, p.qk_dim, p.v_dim, p.kv_rank, p.rot_dim, p.rot_dims);
+  MI_CHECK(!c_norm || ldq >= g.H * g.dq() + g.rank + g.nr, "latent scatter: columns");
+  const LatentRowsIn in{qd, qd + g.H * g.dq(), ldq, ldq};
+  return launch_latent_scatter(in, T, g, Rotation{(const float2*)rot, pos}, c_norm, eps, slots, block_size, q, pool, f32 != 0, (hipStream_t)stream);
+}
+
+int mi_op_delta_rule(const mi_layer_spec* spec, const float* proj, int32_t ldp, int32_t beta, const float* z, int32_t ldz, int32_t gate, const float* conv,
+                     const float* a_log, const float* dt, const float* norm, float eps, float* state, float* ring, int32_t num_slots, const int32_t* slots_host,
+                     const int32_t* pos_host, const int32_t* segs_host, int32_t nseg, int32_t T, int32_t max_chunks, void* out, int32_t ldo, int32_t f32,
+                     void* stream) {
+  MI_CHECK(spec && proj && z && conv && a_log && dt && norm && state && ring && slots_host && pos_host && out && T >= 1 && nseg >= 0, "null argument");
+  MI_CHECK(max_chunks >= 1 && (nseg == 0 || segs_host), "delta rule: segments");
+  const mi_layer_spec& p = *spec;
+  hipStream_t s = (hipStream_t)stream;
+  Arena mem;
+  const DeltaGeom g{p.num_heads, p.num_kv_heads, p.qk_dim, p.v_dim, pad_to(p.qk_dim, 16), pad_to(p.v_dim, 16), p.conv_taps};
+  MI_CHECK(delta_supported(g), "delta rule: sizes");
+  const int seqs = nseg ? nseg : T;
+  for (int i = 0; i < seqs; ++i) MI_CHECK(slots_host[i] >= 0 && slots_host[i] < num_slots, "delta rule: slot out of range");
+  for (int i = 0; i < T; ++i) MI_CHECK(pos_host[i] >= 0, "delta rule: position");
+  std::vector<AttnSeg> segs;
+  AttnSeg* sd = nullptr;
+  if (nseg) {
+    MI_TRY(take_segs(mem, segs_host, nseg, T, 16, 1 << 20, segs, &sd, s));
+    for (const AttnSeg& x : segs) MI_CHECK(x.seq < seqs, "segments: sequence");
+  }
+  int32_t *slots, *pos;
+  float *factors, *o;
+  MI_TRY(mem.take(&slots, (size_t)seqs * 4, s));
+  MI_TRY(mem.take(&pos, (size_t)T * 4, s));
+  MI_TRY(mem.take(&factors, (size_t)max_chunks * delta_factor_floats(g) * 4, s));
+  MI_TRY(mem.take(&o, (size_t)T * g.H * g.dvp * 4, s));
+  MI_HIP(hipMemcpyAsync(slots, slots_host, (size_t)seqs * 4, hipMemcpyHostToDevice, s));
+  MI_HIP(hipMemcpyAsync(pos, pos_host, (size_t)T * 4, hipMemcpyHostToDevice, s));
+  DeltaIn in;
+  in.proj = proj; in.ldp = ldp; in.beta = beta; in.z = z; in.ldz = ldz; in.gate = gate;
+  in.conv = conv; in.a_log = a_log; in.dt = dt; in.norm = norm; in.eps = eps;
+  in.state = state; in.ring = ring; in.slots = slots; in.pos = pos;
+  if (!nseg) {
+    MI_TRY(launch_delta_token(g, in, T, nullptr, out, ldo, f32 != 0, s));
+  } else {
+    MI_TRY(launch_delta_token(g, in, nseg, sd, out, ldo, f32 != 0, s));
+    MI_TRY(launch_delta_prompt(g, in, sd, segs.data(), nseg, factors, max_chunks, o, out, ldo, f32 != 0, s));
+  }
+  MI_HIP(hipStreamSynchronize(s));
+  return MI_OK;
 }
 
 int mi_op_latent_attn(const mi_layer_spec* spec, const float* uk, const float* uv, const void* q, const void* pool, int32_t block_size,
@@ -171,15 +224,16 @@ int mi_op_latent_attn(const mi_layer_spec* spec, const float* uk, const float* u
 }
 
 int mi_op_experts(const void* x, int32_t ldx, int32_t T, int32_t D, int32_t experts, int32_t top, int32_t ff, const float* router, const float* router_b,
-                  const float* gate, const float* up, const float* down, int32_t* ids, float* weights, float* y, int32_t ldy, int32_t f32, int32_t path,
-                  void* stream) {
-  MI_CHECK(x && router && router_b && gate && up && down && ids && weights && y && T >= 1, "null argument");
+                  const float* gate, const float* up, const float* down, int32_t* ids, float* weights, float* y, int32_t ldy, int32_t groups, int32_t keep,
+                  int32_t f32, int32_t path, void* stream) {
+  const bool relu2 = groups > 0;
+  MI_CHECK(x && router && router_b && (gate || relu2) && up && down && ids && weights && y && T >= 1, "null argument");
   MI_CHECK(path == 1 || path == 2, "path: 1 weight streaming (or fp32), 2 grouped");
   MI_CHECK(path == 1 || !f32, "experts: the grouped form is built for bf16");
   hipStream_t s = (hipStream_t)stream;
   Arena mem;
   const size_t el = f32 ? 4 : 2;
-  const int Kd = pad_to(D, 64), N1 = pad_to(2 * ff, 16), K2 = pad_to(ff, 64), N2 = pad_to(D, 16), E16 = pad_to(experts, 16), pairs = T * top;
+  const int Kd = pad_to(D, 64), N1 = pad_to((relu2 ? 1 : 2) * ff, 16), K2 = pad_to(ff, 64), N2 = pad_to(D, 16), E16 = pad_to(experts, 16), pairs = T * top;
   MI_CHECK(ldx >= Kd && ldy >= N2, "experts: strides");
   unsigned char *gu, *dn, *act, *rw;
   uint16_t *y16, *rt;
@@ -201,25 +255,29 @@ int mi_op_experts(const void* x, int32_t ldx, int32_t T, int32_t D, int32_t expe
   MI_TRY(launch_fill_f32(ones, E16, 1.f, s));
   MI_TRY(launch_place_rows(router, experts, D, rw, Kd, f32 != 0, s));
   for (int e = 0; e < experts; ++e) {
-    MI_TRY(launch_place(gate + (size_t)e * ff * D, D, 0, ff, D, gu + (size_t)e * N1 * Kd * el, Kd, f32 != 0, 0, 0, s, 2));
-    MI_TRY(launch_place(up + (size_t)e * ff * D, D, 0, ff, D, gu + (size_t)e * N1 * Kd * el, Kd, f32 != 0, 1, 0, s, 2));
+    if (!relu2) MI_TRY(launch_place(gate + (size_t)e * ff * D, D, 0, ff, D, gu + (size_t)e * N1 * Kd * el, Kd, f32 != 0, 0, 0, s, 2));
+    MI_TRY(launch_place(up + (size_t)e * ff * D, D, 0, ff, D, gu + (size_t)e * N1 * Kd * el, Kd, f32 != 0, relu2 ? 0 : 1, 0, s, relu2 ? 1 : 2));
     MI_TRY(launch_place(down + (size_t)e * D * ff, ff, 0, D, ff, dn + (size_t)e * N2 * K2 * el, K2, f32 != 0, 0, 0, s));
   }
+  RouterRule rule;
+  rule.b = bias;
+  if (relu2) { rule.sigmoid = true; rule.groups = groups; rule.keep = keep; }
+  const int a1 = relu2 ? EXPERT_RELU2 : EXPERT_SILU_GLU;
   const ExpertsLinear l1{gu, experts, N1, Kd}, l2{dn, experts, N2, K2};
   if (path == 1) {
-    MI_TRY(launch_route(x, ldx, T, rw, bias, experts, Kd, top, ids, weights, f32 != 0, s, f32 ? nullptr : z, f32 ? nullptr : tickets));
-    MI_TRY(launch_experts_linear(l1, ids, pairs, x, ldx, top, true, act, K2, f32 != 0, s));
-    MI_TRY(launch_experts_linear(l2, ids, pairs, act, K2, 1, false, y, ldy, f32 != 0, s));
+    MI_TRY(launch_route(x, ldx, T, rw, rule, experts, Kd, top, ids, weights, f32 != 0, s, f32 ? nullptr : z, f32 ? nullptr : tickets));
+    MI_TRY(launch_experts_linear(l1, ids, pairs, x, ldx, top, a1, act, K2, f32 != 0, s));
+    MI_TRY(launch_experts_linear(l2, ids, pairs, act, K2, 1, EXPERT_LINEAR, y, ldy, f32 != 0, s));
   } else {
     MI_TRY(launch_place(router, D, 0, experts, D, rt, Kd, false, 0, 0, s));
     EpiArgs e{};
-    e.scale = ones; e.bias = bias; e.out_f32 = z; e.ld_out = E16;
+    e.scale = ones; e.bias = relu2 ? nullptr : bias; e.out_f32 = z; e.ld_out = E16;
     MI_TRY(launch_gemm(LinearW{rt, E16, Kd, MI_W_BF16}, T, (const uint16_t*)x, ldx, EPI_F32, e, s));
-    MI_TRY(launch_route_pick(z, E16, T, experts, top, ids, weights, s));
+    MI_TRY(launch_route_pick(z, E16, T, rule, experts, top, ids, weights, s));
     const ExpertPlan plan = experts_plan(plan_mem, pairs, experts);
     MI_TRY(launch_experts_sort(plan, ids, pairs, experts, s));
-    MI_TRY(launch_experts_gemm(l1, plan, pairs, (const uint16_t*)x, ldx, top, true, (uint16_t*)act, K2, s));
-    MI_TRY(launch_experts_gemm(l2, plan, pairs, (const uint16_t*)act, K2, 1, false, y16, ldy, s));
+    MI_TRY(launch_experts_gemm(l1, plan, pairs, (const uint16_t*)x, ldx, top, a1, (uint16_t*)act, K2, s));
+    MI_TRY(launch_experts_gemm(l2, plan, pairs, (const uint16_t*)act, K2, 1, EXPERT_LINEAR, y16, ldy, s));
     MI_TRY(launch_bf16_to_f32(y16, y, (size_t)pairs * ldy, s));
   }
   MI_HIP(hipStreamSynchronize(s));

@@ -93,7 +93,7 @@ class BokulornConfig:
         entries = raw["layers"]
         _require(entries, "no layers")
         layers = [_layer(i, e) for i, e in enumerate(entries)]
-        sizes_from = {}
+        owner, sizes_from = [], {}
         for i, entry in enumerate(entries):
             j, seen = i, {i}
             while entries[j].get("weights_of") is not None:      # the layer that has the tensors
@@ -102,10 +102,12 @@ class BokulornConfig:
                 seen.add(j)
             if j != i:
                 _require(layers[i] == layers[j], f"layer {i}: weights_of names a layer with other sizes")
-            layers[i]["weights_of"] = j if j != i else -1
+            owner.append(j)
             if layers[i]["mixer_kind"] == MI_MIX["delta"]:
                 sizes_from[(i, "decay_rank")] = f"l{j}.mix.a1"
                 sizes_from[(i, "gate_rank")] = f"l{j}.mix.g1"
+        for i, j in enumerate(owner):
+            layers[i]["weights_of"] = j if j != i else -1
         width = int(raw["width"])
         stack = dict(layers=layers, width=width, vocab_size=int(raw["vocab"]), max_positions=0, norm_eps=float(raw["norm"]["eps"]),
                      residual_mult=1.0, block_kind=MI_BLOCK["one_norm"], norm_groups=1, norm_offset=1.0,

@@ -16,7 +16,7 @@ from __future__ import annotations
 
 import torch
 
-__all__ = ["rms", "rotate", "latent_kv", "latent_attention", "short_conv", "unit", "decays", "delta_rule", "delta_mixer", "pick",
+__all__ = ["rms", "rotate", "latent_kv", "latent_attention", "short_conv", "unit", "decays", "delta_rule", "delta_heads", "delta_mixer", "pick",
            "expert_ff", "resolve", "residuals_and_logits", "logits"]
 
 
@@ -65,7 +65,7 @@ def latent_attention(q, c, k_rot, w_uk, w_uv, scale, r=lambda t: t):
     return out
 
 
-def latent_mixer(h, m, w, p, eps, r=lambda t: t):
+def latent_mixer(h, m, w, p, eps, per_head, r=lambda t: t):
     """`m` = the layer's mixer entry; w[p + name] its tensors.  The gate has one row per head, or one per element of the heads."""
     T, H, rot = h.shape[0], m["heads"], m.get("rot")
     nr = m.get("rot_dim", 0)
@@ -76,7 +76,7 @@ def latent_mixer(h, m, w, p, eps, r=lambda t: t):
     c, k_rot = latent_kv(h, w[p + "dkv"], w[p + "dkv.norm"], m["kv_rank"], eps, rot if nr else None, r)
     o = latent_attention(q, c, k_rot, w[p + "uk"], w[p + "uv"], m["scale"], r)
     g = torch.sigmoid(h @ w[p + "g"].t())
-    o = o * (g.view(T, H, 1) if g.shape[1] == H and nr else g.view(T, H, m["vdim"]))
+    o = o * g.view(T, H, 1 if per_head else m["vdim"])
     return r(o.reshape(T, -1)) @ w[p + "o"].t()
 
 
@@ -117,16 +117,25 @@ def delta_rule(q, k, v, log_g, beta, state=None):
     return out, S
 
 
-def delta_mixer(h, m, w, p, eps, r=lambda t: t):
-    T, H, G, d, dv = h.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
-    x = {n: short_conv(r(h @ w[p + n].t()), w[p + n + ".conv"]) for n in ("q", "k", "v")}
+def delta_heads(q, k, v, b, z, gate, conv, a_log, dt_bias, w_norm, eps):
+    """From the projections of a whole sequence to the heads' outputs: q, k [T, G d], v [T, H dv], b [T, H], z [T, H d], gate [T, H dv],
+    conv = the three convolutions' weights -> [T, H dv], and the state behind the last token."""
+    T, H = b.shape
+    d, dv = z.shape[1] // H, v.shape[1] // H
+    G = q.shape[1] // d
     of = torch.arange(H) // (H // G)
-    q, k = unit(x["q"].view(T, G, d))[:, of] * d ** -0.5, unit(x["k"].view(T, G, d))[:, of]
-    beta = torch.sigmoid(h @ w[p + "b"].t())
-    z = (r(h @ w[p + "a1"].t()) @ w[p + "a2"].t()).view(T, H, d)
-    o, _ = delta_rule(q, k, x["v"].view(T, H, dv), decays(z, w[p + "A_log"], w[p + "dt_bias"]), beta)
-    gate = torch.sigmoid(r(h @ w[p + "g1"].t()) @ w[p + "g2"].t()).view(T, H, dv)
-    return r((rms(o, eps) * w[p + "norm"] * gate).reshape(T, -1)) @ w[p + "o"].t()
+    q, k, v = (short_conv(x, w) for x, w in zip((q, k, v), conv))
+    q, k = unit(q.view(T, G, d))[:, of] * d ** -0.5, unit(k.view(T, G, d))[:, of]
+    o, S = delta_rule(q, k, v.view(T, H, dv), decays(z.view(T, H, d), a_log, dt_bias), torch.sigmoid(b))
+    return (rms(o, eps) * w_norm * torch.sigmoid(gate).view(T, H, dv)).reshape(T, H * dv), S
+
+
+def delta_mixer(h, m, w, p, eps, r=lambda t: t):
+    z = r(h @ w[p + "a1"].t()) @ w[p + "a2"].t()
+    gate = r(h @ w[p + "g1"].t()) @ w[p + "g2"].t()
+    y, _ = delta_heads(*(h @ w[p + n].t() for n in "qkvb"), z, gate, [w[p + n + ".conv"] for n in "qkv"], w[p + "A_log"], w[p + "dt_bias"],
+                       w[p + "norm"], eps)
+    return r(y) @ w[p + "o"].t()
 
 
 def pick(z, correction, top, groups, keep):
@@ -179,8 +188,10 @@ def residuals_and_logits(cfg, weights, tokens, dtype=torch.float32, rounding=Non
         j = resolve(cfg["layers"], i)
         spec, p = cfg["layers"][j], f"l{j}."
         h = norm(x, p + "norm1")
-        mixer = delta_mixer if spec["type"] == "channel_delta" else latent_mixer
-        y = mixer(h, spec["mixer"], w, p + "mix.", eps, r)
+        if spec["type"] == "channel_delta":
+            y = delta_mixer(h, spec["mixer"], w, p + "mix.", eps, r)
+        else:
+            y = latent_mixer(h, spec["mixer"], w, p + "mix.", eps, spec["type"] == "latent_attention", r)
         if spec.get("mlp") is not None:
             y = y + expert_ff(h, spec["mlp"], w, p + "mlp.", r)
         x = x + y

@@ -308,10 +308,13 @@ class StackBench:
         return self.ready(NativeModel(weight_dtype=0, quant_type=0, quantize_lm_head=0, tp_degree=1, tp_rank=0,
                                       prefill_fp8_activations=0, **self.common(), **_decoder_geometry(SimpleNamespace(**hf))))
 
-    def stack(self, config):
+    def stack(self, config, ranks=None):
+        """ranks: sizes that a checkpoint's tensors would give"""
         from vllm_neuron_amd._native import NativeModel
-        from vllm_neuron_amd.models import config_from_dict
-        return self.ready(NativeModel(stack=dict(config_from_dict(config).stack, compute_dtype=1), **self.common()))
+        from vllm_neuron_amd.models import config_from_dict, fill_sizes
+        c = config_from_dict(config)
+        fill_sizes(c, lambda name: (ranks, config["width"]))
+        return self.ready(NativeModel(stack=dict(c.stack, compute_dtype=1), **self.common()))
 
     @staticmethod
     def keys_seen(n, window):          # keys of the first n queries of a sequence
@@ -368,20 +371,21 @@ class StackBench:
 
     @staticmethod
     def compare(size, window):
-        """tokens/s and `distance` (how much further from its roofline a class is) against the Llama of the size"""
+        """tokens/s and `distance` (how much further from its roofline a class is) against the first model of the size"""
+        first = size["prefill"][0]["model"]
         for table, fr in (("prefill", "roofline_fraction"), ("decode", "hbm_fraction")):
-            base = {(r.get("tokens"), r.get("batch"), r.get("context")): r for r in size[table] if r["model"] == "llama"}
+            base = {(r.get("tokens"), r.get("batch"), r.get("context")): r for r in size[table] if r["model"] == first}
             for r in size[table]:
-                if r["model"] == "llama":
+                if r["model"] == first:
                     continue
                 b = base[r.get("tokens"), r.get("batch"), r.get("context")]
-                r["vs_llama_tokens_per_s"] = round(r["tokens_per_s"] / b["tokens_per_s"], 3)
+                r[f"vs_{first}_tokens_per_s"] = round(r["tokens_per_s"] / b["tokens_per_s"], 3)
                 if "window" in r["model"] and r.get("context", 0) > window:     # the Llama step that reads as many keys
                     b = base[None, r["batch"], window]
                 r["distance"] = {k: round(b[fr][k] / v, 2) for k, v in r[fr].items() if k in b[fr] and v > 0}
 
-    def line(self, design, sizes):
-        print(json.dumps({"metric": f"{design} prefill / decode beside a Llama of equal size", "dtype": "bf16", "data": "synthetic",
+    def line(self, design, sizes, beside="Llama"):
+        print(json.dumps({"metric": f"{design} prefill / decode beside a {beside} of equal size", "dtype": "bf16", "data": "synthetic",
                           "higher_is_better": True, "steps": self.args.steps, "warmup": self.args.warmup, "n_gpus": 1, "sizes": sizes}),
               flush=True)
 
@@ -462,6 +466,69 @@ def rapodra_section(args):
     bench.line("Rapodra", out)
 
 
+# ---- --bokulorn: every mixer of the design beside Rapodra's latent attention, all with experts of equal bytes ----------------------
+# (label, width, heads of 128, latent rank, query rank, expert size of Rapodra's gated experts, layers); 64 experts, 8 per token.  A
+# squared-relu expert has two matrices where a gated one has three: 1.5 x the expert size.
+BOKULORN_SIZES = [("2b-like", 2048, 16, 512, 1024, 768, 8), ("8b-like", 4096, 32, 512, 1536, 1536, 4)]
+BOKULORN_ROT, BOKULORN_LOW = 64, 128
+MFMA_F32_PEAK_TFLOPS = 157.3
+
+
+def bokulorn_section(args):
+    bench, out = StackBench(args), []
+    every, E, top, dim, rot, low = bench.MAX_LEN, RAPODRA_EXPERTS, RAPODRA_TOP, RAPODRA_DIM, BOKULORN_ROT, BOKULORN_LOW
+    for label, width, H, rank, q_rank, eff, layers in BOKULORN_SIZES:
+        size = {"size": label, "layers": layers, "width": width, "heads": [H, dim, rank], "query rank": q_rank, "experts": [E, top, eff],
+                "prefill": [], "decode": []}
+        moe = {"kind": "moe", "router": {"experts": E, "top": top, "groups": {"count": 8, "keep": 4}}, "expert": {"ff": eff * 3 // 2}}
+        hit = lambda B: E * (1 - (1 - top / E) ** B)                   # noqa: E731  (expected number of different experts)
+        for kind in ("rapodra", "latent_attention", "latent_attention_2", "channel_delta"):
+            if args.kinds and kind not in args.kinds.split(","):
+                continue
+            print(f"[bench] {label} {kind}", file=sys.stderr, flush=True)
+            kv = 2 * rank * H * dim
+            if kind == "rapodra":
+                layer = {"type": "latent_attention", "mixer": {"heads": H, "dim": dim, "vdim": dim, "kv_rank": rank, "mask": {"size": every},
+                                                               "scale": dim ** -0.5},
+                         "mlp": {"kind": "moe", "router": {"experts": E, "top": top}, "expert": {"ff": eff}}}
+                m = bench.stack({"architecture": "Rapodra", "width": width, "vocab": STACK_VOCAB, "layers": [layer] * layers, "canon": {"taps": 4},
+                                 "norm": {"eps": 1e-5, "groups": 1}, "logit_softcap": 30.0})
+                proj, row, flops = width * (H * dim + rank) + H * dim * width + kv, rank, 4.0 * H * dim
+            else:
+                mix = {"heads": H, "dim": dim, "vdim": dim}
+                if kind == "channel_delta":
+                    mix.update(kv_heads=H, conv=4)
+                    proj, kv = width * (3 * H * dim + H + 2 * low) + 2 * low * H * dim + H * dim * width, 0
+                else:
+                    mix.update(kv_rank=rank, q_rank=q_rank, scale=dim ** -0.5)
+                    r = rot if kind == "latent_attention" else 0
+                    if r:
+                        mix.update(rot_dim=r, rot={"base": 1e4, "dims": r})
+                    proj = width * (q_rank + rank + r + (H if r else H * dim)) + q_rank * H * (dim + r) + H * dim * width + kv
+                    row, flops = rank + r, 2.0 * H * (2 * dim + r)
+                m = bench.stack({"architecture": "Bokulorn", "width": width, "vocab": STACK_VOCAB, "layers": [{"type": kind, "mixer": mix, "mlp": moe}] * layers,
+                                 "norm": {"eps": 1e-5}, "embedding": {"scale": 1.0}}, ranks=low)
+            weights, expert = proj + E * width, 3 * width * eff
+
+            def work(T):
+                gemm = (2.0 * T * layers * (weights + top * expert), 2.0 * layers * (weights + hit(T) * expert))
+                if kind == "channel_delta":      # three products of the state per token, on the fp32 matrix cores
+                    return {"gemm": gemm, "attn_prefill": (6.0 * layers * T * H * dim * dim * MFMA_BF16_PEAK_TFLOPS / MFMA_F32_PEAK_TFLOPS, 0.0)}
+                return {"gemm": gemm, "attn_prefill": (layers * flops * bench.keys_seen(T, every), 0.0)}
+
+            def mixer_bytes(B, ctx):
+                if kind == "channel_delta":      # the state, read and written
+                    return 8.0 * layers * B * H * dim * dim
+                return 2.0 * layers * (B * ctx * row + rank * H * dim)
+            size["prefill"] += bench.prefill(m, kind, work)
+            size["decode"] += bench.decode(m, kind, mixer_bytes, lambda B: 2.0 * layers * hit(B) * expert)
+            m.close()
+        if not args.kinds:
+            bench.compare(size, every)
+        out.append(size)
+    bench.line("Bokulorn", out, "Rapodra")
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -481,7 +548,13 @@ def main():
     ap.add_argument("--rapodra", action="store_true",
                     help="instead of the headline workload: Rapodra (latent attention; dense and expert feed-forwards) beside a Llama "
                          "of equal size, all bf16")
+    ap.add_argument("--bokulorn", action="store_true",
+                    help="instead of the headline workload: Bokulorn's mixers (latent attention, delta rule), each with experts, beside "
+                         "Rapodra of equal size, all bf16")
+    ap.add_argument("--kinds", default="", help="--bokulorn: only these models (comma-separated; no comparison)")
     args = ap.parse_args()
+    if args.bokulorn:
+        return bokulorn_section(args)
     if args.vimesun:
         return vimesun_section(args)
     if args.rapodra:

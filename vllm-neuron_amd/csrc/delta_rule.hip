@@ -9,9 +9,13 @@ namespace {
 
 constexpr int kC = kDeltaChunk;
 
-__device__ __forceinline__ float silu(float v) { return v / (1.f + expf(-v)); }
+__device__ __forceinline__ float silu(float v) { return v * __builtin_amdgcn_rcpf(1.f + __expf(-v)); }
 __device__ __forceinline__ float sigmoid(float v) { return 1.f / (1.f + expf(-v)); }
-__device__ __forceinline__ float softplus(float v) { return fmaxf(v, 0.f) + log1pf(expf(-fabsf(v))); }
+// max(v, 0) + log(1 + w), w = exp(-|v|): the series where w is small (its first left-out term is w^5 / 5)
+__device__ __forceinline__ float softplus(float v) {
+  const float w = __expf(-fabsf(v)), series = w * (1.f - w * (0.5f - w * (1.f / 3.f - 0.25f * w)));
+  return fmaxf(v, 0.f) + (w < 0.02f ? series : __logf(1.f + w));
+}
 __device__ __forceinline__ float log_decay(float z, float dt, float a_log) { return -expf(a_log) * softplus(z + dt); }
 __device__ __forceinline__ void put1(uint16_t* p, float v) { *p = f32_to_bf16(v); }
 __device__ __forceinline__ void put1(float* p, float v) { *p = v; }
@@ -148,18 +152,31 @@ __device__ __forceinline__ Factors factors_at(float* base, size_t index, int dkp
   return Factors{p, p + 16 * dkp, p + 32 * dkp, p + 48 * dkp, p + 49 * dkp, p + 49 * dkp + 256};
 }
 
-// the input of a convolution `i` rows behind the segment's start (negative: ahead of it)
-__device__ __forceinline__ float conv_in(const DeltaIn& in, const AttnSeg& sg, const float* ring, int taps, int C, int ch, int i) {
-  if (i >= 0) return in.proj[(size_t)(sg.row0 + i) * in.ldp + ch];
-  const int p = sg.pos0 + i;
-  return p >= 0 ? ring[(size_t)(p % taps) * C + ch] : 0.f;
+// where the input of a convolution `i` rows behind the segment's start lies (negative: ahead of it; ahead of the sequence: anywhere
+// valid, conv_known is false).  Addresses are selected, not branched over: loads stay in flight together.
+__device__ __forceinline__ const float* conv_at(const DeltaIn& in, const AttnSeg& sg, const float* ring, int taps, int C, int ch, int i) {
+  const int p = max(sg.pos0 + i, 0) % taps;
+  const float *a = in.proj + (size_t)(sg.row0 + max(i, 0)) * in.ldp + ch, *b = ring + (size_t)p * C + ch;
+  return i >= 0 ? a : b;
 }
+__device__ __forceinline__ bool conv_known(const AttnSeg& sg, int i) { return sg.pos0 + i >= 0; }
+__device__ __forceinline__ float conv_in(const DeltaIn& in, const AttnSeg& sg, const float* ring, int taps, int C, int ch, int i) {
+  const float v = *conv_at(in, sg, ring, taps, C, ch, i);
+  return conv_known(sg, i) ? v : 0.f;
+}
+
+// LDS written by some lanes of a wave, read by others of it
+__device__ __forceinline__ void wave_order() {
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+}
+constexpr int kPairTiles = 36, kPairParts = 7;
 
 template <int TAPS>
 __global__ __launch_bounds__(256) void delta_factors_kernel(DeltaGeom g, DeltaIn in, const AttnSeg* __restrict__ segs, int nseg, int c0, float* __restrict__ out) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
   const int pitch = g.dkp + 4;
-  float *qs = sm, *ks = qs + kC * pitch, *Ls = ks + kC * pitch, *gs = Ls + kC * pitch, *red = gs + kC * pitch;   // red [4][64][8]
+  float *qs = sm, *ks = qs + kC * pitch, *Ls = ks + kC * pitch, *gs = Ls + kC * pitch, *red = gs;   // (red: in place of gs once that is used up)
   __shared__ float As[kC][kC + 1], Ps[kC][kC + 1], Ts[kC][kC + 1], Ms[kC][kC + 1], bs[kC], rn[2 * kC];
   const ChunkAt at = chunk_at(segs, nseg, c0 + blockIdx.x);
   if (!at.ok) return;
@@ -202,19 +219,11 @@ __global__ __launch_bounds__(256) void delta_factors_kernel(DeltaGeom g, DeltaIn
   }
   {
     const float a_log = in.a_log[h];
-    for (int d = tid; d < g.dkp; d += 256) {
-      float zt[kC];
-#pragma unroll
-      for (int t = 0; t < kC; ++t) zt[t] = d < g.dk ? in.z[(size_t)(at.sg.row0 + at.t0 + min(t, n - 1)) * in.ldz + h * g.dk + d] : 0.f;
-      const float dt = d < g.dk ? in.dt[h * g.dk + d] : 0.f;
-      float L = 0.f;
-#pragma unroll
-      for (int t = 0; t < kC; ++t) {
-        const float lg = d < g.dk && t < n ? log_decay(zt[t], dt, a_log) : 0.f;
-        L += lg;
-        Ls[t * pitch + d] = L;
-        gs[t * pitch + d] = expf(lg);
-      }
+    const float* zr = in.z + (size_t)(at.sg.row0 + at.t0) * in.ldz + h * g.dk;
+    for (int i = tid; i < kC * g.dkp; i += 256) {
+      const int t = i / g.dkp, d = i - t * g.dkp, dc = min(d, g.dk - 1);
+      const float lg = log_decay(zr[(size_t)min(t, n - 1) * in.ldz + dc], in.dt[h * g.dk + dc], a_log);
+      Ls[t * pitch + d] = d < g.dk && t < n ? lg : 0.f;
     }
   }
   if (tid < kC) bs[tid] = tid < n ? sigmoid(rows[(size_t)tid * in.ldp + in.beta + h]) : 0.f;
@@ -228,6 +237,17 @@ __global__ __launch_bounds__(256) void delta_factors_kernel(DeltaGeom g, DeltaIn
     s = wave_sum(s);
     if (lane == 0) rn[v] = 1.f / sqrtf(s + 1e-6f) * (v < kC ? 1.f / sqrtf((float)g.dk) : 1.f);
   }
+  for (int d = tid; d < g.dkp; d += 256) {           // running sums of the decays' logarithms, the decays beside them
+    float L = 0.f, lg[kC];
+#pragma unroll
+    for (int t = 0; t < kC; ++t) lg[t] = Ls[t * pitch + d];
+#pragma unroll
+    for (int t = 0; t < kC; ++t) {
+      L += lg[t];
+      Ls[t * pitch + d] = L;
+      gs[t * pitch + d] = __expf(lg[t]);
+    }
+  }
   __syncthreads();
   for (int i = tid; i < 2 * kC * (g.dkp / 4); i += 256) {
     const int v = i / (g.dkp / 4), d = (i % (g.dkp / 4)) * 4;
@@ -237,75 +257,100 @@ __global__ __launch_bounds__(256) void delta_factors_kernel(DeltaGeom g, DeltaIn
     *r = make_float4(x.x * f, x.y * f, x.z * f, x.w * f);
   }
   __syncthreads();
-  {   // pairs: lane (I, J) takes tokens 2 I, 2 I + 1 against 2 J, 2 J + 1, a wave a quarter of the channels
-    const int I = lane >> 3, J = lane & 7, i0 = 2 * I, j0 = 2 * J;
-    float a[4] = {0.f, 0.f, 0.f, 0.f}, p[4] = {0.f, 0.f, 0.f, 0.f};        // (i0,j0) (i0,j1) (i1,j0) (i1,j1)
-    if (J <= I) {
-      const bool diag = I == J;
-      for (int d = wave * (g.dkp / 4); d < (wave + 1) * (g.dkp / 4); d += 4) {
-        const float4 ki0 = *reinterpret_cast<const float4*>(ks + i0 * pitch + d), ki1 = *reinterpret_cast<const float4*>(ks + (i0 + 1) * pitch + d);
-        const float4 qi0 = *reinterpret_cast<const float4*>(qs + i0 * pitch + d), qi1 = *reinterpret_cast<const float4*>(qs + (i0 + 1) * pitch + d);
-        const float4 kj0 = *reinterpret_cast<const float4*>(ks + j0 * pitch + d), kj1 = *reinterpret_cast<const float4*>(ks + (j0 + 1) * pitch + d);
-        const float4 Li = *reinterpret_cast<const float4*>(Ls + i0 * pitch + d), Lj = *reinterpret_cast<const float4*>(Ls + (j0 + 1) * pitch + d);
-        const float4 gi = *reinterpret_cast<const float4*>(gs + (i0 + 1) * pitch + d), gj = *reinterpret_cast<const float4*>(gs + (j0 + 1) * pitch + d);
-        auto one = [&](float k0, float k1, float q0, float q1, float c0, float c1, float li, float lj, float g1, float h1) {
-          const float e = diag ? 0.f : __expf(li - lj);
-          const float e01 = e, e11 = diag ? 1.f : e * g1, e00 = diag ? 1.f : e * h1, e10 = e00 * g1;
-          const float x00 = c0 * e00, x01 = c1 * e01, x10 = c0 * e10, x11 = c1 * e11;
-          a[0] = __builtin_fmaf(k0, x00, a[0]); a[1] = __builtin_fmaf(k0, x01, a[1]); a[2] = __builtin_fmaf(k1, x10, a[2]); a[3] = __builtin_fmaf(k1, x11, a[3]);
-          p[0] = __builtin_fmaf(q0, x00, p[0]); p[1] = __builtin_fmaf(q0, x01, p[1]); p[2] = __builtin_fmaf(q1, x10, p[2]); p[3] = __builtin_fmaf(q1, x11, p[3]);
-        };
-        one(ki0.x, ki1.x, qi0.x, qi1.x, kj0.x, kj1.x, Li.x, Lj.x, gi.x, gj.x);
-        one(ki0.y, ki1.y, qi0.y, qi1.y, kj0.y, kj1.y, Li.y, Lj.y, gi.y, gj.y);
-        one(ki0.z, ki1.z, qi0.z, qi1.z, kj0.z, kj1.z, Li.z, Lj.z, gi.z, gj.z);
-        one(ki0.w, ki1.w, qi0.w, qi1.w, kj0.w, kj1.w, Li.w, Lj.w, gi.w, gj.w);
-      }
+  // pairs: a thread takes one of the 36 tiles of tokens (2 I, 2 I + 1) x (2 J, 2 J + 1), J <= I, and every seventh group of four channels
+  float a[4] = {0.f, 0.f, 0.f, 0.f}, p[4] = {0.f, 0.f, 0.f, 0.f};        // (i0,j0) (i0,j1) (i1,j0) (i1,j1)
+  const int part = tid / kPairTiles, tl = tid - part * kPairTiles;
+  if (part < kPairParts) {
+    int I = 0;
+#pragma unroll
+    for (int k = 1; k < 8; ++k) I += tl >= k * (k + 1) / 2 ? 1 : 0;
+    const int J = tl - I * (I + 1) / 2, i0 = 2 * I, j0 = 2 * J;
+    const bool diag = I == J;
+    for (int d = part * 4; d < g.dkp; d += 4 * kPairParts) {
+      const float4 ki0 = *reinterpret_cast<const float4*>(ks + i0 * pitch + d), ki1 = *reinterpret_cast<const float4*>(ks + (i0 + 1) * pitch + d);
+      const float4 qi0 = *reinterpret_cast<const float4*>(qs + i0 * pitch + d), qi1 = *reinterpret_cast<const float4*>(qs + (i0 + 1) * pitch + d);
+      const float4 kj0 = *reinterpret_cast<const float4*>(ks + j0 * pitch + d), kj1 = *reinterpret_cast<const float4*>(ks + (j0 + 1) * pitch + d);
+      const float4 Li = *reinterpret_cast<const float4*>(Ls + i0 * pitch + d), Lj = *reinterpret_cast<const float4*>(Ls + (j0 + 1) * pitch + d);
+      const float4 gi = *reinterpret_cast<const float4*>(gs + (i0 + 1) * pitch + d), gj = *reinterpret_cast<const float4*>(gs + (j0 + 1) * pitch + d);
+      auto one = [&](float k0, float k1, float q0, float q1, float c0, float c1, float li, float lj, float g1, float h1) {
+        const float e = __expf(li - lj);                   // (diagonal tiles: the entry above the diagonal, left out below)
+        const float e11 = diag ? 1.f : e * g1, e00 = diag ? 1.f : e * h1;
+        const float x00 = c0 * e00, x01 = c1 * e, x10 = x00 * g1, x11 = c1 * e11;
+        a[0] = __builtin_fmaf(k0, x00, a[0]); a[1] = __builtin_fmaf(k0, x01, a[1]); a[2] = __builtin_fmaf(k1, x10, a[2]); a[3] = __builtin_fmaf(k1, x11, a[3]);
+        p[0] = __builtin_fmaf(q0, x00, p[0]); p[1] = __builtin_fmaf(q0, x01, p[1]); p[2] = __builtin_fmaf(q1, x10, p[2]); p[3] = __builtin_fmaf(q1, x11, p[3]);
+      };
+      one(ki0.x, ki1.x, qi0.x, qi1.x, kj0.x, kj1.x, Li.x, Lj.x, gi.x, gj.x);
+      one(ki0.y, ki1.y, qi0.y, qi1.y, kj0.y, kj1.y, Li.y, Lj.y, gi.y, gj.y);
+      one(ki0.z, ki1.z, qi0.z, qi1.z, kj0.z, kj1.z, Li.z, Lj.z, gi.z, gj.z);
+      one(ki0.w, ki1.w, qi0.w, qi1.w, kj0.w, kj1.w, Li.w, Lj.w, gi.w, gj.w);
     }
-    float4* r = reinterpret_cast<float4*>(red + (wave * 64 + lane) * 8);
+  }
+  __syncthreads();
+  if (part < kPairParts) {
+    float4* r = reinterpret_cast<float4*>(red + tid * 8);
     r[0] = make_float4(a[0], a[1], a[2], a[3]);
     r[1] = make_float4(p[0], p[1], p[2], p[3]);
   }
+  // k exp L and q exp L in place of k and q, K' out: a thread takes eight tokens of a channel
+  for (int u = tid; u < 2 * g.dkp; u += 256) {
+    const int d = u < g.dkp ? u : u - g.dkp, t0 = u < g.dkp ? 0 : 8;
+    const float end = Ls[(kC - 1) * pitch + d];
+    float o[8];
+#pragma unroll
+    for (int t = 0; t < 8; ++t) {
+      const int r = (t0 + t) * pitch + d;
+      const float L = Ls[r], e = __expf(L), k = ks[r];
+      o[t] = k * __expf(end - L);
+      ks[r] = k * e;
+      qs[r] *= e;
+    }
+    float* kt = F.k + (d >> 4) * 256 + (d & 15) * 16 + t0;
+    *reinterpret_cast<float4*>(kt) = make_float4(o[0], o[1], o[2], o[3]);
+    *reinterpret_cast<float4*>(kt + 4) = make_float4(o[4], o[5], o[6], o[7]);
+    if (t0 == 0) F.e[d] = __expf(end);
+  }
   __syncthreads();
   {
-    const int i = tid >> 4, j = tid & 15, at8 = ((i >> 1) * 8 + (j >> 1)) * 8 + (i & 1) * 2 + (j & 1);
-    float a = 0.f, p = 0.f;
+    const int i = tid >> 4, j = tid & 15, I = i >> 1, J = j >> 1, at8 = (I * (I + 1) / 2 + J) * 8 + (i & 1) * 2 + (j & 1);
+    float av = 0.f, pv = 0.f;
+    if (j <= i) {
 #pragma unroll
-    for (int w = 0; w < 4; ++w) { a += red[w * 512 + at8]; p += red[w * 512 + at8 + 4]; }
-    As[i][j] = j < i ? a * bs[i] : 0.f;
-    Ps[i][j] = j <= i ? p : 0.f;
+      for (int w = 0; w < kPairParts; ++w) { av += red[w * kPairTiles * 8 + at8]; pv += red[w * kPairTiles * 8 + at8 + 4]; }
+    }
+    As[i][j] = j < i ? av * bs[i] : 0.f;
+    Ps[i][j] = j <= i ? pv : 0.f;
+    Ts[i][j] = 0.f;
   }
   __syncthreads();
-  if (wave == 0) {   // (I + A)^-1, a lane per column, by forward substitution
-    float x[kC];
-    const int j = lane & 15;
-#pragma unroll
-    for (int i = 0; i < kC; ++i) {
-      float v = i == j ? 1.f : 0.f;
-#pragma unroll
-      for (int m = 0; m < i; ++m) v = __builtin_fmaf(-As[i][m], x[m], v);
-      x[i] = v;
-    }
+  if (wave == 0) {   // X = (I + A)^-1: the two diagonal blocks by forward substitution, a lane per column; X21 = -X22 A21 X11
     if (lane < kC) {
+      const int b8 = lane & 8, j = lane & 7;
+      float x[8];
 #pragma unroll
-      for (int i = 0; i < kC; ++i) Ts[i][j] = x[i] * bs[j];
-    }
-  } else {           // k exp L and q exp L in place of k and q, K' out
-    for (int d = tid - 64; d < g.dkp; d += 192) {
-      const float end = Ls[(kC - 1) * pitch + d];
-      float* kt = F.k + (d >> 4) * 256 + (d & 15) * 16;
-      float o[kC];
+      for (int i = 0; i < 8; ++i) {
+        float v = i == j ? 1.f : 0.f;
 #pragma unroll
-      for (int t = 0; t < kC; ++t) {
-        const float L = Ls[t * pitch + d], e = expf(L), k = ks[t * pitch + d];
-        o[t] = k * expf(end - L);
-        ks[t * pitch + d] = k * e;
-        qs[t * pitch + d] *= e;
+        for (int m = 0; m < i; ++m) v = __builtin_fmaf(-As[b8 + i][b8 + m], x[m], v);
+        x[i] = v;
       }
 #pragma unroll
-      for (int t = 0; t < kC; t += 4) *reinterpret_cast<float4*>(kt + t) = make_float4(o[t], o[t + 1], o[t + 2], o[t + 3]);
-      F.e[d] = expf(end);
+      for (int i = 0; i < 8; ++i) Ts[b8 + i][b8 + j] = x[i];
     }
+    wave_order();
+    const int i = lane >> 3, j = lane & 7;
+    float y = 0.f;
+#pragma unroll
+    for (int m = 0; m < 8; ++m) y = __builtin_fmaf(As[8 + i][m], Ts[m][j], y);
+    Ms[i][j] = y;
+    wave_order();
+    y = 0.f;
+#pragma unroll
+    for (int m = 0; m < 8; ++m) y = __builtin_fmaf(-Ts[8 + i][8 + m], Ms[m][j], y);
+    wave_order();
+    Ts[8 + i][j] = y;
   }
+  __syncthreads();
+  if (tid < kC * kC) Ts[tid >> 4][tid & 15] *= bs[tid & 15];
   __syncthreads();
   {
     const int i = tid >> 4, j = tid & 15;
@@ -372,63 +417,116 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaGeom g, DeltaIn in
 #pragma unroll
     for (int r = 0; r < 4; ++r) S[t][r] = sg.pos0 + k0 > 0 && tile[t] < tiles ? S0[(size_t)(tile[t] * 16 + 4 * g4 + r) * g.dvp] : 0.f;
   }
-  float cw[TAPS > 0 ? TAPS : 1];
+  constexpr int NX = TAPS > 0 ? TAPS : 1;
+  float cw[NX];
   if constexpr (TAPS > 0) {
 #pragma unroll
-    for (int j = 0; j < TAPS; ++j) cw[j] = in.conv[(size_t)j * C + ch];
+    for (int j = 0; j < TAPS; ++j) cw[j] = vin ? in.conv[(size_t)j * C + ch] : 0.f;
   }
-  struct Frag { f32x4_t w[NT], q[NT], k[NT], e[NT]; float t, m, x[TAPS > 0 ? TAPS : 1]; };
-  auto load = [&](int k, Frag& f) {
-    const Factors F = factors_at(factors, (size_t)(first + k - c0) * g.H + h, g.dkp);
+  // Factors and convolution inputs of the next kAhead chunks are in flight.  Addresses: a uniform part that moves from chunk to chunk and
+  // lane offsets that do not.
+  constexpr int kAhead = NT <= 2 ? 4 : 2;
+  struct Frag { f32x4_t w[NT], q[NT], k[NT], e[NT]; float t, m, x[NX]; };
+  uint32_t off[NT], eoff[NT], xoff[NX], xoff_last[NX];
+#pragma unroll
+  for (int t = 0; t < NT; ++t) {
+    const int tl = min(tile[t], tiles - 1);            // (past the last tile: S stays zero)
+    off[t] = tl * 256 + c * 16 + 4 * g4;
+    eoff[t] = tl * 16 + 4 * g4;
+  }
+  const uint32_t toff = c * 16 + 4 * wave + g4;
+  const int nk = ceil_div(sg.n, kC), left = sg.n - (nk - 1) * kC;      // chunks of the segment, rows of the last one
+#pragma unroll
+  for (int j = 0; j < NX; ++j) {                       // from one chunk's first row on: the rows start at kC ahead of it
+    const int i = 4 * wave + g4;
+    xoff[j] = (uint32_t)(kC + i - (NX - 1 - j)) * in.ldp + ch;
+    xoff_last[j] = (uint32_t)(kC + min(i, left - 1) - (NX - 1 - j)) * in.ldp + ch;
+  }
+  const uint32_t ooff = (uint32_t)(4 * g4 + wave) * g.H * g.dvp + v;
+  const size_t fstride = (size_t)g.H * factor_floats(g.dkp);
+  const float* f0 = factors + ((size_t)(first - c0) * g.H + h) * factor_floats(g.dkp);      // (of the segment's chunk 0: may lie ahead of the piece)
+  const int dk16 = 16 * g.dkp;
+  auto load_factors = [&](int k, Frag& f) {
+    const float *fw = f0 + (ptrdiff_t)k * fstride, *fq = fw + dk16, *fk = fq + dk16, *fe = fk + dk16, *ft = fe + g.dkp, *fm = ft + 256;
 #pragma unroll
     for (int t = 0; t < NT; ++t) {
-      const int tl = min(tile[t], tiles - 1), off = tl * 256 + c * 16 + 4 * g4;     // (past the last tile: S stays zero)
-      f.w[t] = *reinterpret_cast<const f32x4_t*>(F.w + off);
-      f.q[t] = *reinterpret_cast<const f32x4_t*>(F.q + off);
-      f.k[t] = *reinterpret_cast<const f32x4_t*>(F.k + off);
-      f.e[t] = *reinterpret_cast<const f32x4_t*>(F.e + tl * 16 + 4 * g4);
+      f.w[t] = *reinterpret_cast<const f32x4_t*>(fw + off[t]);
+      f.q[t] = *reinterpret_cast<const f32x4_t*>(fq + off[t]);
+      f.k[t] = *reinterpret_cast<const f32x4_t*>(fk + off[t]);
+      f.e[t] = *reinterpret_cast<const f32x4_t*>(fe + eoff[t]);
     }
-    f.t = F.t[c * 16 + 4 * wave + g4];
-    f.m = F.m[c * 16 + 4 * wave + g4];
-    const int tok = min(k * kC + 4 * wave + g4, sg.n - 1);
+    f.t = ft[toff];
+    f.m = fm[toff];
+  };
+  auto load_first = [&](int k, Frag& f) {              // any chunk, the one at the segment's start too
+    load_factors(k, f);
     if constexpr (TAPS > 0) {
+      const int tok = min(k * kC + 4 * wave + g4, sg.n - 1);
 #pragma unroll
       for (int j = 0; j < TAPS; ++j) f.x[j] = conv_in(in, sg, ring, TAPS, C, ch, tok - (TAPS - 1 - j));
-    } else {
-      float a = 0.f;
-      for (int j = 0; j < g.taps; ++j) a = __builtin_fmaf(in.conv[(size_t)j * C + ch], conv_in(in, sg, ring, g.taps, C, ch, tok - (g.taps - 1 - j)), a);
-      f.x[0] = a;
     }
   };
-  Frag f;
-  load(k0, f);
-  for (int k = k0; k < k1; ++k) {
-    Frag nx;
-    load(min(k + 1, k1 - 1), nx);
+  auto load = [&](int k, Frag& f) {                    // k >= 1
+    load_factors(k, f);
+    if constexpr (TAPS > 0) {
+      const float* xb = in.proj + (size_t)(sg.row0 + (k - 1) * kC) * in.ldp;
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) f.x[j] = xb[k == nk - 1 ? xoff_last[j] : xoff[j]];
+    }
+  };
+  auto value = [&](int k, const Frag& f) {            // the value this lane convolves
+    const int mine = k * kC + 4 * wave + g4;
     float x = 0.f;
     if constexpr (TAPS > 0) {
 #pragma unroll
       for (int j = 0; j < TAPS; ++j) x = __builtin_fmaf(cw[j], f.x[j], x);
     } else {
-      x = f.x[0];
+      for (int j = 0; j < g.taps; ++j) x = __builtin_fmaf(in.conv[(size_t)j * C + ch], conv_in(in, sg, ring, g.taps, C, ch, min(mine, sg.n - 1) - (g.taps - 1 - j)), x);
+      x = vin ? x : 0.f;
     }
-    x = vin && k * kC + 4 * wave + g4 < sg.n ? silu(x) : 0.f;
-    f32x4_t u = {0.f, 0.f, 0.f, 0.f}, ov = u;
+    x = silu(x);
+    return mine < sg.n ? x : 0.f;
+  };
+  auto meet = [] {      // one barrier a chunk, for LDS alone: the loads of later chunks stay in flight across it
+    __builtin_amdgcn_sched_barrier(0);
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+    __builtin_amdgcn_sched_barrier(0);
+  };
+  auto emit = [&](int k, int b) {      // a chunk's output: its partial sums lie in ps[b][1]
+    const float* po = reinterpret_cast<const float*>(&ps[b][1][0][0]);
+    float s = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) s += po[(w * 64 + lane) * 4 + wave];
+    float* ob = o + ((size_t)(sg.row0 + k * kC) * g.H + h) * g.dvp;
+    if (k * kC + 4 * g4 + wave < sg.n) ob[ooff] = s;
+  };
+  float x;
+  f32x4_t ov = {0.f, 0.f, 0.f, 0.f};
+  // u's partial sums go out first; o's products, the next chunk's value and the scaling of S run while they do.  o's own meet at the
+  // next chunk's barrier.
+  auto step = [&](int k, const Frag& f, const Frag& nx) {
+    const int b = k & 1;
+    f32x4_t u = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int t = 0; t < NT; ++t)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        u = __builtin_amdgcn_mfma_f32_16x16x4f32(f.w[t][r], S[t][r], u, 0, 0, 0);
-        ov = __builtin_amdgcn_mfma_f32_16x16x4f32(f.q[t][r], S[t][r], ov, 0, 0, 0);
-      }
+      for (int r = 0; r < 4; ++r) u = __builtin_amdgcn_mfma_f32_16x16x4f32(f.w[t][r], S[t][r], u, 0, 0, 0);
     u = __builtin_amdgcn_mfma_f32_16x16x4f32(f.t, x, u, 0, 0, 0);
-    ov = __builtin_amdgcn_mfma_f32_16x16x4f32(f.m, x, ov, 0, 0, 0);
-    const int b = k & 1;
-    ps[b][0][wave][lane] = u;
     ps[b][1][wave][lane] = ov;
-    __syncthreads();
+    ps[b][0][wave][lane] = u;
+    ov = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int t = 0; t < NT; ++t) { S[t][0] *= f.e[t][0]; S[t][1] *= f.e[t][1]; S[t][2] *= f.e[t][2]; S[t][3] *= f.e[t][3]; }
+    for (int t = 0; t < NT; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) ov = __builtin_amdgcn_mfma_f32_16x16x4f32(f.q[t][r], S[t][r], ov, 0, 0, 0);
+    ov = __builtin_amdgcn_mfma_f32_16x16x4f32(f.m, x, ov, 0, 0, 0);
+    x = value(k + 1, nx);
+    f32x4_t Sg[NT];
+#pragma unroll
+    for (int t = 0; t < NT; ++t) Sg[t] = f32x4_t{S[t][0] * f.e[t][0], S[t][1] * f.e[t][1], S[t][2] * f.e[t][2], S[t][3] * f.e[t][3]};
+    meet();
     u = ps[b][0][0][lane];
 #pragma unroll
     for (int w = 1; w < 4; ++w) {
@@ -436,20 +534,32 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaGeom g, DeltaIn in
       u[0] += a[0]; u[1] += a[1]; u[2] += a[2]; u[3] += a[3];
     }
 #pragma unroll
-    for (int t = 0; t < NT; ++t)
+    for (int r = 0; r < 4; ++r)
 #pragma unroll
-      for (int r = 0; r < 4; ++r)
-        if (tile[t] < tiles) S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.k[t][r], u[r], S[t], 0, 0, 0);
-    {
-      const float* po = reinterpret_cast<const float*>(&ps[b][1][0][0]);
-      const int tok = k * kC + 4 * g4 + wave;
-      float s = 0.f;
+      for (int t = 0; t < NT; ++t)     // (a tile past the last one stays zero)
+        Sg[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(tile[t] < tiles ? f.k[t][r] : 0.f, u[r], Sg[t], 0, 0, 0);
 #pragma unroll
-      for (int w = 0; w < 4; ++w) s += po[(w * 64 + lane) * 4 + wave];
-      if (tok < sg.n) o[(size_t)(sg.row0 + tok) * g.H * g.dvp + h * g.dvp + v] = s;
+    for (int t = 0; t < NT; ++t) S[t] = Sg[t];
+    if (k > k0) emit(k - 1, b);
+  };
+  Frag f[kAhead];
+#pragma unroll
+  for (int i = 0; i < kAhead; ++i) load_first(min(k0 + i, k1 - 1), f[i]);
+  x = value(k0, f[0]);
+  int k = k0;
+  for (; k + kAhead <= k1; k += kAhead) {
+#pragma unroll
+    for (int i = 0; i < kAhead; ++i) {
+      step(k + i, f[i], f[(i + 1) % kAhead]);
+      load(min(k + i + kAhead, k1 - 1), f[i]);
     }
-    f = nx;
   }
+#pragma unroll
+  for (int i = 0; i < kAhead; ++i)
+    if (k + i < k1) step(k + i, f[i], f[(i + 1) % kAhead]);
+  ps[k1 & 1][1][wave][lane] = ov;
+  __syncthreads();
+  emit(k1 - 1, k1 & 1);
 #pragma unroll
   for (int t = 0; t < NT; ++t)
 #pragma unroll
@@ -457,29 +567,41 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaGeom g, DeltaIn in
       if (tile[t] < tiles) S0[(size_t)(tile[t] * 16 + 4 * g4 + r) * g.dvp] = S[t][r];
 }
 
-// norm and gate, a wave per head and token; the work-groups of a segment's last chunk renew its ring
-template <typename T>
+// norm and gate: a wave per head, four of the chunk's tokens at a time; the work-groups of a segment's last chunk renew its ring
+template <typename T, int NV>
 __global__ __launch_bounds__(256) void delta_out_kernel(DeltaGeom g, DeltaIn in, const AttnSeg* __restrict__ segs, int nseg, int c0, const float* __restrict__ o,
                                                         T* __restrict__ y, int ldy) {
   const ChunkAt at = chunk_at(segs, nseg, c0 + blockIdx.x);
   if (!at.ok) return;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, h = blockIdx.y * 4 + wave;
   if (h < g.H) {
-    for (int t = 0; t < at.n; ++t) {
-      const size_t row = at.sg.row0 + at.t0 + t;
-      const float* src = o + row * g.H * g.dvp + h * g.dvp;
-      float x[4], ss = 0.f;
+    float nw[NV];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int v = lane + 64 * i;
-        x[i] = v < g.dv ? src[v] : 0.f;
-        ss = __builtin_fmaf(x[i], x[i], ss);
-      }
-      const float f = 1.f / sqrtf(wave_sum(ss) / (float)g.dv + in.eps);
+    for (int i = 0; i < NV; ++i) nw[i] = in.norm[min(lane + 64 * i, g.dv - 1)];
+    const size_t row0 = at.sg.row0 + at.t0;
+    const float *src = o + row0 * g.H * g.dvp + h * g.dvp, *zr = in.z + row0 * in.ldz + in.gate + h * g.dv;
+    for (int t0 = 0; t0 < at.n; t0 += 4) {
+      float x[4][NV], z[4][NV];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int v = lane + 64 * i;
-        if (v < g.dv) put1(y + row * ldy + h * g.dv + v, x[i] * f * in.norm[v] * sigmoid(in.z[row * in.ldz + in.gate + h * g.dv + v]));
+      for (int t = 0; t < 4; ++t)
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+          const int r = min(t0 + t, at.n - 1), v = min(lane + 64 * i, g.dv - 1);
+          x[t][i] = src[(size_t)r * g.H * g.dvp + v];
+          z[t][i] = zr[(size_t)r * in.ldz + v];
+        }
+#pragma unroll
+      for (int t = 0; t < 4; ++t) {
+        float ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < NV; ++i) ss = __builtin_fmaf(x[t][i], lane + 64 * i < g.dv ? x[t][i] : 0.f, ss);
+        const float f = 1.f / sqrtf(wave_sum(ss) / (float)g.dv + in.eps);
+        if (t0 + t >= at.n) break;
+#pragma unroll
+        for (int i = 0; i < NV; ++i) {
+          const int v = lane + 64 * i;
+          if (v < g.dv) put1(y + (row0 + t0 + t) * ldy + h * g.dv + v, x[t][i] * f * nw[i] * sigmoid(z[t][i]));
+        }
       }
     }
   }
@@ -533,7 +655,7 @@ int launch_delta_prompt(const DeltaGeom& g, const DeltaIn& in, const AttnSeg* sd
   int chunks = 0;
   for (int i = 0; i < nseg; ++i) chunks += sh[i].n < 2 ? 0 : ceil_div(sh[i].n, kC);
   const int nvt = g.dvp / 16, nt = ceil_div(g.dkp / 16, 4);
-  const size_t lds = (size_t)(4 * kC * (g.dkp + 4) + 4 * 64 * 8) * sizeof(float);
+  const size_t lds = (size_t)(3 * kC * (g.dkp + 4) + std::max(kC * (g.dkp + 4), kPairParts * kPairTiles * 8)) * sizeof(float);
   for (int c0 = 0; c0 < chunks; c0 += max_chunks) {
     const int n = std::min(max_chunks, chunks - c0);
     const dim3 gf(n, g.H), gs(g.H * nvt, nseg), go(n, ceil_div(g.H, 4));
@@ -552,8 +674,11 @@ int launch_delta_prompt(const DeltaGeom& g, const DeltaIn& in, const AttnSeg* sd
       default: MI_DF(0);
     }
 #undef MI_DF
-    if (f32) hipLaunchKernelGGL((delta_out_kernel<float>), go, dim3(256), 0, s, g, in, sd, nseg, c0, o, (float*)y, ldy);
-    else hipLaunchKernelGGL((delta_out_kernel<uint16_t>), go, dim3(256), 0, s, g, in, sd, nseg, c0, o, (uint16_t*)y, ldy);
+#define MI_DO(NV) \
+    if (f32) hipLaunchKernelGGL((delta_out_kernel<float, NV>), go, dim3(256), 0, s, g, in, sd, nseg, c0, o, (float*)y, ldy); \
+    else hipLaunchKernelGGL((delta_out_kernel<uint16_t, NV>), go, dim3(256), 0, s, g, in, sd, nseg, c0, o, (uint16_t*)y, ldy)
+    if (g.dv <= 64) { MI_DO(1); } else if (g.dv <= 128) { MI_DO(2); } else { MI_DO(4); }
+#undef MI_DO
     MI_HIP(hipGetLastError());
   }
   return MI_OK;

@@ -79,7 +79,17 @@ __global__ __launch_bounds__(256) void latent_scatter_kernel(LatentRowsIn in, Sl
     const bool vec = ((g.dk | g.nr) & 3) == 0;
     for (int d = (tid & 31) * 4; d < g.dkp; d += 128) {
       float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
-      if (d + 3 >= g.dk && g.nr) {
+      if (vec && d >= g.dk && ((g.dims >> 1) & 3) == 0 && g.nr) {      // four pairs at a time
+        const int i = d - g.dk, half = g.dims >> 1, j = i < half ? i : i - half;
+        if (i < g.dims) {
+          const float4 u = row.at4(c0 + g.dk + j), w = row.at4(c0 + g.dk + j + half);
+          const float4 a = *reinterpret_cast<const float4*>(cs + j), b = *reinterpret_cast<const float4*>(cs + j + 2);    // (cos, sin) of two pairs each
+          v = i < half ? make_float4(u.x * a.x - w.x * a.y, u.y * a.z - w.y * a.w, u.z * b.x - w.z * b.y, u.w * b.z - w.w * b.w)
+                       : make_float4(w.x * a.x + u.x * a.y, w.y * a.z + u.y * a.w, w.z * b.x + u.z * b.y, w.w * b.z + u.w * b.w);
+        } else if (i < g.nr) {
+          v = row.at4(c0 + d);
+        }
+      } else if (d + 3 >= g.dk && g.nr) {
         auto at = [&](int i) {
           if (d + i < g.dk) return row.at(c0 + d + i);
           return d + i < g.dk + g.nr ? rotated(d + i - g.dk, g.dims, cs, [&](int k) { return row.at(c0 + g.dk + k); }) : 0.f;

@@ -104,12 +104,12 @@ constexpr size_t prefill_lds() { return (size_t)64 * (DK + kPitch + DV + kPitch)
 // KS = 2: a second set of four waves takes every other key tile of the same queries (short grids, whose heaviest work-group is what
 // the launch waits for); the two sets' sums meet in LDS at the end.
 template <int DK, int DV, int NCG, int KS2, bool FIXED>
-__global__ __launch_bounds__(256 * KS2) __attribute__((amdgpu_waves_per_eu(DK > 128 ? KS2 : 2, DK > 128 ? KS2 : 2))) void attn_window_prefill_kernel(AttnSpec a, const uint16_t* __restrict__ q, const uint16_t* __restrict__ kpool,
+__global__ __launch_bounds__(256 * KS2) __attribute__((amdgpu_waves_per_eu(DK > 192 || DV > 128 ? KS2 : 2, DK > 192 || DV > 128 ? KS2 : 2))) void attn_window_prefill_kernel(AttnSpec a, const uint16_t* __restrict__ q, const uint16_t* __restrict__ kpool,
                                                                   const uint16_t* __restrict__ vpool, int bs, const int32_t* __restrict__ bt,
                                                                   int MB, const AttnSeg* __restrict__ segs, int nseg,
                                                                   uint16_t* __restrict__ out, int ldo, float s_max, int fold, int min_rows, int bs_shift) {
   constexpr int KP = DK + kPitch, VP = DV + kPitch;    // LDS row pitches (elements)
-  constexpr int KS = DK / 32, DN = DV / 16, KCH = DK / 8, VCH = DV / 8;
+  constexpr int KS = DK / 32, DN = DV / 16, KCH = DK / 8, VCH = DV / 8, KC0 = KCH == 24 ? 16 : KCH;   // (192 = 128 + 64: powers of two)
   constexpr int NKL = 64 * KCH / 256, NVL = 64 * VCH / 256;   // 16-byte loads per thread and tile
   extern __shared__ __attribute__((aligned(16))) unsigned char dsm[];
   const int set = KS2 == 1 ? 0 : (int)threadIdx.x >> 8;
@@ -153,9 +153,9 @@ __global__ __launch_bounds__(256 * KS2) __attribute__((amdgpu_waves_per_eu(DK > 
       if (!in) off[u] = 0;
     }
   };
-  auto load_tile = [&](auto& reg, const uint16_t* pool, const size_t (&base)[4], int rowp, int last, auto chunks) {
+  auto load_tile = [&](u32x4_t* reg, const uint16_t* pool, const size_t (&base)[4], int rowp, int last, auto chunks, int chunk0 = 0) {
     constexpr int CH = decltype(chunks)::value, R = 256 / CH, N = 64 / R;
-    const int row0 = tid / CH, lane_off = (row0 & 15) * rowp + min(tid % CH, last) * 8;
+    const int row0 = tid / CH, lane_off = (row0 & 15) * rowp + min(chunk0 + tid % CH, last) * 8;
 #pragma unroll
     for (int i = 0; i < N; ++i) {
       if constexpr (R >= 16) {
@@ -171,7 +171,8 @@ __global__ __launch_bounds__(256 * KS2) __attribute__((amdgpu_waves_per_eu(DK > 
     size_t base[4];
 #pragma unroll
     for (int u = 0; u < 4; ++u) base[u] = ((size_t)blk[u] * G + kvh) * bs + off[u];
-    load_tile(kr, kpool, base, a.g.dkp, dkc, std::integral_constant<int, KCH>{});
+    load_tile(kr, kpool, base, a.g.dkp, dkc, std::integral_constant<int, KC0>{});
+    if constexpr (KCH > KC0) load_tile(kr + KC0 / 4, kpool, base, a.g.dkp, dkc, std::integral_constant<int, KCH - KC0>{}, KC0);
     load_tile(vr, vpool, base, a.g.dvp, dvc, std::integral_constant<int, VCH>{});
   };
   const int k_own = klo + 64 * set;        // this set's first tile
@@ -213,9 +214,16 @@ __global__ __launch_bounds__(256 * KS2) __attribute__((amdgpu_waves_per_eu(DK > 
     const int k0 = k_own + 64 * n;       // (the second set's last tile may lie beyond the keys: no wave sees a key of it)
     __syncthreads();                     // the previous tile is consumed
 #pragma unroll
-    for (int i = 0; i < NKL; ++i) {
+    for (int i = 0; i < KC0 / 4; ++i) {
       const int idx = tid + 256 * i;
-      *reinterpret_cast<u32x4_t*>(&Ks[(idx / KCH) * KP + (idx % KCH) * 8]) = kr[i];
+      *reinterpret_cast<u32x4_t*>(&Ks[(idx / KC0) * KP + (idx % KC0) * 8]) = kr[i];
+    }
+    if constexpr (KCH > KC0) {
+#pragma unroll
+      for (int i = 0; i < (KCH - KC0) / 4; ++i) {
+        const int idx = tid + 256 * i;
+        *reinterpret_cast<u32x4_t*>(&Ks[(idx / (KCH - KC0)) * KP + (KC0 + idx % (KCH - KC0)) * 8]) = kr[KC0 / 4 + i];
+      }
     }
 #pragma unroll
     for (int i = 0; i < NVL; ++i) {
@@ -720,8 +728,9 @@ int launch_attn_window_prefill(const AttnSpec& a, const uint16_t* q, const uint1
   for (int i = 0; i < nseg; ++i) tiles += sh[i].n >= min_rows ? ceil_div(sh[i].n, 128 / (a.g.H / a.g.G)) : 0;
   const bool half = tiles * a.g.G < 2 * num_cu;
 #define MI_CALL_P(DK, DV, NCG) \
-  half ? launch_prefill_t<DK, DV, 1, (DK > 128 || DV > 128 ? 1 : 2)>(a, q, kpool, vpool, bs, bt, MB, sd, sh, nseg, out, ldo, s, min_rows) \
+  half ? launch_prefill_t<DK, DV, 1, (DK > 192 || DV > 128 ? 1 : 2)>(a, q, kpool, vpool, bs, bt, MB, sd, sh, nseg, out, ldo, s, min_rows) \
        : launch_prefill_t<DK, DV, NCG, 1>(a, q, kpool, vpool, bs, bt, MB, sd, sh, nseg, out, ldo, s, min_rows)
+  if (a.g.dkp > 128 && a.g.dkp <= 192 && a.g.dvp <= 128) return MI_CALL_P(192, 128, 2);
   MI_BY_SIZE(MI_CALL_P);
 #undef MI_CALL_P
 }

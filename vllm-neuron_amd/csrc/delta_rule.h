@@ -38,12 +38,11 @@ struct DeltaIn {
 };
 bool delta_supported(const DeltaGeom& g);
 constexpr int kDeltaChunk = 16;
-// device memory behind delta_prompt: the factors of `chunks` chunks
-size_t delta_factor_floats(const DeltaGeom& g);        // of one chunk
+size_t delta_chunk_floats(const DeltaGeom& g);         // device memory behind a chunk of a prompt: factors, values, outputs
 // token generation: row = sequence (segs null), or the one-row segments of a ragged batch
 int launch_delta_token(const DeltaGeom& g, const DeltaIn& in, int rows, const AttnSeg* segs, void* y, int ldy, bool f32, hipStream_t s);
-// the segments of two rows and more; o [rows][H dvp] scratch; factors: memory for max_chunks chunks
-int launch_delta_prompt(const DeltaGeom& g, const DeltaIn& in, const AttnSeg* segs_dev, const AttnSeg* segs_host, int nseg, float* factors,
-                        int max_chunks, float* o, void* y, int ldy, bool f32, hipStream_t s);
+// the segments of two rows and more; records: memory for max_chunks chunks, more of them go in pieces
+int launch_delta_prompt(const DeltaGeom& g, const DeltaIn& in, const AttnSeg* segs_dev, const AttnSeg* segs_host, int nseg, float* records,
+                        int max_chunks, void* y, int ldy, bool f32, hipStream_t s);
 
 }  // namespace mi

@@ -143,13 +143,14 @@ __device__ __forceinline__ ChunkAt chunk_at(const AttnSeg* segs, int nseg, int c
   return ChunkAt{AttnSeg{0, 0, 0, 0}, 0, 0, false, false};
 }
 
-// factors of a chunk and head, in floats: -W, Q', K' as [dkp / 16] tiles of 16 x 16 (W, Q': token x channel; K': channel x token),
-// exp L_end [dkp], T and P T [16][16]
-struct Factors { float *w, *q, *k, *e, *t, *m; };
-__host__ __device__ __forceinline__ size_t factor_floats(int dkp) { return (size_t)49 * dkp + 512; }
-__device__ __forceinline__ Factors factors_at(float* base, size_t index, int dkp) {
-  float* p = base + index * factor_floats(dkp);
-  return Factors{p, p + 16 * dkp, p + 32 * dkp, p + 48 * dkp, p + 49 * dkp, p + 49 * dkp + 256};
+// The record of a chunk and head, in floats: -W, Q', K' as [dkp / 16] tiles of 16 x 16 (W, Q': token x channel; K': channel x token),
+// exp L_end [dkp], T and P T [16][16], and [dvp / 16] tiles (token x column) of values that the scan replaces by outputs.  A head's
+// records follow each other: the scan reads on without a gap.
+struct Factors { float *w, *q, *k, *e, *t, *m, *v; };
+__host__ __device__ __forceinline__ size_t record_floats(int dkp, int dvp) { return (size_t)49 * dkp + 512 + 16 * dvp; }
+__device__ __forceinline__ Factors factors_at(float* base, size_t index, int dkp, int dvp) {
+  float* p = base + index * record_floats(dkp, dvp);
+  return Factors{p, p + 16 * dkp, p + 32 * dkp, p + 48 * dkp, p + 49 * dkp, p + 49 * dkp + 256, p + 49 * dkp + 512};
 }
 
 // where the input of a convolution `i` rows behind the segment's start lies (negative: ahead of it; ahead of the sequence: anywhere
@@ -181,39 +182,39 @@ __global__ __launch_bounds__(256) void delta_factors_kernel(DeltaGeom g, DeltaIn
   const ChunkAt at = chunk_at(segs, nseg, c0 + blockIdx.x);
   if (!at.ok) return;
   const int h = blockIdx.y, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, n = at.n, C = g.channels(), kvh = h / (g.H / g.G);
-  const Factors F = factors_at(out, (size_t)blockIdx.x * g.H + h, g.dkp);
+  const Factors F = factors_at(out, (size_t)h * gridDim.x + blockIdx.x, g.dkp, g.dvp);
   const float* ring = in.ring + (size_t)in.slots[at.sg.seq] * g.taps * C;
   const float* rows = in.proj + (size_t)(at.sg.row0 + at.t0) * in.ldp;
-  // convolutions: a thread walks one channel down the chunk
-  for (int i = tid; i < 2 * g.dkp; i += 256) {
-    const int part = i < g.dkp ? 0 : 1, d = i - part * g.dkp;
-    float* dst = (part ? ks : qs) + d;
-    if (d >= g.dk) {
-      for (int t = 0; t < kC; ++t) dst[t * pitch] = 0.f;
-      continue;
-    }
-    const int ch = (part * g.G + kvh) * g.dk + d;
+  // convolutions: a thread walks one channel of q, k or v down half the chunk
+  constexpr int kHalf = kC / 2;
+  const int cols = 2 * g.dkp + g.dvp;
+  for (int i = tid; i < 2 * cols; i += 256) {
+    const int t0 = i < cols ? 0 : kHalf, col = i < cols ? i : i - cols;
+    const int part = col < g.dkp ? 0 : col < 2 * g.dkp ? 1 : 2, d = col - part * g.dkp, size = part == 2 ? g.dv : g.dk;
+    const int ch = part == 2 ? 2 * g.G * g.dk + h * g.dv + min(d, size - 1) : (part * g.G + kvh) * g.dk + min(d, size - 1);
+    float* dst = part == 2 ? F.v + (d >> 4) * 256 + (d & 15) : (part ? ks : qs) + d;
+    const int step = part == 2 ? 16 : pitch;
     if constexpr (TAPS > 0) {
-      float x[kC + TAPS - 1], w[TAPS];
+      float x[kHalf + TAPS - 1], w[TAPS];
 #pragma unroll
-      for (int k = 0; k < kC + TAPS - 1; ++k) {
-        const int t = k - (TAPS - 1);
-        x[k] = t < 0 ? conv_in(in, at.sg, ring, TAPS, C, ch, at.t0 + t) : rows[(size_t)min(t, n - 1) * in.ldp + ch];
+      for (int k = 0; k < kHalf + TAPS - 1; ++k) {
+        const int t = t0 + k - (TAPS - 1);
+        x[k] = conv_in(in, at.sg, ring, TAPS, C, ch, at.t0 + min(t, n - 1));
       }
 #pragma unroll
       for (int j = 0; j < TAPS; ++j) w[j] = in.conv[(size_t)j * C + ch];
 #pragma unroll
-      for (int t = 0; t < kC; ++t) {
+      for (int t = 0; t < kHalf; ++t) {
         float a = 0.f;
 #pragma unroll
         for (int j = 0; j < TAPS; ++j) a = __builtin_fmaf(w[j], x[t + j], a);
-        dst[t * pitch] = t < n ? silu(a) : 0.f;
+        dst[(t0 + t) * step] = t0 + t < n && d < size ? silu(a) : 0.f;
       }
     } else {
-      for (int t = 0; t < kC; ++t) {
+      for (int t = t0; t < t0 + kHalf; ++t) {
         float a = 0.f;
         for (int j = 0; j < g.taps; ++j) a = __builtin_fmaf(in.conv[(size_t)j * C + ch], conv_in(in, at.sg, ring, g.taps, C, ch, at.t0 + min(t, n - 1) - (g.taps - 1 - j)), a);
-        dst[t * pitch] = t < n ? silu(a) : 0.f;
+        dst[t * step] = t < n && d < size ? silu(a) : 0.f;
       }
     }
   }
@@ -383,9 +384,9 @@ __global__ __launch_bounds__(256) void delta_factors_kernel(DeltaGeom g, DeltaIn
 // One work-group per (head, 16 value columns, segment): the chunks of the segment in order.  A wave holds NT 16-channel tiles of the
 // state as MFMA accumulators, which are the B operands of the next chunk's products as they stand; the partial sums of u and
 // o over the channels meet in LDS, once per chunk.
-template <int NT, int TAPS>
-__global__ __launch_bounds__(256) void delta_scan_kernel(DeltaGeom g, DeltaIn in, const AttnSeg* __restrict__ segs, int nseg, int c0, int c1, int nvt,
-                                                         float* __restrict__ factors, float* __restrict__ o) {
+template <int NT>
+__global__ __launch_bounds__(256) void delta_scan_kernel(DeltaGeom g, float* __restrict__ state, const int32_t* __restrict__ slots,
+                                                         const AttnSeg* __restrict__ segs, int c0, int nchunks, int nvt, float* __restrict__ records) {
   __shared__ f32x4_t ps[2][2][4][64];
   int id = blockIdx.x, h, vt;
   if (g.H % 8 == 0) {        // the column blocks of a head on one XCD: they read the same factors
@@ -401,91 +402,42 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaGeom g, DeltaIn in
   if (sg.n < 2) return;
   int first = 0;             // the segment's first chunk among all
   for (int i = 0; i < si; ++i) first += segs[i].n < 2 ? 0 : ceil_div(segs[i].n, kC);
-  const int k0 = max(c0 - first, 0), k1 = min(c1 - first, ceil_div(sg.n, kC));
+  const int k0 = max(c0 - first, 0), k1 = min(c0 + nchunks - first, ceil_div(sg.n, kC));
   if (k0 >= k1) return;
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g4 = lane >> 4, c = lane & 15;
-  const int tiles = g.dkp / 16, v = vt * 16 + c, slot = in.slots[sg.seq], C = g.channels();
-  const bool vin = v < g.dv;
-  float* S0 = in.state + ((size_t)slot * g.H + h) * g.dkp * g.dvp + v;
-  const float* ring = in.ring + (size_t)slot * g.taps * C;
-  const int ch = 2 * g.G * g.dk + h * g.dv + min(v, g.dv - 1);
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, g4 = lane >> 4, c = lane & 15, tiles = g.dkp / 16;
+  float* S0 = state + ((size_t)slots[sg.seq] * g.H + h) * g.dkp * g.dvp + vt * 16 + c;
   f32x4_t S[NT];
-  int tile[NT];
-#pragma unroll
-  for (int t = 0; t < NT; ++t) {
-    tile[t] = wave * NT + t;
-#pragma unroll
-    for (int r = 0; r < 4; ++r) S[t][r] = sg.pos0 + k0 > 0 && tile[t] < tiles ? S0[(size_t)(tile[t] * 16 + 4 * g4 + r) * g.dvp] : 0.f;
-  }
-  constexpr int NX = TAPS > 0 ? TAPS : 1;
-  float cw[NX];
-  if constexpr (TAPS > 0) {
-#pragma unroll
-    for (int j = 0; j < TAPS; ++j) cw[j] = vin ? in.conv[(size_t)j * C + ch] : 0.f;
-  }
-  // Factors and convolution inputs of the next kAhead chunks are in flight.  Addresses: a uniform part that moves from chunk to chunk and
-  // lane offsets that do not.
+  // Factors and values of the next kAhead chunks are in flight.  Addresses: a uniform part that moves from chunk to chunk and lane
+  // offsets (bytes) that do not.
   constexpr int kAhead = NT <= 2 ? 4 : 2;
-  struct Frag { f32x4_t w[NT], q[NT], k[NT], e[NT]; float t, m, x[NX]; };
-  uint32_t off[NT], eoff[NT], xoff[NX], xoff_last[NX];
+  struct Frag { f32x4_t w[NT], q[NT], k[NT], e[NT]; float t, m, x; };
+  uint32_t off[NT], eoff[NT];
 #pragma unroll
   for (int t = 0; t < NT; ++t) {
-    const int tl = min(tile[t], tiles - 1);            // (past the last tile: S stays zero)
-    off[t] = tl * 256 + c * 16 + 4 * g4;
-    eoff[t] = tl * 16 + 4 * g4;
+    const int tile = wave * NT + t, tl = min(tile, tiles - 1);            // (past the last tile: S stays zero)
+    off[t] = (tl * 256 + c * 16 + 4 * g4) * 4;
+    eoff[t] = (tl * 16 + 4 * g4) * 4;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) S[t][r] = sg.pos0 + k0 > 0 && tile < tiles ? S0[(size_t)(tile * 16 + 4 * g4 + r) * g.dvp] : 0.f;
   }
-  const uint32_t toff = c * 16 + 4 * wave + g4;
-  const int nk = ceil_div(sg.n, kC), left = sg.n - (nk - 1) * kC;      // chunks of the segment, rows of the last one
-#pragma unroll
-  for (int j = 0; j < NX; ++j) {                       // from one chunk's first row on: the rows start at kC ahead of it
-    const int i = 4 * wave + g4;
-    xoff[j] = (uint32_t)(kC + i - (NX - 1 - j)) * in.ldp + ch;
-    xoff_last[j] = (uint32_t)(kC + min(i, left - 1) - (NX - 1 - j)) * in.ldp + ch;
-  }
-  const uint32_t ooff = (uint32_t)(4 * g4 + wave) * g.H * g.dvp + v;
-  const size_t fstride = (size_t)g.H * factor_floats(g.dkp);
-  const float* f0 = factors + ((size_t)(first - c0) * g.H + h) * factor_floats(g.dkp);      // (of the segment's chunk 0: may lie ahead of the piece)
-  const int dk16 = 16 * g.dkp;
-  auto load_factors = [&](int k, Frag& f) {
-    const float *fw = f0 + (ptrdiff_t)k * fstride, *fq = fw + dk16, *fk = fq + dk16, *fe = fk + dk16, *ft = fe + g.dkp, *fm = ft + 256;
-#pragma unroll
-    for (int t = 0; t < NT; ++t) {
-      f.w[t] = *reinterpret_cast<const f32x4_t*>(fw + off[t]);
-      f.q[t] = *reinterpret_cast<const f32x4_t*>(fq + off[t]);
-      f.k[t] = *reinterpret_cast<const f32x4_t*>(fk + off[t]);
-      f.e[t] = *reinterpret_cast<const f32x4_t*>(fe + eoff[t]);
-    }
-    f.t = ft[toff];
-    f.m = fm[toff];
+  const uint32_t toff = (c * 16 + 4 * wave + g4) * 4, xoff = ((4 * wave + g4) * 16 + c) * 4, ooff = ((4 * g4 + wave) * 16 + c) * 4;
+  auto at = [](float* base, uint32_t bytes) { return reinterpret_cast<unsigned char*>(base) + bytes; };
+  auto record = [&](int k) { return factors_at(records, (size_t)h * nchunks + (first + k - c0), g.dkp, g.dvp); };
+  auto load_w = [&](const Factors& F, Frag& f, int t) { f.w[t] = *reinterpret_cast<const f32x4_t*>(at(F.w, off[t])); };
+  auto load_q = [&](const Factors& F, Frag& f, int t) { f.q[t] = *reinterpret_cast<const f32x4_t*>(at(F.q, off[t])); };
+  auto load_k = [&](const Factors& F, Frag& f, int t) { f.k[t] = *reinterpret_cast<const f32x4_t*>(at(F.k, off[t])); };
+  auto load_e = [&](const Factors& F, Frag& f, int t) { f.e[t] = *reinterpret_cast<const f32x4_t*>(at(F.e, eoff[t])); };
+  auto load_rest = [&](const Factors& F, Frag& f, int i) {
+    if (i == 0) f.t = *reinterpret_cast<const float*>(at(F.t, toff));
+    if (i == 1) f.m = *reinterpret_cast<const float*>(at(F.m, toff));
+    if (i == 2) f.x = *reinterpret_cast<const float*>(at(F.v + vt * 256, xoff));
   };
-  auto load_first = [&](int k, Frag& f) {              // any chunk, the one at the segment's start too
-    load_factors(k, f);
-    if constexpr (TAPS > 0) {
-      const int tok = min(k * kC + 4 * wave + g4, sg.n - 1);
+  auto load = [&](int k, Frag& f) {
+    const Factors F = record(k);
 #pragma unroll
-      for (int j = 0; j < TAPS; ++j) f.x[j] = conv_in(in, sg, ring, TAPS, C, ch, tok - (TAPS - 1 - j));
-    }
-  };
-  auto load = [&](int k, Frag& f) {                    // k >= 1
-    load_factors(k, f);
-    if constexpr (TAPS > 0) {
-      const float* xb = in.proj + (size_t)(sg.row0 + (k - 1) * kC) * in.ldp;
+    for (int t = 0; t < NT; ++t) { load_w(F, f, t); load_q(F, f, t); load_k(F, f, t); load_e(F, f, t); }
 #pragma unroll
-      for (int j = 0; j < TAPS; ++j) f.x[j] = xb[k == nk - 1 ? xoff_last[j] : xoff[j]];
-    }
-  };
-  auto value = [&](int k, const Frag& f) {            // the value this lane convolves
-    const int mine = k * kC + 4 * wave + g4;
-    float x = 0.f;
-    if constexpr (TAPS > 0) {
-#pragma unroll
-      for (int j = 0; j < TAPS; ++j) x = __builtin_fmaf(cw[j], f.x[j], x);
-    } else {
-      for (int j = 0; j < g.taps; ++j) x = __builtin_fmaf(in.conv[(size_t)j * C + ch], conv_in(in, sg, ring, g.taps, C, ch, min(mine, sg.n - 1) - (g.taps - 1 - j)), x);
-      x = vin ? x : 0.f;
-    }
-    x = silu(x);
-    return mine < sg.n ? x : 0.f;
+    for (int i = 0; i < 3; ++i) load_rest(F, f, i);
   };
   auto meet = [] {      // one barrier a chunk, for LDS alone: the loads of later chunks stay in flight across it
     __builtin_amdgcn_sched_barrier(0);
@@ -494,35 +446,48 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaGeom g, DeltaIn in
     asm volatile("" ::: "memory");
     __builtin_amdgcn_sched_barrier(0);
   };
-  auto emit = [&](int k, int b) {      // a chunk's output: its partial sums lie in ps[b][1]
+  auto emit = [&](int k, int b) {      // a chunk's output in place of its values: its partial sums lie in ps[b][1]
     const float* po = reinterpret_cast<const float*>(&ps[b][1][0][0]);
     float s = 0.f;
 #pragma unroll
     for (int w = 0; w < 4; ++w) s += po[(w * 64 + lane) * 4 + wave];
-    float* ob = o + ((size_t)(sg.row0 + k * kC) * g.H + h) * g.dvp;
-    if (k * kC + 4 * g4 + wave < sg.n) ob[ooff] = s;
+    *reinterpret_cast<float*>(at(record(k).v + vt * 256, ooff)) = s;
   };
-  float x;
   f32x4_t ov = {0.f, 0.f, 0.f, 0.f};
-  // u's partial sums go out first; o's products, the next chunk's value and the scaling of S run while they do.  o's own meet at the
-  // next chunk's barrier.
-  auto step = [&](int k, const Frag& f, const Frag& nx) {
+  // u's partial sums go out first; o's products and the scaling of S run while they do.  o's own meet at the next chunk's barrier.
+  // A CU takes a wave's 16-byte loads in at one per 16 clocks: they are dealt out between the products, each as soon as what it
+  // replaces is used up (K' and exp L_end of the chunk before behind the first products).
+  auto pin = [] { __builtin_amdgcn_sched_barrier(0x6); };       // (ALU instructions may cross)
+  auto step = [&](int k, Frag& f, Frag& before, bool more, bool more_before) {
     const int b = k & 1;
+    const Factors Fn = record(k + kAhead), Fb = record(k - 1 + kAhead);
     f32x4_t u = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int t = 0; t < NT; ++t)
+    for (int t = 0; t < NT; ++t) {
 #pragma unroll
-      for (int r = 0; r < 4; ++r) u = __builtin_amdgcn_mfma_f32_16x16x4f32(f.w[t][r], S[t][r], u, 0, 0, 0);
-    u = __builtin_amdgcn_mfma_f32_16x16x4f32(f.t, x, u, 0, 0, 0);
+      for (int r = 0; r < 4; ++r) {
+        u = __builtin_amdgcn_mfma_f32_16x16x4f32(f.w[t][r], S[t][r], u, 0, 0, 0);
+        if (r & 1) {
+          pin();
+          if (more_before) { if (r == 1) load_k(Fb, before, t); else load_e(Fb, before, t); }
+          pin();
+        }
+      }
+    }
+    u = __builtin_amdgcn_mfma_f32_16x16x4f32(f.t, f.x, u, 0, 0, 0);
     ps[b][1][wave][lane] = ov;
     ps[b][0][wave][lane] = u;
+    pin();
     ov = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int t = 0; t < NT; ++t)
+    for (int t = 0; t < NT; ++t) {
 #pragma unroll
       for (int r = 0; r < 4; ++r) ov = __builtin_amdgcn_mfma_f32_16x16x4f32(f.q[t][r], S[t][r], ov, 0, 0, 0);
-    ov = __builtin_amdgcn_mfma_f32_16x16x4f32(f.m, x, ov, 0, 0, 0);
-    x = value(k + 1, nx);
+      pin();
+      if (more) load_w(Fn, f, t);
+      pin();
+    }
+    ov = __builtin_amdgcn_mfma_f32_16x16x4f32(f.m, f.x, ov, 0, 0, 0);
     f32x4_t Sg[NT];
 #pragma unroll
     for (int t = 0; t < NT; ++t) Sg[t] = f32x4_t{S[t][0] * f.e[t][0], S[t][1] * f.e[t][1], S[t][2] * f.e[t][2], S[t][3] * f.e[t][3]};
@@ -534,29 +499,38 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaGeom g, DeltaIn in
       u[0] += a[0]; u[1] += a[1]; u[2] += a[2]; u[3] += a[3];
     }
 #pragma unroll
-    for (int r = 0; r < 4; ++r)
+    for (int r = 0; r < 4; ++r) {
 #pragma unroll
       for (int t = 0; t < NT; ++t)     // (a tile past the last one stays zero)
-        Sg[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(tile[t] < tiles ? f.k[t][r] : 0.f, u[r], Sg[t], 0, 0, 0);
+        Sg[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(wave * NT + t < tiles ? f.k[t][r] : 0.f, u[r], Sg[t], 0, 0, 0);
+      pin();
+      if (more) {
+        if (r < NT) load_q(Fn, f, r);
+        if (r < 3) load_rest(Fn, f, r);
+      }
+      pin();
+    }
 #pragma unroll
     for (int t = 0; t < NT; ++t) S[t] = Sg[t];
     if (k > k0) emit(k - 1, b);
   };
   Frag f[kAhead];
 #pragma unroll
-  for (int i = 0; i < kAhead; ++i) load_first(min(k0 + i, k1 - 1), f[i]);
-  x = value(k0, f[0]);
+  for (int i = 0; i < kAhead; ++i) load(min(k0 + i, k1 - 1), f[i]);
   int k = k0;
-  for (; k + kAhead <= k1; k += kAhead) {
+  for (; k + 2 * kAhead <= k1; k += kAhead) {
+#pragma unroll
+    for (int i = 0; i < kAhead; ++i) step(k + i, f[i], f[(i + kAhead - 1) % kAhead], true, i > 0 || k > k0);
+  }
+  // up to 2 kAhead - 1 chunks are left
+  const bool was = k > k0;
+  for (int j = 0; j < 2; ++j) {
 #pragma unroll
     for (int i = 0; i < kAhead; ++i) {
-      step(k + i, f[i], f[(i + 1) % kAhead]);
-      load(min(k + i + kAhead, k1 - 1), f[i]);
+      const int n = k + j * kAhead + i;
+      if (n < k1) step(n, f[i], f[(i + kAhead - 1) % kAhead], n + kAhead < k1, (n > k || was) && n - 1 + kAhead < k1);
     }
   }
-#pragma unroll
-  for (int i = 0; i < kAhead; ++i)
-    if (k + i < k1) step(k + i, f[i], f[(i + 1) % kAhead]);
   ps[k1 & 1][1][wave][lane] = ov;
   __syncthreads();
   emit(k1 - 1, k1 & 1);
@@ -564,12 +538,12 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaGeom g, DeltaIn in
   for (int t = 0; t < NT; ++t)
 #pragma unroll
     for (int r = 0; r < 4; ++r)
-      if (tile[t] < tiles) S0[(size_t)(tile[t] * 16 + 4 * g4 + r) * g.dvp] = S[t][r];
+      if (wave * NT + t < tiles) S0[(size_t)((wave * NT + t) * 16 + 4 * g4 + r) * g.dvp] = S[t][r];
 }
 
 // norm and gate: a wave per head, four of the chunk's tokens at a time; the work-groups of a segment's last chunk renew its ring
 template <typename T, int NV>
-__global__ __launch_bounds__(256) void delta_out_kernel(DeltaGeom g, DeltaIn in, const AttnSeg* __restrict__ segs, int nseg, int c0, const float* __restrict__ o,
+__global__ __launch_bounds__(256) void delta_out_kernel(DeltaGeom g, DeltaIn in, const AttnSeg* __restrict__ segs, int nseg, int c0, float* __restrict__ records,
                                                         T* __restrict__ y, int ldy) {
   const ChunkAt at = chunk_at(segs, nseg, c0 + blockIdx.x);
   if (!at.ok) return;
@@ -579,7 +553,7 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaGeom g, DeltaIn in,
 #pragma unroll
     for (int i = 0; i < NV; ++i) nw[i] = in.norm[min(lane + 64 * i, g.dv - 1)];
     const size_t row0 = at.sg.row0 + at.t0;
-    const float *src = o + row0 * g.H * g.dvp + h * g.dvp, *zr = in.z + row0 * in.ldz + in.gate + h * g.dv;
+    const float *src = factors_at(records, (size_t)h * gridDim.x + blockIdx.x, g.dkp, g.dvp).v, *zr = in.z + row0 * in.ldz + in.gate + h * g.dv;
     for (int t0 = 0; t0 < at.n; t0 += 4) {
       float x[4][NV], z[4][NV];
 #pragma unroll
@@ -587,7 +561,7 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaGeom g, DeltaIn in,
 #pragma unroll
         for (int i = 0; i < NV; ++i) {
           const int r = min(t0 + t, at.n - 1), v = min(lane + 64 * i, g.dv - 1);
-          x[t][i] = src[(size_t)r * g.H * g.dvp + v];
+          x[t][i] = src[(v >> 4) * 256 + r * 16 + (v & 15)];
           z[t][i] = zr[(size_t)r * in.ldz + v];
         }
 #pragma unroll
@@ -626,7 +600,7 @@ int check_in(const DeltaGeom& g, const DeltaIn& in) {
 bool delta_supported(const DeltaGeom& g) {
   return g.H >= 1 && g.G >= 1 && g.H % g.G == 0 && g.dk >= 1 && g.dk <= 256 && g.dv >= 1 && g.dv <= 256 && g.taps >= 1 && g.taps <= 16;
 }
-size_t delta_factor_floats(const DeltaGeom& g) { return (size_t)g.H * factor_floats(g.dkp); }
+size_t delta_chunk_floats(const DeltaGeom& g) { return (size_t)g.H * record_floats(g.dkp, g.dvp); }
 
 int launch_delta_token(const DeltaGeom& g, const DeltaIn& in, int rows, const AttnSeg* segs, void* y, int ldy, bool f32, hipStream_t s) {
   int rc = check_in(g, in);
@@ -647,11 +621,11 @@ int launch_delta_token(const DeltaGeom& g, const DeltaIn& in, int rows, const At
   return MI_OK;
 }
 
-int launch_delta_prompt(const DeltaGeom& g, const DeltaIn& in, const AttnSeg* sd, const AttnSeg* sh, int nseg, float* factors, int max_chunks,
-                        float* o, void* y, int ldy, bool f32, hipStream_t s) {
+int launch_delta_prompt(const DeltaGeom& g, const DeltaIn& in, const AttnSeg* sd, const AttnSeg* sh, int nseg, float* records, int max_chunks,
+                        void* y, int ldy, bool f32, hipStream_t s) {
   int rc = check_in(g, in);
   if (rc != MI_OK) return rc;
-  MI_CHECK(nseg >= 1 && nseg <= 65535 && factors && max_chunks >= 1 && o && y && ldy >= g.H * g.dv, "delta rule: segments / workspace");
+  MI_CHECK(nseg >= 1 && nseg <= 65535 && records && max_chunks >= 1 && y && ldy >= g.H * g.dv, "delta rule: segments / workspace");
   int chunks = 0;
   for (int i = 0; i < nseg; ++i) chunks += sh[i].n < 2 ? 0 : ceil_div(sh[i].n, kC);
   const int nvt = g.dvp / 16, nt = ceil_div(g.dkp / 16, 4);
@@ -661,11 +635,8 @@ int launch_delta_prompt(const DeltaGeom& g, const DeltaIn& in, const AttnSeg* sd
     const dim3 gf(n, g.H), gs(g.H * nvt, nseg), go(n, ceil_div(g.H, 4));
 #define MI_DF(TAPS) { \
     if (lds > 48 * 1024) { rc = ensure_dynamic_lds(reinterpret_cast<const void*>(delta_factors_kernel<TAPS>), (int)lds); if (rc != MI_OK) return rc; } \
-    hipLaunchKernelGGL((delta_factors_kernel<TAPS>), gf, dim3(256), lds, s, g, in, sd, nseg, c0, factors); \
-    if (nt == 1) hipLaunchKernelGGL((delta_scan_kernel<1, TAPS>), gs, dim3(256), 0, s, g, in, sd, nseg, c0, c0 + n, nvt, factors, o); \
-    else if (nt == 2) hipLaunchKernelGGL((delta_scan_kernel<2, TAPS>), gs, dim3(256), 0, s, g, in, sd, nseg, c0, c0 + n, nvt, factors, o); \
-    else if (nt == 3) hipLaunchKernelGGL((delta_scan_kernel<3, TAPS>), gs, dim3(256), 0, s, g, in, sd, nseg, c0, c0 + n, nvt, factors, o); \
-    else hipLaunchKernelGGL((delta_scan_kernel<4, TAPS>), gs, dim3(256), 0, s, g, in, sd, nseg, c0, c0 + n, nvt, factors, o); }
+    hipLaunchKernelGGL((delta_factors_kernel<TAPS>), gf, dim3(256), lds, s, g, in, sd, nseg, c0, records); }
+#define MI_DS(NT) hipLaunchKernelGGL((delta_scan_kernel<NT>), gs, dim3(256), 0, s, g, in.state, in.slots, sd, c0, n, nvt, records)
     switch (g.taps) {
       case 1: MI_DF(1); break;
       case 2: MI_DF(2); break;
@@ -674,9 +645,14 @@ int launch_delta_prompt(const DeltaGeom& g, const DeltaIn& in, const AttnSeg* sd
       default: MI_DF(0);
     }
 #undef MI_DF
+    if (nt == 1) MI_DS(1);
+    else if (nt == 2) MI_DS(2);
+    else if (nt == 3) MI_DS(3);
+    else MI_DS(4);
+#undef MI_DS
 #define MI_DO(NV) \
-    if (f32) hipLaunchKernelGGL((delta_out_kernel<float, NV>), go, dim3(256), 0, s, g, in, sd, nseg, c0, o, (float*)y, ldy); \
-    else hipLaunchKernelGGL((delta_out_kernel<uint16_t, NV>), go, dim3(256), 0, s, g, in, sd, nseg, c0, o, (uint16_t*)y, ldy)
+    if (f32) hipLaunchKernelGGL((delta_out_kernel<float, NV>), go, dim3(256), 0, s, g, in, sd, nseg, c0, records, (float*)y, ldy); \
+    else hipLaunchKernelGGL((delta_out_kernel<uint16_t, NV>), go, dim3(256), 0, s, g, in, sd, nseg, c0, records, (uint16_t*)y, ldy)
     if (g.dv <= 64) { MI_DO(1); } else if (g.dv <= 128) { MI_DO(2); } else { MI_DO(4); }
 #undef MI_DO
     MI_HIP(hipGetLastError());

@@ -95,9 +95,9 @@ struct Stack {
   std::vector<float*> state_at;       // every run's recurrent state, then its ring (null: none)
   int state_slots = 0;                // 0: no layer has any
   int z_ld = 0, z_gate = 0, low_ld = 0, cq_ld = 0, q2_ld = 0, delta_chunks = 0;
-  size_t delta_o_cols = 0, factor_floats = 0;
+  size_t chunk_floats = 0;
   void *cq = nullptr, *low = nullptr; // normed query latents; the inputs of the decay's and the gate's second product [2][rows][low_ld]
-  float *q2 = nullptr, *z = nullptr, *delta_o = nullptr, *factors = nullptr;
+  float *q2 = nullptr, *z = nullptr, *delta_records = nullptr;
   bool one_norm() const { return cfg.block_kind == MI_BLOCK_ONE_NORM; }
   bool sandwich() const { return cfg.block_kind == MI_BLOCK_SANDWICH; }
   void* attn_scratch = nullptr;

@@ -364,8 +364,7 @@ int delta_layer_create(mi_ctx* c, StackLayer& W) {
   MI_TRY(alloc0(c, &W.o_norm, (size_t)g.dv * 4, wb));
   S->z_ld = std::max(S->z_ld, W.a2.N + W.g2.N);
   S->low_ld = std::max(S->low_ld, std::max(W.a2.K, W.g2.K));
-  S->delta_o_cols = std::max(S->delta_o_cols, (size_t)g.H * g.dvp);
-  S->factor_floats = std::max(S->factor_floats, delta_factor_floats(g));
+  S->chunk_floats = std::max(S->chunk_floats, delta_chunk_floats(g));
   S->cat_ld = std::max(S->cat_ld, W.out.K);
   S->state_slots = c->cfg.max_num_seqs;
   return MI_OK;
@@ -573,7 +572,7 @@ void stack_destroy(mi_ctx* c) {
   free_norm(S->final_norm);
   void* ptrs[] = {S->embed, S->pos, S->x0, S->qkv_out, S->logits_pad, S->n1, S->n2, S->q, S->cat, S->pair, S->attn_scratch, S->residuals,
                   S->y, S->pair_w, S->pair_ids, S->hb, S->act, S->qa, S->lat, S->kv_x, S->kv_k, S->kv_v, S->kv_bt, S->plan,
-                  S->tickets, S->route_z, S->cq, S->low, S->q2, S->z, S->delta_o, S->factors};
+                  S->tickets, S->route_z, S->cq, S->low, S->q2, S->z, S->delta_records};
   for (void* p : ptrs) hipFree(p);
   for (float* p : S->state_at) hipFree(p);
   for (Stack::RotTable& r : S->rot) hipFree(r.t);
@@ -821,8 +820,8 @@ size_t stack_workspace_estimate(const mi_ctx* c) {
   size_t extra = 0;
   if (S->one_norm()) {
     for (const StackRun& r : S->runs) extra += state_floats(c, S->layers[r.layer]) * 4;
-    if (S->state_slots) extra += (size_t)delta_chunks(c) * S->factor_floats * 4;
-    extra += R * ((size_t)S->z_ld + S->delta_o_cols + S->q2_ld) * 4 + R * (2 * (size_t)S->low_ld + S->cq_ld) * S->elem();
+    if (S->state_slots) extra += (size_t)delta_chunks(c) * S->chunk_floats * 4;
+    extra += R * ((size_t)S->z_ld + S->q2_ld) * 4 + R * (2 * (size_t)S->low_ld + S->cq_ld) * S->elem();
     for (const StackLayer& W : S->layers) extra += W.s.mixer_kind == MI_MIX_LATENT ? (size_t)c->cfg.max_model_len * W.s.rot_dims * 4 : 0;
   }
   size_t b = 3 * R * S->ld * 4 + R * S->qkv_ld * 4 + R * (4 * (size_t)S->Kd + S->q_cols + S->cat_ld) * S->elem();
@@ -873,8 +872,7 @@ static int one_norm_alloc(mi_ctx* c) {
     S->delta_chunks = delta_chunks(c);
     MI_TRY(alloc0(c, &S->low, 2 * R * S->low_ld * S->elem(), ws));
     MI_TRY(alloc0(c, &S->z, R * S->z_ld * 4, ws));
-    MI_TRY(alloc0(c, &S->delta_o, R * S->delta_o_cols * 4, ws));
-    MI_TRY(alloc0(c, &S->factors, (size_t)S->delta_chunks * S->factor_floats * 4, ws));
+    MI_TRY(alloc0(c, &S->delta_records, (size_t)S->delta_chunks * S->chunk_floats * 4, ws));
   }
   return MI_OK;
 }
@@ -1225,7 +1223,7 @@ int one_norm_delta(mi_ctx* c, const StackLayer& W, float* state, const Batch& b)
   for (int i = 0; i < b.nseg; ++i) ones += b.segs[i].n == 1;
   const AttnSeg* segs = reinterpret_cast<const AttnSeg*>(c->d_segs);
   if (ones) MI_TRY(launch_delta_token(g, in, b.nseg, segs, S->cat, S->cat_ld, S->f32, s));
-  if (ones < b.nseg) MI_TRY(launch_delta_prompt(g, in, segs, b.segs, b.nseg, S->factors, S->delta_chunks, S->delta_o, S->cat, S->cat_ld, S->f32, s));
+  if (ones < b.nseg) MI_TRY(launch_delta_prompt(g, in, segs, b.segs, b.nseg, S->delta_records, S->delta_chunks, S->cat, S->cat_ld, S->f32, s));
   return MI_OK;
 }
 

@@ -194,11 +194,10 @@ int mi_op_delta_rule(const mi_layer_spec* spec, const float* proj, int32_t ldp, 
     for (const AttnSeg& x : segs) MI_CHECK(x.seq < seqs, "segments: sequence");
   }
   int32_t *slots, *pos;
-  float *factors, *o;
+  float* records;
   MI_TRY(mem.take(&slots, (size_t)seqs * 4, s));
   MI_TRY(mem.take(&pos, (size_t)T * 4, s));
-  MI_TRY(mem.take(&factors, (size_t)max_chunks * delta_factor_floats(g) * 4, s));
-  MI_TRY(mem.take(&o, (size_t)T * g.H * g.dvp * 4, s));
+  MI_TRY(mem.take(&records, (size_t)max_chunks * delta_chunk_floats(g) * 4, s));
   MI_HIP(hipMemcpyAsync(slots, slots_host, (size_t)seqs * 4, hipMemcpyHostToDevice, s));
   MI_HIP(hipMemcpyAsync(pos, pos_host, (size_t)T * 4, hipMemcpyHostToDevice, s));
   DeltaIn in;
@@ -209,7 +208,7 @@ int mi_op_delta_rule(const mi_layer_spec* spec, const float* proj, int32_t ldp, 
     MI_TRY(launch_delta_token(g, in, T, nullptr, out, ldo, f32 != 0, s));
   } else {
     MI_TRY(launch_delta_token(g, in, nseg, sd, out, ldo, f32 != 0, s));
-    MI_TRY(launch_delta_prompt(g, in, sd, segs.data(), nseg, factors, max_chunks, o, out, ldo, f32 != 0, s));
+    MI_TRY(launch_delta_prompt(g, in, sd, segs.data(), nseg, records, max_chunks, out, ldo, f32 != 0, s));
   }
   MI_HIP(hipStreamSynchronize(s));
   return MI_OK;

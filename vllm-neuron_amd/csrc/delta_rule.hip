@@ -10,6 +10,7 @@ namespace {
 constexpr int kC = kDeltaChunk;
 
 __device__ __forceinline__ float silu(float v) { return v * __builtin_amdgcn_rcpf(1.f + __expf(-v)); }
+__device__ __forceinline__ float gate(float v) { return __builtin_amdgcn_rcpf(1.f + __expf(-v)); }
 __device__ __forceinline__ float sigmoid(float v) { return 1.f / (1.f + expf(-v)); }
 // max(v, 0) + log(1 + w), w = exp(-|v|): the series where w is small (its first left-out term is w^5 / 5)
 __device__ __forceinline__ float softplus(float v) {
@@ -126,7 +127,7 @@ __global__ __launch_bounds__(kTokenThreads) void delta_token_kernel(DeltaGeom g,
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int v = vq * 4 + i;
-    if (v < g.dv) put1(y + (size_t)row * ldy + h * g.dv + v, o[i] * f * in.norm[v] * sigmoid(in.z[(size_t)row * in.ldz + in.gate + h * g.dv + v]));
+    if (v < g.dv) put1(y + (size_t)row * ldy + h * g.dv + v, o[i] * f * in.norm[v] * gate(in.z[(size_t)row * in.ldz + in.gate + h * g.dv + v]));
   }
 }
 
@@ -185,47 +186,85 @@ __global__ __launch_bounds__(256) void delta_factors_kernel(DeltaGeom g, DeltaIn
   const Factors F = factors_at(out, (size_t)h * gridDim.x + blockIdx.x, g.dkp, g.dvp);
   const float* ring = in.ring + (size_t)in.slots[at.sg.seq] * g.taps * C;
   const float* rows = in.proj + (size_t)(at.sg.row0 + at.t0) * in.ldp;
-  // convolutions: a thread walks one channel of q, k or v down half the chunk
-  constexpr int kHalf = kC / 2;
+  // Convolutions: a thread walks channels of q, k and v down half the chunk, kItems of them at a time; their inputs and the decays' are
+  // requested together.
+  constexpr int kHalf = kC / 2, kItems = 3, kZ = 8, NX = TAPS > 0 ? kHalf + TAPS - 1 : 1, NW = TAPS > 0 ? TAPS : 1;
   const int cols = 2 * g.dkp + g.dvp;
-  for (int i = tid; i < 2 * cols; i += 256) {
-    const int t0 = i < cols ? 0 : kHalf, col = i < cols ? i : i - cols;
-    const int part = col < g.dkp ? 0 : col < 2 * g.dkp ? 1 : 2, d = col - part * g.dkp, size = part == 2 ? g.dv : g.dk;
-    const int ch = part == 2 ? 2 * g.G * g.dk + h * g.dv + min(d, size - 1) : (part * g.G + kvh) * g.dk + min(d, size - 1);
-    float* dst = part == 2 ? F.v + (d >> 4) * 256 + (d & 15) : (part ? ks : qs) + d;
-    const int step = part == 2 ? 16 : pitch;
-    if constexpr (TAPS > 0) {
-      float x[kHalf + TAPS - 1], w[TAPS];
+  struct Item { int t0, d, ch, size; bool v; float* dst; int step; };
+  auto item = [&](int i) {
+    Item x;
+    x.t0 = i < cols ? 0 : kHalf;
+    const int col = i < cols ? i : min(i - cols, cols - 1), part = col < g.dkp ? 0 : col < 2 * g.dkp ? 1 : 2;
+    x.d = col - part * g.dkp;
+    x.v = part == 2;
+    x.size = x.v ? g.dv : g.dk;
+    x.ch = (x.v ? 2 * g.G * g.dk + h * g.dv : (part * g.G + kvh) * g.dk) + min(x.d, x.size - 1);
+    x.dst = x.v ? F.v + (x.d >> 4) * 256 + (x.d & 15) : (part ? ks : qs) + x.d;
+    x.step = x.v ? 16 : pitch;
+    return x;
+  };
+  // decays: thread = channel zd of tokens zt0, zt0 + zn, ...
+  const float decay = expf(in.a_log[h]);
+  const int zn = 256 / g.dkp, zt0 = tid / g.dkp, zd = tid - zt0 * g.dkp, zdc = min(zd, g.dk - 1);
+  const bool zin = zt0 < zn;
+  const float* zr = in.z + (size_t)(at.sg.row0 + at.t0) * in.ldz + h * g.dk;
+  const float zdt = in.dt[h * g.dk + zdc];
+  auto put_decay = [&](int t, float z) { Ls[t * pitch + zd] = zd < g.dk && t < n ? -decay * softplus(z + zdt) : 0.f; };
+  float z0[kZ];
 #pragma unroll
-      for (int k = 0; k < kHalf + TAPS - 1; ++k) {
-        const int t = t0 + k - (TAPS - 1);
-        x[k] = conv_in(in, at.sg, ring, TAPS, C, ch, at.t0 + min(t, n - 1));
+  for (int u = 0; u < kZ; ++u) z0[u] = zr[(uint32_t)min(zt0 + u * zn, n - 1) * in.ldz + zdc];
+  const bool inside = at.t0 >= TAPS - 1 && n == kC;      // every input is a row of the batch: no clamps, no ring
+  for (int base = 0; base < 2 * cols; base += kItems * 256) {
+    float x[kItems][NX], w[kItems][NW];
+    if constexpr (TAPS > 0) {
+      if (inside) {
+        const float* from = rows - (size_t)(TAPS - 1) * in.ldp;
+#pragma unroll
+        for (int p = 0; p < kItems; ++p) {
+          const Item it = item(base + p * 256 + tid);
+          uint32_t off = (uint32_t)it.t0 * in.ldp + it.ch;
+#pragma unroll
+          for (int k = 0; k < NX; ++k, off += in.ldp) x[p][k] = *reinterpret_cast<const float*>(reinterpret_cast<const unsigned char*>(from) + off * 4);
+        }
+      } else {
+#pragma unroll
+        for (int p = 0; p < kItems; ++p) {
+          const Item it = item(base + p * 256 + tid);
+#pragma unroll
+          for (int k = 0; k < NX; ++k) x[p][k] = conv_in(in, at.sg, ring, TAPS, C, it.ch, at.t0 + min(it.t0 + k - (TAPS - 1), n - 1));
+        }
       }
 #pragma unroll
-      for (int j = 0; j < TAPS; ++j) w[j] = in.conv[(size_t)j * C + ch];
+      for (int p = 0; p < kItems; ++p) {
+        const int ch = item(base + p * 256 + tid).ch;
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) w[p][j] = in.conv[(uint32_t)j * C + ch];
+      }
+    }
+#pragma unroll
+    for (int p = 0; p < kItems; ++p) {
+      const int i = base + p * 256 + tid;
+      if (i >= 2 * cols) continue;
+      const Item it = item(i);
 #pragma unroll
       for (int t = 0; t < kHalf; ++t) {
         float a = 0.f;
+        if constexpr (TAPS > 0) {
 #pragma unroll
-        for (int j = 0; j < TAPS; ++j) a = __builtin_fmaf(w[j], x[t + j], a);
-        dst[(t0 + t) * step] = t0 + t < n && d < size ? silu(a) : 0.f;
-      }
-    } else {
-      for (int t = t0; t < t0 + kHalf; ++t) {
-        float a = 0.f;
-        for (int j = 0; j < g.taps; ++j) a = __builtin_fmaf(in.conv[(size_t)j * C + ch], conv_in(in, at.sg, ring, g.taps, C, ch, at.t0 + min(t, n - 1) - (g.taps - 1 - j)), a);
-        dst[t * step] = t < n && d < size ? silu(a) : 0.f;
+          for (int j = 0; j < TAPS; ++j) a = __builtin_fmaf(w[p][j], x[p][t + j], a);
+        } else {
+          for (int j = 0; j < g.taps; ++j)
+            a = __builtin_fmaf(in.conv[(size_t)j * C + it.ch], conv_in(in, at.sg, ring, g.taps, C, it.ch, at.t0 + min(it.t0 + t, n - 1) - (g.taps - 1 - j)), a);
+        }
+        it.dst[(it.t0 + t) * it.step] = it.t0 + t < n && it.d < it.size ? silu(a) : 0.f;
       }
     }
   }
-  {
-    const float a_log = in.a_log[h];
-    const float* zr = in.z + (size_t)(at.sg.row0 + at.t0) * in.ldz + h * g.dk;
-    for (int i = tid; i < kC * g.dkp; i += 256) {
-      const int t = i / g.dkp, d = i - t * g.dkp, dc = min(d, g.dk - 1);
-      const float lg = log_decay(zr[(size_t)min(t, n - 1) * in.ldz + dc], in.dt[h * g.dk + dc], a_log);
-      Ls[t * pitch + d] = d < g.dk && t < n ? lg : 0.f;
-    }
+  if (zin) {
+#pragma unroll
+    for (int u = 0; u < kZ; ++u)
+      if (zt0 + u * zn < kC) put_decay(zt0 + u * zn, z0[u]);
+    for (int t = zt0 + kZ * zn; t < kC; t += zn) put_decay(t, zr[(uint32_t)min(t, n - 1) * in.ldz + zdc]);
   }
   if (tid < kC) bs[tid] = tid < n ? sigmoid(rows[(size_t)tid * in.ldp + in.beta + h]) : 0.f;
   __syncthreads();
@@ -541,7 +580,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaGeom g, float* __r
       if (wave * NT + t < tiles) S0[(size_t)((wave * NT + t) * 16 + 4 * g4 + r) * g.dvp] = S[t][r];
 }
 
-// norm and gate: a wave per head, four of the chunk's tokens at a time; the work-groups of a segment's last chunk renew its ring
+// norm and gate: a wave per head, eight (four) of the chunk's tokens at a time; the work-groups of a segment's last chunk renew its ring
 template <typename T, int NV>
 __global__ __launch_bounds__(256) void delta_out_kernel(DeltaGeom g, DeltaIn in, const AttnSeg* __restrict__ segs, int nseg, int c0, float* __restrict__ records,
                                                         T* __restrict__ y, int ldy) {
@@ -554,10 +593,11 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaGeom g, DeltaIn in,
     for (int i = 0; i < NV; ++i) nw[i] = in.norm[min(lane + 64 * i, g.dv - 1)];
     const size_t row0 = at.sg.row0 + at.t0;
     const float *src = factors_at(records, (size_t)h * gridDim.x + blockIdx.x, g.dkp, g.dvp).v, *zr = in.z + row0 * in.ldz + in.gate + h * g.dv;
-    for (int t0 = 0; t0 < at.n; t0 += 4) {
-      float x[4][NV], z[4][NV];
+    constexpr int TB = NV <= 2 ? 8 : 4;
+    for (int t0 = 0; t0 < at.n; t0 += TB) {
+      float x[TB][NV], z[TB][NV];
 #pragma unroll
-      for (int t = 0; t < 4; ++t)
+      for (int t = 0; t < TB; ++t)
 #pragma unroll
         for (int i = 0; i < NV; ++i) {
           const int r = min(t0 + t, at.n - 1), v = min(lane + 64 * i, g.dv - 1);
@@ -565,7 +605,7 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaGeom g, DeltaIn in,
           z[t][i] = zr[(size_t)r * in.ldz + v];
         }
 #pragma unroll
-      for (int t = 0; t < 4; ++t) {
+      for (int t = 0; t < TB; ++t) {
         float ss = 0.f;
 #pragma unroll
         for (int i = 0; i < NV; ++i) ss = __builtin_fmaf(x[t][i], lane + 64 * i < g.dv ? x[t][i] : 0.f, ss);
@@ -574,7 +614,7 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaGeom g, DeltaIn in,
 #pragma unroll
         for (int i = 0; i < NV; ++i) {
           const int v = lane + 64 * i;
-          if (v < g.dv) put1(y + (row0 + t0 + t) * ldy + h * g.dv + v, x[t][i] * f * nw[i] * sigmoid(z[t][i]));
+          if (v < g.dv) put1(y + (row0 + t0 + t) * ldy + h * g.dv + v, x[t][i] * f * nw[i] * gate(z[t][i]));
         }
       }
     }

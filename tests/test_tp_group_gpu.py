@@ -404,7 +404,7 @@ def test_exchange_inside_hipgraphs_with_device_flag_waits():
     """The exchange exactly as it will run across GPUs: no host barrier, every shard's token-generation step (publish and
     reduce kernels included) replayed from its own hipGraph, reducers waiting on device flags.  On ONE device this depends
     on how the runtime maps the two shard streams onto hardware queues: when a waiting reduce kernel lands in front of the
-    peer's publish kernel in a shared queue the wait can only end at its time bound.  Measured this round: passes in some
+    peer's publish kernel in a shared queue the wait can only end at its time bound.  Measured: passes in some
     processes, runs into the bound (a clean MI_ECOMM, never a hang) in others -- so a time-out here is reported as a skip;
     anything else (wrong sums, wrong logits, a crash) fails."""
     r = _run_concurrent_child(2, hostbar=False)

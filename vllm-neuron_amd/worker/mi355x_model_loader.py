@@ -514,7 +514,7 @@ def check_draft(stack: dict | None) -> None:
     """The draft's chained steps run one row per sequence with a catch-up row beside it; a convolution's or a recurrence's
     state would need them in order."""
     if stack is not None and (stack.get("conv_taps", 0) > 1 or has_recurrent_state(SimpleNamespace(stack=stack))):
-        raise NotImplementedError("fused speculation: a draft model with sequence state beside its KV blocks is not built")
+        raise NotImplementedError("fused speculation: a draft model with convolution or recurrent state is not built")
 
 
 def _checkpoint_shapes(path: str, cfg: dict):

@@ -52,15 +52,21 @@ struct LatentRows {
 // per head y[t, h] = W_h x[t, h]: x [T, H, K], W [H][N, K] (16 x 32 bf16 tiles or row-major fp32; K % 32 == 0, N % 16 == 0);
 // columns n < n_valid go to y[t * ldy + h * y_head + n]
 int launch_head_linear(const void* w, int H, int N, int K, const void* x, int T, void* y, int ldy, int y_head, int n_valid, bool f32, hipStream_t s);
+// sigmoid(z) on the heads' outputs: row t at z + t ld, an element per head or per element of the heads; z null: none
+struct OutGate {
+  const float* z = nullptr;
+  int ld = 0;
+  bool per_element = false;
+};
 int launch_head_linear_rows(const void* w, int H, int N, int K, const uint16_t* x, const LatentRows& rows, uint16_t* y, int ldy, int y_head,
-                            int n_valid, hipStream_t s);      // bf16, the listed rows only
+                            int n_valid, hipStream_t s, OutGate gate = OutGate());      // bf16, the listed rows only
 // ---- attention over latents, MFMA form (bf16)
 bool latent_attn_supported(const LatentGeom& g);      // rank <= 512, rotated part <= 64
 size_t latent_attn_scratch_bytes(const LatentGeom& g);
 // qa [T, H, cp] = W_uk^T q; lat [T, H, rp] scratch; out [T, ldo]: head h at column h dv
 int launch_latent_attn_rows(const LatentGeom& g, float scale, int window, const uint16_t* qa, const uint16_t* pool, int block_size,
                             const int32_t* block_table, int MB, const int32_t* pos, const LatentRows& rows, int max_ctx, const void* w_uv,
-                            uint16_t* lat, uint16_t* out, int ldo, void* scratch, hipStream_t s);
+                            uint16_t* lat, uint16_t* out, int ldo, void* scratch, hipStream_t s, OutGate gate = OutGate());
 
 // ---- prompts: keys and values of the tokens in sight written out per head, for the windowed context-encoding kernel ---------------
 // Of every segment with at least min_n rows: the latents of positions kv_first .. end, padded to whole kKvBlock rows, gathered into

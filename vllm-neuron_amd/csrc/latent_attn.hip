@@ -39,6 +39,23 @@ __device__ __forceinline__ float rotated(int i, int dims, const float2* cs, F at
   return at(i) * cs[i - half].x + at(i - half) * cs[i - half].y;
 }
 
+// elements i .. i + 3 (i % 4 == 0) of a rotated part of nr, zeros behind it; at4: four at a time, for vec (nr and the part's place
+// multiples of 4), where no pair is split by the quads of either half
+template <typename F, typename F4>
+__device__ __forceinline__ float4 rotated4(int i, int nr, int dims, const float2* cs, bool vec, F at, F4 at4) {
+  const int half = dims >> 1;
+  if (vec && (half & 3) == 0) {
+    if (i >= dims) return i < nr ? at4(i) : make_float4(0.f, 0.f, 0.f, 0.f);
+    const int j = i < half ? i : i - half;
+    const float4 u = at4(j), w = at4(j + half);
+    const float4 a = *reinterpret_cast<const float4*>(cs + j), b = *reinterpret_cast<const float4*>(cs + j + 2);    // (cos, sin) of two pairs each
+    return i < half ? make_float4(u.x * a.x - w.x * a.y, u.y * a.z - w.y * a.w, u.z * b.x - w.z * b.y, u.w * b.z - w.w * b.w)
+                    : make_float4(w.x * a.x + u.x * a.y, w.y * a.z + u.y * a.w, w.z * b.x + u.z * b.y, w.w * b.z + u.w * b.w);
+  }
+  auto one = [&](int k) { return k < nr ? rotated(k, dims, cs, at) : 0.f; };
+  return make_float4(one(i), one(i + 1), one(i + 2), one(i + 3));
+}
+
 // one latent (columns c0 .. of the row) over its root mean square times c_norm, into its pool row; 256 threads
 template <typename T>
 __device__ __forceinline__ void latent_norm_row(const QdRow& row, int c0, const LatentGeom& g, const float2* cs, const float* __restrict__ c_norm, float eps,
@@ -79,16 +96,8 @@ __global__ __launch_bounds__(256) void latent_scatter_kernel(LatentRowsIn in, Sl
     const bool vec = ((g.dk | g.nr) & 3) == 0;
     for (int d = (tid & 31) * 4; d < g.dkp; d += 128) {
       float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
-      if (vec && d >= g.dk && ((g.dims >> 1) & 3) == 0 && g.nr) {      // four pairs at a time
-        const int i = d - g.dk, half = g.dims >> 1, j = i < half ? i : i - half;
-        if (i < g.dims) {
-          const float4 u = row.at4(c0 + g.dk + j), w = row.at4(c0 + g.dk + j + half);
-          const float4 a = *reinterpret_cast<const float4*>(cs + j), b = *reinterpret_cast<const float4*>(cs + j + 2);    // (cos, sin) of two pairs each
-          v = i < half ? make_float4(u.x * a.x - w.x * a.y, u.y * a.z - w.y * a.w, u.z * b.x - w.z * b.y, u.w * b.z - w.w * b.w)
-                       : make_float4(w.x * a.x + u.x * a.y, w.y * a.z + u.y * a.w, w.z * b.x + u.z * b.y, w.w * b.z + u.w * b.w);
-        } else if (i < g.nr) {
-          v = row.at4(c0 + d);
-        }
+      if (vec && d >= g.dk && g.nr) {
+        v = rotated4(d - g.dk, g.nr, g.dims, cs, true, [&](int k) { return row.at(c0 + g.dk + k); }, [&](int k) { return row.at4(c0 + g.dk + k); });
       } else if (d + 3 >= g.dk && g.nr) {
         auto at = [&](int i) {
           if (d + i < g.dk) return row.at(c0 + d + i);
@@ -123,9 +132,19 @@ __device__ __forceinline__ RowAt latent_row(const LatentRows& r, int z) {
   return RowAt{0, 0};    // (not reached: the grid has LatentRows::rows rows)
 }
 
+// factors of the elements d .. d + 3 of head h
+__device__ __forceinline__ float4 gate4(const OutGate& gt, int row, int h, int dv, int d) {
+  if (!gt.z) return make_float4(1.f, 1.f, 1.f, 1.f);
+  const float* z = gt.z + (size_t)row * gt.ld;
+  auto f = [&](int i) { return 1.f / (1.f + expf(-z[gt.per_element ? h * dv + min(d + i, dv - 1) : h])); };
+  if (gt.per_element) return make_float4(f(0), f(1), f(2), f(3));
+  const float v = f(0);
+  return make_float4(v, v, v, v);
+}
+
 // a wave: one 16-row tile of W_h against 16 tokens
 __global__ __launch_bounds__(256) void head_linear_kernel(const uint4* __restrict__ w, int H, int NT, int KT, const uint16_t* __restrict__ x,
-                                                          LatentRows lr, uint16_t* __restrict__ y, int ldy, int y_head, int n_valid) {
+                                                          LatentRows lr, OutGate gt, uint16_t* __restrict__ y, int ldy, int y_head, int n_valid) {
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, g4 = lane >> 4, c = lane & 15;
   const int nt = blockIdx.x * 4 + wave, h = blockIdx.y, z = blockIdx.z * 16 + c, m = latent_row(lr, min(z, lr.rows - 1)).row;
   if (nt >= NT) return;
@@ -145,6 +164,8 @@ __global__ __launch_bounds__(256) void head_linear_kernel(const uint4* __restric
   if (z >= lr.rows) return;
   const int n = nt * 16 + g4 * 4;
   uint16_t* o = y + (size_t)m * ldy + (size_t)h * y_head + n;
+  const float4 f = gate4(gt, m, h, n_valid, n);
+  acc[0] *= f.x; acc[1] *= f.y; acc[2] *= f.z; acc[3] *= f.w;
   if (n + 4 <= n_valid && ((y_head | ldy) & 3) == 0) {
     put4(o, make_float4(acc[0], acc[1], acc[2], acc[3]));
   } else {
@@ -171,32 +192,34 @@ __global__ __launch_bounds__(256) void latent_token_kernel(LatentRowsIn in, Late
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, g4 = lane >> 4, c = lane & 15;
   const int NT = g.cp / 16, KT = g.dkp / 32, ntg = ceil_div(NT, 4), tt = blockIdx.x / ntg, nt = (blockIdx.x % ntg) * 4 + wave, m = tt * 16 + c;
   if (tt * 16 >= rows || nt >= NT) return;
+  const float* X = in.q + (size_t)min(m, rows - 1) * in.ldq + (size_t)h * (g.dk + g.nr);
+  uint16_t* dst = qa + ((size_t)m * g.H + h) * g.cp + nt * 16 + g4 * 4;
+  if (nt * 16 >= g.rp) {                     // the rotated part, as it is
+    if (m >= rows) return;
+    const float* X1 = X + g.dk;
+    put4(dst, rotated4(nt * 16 + g4 * 4 - g.rp, g.nr, g.dims, rot.table + (size_t)rot.pos[m] * (g.dims / 2), true, [&](int k) { return X1[k]; },
+                       [&](int k) { return *reinterpret_cast<const float4*>(X1 + k); }));
+    return;
+  }
   const u32x4_t* W = reinterpret_cast<const u32x4_t*>(w_uk) + ((size_t)h * NT + nt) * KT * 64 + lane;
-  const float* X0 = in.q + (size_t)min(m, rows - 1) * in.ldq + (size_t)h * (g.dk + g.nr);
-  const float* X = X0 + g4 * 8;
-  const float2* cs = g.nr ? rot.table + (size_t)rot.pos[min(m, rows - 1)] * (g.dims / 2) : nullptr;
-  auto turned = [&](int d) {          // four elements of the rotated part
-    auto at = [&](int i) { return rotated(d - g.dk + i, g.dims, cs, [&](int k) { return X0[g.dk + k]; }); };
-    return make_float4(at(0), at(1), at(2), at(3));
-  };
+  X += g4 * 8;
+  const int KD = ceil_div(g.dk, 32);         // (the latent's rows have zeros behind dk)
   f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
-  for (int k0 = 0; k0 < KT; k0 += 4) {       // (past the last tile: the last one's weights against zeros)
+  for (int k0 = 0; k0 < KD; k0 += 4) {       // (past the last tile: the last one's weights against zeros)
     u32x4_t a[4], x[4];
 #pragma unroll
     for (int u = 0; u < 4; ++u) {
-      a[u] = W[min(k0 + u, KT - 1) * 64];
+      a[u] = W[min(k0 + u, KD - 1) * 64];
       float4 x0 = make_float4(0.f, 0.f, 0.f, 0.f), x1 = x0;
       const int d = (k0 + u) * 32 + g4 * 8;
       if (d < g.dk) x0 = *reinterpret_cast<const float4*>(X + (k0 + u) * 32);
-      else if (d < g.dk + g.nr) x0 = turned(d);
       if (d + 4 < g.dk) x1 = *reinterpret_cast<const float4*>(X + (k0 + u) * 32 + 4);
-      else if (d + 4 < g.dk + g.nr) x1 = turned(d + 4);
       x[u] = u32x4_t{pack_bf16x2(x0.x, x0.y), pack_bf16x2(x0.z, x0.w), pack_bf16x2(x1.x, x1.y), pack_bf16x2(x1.z, x1.w)};
     }
 #pragma unroll
     for (int u = 0; u < 4; ++u) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a[u]), __builtin_bit_cast(bf16x8_t, x[u]), acc, 0, 0, 0);
   }
-  if (m < rows) put4(qa + ((size_t)m * g.H + h) * g.cp + nt * 16 + g4 * 4, make_float4(acc[0], acc[1], acc[2], acc[3]));
+  if (m < rows) put4(dst, make_float4(acc[0], acc[1], acc[2], acc[3]));
 }
 
 __global__ __launch_bounds__(64) void head_linear_f32_kernel(const float* __restrict__ w, int H, int N, int K, const float* __restrict__ x,
@@ -449,7 +472,7 @@ __global__ __launch_bounds__(256, HG == 1 ? 2 : 1) void latent_rows_kernel(Laten
 // weight tiles are requested ahead of the merge.
 template <int RW>
 __global__ __launch_bounds__(512) void latent_merge_kernel(LatentGeom g, const float* __restrict__ o_part, const float* __restrict__ ml_part, int NS,
-                                                           LatentRows lr, const uint4* __restrict__ w_uv, uint16_t* __restrict__ out, int ldo) {
+                                                           LatentRows lr, OutGate gt, const uint4* __restrict__ w_uv, uint16_t* __restrict__ out, int ldo) {
   extern __shared__ __attribute__((aligned(16))) unsigned char dsm[];
   uint16_t* os = reinterpret_cast<uint16_t*>(dsm);           // [RW][rp + 8]
   const int h = blockIdx.x, z0 = blockIdx.y * RW, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g4 = lane >> 4, c = lane & 15;
@@ -459,6 +482,8 @@ __global__ __launch_bounds__(512) void latent_merge_kernel(LatentGeom g, const f
   u32x4_t pre[PF];
 #pragma unroll
   for (int u = 0; u < PF; ++u) pre[u] = W0[min(u, KT - 1) * 64];
+  const int row = latent_row(lr, z0 + min(c, n - 1)).row;
+  const float4 gate0 = gate4(gt, row, h, g.dv, wave * 16 + g4 * 4);
   for (int i = tid; i < n * (g.rp / 4); i += 512) {
     const int r = i / (g.rp / 4), d = (i % (g.rp / 4)) * 4;
     const size_t at = ((size_t)(z0 + r) * g.H + h) * NS;
@@ -486,7 +511,6 @@ __global__ __launch_bounds__(512) void latent_merge_kernel(LatentGeom g, const f
   __syncthreads();
   const bool live = c < n;
   const uint16_t* X = os + min(c, n - 1) * pitch + g4 * 8;
-  const int row = latent_row(lr, z0 + min(c, n - 1)).row;
   for (int nt = wave; nt < NT; nt += 8) {
     const u32x4_t* W = reinterpret_cast<const u32x4_t*>(w_uv) + ((size_t)h * NT + nt) * KT * 64 + lane;
     f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
@@ -509,6 +533,8 @@ __global__ __launch_bounds__(512) void latent_merge_kernel(LatentGeom g, const f
       acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, W[kt * 64]), *reinterpret_cast<const bf16x8_t*>(X + kt * 32), acc, 0, 0, 0);
     if (!live) continue;
     const int d = nt * 16 + g4 * 4;
+    const float4 f = nt == wave ? gate0 : gate4(gt, row, h, g.dv, d);
+    acc[0] *= f.x; acc[1] *= f.y; acc[2] *= f.z; acc[3] *= f.w;
     uint16_t* o = out + (size_t)row * ldo + (size_t)h * g.dv + d;
     if (d + 4 <= g.dv && ((g.dv | ldo) & 3) == 0) {
       put4(o, make_float4(acc[0], acc[1], acc[2], acc[3]));
@@ -594,9 +620,9 @@ int launch_latent_token(const LatentRowsIn& in, int rows, const LatentGeom& g, c
 }
 
 int launch_head_linear_rows(const void* w, int H, int N, int K, const uint16_t* x, const LatentRows& rows, uint16_t* y, int ldy, int y_head,
-                            int n_valid, hipStream_t s) {
+                            int n_valid, hipStream_t s, OutGate gt) {
   MI_CHECK(H >= 1 && rows.rows >= 1 && N % 16 == 0 && K % 32 == 0 && n_valid <= N && y_head >= n_valid && ldy >= (H - 1) * y_head + n_valid, "head linear: shape");
-  hipLaunchKernelGGL(head_linear_kernel, dim3(ceil_div(N / 16, 4), H, ceil_div(rows.rows, 16)), dim3(256), 0, s, (const uint4*)w, H, N / 16, K / 32, x, rows, y, ldy, y_head, n_valid);
+  hipLaunchKernelGGL(head_linear_kernel, dim3(ceil_div(N / 16, 4), H, ceil_div(rows.rows, 16)), dim3(256), 0, s, (const uint4*)w, H, N / 16, K / 32, x, rows, gt, y, ldy, y_head, n_valid);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
@@ -617,7 +643,7 @@ size_t latent_attn_scratch_bytes(const LatentGeom& g) { return (size_t)512 * g.H
 
 int launch_latent_attn_rows(const LatentGeom& g, float scale, int window, const uint16_t* qa, const uint16_t* pool, int bs, const int32_t* bt,
                             int MB, const int32_t* pos, const LatentRows& lr, int max_ctx, const void* w_uv, uint16_t* lat, uint16_t* out, int ldo,
-                            void* scratch, hipStream_t s) {
+                            void* scratch, hipStream_t s, OutGate gt) {
   MI_CHECK(latent_attn_supported(g) && lr.rows >= 1 && lr.rows <= 65535 && bs > 0 && bs % 16 == 0 && max_ctx >= 1 && window >= 0 && ldo >= g.H * g.dv, "latent attention: shape");
   const int hgs = ceil_div(g.H, 16), max_keys = window > 0 && window < max_ctx ? window : max_ctx, tiles = ceil_div(max_keys, 64) + 1;
   // head groups that share a tile: as many as leave the chip full
@@ -644,11 +670,11 @@ int launch_latent_attn_rows(const LatentGeom& g, float scale, int window, const 
 #undef MI_LR
 #undef MI_LX
   if (rc != MI_OK) return rc;
-  if (NS == 1) return launch_head_linear_rows(w_uv, g.H, g.dvp, g.rp, lat, lr, out, ldo, g.dv, g.dv, s);
+  if (NS == 1) return launch_head_linear_rows(w_uv, g.H, g.dvp, g.rp, lat, lr, out, ldo, g.dv, g.dv, s, gt);
   const int per = g.H * lr.rows / 256, rw = per <= 1 ? 1 : per <= 2 ? 2 : per <= 4 ? 4 : 16;
   const size_t lds = (size_t)rw * (g.rp + 8) * 2;
   const dim3 grid(g.H, ceil_div(lr.rows, rw));
-#define MI_LM(RW) hipLaunchKernelGGL((latent_merge_kernel<RW>), grid, dim3(512), lds, s, g, op, ml, NS, lr, (const uint4*)w_uv, out, ldo)
+#define MI_LM(RW) hipLaunchKernelGGL((latent_merge_kernel<RW>), grid, dim3(512), lds, s, g, op, ml, NS, lr, gt, (const uint4*)w_uv, out, ldo)
   if (rw == 1) MI_LM(1);
   else if (rw == 2) MI_LM(2);
   else if (rw == 4) MI_LM(4);

@@ -988,7 +988,7 @@ int latent_attention_plain(mi_ctx* c, const StackLayer& W, const void* pool, con
 // Rows of short portions (and token generation) stay in the latent space; longer ones get the keys and values in their sight
 // written out per head, which costs a matrix product over those tokens and then a quarter of the attention arithmetic or less.
 constexpr int kLatentRowsBelow = 64;
-int latent_attention(mi_ctx* c, const StackLayer& W, const uint16_t* pool, const Batch& b) {
+int latent_attention(mi_ctx* c, const StackLayer& W, const uint16_t* pool, const Batch& b, const OutGate& gate = OutGate()) {
   Stack* S = c->stack;
   const mi_model_config& k = c->cfg;
   const LatentGeom& g = W.lg;
@@ -1009,7 +1009,7 @@ int latent_attention(mi_ctx* c, const StackLayer& W, const uint16_t* pool, const
     if (!b.decode || !latent_token_supported(g))   // (token generation: done with the scatter)
       MI_TRY(launch_head_linear_rows(W.w_uk, g.H, g.cp, g.dkp, q, lr, qa, g.H * g.cp, g.cp, g.cp, s));
     MI_TRY(launch_latent_attn_rows(g, W.s.scale, W.s.window, qa, pool, k.block_size, c->d_bt, b.MB, c->d_pos, lr, k.max_model_len, W.w_uv,
-                                   reinterpret_cast<uint16_t*>(S->lat), out, S->cat_ld, S->attn_scratch, s));
+                                   reinterpret_cast<uint16_t*>(S->lat), out, S->cat_ld, S->attn_scratch, s, gate));
   }
   const AttnSpec a{W.kvg, W.s.scale, W.s.window, nullptr, 0, 0};
   uint16_t *kk = reinterpret_cast<uint16_t*>(S->kv_k), *vv = reinterpret_cast<uint16_t*>(S->kv_v);
@@ -1166,7 +1166,7 @@ int one_norm_latent(mi_ctx* c, const StackLayer& W, size_t kv_at, const Batch& b
   if (W.s.q_rank) {
     if (runs_other(c)) {
       Scope sc(c, MI_K_OTHER);
-      MI_TRY(launch_columns(S->qkv_out, W.qkv.N, W.col_q, W.s.q_rank, W.q_norm, S->cfg.norm_eps, b.rows, S->cq, W.uq.K, S->f32, s));
+      MI_TRY(launch_columns(S->qkv_out, W.qkv.N, {W.col_q, W.s.q_rank, W.q_norm, S->cq}, {}, S->cfg.norm_eps, b.rows, W.uq.K, S->f32, s));
     }
     EpiArgs u{};
     u.out_f32 = S->q2; u.ld_out = W.uq.N;
@@ -1183,8 +1183,10 @@ int one_norm_latent(mi_ctx* c, const StackLayer& W, size_t kv_at, const Batch& b
     else
       MI_TRY(launch_latent_scatter(in, b.rows, g, rot, W.c_norm, S->cfg.norm_eps, c->d_slots, c->cfg.block_size, S->q, pool, S->f32, s));
   }
-  MI_TRY(W.fast() ? latent_attention(c, W, reinterpret_cast<const uint16_t*>(pool), b) : latent_attention_plain(c, W, pool, b));
-  if (W.s.out_gate == MI_GATE_NONE || !runs_other(c)) return MI_OK;
+  // (token generation: the gate goes onto the heads' outputs before they are rounded)
+  const OutGate gate{b.decode && W.fast() && W.s.out_gate != MI_GATE_NONE ? S->qkv_out + W.col_g : nullptr, W.qkv.N, W.s.out_gate == MI_GATE_ELEMENT};
+  MI_TRY(W.fast() ? latent_attention(c, W, reinterpret_cast<const uint16_t*>(pool), b, gate) : latent_attention_plain(c, W, pool, b));
+  if (W.s.out_gate == MI_GATE_NONE || gate.z || !runs_other(c)) return MI_OK;
   Scope sc(c, MI_K_OTHER);
   return launch_gate_rows(S->cat, S->cat_ld, b.rows, g.H, g.dv, S->qkv_out + W.col_g, W.qkv.N, W.s.out_gate == MI_GATE_ELEMENT, S->f32, s);
 }
@@ -1199,8 +1201,8 @@ int one_norm_delta(mi_ctx* c, const StackLayer& W, float* state, const Batch& b)
   void* low2 = reinterpret_cast<unsigned char*>(S->low) + (size_t)c->max_rows * S->low_ld * S->elem();
   if (runs_other(c)) {
     Scope sc(c, MI_K_OTHER);
-    MI_TRY(launch_columns(S->qkv_out, W.qkv.N, W.col_a, W.s.decay_rank, nullptr, 0.f, b.rows, S->low, S->low_ld, S->f32, s));
-    MI_TRY(launch_columns(S->qkv_out, W.qkv.N, W.col_g, W.s.gate_rank, nullptr, 0.f, b.rows, low2, S->low_ld, S->f32, s));
+    MI_TRY(launch_columns(S->qkv_out, W.qkv.N, {W.col_a, W.s.decay_rank, nullptr, S->low}, {W.col_g, W.s.gate_rank, nullptr, low2}, 0.f, b.rows, S->low_ld,
+                          S->f32, s));
   }
   const int ldz = W.a2.N + W.g2.N;
   EpiArgs z{};

@@ -53,7 +53,8 @@ int launch_conv_rows(const void* h, const ConvState& conv, const AttnSeg* segs_d
                      void* y, int ldy, bool f32, hipStream_t s);
 
 // y [T, ldy] = columns col .. col + n of x [T, ld] fp32 in the compute type, zeros behind them; w [n]: over their root mean square, times w
-int launch_columns(const float* x, int ld, int col, int n, const float* w, float eps, int T, void* y, int ldy, bool f32, hipStream_t s);
+struct Columns { int col = 0, n = 0; const float* w = nullptr; void* y = nullptr; };      // w null: no norm
+int launch_columns(const float* x, int ld, Columns a, Columns b, float eps, int T, int ldy, bool f32, hipStream_t s);   // b.y null: a alone
 // y[t, h dv + d] *= sigmoid(g[t, ...]): one gate per head, or (per_element) per element; g [T, ldg] fp32, y [T, ldy] in the compute type
 int launch_gate_rows(void* y, int ldy, int T, int H, int dv, const float* g, int ldg, bool per_element, bool f32, hipStream_t s);
 // dst = src + offset

@@ -407,12 +407,32 @@ __global__ __launch_bounds__(256) void conv_rows_kernel(const T* __restrict__ hi
 }
 
 template <typename T>
-__global__ __launch_bounds__(256) void columns_kernel(const float* __restrict__ x, int ld, int n, const float* __restrict__ w, float eps,
-                                                      T* __restrict__ y, int ldy) {
+__global__ __launch_bounds__(256) void columns_kernel(const float* __restrict__ x, int ld, Columns first, Columns second, float eps, int ldy) {
   __shared__ float red[4];
-  const float* src = x + (size_t)blockIdx.x * ld;
-  const int tid = threadIdx.x;
+  const Columns k = blockIdx.y ? second : first;
+  const int tid = threadIdx.x, n = k.n;
+  const float *src = x + (size_t)blockIdx.x * ld + k.col, *w = k.w;
+  T* y = reinterpret_cast<T*>(k.y);
   float f = 1.f;
+  if (((n | k.col | ld) & 3) == 0 && ldy <= 2048) {      // the row in registers
+    float4 v[2], u[2];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int d = (i * 256 + tid) * 4;
+      const bool in = d < n;
+      v[i] = in ? *reinterpret_cast<const float4*>(src + d) : make_float4(0.f, 0.f, 0.f, 0.f);
+      u[i] = in && w ? make_float4(w[d], w[d + 1], w[d + 2], w[d + 3]) : make_float4(1.f, 1.f, 1.f, 1.f);
+      ss += (v[i].x * v[i].x + v[i].y * v[i].y) + (v[i].z * v[i].z + v[i].w * v[i].w);
+    }
+    if (w) f = 1.0f / sqrtf(block_sum(ss, red) / (float)n + eps);
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int d = (i * 256 + tid) * 4;
+      if (d < ldy) put4(y + (size_t)blockIdx.x * ldy + d, v[i].x * f * u[i].x, v[i].y * f * u[i].y, v[i].z * f * u[i].z, v[i].w * f * u[i].w);
+    }
+    return;
+  }
   if (w) {
     float ss = 0.f;
     for (int d = tid; d < n; d += 256) ss = __builtin_fmaf(src[d], src[d], ss);
@@ -425,9 +445,31 @@ __global__ __launch_bounds__(256) void columns_kernel(const float* __restrict__ 
 }
 __device__ __forceinline__ void gate1(uint16_t* p, float g) { *p = f32_to_bf16(bf16_to_f32(*p) * g); }
 __device__ __forceinline__ void gate1(float* p, float g) { *p *= g; }
+__device__ __forceinline__ void gate_quad(uint16_t* p, float4 g) {
+  const uint2 x = *reinterpret_cast<const uint2*>(p);
+  put4(p, bf16_to_f32((uint16_t)x.x) * g.x, bf16_to_f32((uint16_t)(x.x >> 16)) * g.y, bf16_to_f32((uint16_t)x.y) * g.z, bf16_to_f32((uint16_t)(x.y >> 16)) * g.w);
+}
+__device__ __forceinline__ void gate_quad(float* p, float4 g) {
+  const float4 x = *reinterpret_cast<const float4*>(p);
+  put4(p, x.x * g.x, x.y * g.y, x.z * g.z, x.w * g.w);
+}
 template <typename T, bool ELEM>
 __global__ __launch_bounds__(256) void gate_rows_kernel(T* __restrict__ y, int ldy, int n, int dv, const float* __restrict__ g, int ldg) {
   const int t = blockIdx.x;
+  if (((n | dv | ldy | ldg) & 3) == 0) {
+    for (int i = (blockIdx.y * 256 + threadIdx.x) * 4; i < n; i += gridDim.y * 1024) {
+      auto f = [&](float z) { return 1.f / (1.f + expf(-z)); };
+      T* p = y + (size_t)t * ldy + i;
+      if constexpr (ELEM) {
+        const float4 z = *reinterpret_cast<const float4*>(g + (size_t)t * ldg + i);
+        gate_quad(p, make_float4(f(z.x), f(z.y), f(z.z), f(z.w)));
+      } else {
+        const float v = f(g[(size_t)t * ldg + i / dv]);
+        gate_quad(p, make_float4(v, v, v, v));
+      }
+    }
+    return;
+  }
   for (int i = blockIdx.y * 256 + threadIdx.x; i < n; i += gridDim.y * 256)
     gate1(y + (size_t)t * ldy + i, 1.f / (1.f + expf(-g[(size_t)t * ldg + (ELEM ? i : i / dv)])));
 }
@@ -683,10 +725,13 @@ int launch_conv_rows(const void* h, const ConvState& conv, const AttnSeg* sd, co
   return MI_OK;
 }
 
-int launch_columns(const float* x, int ld, int col, int n, const float* w, float eps, int T, void* y, int ldy, bool f32, hipStream_t s) {
-  MI_CHECK(T >= 1 && n >= 1 && col >= 0 && ld >= col + n && ldy >= n && ldy % 4 == 0, "columns: strides");
-  if (f32) hipLaunchKernelGGL((columns_kernel<float>), dim3(T), dim3(256), 0, s, x + col, ld, n, w, eps, (float*)y, ldy);
-  else hipLaunchKernelGGL((columns_kernel<uint16_t>), dim3(T), dim3(256), 0, s, x + col, ld, n, w, eps, (uint16_t*)y, ldy);
+int launch_columns(const float* x, int ld, Columns a, Columns b, float eps, int T, int ldy, bool f32, hipStream_t s) {
+  const bool two = b.y != nullptr;
+  MI_CHECK(T >= 1 && a.y && a.n >= 1 && a.col >= 0 && ld >= a.col + a.n && ldy >= a.n && ldy % 4 == 0, "columns: strides");
+  MI_CHECK(!two || (b.n >= 1 && b.col >= 0 && ld >= b.col + b.n && ldy >= b.n), "columns: strides");
+  const dim3 grid(T, two ? 2 : 1);
+  if (f32) hipLaunchKernelGGL((columns_kernel<float>), grid, dim3(256), 0, s, x, ld, a, b, eps, ldy);
+  else hipLaunchKernelGGL((columns_kernel<uint16_t>), grid, dim3(256), 0, s, x, ld, a, b, eps, ldy);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
@@ -694,7 +739,7 @@ int launch_columns(const float* x, int ld, int col, int n, const float* w, float
 int launch_gate_rows(void* y, int ldy, int T, int H, int dv, const float* g, int ldg, bool per_element, bool f32, hipStream_t s) {
   const int n = H * dv;
   MI_CHECK(T >= 1 && H >= 1 && dv >= 1 && ldy >= n && ldg >= (per_element ? n : H), "gate rows: strides");
-  const dim3 grid(T, std::min(ceil_div(n, 256), 16));
+  const dim3 grid(T, std::min(ceil_div(n, 1024), 16));
   if (f32 && per_element) hipLaunchKernelGGL((gate_rows_kernel<float, true>), grid, dim3(256), 0, s, (float*)y, ldy, n, dv, g, ldg);
   else if (f32) hipLaunchKernelGGL((gate_rows_kernel<float, false>), grid, dim3(256), 0, s, (float*)y, ldy, n, dv, g, ldg);
   else if (per_element) hipLaunchKernelGGL((gate_rows_kernel<uint16_t, true>), grid, dim3(256), 0, s, (uint16_t*)y, ldy, n, dv, g, ldg);

@@ -94,19 +94,21 @@ typedef struct mi_model_config {
 enum { MI_TP_TRANSPORT_P2P = 0, MI_TP_TRANSPORT_RCCL = 1 };
 
 /* ---- layer-stack decoders: a decoder given layer by layer, every size and constant a parameter ----
- * (Vimesun, Rapodra and Bokulorn are such designs; the worker's model registry fills this from their config.json.)
+ * (Vimesun, Rapodra, Bokulorn and Nusovik are such designs; the worker's model registry fills this from their config.json.)
  *     x = embed_scale embed[token] (+ pos[position])          fp32 residual stream
+ *         pos_base > 0: + sin / cos of position * pos_base^(-2 i / width) at elements 2 i / 2 i + 1
  *     block MI_BLOCK_PARALLEL:  x <- x + residual_mult (mixer(norm1 x) + ff(norm2 x))     both of the same x
  *     block MI_BLOCK_SANDWICH:  x <- x + norm1b(mixer(C1(norm1 x))); x <- x + norm2b(ff(C2(norm2 x)))
  *             C(h) = h + causal convolution of h over time, conv_taps taps per channel; the last conv_taps - 1 inputs h
  *             are part of a sequence's state
  *     block MI_BLOCK_ONE_NORM:  h = norm1 x;  x <- x + mixer(h) + ff(h)
+ *     block MI_BLOCK_POST_NORM: x <- x + norm1(mixer(x));  x <- x + norm2(ff(x))
  *     norms:  norm_groups = 0: layer norm with weight and bias; else RMS norm of norm_groups equal parts, each over its
  *             own sqrt(mean square + norm_eps), times a weight (norm_offset = 1: times 1 + weight, also the final norm)
  *     loop:   layers loop_start .. loop_stop - 1 run loop_times times in a row with the same weights, each pass with a
  *             KV pool of its own; ahead of a pass's first layer  x <- W_in [x ; embedding output]
  *     weights_of >= 0: the layer has no tensors of its own, it runs that other layer's with a cache and state of its own
- *     logits = head final_norm(x); logit_softcap > 0: softcap tanh(logits / softcap)
+ *     logits = logit_scale head final_norm(x); logit_softcap > 0: softcap tanh(logits / softcap)
  * Mixers: MI_MIX_ATTENTION, grouped heads with K / V pools; MI_MIX_LATENT, per head k = W_uk c, v = W_uv c of a cached latent
  *     c = RMSnorm(W_dkv h) [kv_rank]; kv_from >= 0: the latents of that earlier layer instead of own ones.
  *     q_rank > 0: queries q = W_uq RMSnorm(W_dq h) [q_rank] instead of W_q h.  rot_dim > 0: a head's query has rot_dim more
@@ -119,6 +121,18 @@ enum { MI_TP_TRANSPORT_P2P = 0, MI_TP_TRANSPORT_RCCL = 1 };
  *     softplus(W_a2 W_a1 h + dt_bias)) (decay_rank rows in W_a1);  S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q;
  *     output W_o (RMSnorm(o) sigmoid(W_g2 W_g1 h)) (gate_rank rows in W_g1).  Everything fp32 but the projections.  S and the
  *     last inputs of the convolution live in a state slot per sequence (seq_ids of the model calls).
+ *   MI_MIX_ATTENTION in post-norm blocks: qk_norm, q and k heads over sqrt(mean square + eps) times a weight per element; qk_bias, biases of
+ *     their projections; keys_as_values, no W_v: a value is the key as projected (ahead of its norm); chunk > 0: a query sees keys of its own
+ *     chunk of that many positions; distance_bias MI_BIAS_TABLE, rel[bucket(i - j), head] joins the score, bucket(n) = n below rel_rows / 2, else
+ *     min(rel_rows - 1, rel_rows / 2 + floor(ln(n / (rel_rows / 2)) / ln(rel_far / (rel_rows / 2)) (rel_rows - rel_rows / 2)));
+ *     softmax_sink MI_SINK_LEARNED, exp(sink[head]) in the denominator; out_gate MI_GATE_HEAD.  beside_kind MI_MIX_SSD: a second mixer of the same x
+ *     beside it, the result mix_mult attention + beside_mult second.
+ *   MI_MIX_SSD (Mamba-2), ssm_heads heads of ssm_dim with a state of ssm_state x ssm_dim each, B and C shared by ssm_groups groups of heads: W_in x =
+ *     [z | x | B | C | dt]; x, B, C through a causal convolution of conv_taps taps with bias and silu; dt = softplus(dt + dt_bias);
+ *     S <- exp(-exp(A_log) dt) S + dt B x^T;  y = S^T C + D x;  y silu(z) in ssm_parts equal parts over their root mean square, times norm; W_o.
+ *   MI_MIX_SCAN (Mamba), ssm_inner channels with ssm_state states each: W_in x = [x | z]; x through the convolution and silu; W_x x = [low, dt_rank | B |
+ *     C]; dt = softplus(W_dt low + bias) per channel; S <- exp(-exp(A_log) dt) S + dt x B;  y = sum S C + D x;  W_o (y silu(z)).
+ *     States and convolution inputs of both live in the sequence's slot, in fp32.
  * Feed-forwards: MI_FF_RELU2 down(max(up x, 0)^2); MI_FF_GLU down(act(gate x, up x)); MI_FF_MOE the softmax-weighted sum of the
  *     experts_top experts with the largest router logits (W_router x + b), each down(act(gate x, up x)).
  *     router_score MI_ROUTE_SIGMOID: s = sigmoid(W_router x); choice scores s + correction; the experts lie in router_groups equal
@@ -126,14 +140,19 @@ enum { MI_TP_TRANSPORT_P2P = 0, MI_TP_TRANSPORT_RCCL = 1 };
  * Gated activations: MI_ACT_SILU g sigmoid(g) u; MI_ACT_SWISH_CLIP, g = min(g, limit), u within +-limit: g sigmoid(alpha g) (u + 1).
  * MI_ACT_RELU2 (experts): no gate, max(up x, 0)^2.
  * Built: parallel blocks of MI_MIX_ATTENTION with layer norms, sandwich blocks of MI_MIX_LATENT with RMS norms and no loop,
- * one-norm blocks of MI_MIX_LATENT (every earlier token in sight) and MI_MIX_DELTA with RMS norms, experts or no feed-forward and no loop.
+ * one-norm blocks of MI_MIX_LATENT (every earlier token in sight) and MI_MIX_DELTA with RMS norms, experts or no feed-forward and no loop,
+ * post-norm blocks of MI_MIX_ATTENTION (alone or beside MI_MIX_SSD) and MI_MIX_SCAN with RMS norms, MI_FF_RELU2 or no feed-forward and no loop.
  * Tensor names ("l<i>." = layer i): embed, pos, loop.in, l<i>.norm1(.b), l<i>.norm2(.b), l<i>.mix.{q,k,v,o},
  * l<i>.mlp.{up,down}, final.norm(.b), head; sandwich blocks: l<i>.norm1, .norm1b, .norm2, .norm2b, .canon1, .canon2
  * [width, taps], l<i>.mix.{q,dkv,dkv.norm,uk,uv,o}, l<i>.mlp.{gate,up,down}, l<i>.mlp.router(.b), l<i>.mlp.e<n>.{gate,up,down};
  * one-norm blocks: l<i>.norm1, l<i>.mix.{dq,dq.norm,uq | q}, l<i>.mix.{dkv,dkv.norm,uk,uv,g,o}, or l<i>.mix.{q,k,v,q.conv,k.conv,v.conv,
- * b,A_log,a1,a2,dt_bias,g1,g2,norm,o}, l<i>.mlp.router, .correction (or .router.b), l<i>.mlp.e<n>.{gate,up,down}. */
-enum { MI_BLOCK_PARALLEL = 0, MI_BLOCK_SANDWICH = 1, MI_BLOCK_ONE_NORM = 2 };
-enum { MI_MIX_ATTENTION = 0, MI_MIX_LATENT = 1, MI_MIX_DELTA = 2 };
+ * b,A_log,a1,a2,dt_bias,g1,g2,norm,o}, l<i>.mlp.router, .correction (or .router.b), l<i>.mlp.e<n>.{gate,up,down};
+ * post-norm blocks: l<i>.norm1, .norm2, l<i>.mlp.{up,down}, l<i>.mix.{q,k,v,q.b,k.b,q.norm,k.norm,rel,sink,g,o} (those the layer has; beside a second
+ * mixer l<i>.mix.left.*, and l<i>.mix.right.{in,conv,conv.b,dt_bias,A_log,D,norm,o}), or l<i>.mix.{in,conv,conv.b,x,dt,dt.b,A_log,D,o}. */
+enum { MI_BLOCK_PARALLEL = 0, MI_BLOCK_SANDWICH = 1, MI_BLOCK_ONE_NORM = 2, MI_BLOCK_POST_NORM = 3 };
+enum { MI_MIX_ATTENTION = 0, MI_MIX_LATENT = 1, MI_MIX_DELTA = 2, MI_MIX_SCAN = 3, MI_MIX_SSD = 4 };
+enum { MI_BIAS_NONE = 0, MI_BIAS_SLOPE = 1, MI_BIAS_TABLE = 2 };
+enum { MI_SINK_NONE = 0, MI_SINK_ONE = 1, MI_SINK_LEARNED = 2 };
 enum { MI_FF_NONE = 0, MI_FF_RELU2 = 1, MI_FF_GLU = 2, MI_FF_MOE = 3 };
 enum { MI_ACT_SILU = 0, MI_ACT_SWISH_CLIP = 1, MI_ACT_RELU2 = 2 };
 enum { MI_GATE_NONE = 0, MI_GATE_HEAD = 1, MI_GATE_ELEMENT = 2 };
@@ -143,8 +162,8 @@ typedef struct mi_layer_spec {
   int32_t window;         /* a query sees keys with 0 <= i - j < window; 0 = every earlier token */
   float scale;            /* of q . k */
   int32_t qk_unit_norm;   /* q and k heads divided by sqrt(mean square + norm_eps) */
-  int32_t distance_bias;  /* 2^(-8 (h + 1) / num_heads) (i - j) taken off the score of head h */
-  int32_t softmax_sink;   /* one added to the softmax denominator */
+  int32_t distance_bias;  /* MI_BIAS_*; SLOPE: 2^(-8 (h + 1) / num_heads) (i - j) taken off the score of head h */
+  int32_t softmax_sink;   /* MI_SINK_*; ONE: one added to the softmax denominator */
   int32_t ff_kind, ff_size;   /* ff_size: of one expert where there are experts */
   int32_t mixer_kind;
   int32_t kv_rank, kv_from;   /* MI_MIX_LATENT; kv_from = -1: own latents */
@@ -157,7 +176,13 @@ typedef struct mi_layer_spec {
   int32_t rot_dim, rot_dims;
   float rot_base;
   int32_t out_gate;           /* MI_GATE_* */
-  int32_t conv_taps, decay_rank, gate_rank;   /* MI_MIX_DELTA */
+  int32_t conv_taps, decay_rank, gate_rank;   /* MI_MIX_DELTA (conv_taps: MI_MIX_SCAN and MI_MIX_SSD too) */
+  int32_t qk_norm, qk_bias, keys_as_values, chunk, rel_rows;   /* post-norm blocks, MI_MIX_ATTENTION */
+  float rel_far;
+  int32_t beside_kind;        /* 0 or MI_MIX_SSD */
+  float mix_mult, beside_mult;
+  int32_t ssm_state, ssm_heads, ssm_dim, ssm_groups, ssm_parts;   /* MI_MIX_SSD (ssm_state: MI_MIX_SCAN too) */
+  int32_t ssm_inner, dt_rank;                                      /* MI_MIX_SCAN */
 } mi_layer_spec;
 typedef struct mi_stack_config {
   int32_t num_layers;
@@ -171,10 +196,11 @@ typedef struct mi_stack_config {
   float logit_softcap;     /* 0 = none */
   int32_t state_lookahead; /* sandwich blocks: a step may write this many positions behind the last accepted one (speculation: k - 1) */
   float embed_scale, norm_offset;
+  float pos_base, logit_scale;   /* post-norm blocks: pos_base 0 = no sinusoidal positions; logit_scale 1 elsewhere */
 } mi_stack_config;
 
 const char* mi_last_error(void);
-int mi_version(void);   /* 7 = this header (+ one-norm blocks, recurrent mixers and their state slots: seq_ids of mi_forward_chunked / mi_forward_rows); 6 (+ sandwich blocks, latent attention, experts in mi_layer_spec / mi_stack_config and their mi_op_*); 5 (+ mi_ctx_create_stack, mi_forward_rows, mi_layer_residuals, mi_op_* of the stack kernels); 4 (+ mi_tp_plan, mi_tp_info); 3 lacked them; 2 lacked tp_device_ids / tp_transport / MI_TP_ALL_RANKS; 1 lacked mi_forward_tokens, mi_op_sample, mi_tp_init_transport */
+int mi_version(void);   /* 8 = this header (+ post-norm blocks, chunks / distance tables / learned sinks, selective scan and state-space duality); 7 (+ one-norm blocks, recurrent mixers and their state slots: seq_ids of mi_forward_chunked / mi_forward_rows); 6 (+ sandwich blocks, latent attention, experts in mi_layer_spec / mi_stack_config and their mi_op_*); 5 (+ mi_ctx_create_stack, mi_forward_rows, mi_layer_residuals, mi_op_* of the stack kernels); 4 (+ mi_tp_plan, mi_tp_info); 3 lacked them; 2 lacked tp_device_ids / tp_transport / MI_TP_ALL_RANKS; 1 lacked mi_forward_tokens, mi_op_sample, mi_tp_init_transport */
 
 int mi_ctx_create(const mi_model_config* cfg, mi_ctx** out);
 /* The same context around a layer stack.  Of cfg only the serving fields are read (pool, batch, buckets, device, graphs);
@@ -475,6 +501,38 @@ int mi_op_delta_rule(const mi_layer_spec* spec, const float* proj, int32_t ldp, 
                      const float* a_log, const float* dt, const float* norm, float eps, float* state, float* ring, int32_t num_slots,
                      const int32_t* slots_host, const int32_t* pos_host, const int32_t* segs_host, int32_t nseg, int32_t T, int32_t max_chunks,
                      void* out, int32_t ldo, int32_t f32, void* stream);
+/* ---- kernels of the post-norm blocks (device pointers but those named host; segs_host, slots_host as above, nseg = 0: token generation) ----
+ * resid [T, ld] = scale table[ids[t]] + sinusoid of pos[t] (base pos_base); out [T, ldy]: the same in the compute type */
+int mi_op_embed_sinusoid(const int32_t* ids, const int32_t* pos, const void* table, float scale, float pos_base, int32_t T, int32_t D, int32_t ld,
+                         float* resid, void* out, int32_t ldy, int32_t f32, void* stream);
+/* mi_op_qkv_scatter with biases [H dk + G dk], norm weights [dk] (any may be NULL) and spec's qk_norm / keys_as_values */
+int mi_op_head_scatter(const float* qkv, int32_t ldq, int32_t T, const mi_layer_spec* spec, const float* bias, const float* q_norm, const float* k_norm,
+                       float eps, const int32_t* slots, int32_t block_size, void* q, void* kpool, void* vpool, int32_t f32, void* stream);
+/* mi_op_window_attn with spec's chunk, sinks [H] (NULL: spec's softmax_sink is a score of 0), rel [rel_rows, H] (NULL: no bias), and the heads' outputs
+ * times mult sigmoid(gate [T, ldg]) (NULL: mult alone) */
+int mi_op_chunk_attn(const mi_layer_spec* spec, const float* sinks, const float* rel, const float* gate, int32_t ldg, float mult, const void* q,
+                     const void* kpool, const void* vpool, int32_t block_size, const int32_t* block_table, int32_t MB, const int32_t* pos,
+                     const int32_t* ctx_lens, const int32_t* segs_host, int32_t nseg, int32_t T, int32_t max_ctx, void* out, int32_t ldo, int32_t f32,
+                     int32_t path, void* stream);
+/* y [T, ldy] = silu(bias + causal convolution of x [T, ldx] over C channels); w [taps][C] (last row: the token itself), ring [slots][taps][C] */
+int mi_op_short_conv(const float* x, int32_t ldx, const float* w, const float* b, int32_t C, int32_t taps, float* ring, int32_t num_slots,
+                     const int32_t* slots_host, const int32_t* pos_host, const int32_t* segs_host, int32_t nseg, int32_t T, void* y, int32_t ldy,
+                     int32_t f32, void* stream);
+/* Selective scan (spec: MI_MIX_SCAN).  x [T, ldx] compute type; low [T, ldl] fp32: dt's low-rank input at column 0, B at col_b, C at col_c; w_dt
+ * [inner, dt_rank], dt_bias, a_log [inner, state], d fp32; z [T, ldz]; state [num_slots][inner][padded state].  y [T, ldy] compute type */
+int mi_op_scan(const mi_layer_spec* spec, const void* x, int32_t ldx, const float* low, int32_t ldl, int32_t col_b, int32_t col_c, const float* w_dt,
+               const float* dt_bias, const float* a_log, const float* d, const float* z, int32_t ldz, float* state, int32_t num_slots,
+               const int32_t* slots_host, const int32_t* pos_host, const int32_t* segs_host, int32_t nseg, int32_t T, void* y, int32_t ldy, int32_t f32,
+               void* stream);
+int32_t mi_op_scan_state(int32_t state);    /* the padded state */
+/* State-space duality (spec: MI_MIX_SSD).  xbc [T, ldx] compute type: [x | B | C] behind the convolution; dt [T, ldt]; state [num_slots][H]
+ * [pad16(state)][pad16(dim)]; max_chunks: chunks of 64 tokens in memory at a time.  y [T, ldy] fp32, ahead of gate and norm */
+int mi_op_ssd(const mi_layer_spec* spec, const void* xbc, int32_t ldx, const float* dt, int32_t ldt, const float* dt_bias, const float* a_log, const float* d,
+              float* state, int32_t num_slots, const int32_t* slots_host, const int32_t* pos_host, const int32_t* segs_host, int32_t nseg, int32_t T,
+              int32_t max_chunks, float* y, int32_t ldy, int32_t f32, void* stream);
+/* out [T, ldo] = y silu(z), in `parts` equal parts over their root mean square, times w [n] */
+int mi_op_gated_norm(const float* y, int32_t ldy, const float* z, int32_t ldz, const float* w, int32_t n, int32_t parts, float eps, int32_t T, void* out,
+                     int32_t ldo, int32_t f32, void* stream);
 /* Latent attention of a ragged batch over that pool: uk [H dk, rank], uv [H dv, rank] fp32.  path: 1 plain, 2 rows in the latent space,
  * 3 keys and values written out (segments of two rows and more).  out [T, H v_dim] (row stride ldo). */
 int mi_op_latent_attn(const mi_layer_spec* spec, const float* uk, const float* uv, const void* q, const void* pool, int32_t block_size,

@@ -14,7 +14,7 @@ import os
 
 import torch  # noqa: F401  (must precede CDLL, see module docstring)
 
-from ._stack_enums import MI_ACT, MI_BLOCK, MI_FF, MI_GATE, MI_MIX, MI_ROUTE  # noqa: F401
+from ._stack_enums import MI_ACT, MI_BIAS, MI_BLOCK, MI_FF, MI_GATE, MI_MIX, MI_ROUTE, MI_SINK  # noqa: F401
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 # MI355X_VLLM_LIB points at another build of the same library (A/B measurements)
@@ -66,7 +66,11 @@ class MiLayerSpec(C.Structure):
                 ("ff_alpha", C.c_float), ("experts", C.c_int32), ("experts_top", C.c_int32),
                 ("router_score", C.c_int32), ("router_groups", C.c_int32), ("router_keep", C.c_int32), ("weights_of", C.c_int32),
                 ("q_rank", C.c_int32), ("rot_dim", C.c_int32), ("rot_dims", C.c_int32), ("rot_base", C.c_float),
-                ("out_gate", C.c_int32), ("conv_taps", C.c_int32), ("decay_rank", C.c_int32), ("gate_rank", C.c_int32)]
+                ("out_gate", C.c_int32), ("conv_taps", C.c_int32), ("decay_rank", C.c_int32), ("gate_rank", C.c_int32),
+                ("qk_norm", C.c_int32), ("qk_bias", C.c_int32), ("keys_as_values", C.c_int32), ("chunk", C.c_int32),
+                ("rel_rows", C.c_int32), ("rel_far", C.c_float), ("beside_kind", C.c_int32), ("mix_mult", C.c_float),
+                ("beside_mult", C.c_float), ("ssm_state", C.c_int32), ("ssm_heads", C.c_int32), ("ssm_dim", C.c_int32),
+                ("ssm_groups", C.c_int32), ("ssm_parts", C.c_int32), ("ssm_inner", C.c_int32), ("dt_rank", C.c_int32)]
 
 
 class MiStackConfig(C.Structure):
@@ -75,7 +79,8 @@ class MiStackConfig(C.Structure):
                 ("residual_mult", C.c_float), ("loop_start", C.c_int32), ("loop_stop", C.c_int32),
                 ("loop_times", C.c_int32), ("compute_dtype", C.c_int32), ("block_kind", C.c_int32),
                 ("norm_groups", C.c_int32), ("conv_taps", C.c_int32), ("logit_softcap", C.c_float),
-                ("state_lookahead", C.c_int32), ("embed_scale", C.c_float), ("norm_offset", C.c_float)]
+                ("state_lookahead", C.c_int32), ("embed_scale", C.c_float), ("norm_offset", C.c_float),
+                ("pos_base", C.c_float), ("logit_scale", C.c_float)]
 
 
 class MiTpPlan(C.Structure):
@@ -137,6 +142,20 @@ _SIGS = {
     "mi_op_experts": (C.c_int, [C.c_void_p] + [C.c_int32] * 6 + [C.c_void_p] * 8 + [C.c_int32] * 5 + [C.c_void_p]),
     "mi_op_delta_rule": (C.c_int, [C.POINTER(MiLayerSpec), C.c_void_p, C.c_int32, C.c_int32, C.c_void_p, C.c_int32, C.c_int32] + [C.c_void_p] * 4
                          + [C.c_float, C.c_void_p, C.c_void_p, C.c_int32] + [C.c_void_p] * 3 + [C.c_int32] * 3 + [C.c_void_p, C.c_int32, C.c_int32, C.c_void_p]),
+    "mi_op_embed_sinusoid": (C.c_int, [C.c_void_p] * 3 + [C.c_float] * 2 + [C.c_int32] * 3 + [C.c_void_p] * 2 + [C.c_int32] * 2 + [C.c_void_p]),
+    "mi_op_head_scatter": (C.c_int, [C.c_void_p, C.c_int32, C.c_int32, C.POINTER(MiLayerSpec)] + [C.c_void_p] * 3
+                           + [C.c_float, C.c_void_p, C.c_int32] + [C.c_void_p] * 3 + [C.c_int32, C.c_void_p]),
+    "mi_op_chunk_attn": (C.c_int, [C.POINTER(MiLayerSpec)] + [C.c_void_p] * 3 + [C.c_int32, C.c_float] + [C.c_void_p] * 3
+                         + [C.c_int32, C.c_void_p, C.c_int32] + [C.c_void_p] * 3 + [C.c_int32] * 3 + [C.c_void_p] + [C.c_int32] * 3 + [C.c_void_p]),
+    "mi_op_short_conv": (C.c_int, [C.c_void_p, C.c_int32, C.c_void_p, C.c_void_p, C.c_int32, C.c_int32, C.c_void_p, C.c_int32]
+                         + [C.c_void_p] * 3 + [C.c_int32] * 2 + [C.c_void_p] + [C.c_int32] * 2 + [C.c_void_p]),
+    "mi_op_scan": (C.c_int, [C.POINTER(MiLayerSpec), C.c_void_p, C.c_int32, C.c_void_p] + [C.c_int32] * 3 + [C.c_void_p] * 5
+                   + [C.c_int32, C.c_void_p, C.c_int32] + [C.c_void_p] * 3 + [C.c_int32] * 2 + [C.c_void_p] + [C.c_int32] * 2 + [C.c_void_p]),
+    "mi_op_scan_state": (C.c_int32, [C.c_int32]),
+    "mi_op_ssd": (C.c_int, [C.POINTER(MiLayerSpec), C.c_void_p, C.c_int32, C.c_void_p, C.c_int32] + [C.c_void_p] * 4 + [C.c_int32]
+                  + [C.c_void_p] * 3 + [C.c_int32] * 3 + [C.c_void_p] + [C.c_int32] * 2 + [C.c_void_p]),
+    "mi_op_gated_norm": (C.c_int, [C.c_void_p, C.c_int32, C.c_void_p, C.c_int32, C.c_void_p, C.c_int32, C.c_int32, C.c_float, C.c_int32, C.c_void_p,
+                                   C.c_int32, C.c_int32, C.c_void_p]),
     "mi_forward_spec": (C.c_int, [C.c_void_p, C.c_void_p, C.c_int32, C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p,
                                   C.c_int32, C.c_void_p, C.c_void_p, C.c_void_p]),
     "mi_replay_decode": (C.c_int, [C.c_void_p, C.c_int32, C.POINTER(C.c_float)]),
@@ -216,7 +235,7 @@ def _ptr(t) -> int:
 
 
 def layer_spec(layer: dict) -> MiLayerSpec:
-    out = MiLayerSpec(weights_of=-1)
+    out = MiLayerSpec(weights_of=-1, mix_mult=1.0, beside_mult=1.0)
     for k, v in layer.items():
         if not hasattr(out, k):
             raise ValueError(f"unknown layer field {k!r}")
@@ -225,7 +244,7 @@ def layer_spec(layer: dict) -> MiLayerSpec:
 
 
 def stack_config(stack: dict) -> MiStackConfig:
-    st = MiStackConfig(embed_scale=1.0)
+    st = MiStackConfig(embed_scale=1.0, logit_scale=1.0)
     layers = [layer_spec(x) for x in stack["layers"]]
     st._keep = (MiLayerSpec * len(layers))(*layers)      # the library copies it during the call
     st.layers, st.num_layers = st._keep, len(layers)

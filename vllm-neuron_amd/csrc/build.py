@@ -15,8 +15,8 @@ import sys
 HERE = os.path.dirname(os.path.abspath(__file__))
 HIPCC = shutil.which("hipcc") or "/opt/rocm/bin/hipcc"
 SOURCES = ["gemv_bf16.hip", "gemv_f8.hip", "gemv_i8.hip", "linear_kernels.hip", "attn_kernels.hip", "misc_kernels.hip", "stack_kernels.hip",
-           "window_attn.hip", "latent_attn.hip", "delta_rule.hip", "experts.hip", "stack.hip", "stack_ops.hip", "model.hip", "tp_group.hip"]
-HEADERS = ["mi_common.h", "linear_device.h", "linear_kernels.h", "attn_kernels.h", "misc_kernels.h", "model_internal.h", "stack_kernels.h", "window_attn.h", "latent_attn.h", "delta_rule.h", "experts.h", "stack.h", "tp_group.h",
+           "window_attn.hip", "latent_attn.hip", "delta_rule.hip", "ssm.hip", "experts.hip", "stack.hip", "stack_ops.hip", "model.hip", "tp_group.hip"]
+HEADERS = ["mi_common.h", "linear_device.h", "linear_kernels.h", "attn_kernels.h", "misc_kernels.h", "model_internal.h", "stack_kernels.h", "window_attn.h", "latent_attn.h", "delta_rule.h", "ssm.h", "experts.h", "stack.h", "tp_group.h",
            os.path.join("..", "..", "include", "mi355x_vllm.h")]
 LIB = os.path.join(HERE, "libmi355x_vllm.so")
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function", "-Wno-unused-value",

@@ -52,12 +52,6 @@ struct LatentRows {
 // per head y[t, h] = W_h x[t, h]: x [T, H, K], W [H][N, K] (16 x 32 bf16 tiles or row-major fp32; K % 32 == 0, N % 16 == 0);
 // columns n < n_valid go to y[t * ldy + h * y_head + n]
 int launch_head_linear(const void* w, int H, int N, int K, const void* x, int T, void* y, int ldy, int y_head, int n_valid, bool f32, hipStream_t s);
-// sigmoid(z) on the heads' outputs: row t at z + t ld, an element per head or per element of the heads; z null: none
-struct OutGate {
-  const float* z = nullptr;
-  int ld = 0;
-  bool per_element = false;
-};
 int launch_head_linear_rows(const void* w, int H, int N, int K, const uint16_t* x, const LatentRows& rows, uint16_t* y, int ldy, int y_head,
                             int n_valid, hipStream_t s, OutGate gate = OutGate());      // bf16, the listed rows only
 // ---- attention over latents, MFMA form (bf16)

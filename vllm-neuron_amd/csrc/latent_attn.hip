@@ -134,9 +134,9 @@ __device__ __forceinline__ RowAt latent_row(const LatentRows& r, int z) {
 
 // factors of the elements d .. d + 3 of head h
 __device__ __forceinline__ float4 gate4(const OutGate& gt, int row, int h, int dv, int d) {
-  if (!gt.z) return make_float4(1.f, 1.f, 1.f, 1.f);
+  if (!gt.z) return make_float4(gt.mult, gt.mult, gt.mult, gt.mult);
   const float* z = gt.z + (size_t)row * gt.ld;
-  auto f = [&](int i) { return 1.f / (1.f + expf(-z[gt.per_element ? h * dv + min(d + i, dv - 1) : h])); };
+  auto f = [&](int i) { return gt.mult / (1.f + expf(-z[gt.per_element ? h * dv + min(d + i, dv - 1) : h])); };
   if (gt.per_element) return make_float4(f(0), f(1), f(2), f(3));
   const float v = f(0);
   return make_float4(v, v, v, v);

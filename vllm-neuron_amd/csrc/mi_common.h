@@ -174,7 +174,7 @@ struct SlabSum {
   const float* row_scale = nullptr; // [T] or null (FP8 activations)
 };
 int device_num_cu(int* out);                                  // CUs of the current device
-int ensure_dynamic_lds(const void* kernel, int bytes);        // hipFuncSetAttribute once per (device, kernel)
+int ensure_dynamic_lds(const void* kernel, int bytes);        // hipFuncSetAttribute where (device, kernel) has fewer so far
 
 // weight tile geometry: a tile is 16 rows x TILE_K(wd) columns = 1 KiB, lane l owns
 // row (l & 15), k-chunk (l >> 4) of 16 bytes.

@@ -3,7 +3,7 @@
 #include "misc_kernels.h"
 
 #include <mutex>
-#include <set>
+#include <map>
 #include <utility>
 
 namespace mi {
@@ -25,13 +25,14 @@ int device_num_cu(int* out) {
 
 int ensure_dynamic_lds(const void* kernel, int bytes) {
   static std::mutex mu;
-  static std::set<std::pair<int, const void*>> done;
+  static std::map<std::pair<int, const void*>, int> done;     // bytes allowed so far
   int dev = 0;
   MI_HIP(hipGetDevice(&dev));
   std::lock_guard<std::mutex> lk(mu);
-  if (done.count({dev, kernel})) return MI_OK;
+  int& have = done[{dev, kernel}];
+  if (have >= bytes) return MI_OK;
   MI_HIP(hipFuncSetAttribute(kernel, hipFuncAttributeMaxDynamicSharedMemorySize, bytes));
-  done.insert({dev, kernel});
+  have = bytes;
   return MI_OK;
 }
 

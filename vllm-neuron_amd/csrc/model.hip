@@ -577,7 +577,7 @@ int capture_or_launch_decode(mi_ctx* c, int B, int MB) {
 extern "C" {
 
 const char* mi_last_error(void) { return mi::g_err.c_str(); }
-int mi_version(void) { return 7; }   // 3: + in-process tensor parallelism (tp_rank = MI_TP_ALL_RANKS, tp_device_ids, tp_transport)
+int mi_version(void) { return 8; }   // 3: + in-process tensor parallelism (tp_rank = MI_TP_ALL_RANKS, tp_device_ids, tp_transport)
 
 int mi_tp_plan(const mi_model_config* cfg, int32_t rank, mi_tp_plan_t* out) {
   MI_CHECK(cfg && out, "null argument");
@@ -695,6 +695,27 @@ int mi_ctx_create(const mi_model_config* cfg, mi_ctx** out) {
   return MI_OK;
 }
 
+static int check_post_norm_layer(const mi_layer_spec& p, const std::string& who) {
+  MI_CHECK(p.ff_kind == MI_FF_NONE || (p.ff_kind == MI_FF_RELU2 && p.ff_size > 0), who + "bad feed-forward");
+  MI_CHECK(p.weights_of < 0, who + "weights_of is built for one-norm blocks");
+  if (p.mixer_kind == MI_MIX_SCAN) {
+    MI_CHECK(p.ssm_inner > 0 && p.dt_rank > 0 && scan_supported(p.ssm_state) && p.conv_taps >= 1 && p.conv_taps <= 16, who + "selective scan: 1 .. 256 states, 1 .. 16 taps");
+    MI_CHECK(!p.beside_kind, who + "a second mixer is built beside attention");
+    return MI_OK;
+  }
+  MI_CHECK(p.mixer_kind == MI_MIX_ATTENTION, who + "this mixer is not built for the block kind");
+  MI_CHECK(p.num_heads > 0 && p.num_kv_heads > 0 && p.num_heads % p.num_kv_heads == 0 && p.qk_dim > 0 && p.v_dim > 0 && p.window >= 0 && p.chunk >= 0, who + "bad attention sizes");
+  MI_CHECK(!p.keys_as_values || p.qk_dim == p.v_dim, who + "values that are the keys have their size");
+  MI_CHECK(p.distance_bias == MI_BIAS_NONE || (p.distance_bias == MI_BIAS_TABLE && p.rel_rows >= 1 && p.rel_far > p.rel_rows / 2), who + "distance table: rel_far must be beyond half its rows");
+  MI_CHECK(p.softmax_sink >= MI_SINK_NONE && p.softmax_sink <= MI_SINK_LEARNED && (p.out_gate == MI_GATE_NONE || p.out_gate == MI_GATE_HEAD), who + "sink / output gate");
+  if (p.beside_kind) {
+    const SsdGeom g = ssd_geom(p.ssm_heads, p.ssm_dim, p.ssm_state, p.ssm_groups);
+    MI_CHECK(p.beside_kind == MI_MIX_SSD && ssd_supported(g) && p.conv_taps >= 1 && p.conv_taps <= 16, who + "state-space duality: heads a multiple of the groups, sizes 1 .. 256, 1 .. 16 taps");
+    MI_CHECK(p.ssm_parts >= 1 && g.inner() % p.ssm_parts == 0 && g.inner() <= 32768, who + "state-space duality: norm groups must divide the heads' columns");
+  }
+  return MI_OK;
+}
+
 int mi_ctx_create_stack(const mi_model_config* cfg, const mi_stack_config* stack, mi_ctx** out) {
   MI_CHECK(cfg && stack && out && stack->layers, "null argument");
   mi_model_config k = *cfg;
@@ -702,18 +723,23 @@ int mi_ctx_create_stack(const mi_model_config* cfg, const mi_stack_config* stack
   MI_CHECK(t.num_layers > 0 && t.width > 0 && t.width <= 32768 && t.vocab_size > 0 && t.max_positions >= 0 && t.norm_eps >= 0.f, "stack: bad geometry");
   MI_CHECK(t.compute_dtype == MI_BF16 || t.compute_dtype == MI_F32, "stack: compute_dtype must be MI_BF16 or MI_F32");
   MI_CHECK(t.loop_times == 0 || (t.loop_times > 0 && t.loop_start >= 0 && t.loop_start < t.loop_stop && t.loop_stop <= t.num_layers), "stack: bad loop");
-  MI_CHECK(t.block_kind >= MI_BLOCK_PARALLEL && t.block_kind <= MI_BLOCK_ONE_NORM, "stack: block_kind");
-  const bool sandwich = t.block_kind == MI_BLOCK_SANDWICH, one_norm = t.block_kind == MI_BLOCK_ONE_NORM;
+  MI_CHECK(t.block_kind >= MI_BLOCK_PARALLEL && t.block_kind <= MI_BLOCK_POST_NORM, "stack: block_kind");
+  const bool sandwich = t.block_kind == MI_BLOCK_SANDWICH, one_norm = t.block_kind == MI_BLOCK_ONE_NORM, post_norm = t.block_kind == MI_BLOCK_POST_NORM;
   if (sandwich) {
     MI_CHECK(t.norm_groups >= 1 && t.width % t.norm_groups == 0, "stack: the norm's groups must divide the width");
     MI_CHECK(t.conv_taps >= 1 && t.conv_taps <= 16 && t.state_lookahead >= 0, "stack: convolutions of 1 .. 16 taps are built");
     MI_CHECK(t.loop_times == 0, "stack: loops are not built for sandwich blocks");
+  } else if (post_norm) {
+    MI_CHECK(t.norm_groups == 1 && t.conv_taps == 0 && t.loop_times == 0 && t.residual_mult == 1.f && t.norm_offset == 0.f && t.max_positions == 0 && t.logit_softcap == 0.f,
+             "stack: post-norm blocks are built with a whole-row RMS norm, sinusoidal or no positions and no loop");
+    MI_CHECK(t.pos_base >= 0.f && t.logit_scale != 0.f, "stack: pos_base / logit_scale");
   } else if (one_norm) {
     MI_CHECK(t.norm_groups == 1 && t.conv_taps == 0 && t.loop_times == 0 && t.residual_mult == 1.f, "stack: one-norm blocks are built with a whole-row RMS norm and no loop");
   } else {
     MI_CHECK(t.norm_groups == 0 && t.conv_taps == 0 && t.max_positions > 0, "stack: parallel blocks are built with layer norms, learned positions and no convolution");
   }
-  MI_CHECK(one_norm || (t.norm_offset == 0.f && t.embed_scale == 1.f), "stack: norm_offset and embed_scale are built for one-norm blocks");
+  MI_CHECK(one_norm || (t.norm_offset == 0.f && (post_norm || t.embed_scale == 1.f)), "stack: norm_offset and embed_scale are built for one-norm blocks, embed_scale for post-norm blocks too");
+  MI_CHECK(post_norm || (t.pos_base == 0.f && t.logit_scale == 1.f), "stack: pos_base and logit_scale are built for post-norm blocks");
   MI_CHECK(t.logit_softcap >= 0.f, "stack: logit_softcap");
   for (int i = 0; i < t.num_layers; ++i) {
     const mi_layer_spec& p = t.layers[i];
@@ -724,6 +750,13 @@ int mi_ctx_create_stack(const mi_model_config* cfg, const mi_stack_config* stack
       MI_CHECK(j >= 0 && j < t.num_layers && t.layers[j].weights_of < 0, who + "weights_of must lead to a layer with tensors of its own");
       continue;
     }
+    if (post_norm) {
+      const int rc = check_post_norm_layer(p, who);
+      if (rc != MI_OK) return rc;
+      continue;
+    }
+    MI_CHECK(!p.qk_norm && !p.qk_bias && !p.keys_as_values && !p.chunk && !p.beside_kind && p.distance_bias <= MI_BIAS_SLOPE && p.softmax_sink <= MI_SINK_ONE,
+             who + "weighted query / key norms, biases, chunks, distance tables, learned sinks and second mixers are built for post-norm blocks");
     MI_CHECK(one_norm ? p.mixer_kind == MI_MIX_LATENT || p.mixer_kind == MI_MIX_DELTA : p.mixer_kind == (sandwich ? MI_MIX_LATENT : MI_MIX_ATTENTION),
              who + "this mixer is not built for the block kind");
     MI_CHECK(p.num_heads > 0 && p.qk_dim > 0 && p.v_dim > 0 && p.window >= 0, who + "bad attention sizes");
@@ -2039,15 +2072,44 @@ int mi_op_embed_pos(const int32_t* ids, const int32_t* pos, const void* table, c
 int mi_op_qkv_scatter(const float* qkv, int32_t ldq, int32_t T, const mi_layer_spec* spec, float eps, const int32_t* slots,
                       int32_t block_size, void* q, void* kpool, void* vpool, int32_t f32, void* stream) {
   MI_CHECK(qkv && spec && slots && q && kpool && vpool && T >= 1, "null argument");
-  return launch_qkv_scatter(qkv, ldq, T, head_geom(*spec), spec->qk_unit_norm != 0, eps, slots, block_size, q, kpool, vpool, f32 != 0, (hipStream_t)stream);
+  return launch_qkv_scatter(qkv, ldq, T, head_geom(*spec), HeadRule{spec->qk_unit_norm != 0}, eps, slots, block_size, q, kpool, vpool, f32 != 0, (hipStream_t)stream);
 }
+static int attn_op(const AttnSpec& a, const OutGate& gate, const void* q, const void* kpool, const void* vpool, int32_t block_size, const int32_t* block_table,
+                   int32_t MB, const int32_t* pos, const int32_t* ctx_lens, const int32_t* segs_host, int32_t nseg, int32_t T, int32_t max_ctx, void* out,
+                   int32_t ldo, int32_t f32, int32_t path, void* stream);
 int mi_op_window_attn(const mi_layer_spec* spec, const float* slopes, const void* q, const void* kpool, const void* vpool,
                       int32_t block_size, const int32_t* block_table, int32_t MB, const int32_t* pos, const int32_t* ctx_lens,
                       const int32_t* segs_host, int32_t nseg, int32_t T, int32_t max_ctx, void* out, int32_t ldo, int32_t f32,
                       int32_t path, void* stream) {
-  MI_CHECK(spec && q && kpool && vpool && block_table && pos && ctx_lens && segs_host && out && nseg >= 1 && T >= 1, "null argument");
+  MI_CHECK(spec, "null argument");
   MI_CHECK(!spec->distance_bias || slopes, "distance bias without slopes");
   const AttnSpec a{head_geom(*spec), spec->scale, spec->window, spec->distance_bias ? slopes : nullptr, spec->qk_unit_norm ? 1 : 0, spec->softmax_sink ? 1 : 0};
+  return attn_op(a, OutGate(), q, kpool, vpool, block_size, block_table, MB, pos, ctx_lens, segs_host, nseg, T, max_ctx, out, ldo, f32, path, stream);
+}
+int mi_op_chunk_attn(const mi_layer_spec* spec, const float* sinks, const float* rel, const float* gate, int32_t ldg, float mult, const void* q,
+                     const void* kpool, const void* vpool, int32_t block_size, const int32_t* block_table, int32_t MB, const int32_t* pos,
+                     const int32_t* ctx_lens, const int32_t* segs_host, int32_t nseg, int32_t T, int32_t max_ctx, void* out, int32_t ldo, int32_t f32,
+                     int32_t path, void* stream) {
+  MI_CHECK(spec && (!rel || (spec->rel_rows >= 1 && spec->rel_far > spec->rel_rows / 2)), "distance table");
+  AttnSpec a{head_geom(*spec), spec->scale, spec->window, nullptr, 0, spec->softmax_sink || sinks ? 1 : 0, spec->chunk, sinks};
+  float* table = nullptr;
+  if (rel) {
+    hipStream_t s = (hipStream_t)stream;
+    const std::vector<int> rows = distance_rows(spec->rel_rows, spec->rel_far, spec->chunk);
+    a.table_n = (int)rows.size();
+    MI_HIP(hipMalloc(reinterpret_cast<void**>(&table), (size_t)spec->num_heads * a.table_n * 4));
+    const int rc = stack_distance_table(rel, rows, spec->rel_rows, spec->num_heads, table, s);
+    if (rc != MI_OK) { hipFree(table); return rc; }
+    a.table = table;
+  }
+  const int rc = attn_op(a, OutGate{gate, ldg, false, mult}, q, kpool, vpool, block_size, block_table, MB, pos, ctx_lens, segs_host, nseg, T, max_ctx, out, ldo, f32, path, stream);
+  hipFree(table);
+  return rc;
+}
+static int attn_op(const AttnSpec& a, const OutGate& gate, const void* q, const void* kpool, const void* vpool, int32_t block_size, const int32_t* block_table,
+                   int32_t MB, const int32_t* pos, const int32_t* ctx_lens, const int32_t* segs_host, int32_t nseg, int32_t T, int32_t max_ctx, void* out,
+                   int32_t ldo, int32_t f32, int32_t path, void* stream) {
+  MI_CHECK(q && kpool && vpool && block_table && pos && ctx_lens && segs_host && out && nseg >= 1 && T >= 1, "null argument");
   std::vector<AttnSeg> segs((size_t)nseg);
   memcpy(segs.data(), segs_host, (size_t)nseg * sizeof(AttnSeg));
   int row = 0;
@@ -2063,15 +2125,16 @@ int mi_op_window_attn(const mi_layer_spec* spec, const float* slopes, const void
   MI_HIP(hipMalloc(&scratch, attn_window_scratch_bytes(nseg, a.g)));
   MI_HIP(hipMemcpyAsync(sd, segs.data(), (size_t)nseg * sizeof(AttnSeg), hipMemcpyHostToDevice, s));
   int rc = MI_OK;
-  if (f32 || path == 1 || !attn_window_supported(a.g)) {
-    rc = launch_attn_plain(a, q, kpool, vpool, block_size, block_table, MB, pos, sd, nseg, T, out, ldo, f32 != 0, s);
+  if (f32 || path == 1 || !attn_window_supported(a.g) || (a.table && !attn_table_supported(a.g, a.table_n))) {
+    rc = launch_attn_plain(a, q, kpool, vpool, block_size, block_table, MB, pos, sd, nseg, T, out, ldo, f32 != 0, s, gate);
   } else {
     const uint16_t *qb = (const uint16_t*)q, *kb = (const uint16_t*)kpool, *vb = (const uint16_t*)vpool;
-    rc = launch_attn_window_prefill(a, qb, kb, vb, block_size, block_table, MB, sd, segs.data(), nseg, (uint16_t*)out, ldo, s);
+    rc = launch_attn_window_prefill(a, qb, kb, vb, block_size, block_table, MB, sd, segs.data(), nseg, (uint16_t*)out, ldo, s, 2, gate);
     for (int i = 0; i < nseg && rc == MI_OK; ++i)
       if (segs[i].n == 1)
         rc = launch_attn_window_decode(a, qb + (size_t)segs[i].row0 * a.g.H * a.g.dkp, kb, vb, block_size, block_table + (size_t)segs[i].seq * MB, MB,
-                                       ctx_lens + segs[i].seq, 1, max_ctx, (uint16_t*)out + (size_t)segs[i].row0 * ldo, ldo, scratch, s);
+                                       ctx_lens + segs[i].seq, 1, max_ctx, (uint16_t*)out + (size_t)segs[i].row0 * ldo, ldo, scratch, s,
+                                       OutGate{gate.z ? gate.z + (size_t)segs[i].row0 * gate.ld : nullptr, gate.ld, false, gate.mult});
   }
   hipStreamSynchronize(s);
   hipFree(sd);

@@ -8,6 +8,7 @@
 #include "experts.h"
 #include "latent_attn.h"
 #include "model_internal.h"
+#include "ssm.h"
 
 namespace mi {
 
@@ -42,6 +43,23 @@ struct StackLayer {
   StackMat uq, a2, g2;
   float *q_norm = nullptr, *conv = nullptr, *a_log = nullptr, *dt = nullptr, *o_norm = nullptr;
   DeltaGeom dg;
+  // post-norm blocks: qkv = every product with x the mixer needs; attention: [q | k (| v) | g], beside it [z | x B C | dt]; selective scan: [x | z].
+  // out = W_o, or [W_o left | W_o right] over [heads x v_dim | second mixer]; n1 / n2 the norms of the sublayers' outputs
+  int col_z = 0, col_x = 0, col_dt = 0;
+  HeadRule heads;
+  float *qk_bias = nullptr, *k_norm = nullptr, *sinks = nullptr, *table = nullptr;
+  std::vector<int> table_rows;                   // row of the checkpoint's distance table by distance
+  StackMat low_in, dt_mat;                       // selective scan: x -> [low | B | C], low -> step sizes of the channels
+  int col_B = 0, col_C = 0;
+  void* w_dt = nullptr;                          // dt_mat row-major [C][rank_p]: token generation
+  float *conv_b = nullptr, *decay = nullptr, *ssm_d = nullptr;   // (decay, bias and norm: a_log, dt, o_norm)
+  ScanGeom scan;
+  SsdGeom ssd;
+  bool has_scan() const { return s.mixer_kind == MI_MIX_SCAN; }
+  bool has_ssd() const { return s.beside_kind == MI_MIX_SSD; }
+  int conv_channels() const { return has_scan() ? scan.C : ssd.channels(); }
+  size_t ssm_state_floats() const { return has_scan() ? scan.state_floats() : has_ssd() ? ssd.state_floats() : 0; }
+  size_t ssm_ring_floats() const { return ssm_state_floats() ? (size_t)s.conv_taps * conv_channels() : 0; }
   const float2* rot = nullptr;                   // cosines and sines of the layer's rotation (Stack::rot)
   int ff_act() const { return s.ff_act == MI_ACT_RELU2 ? EXPERT_RELU2 : EXPERT_SILU_GLU; }
   RouterRule rule() const {
@@ -98,6 +116,14 @@ struct Stack {
   size_t chunk_floats = 0;
   void *cq = nullptr, *low = nullptr; // normed query latents; the inputs of the decay's and the gate's second product [2][rows][low_ld]
   float *q2 = nullptr, *z = nullptr, *delta_records = nullptr;
+  // post-norm blocks
+  double* turns = nullptr;             // sinusoidal positions: turns per position [ceil(width / 2)]
+  void *xc = nullptr;                  // convolution outputs [rows][xc_ld]
+  float *xp = nullptr, *dtp = nullptr, *yssm = nullptr, *ssd_records = nullptr;   // [low | B | C]; step sizes; outputs ahead of gate and norm
+  int xc_ld = 0, xp_ld = 0, dtp_ld = 0, yssm_ld = 0, ssd_chunks = 0;
+  size_t ssd_chunk_floats = 0;
+  bool post_norm() const { return cfg.block_kind == MI_BLOCK_POST_NORM; }
+  bool parallel() const { return cfg.block_kind == MI_BLOCK_PARALLEL; }
   bool one_norm() const { return cfg.block_kind == MI_BLOCK_ONE_NORM; }
   bool sandwich() const { return cfg.block_kind == MI_BLOCK_SANDWICH; }
   void* attn_scratch = nullptr;
@@ -106,6 +132,10 @@ struct Stack {
   size_t elem() const { return f32 ? 4 : 2; }
 };
 
+// *turns [ceil(width / 2)] (device, allocated): base^(-2 i / width) / 2 pi
+int stack_position_turns(int width, float base, double** turns, hipStream_t s);
+// table [H][rows.size()] = rel [rel_rows, H] (device) by distance
+int stack_distance_table(const float* rel, const std::vector<int>& rows, int rel_rows, int H, float* table, hipStream_t s);
 int stack_create(mi_ctx* c, const mi_stack_config& cfg);      // geometry + weight images (zeroed)
 void stack_destroy(mi_ctx* c);
 int stack_load_tensor(mi_ctx* c, const std::string& name, const float* dev, int rows, int cols);   // cols 0: a vector of `rows`

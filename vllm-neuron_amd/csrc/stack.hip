@@ -22,6 +22,13 @@
 //   latent attention: [dkv | dq | g] product; query latent's norm; W_uq; rotation, scatter, attention as above; output gate
 //   delta rule: [q | k | v | b | a1 | g1] product; a2, g2; recurrence               delta_rule.hip
 //   output projection + residual; the experts' weighted sum and a K-split's are left to the next row kernel
+//
+// A post-norm block's run (the sublayers read the stream itself, RMS norms on their outputs):
+//   row: x += norm of the previous sublayer's output; x in the compute type         sandwich_rows
+//   attention: [q | k | g] product, beside it [z | x B C | dt]; norms and scatter; attention with gate; short convolution, recurrence,
+//   gate and norm into the same row (ssm.hip); one output projection for both
+//   selective scan: [x | z] product; short convolution; [low | B | C] product; step sizes; scan (ssm.hip); output projection
+//   up, squared relu, down
 
 #include "stack.h"
 
@@ -108,7 +115,7 @@ int norm_rows(mi_ctx* c, int cur, int rows, const NormOut& a, const NormOut& b) 
 
 bool runs_other(mi_ctx* c) { return c->runs(MI_K_OTHER); }
 
-int attention(mi_ctx* c, const StackLayer& W, size_t kv_at, int rows, bool decode, int MB, const AttnSeg* segs, int nseg) {
+int attention(mi_ctx* c, const StackLayer& W, size_t kv_at, int ldq, int rows, bool decode, int MB, const AttnSeg* segs, int nseg, const OutGate& gate = OutGate()) {
   Stack* S = c->stack;
   const mi_model_config& k = c->cfg;
   unsigned char* base = reinterpret_cast<unsigned char*>(c->kv_pool);
@@ -116,13 +123,14 @@ int attention(mi_ctx* c, const StackLayer& W, size_t kv_at, int rows, bool decod
   unsigned char *kp = base + kv_at * S->elem(), *vp = base + (kv_at + kn) * S->elem();
   if (runs_other(c)) {
     Scope sc(c, MI_K_OTHER);
-    MI_TRY(launch_qkv_scatter(S->qkv_out, S->qkv_ld, rows, W.g, W.s.qk_unit_norm != 0, S->cfg.norm_eps, c->d_slots, k.block_size, S->q, kp, vp, S->f32, c->stream));
+    MI_TRY(launch_qkv_scatter(S->qkv_out, ldq, rows, W.g, W.heads, S->cfg.norm_eps, c->d_slots, k.block_size, S->q, kp, vp, S->f32, c->stream));
   }
   const int ldo = S->cat_ld;
-  if (S->f32 || !attn_window_supported(W.g)) {
+  if (S->f32 || !attn_window_supported(W.g) || (W.attn.table && !attn_table_supported(W.g, W.attn.table_n))) {
+    if (!c->runs(decode ? MI_K_ATTN_DECODE : MI_K_ATTN_PREFILL)) return MI_OK;
     Scope sc(c, decode ? MI_K_ATTN_DECODE : MI_K_ATTN_PREFILL);
     return launch_attn_plain(W.attn, S->q, kp, vp, k.block_size, c->d_bt, MB, c->d_pos, decode ? nullptr : reinterpret_cast<const AttnSeg*>(c->d_segs),
-                             nseg, rows, S->cat, ldo, S->f32, c->stream);
+                             nseg, rows, S->cat, ldo, S->f32, c->stream, gate);
   }
   const uint16_t* q = reinterpret_cast<const uint16_t*>(S->q);
   const uint16_t *kb = reinterpret_cast<const uint16_t*>(kp), *vb = reinterpret_cast<const uint16_t*>(vp);
@@ -131,16 +139,17 @@ int attention(mi_ctx* c, const StackLayer& W, size_t kv_at, int rows, bool decod
   if (decode) {
     if (!c->runs(MI_K_ATTN_DECODE)) return MI_OK;
     Scope sc(c, MI_K_ATTN_DECODE);
-    return launch_attn_window_decode(W.attn, q, kb, vb, k.block_size, c->d_bt, MB, c->d_ctx, rows, k.max_model_len, out, ldo, S->attn_scratch, c->stream);
+    return launch_attn_window_decode(W.attn, q, kb, vb, k.block_size, c->d_bt, MB, c->d_ctx, rows, k.max_model_len, out, ldo, S->attn_scratch, c->stream, gate);
   }
   Scope sc(c, MI_K_ATTN_PREFILL);
-  MI_TRY(launch_attn_window_prefill(W.attn, q, kb, vb, k.block_size, c->d_bt, MB, reinterpret_cast<const AttnSeg*>(c->d_segs), segs, nseg, out, ldo, c->stream));
+  MI_TRY(launch_attn_window_prefill(W.attn, q, kb, vb, k.block_size, c->d_bt, MB, reinterpret_cast<const AttnSeg*>(c->d_segs), segs, nseg, out, ldo, c->stream, 2, gate));
   for (int i = 0; i < nseg;) {   // runs of requests with one token: one token-generation launch each
     int j = i;
     while (j < nseg && segs[j].n == 1) ++j;
     if (j > i)
       MI_TRY(launch_attn_window_decode(W.attn, q + segs[i].row0 * qrow, kb, vb, k.block_size, c->d_bt + (size_t)i * MB, MB, c->d_seg_ctx + i, j - i,
-                                       k.max_model_len, out + (size_t)segs[i].row0 * ldo, ldo, S->attn_scratch, c->stream));
+                                       k.max_model_len, out + (size_t)segs[i].row0 * ldo, ldo, S->attn_scratch, c->stream,
+                                       OutGate{gate.z ? gate.z + (size_t)segs[i].row0 * gate.ld : nullptr, gate.ld, false, gate.mult}));
     i = j > i ? j : i + 1;
   }
   return MI_OK;
@@ -472,7 +481,229 @@ int one_norm_place(mi_ctx* c, StackLayer& W, const std::string& t, const float* 
   return vec(m == "dq.norm" ? W.q_norm : W.c_norm);
 }
 
+// ---- post-norm blocks: geometry and weights of one layer ---------------------------------------------------------------------
+// name of a layer's tensor behind "mix." within the mixer it belongs to: 0 the only or the left one, 1 the right one, -1 neither's
+int mixer_of(const StackLayer& W, const std::string& t, std::string* name) {
+  if (t.compare(0, 4, "mix.") != 0) return -1;
+  *name = t.substr(4);
+  if (!W.s.beside_kind) return 0;
+  for (int i = 0; i < 2; ++i) {
+    const std::string p = i ? "right." : "left.";
+    if (name->compare(0, p.size(), p) == 0) { *name = name->substr(p.size()); return i; }
+  }
+  return -1;
+}
+
+int post_norm_layer_create(mi_ctx* c, StackLayer& W, const std::string& p) {
+  Stack* S = c->stack;
+  const mi_layer_spec& s = W.s;
+  size_t* wb = &c->weight_bytes;
+  auto want = [&](const std::string& n) { S->missing.push_back(p + n); };
+  auto vec = [&](float** v, size_t n) { return alloc0(c, v, n * 4, wb); };
+  MI_TRY(vec(&W.n1.w, S->ld));
+  want("norm1");
+  if (s.ff_kind != MI_FF_NONE) {
+    MI_TRY(vec(&W.n2.w, S->ld));
+    MI_TRY(alloc_mat(c, W.up, s.ff_size, S->D, 1.f));
+    MI_TRY(alloc_mat(c, W.down, S->D, s.ff_size, 1.f));
+    W.ffk = W.down.K;
+    S->act_ld = std::max(S->act_ld, W.ffk);
+    for (const char* n : {"norm2", "mlp.up", "mlp.down"}) want(n);
+  }
+  if (W.has_scan()) {
+    const ScanGeom& g = W.scan = scan_geom(s.ssm_inner, s.ssm_state, s.dt_rank);
+    W.col_z = pad_to(g.C, 16);
+    W.col_B = pad_to(g.rank, 16);
+    W.col_C = W.col_B + pad_to(g.N, 16);
+    MI_TRY(alloc_mat(c, W.qkv, W.col_z + g.C, S->D, 1.f));
+    MI_TRY(alloc_mat(c, W.low_in, W.col_C + g.N, g.C, 1.f));
+    MI_TRY(alloc_mat(c, W.dt_mat, g.C, g.rank, 1.f));
+    MI_TRY(alloc_mat(c, W.out, S->D, g.C, 1.f));
+    MI_TRY(alloc0(c, &W.w_dt, (size_t)g.C * g.rank_p * S->elem(), wb));
+    MI_TRY(vec(&W.decay, (size_t)g.C * g.Np));
+    MI_TRY(vec(&W.dt, g.C));
+    MI_TRY(vec(&W.ssm_d, g.C));
+    S->xc_ld = std::max(S->xc_ld, W.low_in.K);
+    S->xp_ld = std::max(S->xp_ld, W.low_in.N);
+    S->low_ld = std::max(S->low_ld, W.dt_mat.K);
+    S->dtp_ld = std::max(S->dtp_ld, W.dt_mat.N);
+    for (const char* n : {"in", "conv", "conv.b", "x", "dt", "dt.b", "A_log", "D", "o"}) want(std::string("mix.") + n);
+  } else {
+    const std::string m = s.beside_kind ? "mix.left." : "mix.";
+    const int qk = (s.num_heads + s.num_kv_heads) * s.qk_dim;
+    W.g = HeadGeom{s.num_heads, s.num_kv_heads, s.qk_dim, s.v_dim, pad_to(s.qk_dim, 16), pad_to(s.v_dim, 16)};
+    W.attn_cols = pad_to(s.num_heads * s.v_dim, 16);
+    int n = pad_to(qk + (s.keys_as_values ? 0 : s.num_kv_heads * s.v_dim), 16);
+    W.col_g = n;
+    if (s.out_gate) n = W.col_g + pad_to(s.num_heads, 16);
+    if (W.has_ssd()) {
+      const SsdGeom& g = W.ssd = ssd_geom(s.ssm_heads, s.ssm_dim, s.ssm_state, s.ssm_groups);
+      W.col_z = n;
+      W.col_x = W.col_z + pad_to(g.inner(), 16);
+      W.col_dt = W.col_x + pad_to(g.channels(), 16);
+      n = W.col_dt + pad_to(g.H, 16);
+      MI_TRY(vec(&W.a_log, g.H));
+      MI_TRY(vec(&W.dt, g.H));
+      MI_TRY(vec(&W.ssm_d, g.H));
+      MI_TRY(vec(&W.o_norm, g.inner()));
+      S->xc_ld = std::max(S->xc_ld, pad_to(g.channels(), 16));
+      S->yssm_ld = std::max(S->yssm_ld, pad_to(g.inner(), 16));
+      S->ssd_chunk_floats = std::max(S->ssd_chunk_floats, ssd_chunk_floats(g));
+      for (const char* t : {"in", "conv", "conv.b", "dt_bias", "A_log", "D", "norm", "o"}) want(std::string("mix.right.") + t);
+    }
+    MI_TRY(alloc_mat(c, W.qkv, n, S->D, 1.f));
+    MI_TRY(alloc_mat(c, W.out, S->D, W.attn_cols + (W.has_ssd() ? W.ssd.inner() : 0), 1.f));
+    for (const char* t : {"q", "k", "o"}) want(m + t);
+    if (!s.keys_as_values) want(m + "v");
+    W.heads = HeadRule{s.qk_norm || s.qk_unit_norm, nullptr, nullptr, nullptr, s.keys_as_values != 0};
+    if (s.qk_bias) {
+      MI_TRY(vec(&W.qk_bias, qk));
+      W.heads.bias = W.qk_bias;
+      want(m + "q.b"); want(m + "k.b");
+    }
+    if (s.qk_norm) {
+      MI_TRY(vec(&W.q_norm, s.qk_dim));
+      MI_TRY(vec(&W.k_norm, s.qk_dim));
+      W.heads.q_norm = W.q_norm; W.heads.k_norm = W.k_norm;
+      want(m + "q.norm"); want(m + "k.norm");
+    }
+    if (s.out_gate) want(m + "g");
+    if (s.softmax_sink == MI_SINK_LEARNED) {
+      MI_TRY(vec(&W.sinks, s.num_heads));
+      want(m + "sink");
+    }
+    if (s.distance_bias == MI_BIAS_TABLE) {
+      W.table_rows = distance_rows(s.rel_rows, s.rel_far, s.chunk);
+      MI_TRY(vec(&W.table, (size_t)s.num_heads * W.table_rows.size()));
+      want(m + "rel");
+    }
+    W.attn = AttnSpec{W.g, s.scale, s.window, nullptr, 0, s.softmax_sink != MI_SINK_NONE, s.chunk, W.sinks, W.table, (int)W.table_rows.size()};
+    S->q_cols = std::max(S->q_cols, s.num_heads * W.g.dkp);
+  }
+  if (W.ssm_state_floats()) {
+    const int C = W.conv_channels();
+    MI_TRY(vec(&W.conv, (size_t)s.conv_taps * C));
+    MI_TRY(vec(&W.conv_b, C));
+    S->state_slots = c->cfg.max_num_seqs;
+  }
+  S->qkv_ld = std::max(S->qkv_ld, W.qkv.N);
+  S->cat_ld = std::max(S->cat_ld, W.out.K);
+  return MI_OK;
+}
+
+void post_norm_tensor_shape(const Stack* S, const StackLayer& W, const std::string& t, int* rows, int* cols) {
+  const mi_layer_spec& s = W.s;
+  *rows = *cols = 0;
+  auto is = [&](int r, int k) { *rows = r; *cols = k; };
+  const bool ff = s.ff_kind != MI_FF_NONE;
+  if (t == "norm1" || (ff && t == "norm2")) return is(S->D, 0);
+  if (ff && t == "mlp.up") return is(s.ff_size, S->D);
+  if (ff && t == "mlp.down") return is(S->D, s.ff_size);
+  std::string m;
+  const int part = mixer_of(W, t, &m);
+  if (part < 0) return;
+  if (part == 0 && !W.has_scan()) {
+    const int H = s.num_heads, G = s.num_kv_heads, d = s.qk_dim;
+    if (m == "q") is(H * d, S->D);
+    else if (m == "k") is(G * d, S->D);
+    else if (m == "v" && !s.keys_as_values) is(G * s.v_dim, S->D);
+    else if (m == "q.b" && s.qk_bias) is(H * d, 0);
+    else if (m == "k.b" && s.qk_bias) is(G * d, 0);
+    else if ((m == "q.norm" || m == "k.norm") && s.qk_norm) is(d, 0);
+    else if (m == "rel" && s.distance_bias == MI_BIAS_TABLE) is(s.rel_rows, H);
+    else if (m == "sink" && s.softmax_sink == MI_SINK_LEARNED) is(H, 0);
+    else if (m == "g" && s.out_gate) is(H, S->D);
+    else if (m == "o") is(S->D, H * s.v_dim);
+    return;
+  }
+  const int C = W.conv_channels();
+  if (m == "conv") return is(C, s.conv_taps);
+  if (m == "conv.b") return is(C, 0);
+  if (W.has_scan()) {
+    const ScanGeom& g = W.scan;
+    if (m == "in") is(2 * g.C, S->D);
+    else if (m == "x") is(g.rank + 2 * g.N, g.C);
+    else if (m == "dt") is(g.C, g.rank);
+    else if (m == "dt.b" || m == "D") is(g.C, 0);
+    else if (m == "A_log") is(g.C, g.N);
+    else if (m == "o") is(S->D, g.C);
+    return;
+  }
+  const SsdGeom& g = W.ssd;
+  if (m == "in") is(g.inner() + C + g.H, S->D);
+  else if (m == "dt_bias" || m == "A_log" || m == "D") is(g.H, 0);
+  else if (m == "norm") is(g.inner(), 0);
+  else if (m == "o") is(S->D, g.inner());
+}
+
+int post_norm_place(mi_ctx* c, StackLayer& W, const std::string& t, const float* dev, int rows, int cols) {
+  Stack* S = c->stack;
+  const mi_layer_spec& s = W.s;
+  hipStream_t st = c->stream;
+  auto vec = [&](float* dst) { return launch_offset_copy(dev, rows, 0.f, dst, st); };
+  // rows r0 .. + n of the tensor to row0 of the matrix
+  auto part = [&](const StackMat& m, int r0, int n, int row0, int col0 = 0) {
+    return launch_place(dev + (size_t)r0 * cols, cols, 0, n, cols, m.L.w, m.K, S->f32, row0, col0, st);
+  };
+  if (t == "norm1") return vec(W.n1.w);
+  if (t == "norm2") return vec(W.n2.w);
+  if (t == "mlp.up") return part(W.up, 0, rows, 0);
+  if (t == "mlp.down") return part(W.down, 0, rows, 0);
+  std::string m;
+  const int which = mixer_of(W, t, &m);
+  if (which == 0 && !W.has_scan()) {
+    const int qn = s.num_heads * s.qk_dim, kn = s.num_kv_heads * s.qk_dim;
+    if (m == "q") return part(W.qkv, 0, rows, 0);
+    if (m == "k") return part(W.qkv, 0, rows, qn);
+    if (m == "v") return part(W.qkv, 0, rows, qn + kn);
+    if (m == "g") return part(W.qkv, 0, rows, W.col_g);
+    if (m == "o") return part(W.out, 0, rows, 0);
+    if (m == "q.b") return vec(W.qk_bias);
+    if (m == "k.b") return vec(W.qk_bias + qn);
+    if (m == "q.norm") return vec(W.q_norm);
+    if (m == "k.norm") return vec(W.k_norm);
+    if (m == "sink") return vec(W.sinks);
+    return stack_distance_table(dev, W.table_rows, s.rel_rows, s.num_heads, W.table, st);
+  }
+  if (m == "conv") return launch_transpose(dev, rows, cols, W.conv, rows, st);
+  if (m == "conv.b") return vec(W.conv_b);
+  if (m == "D") return vec(W.ssm_d);
+  if (W.has_scan()) {
+    const ScanGeom& g = W.scan;
+    if (m == "in") { MI_TRY(part(W.qkv, 0, g.C, 0)); return part(W.qkv, g.C, g.C, W.col_z); }
+    if (m == "x") {
+      MI_TRY(part(W.low_in, 0, g.rank, 0));
+      MI_TRY(part(W.low_in, g.rank, g.N, W.col_B));
+      return part(W.low_in, g.rank + g.N, g.N, W.col_C);
+    }
+    if (m == "dt") { MI_TRY(launch_place_rows(dev, rows, cols, W.w_dt, g.rank_p, S->f32, st)); return part(W.dt_mat, 0, rows, 0); }
+    if (m == "dt.b") return vec(W.dt);
+    if (m == "A_log") return launch_scan_decay(dev, g, W.decay, st);
+    return part(W.out, 0, rows, 0);
+  }
+  const SsdGeom& g = W.ssd;
+  if (m == "in") {
+    MI_TRY(part(W.qkv, 0, g.inner(), W.col_z));
+    MI_TRY(part(W.qkv, g.inner(), g.channels(), W.col_x));
+    return part(W.qkv, g.inner() + g.channels(), g.H, W.col_dt);
+  }
+  if (m == "o") return part(W.out, 0, rows, 0, W.attn_cols);
+  if (m == "norm") return launch_scaled_copy(dev, rows, s.beside_mult, W.o_norm, st);
+  return vec(m == "A_log" ? W.a_log : W.dt);
+}
+
 }  // namespace
+
+int stack_distance_table(const float* rel, const std::vector<int>& rows, int rel_rows, int H, float* table, hipStream_t s) {
+  std::vector<float> r((size_t)rel_rows * H), t((size_t)H * rows.size());
+  MI_HIP(hipMemcpyAsync(r.data(), rel, r.size() * 4, hipMemcpyDeviceToHost, s));
+  MI_HIP(hipStreamSynchronize(s));
+  for (int h = 0; h < H; ++h)
+    for (size_t n = 0; n < rows.size(); ++n) t[h * rows.size() + n] = r[(size_t)rows[n] * H + h];
+  MI_HIP(hipMemcpyAsync(table, t.data(), t.size() * 4, hipMemcpyHostToDevice, s));
+  MI_HIP(hipStreamSynchronize(s));
+  return MI_OK;
+}
 
 int stack_create(mi_ctx* c, const mi_stack_config& cfg) {
   Stack* S = c->stack = new Stack();
@@ -518,6 +749,10 @@ int stack_create(mi_ctx* c, const mi_stack_config& cfg) {
     StackLayer& W = S->layers[i];
     W.s = cfg.layers[i];
     const mi_layer_spec& s = W.s;
+    if (S->post_norm()) {
+      MI_TRY(post_norm_layer_create(c, W, "l" + std::to_string(i) + "."));
+      continue;
+    }
     if (S->one_norm()) {
       if (s.weights_of < 0) MI_TRY(one_norm_layer_create(c, W, "l" + std::to_string(i) + "."));
       continue;
@@ -542,6 +777,7 @@ int stack_create(mi_ctx* c, const mi_stack_config& cfg) {
       MI_HIP(hipStreamSynchronize(c->stream));
     }
     W.attn = AttnSpec{W.g, s.scale, s.window, W.slopes, s.qk_unit_norm ? 1 : 0, s.softmax_sink ? 1 : 0};
+    W.heads.unit_norm = s.qk_unit_norm != 0;
     S->qkv_ld = std::max(S->qkv_ld, W.qkv.N);
     S->q_cols = std::max(S->q_cols, s.num_heads * W.g.dkp);
     S->cat_ld = std::max(S->cat_ld, W.out.K);
@@ -551,7 +787,7 @@ int stack_create(mi_ctx* c, const mi_stack_config& cfg) {
       for (const char* n : {"norm2", "norm2.b", "mlp.up", "mlp.down"}) want(p + n);
   }
   MI_TRY(alloc_norm(c, S->final_norm));
-  MI_TRY(alloc_mat(c, S->head, cfg.vocab_size, S->D, 1.f));
+  MI_TRY(alloc_mat(c, S->head, cfg.vocab_size, S->D, cfg.logit_scale));
   want("final.norm"); want("head");
   if (cfg.norm_groups == 0) want("final.norm.b");
   MI_HIP(hipStreamSynchronize(c->stream));
@@ -564,15 +800,18 @@ void stack_destroy(mi_ctx* c) {
     free_mat(W.qkv); free_mat(W.up); free_mat(W.out);
     free_mat(W.down); free_mat(W.ukv); free_mat(W.router_t);
     free_norm(W.n1); free_norm(W.n2); free_norm(W.n1b); free_norm(W.n2b);
+    free_mat(W.low_in); free_mat(W.dt_mat);
     free_mat(W.uq); free_mat(W.a2); free_mat(W.g2);
-    void* ps[] = {W.q_norm, W.conv, W.a_log, W.dt, W.o_norm, W.slopes, W.conv1, W.conv2, W.c_norm, W.w_uk, W.w_uv, W.router, W.router_b, W.expert_gu, W.expert_down};
+    void* ps[] = {W.q_norm, W.conv, W.a_log, W.dt, W.o_norm, W.slopes, W.conv1, W.conv2, W.c_norm, W.w_uk, W.w_uv, W.router, W.router_b, W.expert_gu, W.expert_down,
+                  W.qk_bias, W.k_norm, W.sinks, W.table, W.w_dt, W.conv_b, W.decay, W.ssm_d};
     for (void* p : ps) hipFree(p);
   }
   free_mat(S->loop_in); free_mat(S->head);
   free_norm(S->final_norm);
   void* ptrs[] = {S->embed, S->pos, S->x0, S->qkv_out, S->logits_pad, S->n1, S->n2, S->q, S->cat, S->pair, S->attn_scratch, S->residuals,
                   S->y, S->pair_w, S->pair_ids, S->hb, S->act, S->qa, S->lat, S->kv_x, S->kv_k, S->kv_v, S->kv_bt, S->plan,
-                  S->tickets, S->route_z, S->cq, S->low, S->q2, S->z, S->delta_records};
+                  S->tickets, S->route_z, S->cq, S->low, S->q2, S->z, S->delta_records,
+                  S->turns, S->xc, S->xp, S->dtp, S->yssm, S->ssd_records};
   for (void* p : ptrs) hipFree(p);
   for (float* p : S->state_at) hipFree(p);
   for (Stack::RotTable& r : S->rot) hipFree(r.t);
@@ -629,6 +868,13 @@ int stack_load_tensor(mi_ctx* c, const std::string& name, const float* dev, int 
     StackLayer& W = S->layers[l];
     const mi_layer_spec& p = W.s;
     const std::string t = name.substr(at);
+    if (S->post_norm()) {
+      int r = 0, cl = 0;
+      post_norm_tensor_shape(S, W, t, &r, &cl);
+      if (r > 0) return rows == r && cols == cl ? done(post_norm_place(c, W, t, dev, rows, cols)) : bad();
+      set_error("tensor " + name + " is not part of this model's configuration");
+      return MI_EINVAL;
+    }
     if (S->one_norm()) {
       int r = 0, cl = 0;
       if (p.weights_of < 0) one_norm_tensor_shape(S, W, t, &r, &cl);
@@ -681,9 +927,10 @@ int stack_synthetic(mi_ctx* c, uint64_t seed, float std) {
     if (n == "embed" || n == "head") { rows = k.vocab_size; cols = S->D; if (n == "embed") sd = 1.f; }
     else if (n == "pos") { rows = k.max_positions; cols = S->D; sd = 0.1f; }
     else if (n == "loop.in") cols = 2 * S->D;
-    else if (S->one_norm() && n[0] == 'l') {
+    else if ((S->one_norm() || S->post_norm()) && n[0] == 'l') {
       const StackLayer& W = S->layers[atoi(n.c_str() + 1)];
-      one_norm_tensor_shape(S, W, n.substr(n.find('.') + 1), &rows, &cols);
+      if (S->one_norm()) one_norm_tensor_shape(S, W, n.substr(n.find('.') + 1), &rows, &cols);
+      else post_norm_tensor_shape(S, W, n.substr(n.find('.') + 1), &rows, &cols);
       if (n.find(".conv") != std::string::npos) sd = 0.3f;
       is_norm = cols == 0;
     } else if (!is_norm) {
@@ -708,6 +955,7 @@ int stack_synthetic(mi_ctx* c, uint64_t seed, float std) {
     }
     if (is_norm && S->one_norm())     // norms around zero; plain ones; decays, biases and corrections zero
       rc = launch_fill_f32(buf, elems, n.find(".mix.") != std::string::npos && n.find("norm") != std::string::npos ? 1.f : 0.f, c->stream);
+    else if (is_norm && S->post_norm()) rc = launch_fill_f32(buf, elems, n.find("norm") != std::string::npos ? 1.f : 0.f, c->stream);
     else if (is_norm) rc = launch_fill_f32(buf, elems, n.size() > 2 && n.compare(n.size() - 2, 2, ".b") == 0 ? 0.f : 1.f, c->stream);
     else rc = launch_randn(buf, elems, seed, tid, sd, c->stream);
     ++tid;
@@ -729,7 +977,21 @@ void stack_artifact_tensors(mi_ctx* c, std::vector<std::pair<void*, size_t>>& ou
   if (S->cfg.loop_times > 0) mat(S->loop_in);
   for (StackLayer& W : S->layers) {
     if (S->one_norm() && W.s.weights_of >= 0) continue;
-    if (!S->sandwich() && !S->one_norm()) {
+    if (S->post_norm()) {
+      auto put = [&](void* q, size_t elems) { if (q) out.push_back({q, elems * 4}); };
+      const mi_layer_spec& p = W.s;
+      mat(W.qkv); mat(W.out); put(W.n1.w, S->ld); put(W.n2.w, S->ld);
+      for (StackMat* m : {&W.up, &W.down, &W.low_in, &W.dt_mat})
+        if (m->L.w) mat(*m);
+      if (W.w_dt) out.push_back({W.w_dt, (size_t)W.scan.C * W.scan.rank_p * S->elem()});
+      const size_t heads = W.has_scan() ? W.scan.C : W.ssd.H;
+      put(W.decay, (size_t)W.scan.C * W.scan.Np); put(W.dt, heads); put(W.ssm_d, heads); put(W.a_log, heads); put(W.o_norm, W.ssd.inner());
+      put(W.conv, W.ssm_ring_floats()); put(W.conv_b, W.ssm_state_floats() ? W.conv_channels() : 0);
+      put(W.qk_bias, (size_t)(p.num_heads + p.num_kv_heads) * p.qk_dim); put(W.q_norm, p.qk_dim); put(W.k_norm, p.qk_dim);
+      put(W.sinks, p.num_heads); put(W.table, (size_t)p.num_heads * W.table_rows.size());
+      continue;
+    }
+    if (S->parallel()) {
       mat(W.qkv); mat(W.out); norm(W.n1);
       if (W.ff_cols) { mat(W.up); norm(W.n2); }
       continue;
@@ -773,12 +1035,15 @@ int stack_geometry_hash(const mi_ctx* c) {
   mix(g, sizeof g);
   const float f[2] = {k.embed_scale, k.norm_offset};
   if (S->one_norm()) mix(f, sizeof f);
+  const float pf[3] = {k.embed_scale, k.pos_base, k.logit_scale};
+  if (S->post_norm()) mix(pf, sizeof pf);
   for (const StackLayer& W : S->layers) mix(&W.s, sizeof W.s);
   return (int)(h & 0x7fffffff);
 }
 
 static size_t kv_run_elems_per_block(const mi_ctx* c, const StackLayer& W) {
   const Stack* S = c->stack;
+  if (W.has_scan()) return 0;
   if (S->one_norm()) return W.s.mixer_kind == MI_MIX_LATENT ? (size_t)c->cfg.block_size * W.lg.cp : 0;
   if (S->sandwich())   // latents (own ones) and both convolutions' state
     return (W.s.kv_from < 0 ? (size_t)c->cfg.block_size * W.lg.cp : 0) + (size_t)S->conv_keep * S->Kd * (W.s.ff_kind == MI_FF_NONE ? 1 : 2);
@@ -797,7 +1062,8 @@ static size_t stack_scratch(const mi_ctx* c) {
       if (W.fast()) b = std::max(b, latent_attn_scratch_bytes(W.lg));
     return b;
   }
-  for (const StackLayer& W : c->stack->layers) b = std::max(b, attn_window_scratch_bytes(c->cfg.max_num_seqs, W.g));
+  for (const StackLayer& W : c->stack->layers)
+    if (W.g.H) b = std::max(b, attn_window_scratch_bytes(c->cfg.max_num_seqs, W.g));
   return b;
 }
 
@@ -809,15 +1075,22 @@ static int kv_work_rows(const mi_ctx* c) {
 bool stack_has_state(const mi_ctx* c) { return c->stack && c->stack->state_slots > 0; }
 
 static size_t state_floats(const mi_ctx* c, const StackLayer& W) {
+  if (c->stack->post_norm()) return c->stack->state_slots * (W.ssm_state_floats() + W.ssm_ring_floats());
   return W.s.mixer_kind == MI_MIX_DELTA ? c->stack->state_slots * (W.dg.state_floats() + W.dg.ring_floats()) : 0;
 }
 // chunks of prompts whose factors are in memory at a time
 static int delta_chunks(const mi_ctx* c) { return std::min(512, c->max_rows / kDeltaChunk + c->cfg.max_num_seqs); }
 
+static int ssd_chunks(const mi_ctx* c) { return std::min(256, c->max_rows / kSsdChunk + c->cfg.max_num_seqs); }
+
 size_t stack_workspace_estimate(const mi_ctx* c) {
   const Stack* S = c->stack;
   const size_t R = (size_t)c->max_rows;
   size_t extra = 0;
+  if (S->post_norm()) {
+    for (const StackRun& r : S->runs) extra += state_floats(c, S->layers[r.layer]) * 4;
+    extra += R * (size_t)(S->xc_ld + S->low_ld) * S->elem() + R * (size_t)(S->xp_ld + S->dtp_ld + S->yssm_ld) * 4 + (size_t)ssd_chunks(c) * S->ssd_chunk_floats * 4;
+  }
   if (S->one_norm()) {
     for (const StackRun& r : S->runs) extra += state_floats(c, S->layers[r.layer]) * 4;
     if (S->state_slots) extra += (size_t)delta_chunks(c) * S->chunk_floats * 4;
@@ -826,7 +1099,7 @@ size_t stack_workspace_estimate(const mi_ctx* c) {
   }
   size_t b = 3 * R * S->ld * 4 + R * S->qkv_ld * 4 + R * (4 * (size_t)S->Kd + S->q_cols + S->cat_ld) * S->elem();
   b += extra;
-  if (S->sandwich() || S->one_norm()) {
+  if (!S->parallel()) {
     const size_t pairs = R * std::max(1, S->max_top);
     b += (size_t)kv_work_rows(c) * (S->kv_ldx + S->kv_k_cols + S->kv_v_cols) * 2;
     b += pairs * S->ld * 4 + pairs * 16 + R * (S->max_experts + 1) * 4 + R * S->Kd * S->elem() + pairs * S->act_ld * S->elem() + 2 * R * S->lat_cols * S->elem();
@@ -877,6 +1150,40 @@ static int one_norm_alloc(mi_ctx* c) {
   return MI_OK;
 }
 
+// recurrent state, position table and the workspace only post-norm blocks have
+static int post_norm_alloc(mi_ctx* c) {
+  Stack* S = c->stack;
+  const size_t R = (size_t)c->max_rows;
+  size_t* ws = &c->workspace_bytes;
+  for (const StackRun& r : S->runs) {
+    float* p = nullptr;
+    if (const size_t n = state_floats(c, S->layers[r.layer])) MI_TRY(alloc0(c, &p, n * 4, &c->kv_bytes));
+    S->state_at.push_back(p);
+  }
+  if (S->cfg.pos_base > 0.f) MI_TRY(stack_position_turns(S->D, S->cfg.pos_base, &S->turns, c->stream));
+  if (S->xc_ld) MI_TRY(alloc0(c, &S->xc, R * S->xc_ld * S->elem(), ws));
+  if (S->low_ld) {
+    MI_TRY(alloc0(c, &S->low, R * S->low_ld * S->elem(), ws));
+    MI_TRY(alloc0(c, &S->xp, R * S->xp_ld * 4, ws));
+    MI_TRY(alloc0(c, &S->dtp, R * S->dtp_ld * 4, ws));
+  }
+  if (S->yssm_ld) {
+    S->ssd_chunks = ssd_chunks(c);
+    MI_TRY(alloc0(c, &S->yssm, R * S->yssm_ld * 4, ws));
+    MI_TRY(alloc0(c, &S->ssd_records, (size_t)S->ssd_chunks * S->ssd_chunk_floats * 4, ws));
+  }
+  return MI_OK;
+}
+
+int stack_position_turns(int width, float base, double** turns, hipStream_t s) {
+  std::vector<double> t((size_t)(width + 1) / 2);
+  for (size_t i = 0; i < t.size(); ++i) t[i] = std::pow((double)base, -2.0 * (double)i / width) / 6.283185307179586476925286766559;
+  MI_HIP(hipMalloc(reinterpret_cast<void**>(turns), t.size() * 8));
+  MI_HIP(hipMemcpyAsync(*turns, t.data(), t.size() * 8, hipMemcpyHostToDevice, s));
+  MI_HIP(hipStreamSynchronize(s));
+  return MI_OK;
+}
+
 int stack_alloc(mi_ctx* c) {
   Stack* S = c->stack;
   if (!S->missing.empty()) {
@@ -905,12 +1212,13 @@ int stack_alloc(mi_ctx* c) {
     at += kv_run_elems_per_block(c, W) * k.num_blocks;
   }
   if (S->one_norm()) MI_TRY(one_norm_alloc(c));
+  if (S->post_norm()) MI_TRY(post_norm_alloc(c));
   const size_t R = (size_t)c->max_rows;
   size_t* ws = &c->workspace_bytes;
   MI_TRY(alloc0(c, &c->resid[0], R * S->ld * 4, ws));
   MI_TRY(alloc0(c, &c->resid[1], R * S->ld * 4, ws));
   MI_TRY(alloc0(c, &S->n1, R * S->Kd * S->elem(), ws));
-  if (S->sandwich() || S->one_norm()) {
+  if (!S->parallel()) {
     const size_t pairs = R * std::max(1, S->max_top);   // (a dense feed-forward: one "pair" per row)
     MI_TRY(alloc0(c, &S->y, pairs * S->ld * 4, ws));
     MI_TRY(alloc0(c, &S->hb, R * S->Kd * S->elem(), ws));
@@ -1264,6 +1572,143 @@ int one_norm_trunk(mi_ctx* c, const Batch& b, int& cur) {
   return keep(S->runs.size() - 1);
 }
 
+// ---- post-norm blocks ----------------------------------------------------------------------------------------------------------
+int post_norm_conv(mi_ctx* c, const StackLayer& W, float* state, const Batch& b, int col, int ldc) {
+  Stack* S = c->stack;
+  if (!runs_other(c)) return MI_OK;
+  Scope sc(c, MI_K_OTHER);
+  const ShortConv cv{W.conv, W.conv_b, W.s.conv_taps, W.conv_channels(), state + (size_t)S->state_slots * W.ssm_state_floats(), c->d_state};
+  return launch_short_conv(S->qkv_out + col, W.qkv.N, cv, c->d_pos, reinterpret_cast<const AttnSeg*>(c->d_segs), b.segs, b.decode ? 0 : b.nseg, b.rows, S->xc, ldc,
+                           S->f32, c->stream);
+}
+
+int post_norm_scan(mi_ctx* c, const StackLayer& W, float* state, const Batch& b) {
+  Stack* S = c->stack;
+  const ScanGeom& g = W.scan;
+  hipStream_t s = c->stream;
+  EpiArgs e{};
+  e.out_f32 = S->qkv_out; e.ld_out = W.qkv.N;
+  MI_TRY(apply(c, W.qkv, b.rows, S->n1, S->Kd, EPI_F32, e));
+  MI_TRY(post_norm_conv(c, W, state, b, 0, W.low_in.K));
+  EpiArgs x{};
+  x.out_f32 = S->xp; x.ld_out = W.low_in.N;
+  MI_TRY(apply(c, W.low_in, b.rows, S->xc, W.low_in.K, EPI_F32, x));
+  ScanIn in;
+  in.x = S->xc; in.ldx = W.low_in.K;
+  in.low = S->xp; in.ldl = W.low_in.N; in.col_b = W.col_B; in.col_c = W.col_C;
+  in.dt = S->dtp; in.ldt = W.dt_mat.N; in.w_dt = W.w_dt;
+  in.dt_bias = W.dt; in.a2 = W.decay; in.d = W.ssm_d;
+  in.z = S->qkv_out + W.col_z; in.ldz = W.qkv.N;
+  in.state = state; in.slots = c->d_state; in.pos = c->d_pos;
+  int ones = 0;
+  for (int i = 0; i < b.nseg; ++i) ones += b.segs[i].n == 1;
+  const bool prompts = !b.decode && ones < b.nseg;
+  if (prompts) {
+    if (runs_other(c)) {
+      Scope sc(c, MI_K_OTHER);
+      MI_TRY(launch_columns(S->xp, W.low_in.N, {0, g.rank, nullptr, S->low}, {}, 0.f, b.rows, W.dt_mat.K, S->f32, s));
+    }
+    EpiArgs z{};
+    z.out_f32 = S->dtp; z.ld_out = W.dt_mat.N;
+    MI_TRY(apply(c, W.dt_mat, b.rows, S->low, W.dt_mat.K, EPI_F32, z));
+  }
+  const int cls = b.decode ? MI_K_ATTN_DECODE : MI_K_ATTN_PREFILL;
+  if (!c->runs(cls)) return MI_OK;
+  Scope sc(c, cls);
+  if (b.decode) return launch_scan_token(g, in, b.rows, nullptr, S->cat, S->cat_ld, S->f32, s);
+  const AttnSeg* segs = reinterpret_cast<const AttnSeg*>(c->d_segs);
+  if (ones) MI_TRY(launch_scan_token(g, in, b.nseg, segs, S->cat, S->cat_ld, S->f32, s));
+  if (prompts) MI_TRY(launch_scan_prompt(g, in, segs, b.nseg, S->cat, S->cat_ld, S->f32, s));
+  return MI_OK;
+}
+
+// the second mixer of x beside attention: columns attn_cols .. of the concatenated row
+int post_norm_ssd(mi_ctx* c, const StackLayer& W, float* state, const Batch& b) {
+  Stack* S = c->stack;
+  const SsdGeom& g = W.ssd;
+  hipStream_t s = c->stream;
+  const int ldc = pad_to(g.channels(), 16), ldy = pad_to(g.inner(), 16);
+  MI_TRY(post_norm_conv(c, W, state, b, W.col_x, ldc));
+  SsdIn in;
+  in.xbc = S->xc; in.ldx = ldc;
+  in.dt = S->qkv_out + W.col_dt; in.ldt = W.qkv.N;
+  in.dt_bias = W.dt; in.a_log = W.a_log; in.d = W.ssm_d;
+  in.state = state; in.slots = c->d_state; in.pos = c->d_pos;
+  const int cls = b.decode ? MI_K_ATTN_DECODE : MI_K_ATTN_PREFILL;
+  if (c->runs(cls)) {
+    Scope sc(c, cls);
+    if (b.decode) {
+      MI_TRY(launch_ssd_token(g, in, b.rows, nullptr, S->yssm, ldy, S->f32, s));
+    } else {
+      int ones = 0;
+      for (int i = 0; i < b.nseg; ++i) ones += b.segs[i].n == 1;
+      const AttnSeg* segs = reinterpret_cast<const AttnSeg*>(c->d_segs);
+      if (ones) MI_TRY(launch_ssd_token(g, in, b.nseg, segs, S->yssm, ldy, S->f32, s));
+      if (ones < b.nseg) MI_TRY(launch_ssd_prompt(g, in, segs, b.segs, b.nseg, S->ssd_records, S->ssd_chunks, S->yssm, ldy, S->f32, s));
+    }
+  }
+  if (!runs_other(c)) return MI_OK;
+  Scope sc(c, MI_K_OTHER);
+  void* out = reinterpret_cast<unsigned char*>(S->cat) + (size_t)W.attn_cols * S->elem();
+  return launch_gated_norm(S->yssm, ldy, S->qkv_out + W.col_z, W.qkv.N, W.o_norm, g.inner(), W.s.ssm_parts, S->cfg.norm_eps, b.rows, out, S->cat_ld, S->f32, s);
+}
+
+int post_norm_trunk(mi_ctx* c, const Batch& b, int& cur) {
+  Stack* S = c->stack;
+  RowSource src;
+  const float* w_post = nullptr;
+  auto keep = [&](size_t run) -> int {
+    if (S->residuals)
+      MI_HIP(hipMemcpyAsync(S->residuals + run * c->max_rows * S->ld, c->resid[cur], (size_t)b.rows * S->ld * 4, hipMemcpyDeviceToDevice, c->stream));
+    return MI_OK;
+  };
+  // x += norm of the sublayer's output; x in the compute type -> S->n1
+  auto row = [&]() -> int {
+    if (runs_other(c)) {
+      Scope sc(c, MI_K_OTHER);
+      MI_TRY(launch_sandwich_rows(c->resid[cur], c->resid[cur ^ 1], src, w_post, nullptr, b.rows, S->D, S->ld, 1, S->cfg.norm_eps, nullptr, S->n1, S->Kd, S->f32,
+                                  c->stream, true));
+    }
+    cur ^= 1;
+    src = RowSource();
+    return MI_OK;
+  };
+  // a sublayer's output rows -> src
+  auto project = [&](const StackMat& m, const void* x, int ldx, const float* w) -> int {
+    EpiArgs e{};
+    e.out_f32 = S->y; e.ld_out = S->ld;
+    src.y = S->y; src.ld = S->ld;
+    w_post = w;
+    return apply(c, m, b.rows, x, ldx, EPI_F32, e, b.rows >= 384 ? &src.slabs : nullptr);
+  };
+  for (size_t i = 0; i < S->runs.size(); ++i) {
+    const StackLayer& W = S->layers[S->runs[i].layer];
+    if (i > 0) {
+      MI_TRY(row());
+      MI_TRY(keep(i - 1));
+    }
+    if (W.has_scan()) {
+      MI_TRY(post_norm_scan(c, W, S->state_at[i], b));
+    } else {
+      EpiArgs e{};
+      e.out_f32 = S->qkv_out; e.ld_out = W.qkv.N;
+      MI_TRY(apply(c, W.qkv, b.rows, S->n1, S->Kd, EPI_F32, e));
+      const OutGate gate{W.s.out_gate ? S->qkv_out + W.col_g : nullptr, W.qkv.N, false, W.s.mix_mult};
+      MI_TRY(attention(c, W, S->kv_at[i], W.qkv.N, b.rows, b.decode, b.MB, b.segs, b.nseg, gate));
+      if (W.has_ssd()) MI_TRY(post_norm_ssd(c, W, S->state_at[i], b));
+    }
+    MI_TRY(project(W.out, S->cat, S->cat_ld, W.n1.w));
+    if (W.s.ff_kind == MI_FF_NONE) continue;
+    MI_TRY(row());
+    EpiArgs u{};
+    u.act_out = reinterpret_cast<uint16_t*>(S->act); u.ld_act = S->act_ld;
+    MI_TRY(apply(c, W.up, b.rows, S->n1, S->Kd, EPI_RELU2, u));
+    MI_TRY(project(W.down, S->act, S->act_ld, W.n2.w));
+  }
+  MI_TRY(row());
+  return keep(S->runs.size() - 1);
+}
+
 }  // namespace
 
 int stack_trunk(mi_ctx* c, int rows, bool decode, int MB, const AttnSeg* segs, int nseg) {
@@ -1273,7 +1718,13 @@ int stack_trunk(mi_ctx* c, int rows, bool decode, int MB, const AttnSeg* segs, i
   int cur = 0;
   if (runs_other(c)) {
     Scope sc(c, MI_K_OTHER);
-    MI_TRY(launch_embed_pos(c->d_ids, c->d_pos, S->embed, S->pos, S->cfg.embed_scale, S->f32, rows, S->D, S->ld, c->resid[0], S->x0, s));
+    MI_TRY(launch_embed_pos(c->d_ids, c->d_pos, S->embed, S->pos, S->cfg.embed_scale, S->f32, rows, S->D, S->ld, c->resid[0], S->x0, s, S->turns,
+                            S->post_norm() ? S->n1 : nullptr, S->Kd));
+  }
+  if (S->post_norm()) {
+    MI_TRY(post_norm_trunk(c, Batch{rows, decode, MB, segs, nseg}, cur));
+    c->tail_cur = cur;
+    return MI_OK;
   }
   if (S->one_norm()) {
     MI_TRY(one_norm_trunk(c, Batch{rows, decode, MB, segs, nseg}, cur));
@@ -1308,7 +1759,7 @@ int stack_trunk(mi_ctx* c, int rows, bool decode, int MB, const AttnSeg* segs, i
       e.out_f32 = S->qkv_out; e.ld_out = S->qkv_ld;
       MI_TRY(apply(c, W.qkv, rows, S->n1, S->Kd, EPI_F32, e));
     }
-    MI_TRY(attention(c, W, S->kv_at[i], rows, decode, MB, segs, nseg));
+    MI_TRY(attention(c, W, S->kv_at[i], S->qkv_ld, rows, decode, MB, segs, nseg));
     if (W.ff_cols) {
       EpiArgs e{};
       e.act_out = reinterpret_cast<uint16_t*>(reinterpret_cast<unsigned char*>(S->cat) + (size_t)W.attn_cols * S->elem());

@@ -1,6 +1,6 @@
-// Row-wise kernels of the layer-stack decoders (stack.hip): embedding with learned positions, layer norm with up to
+// Row-wise kernels of the layer-stack decoders (stack.hip): embedding with learned or sinusoidal positions, layer norm with up to
 // two affine outputs, the sandwich block's row (post-norm, residual sum, pre-norm, causal convolution), the looped stack's
-// input, per-head unit norm with the KV scatter, and the 32-bit linear layer.
+// input, per-head norms with the KV scatter, and the 32-bit linear layer.
 // Every kernel takes its activations as bf16 (`f32 = false`) or fp32 (`f32 = true`: the 32-bit compute mode).
 #pragma once
 #include "linear_kernels.h"
@@ -9,9 +9,10 @@ namespace mi {
 
 struct AttnSeg { int row0, n, pos0, seq; };   // rows row0 .. + n of the batch = positions pos0 .. of the sequence in block-table row seq
 
-// resid[t, :] = scale E[ids[t], :] (+ P[pos[t], :], ptable not null) in fp32, also to x0 when given; columns D .. ld - 1 are zero
+// resid[t, :] = scale E[ids[t], :] (+ P[pos[t], :], ptable not null) in fp32, also to x0 when given; columns D .. ld - 1 are zero.
+// turns [ceil(D / 2)] (not null): + sin / cos of 2 pi pos[t] turns[i] at elements 2 i / 2 i + 1.  y [T, ldy] (not null): the same row in the compute type
 int launch_embed_pos(const int32_t* ids, const int32_t* pos, const void* table, const void* ptable, float scale, bool f32, int T,
-                     int D, int ld, float* resid, float* x0, hipStream_t s);
+                     int D, int ld, float* resid, float* x0, hipStream_t s, const double* turns = nullptr, void* y = nullptr, int ldy = 0);
 
 struct NormOut {
   const float* w = nullptr;   // [ld], zero beyond D
@@ -45,9 +46,9 @@ struct ConvState {
   const int32_t *bt = nullptr, *pos = nullptr, *slots = nullptr;
 };
 // resid_out = resid_in (+ post-normed src; w_post null: + src as it is); then, with w_pre, y [T, ldy] = h in the compute type, or (conv, every row its own
-// sequence: block-table row = row) a with the state read and renewed.  Without w_pre only the residual sum.
+// sequence: block-table row = row) a with the state read and renewed.  Without w_pre only the residual sum, or (as_is) y = that row itself.
 int launch_sandwich_rows(const float* resid_in, float* resid_out, const RowSource& src, const float* w_post, const float* w_pre, int T,
-                         int D, int ld, int groups, float eps, const ConvState* conv, void* y, int ldy, bool f32, hipStream_t s);
+                         int D, int ld, int groups, float eps, const ConvState* conv, void* y, int ldy, bool f32, hipStream_t s, bool as_is = false);
 // a = h + conv(h) over a ragged batch: h [T, ldy] as launch_sandwich_rows leaves it
 int launch_conv_rows(const void* h, const ConvState& conv, const AttnSeg* segs_dev, const AttnSeg* segs_host, int nseg, int D, int ld,
                      void* y, int ldy, bool f32, hipStream_t s);
@@ -57,8 +58,9 @@ struct Columns { int col = 0, n = 0; const float* w = nullptr; void* y = nullptr
 int launch_columns(const float* x, int ld, Columns a, Columns b, float eps, int T, int ldy, bool f32, hipStream_t s);   // b.y null: a alone
 // y[t, h dv + d] *= sigmoid(g[t, ...]): one gate per head, or (per_element) per element; g [T, ldg] fp32, y [T, ldy] in the compute type
 int launch_gate_rows(void* y, int ldy, int T, int H, int dv, const float* g, int ldg, bool per_element, bool f32, hipStream_t s);
-// dst = src + offset
+// dst = src + offset;  dst = src factor
 int launch_offset_copy(const float* src, int n, float offset, float* dst, hipStream_t s);
+int launch_scaled_copy(const float* src, int n, float factor, float* dst, hipStream_t s);
 
 // y[t] = [x ; x0] in the compute type, the second half at column half
 int launch_pair_rows(const float* x, const float* x0, int T, int D, int ld, int half, void* y, bool f32, hipStream_t s);
@@ -67,9 +69,15 @@ int launch_pair_rows(const float* x, const float* x0, int T, int D, int ld, int 
 struct HeadGeom {
   int H = 0, G = 0, dk = 0, dv = 0, dkp = 0, dvp = 0;
 };
-// qkv [T, ldq] fp32 (q heads, k heads, v heads) -> q [T, H, dkp], K / V pool rows at slots (-1: not written).
-// unit_norm: q and k heads over sqrt(mean square + eps)
-int launch_qkv_scatter(const float* qkv, int ldq, int T, const HeadGeom& g, bool unit_norm, float eps, const int32_t* slots,
+// What happens to the projected heads on their way to the query buffer and the pools
+struct HeadRule {
+  bool unit_norm = false;          // q and k heads over sqrt(mean square + eps) ...
+  const float *q_norm = nullptr, *k_norm = nullptr;   // ... times a weight per element [dk] (null: 1)
+  const float* bias = nullptr;     // [H dk + G dk] added to the q and k heads first (null: none)
+  bool keys_as_values = false;     // no v heads: a value is the key ahead of its norm (dv = dk)
+};
+// qkv [T, ldq] fp32 (q heads, k heads, v heads) -> q [T, H, dkp], K / V pool rows at slots (-1: not written)
+int launch_qkv_scatter(const float* qkv, int ldq, int T, const HeadGeom& g, const HeadRule& rule, float eps, const int32_t* slots,
                        int block_size, void* q, void* kpool, void* vpool, bool f32, hipStream_t s);
 
 // y[m, n] = scale[n] sum_k x[m, k] w[n, k] in true fp32, epilogues EPI_F32 / EPI_RESID / EPI_RELU2 / EPI_GLU_CLIP / EPI_SOFTCAP

@@ -35,7 +35,8 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
 template <typename T>
 __global__ __launch_bounds__(256) void embed_pos_kernel(const int32_t* __restrict__ ids, const int32_t* __restrict__ pos,
                                                         const T* __restrict__ table, const T* __restrict__ ptable, float sc, int D, int ld,
-                                                        float* __restrict__ resid, float* __restrict__ x0) {
+                                                        float* __restrict__ resid, float* __restrict__ x0, const double* __restrict__ turns,
+                                                        T* __restrict__ y, int ldy) {
   const int t = blockIdx.x;
   const T* e = table + (size_t)ids[t] * D;
   const T* p = ptable ? ptable + (size_t)pos[t] * D : nullptr;
@@ -50,6 +51,18 @@ __global__ __launch_bounds__(256) void embed_pos_kernel(const int32_t* __restric
       auto at = [&](int i) { return d + i < D ? __builtin_fmaf(sc, to_f32(e[d + i]), p ? to_f32(p[d + i]) : 0.f) : 0.f; };
       v = make_float4(at(0), at(1), at(2), at(3));
     }
+    if (turns) {       // the angle in whole turns, its fraction exact in fp64
+      const double p0 = (double)pos[t];
+      float sn[2] = {0.f, 0.f}, cs[2] = {0.f, 0.f};
+#pragma unroll
+      for (int i = 0; i < 2; ++i)
+        if (d + 2 * i < D) {
+          const double a = p0 * turns[d / 2 + i];
+          sincospif((float)(2.0 * (a - floor(a))), &sn[i], &cs[i]);
+        }
+      v = make_float4(v.x + sn[0], d + 1 < D ? v.y + cs[0] : 0.f, v.z + sn[1], d + 3 < D ? v.w + cs[1] : 0.f);
+    }
+    if (y) put4(y + (size_t)t * ldy + d, v.x, v.y, v.z, v.w);
     *reinterpret_cast<float4*>(resid + (size_t)t * ld + d) = v;
     if (x0) *reinterpret_cast<float4*>(x0 + (size_t)t * ld + d) = v;
   }
@@ -184,7 +197,7 @@ __device__ __forceinline__ float4 ring_get4(const ConvState& cs, int seq, int p,
 template <typename T>
 __global__ __launch_bounds__(1024) void sandwich_rows_kernel(const float* __restrict__ resid_in, float* __restrict__ resid_out, RowSource src,
                                                             const float* __restrict__ w_post, const float* __restrict__ w_pre, int D, int ld,
-                                                            int G, float eps, ConvState cs, T* __restrict__ y, int ldy) {
+                                                            int G, float eps, ConvState cs, T* __restrict__ y, int ldy, bool as_is) {
   extern __shared__ __attribute__((aligned(16))) float row[];   // ld + max(G, 16) + G floats
   float *red = row + ld, *rstd = red + max(G, 16);
   const int t = blockIdx.x, tid = threadIdx.x, nthr = blockDim.x;
@@ -207,6 +220,7 @@ __global__ __launch_bounds__(1024) void sandwich_rows_kernel(const float* __rest
       x.z = __builtin_fmaf(v.z * r.z, w.z, x.z); x.w = __builtin_fmaf(v.w * r.w, w.w, x.w);
       *reinterpret_cast<float4*>(resid_out + o + d) = x;
     }
+    if (as_is) put4(y + (size_t)t * ldy + d, x.x, x.y, x.z, x.w);
     *reinterpret_cast<float4*>(row + d) = x;
   }
   if (!w_pre) return;
@@ -246,7 +260,7 @@ __global__ __launch_bounds__(1024) void sandwich_token_kernel(const float* __res
   const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
   float4 x = *reinterpret_cast<const float4*>(resid_in + (size_t)t * ld + dd);
   float4 v = add ? source_row4(src, t, dd) : zero;
-  const float4 wp = add && w_post ? *reinterpret_cast<const float4*>(w_post + dd) : zero, wn = *reinterpret_cast<const float4*>(w_pre + dd);
+  const float4 wp = add && w_post ? *reinterpret_cast<const float4*>(w_post + dd) : zero, wn = w_pre ? *reinterpret_cast<const float4*>(w_pre + dd) : zero;
   float4 w[TAPS > 0 ? TAPS : 1];
   raw_t past[TAPS > 1 ? TAPS - 1 : 1];
   int slot = -1;
@@ -279,6 +293,10 @@ __global__ __launch_bounds__(1024) void sandwich_token_kernel(const float* __res
     x.x = __builtin_fmaf(v.x * r, wp.x, x.x); x.y = __builtin_fmaf(v.y * r, wp.y, x.y);
     x.z = __builtin_fmaf(v.z * r, wp.z, x.z); x.w = __builtin_fmaf(v.w * r, wp.w, x.w);
     if (in) *reinterpret_cast<float4*>(resid_out + (size_t)t * ld + d) = x;
+  }
+  if (!w_pre) {         // (the row itself)
+    if (in) put4(y + (size_t)t * ldy + d, x.x, x.y, x.z, x.w);
+    return;
   }
   const float r = rstd(in ? x : zero, red[1]);
   if (!in) return;
@@ -473,9 +491,9 @@ __global__ __launch_bounds__(256) void gate_rows_kernel(T* __restrict__ y, int l
   for (int i = blockIdx.y * 256 + threadIdx.x; i < n; i += gridDim.y * 256)
     gate1(y + (size_t)t * ldy + i, 1.f / (1.f + expf(-g[(size_t)t * ldg + (ELEM ? i : i / dv)])));
 }
-__global__ void offset_copy_kernel(const float* __restrict__ src, int n, float offset, float* __restrict__ dst) {
+__global__ void affine_copy_kernel(const float* __restrict__ src, int n, float factor, float offset, float* __restrict__ dst) {
   const int i = blockIdx.x * blockDim.x + threadIdx.x;
-  if (i < n) dst[i] = src[i] + offset;
+  if (i < n) dst[i] = __builtin_fmaf(src[i], factor, offset);
 }
 
 template <typename T>
@@ -491,36 +509,48 @@ __global__ __launch_bounds__(256) void pair_rows_kernel(const float* __restrict_
   }
 }
 
-// 32 lanes per head: H q heads, G k heads, G v heads of one token row
+// 32 lanes per head: H q heads, G k heads, G v heads (keys_as_values: none, the k heads write both pools) of one token row
 template <typename T>
-__global__ __launch_bounds__(256) void qkv_scatter_kernel(const float* __restrict__ qkv, int ldq, HeadGeom g, int unit_norm, float eps,
+__global__ __launch_bounds__(256) void qkv_scatter_kernel(const float* __restrict__ qkv, int ldq, HeadGeom g, HeadRule rule, float eps,
                                                           const int32_t* __restrict__ slots, int bs, T* __restrict__ q,
                                                           T* __restrict__ kpool, T* __restrict__ vpool) {
   const int t = blockIdx.x, head = blockIdx.y * 8 + (threadIdx.x >> 5), l = threadIdx.x & 31;
-  if (head >= g.H + 2 * g.G) return;     // (whole 32-lane group: the shuffles below stay inside it)
+  if (head >= g.H + (rule.keys_as_values ? 1 : 2) * g.G) return;     // (whole 32-lane group: the shuffles below stay inside it)
   const bool is_q = head < g.H, is_v = head >= g.H + g.G;
   const int kvh = is_v ? head - g.H - g.G : head - g.H;
   const int d_n = is_v ? g.dv : g.dk, d_p = is_v ? g.dvp : g.dkp;
   const float* src = qkv + (size_t)t * ldq + (is_v ? (size_t)(g.H + g.G) * g.dk + (size_t)kvh * g.dv : (size_t)head * g.dk);
+  const float* bias = rule.bias && !is_v ? rule.bias + (size_t)head * g.dk : nullptr;
+  const float* w = is_v ? nullptr : is_q ? rule.q_norm : rule.k_norm;
   const bool vec = (d_n & 3) == 0 && (((is_v ? (g.H + g.G) * g.dk : 0)) & 3) == 0;
-  T* dst;
+  T *dst, *raw = nullptr;
   if (is_q) {
     dst = q + ((size_t)t * g.H + head) * g.dkp;
   } else {
     const int slot = slots[t];
     if (slot < 0) return;
     const int blk = slot / bs, off = slot - blk * bs;
-    dst = (is_v ? vpool : kpool) + (((size_t)blk * g.G + kvh) * bs + off) * d_p;
+    const size_t r = ((size_t)blk * g.G + kvh) * bs + off;
+    dst = (is_v ? vpool : kpool) + r * d_p;
+    if (rule.keys_as_values) raw = vpool + r * d_p;
   }
-  auto get = [&](int d) -> float4 {
-    if (vec) return d < d_n ? *reinterpret_cast<const float4*>(src + d) : make_float4(0.f, 0.f, 0.f, 0.f);
-    return make_float4(d < d_n ? src[d] : 0.f, d + 1 < d_n ? src[d + 1] : 0.f, d + 2 < d_n ? src[d + 2] : 0.f, d + 3 < d_n ? src[d + 3] : 0.f);
+  auto get = [&](const float* p, int d) -> float4 {
+    if (vec) return d < d_n ? *reinterpret_cast<const float4*>(p + d) : make_float4(0.f, 0.f, 0.f, 0.f);
+    return make_float4(d < d_n ? p[d] : 0.f, d + 1 < d_n ? p[d + 1] : 0.f, d + 2 < d_n ? p[d + 2] : 0.f, d + 3 < d_n ? p[d + 3] : 0.f);
+  };
+  auto value = [&](int d) -> float4 {
+    float4 v = get(src, d);
+    if (bias) {
+      const float4 b = get(bias, d);
+      v = make_float4(v.x + b.x, v.y + b.y, v.z + b.z, v.w + b.w);
+    }
+    return v;
   };
   float f = 1.f;
-  if (!is_v && unit_norm) {
+  if (!is_v && rule.unit_norm) {
     float ss = 0.f;
     for (int d = l * 4; d < d_n; d += 128) {
-      const float4 v = get(d);
+      const float4 v = value(d);
       ss += (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
     }
 #pragma unroll
@@ -528,8 +558,9 @@ __global__ __launch_bounds__(256) void qkv_scatter_kernel(const float* __restric
     f = 1.0f / sqrtf(ss / (float)d_n + eps);
   }
   for (int d = l * 4; d < d_p; d += 128) {
-    const float4 v = get(d);
-    put4(dst + d, v.x * f, v.y * f, v.z * f, v.w * f);
+    const float4 v = value(d), k = w ? get(w, d) : make_float4(1.f, 1.f, 1.f, 1.f);
+    put4(dst + d, v.x * f * k.x, v.y * f * k.y, v.z * f * k.z, v.w * f * k.w);
+    if (raw) put4(raw + d, v.x, v.y, v.z, v.w);
   }
 }
 
@@ -628,11 +659,12 @@ __global__ void pack_rows_kernel(const float* __restrict__ src, int ld_src, int 
 }  // namespace
 
 int launch_embed_pos(const int32_t* ids, const int32_t* pos, const void* table, const void* ptable, float scale, bool f32, int T, int D,
-                     int ld, float* resid, float* x0, hipStream_t s) {
+                     int ld, float* resid, float* x0, hipStream_t s, const double* turns, void* y, int ldy) {
+  MI_CHECK(!y || (ldy >= ld && ldy % 4 == 0), "embedding: output stride");
   if (f32)
-    hipLaunchKernelGGL((embed_pos_kernel<float>), dim3(T), dim3(256), 0, s, ids, pos, (const float*)table, (const float*)ptable, scale, D, ld, resid, x0);
+    hipLaunchKernelGGL((embed_pos_kernel<float>), dim3(T), dim3(256), 0, s, ids, pos, (const float*)table, (const float*)ptable, scale, D, ld, resid, x0, turns, (float*)y, ldy);
   else
-    hipLaunchKernelGGL((embed_pos_kernel<uint16_t>), dim3(T), dim3(256), 0, s, ids, pos, (const uint16_t*)table, (const uint16_t*)ptable, scale, D, ld, resid, x0);
+    hipLaunchKernelGGL((embed_pos_kernel<uint16_t>), dim3(T), dim3(256), 0, s, ids, pos, (const uint16_t*)table, (const uint16_t*)ptable, scale, D, ld, resid, x0, turns, (uint16_t*)y, ldy);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
@@ -661,20 +693,21 @@ static int check_conv(const ConvState& c) {
 }
 
 int launch_sandwich_rows(const float* resid_in, float* resid_out, const RowSource& src, const float* w_post, const float* w_pre, int T,
-                         int D, int ld, int groups, float eps, const ConvState* conv, void* y, int ldy, bool f32, hipStream_t s) {
+                         int D, int ld, int groups, float eps, const ConvState* conv, void* y, int ldy, bool f32, hipStream_t s, bool as_is) {
+  MI_CHECK(!as_is || !w_pre, "sandwich rows: a pre-norm, or the row as it is");
   MI_CHECK(T >= 1 && ld % 4 == 0 && ld >= D && ld <= 32768 && groups >= 1 && D % groups == 0, "sandwich rows: row stride / norm groups");
   MI_CHECK(!src.any() || (resid_out && resid_out != resid_in), "sandwich rows: residual output");
   MI_CHECK(!src.slabs.slab || (src.slabs.T == T && src.slabs.N == ld && !src.slabs.bias && !src.slabs.row_scale), "sandwich rows: pending K-split sum of another shape");
   MI_CHECK(src.slabs.slab || !src.any() || src.ld >= ld, "sandwich rows: source stride");
   MI_CHECK(!src.y16 || src.pair_w, "sandwich rows: bf16 sources are built for experts");
-  MI_CHECK(!w_pre || (y && ldy >= ld && ldy % 4 == 0), "sandwich rows: output stride");
+  MI_CHECK(!(w_pre || as_is) || (y && ldy >= ld && ldy % 4 == 0), "sandwich rows: output stride");
   ConvState cs;
   if (conv) {
     int rc = check_conv(*conv);
     if (rc != MI_OK) return rc;
     cs = *conv;
   }
-  if (T <= 32 && w_pre && ld <= 4096 && ld == D && (D / groups) % 256 == 0 && (!conv || conv->taps <= 4)) {
+  if (T <= 32 && (w_pre || as_is) && ld <= 4096 && ld == D && (D / groups) % 256 == 0 && (!conv || conv->taps <= 4)) {
     const int threads = ceil_div(ld / 4, 64) * 64, gs = D / groups;
 #define MI_TOKEN(TAPS) \
     if (f32) hipLaunchKernelGGL((sandwich_token_kernel<float, TAPS>), dim3(T), dim3(threads), 0, s, resid_in, resid_out, src, w_post, w_pre, D, ld, gs, eps, cs, (float*)y, ldy); \
@@ -695,8 +728,8 @@ int launch_sandwich_rows(const float* resid_in, float* resid_out, const RowSourc
   const void* kern = f32 ? reinterpret_cast<const void*>(sandwich_rows_kernel<float>) : reinterpret_cast<const void*>(sandwich_rows_kernel<uint16_t>);
   MI_CHECK(lds <= 160 * 1024, "sandwich rows: row too long");
   if (lds > 64 * 1024) { int rc = ensure_dynamic_lds(kern, 160 * 1024); if (rc != MI_OK) return rc; }
-  if (f32) hipLaunchKernelGGL((sandwich_rows_kernel<float>), dim3(T), dim3(threads), lds, s, resid_in, resid_out, src, w_post, w_pre, D, ld, groups, eps, cs, (float*)y, ldy);
-  else hipLaunchKernelGGL((sandwich_rows_kernel<uint16_t>), dim3(T), dim3(threads), lds, s, resid_in, resid_out, src, w_post, w_pre, D, ld, groups, eps, cs, (uint16_t*)y, ldy);
+  if (f32) hipLaunchKernelGGL((sandwich_rows_kernel<float>), dim3(T), dim3(threads), lds, s, resid_in, resid_out, src, w_post, w_pre, D, ld, groups, eps, cs, (float*)y, ldy, as_is);
+  else hipLaunchKernelGGL((sandwich_rows_kernel<uint16_t>), dim3(T), dim3(threads), lds, s, resid_in, resid_out, src, w_post, w_pre, D, ld, groups, eps, cs, (uint16_t*)y, ldy, as_is);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
@@ -750,7 +783,13 @@ int launch_gate_rows(void* y, int ldy, int T, int H, int dv, const float* g, int
 
 int launch_offset_copy(const float* src, int n, float offset, float* dst, hipStream_t s) {
   MI_CHECK(n >= 1, "offset copy: size");
-  hipLaunchKernelGGL(offset_copy_kernel, dim3(ceil_div(n, 256)), dim3(256), 0, s, src, n, offset, dst);
+  hipLaunchKernelGGL(affine_copy_kernel, dim3(ceil_div(n, 256)), dim3(256), 0, s, src, n, 1.f, offset, dst);
+  MI_HIP(hipGetLastError());
+  return MI_OK;
+}
+int launch_scaled_copy(const float* src, int n, float factor, float* dst, hipStream_t s) {
+  MI_CHECK(n >= 1, "scaled copy: size");
+  hipLaunchKernelGGL(affine_copy_kernel, dim3(ceil_div(n, 256)), dim3(256), 0, s, src, n, factor, 0.f, dst);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
@@ -763,13 +802,15 @@ int launch_pair_rows(const float* x, const float* x0, int T, int D, int ld, int 
   return MI_OK;
 }
 
-int launch_qkv_scatter(const float* qkv, int ldq, int T, const HeadGeom& g, bool unit_norm, float eps, const int32_t* slots,
+int launch_qkv_scatter(const float* qkv, int ldq, int T, const HeadGeom& g, const HeadRule& rule, float eps, const int32_t* slots,
                        int block_size, void* q, void* kpool, void* vpool, bool f32, hipStream_t s) {
-  MI_CHECK(ldq % 4 == 0 && ldq >= (g.H + g.G) * g.dk + g.G * g.dv && g.dkp % 16 == 0 && g.dvp % 16 == 0 && g.dkp >= g.dk && g.dvp >= g.dv,
+  MI_CHECK(!rule.keys_as_values || (g.dv == g.dk && g.dvp == g.dkp), "qkv scatter: values that are the keys have their size");
+  MI_CHECK(rule.unit_norm || (!rule.q_norm && !rule.k_norm), "qkv scatter: norm weights without a norm");
+  MI_CHECK(ldq % 4 == 0 && ldq >= (g.H + g.G) * g.dk + (rule.keys_as_values ? 0 : g.G * g.dv) && g.dkp % 16 == 0 && g.dvp % 16 == 0 && g.dkp >= g.dk && g.dvp >= g.dv,
            "qkv scatter: geometry");
   const dim3 grid(T, ceil_div(g.H + 2 * g.G, 8));
-  if (f32) hipLaunchKernelGGL((qkv_scatter_kernel<float>), grid, dim3(256), 0, s, qkv, ldq, g, (int)unit_norm, eps, slots, block_size, (float*)q, (float*)kpool, (float*)vpool);
-  else hipLaunchKernelGGL((qkv_scatter_kernel<uint16_t>), grid, dim3(256), 0, s, qkv, ldq, g, (int)unit_norm, eps, slots, block_size, (uint16_t*)q, (uint16_t*)kpool, (uint16_t*)vpool);
+  if (f32) hipLaunchKernelGGL((qkv_scatter_kernel<float>), grid, dim3(256), 0, s, qkv, ldq, g, rule, eps, slots, block_size, (float*)q, (float*)kpool, (float*)vpool);
+  else hipLaunchKernelGGL((qkv_scatter_kernel<uint16_t>), grid, dim3(256), 0, s, qkv, ldq, g, rule, eps, slots, block_size, (uint16_t*)q, (uint16_t*)kpool, (uint16_t*)vpool);
   MI_HIP(hipGetLastError());
   return MI_OK;
 }

@@ -1,4 +1,4 @@
-// Per-kernel entry points of the sandwich block's mechanisms (include/mi355x_vllm.h: tests and micro-benchmarks): weights are
+// Per-kernel entry points of the sandwich, one-norm and post-norm blocks' mechanisms (include/mi355x_vllm.h: tests and micro-benchmarks): weights are
 // placed here the way stack.hip places a layer's, then the launchers the model call uses run on the caller's data.
 #include <algorithm>
 #include <cstring>
@@ -212,6 +212,138 @@ int mi_op_delta_rule(const mi_layer_spec* spec, const float* proj, int32_t ldp, 
   }
   MI_HIP(hipStreamSynchronize(s));
   return MI_OK;
+}
+
+// sequences of a recurrent mixer's step: slots and positions on the device
+static int take_sequences(Arena& mem, int32_t num_slots, const int32_t* slots_host, const int32_t* pos_host, const int32_t* segs_host, int nseg, int T,
+                          std::vector<AttnSeg>& segs, AttnSeg** sd, int32_t** slots, int32_t** pos, hipStream_t s) {
+  MI_CHECK(slots_host && pos_host && T >= 1 && nseg >= 0 && (nseg == 0 || segs_host), "sequences: null argument");
+  const int seqs = nseg ? nseg : T;
+  for (int i = 0; i < seqs; ++i) MI_CHECK(slots_host[i] >= 0 && slots_host[i] < num_slots, "state slot out of range");
+  for (int i = 0; i < T; ++i) MI_CHECK(pos_host[i] >= 0, "position");
+  if (nseg) {
+    MI_TRY(take_segs(mem, segs_host, nseg, T, 16, 1 << 20, segs, sd, s));
+    for (const AttnSeg& x : segs) MI_CHECK(x.seq < seqs, "segments: sequence");
+  }
+  MI_TRY(mem.take(slots, (size_t)seqs * 4, s));
+  MI_TRY(mem.take(pos, (size_t)T * 4, s));
+  MI_HIP(hipMemcpyAsync(*slots, slots_host, (size_t)seqs * 4, hipMemcpyHostToDevice, s));
+  MI_HIP(hipMemcpyAsync(*pos, pos_host, (size_t)T * 4, hipMemcpyHostToDevice, s));
+  return MI_OK;
+}
+
+int mi_op_embed_sinusoid(const int32_t* ids, const int32_t* pos, const void* table, float scale, float pos_base, int32_t T, int32_t D, int32_t ld,
+                         float* resid, void* out, int32_t ldy, int32_t f32, void* stream) {
+  MI_CHECK(ids && pos && table && resid && out && T >= 1 && D >= 1 && ld >= D && ld % 4 == 0 && pos_base > 0.f, "bad argument");
+  hipStream_t s = (hipStream_t)stream;
+  double* turns = nullptr;
+  int rc = stack_position_turns(D, pos_base, &turns, s);
+  if (rc == MI_OK) rc = launch_embed_pos(ids, pos, table, nullptr, scale, f32 != 0, T, D, ld, resid, nullptr, s, turns, out, ldy);
+  hipStreamSynchronize(s);
+  hipFree(turns);
+  return rc;
+}
+
+int mi_op_head_scatter(const float* qkv, int32_t ldq, int32_t T, const mi_layer_spec* spec, const float* bias, const float* q_norm, const float* k_norm,
+                       float eps, const int32_t* slots, int32_t block_size, void* q, void* kpool, void* vpool, int32_t f32, void* stream) {
+  MI_CHECK(qkv && spec && slots && q && kpool && vpool && T >= 1, "null argument");
+  const mi_layer_spec& p = *spec;
+  const HeadGeom g{p.num_heads, p.num_kv_heads, p.qk_dim, p.v_dim, pad_to(p.qk_dim, 16), pad_to(p.v_dim, 16)};
+  return launch_qkv_scatter(qkv, ldq, T, g, HeadRule{p.qk_norm || p.qk_unit_norm, q_norm, k_norm, bias, p.keys_as_values != 0}, eps, slots, block_size, q, kpool, vpool,
+                            f32 != 0, (hipStream_t)stream);
+}
+
+int mi_op_short_conv(const float* x, int32_t ldx, const float* w, const float* b, int32_t C, int32_t taps, float* ring, int32_t num_slots,
+                     const int32_t* slots_host, const int32_t* pos_host, const int32_t* segs_host, int32_t nseg, int32_t T, void* y, int32_t ldy,
+                     int32_t f32, void* stream) {
+  hipStream_t s = (hipStream_t)stream;
+  Arena mem;
+  std::vector<AttnSeg> segs;
+  AttnSeg* sd = nullptr;
+  int32_t *slots, *pos;
+  MI_TRY(take_sequences(mem, num_slots, slots_host, pos_host, segs_host, nseg, T, segs, &sd, &slots, &pos, s));
+  MI_TRY(launch_short_conv(x, ldx, ShortConv{w, b, taps, C, ring, slots}, pos, sd, segs.data(), nseg, T, y, ldy, f32 != 0, s));
+  MI_HIP(hipStreamSynchronize(s));
+  return MI_OK;
+}
+
+int32_t mi_op_scan_state(int32_t state) { return scan_geom(1, state, 1).Np; }
+
+int mi_op_scan(const mi_layer_spec* spec, const void* x, int32_t ldx, const float* low, int32_t ldl, int32_t col_b, int32_t col_c, const float* w_dt,
+               const float* dt_bias, const float* a_log, const float* d, const float* z, int32_t ldz, float* state, int32_t num_slots,
+               const int32_t* slots_host, const int32_t* pos_host, const int32_t* segs_host, int32_t nseg, int32_t T, void* y, int32_t ldy, int32_t f32,
+               void* stream) {
+  MI_CHECK(spec && x && low && w_dt && a_log && state && scan_supported(spec->ssm_state) && spec->ssm_inner >= 1 && spec->dt_rank >= 1, "selective scan: arguments");
+  hipStream_t s = (hipStream_t)stream;
+  Arena mem;
+  std::vector<AttnSeg> segs;
+  AttnSeg* sd = nullptr;
+  int32_t *slots, *pos;
+  MI_TRY(take_sequences(mem, num_slots, slots_host, pos_host, segs_host, nseg, T, segs, &sd, &slots, &pos, s));
+  const ScanGeom g = scan_geom(spec->ssm_inner, spec->ssm_state, spec->dt_rank);
+  const size_t el = f32 ? 4 : 2;
+  const int N = pad_to(g.C, 16), K = pad_to(g.rank, 64);
+  unsigned char *wr, *wt, *lo;
+  float *a2, *dt, *ones;
+  MI_TRY(mem.take(&wr, (size_t)g.C * g.rank_p * el, s));
+  MI_TRY(mem.take(&wt, (size_t)N * K * el, s));
+  MI_TRY(mem.take(&lo, (size_t)T * K * el, s));
+  MI_TRY(mem.take(&a2, (size_t)g.C * g.Np * 4, s));
+  MI_TRY(mem.take(&dt, (size_t)T * N * 4, s));
+  MI_TRY(mem.take(&ones, (size_t)N * 4, s));
+  MI_TRY(launch_fill_f32(ones, N, 1.f, s));
+  MI_TRY(launch_place_rows(w_dt, g.C, g.rank, wr, g.rank_p, f32 != 0, s));
+  MI_TRY(launch_place(w_dt, g.rank, 0, g.C, g.rank, wt, K, f32 != 0, 0, 0, s));
+  MI_TRY(launch_scan_decay(a_log, g, a2, s));
+  ScanIn in;
+  in.x = x; in.ldx = ldx; in.low = low; in.ldl = ldl; in.col_b = col_b; in.col_c = col_c;
+  in.dt = dt; in.ldt = N; in.w_dt = wr; in.dt_bias = dt_bias; in.a2 = a2; in.d = d; in.z = z; in.ldz = ldz;
+  in.state = state; in.slots = slots; in.pos = pos;
+  if (!nseg) {
+    MI_TRY(launch_scan_token(g, in, T, nullptr, y, ldy, f32 != 0, s));
+  } else {
+    MI_TRY(launch_columns(low, ldl, {0, g.rank, nullptr, lo}, {}, 0.f, T, K, f32 != 0, s));
+    EpiArgs e{};
+    e.scale = ones; e.out_f32 = dt; e.ld_out = N;
+    if (f32) MI_TRY(launch_linear_f32((const float*)wt, N, K, (const float*)lo, K, T, EPI_F32, e, s));
+    else MI_TRY(launch_gemm(LinearW{wt, N, K, MI_W_BF16}, T, (const uint16_t*)lo, K, EPI_F32, e, s));
+    MI_TRY(launch_scan_token(g, in, nseg, sd, y, ldy, f32 != 0, s));
+    MI_TRY(launch_scan_prompt(g, in, sd, nseg, y, ldy, f32 != 0, s));
+  }
+  MI_HIP(hipStreamSynchronize(s));
+  return MI_OK;
+}
+
+int mi_op_ssd(const mi_layer_spec* spec, const void* xbc, int32_t ldx, const float* dt, int32_t ldt, const float* dt_bias, const float* a_log, const float* d,
+              float* state, int32_t num_slots, const int32_t* slots_host, const int32_t* pos_host, const int32_t* segs_host, int32_t nseg, int32_t T,
+              int32_t max_chunks, float* y, int32_t ldy, int32_t f32, void* stream) {
+  MI_CHECK(spec && max_chunks >= 1, "state-space duality: arguments");
+  hipStream_t s = (hipStream_t)stream;
+  Arena mem;
+  std::vector<AttnSeg> segs;
+  AttnSeg* sd = nullptr;
+  int32_t *slots, *pos;
+  MI_TRY(take_sequences(mem, num_slots, slots_host, pos_host, segs_host, nseg, T, segs, &sd, &slots, &pos, s));
+  const SsdGeom g = ssd_geom(spec->ssm_heads, spec->ssm_dim, spec->ssm_state, spec->ssm_groups);
+  MI_CHECK(ssd_supported(g), "state-space duality: sizes");
+  float* records;
+  MI_TRY(mem.take(&records, (size_t)max_chunks * ssd_chunk_floats(g) * 4, s));
+  SsdIn in;
+  in.xbc = xbc; in.ldx = ldx; in.dt = dt; in.ldt = ldt; in.dt_bias = dt_bias; in.a_log = a_log; in.d = d;
+  in.state = state; in.slots = slots; in.pos = pos;
+  if (!nseg) {
+    MI_TRY(launch_ssd_token(g, in, T, nullptr, y, ldy, f32 != 0, s));
+  } else {
+    MI_TRY(launch_ssd_token(g, in, nseg, sd, y, ldy, f32 != 0, s));
+    MI_TRY(launch_ssd_prompt(g, in, sd, segs.data(), nseg, records, max_chunks, y, ldy, f32 != 0, s));
+  }
+  MI_HIP(hipStreamSynchronize(s));
+  return MI_OK;
+}
+
+int mi_op_gated_norm(const float* y, int32_t ldy, const float* z, int32_t ldz, const float* w, int32_t n, int32_t parts, float eps, int32_t T, void* out,
+                     int32_t ldo, int32_t f32, void* stream) {
+  return launch_gated_norm(y, ldy, z, ldz, w, n, parts, eps, T, out, ldo, f32 != 0, (hipStream_t)stream);
 }
 
 int mi_op_latent_attn(const mi_layer_spec* spec, const float* uk, const float* uv, const void* q, const void* pool, int32_t block_size,

@@ -13,6 +13,7 @@ from types import SimpleNamespace
 
 from .._stack_enums import MI_MIX
 from .bokulorn import BokulornConfig
+from .nusovik import NusovikConfig
 from .rapodra import RapodraConfig
 from .vimesun import VimesunConfig
 
@@ -21,7 +22,7 @@ MULTI_MODAL_MODELS = [f"{family}ForConditionalGeneration" for family in ("Mllama
 
 LLAMA_FAMILY = ("LlamaForCausalLM", "Qwen2ForCausalLM", "MistralForCausalLM")
 # architecture name -> reader of its config.json dictionary
-STACK_DESIGNS = {design.architecture: design.from_dict for design in (VimesunConfig, RapodraConfig, BokulornConfig)}
+STACK_DESIGNS = {design.architecture: design.from_dict for design in (VimesunConfig, RapodraConfig, BokulornConfig, NusovikConfig)}
 SUPPORTED_ARCHITECTURES = LLAMA_FAMILY + tuple(STACK_DESIGNS)
 
 
@@ -51,7 +52,8 @@ def stack_of(config) -> dict | None:
 def has_recurrent_state(config) -> bool:
     """Whether a sequence owns state that is not in KV blocks (a slot per sequence; no prefix to be taken over from the cache)."""
     stack = stack_of(config)
-    return stack is not None and any(x.get("mixer_kind") == MI_MIX["delta"] for x in stack["layers"])
+    recurrent = {MI_MIX["delta"], MI_MIX["scan"], MI_MIX["ssd"]}
+    return stack is not None and any(x.get(k) in recurrent for x in stack["layers"] for k in ("mixer_kind", "beside_kind"))
 
 
 def fill_sizes(config, shape_of) -> None:

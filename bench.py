@@ -529,6 +529,69 @@ def bokulorn_section(args):
     bench.line("Bokulorn", out, "Rapodra")
 
 
+# ---- --nusovik: its two kinds of layer beside Vimesun (the attention, the feed-forward) and Bokulorn's delta rule (the recurrences) --
+# (label, width, q heads, kv heads, head size, feed-forward, second mixer's heads of 64 and groups, scan channels and rank, layers); both
+# Nusovik and Vimesun attend to STACK_WINDOW keys at most.
+NUSOVIK_SIZES = [("1b-like", 2048, 32, 8, 64, 12288, 64, 1, 4096, 128, 8), ("8b-like", 4096, 32, 8, 128, 21504, 128, 8, 8192, 256, 4)]
+NUSOVIK_STATE, NUSOVIK_SCAN_STATE, NUSOVIK_ROWS = 128, 16, 32
+# selective scan, per channel, state and token: four plain vector instructions of 16 lanes a clock and one exponential of 4, on 1024 SIMDs
+SCAN_CLOCKS_PER_STATE, SIMD_CLOCKS_PER_S = 4 / 16 + 1 / 4, 1024 * 2.4e9
+
+
+def nusovik_section(args):
+    bench, out = StackBench(args), []
+    win, N, N1 = STACK_WINDOW, NUSOVIK_STATE, NUSOVIK_SCAN_STATE
+    f32 = MFMA_BF16_PEAK_TFLOPS / MFMA_F32_PEAK_TFLOPS
+    for label, width, nh, nkv, hd, ff, h2, groups, inner, rank, layers in NUSOVIK_SIZES:
+        size = {"size": label, "layers": layers, "width": width, "heads": [nh, nkv, hd], "ff": ff, "second mixer": [h2, 64, N, groups],
+                "scan": [inner, N1, rank], "prefill": [], "decode": []}
+        chunk_keys = lambda T: sum(i % win + 1 for i in range(T))       # noqa: E731
+        dense, H = {"kind": "dense", "ff": ff}, width // 128
+        common = {"width": width, "vocab": STACK_VOCAB, "norm": {"eps": 1e-5}}
+        att = {"heads": nh, "kv_heads": nkv, "dim": hd, "vdim": hd, "scale": hd ** -0.5, "mask": {"size": win}}
+        for kind in ("vimesun", "channel_delta", "parallel", "mamba1"):
+            if args.kinds and kind not in args.kinds.split(","):
+                continue
+            print(f"[bench] {label} {kind}", file=sys.stderr, flush=True)
+            if kind == "vimesun":
+                m = bench.stack({"architecture": "Vimesun", **common, "layers": [{"type": "attention", "mixer": att, "mlp": dense}] * layers,
+                                 "max_positions": bench.MAX_LEN, "residual_mult": 0.5})
+                weights = width * (2 * nh + 2 * nkv) * hd + 2 * width * ff
+                mixer = lambda T: (4.0 * nh * hd * bench.keys_seen(T, win), 0.0)                     # noqa: E731
+                token = lambda B, ctx: 4.0 * B * min(ctx, win) * nkv * hd                            # noqa: E731
+            elif kind == "channel_delta":
+                m = bench.stack({"architecture": "Bokulorn", **common, "embedding": {"scale": 1.0}, "layers": [
+                    {"type": kind, "mixer": {"heads": H, "kv_heads": H, "dim": 128, "vdim": 128, "conv": 4}, "mlp": None}] * layers}, ranks=BOKULORN_LOW)
+                weights = width * (4 * H * 128 + H + 2 * BOKULORN_LOW) + 2 * BOKULORN_LOW * H * 128
+                mixer = lambda T: (6.0 * T * H * 128 * 128 * f32, 0.0)                               # noqa: E731
+                token = lambda B, ctx: 8.0 * B * H * 128 * 128                                       # noqa: E731
+            else:
+                if kind == "parallel":
+                    mix = {"left": dict(att, bias_max=win // 2), "left_scale": 1.0, "right_scale": 1.0,
+                           "right": {"heads": h2, "vdim": 64, "state": N, "groups": groups, "norm_groups": groups, "conv": 4}}
+                    n2 = 2 * h2 * 64 + 2 * groups * N + h2
+                    weights = width * (2 * nh + nkv) * hd + width * nh + width * n2 + width * h2 * 64 + 2 * width * ff
+                    mixer = lambda T: (4.0 * nh * hd * chunk_keys(T) + 4.0 * T * h2 * 64 * N * f32, 0.0)     # noqa: E731
+                    token = lambda B, ctx: 4.0 * B * ((ctx - 1) % win + 1) * nkv * hd + 8.0 * B * h2 * 64 * N  # noqa: E731
+                else:
+                    mix = {"inner": inner, "state": N1, "dt_rank": rank, "conv": 4}
+                    weights = 3 * width * inner + inner * (2 * rank + 2 * N1)
+                    clocks = SCAN_CLOCKS_PER_STATE * inner * N1 / SIMD_CLOCKS_PER_S
+                    mixer = lambda T: (T * clocks * MFMA_BF16_PEAK_TFLOPS * 1e12, T * inner * 12.0)  # noqa: E731
+                    token = lambda B, ctx: 8.0 * B * inner * N1 + 4.0 * inner * N1 + 2.0 * inner * rank      # noqa: E731
+                m = bench.stack({"architecture": "Nusovik", **common, "embedding": {"scale": 1.0}, "logit_scale": 1.0, "layers": [
+                    {"type": kind, "mixer": mix, "mlp": dense if kind == "parallel" else None}] * layers}, ranks=NUSOVIK_ROWS)
+            size["prefill"] += bench.prefill(m, kind, lambda T: {"gemm": (2.0 * T * layers * weights, 2.0 * layers * weights),
+                                                                 "attn_prefill": tuple(layers * x for x in mixer(T))})
+            size["decode"] += bench.decode(m, kind, lambda B, ctx: layers * token(B, ctx))
+            m.close()
+        if not args.kinds:
+            for pair in (("vimesun", "parallel"), ("channel_delta", "mamba1")):
+                bench.compare(dict(size, **{t: [r for k in pair for r in size[t] if r["model"] == k] for t in ("prefill", "decode")}), bench.MAX_LEN)
+        out.append(size)
+    bench.line("Nusovik", out, "Vimesun and a delta rule")
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -551,10 +614,15 @@ def main():
     ap.add_argument("--bokulorn", action="store_true",
                     help="instead of the headline workload: Bokulorn's mixers (latent attention, delta rule), each with experts, beside "
                          "Rapodra of equal size, all bf16")
-    ap.add_argument("--kinds", default="", help="--bokulorn: only these models (comma-separated; no comparison)")
+    ap.add_argument("--nusovik", action="store_true",
+                    help="instead of the headline workload: Nusovik's layers (chunked attention beside a Mamba-2 mixer; selective scan) beside "
+                         "Vimesun and Bokulorn's delta rule, all bf16")
+    ap.add_argument("--kinds", default="", help="--bokulorn, --nusovik: only these models (comma-separated; no comparison)")
     args = ap.parse_args()
     if args.bokulorn:
         return bokulorn_section(args)
+    if args.nusovik:
+        return nusovik_section(args)
     if args.vimesun:
         return vimesun_section(args)
     if args.rapodra:

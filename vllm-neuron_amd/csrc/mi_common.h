@@ -84,7 +84,7 @@ __device__ __forceinline__ bf16x8_t decode8<MI_W_INT8>(uint32_t lo, uint32_t hi)
   return u.v;
 }
 
-// ---- cross-lane sums inside an aligned group of 8 or 16 lanes (DPP, no LDS) ------------
+// ---- cross-lane sums inside an aligned group of 4, 8 or 16 lanes (DPP, no LDS) ------------
 template <int CTRL>
 __device__ __forceinline__ float dpp_add(float v) {
   float t = __builtin_bit_cast(
@@ -94,9 +94,9 @@ __device__ __forceinline__ float dpp_add(float v) {
 // after the call every lane of the group holds the group's sum
 template <int LANES>
 __device__ __forceinline__ float group_sum(float v) {
-  static_assert(LANES == 8 || LANES == 16, "group of 8 or 16 lanes");
+  static_assert(LANES == 4 || LANES == 8 || LANES == 16, "group of 4, 8 or 16 lanes");
   if (LANES == 16) v = dpp_add<0x140>(v);  // row_mirror       i <-> 15-i
-  v = dpp_add<0x141>(v);                   // row_half_mirror  i <-> 7-i (within 8)
+  if (LANES >= 8) v = dpp_add<0x141>(v);   // row_half_mirror  i <-> 7-i (within 8)
   v = dpp_add<0xB1>(v);                    // quad_perm [1,0,3,2]
   v = dpp_add<0x4E>(v);                    // quad_perm [2,3,0,1]
   return v;

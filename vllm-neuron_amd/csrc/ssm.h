@@ -54,7 +54,8 @@ int launch_scan_decay(const float* a_log, const ScanGeom& g, float* a2, hipStrea
 // ---- state-space duality --------------------------------------------------------------------------------------------------------
 // Prompts run in chunks of kSsdChunk tokens.  With L the running sum of dt A inside a chunk and S0 the state ahead of it,
 //   y_i = e^(L_i) S0^T C_i + sum_(j <= i) (C_i.B_j) e^(L_i - L_j) dt_j x_j;   S = e^(L_end) S0 + sum_j e^(L_end - L_j) dt_j B_j x_j^T
-// every exponent is of a number <= 0; L is summed and subtracted in fp64, so that a strong decay leaves the following ones exact.
+// every exponent is of a number <= 0; L is summed in fp64 and kept in two fp32 parts, so that a strong decay leaves the following ones exact.
+// One kernel makes C B^T and the steps of all chunks at once, a second one walks a sequence's chunks with the state in registers.
 struct SsdGeom {
   int H = 0, P = 0, N = 0, G = 0;   // heads, head size, states, groups (sizes up to 256)
   int Pp = 0, Np = 0;               // padded to 16: zeros in the state
@@ -75,8 +76,9 @@ struct SsdIn {
 };
 constexpr int kSsdChunk = 64;
 size_t ssd_chunk_floats(const SsdGeom& g);               // device memory behind a chunk of a prompt
-// y [rows, ldy] fp32, heads concatenated
-int launch_ssd_token(const SsdGeom& g, const SsdIn& in, int rows, const AttnSeg* segs, float* y, int ldy, bool f32, hipStream_t s);
+// y [rows, ldy] fp32, heads concatenated.  conv: the convolution in the same launch, from proj [rows, ldp] (in.xbc is not read)
+int launch_ssd_token(const SsdGeom& g, const SsdIn& in, int rows, const AttnSeg* segs, float* y, int ldy, bool f32, hipStream_t s, const ShortConv* conv = nullptr,
+                     const float* proj = nullptr, int ldp = 0);
 int launch_ssd_prompt(const SsdGeom& g, const SsdIn& in, const AttnSeg* segs_dev, const AttnSeg* segs_host, int nseg, float* records, int max_chunks,
                       float* y, int ldy, bool f32, hipStream_t s);
 // out [rows, ldo] compute type = (y silu(z)), every one of `parts` equal parts of the n columns over its root mean square, times w [n]

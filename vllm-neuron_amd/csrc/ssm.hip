@@ -2,6 +2,7 @@
 #include "ssm.h"
 
 #include <algorithm>
+#include <type_traits>
 
 namespace mi {
 
@@ -9,8 +10,12 @@ namespace {
 
 constexpr float kLog2e = 1.4426950408889634f;
 
-__device__ __forceinline__ float silu(float v) { return v / (1.f + __expf(-v)); }
-__device__ __forceinline__ float softplus(float v) { return fmaxf(v, 0.f) + log1pf(expf(-fabsf(v))); }
+__device__ __forceinline__ float silu(float v) { return v * __builtin_amdgcn_rcpf(1.f + __expf(-v)); }
+// max(v, 0) + log(1 + w), w = exp(-|v|); log(1 + w) as log(u) w / (u - 1) with u = 1 + w as it is rounded: right to the last places however small w is
+__device__ __forceinline__ float softplus(float v) {
+  const float w = __expf(-fabsf(v)), u = 1.f + w, d = u - 1.f;
+  return fmaxf(v, 0.f) + (d > 0.f ? __logf(u) * w * __builtin_amdgcn_rcpf(d) : w);
+}
 __device__ __forceinline__ float to_f32(uint16_t v) { return bf16_to_f32(v); }
 __device__ __forceinline__ float to_f32(float v) { return v; }
 __device__ __forceinline__ void put1(uint16_t* p, float v) { *p = f32_to_bf16(v); }
@@ -101,54 +106,109 @@ __global__ __launch_bounds__(256) void short_conv_kernel(const float* __restrict
 template <int LPC>
 __device__ __forceinline__ float lanes_sum(float v) { return group_sum<LPC>(v); }
 
-// LPC lanes per channel, R consecutive states per lane (Np = LPC R).
-template <typename T, int LPC, int R>
-__global__ __launch_bounds__(256) void scan_token_kernel(ScanGeom g, ScanIn in, const AttnSeg* __restrict__ segs, T* __restrict__ y, int ldy) {
+// LPC lanes per channel, R consecutive states per lane (Np = LPC R), RB rows per work-group: the decays and the step sizes' weights are read
+// once for them, and every row's state is requested before any is used.
+template <typename T, int LPC, int R, int RB>
+__global__ __launch_bounds__(256) void scan_token_kernel(ScanGeom g, ScanIn in, const AttnSeg* __restrict__ segs, int rows, T* __restrict__ y, int ldy) {
   constexpr int CB = 256 / LPC;
-  int row = blockIdx.y, seq = blockIdx.y;
-  if (segs) {
-    const AttnSeg sg = segs[blockIdx.y];
-    if (sg.n != 1) return;
-    row = sg.row0; seq = sg.seq;
+  extern __shared__ __attribute__((aligned(16))) float lows[];     // [RB][rank_p]
+  int row[RB], seq[RB];
+  bool live[RB], any = false;
+#pragma unroll
+  for (int b = 0; b < RB; ++b) {
+    const int i = blockIdx.y * RB + b;
+    live[b] = i < rows;
+    row[b] = seq[b] = min(i, rows - 1);
+    if (segs) {
+      const AttnSeg sg = segs[row[b]];
+      live[b] = live[b] && sg.n == 1;
+      row[b] = sg.row0; seq[b] = sg.seq;
+    }
+    any = any || live[b];
+  }
+  if (!any) return;
+  for (int i = threadIdx.x; i < RB * g.rank_p; i += 256) {
+    const int b = i / g.rank_p, k = i - b * g.rank_p;
+    int r = row[0];
+#pragma unroll
+    for (int q = 1; q < RB; ++q) r = b == q ? row[q] : r;
+    lows[i] = k < g.rank ? round_to(in.low[(size_t)r * in.ldl + k], y) : 0.f;
   }
   const int l = threadIdx.x % LPC, c = blockIdx.x * CB + threadIdx.x / LPC, cc = min(c, g.C - 1);     // (lanes past the last channel repeat it)
-  float* S0 = in.state + ((size_t)in.slots[seq] * g.C + cc) * g.Np + l * R;
-  const float *a2 = in.a2 + (size_t)cc * g.Np + l * R, *lo = in.low + (size_t)row * in.ldl;
-  const bool fresh = in.pos[row] == 0;
-  float S[R], A[R], B[R], Cn[R];
+  const float* a2 = in.a2 + (size_t)cc * g.Np + l * R;
+  float S[RB][R], A[R], B[RB][R], Cn[RB][R], x[RB], z[RB], dot[RB];
+  float* S0[RB];
 #pragma unroll
-  for (int r = 0; r < R; ++r) {
-    S[r] = S0[r];
-    A[r] = a2[r];
-    const int n = min(l * R + r, g.N - 1);           // (beyond the last state: B is taken as zero)
-    B[r] = lo[in.col_b + n];
-    Cn[r] = lo[in.col_c + n];
+  for (int r = 0; r < R; ++r) A[r] = a2[r];
+#pragma unroll
+  for (int b = 0; b < RB; ++b) {
+    S0[b] = in.state + ((size_t)in.slots[seq[b]] * g.C + cc) * g.Np + l * R;
+    const float* lo = in.low + (size_t)row[b] * in.ldl;
+#pragma unroll
+    for (int r = 0; r < R; ++r) S[b][r] = S0[b][r];
+    if (l * R + R <= g.N) {                            // (one load where R allows)
+#pragma unroll
+      for (int r = 0; r < R; ++r) { B[b][r] = lo[in.col_b + l * R + r]; Cn[b][r] = lo[in.col_c + l * R + r]; }
+    } else {
+#pragma unroll
+      for (int r = 0; r < R; ++r) {
+        const int n = min(l * R + r, g.N - 1);
+        B[b][r] = l * R + r < g.N ? lo[in.col_b + n] : 0.f;
+        Cn[b][r] = lo[in.col_c + n];
+      }
+    }
+    x[b] = to_f32(reinterpret_cast<const T*>(in.x)[(size_t)row[b] * in.ldx + cc]);
+    z[b] = in.z[(size_t)row[b] * in.ldz + cc];
+    dot[b] = 0.f;
   }
-  const float x = to_f32(reinterpret_cast<const T*>(in.x)[(size_t)row * in.ldx + cc]), z = in.z[(size_t)row * in.ldz + cc];
+  __syncthreads();
   const T* w = reinterpret_cast<const T*>(in.w_dt) + (size_t)cc * g.rank_p;
-  float dot = 0.f;
   for (int k = l * 8; k < g.rank_p; k += LPC * 8) {
+    const float4 w0 = get4(w + k), w1 = get4(w + k + 4);             // (zero beyond the rank)
 #pragma unroll
-    for (int q = 0; q < 8; q += 4) {
-      const float4 wv = get4(w + k + q);             // (zero beyond the rank)
-      auto at = [&](int i) { return round_to(lo[min(k + q + i, g.rank - 1)], y); };
-      dot = __builtin_fmaf(wv.x, at(0), dot); dot = __builtin_fmaf(wv.y, at(1), dot);
-      dot = __builtin_fmaf(wv.z, at(2), dot); dot = __builtin_fmaf(wv.w, at(3), dot);
+    for (int b = 0; b < RB; ++b) {
+      const float4 u = *reinterpret_cast<const float4*>(lows + b * g.rank_p + k), v = *reinterpret_cast<const float4*>(lows + b * g.rank_p + k + 4);
+      dot[b] = __builtin_fmaf(w0.x, u.x, dot[b]); dot[b] = __builtin_fmaf(w0.y, u.y, dot[b]); dot[b] = __builtin_fmaf(w0.z, u.z, dot[b]); dot[b] = __builtin_fmaf(w0.w, u.w, dot[b]);
+      dot[b] = __builtin_fmaf(w1.x, v.x, dot[b]); dot[b] = __builtin_fmaf(w1.y, v.y, dot[b]); dot[b] = __builtin_fmaf(w1.z, v.z, dot[b]); dot[b] = __builtin_fmaf(w1.w, v.w, dot[b]);
     }
   }
-  const float dt = softplus(lanes_sum<LPC>(dot) + in.dt_bias[cc]), dx = dt * x;
-  float o = 0.f;
+  const float bias = in.dt_bias[cc], skip = in.d[cc];
 #pragma unroll
-  for (int r = 0; r < R; ++r) {
-    const float b = l * R + r < g.N ? B[r] : 0.f;
-    S[r] = __builtin_fmaf(__builtin_amdgcn_exp2f(dt * A[r]), fresh ? 0.f : S[r], dx * b);
-    o = __builtin_fmaf(S[r], Cn[r], o);
+  for (int b = 0; b < RB; ++b) {
+    const float dt = softplus(lanes_sum<LPC>(dot[b]) + bias), dx = dt * x[b];
+    const bool fresh = in.pos[row[b]] == 0;
+    float o = 0.f;
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      S[b][r] = __builtin_fmaf(__builtin_amdgcn_exp2f(dt * A[r]), fresh ? 0.f : S[b][r], dx * B[b][r]);
+      o = __builtin_fmaf(S[b][r], Cn[b][r], o);
+    }
+    o = lanes_sum<LPC>(o);
+    if (!live[b] || c >= g.C) continue;
+#pragma unroll
+    for (int r = 0; r < R; ++r) S0[b][r] = S[b][r];
+    if (l == 0) put1(y + (size_t)row[b] * ldy + c, __builtin_fmaf(skip, x[b], o) * silu(z[b]));
   }
-  o = lanes_sum<LPC>(o);
-  if (c >= g.C) return;
-#pragma unroll
-  for (int r = 0; r < R; ++r) S0[r] = S[r];
-  if (l == 0) put1(y + (size_t)row * ldy + c, __builtin_fmaf(in.d[c], x, o) * silu(z));
+}
+
+// Four values summed over the LPC lanes of a group, lane l left with the sum of value token_of(l)
+template <int LPC>
+__device__ __forceinline__ int token_of(int l) { return LPC == 16 ? (l >> 3) * 2 + ((l >> 2) & 1) : (l >> 2) * 2 + ((l >> 1) & 1); }
+template <int CTRL>
+__device__ __forceinline__ float swap_add(float a, float b, bool upper) {    // lower lanes: a + the partner's a; upper lanes: b + the partner's b
+  const float send = upper ? a : b;
+  return (upper ? b : a) + __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, send), CTRL, 0xf, 0xf, true));
+}
+template <int LPC>
+__device__ __forceinline__ float sum_four(const float (&v)[4], int l) {
+  if constexpr (LPC == 16) {       // partners 15 - l, then 7 - l within eight, then inside quads
+    const float a = swap_add<0x140>(v[0], v[2], l & 8), b = swap_add<0x140>(v[1], v[3], l & 8);
+    const float r = swap_add<0x141>(a, b, l & 4);
+    return dpp_add<0x4E>(dpp_add<0xB1>(r));
+  } else {                         // partners 7 - l, then l ^ 2, then l ^ 1
+    const float a = swap_add<0x141>(v[0], v[2], l & 4), b = swap_add<0x141>(v[1], v[3], l & 4);
+    return dpp_add<0xB1>(swap_add<0x4E>(a, b, l & 2));
+  }
 }
 
 // One work-group: CB channels of one segment, its tokens in order, TB at a time: their step sizes, inputs, B and C go through LDS (the next
@@ -162,6 +222,7 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanGeom g, ScanIn in,
   if (sg.n < 2) return;
   const int tid = threadIdx.x, l = tid % LPC, cl = tid / LPC, c0 = blockIdx.x * CB, cc = min(c0 + cl, g.C - 1);
   float* S0 = in.state + ((size_t)in.slots[sg.seq] * g.C + cc) * g.Np + l * R;
+  const int tok = token_of<LPC>(l);
   float S[R], A[R];
 #pragma unroll
   for (int r = 0; r < R; ++r) {
@@ -213,24 +274,35 @@ __global__ __launch_bounds__(256) void scan_prompt_kernel(ScanGeom g, ScanIn in,
     }
     __syncthreads();
     if (t0 + TB < sg.n) load(t0 + TB);
-#pragma unroll 2
+    // four tokens' operands are read while the four before them are worked off
+    struct Four { float d[4], x[4], b[R][4], c[R][4]; };
+    auto take = [&](Four& f, int t) {
+      auto four = [](float* o, const float* p) { const float4 v = *reinterpret_cast<const float4*>(p); o[0] = v.x; o[1] = v.y; o[2] = v.z; o[3] = v.w; };
+      four(f.d, &dts[cl][t]);
+      four(f.x, &dxs[cl][t]);
+#pragma unroll
+      for (int r = 0; r < R; ++r) { four(f.b[r], &Bs[l * R + r][t]); four(f.c[r], &Cs[l * R + r][t]); }
+    };
+    Four f[2];
+    take(f[0], 0);
+#pragma unroll
     for (int t = 0; t < TB; t += 4) {
-      const float4 d4 = *reinterpret_cast<const float4*>(&dts[cl][t]), x4 = *reinterpret_cast<const float4*>(&dxs[cl][t]);
-      const float da[4] = {d4.x, d4.y, d4.z, d4.w}, xa[4] = {x4.x, x4.y, x4.z, x4.w};
-      float o[4] = {0.f, 0.f, 0.f, 0.f};
+      const Four& q = f[(t >> 2) & 1];
+      if (t + 4 < TB) take(f[((t >> 2) + 1) & 1], t + 4);
+      float e[R][4], o[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int r = 0; r < R; ++r) {
-        const float4 b4 = *reinterpret_cast<const float4*>(&Bs[l * R + r][t]), c4 = *reinterpret_cast<const float4*>(&Cs[l * R + r][t]);
-        const float ba[4] = {b4.x, b4.y, b4.z, b4.w}, ca[4] = {c4.x, c4.y, c4.z, c4.w};
+      for (int r = 0; r < R; ++r)
 #pragma unroll
-        for (int u = 0; u < 4; ++u) {
-          S[r] = __builtin_fmaf(__builtin_amdgcn_exp2f(da[u] * A[r]), S[r], xa[u] * ba[u]);
-          o[u] = __builtin_fmaf(S[r], ca[u], o[u]);
+        for (int u = 0; u < 4; ++u) e[r][u] = __builtin_amdgcn_exp2f(q.d[u] * A[r]);
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+          S[r] = __builtin_fmaf(e[r][u], S[r], q.x[u] * q.b[r][u]);
+          o[u] = __builtin_fmaf(S[r], q.c[r][u], o[u]);
         }
-      }
-#pragma unroll
-      for (int u = 0; u < 4; ++u) o[u] = lanes_sum<LPC>(o[u]);
-      if (l == 0) *reinterpret_cast<float4*>(&ys[cl][t]) = make_float4(o[0], o[1], o[2], o[3]);
+      const float sum = sum_four<LPC>(o, l);
+      if ((l & (LPC / 4 - 1)) == 0) ys[cl][t + tok] = sum;
     }
     __syncthreads();
 #pragma unroll
@@ -260,7 +332,8 @@ constexpr int kQ = kSsdChunk;
 // dg RPT .. + RPT - 1.
 constexpr int kTokenThreads = 512;
 template <typename T, int VQ, int RPT>
-__global__ __launch_bounds__(kTokenThreads) void ssd_token_kernel(SsdGeom g, SsdIn in, const AttnSeg* __restrict__ segs, float* __restrict__ y, int ldy) {
+__global__ __launch_bounds__(kTokenThreads) void ssd_token_kernel(SsdGeom g, SsdIn in, ShortConv cv, const float* __restrict__ proj, int ldp, const AttnSeg* __restrict__ segs,
+                                                                  float* __restrict__ y, int ldy) {
   constexpr int NW = kTokenThreads / 64;
   __shared__ float bs[256], cs[256], xs[256];
   __shared__ __attribute__((aligned(16))) float red[NW][VQ * 4];
@@ -280,13 +353,36 @@ __global__ __launch_bounds__(kTokenThreads) void ssd_token_kernel(SsdGeom g, Ssd
     const int n = dg * RPT + i;
     S[i] = !fresh && vin && n < g.Np ? *reinterpret_cast<const float4*>(S0 + (size_t)n * g.Pp) : make_float4(0.f, 0.f, 0.f, 0.f);
   }
-  const T* xr = reinterpret_cast<const T*>(in.xbc) + (size_t)row * in.ldx;
-  const int inner = g.H * g.P, grp = h / (g.H / g.G);
-  for (int i = tid; i < g.Np; i += kTokenThreads) {
-    bs[i] = i < g.N ? to_f32(xr[inner + grp * g.N + i]) : 0.f;
-    cs[i] = i < g.N ? to_f32(xr[inner + (g.G + grp) * g.N + i]) : 0.f;
+  const int inner = g.H * g.P, hpg = g.H / g.G, grp = h / hpg;
+  if (proj) {      // convolutions of the head's channels and its group's B and C; position p goes to a row of the ring that nobody reads in this launch
+    const int C = cv.C, p = in.pos[row];
+    const float* x = proj + (size_t)row * ldp;
+    float* ring = cv.ring + (size_t)cv.slots[seq] * cv.taps * C;
+    for (int i = tid; i < g.Pp + 2 * g.Np; i += kTokenThreads) {
+      const int part = i < g.Pp ? 0 : i < g.Pp + g.Np ? 1 : 2, d = i - (part == 0 ? 0 : g.Pp + (part - 1) * g.Np);
+      float a = 0.f;
+      if (d < (part ? g.N : g.P)) {
+        const int ch = part == 0 ? h * g.P + d : inner + ((part - 1) * g.G + grp) * g.N + d;
+        const float now = x[ch];
+        a = cv.b[ch];
+        for (int j = 0; j + 1 < cv.taps; ++j) {
+          const int q = p - (cv.taps - 1 - j);
+          const float v = ring[(size_t)(max(q, 0) % cv.taps) * C + ch];
+          a = __builtin_fmaf(cv.w[(size_t)j * C + ch], q >= 0 ? v : 0.f, a);
+        }
+        a = round_to(silu(__builtin_fmaf(cv.w[(size_t)(cv.taps - 1) * C + ch], now, a)), (const T*)nullptr);
+        if (part == 0 || h % hpg == 0) ring[(size_t)(p % cv.taps) * C + ch] = now;
+      }
+      (part == 0 ? xs : part == 1 ? bs : cs)[d] = a;
+    }
+  } else {
+    const T* xr = reinterpret_cast<const T*>(in.xbc) + (size_t)row * in.ldx;
+    for (int i = tid; i < g.Np; i += kTokenThreads) {
+      bs[i] = i < g.N ? to_f32(xr[inner + grp * g.N + i]) : 0.f;
+      cs[i] = i < g.N ? to_f32(xr[inner + (g.G + grp) * g.N + i]) : 0.f;
+    }
+    for (int i = tid; i < g.Pp; i += kTokenThreads) xs[i] = i < g.P ? to_f32(xr[h * g.P + i]) : 0.f;
   }
-  for (int i = tid; i < g.Pp; i += kTokenThreads) xs[i] = i < g.P ? to_f32(xr[h * g.P + i]) : 0.f;
   const float dt = softplus(in.dt[(size_t)row * in.ldt + h] + in.dt_bias[h]), decay = expf(-expf(in.a_log[h]) * dt);
   __syncthreads();
   float4 o = make_float4(0.f, 0.f, 0.f, 0.f);
@@ -326,105 +422,78 @@ __device__ __forceinline__ ChunkAt chunk_at(const AttnSeg* segs, int nseg, int c
   return ChunkAt{AttnSeg{0, 0, 0, 0}, 0, 0, false};
 }
 
-// What a piece of chunks leaves in memory: states [chunk][H][Np][Pp], C B^T [chunk][G][kQ][kQ], the chunk's whole decay [chunk][H]
-struct Records { float *state, *cb, *decay; };
+// What a piece of chunks leaves in memory: C B^T [chunk][G][kQ][kQ], and per head the chunk's steps [chunk][H]
+struct Steps {
+  float hi[kQ], lo[kQ];       // running sum of the decays' logarithms (base 2), in two parts: a difference of two sums is exact to fp32's last place
+  float dt[kQ], e[kQ], w[kQ]; // step size; decay from the chunk's start; dt times the decay up to the chunk's end
+};
+struct Records { float* cb; Steps* steps; };
 __host__ __device__ inline Records records_at(float* base, const SsdGeom& g, int chunks) {
-  float* cb = base + (size_t)chunks * g.H * g.Np * g.Pp;
-  return Records{base, cb, cb + (size_t)chunks * g.G * kQ * kQ};
+  return Records{base, reinterpret_cast<Steps*>(base + (size_t)chunks * g.G * kQ * kQ)};
 }
-// LDS row pitches: rows whose columns 16 lanes read side by side (four rows at once), and rows of which 16 lanes read one column each
-__host__ __device__ inline int wide_pitch(int n) { return (n + 47) / 64 * 64 + 16; }
+// LDS pitch of rows of which 16 lanes read one column each
 __host__ __device__ inline int tall_pitch(int n) { return (n + 63) / 64 * 64 + 4; }
 
-// step sizes of the chunk and the running sum of their decays' logarithms; ends with a barrier
-__device__ __forceinline__ void chunk_steps(const SsdIn& in, int h, const ChunkAt& at, double* L, float* dts) {
-  if (threadIdx.x < 64) {
-    const int t = threadIdx.x;
-    const float dt = t < at.n ? softplus(in.dt[(size_t)(at.sg.row0 + at.t0 + min(t, at.n - 1)) * in.ldt + h] + in.dt_bias[h]) : 0.f;
-    double s = (double)(-expf(in.a_log[h]) * dt);
-#pragma unroll
-    for (int m = 1; m < 64; m *= 2) {
-      const double v = __shfl_up(s, m);
-      if (t >= m) s += v;
-    }
-    L[t] = s;
-    dts[t] = dt;
-  }
-  __syncthreads();
-}
-
-// columns col .. + n of the chunk's rows times weight(row) into LDS rows of `pitch`, zeros up to np and beyond the last row
-template <typename T, typename F>
-__device__ __forceinline__ void stage_rows(float* dst, int pitch, const T* src, int ld, int rows, int n, int np, F weight) {
+// columns col .. + n of the chunk's rows in LDS rows of `pitch`, zeros up to np and beyond the last row
+template <typename T>
+__device__ __forceinline__ void stage_rows(float* dst, int pitch, const T* src, int ld, int rows, int n, int np) {
   const int tid = threadIdx.x;
   if (((n | ld) & 3) == 0 && (reinterpret_cast<uintptr_t>(src) & (4 * sizeof(T) - 1)) == 0) {
     const int q = np / 4;
-    for (int i = tid; i < kQ * q; i += 256) {
-      const int t = i / q, c = (i - t * q) * 4;
-      float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
-      if (t < rows && c < n) {
-        const float f = weight(t);
-        v = get4(src + (size_t)t * ld + c);
-        v = make_float4(v.x * f, v.y * f, v.z * f, v.w * f);
+    constexpr int U = 8;                 // in flight together
+    for (int i0 = tid; i0 < kQ * q; i0 += 256 * U) {
+      float4 v[U];
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int i = min(i0 + 256 * u, kQ * q - 1), t = i / q, c = (i - t * q) * 4;
+        v[u] = get4(src + (size_t)min(t, rows - 1) * ld + min(c, n - 4));
       }
-      *reinterpret_cast<float4*>(dst + t * pitch + c) = v;
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int i = i0 + 256 * u, t = i / q, c = (i - t * q) * 4;
+        if (i < kQ * q) *reinterpret_cast<float4*>(dst + t * pitch + c) = t < rows && c < n ? v[u] : make_float4(0.f, 0.f, 0.f, 0.f);
+      }
     }
     return;
   }
   for (int i = tid; i < kQ * np; i += 256) {
     const int t = i / np, c = i - t * np;
-    dst[t * pitch + c] = t < rows && c < n ? to_f32(src[(size_t)t * ld + c]) * weight(t) : 0.f;
+    dst[t * pitch + c] = t < rows && c < n ? to_f32(src[(size_t)t * ld + c]) : 0.f;
   }
 }
 
-// Of every chunk: what it adds to the state, per head (blockIdx.y < H), and C B^T, per group
+// Of every chunk: C B^T, a work-group per group (blockIdx.y < G), and the heads' steps, a wave per head
 template <typename T>
 __global__ __launch_bounds__(256) void ssd_chunk_kernel(SsdGeom g, SsdIn in, const AttnSeg* __restrict__ segs, int nseg, int c0, float* __restrict__ base) {
   extern __shared__ __attribute__((aligned(16))) float sm[];
-  __shared__ double L[kQ];
-  __shared__ float dts[kQ];
   const ChunkAt at = chunk_at(segs, nseg, c0 + blockIdx.x);
   if (!at.ok) return;
   const Records rec = records_at(base, g, gridDim.x);
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g4 = lane >> 4, c = lane & 15, inner = g.H * g.P;
-  const T* rows = reinterpret_cast<const T*>(in.xbc) + (size_t)(at.sg.row0 + at.t0) * in.ldx;
-  if ((int)blockIdx.y < g.H) {
-    const int h = blockIdx.y, grp = h / (g.H / g.G), bp = wide_pitch(g.Np), xp = wide_pitch(g.Pp);
-    float *Bs = sm, *xs = sm + kQ * bp;
-    chunk_steps(in, h, at, L, dts);
-    const double end = L[kQ - 1];
-    stage_rows(Bs, bp, rows + inner + grp * g.N, in.ldx, at.n, g.N, g.Np, [&](int t) { return dts[t] * expf((float)(end - L[t])); });
-    stage_rows(xs, xp, rows + h * g.P, in.ldx, at.n, g.P, g.Pp, [](int) { return 1.f; });
-    if (tid == 0) rec.decay[(size_t)blockIdx.x * g.H + h] = expf((float)end);
-    __syncthreads();
-    float* out = rec.state + ((size_t)blockIdx.x * g.H + h) * g.Np * g.Pp;
-    const int nt = g.Np / 16, pt = g.Pp / 16;
-    for (int n = wave; n < nt; n += 4)
-      for (int p0 = 0; p0 < pt; p0 += 4) {
-        f32x4_t acc[4] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
-        int off[4];
+  if ((int)blockIdx.y >= g.G) {
+    const int h = (blockIdx.y - g.G) * 4 + wave;
+    if (h >= g.H) return;
+    const float dt = lane < at.n ? softplus(in.dt[(size_t)(at.sg.row0 + at.t0 + min(lane, at.n - 1)) * in.ldt + h] + in.dt_bias[h]) : 0.f;
+    double s = (double)(-expf(in.a_log[h]) * dt);
 #pragma unroll
-        for (int p = 0; p < 4; ++p) off[p] = 16 * min(p0 + p, pt - 1) + c;
-#pragma unroll 4
-        for (int s = 0; s < kQ / 4; ++s) {
-          const float a = Bs[(4 * s + g4) * bp + 16 * n + c];
-#pragma unroll
-          for (int p = 0; p < 4; ++p) acc[p] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, xs[(4 * s + g4) * xp + off[p]], acc[p], 0, 0, 0);
-        }
-#pragma unroll
-        for (int p = 0; p < 4; ++p) {
-#pragma unroll
-          for (int r = 0; r < 4; ++r)
-            if (p0 + p < pt) out[(size_t)(16 * n + 4 * g4 + r) * g.Pp + off[p]] = acc[p][r];
-        }
-      }
+    for (int m = 1; m < 64; m *= 2) {
+      const double v = __shfl_up(s, m);
+      if (lane >= m) s += v;
+    }
+    const double end = __shfl(s, 63), l2 = s * 1.4426950408889634;
+    Steps& st = rec.steps[(size_t)blockIdx.x * g.H + h];
+    st.hi[lane] = (float)l2;
+    st.lo[lane] = (float)(l2 - (double)(float)l2);
+    st.dt[lane] = dt;
+    st.e[lane] = expf((float)s);
+    st.w[lane] = dt * expf((float)(end - s));
     return;
   }
-  const int grp = blockIdx.y - g.H, pitch = tall_pitch(g.Np);
+  const T* rows = reinterpret_cast<const T*>(in.xbc) + (size_t)(at.sg.row0 + at.t0) * in.ldx;
+  const int grp = blockIdx.y, pitch = tall_pitch(g.Np);
   float *Bs = sm, *Cs = sm + kQ * pitch;
-  auto one = [](int) { return 1.f; };
-  stage_rows(Bs, pitch, rows + inner + grp * g.N, in.ldx, at.n, g.N, g.Np, one);
-  stage_rows(Cs, pitch, rows + inner + (g.G + grp) * g.N, in.ldx, at.n, g.N, g.Np, one);
+  stage_rows(Bs, pitch, rows + inner + grp * g.N, in.ldx, at.n, g.N, g.Np);
+  stage_rows(Cs, pitch, rows + inner + (g.G + grp) * g.N, in.ldx, at.n, g.N, g.Np);
   __syncthreads();
   float* out = rec.cb + ((size_t)blockIdx.x * g.G + grp) * kQ * kQ;
   f32x4_t acc[4] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
@@ -439,8 +508,66 @@ __global__ __launch_bounds__(256) void ssd_chunk_kernel(SsdGeom g, SsdIn in, con
     for (int r = 0; r < 4; ++r) out[(16 * wave + 4 * g4 + r) * kQ + 16 * j + c] = acc[j][r];
 }
 
-// The chunks of a segment in order: what a chunk adds is replaced by the state ahead of it; the state behind the last one goes to the slot.
-__global__ __launch_bounds__(256) void ssd_pass_kernel(SsdGeom g, SsdIn in, const AttnSeg* __restrict__ segs, int c0, int nchunks, float* __restrict__ base) {
+// N elements as they lie in memory, in whole registers: taken apart where they are used, so that a load stays in flight until then
+template <typename T, int N>
+struct Words {
+  static constexpr int BYTES = N * (int)sizeof(T), Q = BYTES >= 16 ? 4 : BYTES / 4, NV = BYTES / (4 * Q);
+  typedef __attribute__((ext_vector_type(Q))) unsigned vec_t;
+  vec_t v[NV];
+  __device__ __forceinline__ void load(const T* p) {
+#pragma unroll
+    for (int i = 0; i < NV; ++i) v[i] = reinterpret_cast<const vec_t*>(p)[i];
+  }
+  __device__ __forceinline__ void store(T* p) const {
+#pragma unroll
+    for (int i = 0; i < NV; ++i) reinterpret_cast<vec_t*>(p)[i] = v[i];
+  }
+  __device__ __forceinline__ float at(int i) const {
+    constexpr int E = 4 / (int)sizeof(T);
+    const unsigned w = v[i / E / Q][i / E % Q];
+    return E == 1 ? __builtin_bit_cast(float, w) : i & 1 ? bf16hi_to_f32(w) : bf16lo_to_f32(w);
+  }
+  __device__ __forceinline__ void set(int i, T x) {          // (elements in ascending order)
+    constexpr int E = 4 / (int)sizeof(T);
+    unsigned& w = reinterpret_cast<unsigned*>(v)[i / E];
+    if constexpr (E == 1) w = __builtin_bit_cast(unsigned, x);
+    else w = i & 1 ? w | (unsigned)x << 16 : (unsigned)x;
+  }
+};
+template <typename T, int N> struct alignas(sizeof(T) * N) Pack { T v[N]; };
+
+// LDS of the scan: the waves' shares of a chunk's outputs [2][4][4][64] f32x4, steps [2], x [2][kQ][kXPitch], and per wave B [kQ][b_pitch]
+constexpr int kXPitch = 20;
+template <typename T, int NT>
+constexpr int b_pitch() {      // in elements; rows 4 apart fall into different banks
+  constexpr int dw = 16 * NT * (int)sizeof(T) / 4;
+  return (dw == 8 ? 12 : dw == 16 ? 20 : dw == 32 ? 40 : 68) * 4 / (int)sizeof(T);
+}
+template <typename T, int NT>
+constexpr size_t scan_lds() { return 2 * 16 * 64 * 16 + 2 * sizeof(Steps) + 2 * kQ * kXPitch * 4 + 4 * kQ * b_pitch<T, NT>() * sizeof(T); }
+
+// One work-group per (head, 16 columns, segment): the chunks of the segment in order.  A wave holds NT 16-row tiles of the state as MFMA
+// accumulators, which are the B operands of the next chunk's products as they stand.  Row rho of a wave's tile t is state
+// n = 16 NT wave + NT rho + t: a lane's A operands of all tiles lie side by side, in C (registers, four rows of the tiles at a time) as in
+// B (through LDS, the wave's own columns).  The waves' shares of a chunk's outputs meet in LDS, one barrier per chunk; what the next
+// chunk needs is in flight meanwhile.  VEC: whole 16-byte pieces of rows, aligned.
+template <typename T, int NT, bool VEC>
+__global__ __launch_bounds__(256) void ssd_scan_kernel(SsdGeom g, SsdIn in, const AttnSeg* __restrict__ segs, int c0, int nchunks, int nvt, float* __restrict__ base,
+                                                       float* __restrict__ y, int ldy) {
+  extern __shared__ __attribute__((aligned(16))) unsigned char dsm[];
+  f32x4_t (*ps)[4][4][64] = reinterpret_cast<f32x4_t (*)[4][4][64]>(dsm);
+  Steps* st = reinterpret_cast<Steps*>(dsm + 2 * 16 * 64 * 16);
+  float* xs = reinterpret_cast<float*>(st + 2);
+  constexpr int BP = b_pitch<T, NT>(), W = 16 / (int)sizeof(T), LPR = 16 * NT / W, RPL = 64 / LPR;    // elements per 16 bytes; lanes per row, rows per load of B
+  int id = blockIdx.x, h, vt;
+  if (g.H % 8 == 0) {        // the column blocks of a head on one XCD
+    const int k = id >> 3;
+    h = (id & 7) + 8 * (k / nvt);
+    vt = k % nvt;
+  } else {
+    h = id / nvt;
+    vt = id % nvt;
+  }
   const int si = blockIdx.y;
   const AttnSeg sg = segs[si];
   if (sg.n < 2) return;
@@ -448,84 +575,166 @@ __global__ __launch_bounds__(256) void ssd_pass_kernel(SsdGeom g, SsdIn in, cons
   for (int i = 0; i < si; ++i) first += segs[i].n < 2 ? 0 : ceil_div(segs[i].n, kQ);
   const int k0 = max(c0 - first, 0), k1 = min(c0 + nchunks - first, ceil_div(sg.n, kQ));
   if (k0 >= k1) return;
-  const size_t hs = (size_t)g.Np * g.Pp, at = ((size_t)blockIdx.x * 256 + threadIdx.x) * 4;
-  if (at >= g.H * hs) return;
   const Records rec = records_at(base, g, nchunks);
-  const int h = (int)(at / hs);
-  float* slot = in.state + (size_t)in.slots[sg.seq] * g.H * hs + at;
-  float4 S = sg.pos0 + k0 > 0 ? *reinterpret_cast<const float4*>(slot) : make_float4(0.f, 0.f, 0.f, 0.f);
-  constexpr int kAhead = 4;
-  const int n = k1 - k0, r0 = first + k0 - c0;
-  auto add_at = [&](int k) { return rec.state + (size_t)(r0 + min(k, n - 1)) * g.H * hs + at; };
-  auto decay_at = [&](int k) { return rec.decay[(size_t)(r0 + min(k, n - 1)) * g.H + h]; };
-  float4 add[kAhead];
-  float e[kAhead];
+  const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, g4 = lane >> 4, c = lane & 15;
+  const int grp = h / (g.H / g.G), n0 = 16 * NT * wave, p = 16 * vt + c;
+  T* Bs = reinterpret_cast<T*>(xs + 2 * kQ * kXPitch) + wave * kQ * BP;
+  float* S0 = in.state + ((size_t)in.slots[sg.seq] * g.H + h) * g.Np * g.Pp + p;
+  f32x4_t S[NT];
 #pragma unroll
-  for (int i = 0; i < kAhead; ++i) { add[i] = *reinterpret_cast<const float4*>(add_at(i)); e[i] = decay_at(i); }
-  for (int k = 0; k < n; k += kAhead) {
+  for (int t = 0; t < NT; ++t)
 #pragma unroll
-    for (int i = 0; i < kAhead; ++i) {
-      if (k + i < n) {
-      *reinterpret_cast<float4*>(add_at(k + i)) = S;
-      S = make_float4(__builtin_fmaf(e[i], S.x, add[i].x), __builtin_fmaf(e[i], S.y, add[i].y), __builtin_fmaf(e[i], S.z, add[i].z), __builtin_fmaf(e[i], S.w, add[i].w));
-      if (k + i + kAhead < n) { add[i] = *reinterpret_cast<const float4*>(add_at(k + i + kAhead)); e[i] = decay_at(k + i + kAhead); }
+    for (int r = 0; r < 4; ++r) {
+      const int n = n0 + NT * (4 * g4 + r) + t;
+      S[t][r] = sg.pos0 + k0 > 0 && n < g.Np ? S0[(size_t)min(n, g.Np - 1) * g.Pp] : 0.f;
+    }
+  const T* xbc = reinterpret_cast<const T*>(in.xbc) + (size_t)sg.row0 * in.ldx;
+  const int at_b = g.H * g.P + grp * g.N, at_c = at_b + g.G * g.N, at_x = h * g.P + 16 * vt, bn = n0 + (lane % LPR) * W, xn = (tid & 3) * 4;
+  struct Kept { Words<T, 4 * NT> c[4]; f32x4_t cb[4]; };                             // used from registers
+  struct Passed { Words<T, W> b[LPR]; Words<T, 4> x; float s[2]; };                  // passed on to LDS
+  // columns n .. of a row's part of `size` columns; beyond it: anything (C: its states are zero), or zero (B)
+  auto pack = [](auto& o, const T* row, int n, int size, bool zero) {
+    constexpr int M = (int)(sizeof(o.v) / (sizeof(T)));
+    if constexpr (VEC) {
+      o.load(row + min(n, size - M));
+    } else {
+#pragma unroll
+      for (int i = 0; i < M; ++i) {
+        const T x = row[min(n + i, size - 1)];
+        o.set(i, zero && n + i >= size ? T(0) : x);
       }
     }
-  }
-  *reinterpret_cast<float4*>(slot) = S;
-}
-
-// Outputs of a chunk and head: wave w owns tokens 16 w .. + 15
-template <typename T, int NPT>
-__global__ __launch_bounds__(256) void ssd_out_kernel(SsdGeom g, SsdIn in, const AttnSeg* __restrict__ segs, int nseg, int c0, float* __restrict__ base,
-                                                      float* __restrict__ y, int ldy) {
-  extern __shared__ __attribute__((aligned(16))) float sm[];
-  __shared__ double L[kQ];
-  __shared__ float dts[kQ];
-  const ChunkAt at = chunk_at(segs, nseg, c0 + blockIdx.x);
-  if (!at.ok) return;
-  const Records rec = records_at(base, g, gridDim.x);
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, g4 = lane >> 4, c = lane & 15, inner = g.H * g.P, h = blockIdx.y, grp = h / (g.H / g.G);
-  const int mp = kQ + 4, xp = wide_pitch(g.Pp), cp = tall_pitch(g.Np);
-  float *Ms = sm, *xs = Ms + kQ * mp, *Cs = xs + kQ * xp;
-  const T* rows = reinterpret_cast<const T*>(in.xbc) + (size_t)(at.sg.row0 + at.t0) * in.ldx;
-  const float* cb = rec.cb + ((size_t)blockIdx.x * g.G + grp) * kQ * kQ;
-  chunk_steps(in, h, at, L, dts);
-  stage_rows(xs, xp, rows + h * g.P, in.ldx, at.n, g.P, g.Pp, [](int) { return 1.f; });
-  stage_rows(Cs, cp, rows + inner + (g.G + grp) * g.N, in.ldx, at.n, g.N, g.Np, [&](int t) { return expf((float)L[t]); });
-  for (int k = tid; k < kQ * kQ; k += 256) {
-    const int i = k / kQ, j = k % kQ;
-    Ms[i * mp + j] = j <= i ? cb[k] * expf((float)(L[i] - L[j])) * dts[j] : 0.f;
-  }
-  __syncthreads();
-  if (16 * wave >= at.n) return;
-  f32x4_t acc[NPT];
-  int off[NPT];
+  };
+  constexpr int kSteps = sizeof(Steps) / 4;                // floats of a chunk's steps, shared out to the work-group
+  auto load_passed = [&](int k, Passed& d) {
+    const int n = min(kQ, sg.n - k * kQ), rc = first + k - c0;
+    const T* rows = xbc + (size_t)k * kQ * in.ldx;
+    const float* steps = reinterpret_cast<const float*>(rec.steps + (size_t)rc * g.H + h);
 #pragma unroll
-  for (int p = 0; p < NPT; ++p) {
-    acc[p] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    off[p] = min(16 * p, g.Pp - 16) + c;
-  }
-  for (int s = 0; s < 4 * (wave + 1); ++s) {
-    const float a = Ms[(16 * wave + c) * mp + 4 * s + g4];
+    for (int i = 0; i < 2; ++i) d.s[i] = steps[min(tid + 256 * i, kSteps - 1)];
+    pack(d.x, rows + (size_t)min(tid >> 2, n - 1) * in.ldx + at_x, xn, g.P - 16 * vt, false);
 #pragma unroll
-    for (int p = 0; p < NPT; ++p) acc[p] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, xs[(4 * s + g4) * xp + off[p]], acc[p], 0, 0, 0);
-  }
-  const float* S0 = rec.state + ((size_t)blockIdx.x * g.H + h) * g.Np * g.Pp;
-  for (int s = 0; s < g.Np / 4; ++s) {
-    const float a = Cs[(16 * wave + c) * cp + 4 * s + g4];
+    for (int i = 0; i < LPR; ++i) pack(d.b[i], rows + (size_t)min(RPL * i + lane / LPR, n - 1) * in.ldx + at_b, bn, g.N, true);
+  };
+  auto load_kept = [&](int k, Kept& f) {
+    const int n = min(kQ, sg.n - k * kQ), rc = first + k - c0;
+    const T* rows = xbc + (size_t)k * kQ * in.ldx;
 #pragma unroll
-    for (int p = 0; p < NPT; ++p) acc[p] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, S0[(size_t)(4 * s + g4) * g.Pp + off[p]], acc[p], 0, 0, 0);
-  }
-  const float d = in.d[h];
+    for (int i = 0; i < 4; ++i) {
+      pack(f.c[i], rows + (size_t)min(16 * i + c, n - 1) * in.ldx + at_c, n0 + 4 * NT * g4, g.N, false);
+      // (tiles above the diagonal are left out: the wave's own again)
+      f.cb[i] = *reinterpret_cast<const f32x4_t*>(rec.cb + ((size_t)rc * g.G + grp) * kQ * kQ + (16 * wave + c) * kQ + 16 * min(i, wave) + 4 * g4);
+    }
+  };
+  auto post = [&](const Passed& d, int b) {
+    float* s = reinterpret_cast<float*>(&st[b]);
 #pragma unroll
-  for (int p = 0; p < NPT; ++p) {
+    for (int i = 0; i < 2; ++i)
+      if (tid + 256 * i < kSteps) s[tid + 256 * i] = d.s[i];
+    float xv[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) xv[i] = 16 * vt + xn + i < g.P ? d.x.at(i) : 0.f;
+    *reinterpret_cast<float4*>(xs + (b * kQ + (tid >> 2)) * kXPitch + xn) = make_float4(xv[0], xv[1], xv[2], xv[3]);
+#pragma unroll
+    for (int i = 0; i < LPR; ++i) {
+      Words<T, W> v = d.b[i];
+      if constexpr (VEC) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v.v[0][e] = bn < g.N ? v.v[0][e] : 0u;
+      }
+      v.store(Bs + (RPL * i + lane / LPR) * BP + (lane % LPR) * W);
+    }
+  };
+  const float skip = in.d[h];
+  auto step = [&](int k, Kept& f, Kept& next) {
+    const int b = (k - k0) & 1, n = min(kQ, sg.n - k * kQ);
+    const Steps& q = st[b];
+    Passed d;                  // (behind the last chunk: that one again)
+    load_passed(min(k + 1, k1 - 1), d);
+    load_kept(min(k + 1, k1 - 1), next);
+    __builtin_amdgcn_sched_barrier(0);
+    float x[16];               // tokens 16 i + 4 g4 + r (past the last one: its weight and step are zero)
+#pragma unroll
+    for (int i = 0; i < 16; ++i) x[i] = xs[(b * kQ + 16 * (i >> 2) + 4 * g4 + (i & 3)) * kXPitch + c];
+    // share of the outputs that the state holds
+    f32x4_t o[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) o[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int t = 0; t < NT; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.c[i].at(NT * r + t), S[t][r], o[i], 0, 0, 0);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) ps[b][wave][i][lane] = o[i];
+    // the state behind the chunk
+    const float end = q.e[kQ - 1];
+#pragma unroll
+    for (int t = 0; t < NT; ++t) S[t] = f32x4_t{S[t][0] * end, S[t][1] * end, S[t][2] * end, S[t][3] * end};
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const f32x4_t w = *reinterpret_cast<const f32x4_t*>(q.w + 16 * i + 4 * g4);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float xw = x[4 * i + r] * w[r];
+        const Pack<T, NT> bv = *reinterpret_cast<const Pack<T, NT>*>(Bs + (16 * i + 4 * g4 + r) * BP + NT * c);
+#pragma unroll
+        for (int t = 0; t < NT; ++t) S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(to_f32(bv.v[t]), xw, S[t], 0, 0, 0);
+      }
+    }
+    // what the chunk's own tokens add: the wave's 16 tokens
+    f32x4_t own = {0.f, 0.f, 0.f, 0.f};
+    const float hi = q.hi[16 * wave + c], lo = q.lo[16 * wave + c];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      if (j > wave) break;
+      const f32x4_t hj = *reinterpret_cast<const f32x4_t*>(q.hi + 16 * j + 4 * g4), lj = *reinterpret_cast<const f32x4_t*>(q.lo + 16 * j + 4 * g4),
+                    dj = *reinterpret_cast<const f32x4_t*>(q.dt + 16 * j + 4 * g4);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float dt = 16 * j + 4 * g4 + r <= 16 * wave + c ? dj[r] : 0.f, e = __builtin_amdgcn_exp2f(fminf((hi - hj[r]) + (lo - lj[r]), 0.f));
+        own = __builtin_amdgcn_mfma_f32_16x16x4f32(f.cb[j][r] * e * dt, x[4 * j + r], own, 0, 0, 0);
+      }
+    }
+    float xo[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) xo[r] = xs[(b * kQ + 16 * wave + 4 * g4 + r) * kXPitch + c];
+    const f32x4_t e = *reinterpret_cast<const f32x4_t*>(q.e + 16 * wave + 4 * g4);
+    __builtin_amdgcn_sched_barrier(0);
+    post(d, b ^ 1);                     // (B: the wave's own reads of it are done)
+    __syncthreads();
+    f32x4_t sum = ps[b][0][wave][lane];
+#pragma unroll
+    for (int w = 1; w < 4; ++w) {
+      const f32x4_t a = ps[b][w][wave][lane];
+      sum[0] += a[0]; sum[1] += a[1]; sum[2] += a[2]; sum[3] += a[3];
+    }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int i = 16 * wave + 4 * g4 + r;
-      if (i < at.n && 16 * p + c < g.P) y[(size_t)(at.sg.row0 + at.t0 + i) * ldy + h * g.P + 16 * p + c] = __builtin_fmaf(d, xs[i * xp + 16 * p + c], acc[p][r]);
+      if (i < n && p < g.P) y[(size_t)(sg.row0 + k * kQ + i) * ldy + h * g.P + p] = __builtin_fmaf(e[r], sum[r], __builtin_fmaf(skip, xo[r], own[r]));
     }
+  };
+  Kept f[2];
+  {
+    Passed d;
+    load_passed(k0, d);
+    load_kept(k0, f[0]);
+    post(d, 0);
   }
+  __syncthreads();
+  for (int k = k0; k < k1; k += 2) {
+    step(k, f[0], f[1]);
+    if (k + 1 < k1) step(k + 1, f[1], f[0]);
+  }
+#pragma unroll
+  for (int t = 0; t < NT; ++t)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int n = n0 + NT * (4 * g4 + r) + t;
+      if (n < g.Np) S0[(size_t)n * g.Pp] = S[t][r];
+    }
 }
 
 // one work-group per row; a part is shared out to several waves where there are fewer parts than waves (summed in wave order)
@@ -579,11 +788,11 @@ int check_scan(const ScanGeom& g, const ScanIn& in, const void* y, int ldy) {
   MI_CHECK(in.ldx >= g.C && in.ldz >= g.C && ldy >= g.C && in.col_b >= g.rank && in.col_c >= in.col_b + g.N && in.ldl >= in.col_c + g.N, "selective scan: columns");
   return MI_OK;
 }
-int check_ssd(const SsdGeom& g, const SsdIn& in, const float* y, int ldy) {
+int check_ssd(const SsdGeom& g, const SsdIn& in, const float* y, int ldy, bool convolved = false) {
   MI_CHECK(ssd_supported(g), "state-space duality: heads must be a multiple of the groups, sizes 1 .. 256");
   MI_CHECK(g.Np % 16 == 0 && g.Np >= g.N && g.Np < g.N + 16 && g.Pp % 16 == 0 && g.Pp >= g.P && g.Pp < g.P + 16, "state-space duality: padding");
-  MI_CHECK(in.xbc && in.dt && in.dt_bias && in.a_log && in.d && in.state && in.slots && in.pos && y, "state-space duality: null argument");
-  MI_CHECK(in.ldx >= g.channels() && in.ldt >= g.H && ldy >= g.inner(), "state-space duality: columns");
+  MI_CHECK((convolved || (in.xbc && in.ldx >= g.channels())) && in.dt && in.dt_bias && in.a_log && in.d && in.state && in.slots && in.pos && y, "state-space duality: null argument");
+  MI_CHECK(in.ldt >= g.H && ldy >= g.inner(), "state-space duality: columns");
   return MI_OK;
 }
 
@@ -632,12 +841,24 @@ int launch_scan_token(const ScanGeom& g, const ScanIn& in, int rows, const AttnS
   int rc = check_scan(g, in, y, ldy);
   if (rc != MI_OK) return rc;
   MI_CHECK(rows >= 1 && rows <= 65535 && in.w_dt, "selective scan: rows");
-#define MI_ST(LPC, R) { \
-    const dim3 grid(ceil_div(g.C, 256 / LPC), rows); \
-    if (f32) hipLaunchKernelGGL((scan_token_kernel<float, LPC, R>), grid, dim3(256), 0, s, g, in, segs, (float*)y, ldy); \
-    else hipLaunchKernelGGL((scan_token_kernel<uint16_t, LPC, R>), grid, dim3(256), 0, s, g, in, segs, (uint16_t*)y, ldy); }
-  MI_BY_STATE(MI_ST)
+  // several rows: four of them per work-group; many: four states per lane as well (fewer, wider loads)
+  const bool several = rows >= 3 && g.Np <= 64, many = several && rows > 8;
+  const int rb = several ? 4 : 1;
+  const size_t lds = (size_t)rb * g.rank_p * 4;
+  MI_CHECK(lds <= 48 * 1024, "selective scan: the step sizes' rank is too large");
+#define MI_ST_(LPC, R, RB) { \
+    const dim3 grid(ceil_div(g.C, 256 / LPC), ceil_div(rows, rb)); \
+    if (f32) hipLaunchKernelGGL((scan_token_kernel<float, LPC, R, RB>), grid, dim3(256), lds, s, g, in, segs, rows, (float*)y, ldy); \
+    else hipLaunchKernelGGL((scan_token_kernel<uint16_t, LPC, R, RB>), grid, dim3(256), lds, s, g, in, segs, rows, (uint16_t*)y, ldy); }
+#define MI_ST(LPC, R) MI_ST_(LPC, R, 1)
+  if (!several) {
+    MI_BY_STATE(MI_ST)
+  } else if (g.Np == 8) { if (many) MI_ST_(4, 2, 4) else MI_ST_(8, 1, 4) }
+  else if (g.Np == 16) { if (many) MI_ST_(4, 4, 4) else MI_ST_(16, 1, 4) }
+  else if (g.Np == 32) { if (many) MI_ST_(8, 4, 4) else MI_ST_(16, 2, 4) }
+  else MI_ST_(16, 4, 4)
 #undef MI_ST
+#undef MI_ST_
   MI_HIP(hipGetLastError());
   return MI_OK;
 }
@@ -673,17 +894,21 @@ SsdGeom ssd_geom(int H, int P, int N, int G) { return SsdGeom{H, P, N, G, (P + 1
 bool ssd_supported(const SsdGeom& g) {
   return g.H >= 1 && g.G >= 1 && g.H % g.G == 0 && g.P >= 1 && g.P <= 256 && g.N >= 1 && g.N <= 256;
 }
-size_t ssd_chunk_floats(const SsdGeom& g) { return g.state_floats() + (size_t)g.G * kQ * kQ + g.H; }
+size_t ssd_chunk_floats(const SsdGeom& g) { return (size_t)g.G * kQ * kQ + (size_t)g.H * sizeof(Steps) / 4; }
 
-int launch_ssd_token(const SsdGeom& g, const SsdIn& in, int rows, const AttnSeg* segs, float* y, int ldy, bool f32, hipStream_t s) {
-  int rc = check_ssd(g, in, y, ldy);
+int launch_ssd_token(const SsdGeom& g, const SsdIn& in, int rows, const AttnSeg* segs, float* y, int ldy, bool f32, hipStream_t s, const ShortConv* conv, const float* proj,
+                     int ldp) {
+  int rc = check_ssd(g, in, y, ldy, conv != nullptr);
   if (rc != MI_OK) return rc;
+  MI_CHECK(!conv == !proj && (!conv || (conv->w && conv->b && conv->ring && conv->slots && conv->taps >= 1 && conv->taps <= 16 && conv->C == g.channels() && ldp >= conv->C)),
+           "state-space duality: convolution");
+  const ShortConv cv = conv ? *conv : ShortConv();
   MI_CHECK(rows >= 1 && rows <= 65535, "state-space duality: rows");
   const dim3 grid(g.H, rows);
   const int vq = g.Pp <= 16 ? 4 : g.Pp <= 32 ? 8 : g.Pp <= 64 ? 16 : g.Pp <= 128 ? 32 : 64, need = ceil_div(g.Np, kTokenThreads / vq);
 #define MI_ST(VQ, RPT) \
-  if (f32) hipLaunchKernelGGL((ssd_token_kernel<float, VQ, RPT>), grid, dim3(kTokenThreads), 0, s, g, in, segs, y, ldy); \
-  else hipLaunchKernelGGL((ssd_token_kernel<uint16_t, VQ, RPT>), grid, dim3(kTokenThreads), 0, s, g, in, segs, y, ldy)
+  if (f32) hipLaunchKernelGGL((ssd_token_kernel<float, VQ, RPT>), grid, dim3(kTokenThreads), 0, s, g, in, cv, proj, ldp, segs, y, ldy); \
+  else hipLaunchKernelGGL((ssd_token_kernel<uint16_t, VQ, RPT>), grid, dim3(kTokenThreads), 0, s, g, in, cv, proj, ldp, segs, y, ldy)
   if (vq == 4) { if (need <= 1) { MI_ST(4, 1); } else { MI_ST(4, 2); } }
   else if (vq == 8) { if (need <= 1) { MI_ST(8, 1); } else if (need <= 2) { MI_ST(8, 2); } else { MI_ST(8, 4); } }
   else if (vq == 16) { if (need <= 2) { MI_ST(16, 2); } else if (need <= 4) { MI_ST(16, 4); } else { MI_ST(16, 8); } }
@@ -701,30 +926,28 @@ int launch_ssd_prompt(const SsdGeom& g, const SsdIn& in, const AttnSeg* sd, cons
   MI_CHECK(nseg >= 1 && nseg <= 65535 && records && max_chunks >= 1, "state-space duality: segments / workspace");
   int chunks = 0;
   for (int i = 0; i < nseg; ++i) chunks += sh[i].n < 2 ? 0 : ceil_div(sh[i].n, kQ);
-  const size_t lds_c = (size_t)kQ * std::max(wide_pitch(g.Np) + wide_pitch(g.Pp), 2 * tall_pitch(g.Np)) * 4;
-  const size_t lds_o = (size_t)kQ * (kQ + 4 + wide_pitch(g.Pp) + tall_pitch(g.Np)) * 4;
-  const int npt = g.Pp <= 16 ? 1 : g.Pp <= 32 ? 2 : g.Pp <= 64 ? 4 : g.Pp <= 128 ? 8 : 16;
+  const size_t lds = (size_t)kQ * 2 * tall_pitch(g.Np) * 4;
+  const int nvt = g.Pp / 16, nt = g.Np <= 64 ? 1 : g.Np <= 128 ? 2 : 4;
+  // whole packs of B, C and x, rows and groups aligned to them
+  const int unit = std::max(4 * nt, 8);
+  const bool vec = g.N % unit == 0 && g.inner() % unit == 0 && g.P % 4 == 0 && in.ldx % unit == 0 && (reinterpret_cast<uintptr_t>(in.xbc) & 63) == 0;
   for (int c0 = 0; c0 < chunks; c0 += max_chunks) {
     const int n = std::min(max_chunks, chunks - c0);
-    const dim3 gc(n, g.H + g.G), gp((unsigned)ceil_div((int)(g.state_floats() / 4), 256), nseg), go(n, g.H);
-#define MI_SSD_LDS(KERN, BYTES) \
-    if (BYTES > 48 * 1024) { rc = ensure_dynamic_lds(reinterpret_cast<const void*>(KERN), (int)(BYTES)); if (rc != MI_OK) return rc; }
-#define MI_SSD_CHUNK(T) { auto k = ssd_chunk_kernel<T>; MI_SSD_LDS(k, lds_c) hipLaunchKernelGGL(k, gc, dim3(256), lds_c, s, g, in, sd, nseg, c0, records); }
-#define MI_SSD_OUT(T, NPT) { auto k = ssd_out_kernel<T, NPT>; MI_SSD_LDS(k, lds_o) hipLaunchKernelGGL(k, go, dim3(256), lds_o, s, g, in, sd, nseg, c0, records, y, ldy); }
-#define MI_SSD_OUT_T(NPT) if (f32) MI_SSD_OUT(float, NPT) else MI_SSD_OUT(uint16_t, NPT)
+    const dim3 gc(n, g.G + ceil_div(g.H, 4)), gs(g.H * nvt, nseg);
+#define MI_SSD_CHUNK(T) { auto k = ssd_chunk_kernel<T>; \
+      if (lds > 48 * 1024) { rc = ensure_dynamic_lds(reinterpret_cast<const void*>(k), (int)lds); if (rc != MI_OK) return rc; } \
+      hipLaunchKernelGGL(k, gc, dim3(256), lds, s, g, in, sd, nseg, c0, records); }
+#define MI_SSD_SCAN(T, NT, VEC) { auto k = ssd_scan_kernel<T, NT, VEC>; constexpr size_t bytes = scan_lds<T, NT>(); \
+      if (bytes > 64 * 1024) { rc = ensure_dynamic_lds(reinterpret_cast<const void*>(k), (int)bytes); if (rc != MI_OK) return rc; } \
+      hipLaunchKernelGGL(k, gs, dim3(256), bytes, s, g, in, sd, c0, n, nvt, records, y, ldy); }
+#define MI_SSD_SCAN_V(T, NT) if (vec) MI_SSD_SCAN(T, NT, true) else MI_SSD_SCAN(T, NT, false)
+#define MI_SSD_SCAN_T(NT) if (f32) { MI_SSD_SCAN_V(float, NT) } else { MI_SSD_SCAN_V(uint16_t, NT) }
     if (f32) MI_SSD_CHUNK(float) else MI_SSD_CHUNK(uint16_t)
-    hipLaunchKernelGGL(ssd_pass_kernel, gp, dim3(256), 0, s, g, in, sd, c0, n, records);
-    switch (npt) {
-      case 1: MI_SSD_OUT_T(1); break;
-      case 2: MI_SSD_OUT_T(2); break;
-      case 4: MI_SSD_OUT_T(4); break;
-      case 8: MI_SSD_OUT_T(8); break;
-      default: MI_SSD_OUT_T(16);
-    }
-#undef MI_SSD_OUT_T
-#undef MI_SSD_OUT
+    if (nt == 1) { MI_SSD_SCAN_T(1) } else if (nt == 2) { MI_SSD_SCAN_T(2) } else { MI_SSD_SCAN_T(4) }
+#undef MI_SSD_SCAN_T
+#undef MI_SSD_SCAN_V
+#undef MI_SSD_SCAN
 #undef MI_SSD_CHUNK
-#undef MI_SSD_LDS
     MI_HIP(hipGetLastError());
   }
   return MI_OK;

@@ -1573,11 +1573,14 @@ int one_norm_trunk(mi_ctx* c, const Batch& b, int& cur) {
 }
 
 // ---- post-norm blocks ----------------------------------------------------------------------------------------------------------
+ShortConv short_conv(const mi_ctx* c, const StackLayer& W, float* state) {
+  return ShortConv{W.conv, W.conv_b, W.s.conv_taps, W.conv_channels(), state + (size_t)c->stack->state_slots * W.ssm_state_floats(), c->d_state};
+}
 int post_norm_conv(mi_ctx* c, const StackLayer& W, float* state, const Batch& b, int col, int ldc) {
   Stack* S = c->stack;
   if (!runs_other(c)) return MI_OK;
   Scope sc(c, MI_K_OTHER);
-  const ShortConv cv{W.conv, W.conv_b, W.s.conv_taps, W.conv_channels(), state + (size_t)S->state_slots * W.ssm_state_floats(), c->d_state};
+  const ShortConv cv = short_conv(c, W, state);
   return launch_short_conv(S->qkv_out + col, W.qkv.N, cv, c->d_pos, reinterpret_cast<const AttnSeg*>(c->d_segs), b.segs, b.decode ? 0 : b.nseg, b.rows, S->xc, ldc,
                            S->f32, c->stream);
 }
@@ -1628,7 +1631,7 @@ int post_norm_ssd(mi_ctx* c, const StackLayer& W, float* state, const Batch& b) 
   const SsdGeom& g = W.ssd;
   hipStream_t s = c->stream;
   const int ldc = pad_to(g.channels(), 16), ldy = pad_to(g.inner(), 16);
-  MI_TRY(post_norm_conv(c, W, state, b, W.col_x, ldc));
+  if (!b.decode) MI_TRY(post_norm_conv(c, W, state, b, W.col_x, ldc));
   SsdIn in;
   in.xbc = S->xc; in.ldx = ldc;
   in.dt = S->qkv_out + W.col_dt; in.ldt = W.qkv.N;
@@ -1638,7 +1641,8 @@ int post_norm_ssd(mi_ctx* c, const StackLayer& W, float* state, const Batch& b) 
   if (c->runs(cls)) {
     Scope sc(c, cls);
     if (b.decode) {
-      MI_TRY(launch_ssd_token(g, in, b.rows, nullptr, S->yssm, ldy, S->f32, s));
+      const ShortConv cv = short_conv(c, W, state);
+      MI_TRY(launch_ssd_token(g, in, b.rows, nullptr, S->yssm, ldy, S->f32, s, &cv, S->qkv_out + W.col_x, W.qkv.N));
     } else {
       int ones = 0;
       for (int i = 0; i < b.nseg; ++i) ones += b.segs[i].n == 1;
